@@ -160,8 +160,7 @@ PYBIND11_MODULE(_engine, m) {
       .def_readwrite("vocab_parallel", &EngineConfig::vocab_parallel)
       .def_readwrite("device", &EngineConfig::device)
       .def_readwrite("cu_mask", &EngineConfig::cu_mask)
-      .def_readwrite("kv_fp8", &EngineConfig::kv_fp8)
-      .def_readwrite("stream_priority", &EngineConfig::stream_priority);
+      .def_readwrite("kv_fp8", &EngineConfig::kv_fp8);
 
   py::class_<Engine>(m, "Engine")
       .def(py::init<const EngineConfig&>())

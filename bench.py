@@ -160,7 +160,7 @@ def measure_coresident(steps: int = 256, prompt: int = 128, cu_split: int = 0):
     sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "tools"))
     from bench_coresident import run
 
-    return run(_ap.Namespace(steps=steps, prompt=prompt, cu_split=cu_split, priority=""))
+    return run(_ap.Namespace(steps=steps, prompt=prompt, cu_split=cu_split))
 
 
 def measure_tp(args, rank: int, world: int, device: int, gloo):

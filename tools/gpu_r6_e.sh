@@ -1,5 +1,5 @@
 #!/bin/bash
-# fp8 KV attention with 16 dims per lane (hd 128): numerics + long context; co-resident priority streams
+# fp8 KV attention with 16 dims per lane (hd 128): numerics + long context
 set -o pipefail
 mkdir -p gpurun_out
 export HSA_ENABLE_IPC_MODE_LEGACY=0
@@ -19,7 +19,3 @@ done; done
 BENCH_ARGS="--prompt 32000 --kv-dtype fp8_e4m3" timeout -k 10 700 bash tools/prof_decode.sh > /dev/null 2>&1 || { tail -20 gpurun_out/prof.log; exit 1; }
 cp gpurun_out/prof_summary.txt gpurun_out/prof_mistral_32k_fp8.txt
 head -14 gpurun_out/prof_mistral_32k_fp8.txt
-for pr in mistral tinyllama; do
-  timeout -k 10 300 python tools/bench_coresident.py --steps 512 --priority $pr > gpurun_out/cores_p_$pr.json 2>gpurun_out/cores.err || { tail -20 gpurun_out/cores.err; exit 1; }
-  echo "priority $pr: $(cat gpurun_out/cores_p_$pr.json)"
-done
