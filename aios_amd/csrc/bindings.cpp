@@ -135,6 +135,26 @@ PYBIND11_MODULE(_engine, m) {
   m.def("synchronize", []() { HIP_CHECK(hipDeviceSynchronize()); });
   m.def("resid_norm_parts", &resid_norm_parts, py::arg("d"));
 
+  m.attr("MIX_LATENT") = (int)MIX_LATENT;
+  m.attr("MLP_NONE") = (int)MLP_NONE;
+  m.attr("MLP_GLU") = (int)MLP_GLU;
+  m.attr("ACT_SILU") = (int)ACT_SILU;
+  m.attr("ACT_GELU_TANH") = (int)ACT_GELU_TANH;
+  py::class_<LayerSpec>(m, "LayerSpec")
+      .def(py::init<>())
+      .def_readwrite("mixer", &LayerSpec::mixer)
+      .def_readwrite("heads", &LayerSpec::heads)
+      .def_readwrite("dim", &LayerSpec::dim)
+      .def_readwrite("vdim", &LayerSpec::vdim)
+      .def_readwrite("kv_rank", &LayerSpec::kv_rank)
+      .def_readwrite("scale", &LayerSpec::scale)
+      .def_readwrite("sink", &LayerSpec::sink)
+      .def_readwrite("out_gate", &LayerSpec::out_gate)
+      .def_readwrite("mlp", &LayerSpec::mlp)
+      .def_readwrite("ff", &LayerSpec::ff)
+      .def_readwrite("act", &LayerSpec::act)
+      .def_readwrite("weights_of", &LayerSpec::weights_of);
+
   py::class_<EngineConfig>(m, "EngineConfig")
       .def(py::init<>())
       .def_readwrite("name", &EngineConfig::name)
@@ -160,7 +180,11 @@ PYBIND11_MODULE(_engine, m) {
       .def_readwrite("vocab_parallel", &EngineConfig::vocab_parallel)
       .def_readwrite("device", &EngineConfig::device)
       .def_readwrite("cu_mask", &EngineConfig::cu_mask)
-      .def_readwrite("kv_fp8", &EngineConfig::kv_fp8);
+      .def_readwrite("kv_fp8", &EngineConfig::kv_fp8)
+      .def_readwrite("layers", &EngineConfig::layers)
+      .def_readwrite("max_positions", &EngineConfig::max_positions)
+      .def_readwrite("compute_f32", &EngineConfig::compute_f32)
+      .def_readwrite("kv_pool_tokens", &EngineConfig::kv_pool_tokens);
 
   py::class_<Engine>(m, "Engine")
       .def(py::init<const EngineConfig&>())
@@ -261,6 +285,41 @@ PYBIND11_MODULE(_engine, m) {
       .def("release_slot", &Engine::release_slot)
       .def("block_table", &Engine::block_table)
       .def_property_readonly("kv_blocks_free", &Engine::kv_blocks_free)
+      .def_property_readonly("kv_block_tokens", &Engine::kv_block_tokens)
+      .def_property_readonly("mixed_steps", &Engine::mixed_steps)
+      .def("step",
+           [](Engine& e, const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
+              const std::vector<int>& tokens, const std::vector<int>& want) {
+             std::vector<float> v;
+             {
+               py::gil_scoped_release nogil;
+               v = e.step(slots, starts, counts, tokens, want);
+             }
+             py::array_t<float> a({(py::ssize_t)want.size(), (py::ssize_t)e.config().vocab_size});
+             std::memcpy(a.mutable_data(), v.data(), v.size() * 4);
+             return a;
+           },
+           py::arg("slots"), py::arg("starts"), py::arg("counts"), py::arg("tokens"), py::arg("want"))
+      .def("step_sample",
+           [](Engine& e, const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
+              const std::vector<int>& tokens, const std::vector<int>& sample, const std::vector<float>& temperature,
+              const std::vector<int>& top_k, const std::vector<float>& top_p, const std::vector<uint64_t>& seeds,
+              py::bytes mask) {
+             std::string m = mask;
+             std::vector<uint8_t> mv(m.begin(), m.end());
+             py::gil_scoped_release nogil;
+             return e.step_sample(slots, starts, counts, tokens, sample, temperature, top_k, top_p, seeds, mv);
+           },
+           py::arg("slots"), py::arg("starts"), py::arg("counts"), py::arg("tokens"), py::arg("sample"),
+           py::arg("temperature"), py::arg("top_k"), py::arg("top_p"), py::arg("seeds"), py::arg("mask") = py::bytes())
+      .def("last_residual",
+           [](Engine& e, int rows) {
+             std::vector<float> v = e.last_residual(rows);
+             py::array_t<float> a({(py::ssize_t)rows, (py::ssize_t)e.config().d_model});
+             std::memcpy(a.mutable_data(), v.data(), v.size() * 4);
+             return a;
+           },
+           py::arg("rows"))
       .def_property_readonly("kv_blocks_total", &Engine::kv_blocks_total)
       .def_property_readonly("norm_fused_parts", &Engine::norm_fused_parts)
       .def("capture_graphs", &Engine::capture_graphs, py::arg("max_b"), py::call_guard<py::gil_scoped_release>())

@@ -71,6 +71,13 @@ __device__ __forceinline__ uint16_t f32_to_bf16(float f) {
   u += 0x7fffu + ((u >> 16) & 1u);
   return (uint16_t)(u >> 16);
 }
+// activation of a gated MLP's gate: z * sigmoid(z) (SiLU), or GELU in its tanh form, which is
+// z * sigmoid(2 sqrt(2 / pi) (z + 0.044715 z^3)) since (1 + tanh u) / 2 = sigmoid(2 u)
+enum GluAct : int { ACT_SILU = 0, ACT_GELU_TANH = 1 };
+__device__ __forceinline__ float glu_act(float z, int act) {
+  const float u = act == ACT_GELU_TANH ? 1.5957691216057308f * fmaf(0.044715f * z * z, z, z) : z;
+  return z / (1.f + __expf(-u));
+}
 __device__ __forceinline__ float h2f(uint16_t h) { return __half2float(__ushort_as_half(h)); }
 
 // ---- KV cache element formats: bf16, or OCP fp8 e4m3 (gfx950's e4m3fn, max 448) with a per-layer

@@ -15,6 +15,7 @@
 #include <vector>
 
 #include "common.h"
+#include "layered.h"
 #include "ops.h"
 
 namespace aios {
@@ -52,6 +53,12 @@ struct EngineConfig {
   // CU mask of the engine's stream (hipExtStreamCreateWithCUMask; 32 CUs per word, empty = every CU):
   // co-resident tiers each get their own CUs, and the engine sizes its grids to the mask's CU count
   std::vector<uint32_t> cu_mask;
+  // models described layer by layer (layered.h); empty: a llama-family decoder of the sizes above
+  std::vector<LayerSpec> layers;
+  int max_positions = 0;   // rows of the learned position table (layered models)
+  int compute_f32 = 0;     // everything in 32 bits (layered models)
+  // tokens the cache pool holds (whole blocks); 0: every slot's full context at once
+  int kv_pool_tokens = 0;
 };
 
 // device matrix in repacked layout (owns its buffer)
@@ -177,11 +184,47 @@ class Engine {
   int norm_fused_parts() const { return nrm_parts_; }  // 0: batched-decode RMSNorm not split into the GEMMs
   std::vector<int> block_table(int slot) const;
 
+  int kv_block_tokens() const { return kvb_; }
+
+  // ---- mixed batches (layered models) --------------------------------------------------------------
+  // One step over several sequences: entry e brings counts[e] tokens (consecutive in `tokens`) at
+  // positions starts[e].. of slots[e] -- portions of prompts and single decoded tokens alike, run as one
+  // batch.  `want`: indices into `tokens` whose logits are returned (host, [want][vocab]), ascending.
+  std::vector<float> step(const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
+                          const std::vector<int>& tokens, const std::vector<int>& want);
+  // the same step, sampling the token after the last one of every entry with sample[e] != 0 (at most
+  // max_batch of them) on the device, with the decode steps' sampler and RNG stream (seed, position);
+  // the sampling vectors and mask rows are per sampled entry
+  std::vector<int> step_sample(const std::vector<int>& slots, const std::vector<int>& starts,
+                               const std::vector<int>& counts, const std::vector<int>& tokens,
+                               const std::vector<int>& sample, const std::vector<float>& temperature,
+                               const std::vector<int>& top_k, const std::vector<float>& top_p,
+                               const std::vector<uint64_t>& seeds, const std::vector<uint8_t>& mask);
+  bool mixed_steps() const { return lm_ != nullptr; }
+  // residual stream of the last step's first `rows` rows (after the last layer), before the final norm
+  std::vector<float> last_residual(int rows);
+
   // raw device pointers for tests / custom kernels
   uintptr_t kv_cache_k() const { return (uintptr_t)k_cache_; }
   uintptr_t kv_cache_v() const { return (uintptr_t)v_cache_; }
 
  private:
+  friend class LayeredDecoder;
+  std::unique_ptr<LayeredDecoder> lm_;   // layered models; null: llama family
+  int ldl_ = 0;                          // row stride of logits_
+  int kvb_ = KV_BLOCK;                   // tokens per cache block
+  // every cache pool: base and bytes of one block (copy-on-write and prefix sharing copy whole blocks)
+  struct Pool {
+    char* base;
+    size_t block;
+  };
+  std::vector<Pool> pools_;
+  void init_paging();                    // block tables and the free list
+  size_t init_step_state();              // logits, decode parameters, sampler (workspace bytes)
+  void finalize_layered();
+  int ctx_limit() const;                 // positions a sequence may use
+  void run_step(const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
+                const std::vector<int>& tokens, const std::vector<int>& want, std::vector<float>* logits);
   void enqueue_decode_step(int B);       // uses device arrays d_tokens_/d_pos_/d_seqlen_/d_slot_
   void enqueue_decode_forward(int B);    // ... up to the logits (no sampler)
   void enqueue_sample(int B);            // the step's sampler (sample_mask_: with d_mask_)

@@ -78,6 +78,8 @@ Engine::Engine(const EngineConfig& cfg) : cfg_(cfg) {
     HIP_CHECK(hipStreamCreateWithFlags(&stream_, hipStreamNonBlocking));
   }
 
+  if (!cfg_.layers.empty()) cfg_.n_layers = (int)cfg_.layers.size();
+  if (cfg_.compute_f32 && cfg_.layers.empty()) throw std::runtime_error("compute_f32: layered models only");
   layers_.resize(cfg_.n_layers);
   // B <= 8 decodes through the fused GEMVs; larger batches (up to 64) through the MFMA GEMM path
   if (cfg_.max_batch < 1 || cfg_.max_batch > 64) throw std::runtime_error("max_batch must be 1..64");
@@ -85,9 +87,15 @@ Engine::Engine(const EngineConfig& cfg) : cfg_(cfg) {
   if (cfg_.tp_size <= 1 || cfg_.tie_embeddings) cfg_.vocab_parallel = 0;
   if (cfg_.vocab_parallel && cfg_.vocab_size % cfg_.tp_size)
     throw std::runtime_error("vocab_parallel: vocab_size not divisible by tp_size");
+  if (!cfg_.layers.empty()) {
+    kvb_ = 64;  // one key tile of the latent attention
+    lm_.reset(new LayeredDecoder(*this));
+  }
 }
 
 Engine::~Engine() {
+  if (lm_) (void)hipStreamSynchronize(stream_);
+  lm_.reset();
   try {
     stage_release();
   } catch (...) {
@@ -283,6 +291,7 @@ void Engine::set_tensor(const std::string& name, int qt, int rows, int cols, con
   const CuScope cu_scope(cus_);  // (grids sized to this engine's CU mask)
   if (finalized_) throw std::runtime_error("set_tensor after finalize");
   HIP_CHECK(hipSetDevice(cfg_.device));
+  if (lm_) return lm_->set_tensor(name, qt, rows, cols, host, nbytes);
   static const std::regex blk_re(R"(blk\.(\d+)\.(.+))");
   std::smatch m;
   if (name == "token_embd.weight") {
@@ -355,6 +364,10 @@ void Engine::init_random(const std::string& recipe_in, uint64_t seed) {
   HIP_CHECK(hipSetDevice(cfg_.device));
   std::string r = recipe_in;
   std::transform(r.begin(), r.end(), r.begin(), ::toupper);
+  if (lm_) {
+    if (r != "BF16") throw std::runtime_error("layered models hold bf16 weights (recipe BF16)");
+    return lm_->init_random(seed);
+  }
   const int d = cfg_.d_model, qd = cfg_.n_heads * cfg_.head_dim, kvd = cfg_.n_kv_heads * cfg_.head_dim;
   const int ff = cfg_.d_ff, V = cfg_.vocab_size, NL = cfg_.n_layers;
   auto more_bits = [&](int i) { return i < NL / 8 || i >= 7 * NL / 8 || (i - NL / 8) % 3 == 2; };
@@ -425,6 +438,7 @@ void Engine::init_random(const std::string& recipe_in, uint64_t seed) {
 }
 
 std::vector<std::string> Engine::missing_tensors() const {
+  if (lm_) return lm_->missing();
   std::vector<std::string> miss;
   if (!tok_embd_.valid()) miss.push_back("token_embd.weight");
   if (!out_norm_) miss.push_back("output_norm.weight");
@@ -457,75 +471,29 @@ std::string Engine::weight_type_summary() const {
 
 static std::vector<std::vector<const QMat*>> qkv_groups(const LayerW& L);
 
-void Engine::finalize() {
-  const CuScope cu_scope(cus_);  // (grids sized to this engine's CU mask)
-  TraceRange tr("aios.finalize");
-  HIP_CHECK(hipSetDevice(cfg_.device));
-  stage_release();  // weights are in place: drop the load-time staging buffers
-  auto miss = missing_tensors();
-  if (!miss.empty()) throw std::runtime_error("missing tensors, first: " + miss[0]);
-  if (!output_.valid()) {
-    if (!cfg_.tie_embeddings) cfg_.tie_embeddings = 1;
-    cfg_.vocab_parallel = 0;  // the tied table is the full vocabulary
-    output_ = tok_embd_;  // tied embeddings (GGUF files without output.weight)
-  }
-  const int d = cfg_.d_model, hd = cfg_.head_dim, H = cfg_.n_heads, Hkv = cfg_.n_kv_heads;
-  const int qd = H * hd, kvd = Hkv * hd, V = cfg_.vocab_size, Bm = cfg_.max_batch;
-  if (cfg_.max_ctx % KV_BLOCK) cfg_.max_ctx = (int)align_up(cfg_.max_ctx, KV_BLOCK);  // whole KV blocks
-  // paged KV pool: max_slots * max_ctx / KV_BLOCK blocks always suffice (a mapping or
-  // un-sharing step never needs more distinct blocks than there are table entries) + one null
-  // block that unmapped table entries point to on the device
-  kv_maxb_ = cfg_.max_ctx / KV_BLOCK;
+// block tables and the free list.  By default max_slots * max_ctx / block blocks, which always suffice (a
+// mapping or un-sharing step never needs more distinct blocks than there are table entries), or the
+// blocks of kv_pool_tokens; + one null block that unmapped table entries point to on the device
+void Engine::init_paging() {
+  kv_maxb_ = (cfg_.max_ctx + kvb_ - 1) / kvb_;
   kv_nblocks_ = cfg_.max_slots * kv_maxb_;
+  if (cfg_.kv_pool_tokens > 0) kv_nblocks_ = std::min(kv_nblocks_, (cfg_.kv_pool_tokens + kvb_ - 1) / kvb_);
   bt_.assign((size_t)cfg_.max_slots * kv_maxb_, -1);
   refcnt_.assign(kv_nblocks_, 0);
   free_blocks_.clear();
   for (int b = kv_nblocks_ - 1; b >= 0; --b) free_blocks_.push_back(b);
-  row_bt_host_.assign((size_t)Bm * kv_maxb_, kv_nblocks_);
-  layer_kv_elems_ = (size_t)(kv_nblocks_ + 1) * Hkv * KV_BLOCK * hd;
-  kv_es_ = cfg_.kv_fp8 ? 1 : 2;  // bytes per cached element (fp8 e4m3 or bf16)
-  kv_bytes_ = 2 * layer_kv_elems_ * cfg_.n_layers * kv_es_;
-  if (kv_scale_.size() != (size_t)2 * cfg_.n_layers) kv_scale_.assign((size_t)2 * cfg_.n_layers, 1.f);
-  k_cache_ = (bf16_t*)dmalloc(kv_bytes_ / 2);
-  v_cache_ = (bf16_t*)dmalloc(kv_bytes_ / 2);
-  HIP_CHECK(hipMemset(k_cache_, 0, kv_bytes_ / 2));
-  HIP_CHECK(hipMemset(v_cache_, 0, kv_bytes_ / 2));
-  n_chunks_ = (cfg_.max_ctx + ATTN_CHUNK - 1) / ATTN_CHUNK;
-  {
-    const size_t nc = (size_t)std::max(prefill_rows_, Bm) * H;  // decode attention tickets [row][head]
-    attn_cnt_ = (int*)dmalloc(nc * 4);
-    HIP_CHECK(hipMemset(attn_cnt_, 0, nc * 4));
-  }
-  {
-    const int half = hd / 2;
-    std::vector<float> tab((size_t)cfg_.max_ctx * half * 2);
-    for (int pos = 0; pos < cfg_.max_ctx; ++pos)
-      for (int p = 0; p < half; ++p) {
-        const double th = (double)pos * std::pow((double)cfg_.rope_theta, -2.0 * p / (double)hd);
-        tab[((size_t)pos * half + p) * 2] = (float)std::cos(th);
-        tab[((size_t)pos * half + p) * 2 + 1] = (float)std::sin(th);
-      }
-    rope_cs_ = (float2*)dmalloc(tab.size() * 4);
-    HIP_CHECK(hipMemcpy(rope_cs_, tab.data(), tab.size() * 4, hipMemcpyHostToDevice));
-  }
+  row_bt_host_.assign((size_t)cfg_.max_batch * kv_maxb_, kv_nblocks_);
+}
 
+// what every model's steps need around the forward: logits, the decode parameter block, device block
+// tables, the sampler's scratch, the token history
+size_t Engine::init_step_state() {
+  const int V = cfg_.vocab_size, Bm = cfg_.max_batch;
   size_t ws = 0;
   auto fbuf = [&](size_t n) { ws += n * 4; return (float*)dmalloc(n * 4); };
   auto ibuf = [&](size_t n) { ws += n * 4; int* p = (int*)dmalloc(n * 4); HIP_CHECK(hipMemset(p, 0, n * 4)); return p; };
-  x_ = fbuf((size_t)Bm * d);
-  q_ = fbuf((size_t)Bm * qd);
-  qkv_ = fbuf((size_t)Bm * (qd + 2 * kvd));
-  attn_ = fbuf((size_t)Bm * std::max(qd, d));
-  ff_ = fbuf((size_t)Bm * std::max(cfg_.d_ff, d));
-  // (the BF16 engine stages its x as bf16 whatever act_q8 says: the hand-off serves it too)
-  if ((cfg_.act_q8 || layers_[0].wgu.w.qtype == QT_BF16) && cfg_.d_ff % 8 == 0 &&
-      !(std::getenv("AIOS_FF16") && std::atoi(std::getenv("AIOS_FF16")) == 0)) {
-    gv_ff16_ = (bf16_t*)dmalloc((size_t)Bm * cfg_.d_ff * 2);
-    ws += (size_t)Bm * cfg_.d_ff * 2;
-  }
-  opart_ = fbuf((size_t)Bm * H * n_chunks_ * hd);
-  ml_ = fbuf((size_t)Bm * H * n_chunks_ * 2);
-  logits_ = fbuf((size_t)Bm * V);
+  ldl_ = lm_ ? lm_->logits_ld() : V;
+  logits_ = fbuf((size_t)Bm * ldl_);
   {
     // per-step decode parameters + grammar masks in ONE device block mirrored by a pinned host
     // block: a scheduler decode() uploads all of them with a single async copy (round 1 issued 8
@@ -564,17 +532,97 @@ void Engine::finalize() {
     HIP_CHECK(hipMemcpy(d_bt_, nul.data(), nul.size() * 4, hipMemcpyHostToDevice));
     HIP_CHECK(hipMemcpy(d_row_bt_, nul.data(), (size_t)Bm * kv_maxb_ * 4, hipMemcpyHostToDevice));
   }
-  attn_bt_ = d_row_bt_;
-  attn_bt_rows_ = 1;
-  d_step_ = ibuf(4);
-  d_step_kv_ = ibuf((size_t)Bm * 2);
-  d_step_rope_ = (float2*)fbuf((size_t)Bm * hd);
   d_fpos_ = ibuf(4);
   sample_ws_bytes_ = sample_ws_bytes(Bm, V);
   sample_ws_ = dmalloc(sample_ws_bytes_);
   ws += sample_ws_bytes_;
   sample_cnt_ = ibuf(Bm);
   d_history_ = ibuf((size_t)Bm * (cfg_.max_ctx + 1));
+  return ws;
+}
+
+// layered models: paging and step state as above, the rest is the decoder's
+void Engine::finalize_layered() {
+  cfg_.max_ctx = std::min(cfg_.max_ctx, cfg_.max_positions);
+  init_paging();
+  lm_->finalize();
+  ws_bytes_ += init_step_state();
+  HIP_CHECK(hipDeviceSynchronize());
+  finalized_ = true;
+}
+
+int Engine::ctx_limit() const { return cfg_.max_ctx; }
+
+void Engine::finalize() {
+  const CuScope cu_scope(cus_);  // (grids sized to this engine's CU mask)
+  TraceRange tr("aios.finalize");
+  HIP_CHECK(hipSetDevice(cfg_.device));
+  stage_release();  // weights are in place: drop the load-time staging buffers
+  auto miss = missing_tensors();
+  if (!miss.empty()) throw std::runtime_error("missing tensors, first: " + miss[0]);
+  if (lm_) return finalize_layered();
+  if (!output_.valid()) {
+    if (!cfg_.tie_embeddings) cfg_.tie_embeddings = 1;
+    cfg_.vocab_parallel = 0;  // the tied table is the full vocabulary
+    output_ = tok_embd_;  // tied embeddings (GGUF files without output.weight)
+  }
+  const int d = cfg_.d_model, hd = cfg_.head_dim, H = cfg_.n_heads, Hkv = cfg_.n_kv_heads;
+  const int qd = H * hd, kvd = Hkv * hd, V = cfg_.vocab_size, Bm = cfg_.max_batch;
+  kvb_ = KV_BLOCK;
+  if (cfg_.max_ctx % KV_BLOCK) cfg_.max_ctx = (int)align_up(cfg_.max_ctx, KV_BLOCK);  // whole KV blocks
+  init_paging();
+  layer_kv_elems_ = (size_t)(kv_nblocks_ + 1) * Hkv * KV_BLOCK * hd;
+  kv_es_ = cfg_.kv_fp8 ? 1 : 2;  // bytes per cached element (fp8 e4m3 or bf16)
+  kv_bytes_ = 2 * layer_kv_elems_ * cfg_.n_layers * kv_es_;
+  if (kv_scale_.size() != (size_t)2 * cfg_.n_layers) kv_scale_.assign((size_t)2 * cfg_.n_layers, 1.f);
+  k_cache_ = (bf16_t*)dmalloc(kv_bytes_ / 2);
+  v_cache_ = (bf16_t*)dmalloc(kv_bytes_ / 2);
+  HIP_CHECK(hipMemset(k_cache_, 0, kv_bytes_ / 2));
+  HIP_CHECK(hipMemset(v_cache_, 0, kv_bytes_ / 2));
+  for (int l = 0; l < cfg_.n_layers; ++l)  // one block: [n_kv_heads][KV_BLOCK][hd] contiguous
+    for (bf16_t* base : {k_cache_, v_cache_})
+      pools_.push_back({(char*)kv_layer(base, l), (size_t)Hkv * KV_BLOCK * hd * kv_es_});
+  n_chunks_ = (cfg_.max_ctx + ATTN_CHUNK - 1) / ATTN_CHUNK;
+  {
+    const size_t nc = (size_t)std::max(prefill_rows_, Bm) * H;  // decode attention tickets [row][head]
+    attn_cnt_ = (int*)dmalloc(nc * 4);
+    HIP_CHECK(hipMemset(attn_cnt_, 0, nc * 4));
+  }
+  {
+    const int half = hd / 2;
+    std::vector<float> tab((size_t)cfg_.max_ctx * half * 2);
+    for (int pos = 0; pos < cfg_.max_ctx; ++pos)
+      for (int p = 0; p < half; ++p) {
+        const double th = (double)pos * std::pow((double)cfg_.rope_theta, -2.0 * p / (double)hd);
+        tab[((size_t)pos * half + p) * 2] = (float)std::cos(th);
+        tab[((size_t)pos * half + p) * 2 + 1] = (float)std::sin(th);
+      }
+    rope_cs_ = (float2*)dmalloc(tab.size() * 4);
+    HIP_CHECK(hipMemcpy(rope_cs_, tab.data(), tab.size() * 4, hipMemcpyHostToDevice));
+  }
+
+  size_t ws = 0;
+  auto fbuf = [&](size_t n) { ws += n * 4; return (float*)dmalloc(n * 4); };
+  auto ibuf = [&](size_t n) { ws += n * 4; int* p = (int*)dmalloc(n * 4); HIP_CHECK(hipMemset(p, 0, n * 4)); return p; };
+  x_ = fbuf((size_t)Bm * d);
+  q_ = fbuf((size_t)Bm * qd);
+  qkv_ = fbuf((size_t)Bm * (qd + 2 * kvd));
+  attn_ = fbuf((size_t)Bm * std::max(qd, d));
+  ff_ = fbuf((size_t)Bm * std::max(cfg_.d_ff, d));
+  // (the BF16 engine stages its x as bf16 whatever act_q8 says: the hand-off serves it too)
+  if ((cfg_.act_q8 || layers_[0].wgu.w.qtype == QT_BF16) && cfg_.d_ff % 8 == 0 &&
+      !(std::getenv("AIOS_FF16") && std::atoi(std::getenv("AIOS_FF16")) == 0)) {
+    gv_ff16_ = (bf16_t*)dmalloc((size_t)Bm * cfg_.d_ff * 2);
+    ws += (size_t)Bm * cfg_.d_ff * 2;
+  }
+  opart_ = fbuf((size_t)Bm * H * n_chunks_ * hd);
+  ml_ = fbuf((size_t)Bm * H * n_chunks_ * 2);
+  ws += init_step_state();
+  attn_bt_ = d_row_bt_;
+  attn_bt_rows_ = 1;
+  d_step_ = ibuf(4);
+  d_step_kv_ = ibuf((size_t)Bm * 2);
+  d_step_rope_ = (float2*)fbuf((size_t)Bm * hd);
   const int R = prefill_rows_;
   pf_x_ = fbuf((size_t)R * d);
   pf_q_ = fbuf((size_t)R * qd);
@@ -1148,6 +1196,7 @@ void Engine::enqueue_decode_step(int B) {
 }
 
 void Engine::enqueue_decode_forward(int B) {
+  if (lm_) return lm_->decode_forward(B);
   const int d = cfg_.d_model;
   {
     StepPrep sp{d_pos_, d_slot_, d_bt_, kv_maxb_, rope_cs_, cfg_.head_dim / 2, d_step_kv_, d_step_rope_};
@@ -1166,7 +1215,7 @@ void Engine::enqueue_sample(int B) {
   const int V = cfg_.vocab_size;
   SampleArgs s;
   std::memset(&s, 0, sizeof(s));
-  s.logits = logits_; s.ldl = V; s.B = B; s.V = V;
+  s.logits = logits_; s.ldl = ldl_; s.B = B; s.V = V;
   s.temperature = d_temp_; s.top_k = d_topk_;
   s.seed = sample_seed_;
   s.seed_dev = d_seed_;
@@ -1303,6 +1352,11 @@ std::vector<float> Engine::prefill(int slot, const std::vector<int>& tokens, int
   if (slot < 0 || slot >= cfg_.max_slots) throw std::runtime_error("prefill: bad slot");
   for (int t : tokens)
     if (t < 0 || t >= cfg_.vocab_size) throw std::runtime_error("prefill: token id out of range");
+  if (lm_) {
+    std::vector<float> out;
+    run_step({slot}, {start_pos}, {T}, tokens, want_logits ? std::vector<int>{T - 1} : std::vector<int>{}, &out);
+    return out;
+  }
   kv_prepare_write(slot, start_pos, start_pos + T);
   kv_sync(0);
   if (gemm_prefill_ok(T)) {
@@ -1460,6 +1514,131 @@ std::vector<float> Engine::prefill(int slot, const std::vector<int>& tokens, int
   return out;
 }
 
+// Layered models: the step's entries cut into passes of at most step_rows() rows, in order (a later part of a
+// prompt reads the cache its earlier part wrote).  logits: host copy of the wanted rows; null: they are left
+// in logits rows 0.. (at most max_batch of them).
+void Engine::run_step(const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
+                      const std::vector<int>& tokens, const std::vector<int>& want, std::vector<float>* logits) {
+  const CuScope cu_scope(cus_);
+  TraceRange tr("aios.step");
+  if (!lm_) throw std::runtime_error("step: only layered models run mixed batches");
+  if (!finalized_) throw std::runtime_error("engine not finalized");
+  HIP_CHECK(hipSetDevice(cfg_.device));
+  const int E = (int)slots.size(), V = cfg_.vocab_size, Bm = cfg_.max_batch;
+  if ((int)starts.size() != E || (int)counts.size() != E) throw std::runtime_error("step: size mismatch");
+  size_t total = 0;
+  std::set<int> seen;
+  for (int e = 0; e < E; ++e) {
+    if (slots[e] < 0 || slots[e] >= cfg_.max_slots) throw std::runtime_error("step: bad slot");
+    if (!seen.insert(slots[e]).second) throw std::runtime_error("step: a slot appears twice");
+    if (counts[e] < 1 || starts[e] < 0 || starts[e] + counts[e] > ctx_limit())
+      throw std::runtime_error("step: context overflow");
+    total += counts[e];
+  }
+  if (total != tokens.size()) throw std::runtime_error("step: token count mismatch");
+  for (int t : tokens)
+    if (t < 0 || t >= V) throw std::runtime_error("step: token id out of range");
+  for (size_t i = 0; i < want.size(); ++i)
+    if (want[i] < (i ? want[i - 1] + 1 : 0) || want[i] >= (int)total) throw std::runtime_error("step: bad wanted index");
+  if (!logits && (int)want.size() > Bm) throw std::runtime_error("step: more sampled rows than max_batch");
+  for (int e = 0; e < E; ++e) kv_prepare_write(slots[e], starts[e], starts[e] + counts[e]);
+  kv_sync(0);
+  if (logits) logits->resize(want.size() * (size_t)V);
+  int e = 0, off = 0;       // next entry and tokens of it already run
+  size_t base = 0, w0 = 0;  // flat index of the pass's first token, wanted rows done
+  while (e < E) {
+    std::vector<LayeredDecoder::Piece> pieces;
+    int rows = 0;
+    while (e < E && rows < lm_->step_rows()) {
+      const int n = std::min(counts[e] - off, lm_->step_rows() - rows);
+      pieces.push_back({slots[e], starts[e] + off, n, tokens.data() + base + rows});
+      rows += n;
+      off += n;
+      if (off == counts[e]) {
+        ++e;
+        off = 0;
+      }
+    }
+    std::vector<int> first;
+    lm_->forward(pieces, first);
+    std::vector<int> xrows;
+    size_t p = 0, at = base;
+    for (size_t w = w0; w < want.size() && want[w] < (int)(base + rows); ++w) {
+      while (want[w] >= (int)(at + pieces[p].n)) at += pieces[p++].n;
+      xrows.push_back(first[p] + want[w] - (int)at);
+    }
+    lm_->collect(xrows, logits ? 0 : (int)w0);
+    if (logits)
+      for (int i = 0; i < (int)xrows.size(); i += Bm) {
+        const int n = std::min(Bm, (int)xrows.size() - i);
+        lm_->head(n, i);
+        HIP_CHECK(hipMemcpy2DAsync(logits->data() + (w0 + i) * (size_t)V, (size_t)V * 4, logits_, (size_t)ldl_ * 4,
+                                   (size_t)V * 4, n, hipMemcpyDeviceToHost, stream_));
+      }
+    HIP_CHECK(hipStreamSynchronize(stream_));  // (the pinned step block is written again by the next pass)
+    w0 += xrows.size();
+    base += rows;
+  }
+  if (!logits && !want.empty()) lm_->head((int)want.size());
+}
+
+std::vector<float> Engine::step(const std::vector<int>& slots, const std::vector<int>& starts,
+                                const std::vector<int>& counts, const std::vector<int>& tokens,
+                                const std::vector<int>& want) {
+  std::vector<float> out;
+  run_step(slots, starts, counts, tokens, want, &out);
+  return out;
+}
+
+std::vector<int> Engine::step_sample(const std::vector<int>& slots, const std::vector<int>& starts,
+                                     const std::vector<int>& counts, const std::vector<int>& tokens,
+                                     const std::vector<int>& sample, const std::vector<float>& temperature,
+                                     const std::vector<int>& top_k, const std::vector<float>& top_p,
+                                     const std::vector<uint64_t>& seeds, const std::vector<uint8_t>& mask) {
+  const CuScope cu_scope(cus_);
+  if (sample.size() != slots.size() || counts.size() != slots.size() || starts.size() != slots.size())
+    throw std::runtime_error("step_sample: size mismatch");
+  std::vector<int> want, pos;
+  int at = 0;
+  for (size_t e = 0; e < slots.size(); ++e) {
+    at += counts[e];
+    if (sample[e]) {
+      want.push_back(at - 1);
+      pos.push_back(starts[e] + counts[e] - 1);
+    }
+  }
+  const int B = (int)want.size();
+  if ((int)temperature.size() != B || (int)top_k.size() != B || (int)top_p.size() != B || (int)seeds.size() != B)
+    throw std::runtime_error("step_sample: sampling vectors are per sampled entry");
+  const size_t mbytes = (size_t)B * ((cfg_.vocab_size + 7) / 8);
+  if (!mask.empty() && mask.size() != mbytes) throw std::runtime_error("step_sample: mask size mismatch");
+  run_step(slots, starts, counts, tokens, want, nullptr);
+  if (B == 0) return {};
+  // rows 0.. of the parameter block: the next decode re-uploads every row it uses
+  HIP_CHECK(hipMemcpyAsync(d_temp_, temperature.data(), B * 4, hipMemcpyHostToDevice, stream_));
+  HIP_CHECK(hipMemcpyAsync(d_topk_, top_k.data(), B * 4, hipMemcpyHostToDevice, stream_));
+  HIP_CHECK(hipMemcpyAsync(d_topp_, top_p.data(), B * 4, hipMemcpyHostToDevice, stream_));
+  HIP_CHECK(hipMemcpyAsync(d_seeds_, seeds.data(), (size_t)B * 8, hipMemcpyHostToDevice, stream_));
+  HIP_CHECK(hipMemcpyAsync(d_pos_, pos.data(), B * 4, hipMemcpyHostToDevice, stream_));
+  if (!mask.empty()) HIP_CHECK(hipMemcpyAsync(d_mask_, mask.data(), mbytes, hipMemcpyHostToDevice, stream_));
+  SampleArgs s;
+  std::memset(&s, 0, sizeof(s));
+  s.logits = logits_; s.ldl = ldl_; s.B = B; s.V = cfg_.vocab_size;
+  s.temperature = d_temp_; s.top_k = d_topk_; s.seeds = d_seeds_;
+  s.tokens = d_tokens_; s.pos = d_pos_; s.advance = 0;
+  s.mask = mask.empty() ? nullptr : d_mask_;
+  s.top_p = d_topp_; s.ws = sample_ws_; s.ws_bytes = sample_ws_bytes_; s.counters = sample_cnt_;
+  launch_sample(s, stream_);
+  HIP_CHECK(hipMemcpyAsync(h_tok_out_, d_tokens_, B * 4, hipMemcpyDeviceToHost, stream_));
+  HIP_CHECK(hipStreamSynchronize(stream_));
+  return std::vector<int>(h_tok_out_, h_tok_out_ + B);
+}
+
+std::vector<float> Engine::last_residual(int rows) {
+  if (!lm_) throw std::runtime_error("last_residual: layered models only");
+  return lm_->residual(rows);
+}
+
 std::vector<int> Engine::decode(const std::vector<int>& slots, const std::vector<int>& tokens,
                                 const std::vector<int>& pos, const std::vector<float>& temperature,
                                 const std::vector<int>& top_k, uint64_t seed, const std::vector<uint8_t>& mask,
@@ -1536,7 +1715,7 @@ std::vector<int> Engine::resample(int B, const std::vector<float>& temperature, 
   }
   SampleArgs s;
   std::memset(&s, 0, sizeof(s));
-  s.logits = logits_; s.ldl = cfg_.vocab_size; s.B = B; s.V = cfg_.vocab_size;
+  s.logits = logits_; s.ldl = ldl_; s.B = B; s.V = cfg_.vocab_size;
   s.temperature = d_temp_; s.top_k = d_topk_; s.seed_dev = d_seed_; s.seeds = d_seeds_;
   s.tokens = d_tokens_; s.pos = d_pos_; s.advance = 0;
   s.mask = mask.empty() ? nullptr : d_mask_;
@@ -1571,7 +1750,7 @@ int Engine::sample_first(int pos, float temperature, int top_k, float top_p, uin
   if (!mask.empty()) HIP_CHECK(hipMemcpyAsync(d_mask_, mask.data(), mbytes, hipMemcpyHostToDevice, stream_));
   SampleArgs s;
   std::memset(&s, 0, sizeof(s));
-  s.logits = logits_; s.ldl = cfg_.vocab_size; s.B = 1; s.V = cfg_.vocab_size;
+  s.logits = logits_; s.ldl = ldl_; s.B = 1; s.V = cfg_.vocab_size;
   s.temperature = d_temp_; s.top_k = d_topk_; s.seeds = d_seeds_;
   s.tokens = d_tokens_; s.pos = d_fpos_; s.advance = 0;
   s.mask = mask.empty() ? nullptr : d_mask_;
@@ -1584,8 +1763,9 @@ int Engine::sample_first(int pos, float temperature, int top_k, float top_p, uin
 }
 
 std::vector<float> Engine::last_logits(int B) {
+  const size_t row = (size_t)cfg_.vocab_size * 4;
   std::vector<float> out((size_t)B * cfg_.vocab_size);
-  HIP_CHECK(hipMemcpyAsync(out.data(), logits_, out.size() * 4, hipMemcpyDeviceToHost, stream_));
+  HIP_CHECK(hipMemcpy2DAsync(out.data(), row, logits_, (size_t)ldl_ * 4, row, B, hipMemcpyDeviceToHost, stream_));
   HIP_CHECK(hipStreamSynchronize(stream_));
   return out;
 }
@@ -1809,7 +1989,7 @@ void Engine::reset_graphs() {
 
 // ---- paged KV ----------------------------------------------------------------------------------
 int Engine::kv_alloc() {
-  if (free_blocks_.empty()) throw std::runtime_error("paged KV: pool exhausted");  // cannot happen, see finalize
+  if (free_blocks_.empty()) throw std::runtime_error("paged KV: pool exhausted");  // (only with kv_pool_tokens, see init_paging)
   const int b = free_blocks_.back();
   free_blocks_.pop_back();
   refcnt_[b] = 1;
@@ -1821,21 +2001,18 @@ void Engine::kv_unref(int blk) {
   if (--refcnt_[blk] == 0) free_blocks_.push_back(blk);
 }
 
-// one block of every layer's K and V pool: [n_kv_heads][KV_BLOCK][hd] contiguous
+// one block of every cache pool
 void Engine::kv_copy_block(int src, int dst) {
-  const size_t blk = (size_t)cfg_.n_kv_heads * KV_BLOCK * cfg_.head_dim * kv_es_;  // bytes
-  for (int l = 0; l < cfg_.n_layers; ++l)
-    for (bf16_t* base : {k_cache_, v_cache_}) {
-      char* lb = (char*)kv_layer(base, l);
-      HIP_CHECK(hipMemcpyAsync(lb + (size_t)dst * blk, lb + (size_t)src * blk, blk, hipMemcpyDeviceToDevice, stream_));
-    }
+  for (const Pool& p : pools_)
+    HIP_CHECK(hipMemcpyAsync(p.base + (size_t)dst * p.block, p.base + (size_t)src * p.block, p.block,
+                             hipMemcpyDeviceToDevice, stream_));
 }
 
 void Engine::kv_prepare_write(int slot, int from, int to) {
   if (slot < 0 || slot >= cfg_.max_slots) throw std::runtime_error("paged KV: bad slot");
   if (to <= from) return;
   int* row = bt_.data() + (size_t)slot * kv_maxb_;
-  for (int j = from / KV_BLOCK; j <= (to - 1) / KV_BLOCK && j < kv_maxb_; ++j) {
+  for (int j = from / kvb_; j <= (to - 1) / kvb_ && j < kv_maxb_; ++j) {
     if (row[j] < 0) {
       row[j] = kv_alloc();
       bt_dirty_ = true;
@@ -1851,7 +2028,7 @@ void Engine::kv_prepare_write(int slot, int from, int to) {
 
 // Upload the slot table (when dirty) and the row table of decode rows 0..B-1 (when it changed).
 // Blocking uploads with the stream drained first: the captured decode graph reads the tables in
-// place, and a table changes only every KV_BLOCK tokens of a sequence or when rows change.
+// place, and a table changes only every block's tokens of a sequence or when rows change.
 void Engine::kv_sync(int B) {
   bool rows_changed = false;
   std::vector<int> rows((size_t)B * kv_maxb_);
@@ -1892,12 +2069,12 @@ void Engine::copy_slot(int src, int dst, int n) {
     kv_unref(d[j]);
     d[j] = -1;
   }
-  const int full = std::max(n, 0) / KV_BLOCK;
+  const int full = std::max(n, 0) / kvb_;
   for (int j = 0; j < full; ++j) {
     d[j] = s[j];
     if (d[j] >= 0) ++refcnt_[d[j]];
   }
-  if (n > 0 && n % KV_BLOCK && s[full] >= 0) {  // the partial block: private copy
+  if (n > 0 && n % kvb_ && s[full] >= 0) {  // the partial block: private copy
     d[full] = kv_alloc();
     kv_copy_block(s[full], d[full]);
   }

@@ -14,6 +14,8 @@ enum GemvEpilogue : int {
   EPI_QKV = 3,     // (+bias) RoPE on Q/K, Q -> y, K/V -> bf16 KV cache at pos[b]
   EPI_TP_RESID = 4,  // TP row-parallel O / down at batch 1: y[n] += sum over ranks of acc (the one-shot
                      //   all-reduce in the row-pair kernel's epilogue, GemvArgs::tp, gemv_q8.h)
+  EPI_STORE_GLU = 5,  // rows below glu_row0: y[b][n] = acc; above: interleaved gate/up pairs through the GLU
+                      //   to y16[b][(n - glu_row0) / 2] (row stride ldy16) -- the BF16 engine only
 };
 
 struct ArDevCtx;  // comm.h
@@ -44,6 +46,8 @@ struct GemvArgs {
   int ldy;
   bf16_t* y16;                  // EPI_SWIGLU: bf16 output [B][ldy] written instead of y (or null)
   int epi;
+  int act;                      // gate activation of the GLU epilogues (GluAct)
+  int glu_row0, ldy16;          // EPI_STORE_GLU
   // QKV epilogue
   const float* bias;            // [N] or null
   int head_dim, q_dim, kv_dim, n_kv_heads, max_ctx;

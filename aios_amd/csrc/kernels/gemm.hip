@@ -156,7 +156,9 @@ __global__ void __launch_bounds__(BM * BN / 64) gemm_big_kernel(GemmQArgs a) {
         if constexpr (EPI == GEPI_SWIGLU_BF16) {
           // interleaved gate/up columns: even lane = gate, odd lane = its up partner
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-          if (m < a.M && !(l32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+          if (m < a.M && !(l32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+        } else if constexpr (EPI == GEPI_STORE16) {
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
         } else if (m < a.M) {
           float* c = a.C + (size_t)m * a.ldc + n;
           if (S > 1) unsafeAtomicAdd(c, v);
@@ -192,7 +194,7 @@ static void launch_big_tiles(const GemmQArgs& a, hipStream_t st) {
     const int per_cu = std::max(1, 163840 / ((BM + BN) * 256));  // LDS-resident workgroups per CU
     S = tiles >= cus * per_cu / 2 ? 1 : std::max(1, std::min(a.K / 64 / 8, (cus * per_cu) / tiles));
   }
-  if (a.epi == GEPI_SWIGLU_BF16) S = 1;  // nonlinear epilogue needs the full sum
+  if (a.epi == GEPI_SWIGLU_BF16 || a.epi == GEPI_STORE16) S = 1;  // these epilogues need the full sum
   S = std::max(1, std::min(S, a.K / 64));
   if (S > 1 && a.epi == GEPI_STORE)
     HIP_CHECK(hipMemset2DAsync(a.C, (size_t)a.ldc * 4, 0, (size_t)a.N * 4, a.M, st));
@@ -203,6 +205,12 @@ static void launch_big_tiles(const GemmQArgs& a, hipStream_t st) {
     case GEPI_SWIGLU_BF16:
       hipLaunchKernelGGL((gemm_big_kernel<QT, BM, BN, GEPI_SWIGLU_BF16>), grid, dim3(NT), 0, st, a);
       break;
+    case GEPI_STORE16:
+      if constexpr (QT == QT_BF16) {
+        hipLaunchKernelGGL((gemm_big_kernel<QT, BM, BN, GEPI_STORE16>), grid, dim3(NT), 0, st, a);
+        break;
+      }
+      throw std::runtime_error("gemm: the bf16 store epilogue is for bf16 weights");
     default: throw std::runtime_error("gemm: bad epilogue");
   }
 }
@@ -241,8 +249,8 @@ static void launch_one(const GemmQArgs& a, hipStream_t st) {
   static const int skinny_max = env_int("AIOS_GEMM_SKINNY_MAX_M", 64);
   if (launch_gemm_ring(a, st)) return;
   if (a.M <= skinny_max && launch_gemm_skinny(a, st)) return;
-  if (a.epi == GEPI_QKV || a.epi == GEPI_ACCUM_NORM || a.nrm_in)
-    throw std::runtime_error("gemm: the QKV / fused-RMSNorm epilogues need the skinny (M <= 64) kernel");
+  if (a.epi == GEPI_QKV || a.epi == GEPI_ACCUM_NORM || a.epi == GEPI_STORE_GLU || a.nrm_in)
+    throw std::runtime_error("gemm: the QKV / fused-RMSNorm / store + GLU epilogues need the skinny (M <= 64) kernel");
   switch (a.seg[0].qtype) {
     case QT_Q4_K: launch_big<QT_Q4_K>(a, st); break;
     case QT_Q5_K: launch_big<QT_Q5_K>(a, st); break;

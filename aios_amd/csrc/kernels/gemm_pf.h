@@ -392,7 +392,9 @@ __device__ __forceinline__ void pf_body(const GemmQArgs& a, int m0, int n0, int 
         if constexpr (EPI == GEPI_SWIGLU_BF16) {
           // interleaved gate/up columns: even lane = gate, odd lane = its up partner
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-          if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+          if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+        } else if constexpr (EPI == GEPI_STORE16) {
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r16 & 1));
         } else if (m < a.M) {
@@ -590,7 +592,9 @@ __device__ __forceinline__ void pf_body32(const GemmQArgs& a, int m0, int n0, in
       const float v = acc[i][e];
       if constexpr (EPI == GEPI_SWIGLU_BF16) {
         const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-        if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+        if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+      } else if constexpr (EPI == GEPI_STORE16) {
+        if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
       } else if (m < a.M) {
         float* cp = a.C + (size_t)m * a.ldc + n;
         if (S > 1) unsafeAtomicAdd(cp, v);
@@ -899,7 +903,9 @@ __device__ __forceinline__ void pf4_body(const GemmQArgs& a, int m0, int n0, int
         const float v = acc[i][c][e];
         if constexpr (EPI == GEPI_SWIGLU_BF16) {
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-          if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+          if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+        } else if constexpr (EPI == GEPI_STORE16) {
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r32 & 1));
         } else if (m < a.M) {
@@ -1075,7 +1081,9 @@ __device__ __forceinline__ void pf8_body(const GemmQArgs& a, int m0, int n0, int
         const float v = acc[i][c][e];
         if constexpr (EPI == GEPI_SWIGLU_BF16) {
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-          if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+          if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+        } else if constexpr (EPI == GEPI_STORE16) {
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r16 & 1));
         } else if (m < a.M) {
@@ -1362,7 +1370,9 @@ __device__ __forceinline__ void pf8c_body(const GemmQArgs& a, int m0, int n0, in
         const float v = acc[i][c][e];
         if constexpr (EPI == GEPI_SWIGLU_BF16) {
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-          if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+          if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+        } else if constexpr (EPI == GEPI_STORE16) {
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r16 & 1));
         } else if (m < a.M) {
@@ -1555,7 +1565,9 @@ __device__ __forceinline__ void pf8d_body(const GemmQArgs& a, int m0, int n0, in
       const float v = acc[i][e];
       if constexpr (EPI == GEPI_SWIGLU_BF16) {
         const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
-        if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(v / (1.f + __expf(-v)) * up);
+        if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
+      } else if constexpr (EPI == GEPI_STORE16) {
+        if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
       } else if (m < a.M) {
         float* cp = a.C + (size_t)m * a.ldc + n;
         if (S > 1) unsafeAtomicAdd(cp, v);
@@ -1660,7 +1672,7 @@ __global__ void __launch_bounds__(512) gemm_pf8t_kernel(GemmQArgs a, int F) {
 // full tiles before the tail of a 256 x BN launch, or -1 (no tail split for this shape / plan)
 inline int pf_tail_full(const GemmQArgs& a, int BN, int S) {
   const char* e = std::getenv("AIOS_GEMM_PF_TAIL");  // (read per call: tests compare both)
-  if ((e && std::atoi(e) == 0) || S != 1 || a.epi == GEPI_QKV) return -1;
+  if ((e && std::atoi(e) == 0) || S != 1 || a.epi == GEPI_QKV || a.epi == GEPI_STORE16) return -1;
   const int T = (a.N / BN) * ((a.M + 255) / 256), C = device_cu_count(), R = T % C;
   return (T > C && R > 0 && 2 * R <= C) ? T - R : -1;
 }
@@ -1788,6 +1800,9 @@ void pf8_launch(const GemmQArgs& a, int S, hipStream_t st) {
     case GEPI_STORE: hipLaunchKernelGGL((gemm_pf8_kernel<QT0, QT1, BM, GEPI_STORE>), grid, block, lds, st, a); break;
     case GEPI_ACCUM: hipLaunchKernelGGL((gemm_pf8_kernel<QT0, QT1, BM, GEPI_ACCUM>), grid, block, lds, st, a); break;
     case GEPI_QKV: hipLaunchKernelGGL((gemm_pf8_kernel<QT0, QT1, BM, GEPI_QKV>), grid, block, lds, st, a); break;
+    case GEPI_STORE16:
+      if constexpr (QT0 == QT_BF16) hipLaunchKernelGGL((gemm_pf8_kernel<QT0, QT1, BM, GEPI_STORE16>), grid, block, lds, st, a);
+      break;
     default: hipLaunchKernelGGL((gemm_pf8_kernel<QT0, QT1, BM, GEPI_SWIGLU_BF16>), grid, block, lds, st, a); break;
   }
 }
@@ -1883,6 +1898,9 @@ void pf4_launch(const GemmQArgs& a, int S, hipStream_t st) {
     case GEPI_STORE: hipLaunchKernelGGL((gemm_pf4_kernel<QT0, QT1, BM, WC, GEPI_STORE>), grid, block, lds, st, a); break;
     case GEPI_ACCUM: hipLaunchKernelGGL((gemm_pf4_kernel<QT0, QT1, BM, WC, GEPI_ACCUM>), grid, block, lds, st, a); break;
     case GEPI_QKV: hipLaunchKernelGGL((gemm_pf4_kernel<QT0, QT1, BM, WC, GEPI_QKV>), grid, block, lds, st, a); break;
+    case GEPI_STORE16:
+      if constexpr (QT0 == QT_BF16) hipLaunchKernelGGL((gemm_pf4_kernel<QT0, QT1, BM, WC, GEPI_STORE16>), grid, block, lds, st, a);
+      break;
     default: hipLaunchKernelGGL((gemm_pf4_kernel<QT0, QT1, BM, WC, GEPI_SWIGLU_BF16>), grid, block, lds, st, a); break;
   }
 }

@@ -96,7 +96,7 @@ static std::map<PfKey, PfPlan>& pf_tuned_s1() {
 // arrival order, so the low bits of a prefill could differ run to run even with the same plan)
 static bool pf_deterministic() { return pf_env("AIOS_GEMM_PF_DETERMINISTIC", 0) != 0; }
 static bool pf_no_split(const GemmQArgs& a) {
-  return a.epi == GEPI_SWIGLU_BF16 || a.epi == GEPI_QKV || pf_deterministic();
+  return a.epi == GEPI_SWIGLU_BF16 || a.epi == GEPI_QKV || a.epi == GEPI_STORE16 || pf_deterministic();
 }
 // stream-K: STORE / ACCUM launches whose tiles leave CUs idle, with an even K-step count per tile
 // (every stream-K segment then spans >= 2 steps / 256-blocks); AIOS_GEMM_PF_SK=0 keeps it out of plans
@@ -208,7 +208,10 @@ bool launch_gemm_pf(const GemmQArgs& a, hipStream_t st) {
 
 static bool pf_eligible(const GemmQArgs& a) {
   if (a.nseg < 1 || a.M < 1) return false;
-  if (a.epi != GEPI_STORE && a.epi != GEPI_ACCUM && a.epi != GEPI_SWIGLU_BF16 && a.epi != GEPI_QKV) return false;
+  if (a.epi != GEPI_STORE && a.epi != GEPI_ACCUM && a.epi != GEPI_SWIGLU_BF16 && a.epi != GEPI_QKV &&
+      a.epi != GEPI_STORE16)
+    return false;
+  if (a.epi == GEPI_STORE16 && (!a.C16 || a.seg[0].qtype != QT_BF16)) return false;
   if (a.epi == GEPI_QKV && (a.kv_fp8 || a.col0 != 0 || !a.q_out || !a.k_cache || !a.v_cache || !a.pos || !a.rope_cs ||
                             a.head_dim % 2 || a.N != a.q_dim + 2 * a.kv_dim))
     return false;
@@ -225,7 +228,7 @@ static bool pf_eligible(const GemmQArgs& a) {
                   (qt0 == QT_Q8_0 && qt1 == QT_Q8_0);
   if (!bf && !kq) return false;
   if (a.epi == GEPI_SWIGLU_BF16 && (!a.C16 || a.nseg != 1)) return false;
-  if (a.epi != GEPI_SWIGLU_BF16 && a.epi != GEPI_QKV && !a.C) return false;
+  if (a.epi != GEPI_SWIGLU_BF16 && a.epi != GEPI_QKV && a.epi != GEPI_STORE16 && !a.C) return false;
   return true;
 }
 

@@ -354,6 +354,7 @@ static bool rg_launch(const GemmQArgs& a, hipStream_t st) {
 bool launch_gemm_ring(const GemmQArgs& a, hipStream_t st) {
   static const int on = rg_env("AIOS_GEMM_RING", 1);
   static const int min_m = rg_env("AIOS_GEMM_RING_MIN_M", 2);
+  if (a.epi == GEPI_STORE16 || a.epi == GEPI_STORE_GLU) return false;
   if (!on || a.M < min_m || a.M > 32 || a.N % 128 || a.K % 256 || a.lda % 8) return false;
   if (a.nrm_in && (a.nrm_parts <= 0 || a.nrm_parts > 64 || a.nrm_parts % 4)) return false;
   if (a.epi == GEPI_SWIGLU_BF16 && a.ldc % 2) return false;

@@ -290,6 +290,12 @@ static void sk_launch(const GemmQArgs& a, int S, hipStream_t st) {
       case GEPI_QKV: SK_GO(GEPI_QKV); break;
       case GEPI_ACCUM: SK_GO(GEPI_ACCUM); break;
       case GEPI_ACCUM_NORM: SK_GO(GEPI_ACCUM_NORM); break;
+      case GEPI_STORE16:
+        if constexpr (QT0 == QT_BF16) SK_GO(GEPI_STORE16);
+        break;
+      case GEPI_STORE_GLU:
+        if constexpr (QT0 == QT_BF16) SK_GO(GEPI_STORE_GLU);
+        break;
       default: SK_GO(GEPI_SWIGLU_BF16); break;
     }
   }
@@ -315,6 +321,8 @@ static int sk_rb(const GemmQArgs& a) {
 static bool sk_fits(const GemmQArgs& a) {
   if (a.M > 64 || a.N % 64) return false;
   if (a.epi == GEPI_SWIGLU_BF16 && a.ldc % 2) return false;
+  if ((a.epi == GEPI_STORE16 || a.epi == GEPI_STORE_GLU) && a.seg[0].qtype != QT_BF16) return false;
+  if (a.epi == GEPI_STORE_GLU && (a.glu_n0 % 4 || a.ldc16 % 2)) return false;
   if ((a.epi != GEPI_SWIGLU_BF16 && a.ldc % 4) || a.lda % 8) return false;
   if (a.nrm_in && (a.nrm_parts % 4 || a.nrm_parts > 64)) return false;
   if (a.epi == GEPI_ACCUM_NORM && (!a.nrm_g || !a.nrm_out16 || !a.nrm_part || a.N / (16 * sk_rb(a)) != a.nrm_parts))

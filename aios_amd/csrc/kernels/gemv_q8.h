@@ -478,9 +478,13 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
       if (grow + 1 < nrow) unsafeAtomicAdd(a.y + grow + 1, v1);
       break;
     case EPI_SWIGLU: {
-      const float h = v0 / (1.f + __expf(-v0)) * v1;
+      const float h = glu_act(v0, a.act) * v1;
       if (a.y16) a.y16[grow >> 1] = f32_to_bf16(h);
       else a.y[grow >> 1] = h;
+    } break;
+    case EPI_STORE_GLU: {
+      if (grow < a.glu_row0) *(float2*)(a.y + grow) = make_float2(v0, v1);
+      else a.y16[(grow - a.glu_row0) >> 1] = f32_to_bf16(glu_act(v0, a.act) * v1);
     } break;
     case EPI_QKV: {
       if (a.bias) {

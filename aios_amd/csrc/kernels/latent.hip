@@ -1,0 +1,594 @@
+// Latent attention, absorbed form (latent.h), and the small launches of the layered decoders.
+//
+// A decode layer is three launches between the projection GEMVs:
+//   latent_prep   one wave per row normalises the latent and writes it into the paged cache; further
+//                 workgroups fold the queries into the latent space (q_a = Wuk_h^T q_h, MFMA with up to
+//                 16 tokens as rows);
+//   latent_attn   all heads share the cached vectors, so 16 (token, head) rows form one MFMA tile: the
+//                 64-key tile of c staged in LDS serves as keys (read row-major) and, through the
+//                 transposed LDS reads, as values.  Keys are split over workgroups;
+//   latent_out    sums the splits, normalises (the sink joins the denominator here), multiplies by
+//                 Wuv_h and by the output gate.
+// Scores, softmax weights, their sum and the latent norm are fp32.  The weights enter the value product
+// as two bf16 terms (p = hi + lo, 16 significant bits), so that product adds no rounding of its own.
+#include <algorithm>
+#include <cmath>
+
+#include "../latent.h"
+#include "gemm_common.h"
+
+namespace aios {
+
+typedef short lv4i16 __attribute__((ext_vector_type(4)));
+typedef short lv8i16 __attribute__((ext_vector_type(8)));
+typedef unsigned int lu32x4 __attribute__((ext_vector_type(4)));
+
+constexpr float LOG2E = 1.4426950408889634f;
+
+__device__ __forceinline__ float lat_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+
+// ---- prep: latent norm + cache write, query absorption --------------------------------------------
+template <bool F32>
+__device__ __forceinline__ void latent_cache_row(const LatentAttnArgs& a, int row) {
+  const int lane = threadIdx.x & 63;
+  const float* x = a.qdg + (size_t)row * a.ld + a.dkv_off;
+  float s = 0.f;
+  for (int i = lane; i < a.rank; i += 64) s = fmaf(x[i], x[i], s);
+  s = wave_sum(s);
+  const float inv = 1.f / sqrtf(s / (float)a.rank + a.eps);
+  const int pos = a.pos[row], blk = a.bt[(size_t)a.slot[row] * a.maxb + pos / a.kvb];
+  const size_t base = ((size_t)blk * a.kvb + pos % a.kvb) * a.rp;
+  for (int i = lane; i < a.rp; i += 64) {
+    const float c = i < a.rank ? x[i] * inv * a.norm_w[i] : 0.f;
+    if constexpr (F32) ((float*)a.pool)[base + i] = c;
+    else ((bf16_t*)a.pool)[base + i] = f32_to_bf16(c);
+  }
+}
+
+// 8 consecutive floats -> one bf16x8 fragment
+__device__ __forceinline__ gbf16x8 frag_f32(const float* p) {
+  const float4 x0 = *(const float4*)p, x1 = *(const float4*)(p + 4);
+  const uint4 u = make_uint4(pk_bf16(x0.x, x0.y), pk_bf16(x0.z, x0.w), pk_bf16(x1.x, x1.y), pk_bf16(x1.z, x1.w));
+  return __builtin_bit_cast(gbf16x8, u);
+}
+
+// grid: ceil(rows / 4) cache workgroups, then row tiles x heads x (rp / 64) absorb workgroups (4 waves of
+// 16 latent columns each)
+__global__ void __launch_bounds__(256) latent_prep_kernel(LatentAttnArgs a, int rows, int ncache) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  if ((int)blockIdx.x < ncache) {
+    const int row = blockIdx.x * 4 + wave;
+    if (row < rows) latent_cache_row<false>(a, row);
+    return;
+  }
+  int b = blockIdx.x - ncache;
+  const int nr = a.rp >> 6;
+  const int rt = b % nr;
+  b /= nr;
+  const int h = b % a.H, mt = b / a.H;
+  const int r16 = lane & 15, q = lane >> 4;
+  const int m = min(mt * 16 + r16, a.n - 1);  // (clamped rows are computed and not stored)
+  const int r = rt * 64 + wave * 16 + r16;
+  const float* qp = a.qdg + (size_t)m * a.ld + h * a.dkp + 8 * q;
+  const bf16_t* wp = a.wukT + ((size_t)h * a.rp + r) * a.dkp + 8 * q;
+  gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < a.dkp; k += 32) {
+    const gbf16x8 af = frag_f32(qp + k);
+    const gbf16x8 bf = __builtin_bit_cast(gbf16x8, *(const lu32x4*)(wp + k));
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af, bf, acc, 0, 0, 0);
+  }
+  bf16_t* out = (bf16_t*)a.qa;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int t = mt * 16 + 4 * q + j;
+    if (t < a.n) out[((size_t)t * a.H + h) * a.rp + r] = f32_to_bf16(acc[j]);
+  }
+}
+
+// fp32: the same two roles; absorption as one wave per (token, head), lanes over the latent columns
+__global__ void __launch_bounds__(256) latent_prep_f32_kernel(LatentAttnArgs a, int rows, int ncache) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  if ((int)blockIdx.x < ncache) {
+    const int row = blockIdx.x * 4 + wave;
+    if (row < rows) latent_cache_row<true>(a, row);
+    return;
+  }
+  const int f = (blockIdx.x - ncache) * 4 + wave;
+  if (f >= a.n * a.H) return;
+  const int t = f / a.H, h = f - t * a.H;
+  const float* qp = a.qdg + (size_t)t * a.ld + h * a.dkp;
+  for (int r = lane; r < a.rp; r += 64) {
+    const bf16_t* wp = a.wukT + ((size_t)h * a.rp + r) * a.dkp;
+    float s = 0.f;
+    for (int d = 0; d < a.dkp; ++d) s = fmaf(qp[d], bf16_to_f32(wp[d]), s);
+    ((float*)a.qa)[(size_t)f * a.rp + r] = s;
+  }
+}
+
+void launch_latent_prep(const LatentAttnArgs& a, int rows, hipStream_t st) {
+  const int ncache = (rows + 3) / 4;
+  if (a.f32) {
+    hipLaunchKernelGGL(latent_prep_f32_kernel, dim3(ncache + (a.n * a.H + 3) / 4), dim3(256), 0, st, a, rows, ncache);
+  } else {
+    const int nab = (a.n + 15) / 16 * a.H * (a.rp / 64);
+    hipLaunchKernelGGL(latent_prep_kernel, dim3(ncache + nab), dim3(256), 0, st, a, rows, ncache);
+  }
+}
+
+// ---- attention ---------------------------------------------------------------------------------
+int latent_tiles_per_token(int H) { return (H + 15) / 16; }
+
+__device__ __forceinline__ LatentTile latent_tile(const LatentAttnArgs& a, int t) {
+  if (a.tiles) return a.tiles[t];
+  const int tpt = (a.H + 15) >> 4, row = t / tpt, i = t - row * tpt;
+  return LatentTile{row * a.H + 16 * i, min(16, a.H - 16 * i)};
+}
+
+constexpr int LT_KT = 64;  // keys per tile; a cache block is a whole number of tiles
+
+// NT: 16-column tiles of the latent per wave (rp = 64 NT)
+template <int NT>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NT <= 8 ? 2 : 1))) latent_attn_kernel(LatentAttnArgs a) {
+  constexpr int RP = 64 * NT, KS = 2 * NT;
+  constexpr int LDR = RP + 16;          // padded LDS row of the tile (bf16)
+  constexpr int SROW = LT_KT + 4;       // padded LDS row of the scores (fp32)
+  constexpr int PPK = RP / 8, PPT = LT_KT * PPK / 256;
+  extern __shared__ __attribute__((aligned(16))) uint8_t lat_smem[];
+  bf16_t* sC = (bf16_t*)lat_smem;
+  float* sS = (float*)(lat_smem + (size_t)LT_KT * LDR * 2);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int r16 = lane & 15, q = lane >> 4;
+  const LatentTile tl = latent_tile(a, blockIdx.x);
+  const int split = blockIdx.y;
+  const int nf = a.n * a.H;
+  const int f = tl.f0 + min(r16, tl.nv - 1);
+  const int tok = f / a.H;
+  const int mypos = a.pos[tok];
+  const int slot = a.slot[tok];
+  const int len = a.pos[(tl.f0 + tl.nv - 1) / a.H] + 1;
+  const int nkt = (len + LT_KT - 1) / LT_KT, per = (nkt + a.nsplit - 1) / a.nsplit;
+  const int kt0 = split * per, kt1 = min(kt0 + per, nkt);
+  float* mlp = a.ml + ((size_t)split * nf + tl.f0) * 2;
+  if (kt0 >= kt1) {  // (whole workgroup, before any barrier)
+    if (tid < tl.nv) *(float2*)(mlp + 2 * tid) = make_float2(-INFINITY, 0.f);
+    return;
+  }
+  const int* bt = a.bt + (size_t)slot * a.maxb;
+  gbf16x8 qf[KS];
+  {
+    const bf16_t* qp = (const bf16_t*)a.qa + (size_t)f * RP + 8 * q;
+#pragma unroll
+    for (int s = 0; s < KS; ++s) qf[s] = __builtin_bit_cast(gbf16x8, *(const lu32x4*)(qp + 32 * s));
+  }
+  lu32x4 rg[PPT];
+  auto load = [&](int kt) {
+    const int k0 = kt * LT_KT;
+    const bf16_t* base = (const bf16_t*)a.pool + ((size_t)bt[k0 / a.kvb] * a.kvb + k0 % a.kvb) * RP;
+    const int last = len - 1 - k0;  // (keys past the end re-read the last one: finite, weight 0)
+    static_for<PPT>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      const int idx = tid + 256 * i, key = min(idx / PPK, last), c = idx % PPK;
+      rg[i] = *(const lu32x4*)(base + (size_t)key * RP + c * 8);
+    });
+  };
+  gf32x4 o[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) o[t] = gf32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run = -INFINITY, l_run = 0.f;
+  const float sc = a.scale * LOG2E;
+  load(kt0);
+  for (int kt = kt0; kt < kt1; ++kt) {
+    static_for<PPT>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      const int idx = tid + 256 * i, key = idx / PPK, c = idx % PPK;
+      *(lu32x4*)(sC + key * LDR + c * 8) = rg[i];
+    });
+    __syncthreads();
+    if (kt + 1 < kt1) load(kt + 1);
+    // ---- scores of this wave's 16 keys
+    {
+      gf32x4 s4 = {0.f, 0.f, 0.f, 0.f};
+      const bf16_t* kr = sC + (wave * 16 + r16) * LDR + 8 * q;
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        const gbf16x8 kf = __builtin_bit_cast(gbf16x8, *(const lu32x4*)(kr + 32 * s));
+        s4 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[s], kf, s4, 0, 0, 0);
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) sS[(4 * q + j) * SROW + wave * 16 + r16] = s4[j];
+    }
+    __syncthreads();
+    // ---- every wave: online softmax of row r16, keys 32 ks + 8 q + i -- the value product's A layout
+    float p[16];
+    float mx = -INFINITY;
+    const int key0 = kt * LT_KT + 8 * q;
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      const float4 x0 = *(const float4*)(sS + r16 * SROW + 32 * ks + 8 * q);
+      const float4 x1 = *(const float4*)(sS + r16 * SROW + 32 * ks + 8 * q + 4);
+      const float v[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        p[8 * ks + i] = key0 + 32 * ks + i <= mypos ? v[i] * sc : -INFINITY;
+        mx = fmaxf(mx, p[8 * ks + i]);
+      }
+    }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m_run, mx);
+    const float ms = mn == -INFINITY ? 0.f : mn;  // (a row with no visible key yet: weights exp2(-inf) = 0)
+    const float alpha = lat_exp2(m_run - ms);
+    float ps = 0.f;
+    gbf16x8 ph[2], pl[2];
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float e = lat_exp2(p[8 * ks + i] - ms);
+        ps += e;
+        const __bf16 hi = (__bf16)e;
+        ph[ks][i] = hi;
+        pl[ks][i] = (__bf16)(e - (float)hi);
+      }
+    ps += __shfl_xor(ps, 16, 64);
+    ps += __shfl_xor(ps, 32, 64);
+    l_run = l_run * alpha + ps;
+    if (__any(mn != m_run)) {
+      float al[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) al[j] = __shfl(alpha, 4 * q + j, 64);
+#pragma unroll
+      for (int t = 0; t < NT; ++t)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[t][j] *= al[j];
+    }
+    m_run = mn;
+    // ---- values: this wave's NT column tiles
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      // lane 4 i + p of a 16-lane group addresses key 32 ks + 8 q + i (then + 4), columns 4 p .. + 3, and
+      // receives column r16 of the four keys
+      const bf16_t* vb = sC + (32 * ks + 8 * q + (r16 >> 2)) * LDR + wave * 16 * NT + 4 * (r16 & 3);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        const lv4i16 x0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) lv4i16*)(vb + 16 * t));
+        const lv4i16 x1 =
+            __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) lv4i16*)(vb + 16 * t + 4 * LDR));
+        const gbf16x8 vf = __builtin_bit_cast(gbf16x8, __builtin_shufflevector(x0, x1, 0, 1, 2, 3, 4, 5, 6, 7));
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ph[ks], vf, o[t], 0, 0, 0);
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pl[ks], vf, o[t], 0, 0, 0);
+      }
+    }
+    __syncthreads();  // tile and scores are free
+  }
+  float* op = a.opart + ((size_t)split * nf + tl.f0) * RP + wave * 16 * NT + r16;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int m = 4 * q + j;
+    if (m < tl.nv)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) op[(size_t)m * RP + 16 * t] = o[t][j];
+  }
+  if (tid < tl.nv) *(float2*)(mlp + 2 * tid) = make_float2(m_run, l_run);
+}
+
+// plain form (fp32 cache, or a rank beyond the matrix-core kernels): one workgroup per (token, head), keys
+// round-robin over the waves, the latent columns over the lanes (NR = rp / 64 each)
+template <int NR, bool F32>
+__global__ void __launch_bounds__(256) latent_attn_plain_kernel(LatentAttnArgs a) {
+  constexpr int RP = 64 * NR;
+  __shared__ float sm[4], sl[4];
+  extern __shared__ __attribute__((aligned(16))) float so[];  // [4][RP]
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int f = blockIdx.x, tok = f / a.H;
+  const int len = a.pos[tok] + 1, nf = a.n * a.H;
+  const int* bt = a.bt + (size_t)a.slot[tok] * a.maxb;
+  float qv[NR], o[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const size_t qi = (size_t)f * RP + 64 * i + lane;
+    qv[i] = F32 ? ((const float*)a.qa)[qi] : bf16_to_f32(((const bf16_t*)a.qa)[qi]);
+    o[i] = 0.f;
+  }
+  float m = -INFINITY, l = 0.f;
+  const float sc = a.scale * LOG2E;
+  for (int key = wave; key < len; key += 4) {
+    const size_t base = ((size_t)bt[key / a.kvb] * a.kvb + key % a.kvb) * RP + lane;
+    float c[NR], s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      c[i] = F32 ? ((const float*)a.pool)[base + 64 * i] : bf16_to_f32(((const bf16_t*)a.pool)[base + 64 * i]);
+      s = fmaf(c[i], qv[i], s);
+    }
+    s = wave_sum(s) * sc;
+    const float mn = fmaxf(m, s), alpha = exp2f(m - mn), p = exp2f(s - mn);
+    l = l * alpha + p;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) o[i] = fmaf(p, c[i], o[i] * alpha);
+    m = mn;
+  }
+  if (lane == 0) {
+    sm[wave] = m;
+    sl[wave] = l;
+  }
+#pragma unroll
+  for (int i = 0; i < NR; ++i) so[wave * RP + 64 * i + lane] = o[i];
+  __syncthreads();
+  const float M = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));  // (key 0 is visible: finite)
+  float w[4], L = 0.f;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    w[k] = exp2f(sm[k] - M);
+    L += w[k] * sl[k];
+  }
+  for (int i = threadIdx.x; i < RP; i += 256)
+    a.opart[(size_t)f * RP + i] = (so[i] * w[0] + so[RP + i] * w[1]) + (so[2 * RP + i] * w[2] + so[3 * RP + i] * w[3]);
+  if (threadIdx.x == 0) *(float2*)(a.ml + 2 * (size_t)f) = make_float2(M, L);
+  (void)nf;
+}
+
+bool latent_attn_mfma(int rp) { return rp <= 1024; }
+
+template <int NT>
+static void latent_attn_go(const LatentAttnArgs& a, hipStream_t st) {
+  const size_t lds = (size_t)LT_KT * (64 * NT + 16) * 2 + 16 * (LT_KT + 4) * 4;
+  hipLaunchKernelGGL((latent_attn_kernel<NT>), dim3(a.n_tiles, a.nsplit), dim3(256), lds, st, a);
+}
+template <int NR, bool F32>
+static void latent_plain_go(const LatentAttnArgs& a, hipStream_t st) {
+  hipLaunchKernelGGL((latent_attn_plain_kernel<NR, F32>), dim3(a.n * a.H), dim3(256), (size_t)4 * 64 * NR * 4, st, a);
+}
+template <bool F32>
+static void latent_plain(const LatentAttnArgs& a, hipStream_t st) {
+  if (a.nsplit != 1) throw std::runtime_error("latent attention: the plain kernel does not split keys");
+  switch (a.rp / 64) {
+    case 1: return latent_plain_go<1, F32>(a, st);
+    case 2: return latent_plain_go<2, F32>(a, st);
+    case 3: return latent_plain_go<3, F32>(a, st);
+    case 4: return latent_plain_go<4, F32>(a, st);
+    case 6: return latent_plain_go<6, F32>(a, st);
+    case 8: return latent_plain_go<8, F32>(a, st);
+    case 12: return latent_plain_go<12, F32>(a, st);
+    case 16: return latent_plain_go<16, F32>(a, st);
+    case 32: return latent_plain_go<32, F32>(a, st);
+  }
+  throw std::runtime_error("latent attention: unsupported padded rank " + std::to_string(a.rp));
+}
+
+void launch_latent_attn(const LatentAttnArgs& a, hipStream_t st) {
+  if (a.n < 1) return;
+  if (a.kvb % LT_KT) throw std::runtime_error("latent attention: cache block must be a multiple of 64 tokens");
+  if (a.f32) return latent_plain<true>(a, st);
+  switch (a.rp / 64) {
+    case 1: return latent_attn_go<1>(a, st);
+    case 2: return latent_attn_go<2>(a, st);
+    case 3: return latent_attn_go<3>(a, st);
+    case 4: return latent_attn_go<4>(a, st);
+    case 6: return latent_attn_go<6>(a, st);
+    case 8: return latent_attn_go<8>(a, st);
+    case 12: return latent_attn_go<12>(a, st);
+    case 16: return latent_attn_go<16>(a, st);
+  }
+  latent_plain<false>(a, st);
+}
+
+// ---- combine + Wuv + gate ------------------------------------------------------------------------
+constexpr int LO_SMAX = 64;  // key splits at most
+
+// softmax coefficients of (token t, head h): coef[s] = exp2(m_s - M) / (sum + sink) into c (lane s)
+__device__ __forceinline__ float latent_coef(const LatentAttnArgs& a, int t, int h, int lane) {
+  const size_t nf = (size_t)a.n * a.H, f = (size_t)t * a.H + h;
+  float m = -INFINITY, l = 0.f;
+  if (lane < a.nsplit) {
+    const float2 v = *(const float2*)(a.ml + (lane * nf + f) * 2);
+    m = v.x;
+    l = v.y;
+  }
+  float M = wave_max(m);
+  const float sk = a.sink ? a.sink[h] * LOG2E : -INFINITY;
+  M = fmaxf(M, sk);
+  const float e = exp2f(m - M);
+  const float den = wave_sum(l * e) + exp2f(sk - M);
+  return l > 0.f ? e / den : 0.f;
+}
+
+// KW: waves that share a 16-column tile's K (4: 16 output columns per workgroup, for few rows; 1: 64)
+template <int KW>
+__global__ void __launch_bounds__(256) latent_out_kernel(LatentAttnArgs a) {
+  extern __shared__ __attribute__((aligned(16))) uint8_t lo_smem[];
+  const int xrow = a.rp + 8;
+  bf16_t* sX = (bf16_t*)lo_smem;                         // [16][rp + 8]
+  float* sw = (float*)(lo_smem + (size_t)16 * xrow * 2); // [16][nsplit]
+  float* sred = sw + 16 * LO_SMAX;                       // [4][16][16] (KW == 4)
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int r16 = lane & 15, q = lane >> 4;
+  const int h = blockIdx.y, t0 = blockIdx.z * 16;
+  const int nt = min(16, a.n - t0);
+  const int col = KW == 4 ? blockIdx.x * 16 + r16 : blockIdx.x * 64 + wave * 16 + r16;
+  const bool cok = col < a.dvp;
+  for (int m = wave; m < nt; m += 4) {
+    const float c = latent_coef(a, t0 + m, h, lane);
+    if (lane < a.nsplit) sw[m * LO_SMAX + lane] = c;
+  }
+  __syncthreads();
+  const size_t nf = (size_t)a.n * a.H;
+  const int q4 = a.rp >> 2;
+  for (int idx = tid; idx < 16 * q4; idx += 256) {
+    const int m = idx / q4, c4 = 4 * (idx - m * q4);
+    float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (m < nt) {
+      const float* p = a.opart + ((size_t)(t0 + m) * a.H + h) * a.rp + c4;
+      for (int k = 0; k < a.nsplit; ++k) {
+        const float w = sw[m * LO_SMAX + k];
+        if (w != 0.f) {  // (splits without a key of this row were not written)
+          const float4 v = *(const float4*)(p + (size_t)k * nf * a.rp);
+          s.x = fmaf(w, v.x, s.x); s.y = fmaf(w, v.y, s.y); s.z = fmaf(w, v.z, s.z); s.w = fmaf(w, v.w, s.w);
+        }
+      }
+    }
+    *(uint2*)(sX + m * xrow + c4) = make_uint2(pk_bf16(s.x, s.y), pk_bf16(s.z, s.w));
+  }
+  __syncthreads();
+  gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  const bf16_t* wp = a.wuv + ((size_t)h * a.dvp + (cok ? col : 0)) * a.rp + 8 * q;
+  const bf16_t* xp = sX + r16 * xrow + 8 * q;
+  const int ks = a.rp >> 5;
+  for (int s = KW == 4 ? wave : 0; s < ks; s += KW == 4 ? 4 : 1) {
+    const gbf16x8 af = __builtin_bit_cast(gbf16x8, *(const lu32x4*)(xp + 32 * s));
+    const gbf16x8 bf = __builtin_bit_cast(gbf16x8, *(const lu32x4*)(wp + 32 * s));
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af, bf, acc, 0, 0, 0);
+  }
+  if constexpr (KW == 4) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) sred[(wave * 16 + 4 * q + j) * 16 + r16] = acc[j];
+    __syncthreads();
+    if (wave != 0) return;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      float s = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) s += sred[(w * 16 + 4 * q + j) * 16 + r16];
+      acc[j] = s;
+    }
+  }
+  if (!cok) return;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int t = t0 + 4 * q + j;
+    if (t >= a.n) continue;
+    float v = acc[j];
+    const int c = h * a.dvp + col;
+    if (a.g_off >= 0) v *= sigmoid_f(a.qdg[(size_t)t * a.ld + a.g_off + c]);
+    ((bf16_t*)a.out)[(size_t)t * a.ldo + c] = f32_to_bf16(v);
+  }
+}
+
+// fp32: one workgroup per (token, head); the normalised latent sum in LDS, one wave per value column
+__global__ void __launch_bounds__(256) latent_out_f32_kernel(LatentAttnArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lof_smem[];  // [rp]
+  __shared__ float sw[LO_SMAX];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int f = blockIdx.x, t = f / a.H, h = f - t * a.H;
+  if (wave == 0) {
+    const float c = latent_coef(a, t, h, lane);
+    if (lane < a.nsplit) sw[lane] = c;
+  }
+  __syncthreads();
+  const size_t nf = (size_t)a.n * a.H;
+  for (int i = threadIdx.x; i < a.rp; i += 256) {
+    float s = 0.f;
+    for (int k = 0; k < a.nsplit; ++k)
+      if (sw[k] != 0.f) s = fmaf(sw[k], a.opart[(k * nf + f) * a.rp + i], s);
+    lof_smem[i] = s;
+  }
+  __syncthreads();
+  for (int d = wave; d < a.dvp; d += 4) {
+    const bf16_t* wp = a.wuv + ((size_t)h * a.dvp + d) * a.rp;
+    float s = 0.f;
+    for (int i = lane; i < a.rp; i += 64) s = fmaf(bf16_to_f32(wp[i]), lof_smem[i], s);
+    s = wave_sum(s);
+    if (lane == 0) {
+      const int c = h * a.dvp + d;
+      if (a.g_off >= 0) s *= sigmoid_f(a.qdg[(size_t)t * a.ld + a.g_off + c]);
+      ((float*)a.out)[(size_t)t * a.ldo + c] = s;
+    }
+  }
+}
+
+void launch_latent_out(const LatentAttnArgs& a, hipStream_t st) {
+  if (a.n < 1) return;
+  if (a.nsplit < 1 || a.nsplit > LO_SMAX) throw std::runtime_error("latent attention: bad key split");
+  if (a.f32) {
+    hipLaunchKernelGGL(latent_out_f32_kernel, dim3(a.n * a.H), dim3(256), (size_t)a.rp * 4, st, a);
+    return;
+  }
+  const int zt = (a.n + 15) / 16;
+  const size_t lds = (size_t)16 * (a.rp + 8) * 2 + (16 * LO_SMAX + 4 * 16 * 16) * 4;
+  const int wg64 = (a.dvp + 63) / 64 * a.H * zt;
+  if (wg64 < 2 * device_cu_count())
+    hipLaunchKernelGGL(latent_out_kernel<4>, dim3((a.dvp + 15) / 16, a.H, zt), dim3(256), lds, st, a);
+  else
+    hipLaunchKernelGGL(latent_out_kernel<1>, dim3((a.dvp + 63) / 64, a.H, zt), dim3(256), lds, st, a);
+}
+
+// ---- expanded form: gather -----------------------------------------------------------------------
+__global__ void latent_gather_kernel(const bf16_t* __restrict__ pool, const int* __restrict__ bt, int kvb, int S, int rp,
+                                     bf16_t* __restrict__ out) {
+  const int p8 = rp >> 3;
+  const size_t n = (size_t)S * p8;
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+    const int key = (int)(i / p8), c = (int)(i - (size_t)key * p8);
+    *(uint4*)(out + (size_t)key * rp + 8 * c) =
+        *(const uint4*)(pool + ((size_t)bt[key / kvb] * kvb + key % kvb) * rp + 8 * c);
+  }
+}
+void launch_latent_gather(const bf16_t* pool, const int* bt, int maxb, int kvb, int slot, int S, int rp, bf16_t* out,
+                          hipStream_t st) {
+  const size_t n = (size_t)S * (rp / 8);
+  const int g = (int)std::min<size_t>(2048, (n + 255) / 256);
+  hipLaunchKernelGGL(latent_gather_kernel, dim3(g), dim3(256), 0, st, pool, bt + (size_t)slot * maxb, kvb, S, rp, out);
+}
+
+// ---- layered decoders: embedding, row gather, weight transpose, fp32 GLU ---------------------------
+__global__ void embed_pos_kernel(const bf16_t* __restrict__ table, const bf16_t* __restrict__ pos_table,
+                                 const int* __restrict__ tokens, const int* __restrict__ pos, int d, float* __restrict__ x) {
+  const int i = blockIdx.y;
+  const bf16_t* e = table + (size_t)tokens[i] * d;
+  const bf16_t* p = pos_table ? pos_table + (size_t)pos[i] * d : nullptr;
+  for (int k = (blockIdx.x * blockDim.x + threadIdx.x) * 4; k < d; k += gridDim.x * blockDim.x * 4) {
+    const uint2 u = *(const uint2*)(e + k);
+    float4 v = make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
+                           __uint_as_float(u.y & 0xffff0000u));
+    if (p) {
+      const uint2 w = *(const uint2*)(p + k);
+      v.x += __uint_as_float(w.x << 16);
+      v.y += __uint_as_float(w.x & 0xffff0000u);
+      v.z += __uint_as_float(w.y << 16);
+      v.w += __uint_as_float(w.y & 0xffff0000u);
+    }
+    *(float4*)(x + (size_t)i * d + k) = v;
+  }
+}
+void launch_embed_pos(const bf16_t* table, const bf16_t* pos_table, const int* tokens, const int* pos, int n, int d,
+                      float* x, hipStream_t st) {
+  hipLaunchKernelGGL(embed_pos_kernel, dim3((d / 4 + 255) / 256, n), dim3(256), 0, st, table, pos_table, tokens, pos, d, x);
+}
+
+__global__ void gather_rows_kernel(const float* __restrict__ x, int d, const int* __restrict__ rows, float* __restrict__ y) {
+  const float* s = x + (size_t)rows[blockIdx.x] * d;
+  for (int k = threadIdx.x * 4; k < d; k += blockDim.x * 4) *(float4*)(y + (size_t)blockIdx.x * d + k) = *(const float4*)(s + k);
+}
+void launch_gather_rows(const float* x, int d, const int* rows, int n, float* y, hipStream_t st) {
+  hipLaunchKernelGGL(gather_rows_kernel, dim3(n), dim3(256), 0, st, x, d, rows, y);
+}
+
+__global__ void transpose_heads_kernel(const bf16_t* __restrict__ w, int rows, int cols, bf16_t* __restrict__ out) {
+  const size_t per = (size_t)rows * cols;
+  const bf16_t* s = w + blockIdx.y * per;
+  bf16_t* o = out + blockIdx.y * per;
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < per; i += (size_t)gridDim.x * blockDim.x) {
+    const int r = (int)(i / cols), c = (int)(i - (size_t)r * cols);
+    o[(size_t)c * rows + r] = s[i];
+  }
+}
+void launch_transpose_heads(const bf16_t* w, int H, int rows, int cols, bf16_t* out, hipStream_t st) {
+  const int g = (int)std::min<size_t>(256, ((size_t)rows * cols + 255) / 256);
+  hipLaunchKernelGGL(transpose_heads_kernel, dim3(g, H), dim3(256), 0, st, w, rows, cols, out);
+}
+
+__global__ void glu_f32_kernel(const float* __restrict__ gu, int ldg, float* __restrict__ out, int ldo, int n, int act) {
+  const float* g = gu + (size_t)blockIdx.y * ldg;
+  float* o = out + (size_t)blockIdx.y * ldo;
+  for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < n; i += gridDim.x * blockDim.x) {
+    const float2 v = *(const float2*)(g + 2 * i);
+    const float z = v.x;
+    const float u = act == ACT_GELU_TANH ? 1.5957691216057308f * fmaf(0.044715f * z * z, z, z) : z;
+    o[i] = z / (1.f + expf(-u)) * v.y;
+  }
+}
+void launch_glu_f32(const float* gu, int ldg, float* out, int ldo, int rows, int n, int act, hipStream_t st) {
+  hipLaunchKernelGGL(glu_f32_kernel, dim3(std::min(64, (n + 255) / 256), rows), dim3(256), 0, st, gu, ldg, out, ldo, n, act);
+}
+
+}  // namespace aios

@@ -30,8 +30,16 @@ __device__ __forceinline__ bool sk_epilogue(const GemmQArgs& a, gf32x4 (&acc)[MT
     if (m >= a.M) return 0.f;
     if (nrm) v *= inv_s[m];
     if constexpr (EPI == GEPI_SWIGLU_BF16) {
-      const uint32_t pk = pk_bf16(v[0] / (1.f + __expf(-v[0])) * v[1], v[2] / (1.f + __expf(-v[2])) * v[3]);
+      const uint32_t pk = pk_bf16(glu_act(v[0], a.act) * v[1], glu_act(v[2], a.act) * v[3]);
       *(uint32_t*)(a.C16 + (size_t)m * a.ldc + (n >> 1)) = pk;
+    } else if constexpr (EPI == GEPI_STORE16) {
+      *(uint2*)(a.C16 + (size_t)m * a.ldc + n) = make_uint2(pk_bf16(v[0], v[1]), pk_bf16(v[2], v[3]));
+    } else if constexpr (EPI == GEPI_STORE_GLU) {
+      if (n < a.glu_n0)  // (a multiple of 4: the lane's 4 columns are on one side)
+        *(float4*)(a.C + (size_t)m * a.ldc + n) = make_float4(v[0], v[1], v[2], v[3]);
+      else
+        *(uint32_t*)(a.C16 + (size_t)m * a.ldc16 + ((n - a.glu_n0) >> 1)) =
+            pk_bf16(glu_act(v[0], a.act) * v[1], glu_act(v[2], a.act) * v[3]);
     } else if constexpr (EPI == GEPI_QKV) {
       // the lane's 4 consecutive columns are two RoPE pairs (2i, 2i + 1)
       const int hd = a.head_dim, pos = a.pos[m], slot = a.slot ? a.slot[m] : 0;

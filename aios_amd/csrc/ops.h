@@ -190,7 +190,13 @@ void launch_gemm(const GemmArgs& a, hipStream_t st);
 bool gemm_supports(int qt);
 
 // multi-segment GEMM with fused epilogues (the prefill path): C = A x [W0; W1; W2]^T
-enum GemmEpi { GEPI_STORE = 0, GEPI_ACCUM = 1, GEPI_SWIGLU_BF16 = 2, GEPI_QKV = 3, GEPI_ACCUM_NORM = 4 };
+// GEPI_STORE16 (bf16 weights): C16[m][n] = bf16.  GEPI_STORE_GLU (bf16 weights, M <= 64): one launch for
+// projections that share their input -- columns below glu_n0 to C in fp32, the interleaved gate / up
+// columns from there on through the GLU to C16[m][(n - glu_n0) / 2] (row stride ldc16).
+enum GemmEpi {
+  GEPI_STORE = 0, GEPI_ACCUM = 1, GEPI_SWIGLU_BF16 = 2, GEPI_QKV = 3, GEPI_ACCUM_NORM = 4, GEPI_STORE16 = 5,
+  GEPI_STORE_GLU = 6
+};
 struct GemmQArgs {
   const bf16_t* A;   // [M][lda] bf16
   int lda;
@@ -199,9 +205,11 @@ struct GemmQArgs {
   int nseg;
   int M, N, K;
   float* C;          // [M][ldc] fp32 (STORE / ACCUM)
-  bf16_t* C16;       // [M][ldc] bf16 (SWIGLU_BF16: column n/2 = silu(col n) * col n+1)
+  bf16_t* C16;       // [M][ldc] bf16 (SWIGLU_BF16: column n/2 = act(col n) * col n+1)
   int ldc;
   int epi;
+  int act;           // gate activation of the GLU epilogues (GluAct)
+  int glu_n0, ldc16; // GEPI_STORE_GLU
   int ksplit;        // K split over workgroups: 0 = auto, 1 = off
   // skinny (M <= 64) split-K: fp32 partial slabs [S][tiles][16*Mt][rows] + per-tile arrival
   // tickets (zero-initialised, re-armed by each tile's last arriver).  Null -> no split.

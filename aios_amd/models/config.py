@@ -14,12 +14,28 @@ shapes (no network: checkpoints cannot be downloaded).
 from __future__ import annotations
 
 import dataclasses
-from typing import Dict, Optional
+from typing import Dict, Optional, Tuple
 
 from ..gguf.quants import GGMLType
 
 ROPE_NORM = 0   # llama/mistral GGUF: adjacent pairs (x[2i], x[2i+1]) (converter pre-permutes Q/K)
 ROPE_NEOX = 2   # qwen: (x[i], x[i + rot/2])
+
+
+@dataclasses.dataclass(frozen=True)
+class LayerConfig:
+    """One layer of a model described layer by layer (csrc/layered.h LayerSpec)."""
+    mixer: str = "latent"          # latent attention
+    heads: int = 1
+    dim: int = 64                  # query-key dimensions per head
+    vdim: int = 64                 # value dimensions per head
+    kv_rank: int = 64              # width of the cached latent
+    scale: float = 0.125           # of q . k
+    sink: bool = True              # a learned logit per head in the softmax's denominator
+    out_gate: bool = True          # head outputs times sigmoid(Wg h)
+    ff: int = 256                  # hidden width of the gated MLP; 0: none
+    act: str = "gelu_tanh"         # of the gate: "gelu_tanh" | "silu"
+    weights_of: int = -1           # layer whose weights this one uses, or -1
 
 
 @dataclasses.dataclass
@@ -44,6 +60,8 @@ class ModelConfig:
     eos_id: int = 2
     tokenizer_model: str = "llama"  # "llama" (SPM) or "gpt2" (byte-level BPE)
     chat_template: str = "zephyr"
+    # models described layer by layer; empty: a llama-family decoder of the sizes above
+    layers: Tuple[LayerConfig, ...] = ()
 
     @property
     def q_dim(self) -> int:
@@ -58,6 +76,13 @@ class ModelConfig:
         return self.q_dim + 2 * self.kv_dim
 
     def n_params(self) -> int:
+        if self.layers:
+            n = 2 * self.vocab_size * self.d_model + self.max_ctx * self.d_model
+            for l in self.layers:
+                if l.weights_of < 0:
+                    n += self.d_model * (l.heads * (l.dim + 2 * l.vdim) + l.kv_rank + 3 * l.ff)
+                    n += l.kv_rank * l.heads * (l.dim + l.vdim)
+            return n
         per_layer = self.d_model * (self.qkv_dim + self.q_dim) + 3 * self.d_model * self.d_ff + 2 * self.d_model
         emb = self.vocab_size * self.d_model * (1 if self.tie_embeddings else 2)
         return self.n_layers * per_layer + emb + self.d_model
@@ -99,6 +124,13 @@ class ModelConfig:
             tokenizer_model=str(reader.get("tokenizer.ggml.model", "llama")),
             chat_template=tmpl if isinstance(tmpl, str) else "zephyr",
         )
+
+
+def _gefazen(name: str, vocab: int, width: int, n_layers: int, max_ctx: int, **layer) -> ModelConfig:
+    l = LayerConfig(scale=layer["dim"] ** -0.5, **layer)
+    return ModelConfig(name=name, arch="gefazen", vocab_size=vocab, d_model=width, n_layers=n_layers, n_heads=l.heads,
+                       n_kv_heads=1, head_dim=l.dim, d_ff=l.ff, max_ctx=max_ctx, bos_id=-1, eos_id=-1,
+                       layers=(l,) * n_layers)
 
 
 PRESETS: Dict[str, ModelConfig] = {
@@ -148,6 +180,11 @@ PRESETS: Dict[str, ModelConfig] = {
         name="test-llama3-shape", vocab_size=128256, d_model=512, n_layers=2, n_heads=4, n_kv_heads=1, head_dim=128,
         d_ff=1536, rope_theta=5e5, max_ctx=512, bos_id=128000, eos_id=128009, tokenizer_model="gpt2",
         chat_template="llama3"),
+    # Gefazen at the widths of the two tiers above (random-init only): TinyLlama's and Mistral-7B's
+    # width, depth, heads and MLP, a 512-wide latent
+    "gefazen-1b": _gefazen("gefazen-1b", 32000, 2048, 22, 4096, heads=32, dim=64, vdim=64, kv_rank=512, ff=5632),
+    "gefazen-7b": _gefazen("gefazen-7b", 32000, 4096, 32, 32768, heads=32, dim=128, vdim=128, kv_rank=512, ff=14336),
+    "test-gefazen": _gefazen("test-gefazen", 700, 512, 3, 512, heads=4, dim=64, vdim=32, kv_rank=64, ff=1024),
     "test-mistral-shape": ModelConfig(
         name="test-mistral-shape", vocab_size=1024, d_model=1024, n_layers=2, n_heads=8, n_kv_heads=2,
         head_dim=128, d_ff=2048, rope_theta=1e6, max_ctx=512, chat_template="mistral"),

@@ -1,0 +1,56 @@
+"""Registry of the model designs a checkpoint folder can hold.
+
+A folder checkpoint is `config.json` + `model.safetensors`; its `architecture` names the entry here that
+reads the configuration into a `ModelConfig` and maps tensor names to the engine's.  (A GGUF file
+carries its own architecture and names: `ModelConfig.from_gguf`.)
+"""
+from __future__ import annotations
+
+import dataclasses
+import importlib
+import json
+import os
+from typing import Callable, Dict, Tuple
+
+from .config import ModelConfig
+
+
+@dataclasses.dataclass(frozen=True)
+class Architecture:
+    parse: Callable[[dict, str], ModelConfig]         # (config.json, model name) -> ModelConfig
+    tensor_names: Callable[[dict], Dict[str, str]]    # config.json -> {checkpoint name: engine name}
+
+
+# architecture -> module under aios_amd.models that defines ARCHITECTURE
+_MODULES = {"gefazen": "gefazen"}
+
+
+def architectures():
+    return sorted(_MODULES)
+
+
+def get(name: str) -> Architecture:
+    mod = _MODULES.get(str(name).lower())
+    if mod is None:
+        raise ValueError(f"unknown model architecture {name!r}; have {architectures()}")
+    return importlib.import_module(f"{__package__}.{mod}").ARCHITECTURE
+
+
+def is_checkpoint_dir(path: str) -> bool:
+    """Whether `path` is a folder checkpoint of a registered architecture."""
+    f = os.path.join(path, "config.json")
+    if not (os.path.isfile(f) and os.path.isfile(os.path.join(path, "model.safetensors"))):
+        return False
+    try:
+        with open(f) as fh:
+            return str(json.load(fh).get("architecture", "")).lower() in _MODULES
+    except (OSError, ValueError, AttributeError):
+        return False
+
+
+def load_config(path: str, name: str = "") -> Tuple[ModelConfig, dict, Architecture]:
+    """(ModelConfig, raw config.json, architecture) of a folder checkpoint."""
+    with open(os.path.join(path, "config.json")) as f:
+        raw = json.load(f)
+    arch = get(raw.get("architecture", ""))
+    return arch.parse(raw, name or os.path.basename(os.path.normpath(path))), raw, arch

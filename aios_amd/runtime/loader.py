@@ -26,6 +26,7 @@ log = logging.getLogger("aios.runtime.loader")
 
 COLUMN_PARALLEL = ("attn_q.weight", "attn_k.weight", "attn_v.weight", "ffn_gate.weight", "ffn_up.weight",
                    "attn_q.bias", "attn_k.bias", "attn_v.bias")
+_ST_TYPES = {"BF16": GGMLType.BF16, "F16": GGMLType.F16, "F32": GGMLType.F32}
 ROW_PARALLEL = ("attn_output.weight", "ffn_down.weight")
 
 
@@ -57,15 +58,23 @@ def shard_tensor(name: str, raw: np.ndarray, ggml_type: int, rows: int, cols: in
 
 def load_engine(path: str, max_ctx: Optional[int] = None, max_slots: int = 4, max_batch: int = 8, device: int = 0,
                 tp_rank: int = 0, tp_size: int = 1, name: Optional[str] = None, verbose: bool = False,
-                act_q8: bool = True, cu_mask: Optional[list] = None, kv_dtype: str = "bf16"):
-    """Load a GGUF file into a native Engine on `device`. Returns (engine, ModelConfig, reader)."""
+                act_q8: bool = True, cu_mask: Optional[list] = None, kv_dtype: str = "bf16", compute: str = "bf16",
+                kv_pool_tokens: int = 0):
+    """Load a GGUF file, or a folder checkpoint (config.json + model.safetensors of a registered
+    architecture), into a native Engine on `device`.  Returns (engine, ModelConfig, reader)."""
+    if os.path.isdir(path):
+        return _load_dir(path, max_ctx, name, verbose,
+                         dict(max_slots=max_slots, max_batch=max_batch, device=device, tp_rank=tp_rank, tp_size=tp_size,
+                              act_q8=act_q8, cu_mask=cu_mask, kv_dtype=kv_dtype, compute=compute,
+                              kv_pool_tokens=kv_pool_tokens))
     m = native.require()
     t0 = time.time()
     r = GGUFReader(path)
     cfg = ModelConfig.from_gguf(r, name=name)
     ec = native.engine_config(cfg, max_ctx=max_ctx or min(cfg.max_ctx, 4096), max_slots=max_slots,
                               max_batch=max_batch, device=device, tp_rank=tp_rank, tp_size=tp_size,
-                              act_q8=act_q8, cu_mask=cu_mask, kv_dtype=kv_dtype)
+                              act_q8=act_q8, cu_mask=cu_mask, kv_dtype=kv_dtype, compute=compute,
+                              kv_pool_tokens=kv_pool_tokens)
     eng = m.Engine(ec)
     vp = bool(ec.vocab_parallel)
     for tname, ti in r.tensors.items():
@@ -73,6 +82,30 @@ def load_engine(path: str, max_ctx: Optional[int] = None, max_slots: int = 4, ma
         rows, cols = ti.rows, ti.cols
         raw, rows, cols = shard_tensor(tname, raw, int(ti.ggml_type), rows, cols, tp_rank, tp_size, vp)
         eng.set_tensor(tname, int(ti.ggml_type), rows, cols, raw)
+    finalize(eng)
+    if verbose:
+        print(f"[loader] {cfg.name}: {eng.weight_bytes / 1e9:.2f} GB weights, {eng.kv_bytes / 1e9:.2f} GB KV, "
+              f"{time.time() - t0:.1f}s")
+    return eng, cfg, r
+
+
+def _load_dir(path: str, max_ctx: Optional[int], name: Optional[str], verbose: bool, engine_kw: dict):
+    from ..models import registry
+    from .safetensors import SafetensorsReader
+
+    t0 = time.time()
+    cfg, raw, arch = registry.load_config(path, name or "")
+    m = native.require()
+    eng = m.Engine(native.engine_config(cfg, max_ctx=min(max_ctx or cfg.max_ctx, cfg.max_ctx), **engine_kw))
+    r = SafetensorsReader(os.path.join(path, "model.safetensors"))
+    for src, dst in arch.tensor_names(raw).items():
+        if src not in r.tensors:
+            raise ValueError(f"{path}: tensor {src} is missing")
+        t = r.tensors[src]
+        if t.dtype not in _ST_TYPES:
+            raise ValueError(f"{path}: tensor {src} has unsupported dtype {t.dtype}")
+        rows, cols = (1, t.shape[0]) if len(t.shape) == 1 else t.shape
+        eng.set_tensor(dst, int(_ST_TYPES[t.dtype]), rows, cols, r.raw(src))
     finalize(eng)
     if verbose:
         print(f"[loader] {cfg.name}: {eng.weight_bytes / 1e9:.2f} GB weights, {eng.kv_bytes / 1e9:.2f} GB KV, "
@@ -108,14 +141,16 @@ def finalize(eng):
 
 def random_engine(cfg: ModelConfig, recipe: str = "Q4_K_M", seed: int = 0, max_ctx: Optional[int] = None,
                   max_slots: int = 4, max_batch: int = 8, device: int = 0, tp_rank: int = 0, tp_size: int = 1,
-                  act_q8: bool = True, cu_mask: Optional[list] = None, kv_dtype: str = "bf16"):
+                  act_q8: bool = True, cu_mask: Optional[list] = None, kv_dtype: str = "bf16", compute: str = "bf16",
+                  kv_pool_tokens: int = 0):
     """Engine with random-init weights of `cfg`'s architecture generated directly in HBM (cu_mask: the
     CUs its stream may use, native.cu_mask_words)."""
     m = native.require()
     ec = native.engine_config(cfg, max_ctx=max_ctx or min(cfg.max_ctx, 4096), max_slots=max_slots,
                               max_batch=max_batch, device=device, tp_rank=tp_rank, tp_size=tp_size,
-                              act_q8=act_q8, cu_mask=cu_mask, kv_dtype=kv_dtype)
+                              act_q8=act_q8, cu_mask=cu_mask, kv_dtype=kv_dtype, compute=compute,
+                              kv_pool_tokens=kv_pool_tokens)
     eng = m.Engine(ec)
-    eng.init_random(recipe, seed)
+    eng.init_random("BF16" if cfg.layers else recipe, seed)  # (layered models hold bf16 weights)
     finalize(eng)
     return eng

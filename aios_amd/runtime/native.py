@@ -57,7 +57,7 @@ def gpu_available() -> bool:
         return False
 
 
-def require():
+def require(formats: str = "all"):
     """The native engine, loudly: on a GPU box a missing extension is an error."""
     return load(build_if_missing=True)
 
@@ -94,10 +94,11 @@ def cu_mask_words(n: int, first: int = 0, total: int = 256) -> list:
 
 def engine_config(cfg, max_ctx: Optional[int] = None, max_slots: int = 4, max_batch: int = 8, device: int = 0,
                   tp_rank: int = 0, tp_size: int = 1, act_q8: bool = True, vocab_parallel: bool = True,
-                  cu_mask: Optional[list] = None, kv_dtype: str = "bf16"):
+                  cu_mask: Optional[list] = None, kv_dtype: str = "bf16", compute: str = "bf16", kv_pool_tokens: int = 0):
     """aios_amd.models.config.ModelConfig -> native EngineConfig (per-rank shapes under TP).
     Under TP the lm_head is vocab-parallel (V/tp rows per rank + logits all-gather) unless the
-    embeddings are tied or V is not divisible by tp."""
+    embeddings are tied or V is not divisible by tp.  compute "float32" (layered models): everything
+    in 32 bits.  kv_pool_tokens: tokens the cache pool holds (0: every slot's full context)."""
     m = require()
     ec = m.EngineConfig()
     ec.name = cfg.name
@@ -128,4 +129,29 @@ def engine_config(cfg, max_ctx: Optional[int] = None, max_slots: int = 4, max_ba
         ec.cu_mask = [int(w) & 0xFFFFFFFF for w in cu_mask]
     ec.kv_fp8 = kv_fp8_flag(kv_dtype)
     ec.act_q8 = int(act_q8)
+    ec.kv_pool_tokens = int(kv_pool_tokens)
+    if compute not in ("bf16", "bfloat16", "f32", "float32"):
+        raise ValueError(f"compute must be bfloat16 or float32, not {compute!r}")
+    ec.compute_f32 = int(compute in ("f32", "float32"))
+    if ec.compute_f32 and not cfg.layers:
+        raise ValueError(f"{cfg.name}: only layered models compute in 32 bits")
+    if cfg.layers:
+        if tp_size > 1:
+            raise ValueError(f"{cfg.name}: layered models run on one GPU (no tensor parallelism)")
+        if ec.kv_fp8:
+            raise ValueError(f"{cfg.name}: the latent cache has no fp8 form (kv_dtype bf16)")
+        ec.max_positions = int(cfg.max_ctx)
+        ec.layers = [_layer_spec(m, l) for l in cfg.layers]
     return ec
+
+
+def _layer_spec(m, l):
+    s = m.LayerSpec()
+    s.mixer = {"latent": m.MIX_LATENT}[l.mixer]
+    s.heads, s.dim, s.vdim, s.kv_rank = l.heads, l.dim, l.vdim, l.kv_rank
+    s.scale = float(l.scale)
+    s.sink, s.out_gate = int(l.sink), int(l.out_gate)
+    s.mlp, s.ff = (m.MLP_GLU, l.ff) if l.ff else (m.MLP_NONE, 0)
+    s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU}[l.act]
+    s.weights_of = l.weights_of
+    return s
