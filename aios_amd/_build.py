@@ -33,21 +33,29 @@ def ext_suffix() -> str:
     return sysconfig.get_config_var("EXT_SUFFIX") or ".so"
 
 
-def target_path() -> Path:
-    return PKG / ("_engine" + ext_suffix())
+# formats="all": every GGUF weight format; "bf16": the bf16 kernels alone (folder checkpoints hold bf16
+# weights, and the quantised formats' kernels take most of a full build) -- a module of its own, used
+# where no full build is there
+FORMATS = {"all": "_engine", "bf16": "_engine_bf16"}
+_QUANT_SOURCES = ("gemv_kquant.hip", "gemv_kquant2.hip", "gemv_legacy.hip", "gemm_pf_mix.hip", "gemm_pf_q4k.hip",
+                  "gemm_pf_q5k.hip", "gemm_pf_q6k.hip", "gemm_pf_q8q4.hip", "microbench.hip")
 
 
-def _sources():
+def target_path(formats: str = "all") -> Path:
+    return PKG / (FORMATS[formats] + ext_suffix())
+
+
+def _sources(formats: str = "all"):
     srcs = sorted((CSRC / "kernels").glob("*.hip")) + [CSRC / "engine.hip", CSRC / "layered.hip", CSRC / "grammar.cpp", CSRC / "rccl_comm.cpp",
                                                       CSRC / "bindings.cpp"]
-    return srcs
+    return [s for s in srcs if formats == "all" or s.name not in _QUANT_SOURCES]
 
 
 def _headers():
     return list(CSRC.rglob("*.h"))
 
 
-def _flags():
+def _flags(formats: str = "all"):
     import pybind11
 
     return [
@@ -64,7 +72,8 @@ def _flags():
         f"-I{CSRC}",
         f"-I{pybind11.get_include()}",
         f"-I{sysconfig.get_paths()['include']}",
-    ] + (["-DAIOS_GEMV_PROBES=1", "-DAIOS_ATTN_PROBES=1", "-DAIOS_SAMPLE_PROBES=1"] if os.environ.get("AIOS_BUILD_PROBES") == "1" else [])
+    ] + (["-DAIOS_BF16_ONLY=1", "-DAIOS_MODULE=" + FORMATS[formats]] if formats == "bf16" else []) + (
+        ["-DAIOS_GEMV_PROBES=1", "-DAIOS_ATTN_PROBES=1", "-DAIOS_SAMPLE_PROBES=1"] if os.environ.get("AIOS_BUILD_PROBES") == "1" else [])
     # (AIOS_BUILD_PROBES=1: the microbenchmark / phase-stamp hooks the probe tools use -- tools/attn_probe.py
     # --stamps, tools/gemv_cu_probe.py ring mode; compiled out of production builds)
 
@@ -113,19 +122,20 @@ def _compile(src: Path, flags, hipcc, build_dir: Path = None) -> Path:
     return obj
 
 
-def build(verbose: bool = True, jobs: int | None = None, build_dir: Path | None = None, out: Path | None = None) -> Path:
+def build(verbose: bool = True, jobs: int | None = None, build_dir: Path | None = None, out: Path | None = None,
+          formats: str = "all") -> Path:
     """Compile every HIP / C++ source of the engine for gfx950 (incrementally: an object is rebuilt when
     its source or a header it includes is newer) and link the extension.  build_dir / out: a clean
     build elsewhere (tests/test_build.py), leaving the in-tree objects and .so alone."""
-    build_dir = Path(build_dir) if build_dir else BUILD
+    build_dir = Path(build_dir) if build_dir else (BUILD if formats == "all" else BUILD.with_name("native-" + formats))
     build_dir.mkdir(parents=True, exist_ok=True)
     hipcc = _hipcc()
-    flags = _flags()
-    srcs = _sources()
+    flags = _flags(formats)
+    srcs = _sources(formats)
     jobs = jobs or min(len(srcs), max(1, (os.cpu_count() or 4)), 16)
     with cf.ThreadPoolExecutor(jobs) as ex:
         objs = list(ex.map(lambda s: _compile(s, flags, hipcc, build_dir), srcs))
-    out = Path(out) if out else target_path()
+    out = Path(out) if out else target_path(formats)
     newest = max(o.stat().st_mtime for o in objs)
     if not out.exists() or out.stat().st_mtime < newest:
         tmp = out.with_suffix(".tmp.so")

@@ -15,11 +15,13 @@
 namespace py = pybind11;
 using namespace aios;
 
+#ifndef AIOS_BF16_ONLY
 namespace aios {
 double bench_launch_chain(int n_kernels, int blocks, int use_graph, int reps);
 double bench_stream_read(size_t bytes, int nbuf, int wg_per_cu, int u, int threads, int reps);
 double bench_stream_read_part(size_t bytes, int nbuf, int mode, int threads, int reps);
 }
+#endif
 
 namespace {
 
@@ -105,7 +107,10 @@ struct PyQMatrix {
 
 }  // namespace
 
-PYBIND11_MODULE(_engine, m) {
+#ifndef AIOS_MODULE
+#define AIOS_MODULE _engine
+#endif
+PYBIND11_MODULE(AIOS_MODULE, m) {
   m.doc() = "aiOS-MI355X native inference engine (gfx950 HIP kernels + C++ runtime)";
   m.attr("QT_F32") = (int)QT_F32;
   m.attr("QT_F16") = (int)QT_F16;
@@ -119,6 +124,7 @@ PYBIND11_MODULE(_engine, m) {
   m.attr("EPI_RESID") = (int)EPI_RESID;
   m.attr("EPI_SWIGLU") = (int)EPI_SWIGLU;
   m.attr("EPI_QKV") = (int)EPI_QKV;
+  m.attr("EPI_STORE_GLU") = (int)EPI_STORE_GLU;
   m.attr("KV_BLOCK") = KV_BLOCK;
   m.attr("ATTN_CHUNK") = (int)ATTN_CHUNK;
 
@@ -453,7 +459,7 @@ PYBIND11_MODULE(_engine, m) {
   m.def("gemv",
         [](std::vector<PyQMatrix*> segs, int B, uintptr_t x, int ldx, uintptr_t norm_w, float eps, uintptr_t y,
            int ldy, int epi, uintptr_t st, int force_v1, int act_q8, int tune_grid, int tune_u, int tune_ksplit, int tune_dbg,
-           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16) {
+           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16) {
           GemvArgs a;
           std::memset(&a, 0, sizeof(a));
           a.nseg = (int)segs.size();
@@ -465,12 +471,14 @@ PYBIND11_MODULE(_engine, m) {
           a.tune_grid = tune_grid; a.tune_u = tune_u; a.tune_ksplit = tune_ksplit; a.tune_dbg = tune_dbg;
           a.kernel_sel = kernel_sel; a.dbg_ts = (unsigned long long*)dbg_ts;
           a.x16 = (const bf16_t*)x16; a.y16 = (bf16_t*)y16;  // bf16 input / SwiGLU output (hand-off kernels)
+          a.act = act; a.glu_row0 = glu_row0; a.ldy16 = ldy16;
           launch_gemv(a, S(st));
         },
         py::arg("segs"), py::arg("B"), py::arg("x"), py::arg("ldx"), py::arg("norm_w"), py::arg("eps"), py::arg("y"),
         py::arg("ldy"), py::arg("epi"), py::arg("stream"), py::arg("force_v1") = 0, py::arg("act_q8") = 0,
         py::arg("tune_grid") = 0, py::arg("tune_u") = 0, py::arg("tune_ksplit") = 0, py::arg("tune_dbg") = 0,
-        py::arg("kernel_sel") = 0, py::arg("dbg_ts") = 0, py::arg("x16") = 0, py::arg("y16") = 0);
+        py::arg("kernel_sel") = 0, py::arg("dbg_ts") = 0, py::arg("x16") = 0, py::arg("y16") = 0, py::arg("act") = 0,
+        py::arg("glu_row0") = 0, py::arg("ldy16") = 0);
   m.def("gemv_bf16_engine_fits",
         [](std::vector<PyQMatrix*> segs, int B, int epi) {
           GemvArgs a;
@@ -613,7 +621,7 @@ PYBIND11_MODULE(_engine, m) {
   m.def(
       "gemm_q",
       [](uintptr_t A, int lda, std::vector<PyQMatrix*> segs, int M, uintptr_t C, uintptr_t C16, int ldc, int epi,
-         uintptr_t st, int ksplit, uintptr_t dbg_ts) {
+         uintptr_t st, int ksplit, uintptr_t dbg_ts, int act, int glu_n0, int ldc16) {
         GemmQArgs a;
         std::memset(&a, 0, sizeof(a));
         if (segs.empty() || segs.size() > 3) throw std::runtime_error("gemm_q: 1..3 segments");
@@ -623,12 +631,14 @@ PYBIND11_MODULE(_engine, m) {
         a.M = M; a.N = n0; a.K = segs[0]->w.cols;
         a.C = (float*)C; a.C16 = (bf16_t*)C16; a.ldc = ldc; a.epi = epi; a.ksplit = ksplit;
         a.dbg_ts = (unsigned long long*)dbg_ts;
+        a.act = act; a.glu_n0 = glu_n0; a.ldc16 = ldc16;
         GemmWs& g = gemm_ws(M, a.N);
         a.ws = g.ws; a.ws_bytes = g.bytes; a.cnt = g.cnt; a.cnt_len = g.cnt_len;
         launch_gemm_q(a, S(st));
       },
       py::arg("A"), py::arg("lda"), py::arg("segs"), py::arg("M"), py::arg("C"), py::arg("C16"), py::arg("ldc"),
-      py::arg("epi"), py::arg("stream"), py::arg("ksplit") = 0, py::arg("dbg_ts") = 0);
+      py::arg("epi"), py::arg("stream"), py::arg("ksplit") = 0, py::arg("dbg_ts") = 0, py::arg("act") = 0,
+      py::arg("glu_n0") = 0, py::arg("ldc16") = 0);
   m.def(
       "gemm_pf_plan",
       [](std::vector<PyQMatrix*> segs, int M, int epi, int ksplit) {
@@ -644,6 +654,7 @@ PYBIND11_MODULE(_engine, m) {
         return py::make_tuple(bm, bn, sp);
       },
       py::arg("segs"), py::arg("M"), py::arg("epi"), py::arg("ksplit") = 0);
+#ifndef AIOS_BF16_ONLY
   m.def(
       "gemm_pf_probe",
       [](uintptr_t A, int lda, PyQMatrix* w, int M, uintptr_t C, int probe, uintptr_t st) {
@@ -653,9 +664,12 @@ PYBIND11_MODULE(_engine, m) {
         a.K = w->w.cols; a.C = (float*)C; a.ldc = a.N; a.epi = GEPI_STORE;
         return gemm_pf_probe(a, probe, S(st));
       });
+#endif
   m.attr("GEPI_STORE") = (int)GEPI_STORE;
   m.attr("GEPI_ACCUM") = (int)GEPI_ACCUM;
   m.attr("GEPI_SWIGLU_BF16") = (int)GEPI_SWIGLU_BF16;
+  m.attr("GEPI_STORE16") = (int)GEPI_STORE16;
+  m.attr("GEPI_STORE_GLU") = (int)GEPI_STORE_GLU;
   m.def(
       "attn_prefill",
       [](uintptr_t q, uintptr_t k, uintptr_t v, int slot, int start, int T, int H, int Hkv, int hd, int max_ctx,
@@ -674,6 +688,62 @@ PYBIND11_MODULE(_engine, m) {
       py::arg("st"), py::arg("block_table") = 0, py::arg("kv_fp8") = 0, py::arg("k_scale") = 1.f,
       py::arg("v_scale") = 1.f);
   m.def("attn_prefill_supports", &attn_prefill_supports);
+
+  // ------------------------------------------------------------------ latent attention
+  // the absorbed path over a paged cache: prep (latents of `rows` rows into the cache, queries of the first
+  // n absorbed), attention, output.  tiles: (first flat row, rows) pairs on the device or 0 (every row its
+  // own sequence)
+  m.def(
+      "latent_attention",
+      [](int n, int rows, int H, int dk, int dkp, int dvp, int rank, int rp, float scale, float eps, uintptr_t norm_w,
+         uintptr_t sink, uintptr_t qdg, int ld, int dkv_off, int g_off, uintptr_t pos, uintptr_t slot, uintptr_t pool,
+         uintptr_t bt, int maxb, int kvb, int f32, uintptr_t wukT, uintptr_t wuv, uintptr_t qa, uintptr_t tiles,
+         int n_tiles, int nsplit, uintptr_t opart, uintptr_t ml, uintptr_t out, int ldo, uintptr_t st) {
+        LatentAttnArgs a;
+        std::memset(&a, 0, sizeof(a));
+        a.n = n; a.H = H; a.dk = dk; a.dkp = dkp; a.dvp = dvp; a.rank = rank; a.rp = rp; a.scale = scale; a.eps = eps;
+        a.norm_w = (const float*)norm_w; a.sink = (const float*)sink; a.qdg = (const float*)qdg; a.ld = ld;
+        a.dkv_off = dkv_off; a.g_off = g_off; a.pos = (const int*)pos; a.slot = (const int*)slot; a.pool = (void*)pool;
+        a.bt = (const int*)bt; a.maxb = maxb; a.kvb = kvb; a.f32 = f32; a.wukT = (const bf16_t*)wukT;
+        a.wuv = (const bf16_t*)wuv; a.qa = (void*)qa; a.tiles = (const LatentTile*)tiles; a.n_tiles = n_tiles;
+        a.nsplit = nsplit; a.opart = (float*)opart; a.ml = (float*)ml; a.out = (void*)out; a.ldo = ldo;
+        if (dkp % 32 || dvp % 32 || rp % 64 || n > rows) throw std::runtime_error("latent_attention: bad padding");
+        launch_latent_prep(a, rows, S(st));
+        launch_latent_attn(a, S(st));
+        launch_latent_out(a, S(st));
+      },
+      py::arg("n"), py::arg("rows"), py::arg("H"), py::arg("dk"), py::arg("dkp"), py::arg("dvp"), py::arg("rank"),
+      py::arg("rp"), py::arg("scale"), py::arg("eps"), py::arg("norm_w"), py::arg("sink"), py::arg("qdg"), py::arg("ld"),
+      py::arg("dkv_off"), py::arg("g_off"), py::arg("pos"), py::arg("slot"), py::arg("pool"), py::arg("bt"),
+      py::arg("maxb"), py::arg("kvb"), py::arg("f32"), py::arg("wukT"), py::arg("wuv"), py::arg("qa"), py::arg("tiles"),
+      py::arg("n_tiles"), py::arg("nsplit"), py::arg("opart"), py::arg("ml"), py::arg("out"), py::arg("ldo"),
+      py::arg("stream"));
+  m.def(
+      "mha_prefill",
+      [](uintptr_t q, int ldq, uintptr_t k, uintptr_t v, int ldkv, int H, int dkp, int dvp, int start, int T, float scale,
+         uintptr_t sink, uintptr_t gate, uintptr_t out, int ldo, uintptr_t st) {
+        MhaPrefillArgs a;
+        a.q = (const float*)q; a.ldq = ldq; a.k = (const bf16_t*)k; a.v = (const bf16_t*)v; a.ldkv = ldkv; a.H = H;
+        a.dkp = dkp; a.dvp = dvp; a.start = start; a.T = T; a.scale = scale; a.sink = (const float*)sink;
+        a.gate = (const float*)gate; a.out = (bf16_t*)out; a.ldo = ldo;
+        launch_mha_prefill(a, S(st));
+      },
+      py::arg("q"), py::arg("ldq"), py::arg("k"), py::arg("v"), py::arg("ldkv"), py::arg("H"), py::arg("dkp"),
+      py::arg("dvp"), py::arg("start"), py::arg("T"), py::arg("scale"), py::arg("sink"), py::arg("gate"), py::arg("out"),
+      py::arg("ldo"), py::arg("stream"));
+  m.def("gemm_f32",
+        [](uintptr_t A, int lda, uintptr_t W, int ldw, int M, int N, int K, uintptr_t C, int ldc, int accumulate,
+           uintptr_t st) {
+          launch_gemm_f32((const float*)A, lda, (const bf16_t*)W, ldw, M, N, K, (float*)C, ldc, accumulate, S(st));
+        });
+  m.def("embed_pos", [](uintptr_t table, uintptr_t pos_table, uintptr_t tokens, uintptr_t pos, int n, int d, uintptr_t x,
+                        uintptr_t st) {
+    launch_embed_pos((const bf16_t*)table, (const bf16_t*)pos_table, (const int*)tokens, (const int*)pos, n, d, (float*)x,
+                     S(st));
+  });
+  m.def("glu_f32", [](uintptr_t gu, int ldg, uintptr_t out, int ldo, int rows, int n, int act, uintptr_t st) {
+    launch_glu_f32((const float*)gu, ldg, (float*)out, ldo, rows, n, act, S(st));
+  });
 
   // ------------------------------------------------------------------ JSON-mode grammar (K10)
   py::class_<JsonState>(m, "JsonState")
@@ -715,10 +785,12 @@ PYBIND11_MODULE(_engine, m) {
       .def_property_readonly("cache_size", &JsonGrammar::cache_size);
   m.def("gemm_pf_export", &gemm_pf_export);
   m.def("gemm_pf_import", &gemm_pf_import, py::arg("plans"));
+#ifndef AIOS_BF16_ONLY
   m.def("bench_stream_read_part", &aios::bench_stream_read_part, py::arg("bytes"), py::arg("nbuf"), py::arg("mode"),
         py::arg("threads") = 512, py::arg("reps") = 20);
   m.def("bench_stream_read", &aios::bench_stream_read, py::arg("bytes"), py::arg("nbuf"), py::arg("wg_per_cu"),
         py::arg("u"), py::arg("threads"), py::arg("reps"));
   m.def("bench_launch_chain", &aios::bench_launch_chain, py::arg("n_kernels"), py::arg("blocks"), py::arg("use_graph"),
         py::arg("reps"), py::call_guard<py::gil_scoped_release>());
+#endif
 }

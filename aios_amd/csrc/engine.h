@@ -222,7 +222,6 @@ class Engine {
   void init_paging();                    // block tables and the free list
   size_t init_step_state();              // logits, decode parameters, sampler (workspace bytes)
   void finalize_layered();
-  int ctx_limit() const;                 // positions a sequence may use
   void run_step(const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
                 const std::vector<int>& tokens, const std::vector<int>& want, std::vector<float>* logits);
   void enqueue_decode_step(int B);       // uses device arrays d_tokens_/d_pos_/d_seqlen_/d_slot_

@@ -551,8 +551,6 @@ void Engine::finalize_layered() {
   finalized_ = true;
 }
 
-int Engine::ctx_limit() const { return cfg_.max_ctx; }
-
 void Engine::finalize() {
   const CuScope cu_scope(cus_);  // (grids sized to this engine's CU mask)
   TraceRange tr("aios.finalize");
@@ -1531,7 +1529,7 @@ void Engine::run_step(const std::vector<int>& slots, const std::vector<int>& sta
   for (int e = 0; e < E; ++e) {
     if (slots[e] < 0 || slots[e] >= cfg_.max_slots) throw std::runtime_error("step: bad slot");
     if (!seen.insert(slots[e]).second) throw std::runtime_error("step: a slot appears twice");
-    if (counts[e] < 1 || starts[e] < 0 || starts[e] + counts[e] > ctx_limit())
+    if (counts[e] < 1 || starts[e] < 0 || starts[e] + counts[e] > cfg_.max_ctx)
       throw std::runtime_error("step: context overflow");
     total += counts[e];
   }

@@ -252,12 +252,14 @@ static void launch_one(const GemmQArgs& a, hipStream_t st) {
   if (a.epi == GEPI_QKV || a.epi == GEPI_ACCUM_NORM || a.epi == GEPI_STORE_GLU || a.nrm_in)
     throw std::runtime_error("gemm: the QKV / fused-RMSNorm / store + GLU epilogues need the skinny (M <= 64) kernel");
   switch (a.seg[0].qtype) {
+#ifndef AIOS_BF16_ONLY
     case QT_Q4_K: launch_big<QT_Q4_K>(a, st); break;
     case QT_Q5_K: launch_big<QT_Q5_K>(a, st); break;
     case QT_Q6_K: launch_big<QT_Q6_K>(a, st); break;
     case QT_Q4_0: launch_big<QT_Q4_0>(a, st); break;
     case QT_Q8_0: launch_big<QT_Q8_0>(a, st); break;
     case QT_F16: launch_big<QT_F16>(a, st); break;
+#endif
     case QT_BF16: launch_big<QT_BF16>(a, st); break;
     default: throw std::runtime_error("gemm: unsupported weight format");
   }

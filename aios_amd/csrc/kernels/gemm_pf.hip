@@ -13,14 +13,16 @@
 
 namespace aios {
 
+extern template bool pf_launch_fmt<QT_BF16, QT_BF16>(const GemmQArgs&, int, int, int, hipStream_t);
+#ifndef AIOS_BF16_ONLY
 extern template bool pf_launch_fmt<QT_Q4_K, QT_Q4_K>(const GemmQArgs&, int, int, int, hipStream_t);
 extern template bool pf_launch_fmt<QT_Q6_K, QT_Q6_K>(const GemmQArgs&, int, int, int, hipStream_t);
 extern template bool pf_launch_fmt<QT_Q4_K, QT_Q6_K>(const GemmQArgs&, int, int, int, hipStream_t);
-extern template bool pf_launch_fmt<QT_BF16, QT_BF16>(const GemmQArgs&, int, int, int, hipStream_t);
 extern template bool pf_launch_fmt<QT_Q5_K, QT_Q5_K>(const GemmQArgs&, int, int, int, hipStream_t);
 extern template bool pf_launch_fmt<QT_Q5_K, QT_Q6_K>(const GemmQArgs&, int, int, int, hipStream_t);
 extern template bool pf_launch_fmt<QT_Q4_0, QT_Q4_0>(const GemmQArgs&, int, int, int, hipStream_t);
 extern template bool pf_launch_fmt<QT_Q8_0, QT_Q8_0>(const GemmQArgs&, int, int, int, hipStream_t);
+#endif
 
 static int pf_env(const char* name, int dflt) {
   const char* e = std::getenv(name);
@@ -185,6 +187,7 @@ static bool pf_run(const GemmQArgs& a, const PfPlan& p, hipStream_t st) {
   if (p.s != 1 && a.epi == GEPI_QKV) return false;  // (plans keep S = 1 for it; a pinned split declines)
   if (p.s != 1 && a.epi == GEPI_STORE)
     HIP_CHECK(hipMemset2DAsync(a.C, (size_t)a.ldc * 4, 0, (size_t)a.N * 4, a.M, st));
+#ifndef AIOS_BF16_ONLY
   if (qt0 == QT_Q4_K && qt1 == QT_Q4_K) return pf_launch_fmt<QT_Q4_K, QT_Q4_K>(a, p.bm, p.bn, p.s, st);
   if (qt0 == QT_Q6_K && qt1 == QT_Q6_K) return pf_launch_fmt<QT_Q6_K, QT_Q6_K>(a, p.bm, p.bn, p.s, st);
   if (qt0 == QT_Q4_K && qt1 == QT_Q6_K) return pf_launch_fmt<QT_Q4_K, QT_Q6_K>(a, p.bm, p.bn, p.s, st);
@@ -192,6 +195,7 @@ static bool pf_run(const GemmQArgs& a, const PfPlan& p, hipStream_t st) {
   if (qt0 == QT_Q5_K && qt1 == QT_Q6_K) return pf_launch_fmt<QT_Q5_K, QT_Q6_K>(a, p.bm, p.bn, p.s, st);
   if (qt0 == QT_Q4_0 && qt1 == QT_Q4_0) return pf_launch_fmt<QT_Q4_0, QT_Q4_0>(a, p.bm, p.bn, p.s, st);
   if (qt0 == QT_Q8_0 && qt1 == QT_Q8_0) return pf_launch_fmt<QT_Q8_0, QT_Q8_0>(a, p.bm, p.bn, p.s, st);
+#endif
   if (qt0 != QT_BF16) return false;
   return pf_launch_fmt<QT_BF16, QT_BF16>(a, p.bm, p.bn, p.s, st);
 }

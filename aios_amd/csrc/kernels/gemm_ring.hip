@@ -366,6 +366,9 @@ bool launch_gemm_ring(const GemmQArgs& a, hipStream_t st) {
   const int qt0 = a.seg[0].qtype, qt1 = a.seg[a.nseg - 1].qtype;
   for (int s = 0; s + 1 < a.nseg; ++s)
     if (a.seg[s].qtype != qt0) return false;
+#ifdef AIOS_BF16_ONLY
+  return false;
+#else
   auto go = [&](auto mt, auto xr) {
     constexpr int MT = decltype(mt)::value;
     constexpr bool XR = decltype(xr)::value;
@@ -380,6 +383,7 @@ bool launch_gemm_ring(const GemmQArgs& a, hipStream_t st) {
   if (a.M <= RG_XR_ROWS && xr_on && go(std::integral_constant<int, 1>{}, std::true_type{})) return true;
   if (a.M <= 16) return go(std::integral_constant<int, 1>{}, std::false_type{});
   return go(std::integral_constant<int, 2>{}, std::false_type{});
+#endif
 }
 
 }  // namespace aios

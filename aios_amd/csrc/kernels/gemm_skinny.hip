@@ -388,6 +388,9 @@ bool launch_gemm_skinny(const GemmQArgs& a, hipStream_t st) {
   if (!sk_fits(a)) return false;
   bool same = true;
   for (int s = 1; s < a.nseg; ++s) same &= a.seg[s].qtype == a.seg[0].qtype;
+#ifdef AIOS_BF16_ONLY
+  return same && a.seg[0].qtype == QT_BF16 && sk_qt<QT_BF16, QT_BF16>(a, st);
+#else
   if (!same) return gemm_skinny_mixed_ok(a) && sk_qt<QT_Q4_K, QT_Q6_K>(a, st);
   switch (a.seg[0].qtype) {
     case QT_Q4_K: return sk_qt<QT_Q4_K, QT_Q4_K>(a, st);
@@ -399,6 +402,7 @@ bool launch_gemm_skinny(const GemmQArgs& a, hipStream_t st) {
     case QT_BF16: return sk_qt<QT_BF16, QT_BF16>(a, st);
     default: return false;
   }
+#endif
 }
 
 }  // namespace aios

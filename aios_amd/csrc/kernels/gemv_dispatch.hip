@@ -1,4 +1,5 @@
-// Host dispatcher: (segment-0 format, last-segment format) -> kernel instantiation.
+// Host dispatcher: (segment-0 format, last-segment format) -> kernel instantiation.  AIOS_BF16_ONLY builds
+// hold the bf16 kernels alone (folder checkpoints: _build.build(formats="bf16")).
 #include <stdexcept>
 #include <string>
 
@@ -29,6 +30,7 @@ bool gemv_q8_0_engine_fits(const GemvArgs&);
 bool gemv_engine_fits(const GemvArgs& a) {
   const int qt0 = a.seg[0].qtype, qt1 = a.seg[a.nseg - 1].qtype;
   if (qt0 == QT_F16 || qt0 == QT_BF16) return true;
+#ifndef AIOS_BF16_ONLY
   if (qt0 == qt1) {
     switch (qt0) {
       case QT_Q4_K: return gemv_q4k_q4k_engine_fits(a);
@@ -41,6 +43,7 @@ bool gemv_engine_fits(const GemvArgs& a) {
     if (qt0 == QT_Q4_K) return gemv_q4k_q6k_engine_fits(a);
     if (qt0 == QT_Q5_K) return gemv_q5k_q6k_engine_fits(a);
   }
+#endif
   return false;
 }
 
@@ -55,6 +58,7 @@ bool gemv_tpf_q8_0(const GemvArgs&, hipStream_t);
 // plain GEMV and a separate all-reduce
 bool launch_gemv_tp_fused(const GemvArgs& a, hipStream_t st) {
   if (a.nseg != 1 || a.epi != EPI_TP_RESID) return false;
+#ifndef AIOS_BF16_ONLY
   switch (a.seg[0].qtype) {
     case QT_Q4_K: return gemv_tpf_q4k(a, st);
     case QT_Q6_K: return gemv_tpf_q6k(a, st);
@@ -62,6 +66,7 @@ bool launch_gemv_tp_fused(const GemvArgs& a, hipStream_t st) {
     case QT_Q4_0: return gemv_tpf_q4_0(a, st);
     case QT_Q8_0: return gemv_tpf_q8_0(a, st);
   }
+#endif
   return false;
 }
 
@@ -84,6 +89,9 @@ void launch_gemv(const GemvArgs& a, hipStream_t st) {
   }
   if (a.N % 2) throw std::runtime_error("gemv: N must be even");
   if (a.K % 16) throw std::runtime_error("gemv: K must be a multiple of 16");
+#ifdef AIOS_BF16_ONLY
+  if (qt0 == QT_BF16 && qt1 == QT_BF16) return gemv_bf16(a, st);
+#else
   if (qt0 == qt1) {
     switch (qt0) {
       case QT_Q4_K: return gemv_q4k_q4k(a, st);
@@ -98,6 +106,7 @@ void launch_gemv(const GemvArgs& a, hipStream_t st) {
     if (qt0 == QT_Q4_K) return gemv_q4k_q6k(a, st);
     if (qt0 == QT_Q5_K) return gemv_q5k_q6k(a, st);
   }
+#endif
   throw std::runtime_error("gemv: unsupported format pair " + std::to_string(qt0) + "/" + std::to_string(qt1));
 }
 }  // namespace aios

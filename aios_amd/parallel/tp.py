@@ -424,13 +424,18 @@ def env_rank_world():
 
 
 # ------------------------------------------------------------------------------ runtime launcher
-def spec_kv_dtype(path: str) -> str:
-    """the '#...&kv=fp8_e4m3' fragment of a model spec (default: AIOS_KV_DTYPE, else bf16)"""
+def spec_option(path: str, key: str, default: str) -> str:
+    """the value of '#...&key=value' in a model spec"""
     for kv in filter(None, path.partition("#")[2].split("&")):
         k, _, v = kv.partition("=")
-        if k == "kv":
+        if k == key:
             return v
-    return os.environ.get("AIOS_KV_DTYPE", "bf16")
+    return default
+
+
+def spec_kv_dtype(path: str) -> str:
+    """the '#...&kv=fp8_e4m3' fragment of a model spec (default: AIOS_KV_DTYPE, else bf16)"""
+    return spec_option(path, "kv", os.environ.get("AIOS_KV_DTYPE", "bf16"))
 
 
 def parse_spec(path: str):

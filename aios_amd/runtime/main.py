@@ -2,7 +2,8 @@
 
 * builds the ModelManager on the local MI355X,
 * auto-loads every `*.gguf` in $AIOS_MODEL_DIR (default /var/lib/aios/models/) with the
-  reference's size-based context heuristic, plus `AIOS_SYNTHETIC_MODELS` entries
+  reference's size-based context heuristic, every folder checkpoint there (config.json +
+  model.safetensors of a registered architecture, models/registry.py), plus `AIOS_SYNTHETIC_MODELS` entries
   (`name=synthetic:preset[:recipe]`, comma separated),
 * serves aios.runtime.AIRuntime on [::]:50055 (AIOS_RUNTIME_ADDR), with a 10 s health loop
   that marks models whose engine died as errored.
@@ -16,6 +17,7 @@ import os
 import signal
 from pathlib import Path
 
+from ..models import registry
 from ..rpc.client import Stub, channel
 from ..rpc.schema import pb
 from ..rpc.server import RpcServer
@@ -54,6 +56,13 @@ async def auto_load(svc: AIRuntimeService, model_dir: str, cfg=None):
             req_name = f.stem
             log.info("auto-loading %s", f)
             m = await svc.mgr.load_model(req_name, str(f))
+            if m.status == "ready" and svc.http:
+                await svc.start_http(m)
+        for f in sorted(p for p in d.iterdir() if p.is_dir() and registry.is_checkpoint_dir(str(p))):
+            if str(f) in loaded:
+                continue
+            log.info("auto-loading %s", f)
+            m = await svc.mgr.load_model(f.name, str(f))
             if m.status == "ready" and svc.http:
                 await svc.start_http(m)
     for spec in filter(None, os.environ.get("AIOS_SYNTHETIC_MODELS", "").split(",")):

@@ -14,8 +14,10 @@ processes: each model is an in-process native Engine + tokenizer + chat template
   * replicas: one tier may run as several engines on different GPUs of the node (request-level
     data parallelism, SURVEY §2.9 DP row); routing picks the least-loaded ready replica.
 
-Model paths: a GGUF file, or `synthetic:<preset>[:<recipe>]` for a random-init model of a named
-architecture (tests/benchmarks without network access).
+Model paths: a GGUF file, a folder checkpoint of a registered architecture (config.json +
+model.safetensors, models/registry.py), or `synthetic:<preset>[:<recipe>]` for a random-init model of a
+named architecture (tests/benchmarks without network access).  Options follow a '#', joined by '&':
+`tp=N`, `cpu`, `kv=fp8`, `compute=float32` (layered models), `kv_tokens=N` (size of the cache pool).
 """
 from __future__ import annotations
 
@@ -114,6 +116,19 @@ def tier_context(cfg, path: str = "") -> int:
     return min(cfg.max_ctx, context_for_size(nbytes))
 
 
+def synthetic_tokenizer(cfg):
+    """(tokenizer, chat template) of a model without a tokenizer of its own: exactly cfg.vocab_size tokens
+    of the synthetic vocabulary."""
+    from ..models.synthetic import synthetic_vocab
+    from . import chat_template
+    from .tokenizer import SpmTokenizer
+
+    n = cfg.vocab_size
+    toks, scores, types = (v[:n] for v in synthetic_vocab(n))
+    tok = SpmTokenizer(toks, scores, types, cfg.bos_id, cfg.eos_id)
+    return tok, chat_template.for_model(cfg.chat_template if cfg.chat_template in chat_template.BUILTIN else "zephyr", tok)
+
+
 class ModelManager:
     def __init__(self, device: int = 0, max_batch: int = 16, max_slots: int = 16, base_port: int = BASE_PORT):
         self.device = device
@@ -187,12 +202,14 @@ class ModelManager:
         from .tokenizer import SpmTokenizer, from_gguf
 
         E = native.require()
-        from ..parallel.tp import launch_tp, parse_spec, spec_kv_dtype
+        from ..parallel.tp import launch_tp, parse_spec, spec_kv_dtype, spec_option
 
         device = self.device if m.device < 0 else m.device
 
         base, tp, act_q8 = parse_spec(m.path)
         kv_dtype = spec_kv_dtype(m.path)
+        compute = spec_option(m.path, "compute", "bf16")
+        kv_pool = int(spec_option(m.path, "kv_tokens", "0"))
         faults = FaultSpec.from_env(m.name)
         if faults is not None:
             faults.check("load")
@@ -226,19 +243,21 @@ class ModelManager:
             ctx = context_length or tier_context(cfg)
             eng = random_engine(cfg, recipe, seed=_synth_seed(m.group or m.name), max_ctx=ctx,
                                 max_slots=self.max_slots, max_batch=self.max_batch, device=device, act_q8=act_q8,
-                                kv_dtype=kv_dtype)
-            toks, scores, types = synthetic_vocab(cfg.vocab_size)
-            tok = SpmTokenizer(toks, scores, types, cfg.bos_id, cfg.eos_id)
-            tmpl = chat_template.for_model(cfg.chat_template if cfg.chat_template in chat_template.BUILTIN else "zephyr",
-                                           tok)
+                                kv_dtype=kv_dtype, compute=compute, kv_pool_tokens=kv_pool)
+            tok, tmpl = synthetic_tokenizer(cfg)
         else:
             if not os.path.exists(base):
                 raise FileNotFoundError(base)
-            ctx = context_length or context_for_size(os.path.getsize(base))
+            # (a folder checkpoint without an explicit context: the model's own position range)
+            ctx = context_length or (None if os.path.isdir(base) else context_for_size(os.path.getsize(base)))
             eng, cfg, reader = load_engine(base, max_ctx=ctx, max_slots=self.max_slots, max_batch=self.max_batch,
-                                           device=device, name=m.name, act_q8=act_q8, kv_dtype=kv_dtype)
-            tok = from_gguf(reader)
-            tmpl = chat_template.for_model(reader, tok)
+                                           device=device, name=m.name, act_q8=act_q8, kv_dtype=kv_dtype,
+                                           compute=compute, kv_pool_tokens=kv_pool)
+            if os.path.isdir(base):
+                tok, tmpl = synthetic_tokenizer(cfg)  # (these checkpoints carry no tokenizer)
+            else:
+                tok = from_gguf(reader)
+                tmpl = chat_template.for_model(reader, tok)
         if not cpu:
             m.engine, m.config, m.tokenizer, m.template = eng, cfg, tok, tmpl
         if faults is not None:
@@ -363,6 +382,8 @@ class ModelManager:
         from .tokenizer import SpmTokenizer, from_gguf
 
         slots = min(self.max_slots, 4)
+        if os.path.isdir(base) or (base.startswith("synthetic:") and get_preset(base.split(":")[1]).layers):
+            raise RuntimeError(f"{m.name}: layered models run on the GPU only")
         if base.startswith("synthetic:"):
             parts = base.split(":")
             cfg = get_preset(parts[1])

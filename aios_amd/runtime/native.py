@@ -17,7 +17,9 @@ _mod = None
 _err: Optional[BaseException] = None
 
 
-def load(build_if_missing: bool = True):
+def load(build_if_missing: bool = True, formats: str = "all"):
+    """The extension with the kernels of every weight format; formats="bf16": also the smaller build of the
+    bf16 kernels alone, which is what is compiled then if neither is there."""
     global _mod, _err
     if _mod is not None:
         return _mod
@@ -25,17 +27,19 @@ def load(build_if_missing: bool = True):
         import torch  # noqa: F401  (see module docstring)
     except Exception:  # pragma: no cover - torch is present in this image
         pass
-    try:
-        _mod = importlib.import_module("aios_amd._engine")
-        return _mod
-    except ImportError as e:
-        _err = e
+    names = ["_engine"] + (["_engine_bf16"] if formats == "bf16" else [])
+    for n in names:
+        try:
+            _mod = importlib.import_module("aios_amd." + n)
+            return _mod
+        except ImportError as e:
+            _err = e
     if build_if_missing and os.environ.get("AIOS_NO_AUTOBUILD") != "1":
         from .. import _build
 
-        _build.build(verbose=False)
+        _build.build(verbose=False, formats=formats)
         importlib.invalidate_caches()
-        _mod = importlib.import_module("aios_amd._engine")
+        _mod = importlib.import_module("aios_amd." + names[-1])
         return _mod
     raise ImportError(f"aios_amd native engine not built: {_err}")
 
@@ -59,7 +63,7 @@ def gpu_available() -> bool:
 
 def require(formats: str = "all"):
     """The native engine, loudly: on a GPU box a missing extension is an error."""
-    return load(build_if_missing=True)
+    return load(build_if_missing=True, formats=formats)
 
 
 KV_DTYPES = ("bf16", "fp8", "fp8_e4m3")

@@ -12,6 +12,10 @@ with an in-process worker per model that owns the native Engine:
   prefilled AIOS_PREFILL_CHUNK tokens (default 512) per scheduler iteration between batched
   decode steps, so a 3k-token admission does not stall every running stream for its whole
   prefill; with nothing decoding the prompt goes through in one call;
+* engines that run mixed batches (Engine.mixed_steps) take the prompt chunks of several admitted
+  sequences and the decode token of every running one in ONE step instead of alternating the two;
+* a cache pool smaller than every slot's full context (kv_pool_tokens) admits a request only when its
+  blocks are certain to be available, and takes cached prefixes of idle slots back for it;
 * each iteration runs ONE batched decode step (hipGraph replay) for every decoding sequence, so
   concurrent agents/reasoning loops share each weight pass;
 * JSON mode (the reference's `response_format: json_object`) builds the allowed-token mask per
@@ -123,6 +127,12 @@ class Scheduler:
         self.timing = dict(mask_s=0.0, engine_decode_s=0.0, accept_s=0.0, prefill_s=0.0)
         self.step_log: Deque = collections.deque(maxlen=4096)  # (end time, batch) per decode step
         self.share_prefix = hasattr(engine, "copy_slot")
+        self.mixed = bool(getattr(engine, "mixed_steps", False))
+        # a pool that cannot hold every slot's full context: blocks are reserved per request
+        self.kv_block = int(getattr(engine, "kv_block_tokens", 0) or 0)
+        self.kv_total = int(getattr(engine, "kv_blocks_total", 0) or 0)
+        self.kv_limited = self.kv_block > 0 and self.kv_total < max_slots * -(-max_ctx // self.kv_block)
+        self.kv_reserved: Dict[int, int] = {}  # slot -> blocks its running request may use
         self.min_shared_prefix = int(os.environ.get("AIOS_MIN_SHARED_PREFIX", "128"))
         self.cv = threading.Condition()
         self.stop_flag = False
@@ -174,8 +184,9 @@ class Scheduler:
                         self._done(r, GenResult("", [], len(r.prompt_ids), 0, "cancelled"))
                     return
                 admit = []
-                while (self.queue and self.free_slots and
-                       len(self.active) + len(self.prefilling) + len(admit) < self.max_batch):
+                while (self.queue and len(self.free_slots) > len(admit) and
+                       len(self.active) + len(self.prefilling) + len(admit) < self.max_batch and
+                       self._kv_fits(self.queue[0], admit)):
                     admit.append(self.queue.popleft())
             if admit or self.prefilling:
                 self._drain()  # (no other engine call while a pipelined step is in flight)
@@ -189,6 +200,18 @@ class Scheduler:
                     log.exception("admission failed")
                     self._engine_failed(e)
                     self._done(r, GenResult("", [], len(r.prompt_ids), 0, "error", error=str(e)))
+            if self.mixed and self.prefilling and self.active:
+                try:
+                    t0 = time.time()
+                    self._mixed_step()
+                    self.last_progress = time.time()
+                    self._step_ms.append((self.last_progress - t0) * 1e3)
+                except Exception as e:  # noqa: BLE001
+                    log.exception("mixed step failed")
+                    self._engine_failed(e)
+                    for s in list(self.active) + list(self.prefilling):
+                        self._finish(s, "error", str(e))
+                continue
             if self.prefilling:
                 seq = self.prefilling[0]
                 try:
@@ -212,6 +235,36 @@ class Scheduler:
                     self._pending = None
                     for s in list(self.active):
                         self._finish(s, "error", str(e))
+
+    # ------------------------------------------------------------------ limited cache pool
+    def _kv_need(self, r: GenRequest) -> int:
+        """Blocks a request may come to use: its prompt, every token it may generate, and the position a
+        pipelined step writes ahead."""
+        n = min(len(r.prompt_ids) + max(1, r.max_tokens) + 1, self.max_ctx)
+        return -(-n // self.kv_block)
+
+    def _kv_fits(self, r: GenRequest, admitted: List[GenRequest]) -> bool:
+        if not self.kv_limited:
+            return True
+        need = self._kv_need(r)
+        if need > self.kv_total:
+            return True  # (never fits: _admit reports it)
+        return need + sum(self.kv_reserved.values()) + sum(self._kv_need(a) for a in admitted) <= self.kv_total
+
+    def _kv_reserve(self, slot: int, need: int):
+        """Reserve `need` blocks for the request entering `slot`; cached prefixes of idle slots give way
+        until the pool's free blocks cover everything the running requests may still map."""
+        self.kv_reserved[slot] = need
+        held = set()
+        for s in self.kv_reserved:
+            held.update(b for b in self.engine.block_table(s) if b >= 0)
+        idle = [s for s in self.free_slots if s not in self.kv_reserved]
+        idle.sort(key=lambda s: len(self.slot_cache[s]))
+        for s in idle:
+            if self.engine.kv_blocks_free >= sum(self.kv_reserved.values()) - len(held):
+                break
+            self.engine.release_slot(s)
+            self.slot_cache[s] = []
 
     @staticmethod
     def _common(c: List[int], ids: List[int]) -> int:
@@ -251,8 +304,13 @@ class Scheduler:
             raise ValueError(f"prompt of {len(ids)} tokens exceeds the context window ({self.max_ctx})")
         r.max_tokens = max(1, min(r.max_tokens, self.max_ctx - len(ids)))
         r.min_tokens = min(r.min_tokens, r.max_tokens)
+        if self.kv_limited and self._kv_need(r) > self.kv_total:
+            raise ValueError(f"request of {len(ids)} + {r.max_tokens} tokens exceeds the cache pool "
+                             f"({self.kv_total * self.kv_block} tokens)")
         slot, common = self._pick_slot(ids)
         self.free_slots.remove(slot)
+        if self.kv_limited:
+            self._kv_reserve(slot, self._kv_need(r))
         seq = _Seq(r, slot)
         seq.cached = common
         seq.pos = common
@@ -267,6 +325,7 @@ class Scheduler:
                 if seq in self.prefilling:  # the caller reports the error; the slot goes back
                     self.prefilling.remove(seq)
                     self.free_slots.append(slot)
+                    self.kv_reserved.pop(slot, None)
                 raise
 
     def _prefill_chunk(self, seq: _Seq, whole: bool = False):
@@ -288,7 +347,6 @@ class Scheduler:
         self.stats["prefill_tokens"] += n
         if not last:
             return
-        self.prefilling.remove(seq)
         mask = None
         if r.json_mode and self.grammar is not None:
             seq.grammar_state = self.grammar.initial()
@@ -302,9 +360,60 @@ class Scheduler:
         else:
             rng = np.random.default_rng([seq.seed & 0xFFFFFFFF, seq.pos - 1])
             tok = host_sampler.sample(logits, r.temperature, r.top_k, r.top_p, mask, rng)
+        self._begin_decode(seq, tok)
+
+    def _begin_decode(self, seq: _Seq, tok: int):
+        """seq's prompt is in the cache and its first token sampled: it joins the decoding set."""
+        self.prefilling.remove(seq)
         seq.t_first = time.time()
         self.active.append(seq)
         self._accept(seq, tok)
+
+    def _mixed_step(self):
+        """One engine step with the next prompt chunks (prefill_chunk tokens in all) of the admitted
+        sequences and one decode token of every running one; samples every row that has a next token."""
+        t0 = time.perf_counter()
+        rows = list(self.active)
+        chunks, budget = [], max(1, self.prefill_chunk)
+        for seq in list(self.prefilling):
+            if seq.req.cancelled:
+                self._finish(seq, "cancelled")
+                continue
+            n = min(len(seq.todo), budget)
+            if n == 0:
+                break
+            budget -= n
+            chunks.append((seq, n))
+        done = [seq for seq, n in chunks if n == len(seq.todo)]  # prompts this step completes
+        for seq in done:
+            if seq.req.json_mode and self.grammar is not None:
+                seq.grammar_state = self.grammar.initial()
+        sampled = rows + done
+        tokens: List[int] = [s.last for s in rows]
+        for seq, n in chunks:
+            tokens.extend(seq.todo[:n])
+        mask = self._masks(sampled)
+        t1 = time.perf_counter()
+        out = self.engine.step_sample(
+            [s.slot for s in rows] + [s.slot for s, _ in chunks], [s.pos for s in rows] + [s.pos for s, _ in chunks],
+            [1] * len(rows) + [n for _, n in chunks], tokens,
+            [1] * len(rows) + [int(n == len(s.todo)) for s, n in chunks],
+            [float(s.req.temperature) for s in sampled],
+            [int(s.req.top_k) if s.req.temperature > 0 else 0 for s in sampled],
+            [float(s.req.top_p) if 0.0 < s.req.top_p < 1.0 else 1.0 for s in sampled], [s.seed for s in sampled], mask)
+        t2 = time.perf_counter()
+        self.timing["mask_s"] += t1 - t0
+        self.timing["prefill_s" if not rows else "engine_decode_s"] += t2 - t1
+        self.step_log.append((t2, len(rows)))
+        for seq, n in chunks:
+            chunk, seq.todo = seq.todo[:n], seq.todo[n:]
+            seq.pos += n
+            self.slot_cache[seq.slot].extend(chunk)
+            self.stats["prefill_tokens"] += n
+        if rows:
+            self._take(rows, out[:len(rows)])
+        for seq, tok in zip(done, out[len(rows):]):
+            self._begin_decode(seq, int(tok))
 
     def _accept(self, seq: _Seq, tok: int) -> bool:
         """Record a sampled token; returns False when the sequence finished."""
@@ -506,6 +615,7 @@ class Scheduler:
         if seq in self.prefilling:
             self.prefilling.remove(seq)
         self.free_slots.append(seq.slot)
+        self.kv_reserved.pop(seq.slot, None)
         r = seq.req
         text = self.tok.decode(seq.out)
         if r.on_delta is not None and len(text) > len(seq.emitted) and text.startswith(seq.emitted):

@@ -39,7 +39,7 @@ HOT = [
 
 def _engine_so():
     for f in sorted(os.listdir(SO)):
-        if f.startswith("_engine") and f.endswith(".so"):
+        if f.startswith("_engine.") and f.endswith(".so"):
             return os.path.join(SO, f)
     raise FileNotFoundError("no built engine under aios_amd/ (run __graft_entry__.build())")
 
