@@ -102,7 +102,7 @@ def test_oracle_mechanisms_by_hand():
 @pytest.mark.parametrize("fault", ["no sink", "no gate", "no position", "position off by one", "one key short",
                                    "sequential layer", "silu", "no latent norm", "own weights", "scale"])
 def test_a_fault_in_any_mechanism_shows(fault, monkeypatch):
-    """Planted in the oracle: the logits move by far more than the GPU tests' tolerances (2e-2 in bf16)."""
+    """Planted in the oracle: the logits move by far more than the GPU tests' tolerances (3e-2 in bf16)."""
     cfg = MIXED
     w = O.random_weights(cfg, 1, qk_gain=2.0)
     ids = [int(t) for t in np.random.default_rng(1).integers(0, 211, 40)]
