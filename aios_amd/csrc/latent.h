@@ -8,14 +8,14 @@
 //   expanded  k and v of the whole context are computed once per call and a flash attention runs on
 //             them: fewer operations per (query, key) pair, for long portions of a prompt.
 // Every head dimension is padded with zeros: dkp / dvp (query-key / value) to multiples of 32, the
-// rank to rp, a multiple of 64, so the kernels have no ragged dimension.
+// rank to rp, a multiple of 128, so the kernels have no ragged dimension.
 #pragma once
 #include "ops.h"
 
 namespace aios {
 
-// 16 query rows (a row = one head of one token) of one sequence: flat rows [f0, f0 + nv), nv <= 16, of
-// the flattened [token][head] row space
+// query rows (a row = one head of one token) of one sequence: flat rows [f0, f0 + nv) of the flattened
+// [token][head] row space, nv <= 16
 struct LatentTile {
   int f0, nv;
 };
@@ -51,7 +51,6 @@ void launch_latent_attn(const LatentAttnArgs& a, hipStream_t st);
 // partial sums -> softmax normalisation with the sink, Wuv, output gate
 void launch_latent_out(const LatentAttnArgs& a, hipStream_t st);
 bool latent_attn_mfma(int rp);  // the matrix-core kernels serve this padded rank (else the plain one, rank <= 2048)
-int latent_tiles_per_token(int H);
 
 // the first S cached vectors of a slot, contiguous: out [S][rp] (bf16 cache)
 void launch_latent_gather(const bf16_t* pool, const int* bt, int maxb, int kvb, int slot, int S, int rp, bf16_t* out,

@@ -83,7 +83,7 @@ class LayeredDecoder {
     const int *tokens, *pos, *slot;
     int n, n_abs;                         // rows, rows on the absorbed path (they come first)
     bool decode;
-    std::map<int, std::pair<int, int>> tiles;  // heads -> (first tile, count), step batches
+    std::map<int, std::pair<int, int>> tiles;  // step batches: heads -> (first tile, count)
     int max_len;                          // of the absorbed rows
     std::vector<std::pair<int, Piece>> pf;  // expanded path: first row, piece
   };

@@ -26,7 +26,7 @@ static int env_or(const char* name, int dflt) {
 }
 // padded latent widths the attention kernels are built for
 static int pad_rank(int r) {
-  for (int t : {1, 2, 3, 4, 6, 8, 12, 16, 32})
+  for (int t : {2, 4, 6, 8, 12, 16, 32})
     if (r <= 64 * t) return 64 * t;
   throw std::runtime_error("latent attention: kv_rank above 2048");
 }
@@ -343,7 +343,7 @@ void LayeredDecoder::finalize() {
   std::set<int> hs;
   for (const Dims& D : dims_) hs.insert(D.H);
   size_t tiles = 0;
-  for (int h : hs) tiles += (size_t)R * latent_tiles_per_token(h) + R;
+  for (int h : hs) tiles += (size_t)R * ((h + 15) / 16) + R;
   step_ints_ = (size_t)4 * R + 2 * tiles;
   HIP_CHECK(hipHostMalloc((void**)&h_step_, step_ints_ * 4, hipHostMallocDefault));
   d_step_ = (int*)falloc(step_ints_);
@@ -416,11 +416,12 @@ void LayeredDecoder::gemm16(const bf16_t* A, int lda, const bf16_t* w, int M, in
   e_.gemm(g);
 }
 
-// key splits of an absorbed attention launch: about two workgroups per CU, at least one 64-key tile each;
-// tiles x splits stays below tiles + 512, which bounds the partial sums' buffer
+// key splits of an absorbed attention launch: one round of workgroups (two per CU), at least two 32-key tiles
+// each (one for a token or two); rows x splits stays below rows + 16 x 512, which bounds the partial sums' buffer
 int LayeredDecoder::key_split(int tiles, int max_len) const {
   const int want = (512 + tiles - 1) / std::max(tiles, 1);
-  return std::max(1, std::min({want, (max_len + 63) / 64, 64}));
+  const int keys = tiles <= 4 ? 32 : 64;
+  return std::max(1, std::min({want, (max_len + keys - 1) / keys, max_len <= 4096 ? 32 : 64}));
 }
 
 LatentAttnArgs LayeredDecoder::latent_args(int i, const RowSet& r) {
@@ -443,7 +444,7 @@ LatentAttnArgs LayeredDecoder::latent_args(int i, const RowSet& r) {
   a.wuv = w.ukv + (size_t)D.qn * D.rp;
   a.qa = qa_;
   if (r.decode) {
-    a.n_tiles = r.n * latent_tiles_per_token(D.H);
+    a.n_tiles = r.n * ((D.H + 15) / 16);
   } else {
     const auto t = r.tiles.at(D.H);
     a.tiles = st_tiles_ + t.first;

@@ -92,7 +92,7 @@ def test_latent_attention_kernel(H, dk, dv, rank, sink, gate, f32):
     g = torch.Generator().manual_seed(H * 1000 + rank)
     rnd = lambda *s: torch.randn(*s, generator=g)
     dkp, dvp = pad(dk, 32), pad(dv, 32)
-    rp = next(64 * t for t in (1, 2, 3, 4, 6, 8, 12, 16, 32) if rank <= 64 * t)
+    rp = next(64 * t for t in (2, 4, 6, 8, 12, 16, 32) if rank <= 64 * t)
     lens, portion, kvb, maxb = [1, 64, 65, 200], 7, 64, 6
     seqs = [(i, l - 1, 1) for i, l in enumerate(lens)] + [(4, 122, portion)]  # slot, start, new tokens
     n = sum(s[2] for s in seqs)
