@@ -60,6 +60,10 @@ def parse():
                     help="skip the goal->plan latency secondary (BASELINE.json's agent metric)")
     ap.add_argument("--tp-model", default="llama3-70b")
     ap.add_argument("--tp-steps", type=int, default=64)
+    ap.add_argument("--design", default="", choices=("", "gefazen"),
+                    help="instead of the headline: prefill and decode throughput of this design at the sizes of two real "
+                         "models' layers (random weights), beside the llama-family model of equal size with bf16 weights; "
+                         "one JSON line per measurement, one GPU")
     ap.add_argument("--dry-run", action="store_true",
                     help="launcher check: set up the ranks and their process group, print one line per rank, "
                          "touch no GPU")
@@ -116,6 +120,72 @@ def measure(preset: str, recipe: str, batch: int, prompt: int, steps: int, warmu
                 workspace_gb=round(eng.workspace_bytes / 1e9, 3))
     del eng
     return dt, info
+
+
+# --design: (preset of the design, llama-family preset of equal width, depth, heads and MLP)
+DESIGN_PAIRS = {"gefazen": (("gefazen-1b", "tinyllama-1.1b"), ("gefazen-7b", "mistral-7b"))}
+DESIGN_DECODE = ((1, 128), (1, 2048), (4, 2048), (16, 1024), (32, 1024))   # (sequences, context)
+DESIGN_PREFILL = (128, 512, 2048)
+
+
+def measure_design(args):
+    """Both sides of every pair in turn, three rounds, medians: captured greedy decode of `steps` tokens, and
+    whole prompts through Engine.prefill."""
+    import statistics
+
+    from aios_amd.models.config import get_preset
+    from aios_amd.runtime.loader import random_engine
+
+    steps, warmup, rounds = min(args.steps, 64), min(args.warmup, 8), 3
+
+    def prompt(cfg, n, s=0):
+        return [(7 * i + 13 * s) % (cfg.vocab_size - 3) + 3 for i in range(n)]
+
+    def engines(pair, batch, ctx):
+        for p in pair:
+            cfg = get_preset(p)
+            yield cfg, random_engine(cfg, "BF16", seed=1234, max_ctx=(ctx + rounds * (warmup + steps) + 127) // 128 * 128,
+                                     max_slots=batch, max_batch=batch)
+
+    def report(pair, what, batch, ctx, unit, rate, ms):
+        d = {"bench": f"{what} {pair[0]} beside {pair[1]}", "batch": batch, "context": ctx, "unit": unit, "dtype": "bf16",
+             "data": "synthetic (random-init bf16 weights)"}
+        for p, r, m in zip(pair, rate, ms):
+            d[p] = {"value": round(r, 1), "ms": round(m, 3)}
+        d["ratio"] = round(rate[0] / rate[1], 3)
+        print(json.dumps(d), flush=True)
+
+    for pair in DESIGN_PAIRS[args.design]:
+        for batch, ctx in DESIGN_DECODE:
+            side = list(engines(pair, batch, ctx))
+            dts = [[], []]
+            for cfg, eng in side:
+                for s in range(batch):
+                    eng.prefill(s, prompt(cfg, ctx, s), 0, False)
+                eng.decode_loop_prepare(list(range(batch)), [5] * batch, [ctx] * batch)
+            for _ in range(rounds):
+                for i, (cfg, eng) in enumerate(side):
+                    eng.decode_loop_run(batch, warmup, True)
+                    eng.synchronize()
+                    t0 = time.perf_counter()
+                    eng.decode_loop_run(batch, steps, True)
+                    eng.synchronize()
+                    dts[i].append((time.perf_counter() - t0) / steps)
+            dt = [statistics.median(x) for x in dts]
+            report(pair, "decode", batch, ctx, "tokens/s", [batch / x for x in dt], [x * 1e3 for x in dt])
+            del side, eng
+        side = list(engines(pair, 1, max(DESIGN_PREFILL)))
+        for n in DESIGN_PREFILL:
+            dts = [[], []]
+            for r in range(rounds + 1):
+                for i, (cfg, eng) in enumerate(side):
+                    t0 = time.perf_counter()
+                    eng.prefill(0, prompt(cfg, n), 0, True)
+                    if r:
+                        dts[i].append(time.perf_counter() - t0)
+            dt = [statistics.median(x) for x in dts]
+            report(pair, "prefill", 1, n, "tokens/s", [n / x for x in dt], [x * 1e3 for x in dt])
+        del side, eng
 
 
 def measure_goal_plan(goals: int = 16, timeout_s: float = 90.0):
@@ -261,6 +331,11 @@ def main():
         print(json.dumps({"rank": rank, "world": world, "device": device, "ranks_share_gpu": share}), flush=True)
         return
     torch.cuda.set_device(device)
+    if args.design:
+        if world > 1:
+            raise SystemExit("bench.py: --design measures one GPU")
+        measure_design(args)
+        return
     if world > 1:
         import torch.distributed as td
 

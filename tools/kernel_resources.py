@@ -34,6 +34,10 @@ HOT = [
     "aios::gemm_ring_kernel<*",
     "aios::sample_kernel*",
     "aios::get_rows_step_kernel*",
+    "aios::latent_prep_kernel*",
+    "aios::latent_attn_kernel<*",
+    "aios::latent_combine_kernel*",
+    "aios::latent_out_kernel<*",
 ]
 
 
