@@ -1,6 +1,7 @@
 """Gefazen on the CPU: configuration, registry, checkpoint reader, trace replay bookkeeping, the scheduler's
 mixed steps and limited cache pool (fake engine), and the oracle the GPU tests compare against -- including
 that each mechanism, left out or shifted by one, would show in the logits those tests look at."""
+import asyncio
 import json
 import math
 import threading
@@ -290,3 +291,11 @@ def test_scheduler_limited_pool_waits_evicts_and_rejects():
         assert r.token_ids == expected([4] * 20, 5)
     finally:
         sched.close()
+
+
+def test_cpu_backend_refuses_layered_models(tmp_path):
+    from aios_amd.runtime.model_manager import ModelManager
+
+    folder = write_model(tmp_path / "m", MIXED, O.random_weights(MIXED))
+    m = asyncio.run(ModelManager(max_batch=2, max_slots=2).load_model("gefazen-cpu", folder + "#cpu"))
+    assert m.status == "error" and "GPU only" in m.error
