@@ -144,6 +144,11 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.attr("MIX_LATENT") = (int)MIX_LATENT;
   m.attr("MLP_NONE") = (int)MLP_NONE;
   m.attr("MLP_GLU") = (int)MLP_GLU;
+  m.attr("MLP_MOE") = (int)MLP_MOE;
+  m.attr("MIX_MINGRU") = (int)MIX_MINGRU;
+  m.attr("GATE_NONE") = (int)GATE_NONE;
+  m.attr("GATE_ELEMENT") = (int)GATE_ELEMENT;
+  m.attr("GATE_HEAD") = (int)GATE_HEAD;
   m.attr("ACT_SILU") = (int)ACT_SILU;
   m.attr("ACT_GELU_TANH") = (int)ACT_GELU_TANH;
   py::class_<LayerSpec>(m, "LayerSpec")
@@ -159,6 +164,20 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       .def_readwrite("mlp", &LayerSpec::mlp)
       .def_readwrite("ff", &LayerSpec::ff)
       .def_readwrite("act", &LayerSpec::act)
+      .def_readwrite("parallel", &LayerSpec::parallel)
+      .def_readwrite("norm_scalar", &LayerSpec::norm_scalar)
+      .def_readwrite("post_norm", &LayerSpec::post_norm)
+      .def_readwrite("resid_gate", &LayerSpec::resid_gate)
+      .def_readwrite("rot_dim", &LayerSpec::rot_dim)
+      .def_readwrite("rot_dims", &LayerSpec::rot_dims)
+      .def_readwrite("rot_base", &LayerSpec::rot_base)
+      .def_readwrite("window", &LayerSpec::window)
+      .def_readwrite("width", &LayerSpec::width)
+      .def_readwrite("experts", &LayerSpec::experts)
+      .def_readwrite("top", &LayerSpec::top)
+      .def_readwrite("shared_ff", &LayerSpec::shared_ff)
+      .def_readwrite("correction", &LayerSpec::correction)
+      .def_readwrite("router_scale", &LayerSpec::router_scale)
       .def_readwrite("weights_of", &LayerSpec::weights_of);
 
   py::class_<EngineConfig>(m, "EngineConfig")
@@ -189,6 +208,14 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       .def_readwrite("kv_fp8", &EngineConfig::kv_fp8)
       .def_readwrite("layers", &EngineConfig::layers)
       .def_readwrite("max_positions", &EngineConfig::max_positions)
+      .def_readwrite("embed_scale", &EngineConfig::embed_scale)
+      .def_readwrite("logit_scale", &EngineConfig::logit_scale)
+      .def_readwrite("bigram_buckets", &EngineConfig::bigram_buckets)
+      .def_readwrite("bigram_prev", &EngineConfig::bigram_prev)
+      .def_readwrite("bigram_cur", &EngineConfig::bigram_cur)
+      .def_readwrite("loop_start", &EngineConfig::loop_start)
+      .def_readwrite("loop_stop", &EngineConfig::loop_stop)
+      .def_readwrite("loop_times", &EngineConfig::loop_times)
       .def_readwrite("compute_f32", &EngineConfig::compute_f32)
       .def_readwrite("kv_pool_tokens", &EngineConfig::kv_pool_tokens);
 
@@ -293,6 +320,10 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       .def_property_readonly("kv_blocks_free", &Engine::kv_blocks_free)
       .def_property_readonly("kv_block_tokens", &Engine::kv_block_tokens)
       .def_property_readonly("mixed_steps", &Engine::mixed_steps)
+      .def_property_readonly("recurrent", &Engine::recurrent)
+      .def("resumable", &Engine::resumable, py::arg("slot"), py::arg("n"))
+      .def_property_readonly("layer_runs", &Engine::layer_runs)
+      .def("set_run_limit", &Engine::set_run_limit, py::arg("n"))
       .def("step",
            [](Engine& e, const std::vector<int>& slots, const std::vector<int>& starts, const std::vector<int>& counts,
               const std::vector<int>& tokens, const std::vector<int>& want) {
@@ -689,6 +720,111 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       py::arg("v_scale") = 1.f);
   m.def("attn_prefill_supports", &attn_prefill_supports);
 
+  // ------------------------------------------------------------------ layered decoders' row operations
+  auto next_args = [](int kind, uintptr_t g, uintptr_t out, int ldo) {
+    NextArgs x;
+    x.kind = kind; x.g = (const float*)g; x.out = (void*)out; x.ldo = ldo;
+    return x;
+  };
+  m.attr("NEXT_NONE") = (int)NEXT_NONE;
+  m.attr("NEXT_NORM") = (int)NEXT_NORM;
+  m.attr("NEXT_RAW") = (int)NEXT_RAW;
+  m.def(
+      "embed_rows",
+      [next_args](int rows, uintptr_t table, float scale, uintptr_t pair_table, int buckets, long long mul_prev,
+                  long long mul_cur, uintptr_t tokens, uintptr_t pos, uintptr_t slot, uintptr_t run, uintptr_t last, int slots,
+                  int dp, int d, float eps, uintptr_t x, uintptr_t keep, int ld_keep, int f32, int next, uintptr_t g,
+                  uintptr_t out, int ldo, uintptr_t st) {
+        EmbedArgs a;
+        std::memset((void*)&a, 0, sizeof(a));
+        a.table = (const bf16_t*)table; a.scale = scale; a.pair_table = (const bf16_t*)pair_table; a.buckets = buckets;
+        a.mul_prev = mul_prev; a.mul_cur = mul_cur; a.tokens = (const int*)tokens; a.pos = (const int*)pos;
+        a.slot = (const int*)slot; a.run = (const int*)run; a.last = (int*)last; a.slots = slots; a.dp = dp; a.d = d;
+        a.eps = eps; a.x = (float*)x; a.keep = (void*)keep; a.ld_keep = ld_keep; a.f32 = f32;
+        a.next = next_args(next, g, out, ldo);
+        launch_embed_rows(a, rows, S(st));
+      },
+      py::arg("rows"), py::arg("table"), py::arg("scale"), py::arg("pair_table"), py::arg("buckets"), py::arg("mul_prev"),
+      py::arg("mul_cur"), py::arg("tokens"), py::arg("pos"), py::arg("slot"), py::arg("run"), py::arg("last"),
+      py::arg("slots"), py::arg("dp"), py::arg("d"), py::arg("eps"), py::arg("x"), py::arg("keep"), py::arg("ld_keep"),
+      py::arg("f32"), py::arg("next"), py::arg("g"), py::arg("out"), py::arg("ldo"), py::arg("stream"));
+  m.def(
+      "row_close",
+      [next_args](int rows, uintptr_t x, int dp, int d, float eps, uintptr_t y, uintptr_t ye, uintptr_t pair, uintptr_t wt,
+                  int top, uintptr_t gate, int ldg, uintptr_t gate_bias, uintptr_t post, int replace, uintptr_t add, int f32,
+                  int next, uintptr_t g, uintptr_t out, int ldo, uintptr_t st) {
+        RowCloseArgs a;
+        std::memset((void*)&a, 0, sizeof(a));
+        a.x = (float*)x; a.dp = dp; a.d = d; a.eps = eps; a.y = (const float*)y; a.ye = (const void*)ye;
+        a.pair = (const int*)pair; a.wt = (const float*)wt; a.top = top; a.gate = (const float*)gate; a.ldg = ldg;
+        a.gate_bias = (const float*)gate_bias; a.post = (const float*)post; a.replace = replace; a.add = (const float*)add;
+        a.f32 = f32;
+        a.next = next_args(next, g, out, ldo);
+        launch_row_close(a, rows, S(st));
+      },
+      py::arg("rows"), py::arg("x"), py::arg("dp"), py::arg("d"), py::arg("eps"), py::arg("y"), py::arg("ye") = 0,
+      py::arg("pair") = 0, py::arg("wt") = 0, py::arg("top") = 0, py::arg("gate") = 0, py::arg("ldg") = 0,
+      py::arg("gate_bias") = 0, py::arg("post") = 0, py::arg("replace") = 0, py::arg("add") = 0, py::arg("f32") = 0,
+      py::arg("next") = 0, py::arg("g") = 0, py::arg("out") = 0, py::arg("ldo") = 0, py::arg("stream") = 0);
+  // minGRU over portions: (first row, rows, slot, first position) each, cut into chunks here; `work`: device
+  // scratch for the chunk list (24 bytes a chunk), `agg`: [chunks][3][w] floats.  decode: pieces empty, n rows
+  m.attr("SCAN_CHUNK") = SCAN_CHUNK;
+  m.def(
+      "mingru",
+      [](const std::vector<std::vector<int>>& pieces, int n, uintptr_t pos, uintptr_t slot, uintptr_t in, int ld, int z_off,
+         int u_off, int g_off, uintptr_t zb, uintptr_t ub, int w, uintptr_t state, int slots, uintptr_t agg, uintptr_t work,
+         uintptr_t out, int ldo, int f32, uintptr_t st) {
+        MinGruArgs a;
+        std::memset(&a, 0, sizeof(a));
+        a.in = (const float*)in; a.ld = ld; a.z_off = z_off; a.u_off = u_off; a.g_off = g_off; a.zb = (const float*)zb;
+        a.ub = (const float*)ub; a.w = w; a.state = (float*)state; a.slots = slots; a.pos = (const int*)pos;
+        a.slot = (const int*)slot; a.agg = (float*)agg; a.out = (void*)out; a.ldo = ldo; a.f32 = f32; a.n = n;
+        std::vector<ScanChunk> c;
+        for (const auto& p : pieces) {
+          const int c0 = (int)c.size();
+          if (p.size() != 4 || p[2] < 0 || p[2] >= slots) throw std::runtime_error("mingru: bad piece");
+          for (int k = 0; k < p[1]; k += SCAN_CHUNK)
+            c.push_back(ScanChunk{p[0] + k, std::min(SCAN_CHUNK, p[1] - k), p[2], p[3] + k, c0, k + SCAN_CHUNK >= p[1]});
+          if (p[1] > SCAN_CHUNK) a.split = 1;
+        }
+        if (!c.empty()) {
+          HIP_CHECK(hipMemcpyAsync((void*)work, c.data(), c.size() * sizeof(ScanChunk), hipMemcpyHostToDevice, S(st)));
+          HIP_CHECK(hipStreamSynchronize(S(st)));
+          a.chunks = (const ScanChunk*)work;
+          a.n = (int)c.size();
+        }
+        launch_mingru(a, S(st));
+      },
+      py::arg("pieces"), py::arg("n"), py::arg("pos"), py::arg("slot"), py::arg("inp"), py::arg("ld"), py::arg("z_off"),
+      py::arg("u_off"), py::arg("g_off"), py::arg("zb"), py::arg("ub"), py::arg("w"), py::arg("state"), py::arg("slots"),
+      py::arg("agg"), py::arg("work"), py::arg("out"), py::arg("ldo"), py::arg("f32"), py::arg("stream"));
+  // the routed experts of n tokens; few: launch_moe_few (y), else launch_moe_grouped (ye, pair, wt)
+  m.attr("MOE_FEW") = MOE_FEW;
+  m.def("moe_tile_rows", &moe_tile_rows);
+  m.def("moe_max_tiles", &moe_max_tiles);
+  m.def(
+      "moe",
+      [](bool few, int n, int experts, int top, float scale, uintptr_t logits, int ldl, uintptr_t corr, int dp, int ff, int act,
+         uintptr_t h, int ldh, uintptr_t wgu, uintptr_t wdn, uintptr_t sel, uintptr_t wt, uintptr_t pair, uintptr_t token,
+         uintptr_t tiles, uintptr_t n_tiles, int max_tiles, uintptr_t act_out, uintptr_t ye, uintptr_t gu32, int f32,
+         uintptr_t sh_act, int ld_sh, int sh_ff, uintptr_t sh_dn, uintptr_t y, uintptr_t st) {
+        MoeArgs a;
+        std::memset(&a, 0, sizeof(a));
+        a.n = n; a.experts = experts; a.top = top; a.scale = scale; a.logits = (const float*)logits; a.ldl = ldl;
+        a.corr = (const float*)corr; a.dp = dp; a.ff = ff; a.act = act; a.h = (const void*)h; a.ldh = ldh;
+        a.wgu = (const bf16_t*)wgu; a.wdn = (const bf16_t*)wdn; a.sel = (int*)sel; a.wt = (float*)wt; a.pair = (int*)pair;
+        a.token = (int*)token; a.tiles = (int4*)tiles; a.n_tiles = (int*)n_tiles; a.max_tiles = max_tiles;
+        a.act_out = (void*)act_out; a.ye = (void*)ye; a.gu32 = (float*)gu32; a.f32 = f32; a.sh_act = (const bf16_t*)sh_act;
+        a.ld_sh = ld_sh; a.sh_ff = sh_ff; a.sh_dn = (const bf16_t*)sh_dn; a.y = (float*)y;
+        if (few) launch_moe_few(a, S(st));
+        else launch_moe_grouped(a, S(st));
+      },
+      py::arg("few"), py::arg("n"), py::arg("experts"), py::arg("top"), py::arg("scale"), py::arg("logits"), py::arg("ldl"),
+      py::arg("corr"), py::arg("dp"), py::arg("ff"), py::arg("act"), py::arg("h"), py::arg("ldh"), py::arg("wgu"),
+      py::arg("wdn"), py::arg("sel"), py::arg("wt"), py::arg("pair"), py::arg("token"), py::arg("tiles"), py::arg("n_tiles"),
+      py::arg("max_tiles"), py::arg("act_out"), py::arg("ye"), py::arg("gu32"), py::arg("f32"), py::arg("sh_act") = 0,
+      py::arg("ld_sh") = 0, py::arg("sh_ff") = 0, py::arg("sh_dn") = 0, py::arg("y") = 0, py::arg("stream") = 0);
+
   // ------------------------------------------------------------------ latent attention
   // the absorbed path over a paged cache: prep (latents of `rows` rows into the cache, queries of the first
   // n absorbed), attention, output.  tiles: (first flat row, rows) pairs on the device or 0 (every row its
@@ -698,9 +834,13 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       [](int n, int rows, int H, int dk, int dkp, int dvp, int rank, int rp, float scale, float eps, uintptr_t norm_w,
          uintptr_t sink, uintptr_t qdg, int ld, int dkv_off, int g_off, uintptr_t pos, uintptr_t slot, uintptr_t pool,
          uintptr_t bt, int maxb, int kvb, int f32, uintptr_t wukT, uintptr_t wuv, uintptr_t qa, uintptr_t tiles,
-         int n_tiles, int nsplit, uintptr_t opart, uintptr_t ml, uintptr_t out, int ldo, uintptr_t st) {
+         int n_tiles, int nsplit, uintptr_t opart, uintptr_t ml, uintptr_t out, int ldo, uintptr_t st, int rot, int roff,
+         int qrot, uintptr_t rope, int window, int head_gate) {
         LatentAttnArgs a;
         std::memset(&a, 0, sizeof(a));
+        a.rot = rot; a.roff = roff; a.qrot = qrot; a.rope = (const float2*)rope; a.window = window; a.head_gate = head_gate;
+        if (rot % 2 || roff % 8 || qrot % 8 || (rot && (!rope || roff + rot > rp || qrot + rot > dkp)))
+          throw std::runtime_error("latent_attention: bad rotated part");
         a.n = n; a.H = H; a.dk = dk; a.dkp = dkp; a.dvp = dvp; a.rank = rank; a.rp = rp; a.scale = scale; a.eps = eps;
         a.norm_w = (const float*)norm_w; a.sink = (const float*)sink; a.qdg = (const float*)qdg; a.ld = ld;
         a.dkv_off = dkv_off; a.g_off = g_off; a.pos = (const int*)pos; a.slot = (const int*)slot; a.pool = (void*)pool;
@@ -717,12 +857,17 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       py::arg("dkv_off"), py::arg("g_off"), py::arg("pos"), py::arg("slot"), py::arg("pool"), py::arg("bt"),
       py::arg("maxb"), py::arg("kvb"), py::arg("f32"), py::arg("wukT"), py::arg("wuv"), py::arg("qa"), py::arg("tiles"),
       py::arg("n_tiles"), py::arg("nsplit"), py::arg("opart"), py::arg("ml"), py::arg("out"), py::arg("ldo"),
-      py::arg("stream"));
+      py::arg("stream"), py::arg("rot") = 0, py::arg("roff") = 0, py::arg("qrot") = 0, py::arg("rope") = 0,
+      py::arg("window") = 0, py::arg("head_gate") = 0);
   m.def(
       "mha_prefill",
       [](uintptr_t q, int ldq, uintptr_t k, uintptr_t v, int ldkv, int H, int dkp, int dvp, int start, int T, float scale,
-         uintptr_t sink, uintptr_t gate, uintptr_t out, int ldo, uintptr_t st) {
+         uintptr_t sink, uintptr_t gate, uintptr_t out, int ldo, uintptr_t st, int window, int rot, int qrot, int pos0,
+         uintptr_t rope, int head_gate) {
         MhaPrefillArgs a;
+        std::memset(&a, 0, sizeof(a));
+        a.window = window; a.rot = rot; a.qrot = qrot; a.pos0 = pos0; a.rope = (const float2*)rope; a.head_gate = head_gate;
+        if (rot && (!rope || qrot + rot > dkp)) throw std::runtime_error("mha_prefill: bad rotated part");
         a.q = (const float*)q; a.ldq = ldq; a.k = (const bf16_t*)k; a.v = (const bf16_t*)v; a.ldkv = ldkv; a.H = H;
         a.dkp = dkp; a.dvp = dvp; a.start = start; a.T = T; a.scale = scale; a.sink = (const float*)sink;
         a.gate = (const float*)gate; a.out = (bf16_t*)out; a.ldo = ldo;
@@ -730,7 +875,8 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       },
       py::arg("q"), py::arg("ldq"), py::arg("k"), py::arg("v"), py::arg("ldkv"), py::arg("H"), py::arg("dkp"),
       py::arg("dvp"), py::arg("start"), py::arg("T"), py::arg("scale"), py::arg("sink"), py::arg("gate"), py::arg("out"),
-      py::arg("ldo"), py::arg("stream"));
+      py::arg("ldo"), py::arg("stream"), py::arg("window") = 0, py::arg("rot") = 0,
+      py::arg("qrot") = 0, py::arg("pos0") = 0, py::arg("rope") = 0, py::arg("head_gate") = 0);
   m.def("gemm_f32",
         [](uintptr_t A, int lda, uintptr_t W, int ldw, int M, int N, int K, uintptr_t C, int ldc, int accumulate,
            uintptr_t st) {
@@ -738,8 +884,11 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
         });
   m.def("embed_pos", [](uintptr_t table, uintptr_t pos_table, uintptr_t tokens, uintptr_t pos, int n, int d, uintptr_t x,
                         uintptr_t st) {
-    launch_embed_pos((const bf16_t*)table, (const bf16_t*)pos_table, (const int*)tokens, (const int*)pos, n, d, (float*)x,
-                     S(st));
+    EmbedArgs a;
+    std::memset((void*)&a, 0, sizeof(a));
+    a.table = (const bf16_t*)table; a.scale = 1.f; a.pos_table = (const bf16_t*)pos_table; a.tokens = (const int*)tokens;
+    a.pos = (const int*)pos; a.dp = a.d = d; a.x = (float*)x;
+    launch_embed_rows(a, n, S(st));
   });
   m.def("glu_f32", [](uintptr_t gu, int ldg, uintptr_t out, int ldo, int rows, int n, int act, uintptr_t st) {
     launch_glu_f32((const float*)gu, ldg, (float*)out, ldo, rows, n, act, S(st));

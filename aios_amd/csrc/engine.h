@@ -55,7 +55,14 @@ struct EngineConfig {
   std::vector<uint32_t> cu_mask;
   // models described layer by layer (layered.h); empty: a llama-family decoder of the sizes above
   std::vector<LayerSpec> layers;
-  int max_positions = 0;   // rows of the learned position table (layered models)
+  int max_positions = 0;   // rows of the learned position table (layered models; 0: none)
+  // layered models: scale of the token embedding and of the logits; an embedding of (previous, current) token
+  // pairs, row (previous * bigram_prev + token * bigram_cur) mod bigram_buckets (0: none); layers
+  // [loop_start, loop_stop) run loop_times times in a row, every pass entered by x = W_in [x; embedding] + step
+  float embed_scale = 1.f, logit_scale = 1.f;
+  int bigram_buckets = 0;
+  long long bigram_prev = 0, bigram_cur = 0;
+  int loop_start = 0, loop_stop = 0, loop_times = 0;
   int compute_f32 = 0;     // everything in 32 bits (layered models)
   // tokens the cache pool holds (whole blocks); 0: every slot's full context at once
   int kv_pool_tokens = 0;
@@ -201,6 +208,13 @@ class Engine {
                                const std::vector<int>& top_k, const std::vector<float>& top_p,
                                const std::vector<uint64_t>& seeds, const std::vector<uint8_t>& mask);
   bool mixed_steps() const { return lm_ != nullptr; }
+  // Models with a recurrent state: a slot can only go on where its state stands.  resumable: whether position n
+  // of the slot can run next -- 0 (a new sequence), the state's own position, or the single token it ran last
+  // once more (a queued step whose result was dropped)
+  bool recurrent() const { return lm_ && lm_->recurrent(); }
+  bool resumable(int slot, int n) const;
+  int layer_runs() const { return lm_ ? lm_->layer_runs() : cfg_.n_layers; }
+  void set_run_limit(int n);  // layered models: stop after n layer runs (inspection; n < 0: all)
   // residual stream of the last step's first `rows` rows (after the last layer), before the final norm
   std::vector<float> last_residual(int rows);
 
@@ -219,6 +233,13 @@ class Engine {
     size_t block;
   };
   std::vector<Pool> pools_;
+  struct SlotState {
+    int pos = 0;        // tokens the slot's recurrent state has taken in
+    bool again = false; // the last of them ran alone: it may run again
+  };
+  std::vector<SlotState> state_;
+  void check_state(int slot, int from) const;             // throws where the slot cannot go on at `from`
+  void move_state(int slot, int from, int to, bool singles);
   void init_paging();                    // block tables and the free list
   size_t init_step_state();              // logits, decode parameters, sampler (workspace bytes)
   void finalize_layered();

@@ -543,7 +543,8 @@ size_t Engine::init_step_state() {
 
 // layered models: paging and step state as above, the rest is the decoder's
 void Engine::finalize_layered() {
-  cfg_.max_ctx = std::min(cfg_.max_ctx, cfg_.max_positions);
+  if (cfg_.max_positions) cfg_.max_ctx = std::min(cfg_.max_ctx, cfg_.max_positions);
+  state_.assign(cfg_.max_slots, SlotState{});
   init_paging();
   lm_->finalize();
   ws_bytes_ += init_step_state();
@@ -1539,7 +1540,11 @@ void Engine::run_step(const std::vector<int>& slots, const std::vector<int>& sta
   for (size_t i = 0; i < want.size(); ++i)
     if (want[i] < (i ? want[i - 1] + 1 : 0) || want[i] >= (int)total) throw std::runtime_error("step: bad wanted index");
   if (!logits && (int)want.size() > Bm) throw std::runtime_error("step: more sampled rows than max_batch");
-  for (int e = 0; e < E; ++e) kv_prepare_write(slots[e], starts[e], starts[e] + counts[e]);
+  for (int e = 0; e < E; ++e) check_state(slots[e], starts[e]);
+  for (int e = 0; e < E; ++e) {
+    kv_prepare_write(slots[e], starts[e], starts[e] + counts[e]);
+    move_state(slots[e], starts[e], starts[e] + counts[e], counts[e] == 1);
+  }
   kv_sync(0);
   if (logits) logits->resize(want.size() * (size_t)V);
   int e = 0, off = 0;       // next entry and tokens of it already run
@@ -1632,6 +1637,32 @@ std::vector<int> Engine::step_sample(const std::vector<int>& slots, const std::v
   return std::vector<int>(h_tok_out_, h_tok_out_ + B);
 }
 
+// ---- recurrent state ---------------------------------------------------------------------------------
+bool Engine::resumable(int slot, int n) const {
+  if (slot < 0 || slot >= cfg_.max_slots) throw std::runtime_error("resumable: bad slot");
+  if (!recurrent() || n == 0) return true;
+  const SlotState& s = state_[slot];
+  return n == s.pos || (s.again && n == s.pos - 1);
+}
+
+void Engine::check_state(int slot, int from) const {
+  if (!resumable(slot, from))
+    throw std::runtime_error("slot " + std::to_string(slot) + ": its recurrent state stands at position " +
+                             std::to_string(state_[slot].pos) + ", not at " + std::to_string(from));
+}
+
+void Engine::move_state(int slot, int from, int to, bool singles) {
+  if (!recurrent() || to <= from) return;
+  state_[slot].pos = to;
+  state_[slot].again = singles;
+}
+
+void Engine::set_run_limit(int n) {
+  if (!lm_) throw std::runtime_error("set_run_limit: layered models only");
+  reset_graphs();
+  lm_->set_run_limit(n);
+}
+
 std::vector<float> Engine::last_residual(int rows) {
   if (!lm_) throw std::runtime_error("last_residual: layered models only");
   return lm_->residual(rows);
@@ -1655,6 +1686,7 @@ std::vector<int> Engine::decode(const std::vector<int>& slots, const std::vector
     if (tokens[b] < 0 || tokens[b] >= cfg_.vocab_size) throw std::runtime_error("decode: token out of range");
     sl[b] = pos[b] + 1;
   }
+  for (int b = 0; b < B; ++b) check_state(slots[b], pos[b]);
   row_slots_ = slots;
   row_pos_ = pos;
   const int Bm = cfg_.max_batch;
@@ -1803,8 +1835,10 @@ void Engine::decode_loop_run(int B, int n_steps, bool use_graph) {
   HIP_CHECK(hipSetDevice(cfg_.device));
   if ((int)row_slots_.size() < B) throw std::runtime_error("decode_loop_run: rows not prepared");
   // map (and un-share) the blocks the n steps will write, before any of them is enqueued
+  for (int b = 0; b < B; ++b) check_state(row_slots_[b], row_pos_[b]);
   for (int b = 0; b < B; ++b) {
     kv_prepare_write(row_slots_[b], row_pos_[b], std::min(row_pos_[b] + n_steps, cfg_.max_ctx));
+    move_state(row_slots_[b], row_pos_[b], std::min(row_pos_[b] + n_steps, cfg_.max_ctx), true);
     row_pos_[b] = std::min(row_pos_[b] + n_steps, cfg_.max_ctx);
   }
   kv_sync(B);
@@ -1877,6 +1911,7 @@ void Engine::decode_submit(const std::vector<int>& slots, const std::vector<int>
     if (!tokens.empty() && (tokens[b] < 0 || tokens[b] >= cfg_.vocab_size))
       throw std::runtime_error("decode_submit: token out of range");
   }
+  for (int b = 0; b < B; ++b) check_state(slots[b], pos[b]);
   const int Bm = cfg_.max_batch;
   par_buf_ ^= 1;  // the other half: the previous submit's copy may not have run yet
   char* hpar = h_par_ + (size_t)par_buf_ * par_bytes_;
@@ -1906,6 +1941,7 @@ void Engine::decode_submit(const std::vector<int>& slots, const std::vector<int>
   row_pos_ = pos;
   for (int b = 0; b < B; ++b) {
     kv_prepare_write(slots[b], pos[b], pos[b] + 1);
+    move_state(slots[b], pos[b], pos[b] + 1, true);
     row_pos_[b] = pos[b] + 1;
   }
   kv_sync(B);
@@ -2061,6 +2097,11 @@ void Engine::copy_slot(int src, int dst, int n) {
   if (src == dst) return;
   HIP_CHECK(hipSetDevice(cfg_.device));
   n = std::min(n, cfg_.max_ctx);
+  if (recurrent()) {
+    if (!resumable(src, n)) throw std::runtime_error("copy_slot: the source's recurrent state is not at this length");
+    if (n > 0) lm_->copy_state(src, dst);
+    state_[dst] = n > 0 ? state_[src] : SlotState{};
+  }
   int* s = bt_.data() + (size_t)src * kv_maxb_;
   int* d = bt_.data() + (size_t)dst * kv_maxb_;
   for (int j = 0; j < kv_maxb_; ++j) {  // dst's old content is dropped
@@ -2083,6 +2124,7 @@ void Engine::copy_slot(int src, int dst, int n) {
 
 void Engine::release_slot(int slot) {
   if (slot < 0 || slot >= cfg_.max_slots) throw std::runtime_error("release_slot: bad slot");
+  if (!state_.empty()) state_[slot] = SlotState{};
   int* row = bt_.data() + (size_t)slot * kv_maxb_;
   for (int j = 0; j < kv_maxb_; ++j) {
     if (row[j] >= 0) bt_dirty_ = true;

@@ -1,7 +1,7 @@
 // Causal flash attention over contiguous per-head keys and values (latent.h, expanded form): one
 // sequence's T new tokens over keys [0, start + T), query-key and value dimensions of their own, an
-// optional sink logit per head (it starts the running maximum and sum: it has no key and no value) and
-// an optional output gate.
+// optional sliding window, sink logit per head (it starts the running maximum and sum: it has no key and no
+// value) and output gate, and an optional rotation of part of the queries.
 //
 // Four waves of 32 query rows; 64-key tiles of K and V in two LDS buffers, fed by two register buffers, one
 // barrier per tile -- the pipeline of the paged GQA kernel (attention_prefill.hip), whose S^T = K Q^T /
@@ -48,6 +48,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
   const bool qvalid = tq < a.T;
   const int tql = qvalid ? tq : a.T - 1;
   const int qpos = a.start + tql;
+  const int qlow = a.window ? max(0, qpos - a.window + 1) : 0;  // first visible key
   gbf16x8 qf[KS];
   const float sc = a.scale * 1.4426950408889634f;
   {
@@ -56,7 +57,22 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
     for (int s = 0; s < KS; ++s) {
       uint4 u = make_uint4(0, 0, 0, 0);
       if (16 * s < a.dkp) {
-        const float4 x0 = *(const float4*)(qp + 16 * s), x1 = *(const float4*)(qp + 16 * s + 4);
+        float4 x0 = *(const float4*)(qp + 16 * s), x1 = *(const float4*)(qp + 16 * s + 4);
+        const int i0 = 16 * s + 8 * half - a.qrot;  // place in the rotated part (eight numbers are in or out together)
+        if (i0 >= 0 && i0 < a.rot) {
+          const float2* cs = a.rope + (size_t)(a.pos0 + tql) * (a.rot >> 1) + (i0 >> 1);
+          auto turn = [&](float& x, float& y, int i) {
+            if (i0 + 2 * i >= a.rot) return;
+            const float2 t = cs[i];
+            const float u = x, v = y;
+            x = u * t.x - v * t.y;
+            y = v * t.x + u * t.y;
+          };
+          turn(x0.x, x0.y, 0);
+          turn(x0.z, x0.w, 1);
+          turn(x1.x, x1.y, 2);
+          turn(x1.z, x1.w, 3);
+        }
         u = make_uint4(pk_bf16(x0.x * sc, x0.y * sc), pk_bf16(x0.z * sc, x0.w * sc), pk_bf16(x1.x * sc, x1.y * sc),
                        pk_bf16(x1.z * sc, x1.w * sc));
       }
@@ -73,6 +89,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
 
   const int last_pos = a.start + min(a.T, t0 + 128) - 1;  // highest query position of the block
   const int ntiles = last_pos / MH_KT + 1;
+  const int kt0 = a.window ? max(0, a.start + t0 - a.window + 1) / MH_KT : 0;  // tile of the block's first visible key
   const int last_key = a.start + a.T - 1;
   constexpr int KP = MH_KT * DK / 8 / 256, VP = MH_KT * DV / 8 / 256;  // 16-B pieces per thread
   struct Regs {
@@ -125,26 +142,27 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
       }
     }
     const int kbase = kt * MH_KT;
-    const bool full = kbase + MH_KT - 1 <= qpos;
+    const bool full = kbase + MH_KT - 1 <= qpos && kbase >= qlow;
     float mx = -INFINITY;
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int key = kbase + t * 32 + (r & 3) + 8 * (r >> 2) + 4 * half;
-        if (!full && key > qpos) st[t][r] = -INFINITY;
+        if (!full && (key > qpos || key < qlow)) st[t][r] = -INFINITY;
         mx = fmaxf(mx, st[t][r]);
       }
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float mn = fmaxf(m_run, mx);  // finite: key 0 (in tile 0) is visible to every row
-    const float alpha = __builtin_amdgcn_exp2f(m_run - mn);
+    const float mn = fmaxf(m_run, mx);
+    const float ms = mn == -INFINITY ? 0.f : mn;  // (no visible key yet: a window that starts in a later tile)
+    const float alpha = __builtin_amdgcn_exp2f(m_run - ms);
     float ps = 0.f;
     uint32_t pb[2][8], pl[2][8];  // P^T as packed bf16 pairs (hi, lo), accumulator order
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int r = 0; r < 16; r += 2) {
-        const float p0 = __builtin_amdgcn_exp2f(st[t][r] - mn), p1 = __builtin_amdgcn_exp2f(st[t][r + 1] - mn);
+        const float p0 = __builtin_amdgcn_exp2f(st[t][r] - ms), p1 = __builtin_amdgcn_exp2f(st[t][r + 1] - ms);
         ps += p0 + p1;
         const uint32_t hi = pk_bf16(p0, p1);
         pb[t][r >> 1] = hi;
@@ -182,11 +200,11 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
   bf16_t* L0 = mh_smem;
   bf16_t* L1 = mh_smem + TILE_ELEMS;
   Regs A, B;
-  load(A, 0);
-  load(B, 1);
+  load(A, kt0);
+  load(B, kt0 + 1);
   stage(A, L0);
   __syncthreads();
-  for (int kt = 0; kt < ntiles; kt += 2) {  // (an odd count computes one fully masked pad tile)
+  for (int kt = kt0; kt < ntiles; kt += 2) {  // (an odd count computes one fully masked pad tile)
     load(A, kt + 2);
     math(L0, kt);
     stage(B, L1);
@@ -199,7 +217,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
   if (!qvalid) return;
   const float inv = 1.f / l_run;
   bf16_t* op = a.out + (size_t)tq * a.ldo + (size_t)h * a.dvp;
-  const float* gp = a.gate ? a.gate + (size_t)tq * a.ldq + (size_t)h * a.dvp : nullptr;
+  const float* gp = a.gate ? a.gate + (size_t)tq * a.ldq + (a.head_gate ? h : (size_t)h * a.dvp) : nullptr;
 #pragma unroll
   for (int i = 0; i < OT; ++i)
 #pragma unroll
@@ -210,7 +228,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = o[i][r + e] * inv;
         if (gp) {
-          const float4 g = *(const float4*)(gp + d);
+          const float4 g = a.head_gate ? make_float4(gp[0], gp[0], gp[0], gp[0]) : *(const float4*)(gp + d);
           v[0] *= 1.f / (1.f + __expf(-g.x));
           v[1] *= 1.f / (1.f + __expf(-g.y));
           v[2] *= 1.f / (1.f + __expf(-g.z));
@@ -240,6 +258,7 @@ static void mha_dv(const MhaPrefillArgs& a, hipStream_t st) {
 
 void launch_mha_prefill(const MhaPrefillArgs& a, hipStream_t st) {
   if (!mha_prefill_supports(a.dkp, a.dvp)) throw std::runtime_error("mha_prefill: unsupported head dimensions");
+  if (a.rot % 2 || a.qrot % 8) throw std::runtime_error("mha_prefill: bad rotated part");
   if (a.ldkv % 8 || a.ldq % 4 || a.ldo % 4) throw std::runtime_error("mha_prefill: misaligned rows");
   if (a.T < 1) return;
   if (a.dkp <= 64) mha_dv<64>(a, st);

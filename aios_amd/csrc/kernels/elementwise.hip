@@ -113,6 +113,17 @@ void launch_f32_to_bf16(const float* x, bf16_t* y, size_t n, hipStream_t st) {
   hipLaunchKernelGGL(f32_to_bf16_kernel, dim3(g), dim3(256), 0, st, x, y, n);
 }
 
+__global__ void zero_rows_kernel(float* __restrict__ y, int ldy, int n) {
+  float* r = y + (size_t)blockIdx.y * ldy;
+  for (int i = 4 * (blockIdx.x * blockDim.x + threadIdx.x); i < n; i += 4 * gridDim.x * blockDim.x)
+    *(float4*)(r + i) = make_float4(0.f, 0.f, 0.f, 0.f);
+}
+void launch_zero_rows(float* y, int ldy, int rows, int n, hipStream_t st) {
+  if (n % 4 || ldy % 4 || ((uintptr_t)y & 15)) throw std::runtime_error("zero_rows: rows must be 16-byte aligned");
+  if (rows < 1 || n < 1) return;
+  hipLaunchKernelGGL(zero_rows_kernel, dim3(std::min(64, (n / 4 + 255) / 256), rows), dim3(256), 0, st, y, ldy, n);
+}
+
 __global__ void add_kernel(float* __restrict__ y, const float* __restrict__ x, size_t n) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) y[i] += x[i];
 }

@@ -197,7 +197,7 @@ static void launch_big_tiles(const GemmQArgs& a, hipStream_t st) {
   if (a.epi == GEPI_SWIGLU_BF16 || a.epi == GEPI_STORE16) S = 1;  // these epilogues need the full sum
   S = std::max(1, std::min(S, a.K / 64));
   if (S > 1 && a.epi == GEPI_STORE)
-    HIP_CHECK(hipMemset2DAsync(a.C, (size_t)a.ldc * 4, 0, (size_t)a.N * 4, a.M, st));
+    launch_zero_rows(a.C, a.ldc, a.M, a.N, st);  // (a kernel: the launch may be captured)
   const dim3 grid(tiles, S);
   switch (a.epi) {
     case GEPI_STORE: hipLaunchKernelGGL((gemm_big_kernel<QT, BM, BN, GEPI_STORE>), grid, dim3(NT), 0, st, a); break;

@@ -9,13 +9,29 @@ namespace aios {
 
 constexpr int GF_T = 64, GF_K = 16, GF_LD = GF_K + 1;
 
+// rows of a grouped product (launch_gemm_f32_grouped); tiles null: plain rows
+struct GroupRows {
+  const int4* tiles;
+  const int* n_tiles;
+  const int* token;
+};
+
 // 64 x 64 tile, four waves of 32 x 32 (2 x 2 accumulators)
 __global__ void __launch_bounds__(256) gemm_f32_kernel(const float* __restrict__ A, int lda, const bf16_t* __restrict__ W,
-                                                       int ldw, int M, int N, int K, float* __restrict__ C, int ldc, int acc_c) {
+                                                       int ldw, int M, int N, int K, float* __restrict__ C, int ldc, int acc_c,
+                                                       GroupRows gr) {
   __shared__ float sA[GF_T * GF_LD], sB[GF_T * GF_LD];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int r16 = lane & 15, q = lane >> 4;
-  const int m0 = blockIdx.y * GF_T, n0 = blockIdx.x * GF_T;
+  int m0 = blockIdx.y * GF_T;
+  const int n0 = blockIdx.x * GF_T;
+  if (gr.tiles) {
+    if ((int)blockIdx.y >= *gr.n_tiles) return;
+    const int4 t = gr.tiles[blockIdx.y];
+    m0 = t.y;
+    M = t.y + t.z;
+    W += (size_t)t.x * N * ldw;
+  }
   const int wm = (wave >> 1) * 32, wn = (wave & 1) * 32;
   gf32x4 acc[2][2];
 #pragma unroll
@@ -23,10 +39,12 @@ __global__ void __launch_bounds__(256) gemm_f32_kernel(const float* __restrict__
 #pragma unroll
     for (int j = 0; j < 2; ++j) acc[i][j] = gf32x4{0.f, 0.f, 0.f, 0.f};
   const int lr = tid >> 2, lc = (tid & 3) * 4;  // this thread's row and first column of each staged tile
+  const float* arow = A;
+  if (m0 + lr < M) arow = A + (size_t)(gr.token ? gr.token[m0 + lr] : m0 + lr) * lda;
   for (int k0 = 0; k0 < K; k0 += GF_K) {
     float4 av = make_float4(0.f, 0.f, 0.f, 0.f);
     uint2 bv = make_uint2(0, 0);
-    if (m0 + lr < M) av = *(const float4*)(A + (size_t)(m0 + lr) * lda + k0 + lc);
+    if (m0 + lr < M) av = *(const float4*)(arow + k0 + lc);
     if (n0 + lr < N) bv = *(const uint2*)(W + (size_t)(n0 + lr) * ldw + k0 + lc);
     __syncthreads();
     float* pa = sA + lr * GF_LD + lc;
@@ -71,7 +89,15 @@ void launch_gemm_f32(const float* A, int lda, const bf16_t* W, int ldw, int M, i
   if (K % GF_K || lda % 4 || ldw % 4) throw std::runtime_error("gemm_f32: K must be a multiple of 16, rows 16-byte aligned");
   if (M < 1 || N < 1) return;
   hipLaunchKernelGGL(gemm_f32_kernel, dim3((N + GF_T - 1) / GF_T, (M + GF_T - 1) / GF_T), dim3(256), 0, st, A, lda, W, ldw,
-                     M, N, K, C, ldc, accumulate);
+                     M, N, K, C, ldc, accumulate, GroupRows{nullptr, nullptr, nullptr});
+}
+
+void launch_gemm_f32_grouped(const float* A, int lda, const int* token, const bf16_t* W, const int4* tiles, const int* n_tiles,
+                             int max_tiles, int N, int K, float* C, hipStream_t st) {
+  if (K % GF_K || lda % 4) throw std::runtime_error("gemm_f32: K must be a multiple of 16, rows 16-byte aligned");
+  if (max_tiles < 1 || N < 1) return;
+  hipLaunchKernelGGL(gemm_f32_kernel, dim3((N + GF_T - 1) / GF_T, max_tiles), dim3(256), 0, st, A, lda, W, K, 0, N, K, C, N, 0,
+                     GroupRows{tiles, n_tiles, token});
 }
 
 }  // namespace aios

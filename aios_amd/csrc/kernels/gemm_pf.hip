@@ -186,7 +186,7 @@ static bool pf_run(const GemmQArgs& a, const PfPlan& p, hipStream_t st) {
   const int qt0 = a.seg[0].qtype, qt1 = a.seg[a.nseg - 1].qtype;
   if (p.s != 1 && a.epi == GEPI_QKV) return false;  // (plans keep S = 1 for it; a pinned split declines)
   if (p.s != 1 && a.epi == GEPI_STORE)
-    HIP_CHECK(hipMemset2DAsync(a.C, (size_t)a.ldc * 4, 0, (size_t)a.N * 4, a.M, st));
+    launch_zero_rows(a.C, a.ldc, a.M, a.N, st);  // (a kernel: the launch may be captured)
 #ifndef AIOS_BF16_ONLY
   if (qt0 == QT_Q4_K && qt1 == QT_Q4_K) return pf_launch_fmt<QT_Q4_K, QT_Q4_K>(a, p.bm, p.bn, p.s, st);
   if (qt0 == QT_Q6_K && qt1 == QT_Q6_K) return pf_launch_fmt<QT_Q6_K, QT_Q6_K>(a, p.bm, p.bn, p.s, st);

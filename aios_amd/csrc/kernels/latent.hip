@@ -30,8 +30,25 @@ __device__ __forceinline__ float lat_exp2(float x) { return __builtin_amdgcn_exp
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 
 // ---- prep: latent norm + cache write, query absorption --------------------------------------------
-// one wave per row; the row stays in registers between its sum of squares and the scaled store.  Columns past
-// the rank are zero in x and in the weight, so only the mean's divisor knows the rank
+// (cos, sin) turns of the two pairs in v, whose first number is number i0 of the rotated part (i0 % 4 == 0)
+__device__ __forceinline__ float4 rope4(float4 v, const float2* cs, int i0, int rot) {
+  if (i0 < rot) {
+    const float2 t = cs[i0 >> 1];
+    const float x = v.x, y = v.y;
+    v.x = x * t.x - y * t.y;
+    v.y = y * t.x + x * t.y;
+  }
+  if (i0 + 2 < rot) {
+    const float2 t = cs[(i0 >> 1) + 1];
+    const float x = v.z, y = v.w;
+    v.z = x * t.x - y * t.y;
+    v.w = y * t.x + x * t.y;
+  }
+  return v;
+}
+
+// one wave per row; the row stays in registers between its sum of squares and the scaled store.  Columns between
+// the rank and the rotated part are zero in x and in the weight, so only the mean's divisor knows the rank
 template <bool F32>
 __device__ __forceinline__ void latent_cache_row(const LatentAttnArgs& a, int row) {
   const int lane = threadIdx.x & 63;
@@ -48,9 +65,11 @@ __device__ __forceinline__ void latent_cache_row(const LatentAttnArgs& a, int ro
     }
   }
   const int blk = a.bt[(size_t)slot * a.maxb + pos / a.kvb];
+  const int cend = a.rot ? a.roff : a.rp;
   float s = 0.f;
 #pragma unroll
-  for (int i = 0; i < 8; ++i) s += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+  for (int i = 0; i < 8; ++i)
+    if (256 * i + 4 * lane < cend) s += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
   s = wave_sum(s);
   const float inv = 1.f / sqrtf(s / (float)a.rank + a.eps);
   const size_t base = ((size_t)blk * a.kvb + pos % a.kvb) * a.rp;
@@ -58,15 +77,20 @@ __device__ __forceinline__ void latent_cache_row(const LatentAttnArgs& a, int ro
   for (int i = 0; i < 8; ++i) {
     const int c = 256 * i + 4 * lane;
     if (c >= a.rp) break;
-    const float4 o = make_float4(v[i].x * inv * g[i].x, v[i].y * inv * g[i].y, v[i].z * inv * g[i].z, v[i].w * inv * g[i].w);
+    float4 o = make_float4(v[i].x * inv * g[i].x, v[i].y * inv * g[i].y, v[i].z * inv * g[i].z, v[i].w * inv * g[i].w);
+    if (c >= cend) o = rope4(v[i], a.rope + (size_t)pos * (a.rot >> 1), c - a.roff, a.rot);
     if constexpr (F32) *(float4*)((float*)a.pool + base + c) = o;
     else *(uint2*)((bf16_t*)a.pool + base + c) = make_uint2(pk_bf16(o.x, o.y), pk_bf16(o.z, o.w));
   }
 }
 
-// 8 consecutive floats -> one bf16x8 fragment
-__device__ __forceinline__ gbf16x8 frag_f32(const float* p) {
-  const float4 x0 = *(const float4*)p, x1 = *(const float4*)(p + 4);
+// 8 consecutive floats -> one bf16x8 fragment; they are numbers i0 .. of the rotated part (i0 < 0: none of it)
+__device__ __forceinline__ gbf16x8 frag_f32(const float* p, const float2* cs, int i0, int rot) {
+  float4 x0 = *(const float4*)p, x1 = *(const float4*)(p + 4);
+  if (i0 >= 0) {
+    x0 = rope4(x0, cs, i0, rot);
+    x1 = rope4(x1, cs, i0 + 4, rot);
+  }
   const uint4 u = make_uint4(pk_bf16(x0.x, x0.y), pk_bf16(x0.z, x0.w), pk_bf16(x1.x, x1.y), pk_bf16(x1.z, x1.w));
   return __builtin_bit_cast(gbf16x8, u);
 }
@@ -90,6 +114,8 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatentAttnArgs a, int 
   const int r = rt * 64 + wave * 16 + r16;
   const float* qp = a.qdg + (size_t)m * a.ld + h * a.dkp + 8 * q;
   const bf16_t* wp = a.wukT + ((size_t)h * a.rp + r) * a.dkp + 8 * q;
+  const float2* cs = a.rot ? a.rope + (size_t)a.pos[m] * (a.rot >> 1) : nullptr;
+  const int qrot = a.rot ? a.qrot : a.dkp;
   gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < a.dkp; k0 += 128) {  // (four K-steps' loads in flight together; steps past dkp re-read)
     gbf16x8 af[4], bf[4];
@@ -97,7 +123,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatentAttnArgs a, int 
     for (int i = 0; i < 4; ++i) {
       const int k = min(k0 + 32 * i, a.dkp - 32);
       bf[i] = __builtin_bit_cast(gbf16x8, *(const lu32x4*)(wp + k));
-      af[i] = frag_f32(qp + k);
+      af[i] = frag_f32(qp + k, cs, k + 8 * q - qrot, a.rot);
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i)
@@ -123,10 +149,19 @@ __global__ void __launch_bounds__(256) latent_prep_f32_kernel(LatentAttnArgs a, 
   if (f >= a.n * a.H) return;
   const int t = f / a.H, h = f - t * a.H;
   const float* qp = a.qdg + (size_t)t * a.ld + h * a.dkp;
+  const float2* cs = a.rot ? a.rope + (size_t)a.pos[t] * (a.rot >> 1) : nullptr;
+  const int qrot = a.rot ? a.qrot : a.dkp;
   for (int r = lane; r < a.rp; r += 64) {
     const bf16_t* wp = a.wukT + ((size_t)h * a.rp + r) * a.dkp;
     float s = 0.f;
-    for (int d = 0; d < a.dkp; ++d) s = fmaf(qp[d], bf16_to_f32(wp[d]), s);
+    for (int d = 0; d < a.dkp; d += 4) {
+      float4 v = *(const float4*)(qp + d);
+      if (d >= qrot) v = rope4(v, cs, d - qrot, a.rot);
+      s = fmaf(v.x, bf16_to_f32(wp[d]), s);
+      s = fmaf(v.y, bf16_to_f32(wp[d + 1]), s);
+      s = fmaf(v.z, bf16_to_f32(wp[d + 2]), s);
+      s = fmaf(v.w, bf16_to_f32(wp[d + 3]), s);
+    }
     ((float*)a.qa)[(size_t)f * a.rp + r] = s;
   }
 }
@@ -192,8 +227,10 @@ latent_attn_kernel(LatentAttnArgs a) {
   const int nf = a.n * a.H;
   const int len = a.pos[(tl.f0 + tl.nv - 1) / a.H] + 1;
   const int* bt = a.bt + (size_t)a.slot[tl.f0 / a.H] * a.maxb;
-  const int nkt = (len + LT_KT - 1) / LT_KT, per = (nkt + a.nsplit - 1) / a.nsplit;
-  const int kt0 = split * per, kt1 = min(kt0 + per, nkt);
+  // (windowed: from the tile of the first key that the tile's first row sees)
+  const int klo = a.window ? max(0, a.pos[tl.f0 / a.H] - a.window + 1) / LT_KT : 0;
+  const int nkt = (len + LT_KT - 1) / LT_KT, per = (nkt - klo + a.nsplit - 1) / a.nsplit;
+  const int kt0 = klo + split * per, kt1 = min(kt0 + per, nkt);
   float* mlp = a.ml + ((size_t)split * nf + tl.f0) * 2;
   if (kt0 >= kt1) {  // (whole workgroup, before any barrier)
     if (tid < tl.nv) *(float2*)(mlp + 2 * tid) = make_float2(-INFINITY, 0.f);
@@ -244,6 +281,7 @@ latent_attn_kernel(LatentAttnArgs a) {
   gbf16x8 qf[KS];  // this wave's columns of the query rows
   const int f = tl.f0 + min(r16, tl.nv - 1);
   const int mypos = a.pos[f / a.H];
+  const int mylow = a.window ? mypos - a.window + 1 : 0;  // first visible key
   {
     const bf16_t* qp = (const bf16_t*)a.qa + (size_t)f * RP + wave * SH::CW + 8 * q;
 #pragma unroll
@@ -288,7 +326,7 @@ latent_attn_kernel(LatentAttnArgs a) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         const float v = i < 4 ? x0[i & 3] : x1[i & 3];
-        p[i] = key0 + i <= mypos ? v * sc : -INFINITY;
+        p[i] = key0 + i <= mypos && key0 + i >= mylow ? v * sc : -INFINITY;
         mx = fmaxf(mx, p[i]);
       }
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -365,7 +403,8 @@ __global__ void __launch_bounds__(256) latent_attn_plain_kernel(LatentAttnArgs a
   }
   float m = -INFINITY, l = 0.f;
   const float sc = a.scale * LOG2E;
-  for (int key = wave; key < len; key += 4) {
+  const int low = a.window ? max(0, len - a.window) : 0;
+  for (int key = low + wave; key < len; key += 4) {
     const size_t base = ((size_t)bt[key / a.kvb] * a.kvb + key % a.kvb) * RP + lane;
     float c[NR], s = 0.f;
 #pragma unroll
@@ -387,7 +426,7 @@ __global__ void __launch_bounds__(256) latent_attn_plain_kernel(LatentAttnArgs a
 #pragma unroll
   for (int i = 0; i < NR; ++i) so[wave * RP + 64 * i + lane] = o[i];
   __syncthreads();
-  const float M = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));  // (key 0 is visible: finite)
+  const float M = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));  // (the token's own key is visible: finite)
   float w[4], L = 0.f;
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
@@ -419,6 +458,7 @@ static void latent_plain(const LatentAttnArgs& a, hipStream_t st) {
     case 4: return latent_plain_go<4, F32>(a, st);
     case 6: return latent_plain_go<6, F32>(a, st);
     case 8: return latent_plain_go<8, F32>(a, st);
+    case 10: return latent_plain_go<10, F32>(a, st);
     case 12: return latent_plain_go<12, F32>(a, st);
     case 16: return latent_plain_go<16, F32>(a, st);
     case 32: return latent_plain_go<32, F32>(a, st);
@@ -435,6 +475,7 @@ void launch_latent_attn(const LatentAttnArgs& a, hipStream_t st) {
     case 4: return latent_attn_go<4>(a, st);
     case 6: return latent_attn_go<6>(a, st);
     case 8: return latent_attn_go<8>(a, st);
+    case 10: return latent_attn_go<10>(a, st);
     case 12: return latent_attn_go<12>(a, st);
     case 16: return latent_attn_go<16>(a, st);
   }
@@ -600,7 +641,7 @@ __global__ void __launch_bounds__(256) latent_out_kernel(LatentAttnArgs a) {
     if (t >= a.n) continue;
     float v = acc[j];
     const int c = h * a.dvp + col;
-    if (a.g_off >= 0) v *= sigmoid_f(a.qdg[(size_t)t * a.ld + a.g_off + c]);
+    if (a.g_off >= 0) v *= sigmoid_f(a.qdg[(size_t)t * a.ld + a.g_off + (a.head_gate ? h : c)]);
     ((bf16_t*)a.out)[(size_t)t * a.ldo + c] = f32_to_bf16(v);
   }
 }
@@ -631,7 +672,7 @@ __global__ void __launch_bounds__(256) latent_out_f32_kernel(LatentAttnArgs a) {
     s = wave_sum(s);
     if (lane == 0) {
       const int c = h * a.dvp + d;
-      if (a.g_off >= 0) s *= sigmoid_f(a.qdg[(size_t)t * a.ld + a.g_off + c]);
+      if (a.g_off >= 0) s *= sigmoid_f(a.qdg[(size_t)t * a.ld + a.g_off + (a.head_gate ? h : c)]);
       ((float*)a.out)[(size_t)t * a.ldo + c] = s;
     }
   }
@@ -659,48 +700,25 @@ void launch_latent_out(const LatentAttnArgs& a, hipStream_t st) {
 }
 
 // ---- expanded form: gather -----------------------------------------------------------------------
-__global__ void latent_gather_kernel(const bf16_t* __restrict__ pool, const int* __restrict__ bt, int kvb, int S, int rp,
-                                     bf16_t* __restrict__ out) {
+__global__ void latent_gather_kernel(const bf16_t* __restrict__ pool, const int* __restrict__ bt, int kvb, int k0, int S,
+                                     int rp, bf16_t* __restrict__ out) {
   const int p8 = rp >> 3;
   const size_t n = (size_t)S * p8;
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
     const int key = (int)(i / p8), c = (int)(i - (size_t)key * p8);
+    const int at = k0 + key;
     *(uint4*)(out + (size_t)key * rp + 8 * c) =
-        *(const uint4*)(pool + ((size_t)bt[key / kvb] * kvb + key % kvb) * rp + 8 * c);
+        *(const uint4*)(pool + ((size_t)bt[at / kvb] * kvb + at % kvb) * rp + 8 * c);
   }
 }
-void launch_latent_gather(const bf16_t* pool, const int* bt, int maxb, int kvb, int slot, int S, int rp, bf16_t* out,
+void launch_latent_gather(const bf16_t* pool, const int* bt, int maxb, int kvb, int slot, int k0, int S, int rp, bf16_t* out,
                           hipStream_t st) {
   const size_t n = (size_t)S * (rp / 8);
   const int g = (int)std::min<size_t>(2048, (n + 255) / 256);
-  hipLaunchKernelGGL(latent_gather_kernel, dim3(g), dim3(256), 0, st, pool, bt + (size_t)slot * maxb, kvb, S, rp, out);
+  hipLaunchKernelGGL(latent_gather_kernel, dim3(g), dim3(256), 0, st, pool, bt + (size_t)slot * maxb, kvb, k0, S, rp, out);
 }
 
-// ---- layered decoders: embedding, row gather, weight transpose, fp32 GLU ---------------------------
-__global__ void embed_pos_kernel(const bf16_t* __restrict__ table, const bf16_t* __restrict__ pos_table,
-                                 const int* __restrict__ tokens, const int* __restrict__ pos, int d, float* __restrict__ x) {
-  const int i = blockIdx.y;
-  const bf16_t* e = table + (size_t)tokens[i] * d;
-  const bf16_t* p = pos_table ? pos_table + (size_t)pos[i] * d : nullptr;
-  for (int k = (blockIdx.x * blockDim.x + threadIdx.x) * 4; k < d; k += gridDim.x * blockDim.x * 4) {
-    const uint2 u = *(const uint2*)(e + k);
-    float4 v = make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
-                           __uint_as_float(u.y & 0xffff0000u));
-    if (p) {
-      const uint2 w = *(const uint2*)(p + k);
-      v.x += __uint_as_float(w.x << 16);
-      v.y += __uint_as_float(w.x & 0xffff0000u);
-      v.z += __uint_as_float(w.y << 16);
-      v.w += __uint_as_float(w.y & 0xffff0000u);
-    }
-    *(float4*)(x + (size_t)i * d + k) = v;
-  }
-}
-void launch_embed_pos(const bf16_t* table, const bf16_t* pos_table, const int* tokens, const int* pos, int n, int d,
-                      float* x, hipStream_t st) {
-  hipLaunchKernelGGL(embed_pos_kernel, dim3((d / 4 + 255) / 256, n), dim3(256), 0, st, table, pos_table, tokens, pos, d, x);
-}
-
+// ---- layered decoders: row gather, weight transpose, fp32 GLU ---------------------------
 __global__ void gather_rows_kernel(const float* __restrict__ x, int d, const int* __restrict__ rows, float* __restrict__ y) {
   const float* s = x + (size_t)rows[blockIdx.x] * d;
   for (int k = threadIdx.x * 4; k < d; k += blockDim.x * 4) *(float4*)(y + (size_t)blockIdx.x * d + k) = *(const float4*)(s + k);

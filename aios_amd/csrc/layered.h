@@ -12,25 +12,42 @@
 
 #include "common.h"
 #include "latent.h"
+#include "mixers.h"
 #include "ops.h"
 
 namespace aios {
 
-enum MixerKind : int { MIX_LATENT = 1 };
-enum MlpKind : int { MLP_NONE = 0, MLP_GLU = 1 };
+enum MixerKind : int { MIX_LATENT = 1, MIX_MINGRU = 2 };
+enum MlpKind : int { MLP_NONE = 0, MLP_GLU = 1, MLP_MOE = 2 };
+enum OutGate : int { GATE_NONE = 0, GATE_ELEMENT = 1, GATE_HEAD = 2 };
 
-// One layer: a mixer and a feed-forward that read the same normalised input and are added to the
-// residual together (x += mixer(norm(x)) + mlp(norm(x))).
+// One layer: a mixer and a feed-forward.  Parallel: both read the same normalised input and are added to the
+// residual together (x += mixer(norm(x)) + mlp(norm(x))).  Otherwise one after the other, each
+//   x += post( f(h) * sigmoid(Wr h + br) ),  h = norm(x)
+// with the gate (resid_gate) and the norm of the result (post_norm) where the layer has them.
 struct LayerSpec {
   int mixer = MIX_LATENT;
-  int heads = 1, dim = 64, vdim = 64;  // query-key and value dimensions per head
-  int kv_rank = 64;                    // latent width (MIX_LATENT)
+  int parallel = 1;
+  int norm_scalar = 0;                 // norms of the sublayers: one number instead of one per column
+  int post_norm = 0, resid_gate = 0;
+  // MIX_LATENT
+  int heads = 1, dim = 64, vdim = 64;  // (unrotated) query-key and value dimensions per head
+  int kv_rank = 64;                    // latent width
+  int rot_dim = 0, rot_dims = 0;       // rotated query-key dimensions (0: none), the first rot_dims of which turn
+  double rot_base = 10000.0;
+  int window = 0;                      // keys a token sees, itself included (0: all before it)
   float scale = 0.125f;                // of q . k
   int sink = 1;                        // a learned logit per head joins the softmax's denominator
-  int out_gate = 1;                    // head outputs times sigmoid(Wg h)
+  int out_gate = GATE_ELEMENT;         // head outputs times sigmoid(Wg h): a number each, or one per head
+  // MIX_MINGRU
+  int width = 64;                      // of the state
   int mlp = MLP_GLU;
-  int ff = 256;
+  int ff = 256;                        // MLP_GLU: hidden width; MLP_MOE: of every expert
   int act = ACT_GELU_TANH;             // GluAct of the gate
+  int experts = 0, top = 0;            // MLP_MOE
+  int shared_ff = 0;                   // hidden width of the expert that runs for every token (0: none)
+  int correction = 0;                  // a learned number per expert joins the choice, not the weights
+  float router_scale = 1.f;
   int weights_of = -1;                 // layer whose weights this one uses (its cache is its own), or -1
 };
 
@@ -64,35 +81,67 @@ class LayeredDecoder {
   void collect(const std::vector<int>& rows, int at);  // x rows -> head input rows [at, ...)
   void head(int B, int from = 0);                      // logits of head input rows [from, from + B)
   std::vector<float> residual(int rows);               // host copy of x rows [0, rows), width columns
+  bool recurrent() const { return recurrent_; }        // a slot's state is more than its cached tokens
+  void copy_state(int src, int dst);                   // recurrent state and last tokens of a slot
+  int layer_runs() const { return (int)runs_.size(); }
+  void set_run_limit(int n) { run_limit_ = n; }        // stop after n layer runs (n < 0: all)
 
  private:
   struct Dims {
-    int H, dk, dv, rank, ff;
-    int dkp, dvp, rp, qn, gn, fp;  // padded; qn / gn: rows of all heads' queries / values
-    int n1, nin, kout;             // input projections without / with gate and up; columns of the output matrix
+    // latent attention; padded: dkp, dvp, rp.  A head's query is [dk | rotated at qrot], the cached row
+    // [latent | rotated at roff]; qn / gn: rows of all heads' queries / values (gn: columns the mixer leaves)
+    int H, dk, dv, rank, rot, qrot, roff, dkp, dvp, rp, qn, gn;
+    int wp;                   // minGRU: padded width
+    int ff, fp, shf, shp;     // feed-forward and shared expert, padded
+    int gate_off, rg_off;     // columns of the output gate and of the residual gate in the input product
+    int n1;                   // input product without gate / up
+    int nin, kout;            // parallel: with gate / up; columns of the joint output matrix
+    int n2, router_off, glu;  // sequential: the feed-forward's input product [residual gate | router], GLU width (padded)
   };
   struct Weights {
     bool own = false;
-    float *norm = nullptr, *kv_norm = nullptr, *sink = nullptr;
-    bf16_t *in = nullptr;    // [nin][dp]: q | kv down | output gate | gate / up interleaved
-    bf16_t *out = nullptr;   // [dp][kout]: attention output | MLP down
+    float *norm = nullptr, *norm2 = nullptr, *post = nullptr, *post2 = nullptr, *kv_norm = nullptr, *sink = nullptr;
+    float *rgb = nullptr, *rgb2 = nullptr, *zb = nullptr, *ub = nullptr, *corr = nullptr;
+    bf16_t *in = nullptr;    // parallel [nin][dp]: q | kv down | output gate | gate / up interleaved
+                             // sequential [n1][dp]: q | kv down | output gate | residual gate, or z | u | g | residual gate
+    bf16_t *out = nullptr;   // [dp][kout]: attention output | MLP down; sequential [dp][gn]
+    bf16_t *in2 = nullptr;   // [n2 + 2 glu][dp]: residual gate | router | gate / up interleaved
+    bf16_t *out2 = nullptr;  // [dp][glu]
+    bf16_t *egu = nullptr;   // [experts][2 fp][dp] gate / up interleaved
+    bf16_t *edn = nullptr;   // [experts][dp][fp]
     bf16_t *ukv = nullptr;   // [qn + gn][rp]: key | value up-projections
     bf16_t *ukT = nullptr;   // [H][rp][dkp]
   };
+  // one pass of one layer; a looped layer has a cache or state per pass
+  struct Run {
+    int layer, pass;         // pass: -1 outside the loop
+    char* pool;              // cache (latent attention)
+    float* state;            // [2][slots][wp] (minGRU)
+  };
   struct RowSet {
-    const int *tokens, *pos, *slot;
+    const int *tokens, *pos, *slot, *run;  // run: rows of the sequence from its first row (null: one each)
     int n, n_abs;                         // rows, rows on the absorbed path (they come first)
     bool decode;
     std::map<int, std::pair<int, int>> tiles;  // step batches: heads -> (first tile, count)
     int max_len;                          // of the absorbed rows
     std::vector<std::pair<int, Piece>> pf;  // expanded path: first row, piece
+    int n_chunks, split;                  // step batches: chunks of the recurrences
   };
-  void layer(int i, const RowSet& r);
-  void layer16(int i, const RowSet& r);
-  void layer32(int i, const RowSet& r);
-  void attention(int i, const RowSet& r);
+  void layer16(int k, const RowSet& r);  // k: run
+  void layer32(int k, const RowSet& r);
+  void layer_seq(int k, const RowSet& r);
+  void feed_forward(int k, const RowSet& r, RowCloseArgs& c);
+  void recurrence(int k, const RowSet& r);
+  void attention(int k, const RowSet& r);
   void run(const RowSet& r);
-  LatentAttnArgs latent_args(int i, const RowSet& r);
+  NextArgs next_of(int k, bool decode);  // what the residual becomes before run k (the head's input after the last)
+  RowCloseArgs close_args() const;
+  LatentAttnArgs latent_args(int k, const RowSet& r);
+  // y[n][N] (ldy) = operand rows x w^T, through the GEMV, the short or the prefill GEMM
+  void project(const void* a, int lda, const bf16_t* w, int n, int N, int K, float* y, int ldy);
+  void alloc_layer(int i);
+  std::vector<float> rope_table(int rot, int dims, double base) const;
+  int span(const Piece& p) const;        // keys the expanded path of a piece needs at most
   QWeight mat(const bf16_t* p, int rows, int cols) const;
   void gemm16(const bf16_t* A, int lda, const bf16_t* w, int M, int N, int K, int epi, float* C, int ldc, bf16_t* C16,
               int act = 0);
@@ -102,8 +151,8 @@ class LayeredDecoder {
   float* falloc(size_t n);
   void place(bf16_t* dst, int dpitch, const bf16_t* src, int spitch, int width, int height, bool device);
   void put(const std::string& name, int rows, int cols, const bf16_t* src, bool device);
-  void put_vec(float* dst, int n, const bf16_t* src, bool device);
-  std::vector<std::pair<std::string, std::pair<int, int>>> tensor_list() const;
+  void put_vec(float* dst, int n, const bf16_t* src, bool device, int spread = 0, float mul = 1.f);
+  void list_tensors();
   void tune();
 
   Engine& e_;
@@ -111,9 +160,15 @@ class LayeredDecoder {
   std::vector<Dims> dims_;
   std::vector<int> owner_;
   std::vector<Weights> w_;
-  std::vector<char*> pool_;
-  bf16_t *embd_ = nullptr, *posw_ = nullptr, *headw_ = nullptr;
-  float* out_norm_ = nullptr;
+  std::vector<Run> runs_;
+  bool seq_ = false, recurrent_ = false, head_ready_ = false;
+  int run_limit_ = -1, max_window_ = 0;  // max_window_: largest window, 0 if a layer has none
+  bf16_t *embd_ = nullptr, *posw_ = nullptr, *headw_ = nullptr, *pairw_ = nullptr, *loopw_ = nullptr;
+  float *out_norm_ = nullptr, *loop_step_ = nullptr;
+  std::vector<float2*> rope_;            // per layer
+  int* last_tok_ = nullptr;              // [2][slots]
+  std::vector<std::pair<std::string, std::pair<int, int>>> tensors_;  // name, (rows, columns)
+  std::map<std::string, std::pair<int, int>> shape_;
   std::set<std::string> have_;
 
   int step_rows_ = 0, pf_min_ = 0, pf_max_ctx_ = 0;
@@ -122,6 +177,12 @@ class LayeredDecoder {
         *cat32_ = nullptr;
   bf16_t *h16_ = nullptr, *cat16_ = nullptr, *cfull_ = nullptr, *kv_ = nullptr;
   void* qa_ = nullptr;
+  // sequential layers: sublayer result, loop entry operand [rows][2 dp], recurrences' chunk transitions, experts
+  float *y_ = nullptr, *agg_ = nullptr, *moe_wt_ = nullptr, *moe_gu32_ = nullptr;
+  void *xin_ = nullptr, *moe_act_ = nullptr, *moe_ye_ = nullptr;
+  int *moe_sel_ = nullptr, *moe_pair_ = nullptr, *moe_token_ = nullptr, *moe_ntiles_ = nullptr;
+  int4* moe_tiles_ = nullptr;
+  int moe_max_tiles_ = 0;
   // RMSNorm split across the short GEMMs (GemmQArgs nrm_*): set when the residual in x_ already went
   // through bf16(x * g_next) and per-tile sums
   bf16_t* xn16_ = nullptr;
@@ -131,7 +192,9 @@ class LayeredDecoder {
   // step parameters: one pinned block, one copy
   int *h_step_ = nullptr, *d_step_ = nullptr;
   size_t step_ints_ = 0;
-  int *st_tokens_ = nullptr, *st_pos_ = nullptr, *st_slot_ = nullptr, *st_want_ = nullptr;
+  int *st_tokens_ = nullptr, *st_pos_ = nullptr, *st_slot_ = nullptr, *st_want_ = nullptr, *st_run_ = nullptr;
+  ScanChunk* st_chunks_ = nullptr;
+  int max_chunks_ = 0;
   LatentTile* st_tiles_ = nullptr;
 };
 

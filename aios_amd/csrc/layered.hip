@@ -6,6 +6,10 @@
 //               [attention out | MLP down] adding to the residual          -- 5 launches
 //   5-64 rows   the same two products through the skinny MFMA GEMM, the RMSNorm split across them
 //   more rows   prefill GEMMs; long portions take the expanded attention (latent.h)
+// Sequential layers (mixer, then feed-forward, each closed by its residual gate and norms): every product reads a
+// bf16 operand that the row operation before it wrote (mixers.h), so a layer is
+//   input product (+ residual gate rows) | mixer | output product | close | input product (+ residual gate and
+//   router rows, GLU in its epilogue) | experts | down product | close
 // 32-bit engine: the same steps in fp32, absorbed attention for every row.
 #include "layered.h"
 
@@ -20,15 +24,17 @@
 namespace aios {
 
 static int up(int x, int a) { return (x + a - 1) / a * a; }
+// rows of a product of its own: whole tiles of the prefill GEMM
+static int up_n(int x) { return x <= 1024 ? up(x, 128) : up(x, 256); }
 static int env_or(const char* name, int dflt) {
   const char* e = std::getenv(name);
   return e ? std::atoi(e) : dflt;
 }
 // padded latent widths the attention kernels are built for
 static int pad_rank(int r) {
-  for (int t : {2, 4, 6, 8, 12, 16, 32})
+  for (int t : {2, 4, 6, 8, 10, 12, 16, 32})
     if (r <= 64 * t) return 64 * t;
-  throw std::runtime_error("latent attention: kv_rank above 2048");
+  throw std::runtime_error("latent attention: cached rows above 2048 numbers");
 }
 
 LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
@@ -39,12 +45,19 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
   v_ = c.vocab_size;
   vp_ = up(v_, 64);
   f32_ = c.compute_f32;
-  if (d_ < 1 || v_ < 1 || c.max_positions < 1) throw std::runtime_error("layered model: bad sizes");
+  if (d_ < 1 || v_ < 1 || c.max_positions < 0 || c.max_ctx < 1) throw std::runtime_error("layered model: bad sizes");
   if (c.tp_size > 1) throw std::runtime_error("layered models run on one GPU (no tensor parallelism)");
   if (c.kv_fp8) throw std::runtime_error("layered models: the latent cache has no fp8 form");
+  if (c.loop_times > 0 && !(c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= nl_))
+    throw std::runtime_error("layered model: bad loop");
+  if (c.bigram_buckets < 0) throw std::runtime_error("layered model: bad pair table");
+  seq_ = !c.layers[0].parallel;
+  recurrent_ = c.bigram_buckets > 0;
   dims_.resize(nl_);
   owner_.resize(nl_);
   w_.resize(nl_);
+  rope_.assign(nl_, nullptr);
+  bool all_windowed = true;
   for (int i = 0; i < nl_; ++i) {
     int o = i;
     for (int hop = 0; c.layers[o].weights_of >= 0; ++hop) {
@@ -53,47 +66,128 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
     }
     owner_[i] = o;
     const LayerSpec &s = c.layers[i], &t = c.layers[o];
-    if (s.mixer != MIX_LATENT) throw std::runtime_error("unknown mixer kind");
-    if (s.heads != t.heads || s.dim != t.dim || s.vdim != t.vdim || s.kv_rank != t.kv_rank || s.mlp != t.mlp ||
-        (s.mlp != MLP_NONE && s.ff != t.ff))
-      throw std::runtime_error("layer " + std::to_string(i) + ": sizes differ from the layer whose weights it uses");
-    if (s.heads < 1 || s.dim < 1 || s.vdim < 1 || s.kv_rank < 1 || (s.mlp != MLP_NONE && s.ff < 1))
-      throw std::runtime_error("layer " + std::to_string(i) + ": bad sizes");
+    const std::string at = "layer " + std::to_string(i) + ": ";
+    if (!s.parallel != seq_) throw std::runtime_error(at + "parallel and sequential layers in one model");
+    if (s.mixer != t.mixer || s.heads != t.heads || s.dim != t.dim || s.vdim != t.vdim || s.kv_rank != t.kv_rank ||
+        s.rot_dim != t.rot_dim || s.out_gate != t.out_gate || s.sink != t.sink || s.width != t.width || s.mlp != t.mlp ||
+        s.post_norm != t.post_norm || s.resid_gate != t.resid_gate || s.norm_scalar != t.norm_scalar ||
+        (s.mlp != MLP_NONE && (s.ff != t.ff || s.experts != t.experts || s.shared_ff != t.shared_ff || s.correction != t.correction)))
+      throw std::runtime_error(at + "sizes differ from the layer whose weights it uses");
+    if (s.mlp != MLP_NONE && s.ff < 1) throw std::runtime_error(at + "bad sizes");
+    if (s.mlp == MLP_MOE && (s.experts < 1 || s.experts > MOE_MAX_EXPERTS || s.top < 1 || s.top > std::min(s.experts, MOE_MAX_TOP) ||
+                             s.shared_ff < 0))
+      throw std::runtime_error(at + "bad number of experts");
+    if (s.parallel && (s.mixer != MIX_LATENT || s.mlp == MLP_MOE || s.post_norm || s.resid_gate))
+      throw std::runtime_error(at + "a parallel layer is latent attention beside a dense MLP");
     Dims& D = dims_[i];
-    D.H = s.heads;
-    D.dk = s.dim;
-    D.dv = s.vdim;
-    D.rank = s.kv_rank;
+    std::memset(&D, 0, sizeof(D));
+    int n;  // columns of the mixer's input product
+    if (s.mixer == MIX_LATENT) {
+      if (s.heads < 1 || s.dim < 1 || s.vdim < 1 || s.kv_rank < 1 || s.window < 0) throw std::runtime_error(at + "bad sizes");
+      if (s.rot_dim < 0 || s.rot_dim % 2 || s.rot_dims < 0 || s.rot_dims % 2 || s.rot_dims > s.rot_dim)
+        throw std::runtime_error(at + "bad rotated dimensions");
+      D.H = s.heads;
+      D.dk = s.dim;
+      D.dv = s.vdim;
+      D.rank = s.kv_rank;
+      D.rot = s.rot_dim;
+      D.qrot = up(D.dk, 8);
+      D.roff = up(D.rank, 8);
+      D.dkp = up(D.rot ? D.qrot + D.rot : D.dk, 32);
+      D.dvp = up(D.dv, 32);
+      D.rp = pad_rank(D.rot ? D.roff + D.rot : D.rank);
+      D.qn = up(D.H * D.dkp, 64);
+      D.gn = up(D.H * D.dvp, 64);
+      D.gate_off = D.qn + D.rp;
+      n = D.gate_off + (s.out_gate == GATE_ELEMENT ? D.gn : s.out_gate == GATE_HEAD ? up(D.H, 64) : 0);
+      if (s.window) max_window_ = std::max(max_window_, s.window);
+      else all_windowed = false;
+    } else if (s.mixer == MIX_MINGRU) {
+      if (s.width < 1) throw std::runtime_error(at + "bad sizes");
+      D.wp = up(s.width, 64);
+      D.gn = D.wp;
+      n = 3 * D.wp;
+      recurrent_ = true;
+    } else {
+      throw std::runtime_error("unknown mixer kind");
+    }
     D.ff = s.mlp != MLP_NONE ? s.ff : 0;
-    D.dkp = up(D.dk, 32);
-    D.dvp = up(D.dv, 32);
-    D.rp = pad_rank(D.rank);
-    D.qn = up(D.H * D.dkp, 64);
-    D.gn = up(D.H * D.dvp, 64);
     D.fp = up(D.ff, 64);
-    D.n1 = D.qn + D.rp + D.gn;
-    D.nin = D.n1 + 2 * D.fp;
-    D.kout = D.gn + D.fp;
+    if (s.parallel) {
+      D.n1 = n;
+      D.nin = D.n1 + 2 * D.fp;
+      D.kout = D.gn + D.fp;
+      continue;
+    }
+    D.rg_off = n;
+    D.n1 = up_n(n + (s.resid_gate ? dp_ : 0));
+    D.kout = D.gn;
+    D.shf = s.mlp == MLP_MOE ? s.shared_ff : 0;
+    D.shp = up(D.shf, 64);
+    D.glu = s.mlp == MLP_MOE ? D.shp : D.fp;
+    D.router_off = s.resid_gate ? dp_ : 0;
+    D.n2 = up_n(D.router_off + (s.mlp == MLP_MOE ? up(s.experts, 64) : 0));
   }
+  if (!all_windowed) max_window_ = 0;
+  for (int i = 0; i < nl_; ++i) {
+    const bool looped = c.loop_times > 0 && i >= c.loop_start && i < c.loop_stop;
+    if (looped && i == c.loop_start)
+      for (int t = 0; t < c.loop_times; ++t)
+        for (int j = c.loop_start; j < c.loop_stop; ++j) runs_.push_back({j, t, nullptr, nullptr});
+    if (!looped) runs_.push_back({i, -1, nullptr, nullptr});
+  }
+  if (c.loop_times > 0 && !seq_) throw std::runtime_error("layered model: a loop of parallel layers");
   embd_ = balloc((size_t)v_ * dp_);
-  posw_ = balloc((size_t)c.max_positions * dp_);
+  if (c.max_positions) posw_ = balloc((size_t)c.max_positions * dp_);
+  if (c.bigram_buckets) pairw_ = balloc((size_t)(c.bigram_buckets + 1) * dp_);
+  if (c.loop_times > 0) {
+    loopw_ = balloc((size_t)dp_ * 2 * dp_);
+    loop_step_ = falloc((size_t)c.loop_times * dp_);
+  }
   headw_ = balloc((size_t)vp_ * dp_);
   out_norm_ = falloc(dp_);
-  for (int i = 0; i < nl_; ++i) {
-    if (owner_[i] != i) continue;
-    const Dims& D = dims_[i];
-    Weights& w = w_[i];
-    w.own = true;
-    w.norm = falloc(dp_);
+  for (int i = 0; i < nl_; ++i)
+    if (owner_[i] == i) alloc_layer(i);
+  e_.weight_bytes_ = 0;
+  list_tensors();
+  for (const auto& t : tensors_) e_.weight_bytes_ += (size_t)t.second.first * t.second.second * 2;
+}
+
+void LayeredDecoder::alloc_layer(int i) {
+  const Dims& D = dims_[i];
+  const LayerSpec& s = e_.cfg_.layers[i];
+  Weights& w = w_[i];
+  w.own = true;
+  w.norm = falloc(dp_);
+  if (s.mixer == MIX_LATENT) {
     w.kv_norm = falloc(D.rp);
     w.sink = falloc(D.H);
-    w.in = balloc((size_t)D.nin * dp_);
-    w.out = balloc((size_t)dp_ * D.kout);
     w.ukv = balloc((size_t)(D.qn + D.gn) * D.rp);
     w.ukT = balloc((size_t)D.H * D.rp * D.dkp);
+  } else {
+    w.zb = falloc(D.wp);
+    w.ub = falloc(D.wp);
   }
-  e_.weight_bytes_ = 0;
-  for (const auto& t : tensor_list()) e_.weight_bytes_ += (size_t)t.second.first * t.second.second * 2;
+  if (s.parallel) {
+    w.in = balloc((size_t)D.nin * dp_);
+    w.out = balloc((size_t)dp_ * D.kout);
+    return;
+  }
+  w.in = balloc((size_t)D.n1 * dp_);
+  w.out = balloc((size_t)dp_ * D.kout);
+  if (s.post_norm) w.post = falloc(dp_);
+  if (s.resid_gate) w.rgb = falloc(dp_);
+  if (s.mlp == MLP_NONE) return;
+  w.norm2 = falloc(dp_);
+  if (s.post_norm) w.post2 = falloc(dp_);
+  if (s.resid_gate) w.rgb2 = falloc(dp_);
+  w.in2 = balloc((size_t)(D.n2 + 2 * D.glu) * dp_);
+  if (D.glu) w.out2 = balloc((size_t)dp_ * D.glu);
+  if (s.mlp == MLP_MOE) {
+    w.corr = falloc(s.experts);
+    w.egu = balloc((size_t)s.experts * 2 * D.fp * dp_);
+    w.edn = balloc((size_t)s.experts * dp_ * D.fp);
+  }
 }
 
 LayeredDecoder::~LayeredDecoder() {
@@ -119,7 +213,8 @@ void LayeredDecoder::place(bf16_t* dst, int dpitch, const bf16_t* src, int spitc
                         device ? hipMemcpyDeviceToDevice : hipMemcpyHostToDevice));
 }
 
-void LayeredDecoder::put_vec(float* dst, int n, const bf16_t* src, bool device) {
+// src's n numbers times `mul`, or (spread > 0) its one number that many times
+void LayeredDecoder::put_vec(float* dst, int n, const bf16_t* src, bool device, int spread, float mul) {
   std::vector<bf16_t> h(n);
   std::vector<float> f(n);
   if (device) HIP_CHECK(hipMemcpy(h.data(), src, (size_t)n * 2, hipMemcpyDeviceToHost));
@@ -127,105 +222,198 @@ void LayeredDecoder::put_vec(float* dst, int n, const bf16_t* src, bool device) 
   for (int i = 0; i < n; ++i) {
     const uint32_t u = (uint32_t)h[i] << 16;
     std::memcpy(&f[i], &u, 4);
+    f[i] *= mul;
   }
-  HIP_CHECK(hipMemcpy(dst, f.data(), (size_t)n * 4, hipMemcpyHostToDevice));
+  if (spread > 0) f.assign(spread, f[0]);
+  HIP_CHECK(hipMemcpy(dst, f.data(), f.size() * 4, hipMemcpyHostToDevice));
 }
 
 // every tensor of the model: name, (rows, cols)
-std::vector<std::pair<std::string, std::pair<int, int>>> LayeredDecoder::tensor_list() const {
-  std::vector<std::pair<std::string, std::pair<int, int>>> t;
-  auto add = [&](const std::string& n, int r, int c) { t.push_back({n, {r, c}}); };
+void LayeredDecoder::list_tensors() {
+  const EngineConfig& c = e_.cfg_;
+  auto add = [&](const std::string& n, int r, int cl) {
+    tensors_.push_back({n, {r, cl}});
+    shape_[n] = {r, cl};
+  };
+  const int norm_final = c.layers[0].norm_scalar ? 1 : d_;
   add("token_embd.weight", v_, d_);
-  add("position_embd.weight", e_.cfg_.max_positions, d_);
-  add("output_norm.weight", 1, d_);
+  if (posw_) add("position_embd.weight", c.max_positions, d_);
+  if (pairw_) add("bigram_embd.weight", c.bigram_buckets + 1, d_);
+  if (loopw_) {
+    add("loop_in.weight", d_, 2 * d_);
+    add("loop_step.weight", c.loop_times, d_);
+  }
+  add("output_norm.weight", 1, norm_final);
   add("output.weight", v_, d_);
   for (int i = 0; i < nl_; ++i) {
     if (owner_[i] != i) continue;
     const Dims& D = dims_[i];
-    const LayerSpec& s = e_.cfg_.layers[i];
+    const LayerSpec& s = c.layers[i];
     const std::string p = "blk." + std::to_string(i) + ".";
-    add(p + "attn_norm.weight", 1, d_);
-    add(p + "attn_q.weight", D.H * D.dk, d_);
-    add(p + "attn_kv_a.weight", D.rank, d_);
-    add(p + "attn_kv_a_norm.weight", 1, D.rank);
-    add(p + "attn_k_b.weight", D.H * D.dk, D.rank);
-    add(p + "attn_v_b.weight", D.H * D.dv, D.rank);
-    if (s.sink) add(p + "attn_sinks.weight", 1, D.H);
-    if (s.out_gate) add(p + "attn_gate.weight", D.H * D.dv, d_);
-    add(p + "attn_output.weight", d_, D.H * D.dv);
-    if (D.ff) {
+    const int nw = s.norm_scalar ? 1 : d_;
+    add(p + "attn_norm.weight", 1, nw);
+    if (s.mixer == MIX_LATENT) {
+      add(p + "attn_q.weight", D.H * (D.dk + D.rot), d_);
+      add(p + "attn_kv_a.weight", D.rank + D.rot, d_);
+      add(p + "attn_kv_a_norm.weight", 1, D.rank);
+      add(p + "attn_k_b.weight", D.H * D.dk, D.rank);
+      add(p + "attn_v_b.weight", D.H * D.dv, D.rank);
+      if (s.sink) add(p + "attn_sinks.weight", 1, D.H);
+      if (s.out_gate) add(p + "attn_gate.weight", s.out_gate == GATE_HEAD ? D.H : D.H * D.dv, d_);
+      add(p + "attn_output.weight", d_, D.H * D.dv);
+    } else {
+      for (const char* n : {"z", "x"}) {
+        add(p + "rnn_" + n + ".weight", s.width, d_);
+        add(p + "rnn_" + n + ".bias", 1, s.width);
+      }
+      add(p + "rnn_gate.weight", s.width, d_);
+      add(p + "rnn_output.weight", d_, s.width);
+    }
+    auto closing = [&](const std::string& sub) {
+      if (s.post_norm) add(p + sub + "_post_norm.weight", 1, nw);
+      if (s.resid_gate) {
+        add(p + sub + "_resid_gate.weight", d_, d_);
+        add(p + sub + "_resid_gate.bias", 1, d_);
+      }
+    };
+    if (!s.parallel) closing("attn");
+    if (s.mlp == MLP_NONE) continue;
+    if (!s.parallel) {
+      add(p + "ffn_norm.weight", 1, nw);
+      closing("ffn");
+    }
+    if (s.mlp == MLP_GLU) {
       add(p + "ffn_gate.weight", D.ff, d_);
       add(p + "ffn_up.weight", D.ff, d_);
       add(p + "ffn_down.weight", d_, D.ff);
+      continue;
+    }
+    add(p + "ffn_gate_inp.weight", s.experts, d_);
+    if (s.correction) add(p + "exp_probs_b.bias", 1, s.experts);
+    if (s.shared_ff) {
+      add(p + "ffn_gate_shexp.weight", D.shf, d_);
+      add(p + "ffn_up_shexp.weight", D.shf, d_);
+      add(p + "ffn_down_shexp.weight", d_, D.shf);
+    }
+    for (int x = 0; x < s.experts; ++x) {
+      const std::string n = "." + std::to_string(x) + ".weight";
+      add(p + "ffn_gate" + n, D.ff, d_);
+      add(p + "ffn_up" + n, D.ff, d_);
+      add(p + "ffn_down" + n, d_, D.ff);
     }
   }
-  return t;
 }
 
 void LayeredDecoder::put(const std::string& name, int rows, int cols, const bf16_t* src, bool device) {
+  const EngineConfig& c = e_.cfg_;
   if (name == "token_embd.weight") return place(embd_, dp_, src, cols, cols, rows, device);
   if (name == "position_embd.weight") return place(posw_, dp_, src, cols, cols, rows, device);
+  if (name == "bigram_embd.weight") return place(pairw_, dp_, src, cols, cols, rows, device);
   if (name == "output.weight") return place(headw_, dp_, src, cols, cols, rows, device);
-  if (name == "output_norm.weight") return put_vec(out_norm_, cols, src, device);
+  // (the logits' scale goes with the norm before the head)
+  if (name == "output_norm.weight") return put_vec(out_norm_, cols, src, device, cols < d_ ? d_ : 0, c.logit_scale);
+  if (name == "loop_in.weight") {
+    place(loopw_, 2 * dp_, src, cols, d_, rows, device);
+    return place(loopw_ + dp_, 2 * dp_, src + d_, cols, d_, rows, device);
+  }
+  if (name == "loop_step.weight") {
+    for (int t = 0; t < rows; ++t) put_vec(loop_step_ + (size_t)t * dp_, cols, src + (size_t)t * cols, device);
+    return;
+  }
   const size_t dot = name.find('.', 4);
   const int i = std::stoi(name.substr(4, dot - 4));
   const std::string t = name.substr(dot + 1);
   const Dims& D = dims_[i];
+  const LayerSpec& s = c.layers[i];
   Weights& w = w_[i];
-  // heads of per_head rows each, spread to pad rows each
-  auto heads = [&](bf16_t* dst, int dpitch, int per_head, int pad) {
+  // heads of per_head rows each, `take` of them from row `from` spread to pad rows each
+  auto heads = [&](bf16_t* dst, int dpitch, int per_head, int pad, int from = 0, int take = -1) {
     for (int h = 0; h < D.H; ++h)
-      place(dst + (size_t)h * pad * dpitch, dpitch, src + (size_t)h * per_head * cols, cols, cols, per_head, device);
+      place(dst + (size_t)h * pad * dpitch, dpitch, src + ((size_t)h * per_head + from) * cols, cols, cols,
+            take < 0 ? per_head : take, device);
   };
-  if (t == "attn_norm.weight") put_vec(w.norm, cols, src, device);
+  auto rows_at = [&](bf16_t* m, int row) { place(m + (size_t)row * dp_, dp_, src, cols, cols, rows, device); };
+  auto norm = [&](float* dst) { put_vec(dst, cols, src, device, cols < d_ ? d_ : 0); };
+  auto glu = [&](bf16_t* m, int row0, int up_row) {  // gate and up rows interleaved from row0
+    place(m + (size_t)(row0 + up_row) * dp_, 2 * dp_, src, cols, cols, rows, device);
+  };
+  bf16_t* gu = s.parallel ? w.in : w.in2;
+  const int gu0 = s.parallel ? D.n1 : D.n2;
+  if (t == "attn_norm.weight") norm(w.norm);
+  else if (t == "ffn_norm.weight") norm(w.norm2);
+  else if (t == "attn_post_norm.weight") norm(w.post);
+  else if (t == "ffn_post_norm.weight") norm(w.post2);
   else if (t == "attn_kv_a_norm.weight") put_vec(w.kv_norm, cols, src, device);
   else if (t == "attn_sinks.weight") put_vec(w.sink, cols, src, device);
-  else if (t == "attn_q.weight") heads(w.in, dp_, D.dk, D.dkp);
-  else if (t == "attn_kv_a.weight") place(w.in + (size_t)D.qn * dp_, dp_, src, cols, cols, rows, device);
-  else if (t == "attn_gate.weight") heads(w.in + (size_t)(D.qn + D.rp) * dp_, dp_, D.dv, D.dvp);
-  else if (t == "ffn_gate.weight") place(w.in + (size_t)D.n1 * dp_, 2 * dp_, src, cols, cols, rows, device);
-  else if (t == "ffn_up.weight") place(w.in + (size_t)(D.n1 + 1) * dp_, 2 * dp_, src, cols, cols, rows, device);
+  else if (t == "attn_q.weight") {
+    heads(w.in, dp_, D.dk + D.rot, D.dkp, 0, D.dk);
+    if (D.rot) heads(w.in + (size_t)D.qrot * dp_, dp_, D.dk + D.rot, D.dkp, D.dk, D.rot);
+  } else if (t == "attn_kv_a.weight") {
+    place(w.in + (size_t)D.qn * dp_, dp_, src, cols, cols, D.rank, device);
+    if (D.rot) place(w.in + (size_t)(D.qn + D.roff) * dp_, dp_, src + (size_t)D.rank * cols, cols, cols, D.rot, device);
+  } else if (t == "attn_gate.weight") {
+    if (s.out_gate == GATE_HEAD) rows_at(w.in, D.gate_off);
+    else heads(w.in + (size_t)D.gate_off * dp_, dp_, D.dv, D.dvp);
+  } else if (t == "rnn_z.weight") rows_at(w.in, 0);
+  else if (t == "rnn_x.weight") rows_at(w.in, D.wp);
+  else if (t == "rnn_gate.weight") rows_at(w.in, 2 * D.wp);
+  else if (t == "rnn_z.bias") put_vec(w.zb, cols, src, device);
+  else if (t == "rnn_x.bias") put_vec(w.ub, cols, src, device);
+  else if (t == "rnn_output.weight") place(w.out, D.kout, src, cols, cols, rows, device);
+  else if (t == "attn_resid_gate.weight") rows_at(w.in, D.rg_off);
+  else if (t == "ffn_resid_gate.weight") rows_at(w.in2, 0);
+  else if (t == "attn_resid_gate.bias") put_vec(w.rgb, cols, src, device);
+  else if (t == "ffn_resid_gate.bias") put_vec(w.rgb2, cols, src, device);
+  else if (t == "ffn_gate_inp.weight") rows_at(w.in2, D.router_off);
+  else if (t == "exp_probs_b.bias") put_vec(w.corr, cols, src, device);
+  else if (t == "ffn_gate.weight" || t == "ffn_gate_shexp.weight") glu(gu, gu0, 0);
+  else if (t == "ffn_up.weight" || t == "ffn_up_shexp.weight") glu(gu, gu0, 1);
   else if (t == "attn_k_b.weight") heads(w.ukv, D.rp, D.dk, D.dkp);
   else if (t == "attn_v_b.weight") heads(w.ukv + (size_t)D.qn * D.rp, D.rp, D.dv, D.dvp);
   else if (t == "attn_output.weight")
     for (int h = 0; h < D.H; ++h) place(w.out + (size_t)h * D.dvp, D.kout, src + (size_t)h * D.dv, cols, D.dv, rows, device);
-  else if (t == "ffn_down.weight") place(w.out + D.gn, D.kout, src, cols, cols, rows, device);
-  else throw std::runtime_error("unknown layer tensor " + name);
+  else if (t == "ffn_down.weight" && s.parallel) place(w.out + D.gn, D.kout, src, cols, cols, rows, device);
+  else if (t == "ffn_down.weight" || t == "ffn_down_shexp.weight") place(w.out2, D.glu, src, cols, cols, rows, device);
+  else if (t.compare(0, 4, "ffn_") == 0 && s.mlp == MLP_MOE) {  // ffn_{gate,up,down}.<expert>.weight
+    const size_t d1 = t.find('.');
+    const int x = std::stoi(t.substr(d1 + 1));
+    const std::string kind = t.substr(0, d1);
+    if (kind == "ffn_down") place(w.edn + (size_t)x * dp_ * D.fp, D.fp, src, cols, cols, rows, device);
+    else glu(w.egu + (size_t)x * 2 * D.fp * dp_, 0, kind == "ffn_up");
+  } else throw std::runtime_error("unknown layer tensor " + name);
 }
 
 void LayeredDecoder::set_tensor(const std::string& name, int qt, int rows, int cols, const void* host, size_t nbytes) {
   if (qt != QT_BF16) throw std::runtime_error(name + ": layered models load bf16 tensors");
   if (nbytes != (size_t)rows * cols * 2) throw std::runtime_error(name + ": byte size mismatch");
-  for (const auto& t : tensor_list())
-    if (t.first == name) {
-      if (t.second.first != rows || t.second.second != cols)
-        throw std::runtime_error(name + ": shape " + std::to_string(rows) + " x " + std::to_string(cols) + ", expected " +
-                                 std::to_string(t.second.first) + " x " + std::to_string(t.second.second));
-      put(name, rows, cols, (const bf16_t*)host, false);
-      have_.insert(name);
-      return;
-    }
-  throw std::runtime_error("unknown tensor " + name);
+  const auto t = shape_.find(name);
+  if (t == shape_.end()) throw std::runtime_error("unknown tensor " + name);
+  if (t->second.first != rows || t->second.second != cols)
+    throw std::runtime_error(name + ": shape " + std::to_string(rows) + " x " + std::to_string(cols) + ", expected " +
+                             std::to_string(t->second.first) + " x " + std::to_string(t->second.second));
+  put(name, rows, cols, (const bf16_t*)host, false);
+  have_.insert(name);
 }
 
 void LayeredDecoder::init_random(uint64_t seed) {
   uint64_t s = seed * 1000003ULL;
-  for (const auto& t : tensor_list()) {
+  for (const auto& t : tensors_) {
     const int rows = t.second.first, cols = t.second.second;
     const size_t n = (size_t)rows * cols;
     const bool norm = t.first.find("norm") != std::string::npos, sink = t.first.find("sinks") != std::string::npos;
+    const bool bias = t.first.find(".bias") != std::string::npos;
     bf16_t* tmp = nullptr;
-    if (norm || sink) {
+    if (norm || sink || bias) {
       float* f = nullptr;
       HIP_CHECK(hipMalloc(&f, n * 4));
       HIP_CHECK(hipMalloc(&tmp, n * 2 + 16));
-      fill_random_f32(f, n, ++s, norm ? 1.f : 0.f, norm ? 0.1f : 1.f, e_.stream_);
+      fill_random_f32(f, n, ++s, norm ? 1.f : 0.f, norm ? 0.1f : bias ? 0.05f : 1.f, e_.stream_);
       launch_f32_to_bf16(f, tmp, n, e_.stream_);
       HIP_CHECK(hipStreamSynchronize(e_.stream_));
       HIP_CHECK(hipFree(f));
     } else {
       HIP_CHECK(hipMalloc(&tmp, n * 2));
-      fill_random_weight(mat(tmp, rows, cols), ++s, t.first == "token_embd.weight" ? 1.f : 0.02f, e_.stream_);
+      fill_random_weight(mat(tmp, rows, cols), ++s, t.first == "token_embd.weight" || t.first == "bigram_embd.weight" ? 1.f : 0.02f, e_.stream_);
       HIP_CHECK(hipStreamSynchronize(e_.stream_));
     }
     put(t.first, rows, cols, tmp, true);
@@ -237,7 +425,7 @@ void LayeredDecoder::init_random(uint64_t seed) {
 
 std::vector<std::string> LayeredDecoder::missing() const {
   std::vector<std::string> m;
-  for (const auto& t : tensor_list())
+  for (const auto& t : tensors_)
     if (!have_.count(t.first)) m.push_back(t.first);
   return m;
 }
@@ -252,35 +440,87 @@ QWeight LayeredDecoder::mat(const bf16_t* p, int rows, int cols) const {
 }
 
 // ---- workspace ----------------------------------------------------------------------------------------
+// (cos, sin) of every position and pair; pairs past `dims` do not turn
+std::vector<float> LayeredDecoder::rope_table(int rot, int dims, double base) const {
+  const int half = rot / 2, n = e_.cfg_.max_ctx;
+  std::vector<float> t((size_t)n * half * 2);
+  for (int i = 0; i < half; ++i) {
+    const double f = 2 * i < dims ? std::pow(base, -2.0 * i / dims) : 0.0;
+    for (int p = 0; p < n; ++p) {
+      t[((size_t)p * half + i) * 2] = (float)std::cos(p * f);
+      t[((size_t)p * half + i) * 2 + 1] = (float)std::sin(p * f);
+    }
+  }
+  return t;
+}
+
 void LayeredDecoder::finalize() {
   const EngineConfig& c = e_.cfg_;
   const int Bm = c.max_batch;
   hipStream_t st = e_.stream_;
-  for (int i = 0; i < nl_; ++i)
-    if (w_[i].own) launch_transpose_heads(w_[i].ukv, dims_[i].H, dims_[i].dkp, dims_[i].rp, w_[i].ukT, st);
-  // cache pools: one per layer (weights may be shared, the cached vectors are not)
-  const int es = f32_ ? 4 : 2;
-  pool_.resize(nl_);
-  e_.kv_bytes_ = 0;
+  std::map<std::pair<std::pair<int, int>, double>, float2*> ropes;
   for (int i = 0; i < nl_; ++i) {
-    const size_t block = (size_t)e_.kvb_ * dims_[i].rp * es, bytes = (size_t)(e_.kv_nblocks_ + 1) * block;
-    pool_[i] = (char*)e_.dmalloc(bytes);
-    HIP_CHECK(hipMemset(pool_[i], 0, bytes));
-    e_.pools_.push_back({pool_[i], block});
+    const Dims& D = dims_[i];
+    const LayerSpec& s = c.layers[i];
+    if (s.mixer != MIX_LATENT) continue;
+    if (D.rot) {
+      float2*& t = ropes[{{s.rot_dim, s.rot_dims}, s.rot_base}];
+      if (!t) {
+        const std::vector<float> h = rope_table(s.rot_dim, s.rot_dims, s.rot_base);
+        t = (float2*)e_.dmalloc(h.size() * 4);
+        HIP_CHECK(hipMemcpy(t, h.data(), h.size() * 4, hipMemcpyHostToDevice));
+      }
+      rope_[i] = t;
+    }
+    if (!w_[i].own) continue;
+    if (D.rot) {  // the rotated part of the cached row is a head's rotated key as it is
+      std::vector<bf16_t> one((size_t)D.rot * D.rot, 0);
+      for (int k = 0; k < D.rot; ++k) one[(size_t)k * D.rot + k] = 0x3f80;
+      for (int h = 0; h < D.H; ++h)
+        place(w_[i].ukv + ((size_t)h * D.dkp + D.qrot) * D.rp + D.roff, D.rp, one.data(), D.rot, D.rot, D.rot, false);
+    }
+    launch_transpose_heads(w_[i].ukv, D.H, D.dkp, D.rp, w_[i].ukT, st);
+  }
+  // a cache pool or a state per run (weights may be shared, what they leave behind is not)
+  const int es = f32_ ? 4 : 2;
+  e_.kv_bytes_ = 0;
+  for (Run& k : runs_) {
+    const Dims& D = dims_[k.layer];
+    if (c.layers[k.layer].mixer == MIX_MINGRU) {
+      k.state = falloc((size_t)2 * c.max_slots * D.wp);
+      e_.kv_bytes_ += (size_t)2 * c.max_slots * D.wp * 4;
+      continue;
+    }
+    const size_t block = (size_t)e_.kvb_ * D.rp * es, bytes = (size_t)(e_.kv_nblocks_ + 1) * block;
+    k.pool = (char*)e_.dmalloc(bytes);
+    HIP_CHECK(hipMemset(k.pool, 0, bytes));
+    e_.pools_.push_back({k.pool, block});
     e_.kv_bytes_ += bytes;
   }
+  if (pairw_) last_tok_ = (int*)falloc((size_t)2 * c.max_slots);
   step_rows_ = std::max(Bm, std::min(2048, c.max_slots * c.max_ctx));
   if (const char* v = std::getenv("AIOS_STEP_ROWS")) step_rows_ = std::max(Bm, std::atoi(v));
   const int R = step_rows_;
-  int n1 = 0, nin = 0, kout = 0, fp = 0, maxH = 0;
+  int n1 = 0, nin = 0, kout = 0, fp = 0, wp = 0;
   size_t qa = 0, part = 0, kvw = 0, flat = 0;
+  size_t e_act = 0, e_gu = 0, pairs = 0;  // experts
   int rp = 0;
-  for (const Dims& D : dims_) {
-    n1 = std::max(n1, D.n1);
-    nin = std::max(nin, D.nin);
-    kout = std::max(kout, D.kout);
-    fp = std::max(fp, D.fp);
-    maxH = std::max(maxH, D.H);
+  for (int i = 0; i < nl_; ++i) {
+    const Dims& D = dims_[i];
+    const LayerSpec& s = c.layers[i];
+    n1 = std::max({n1, D.n1, D.n2});
+    nin = std::max({nin, D.nin, D.n1, D.n2 + 2 * D.glu});
+    kout = std::max({kout, D.kout, D.glu});
+    fp = std::max(fp, seq_ ? D.glu : D.fp);
+    wp = std::max(wp, D.wp);
+    if (s.mlp == MLP_MOE) {
+      const size_t P = (size_t)R * s.top;
+      pairs = std::max(pairs, P);
+      e_act = std::max(e_act, P * D.fp);
+      e_gu = std::max(e_gu, P * 2 * D.fp);
+      moe_max_tiles_ = std::max(moe_max_tiles_, s.experts + (int)(P / 16));
+    }
+    if (s.mixer != MIX_LATENT) continue;
     rp = std::max(rp, D.rp);
     qa = std::max(qa, (size_t)R * D.H * D.rp);
     const size_t fl = std::max((size_t)R * D.H, (size_t)16 * 1024);  // (key_split: rows x splits)
@@ -294,7 +534,36 @@ void LayeredDecoder::finalize() {
   opart_ = falloc(part);
   ml_ = falloc(flat * 2);
   e_.ws_bytes_ = ((size_t)R * (2 * dp_ + n1) + part + 2 * flat) * 4;
-  pf_max_ctx_ = std::min(c.max_ctx, 32768);
+  pf_max_ctx_ = std::min(c.max_ctx, max_window_ ? std::min(32768, R + max_window_) : 32768);
+  auto operand = [&](size_t n) {  // a product's operand: bf16, or fp32 in the 32-bit engine
+    e_.ws_bytes_ += n * es;
+    return f32_ ? (void*)falloc(n) : (void*)balloc(n);
+  };
+  max_chunks_ = R / SCAN_CHUNK + c.max_slots + 1;
+  if (seq_) {
+    y_ = falloc((size_t)R * dp_);
+    e_.ws_bytes_ += (size_t)R * dp_ * 4;
+    if (loopw_) xin_ = operand((size_t)R * 2 * dp_);
+    if (wp) {
+      agg_ = falloc((size_t)max_chunks_ * 3 * wp);
+      e_.ws_bytes_ += (size_t)max_chunks_ * 3 * wp * 4;
+    }
+    if (pairs) {
+      moe_sel_ = (int*)falloc(pairs);
+      moe_pair_ = (int*)falloc(pairs);
+      moe_token_ = (int*)falloc(pairs);
+      moe_wt_ = falloc(pairs);
+      moe_tiles_ = (int4*)falloc((size_t)4 * moe_max_tiles_);
+      moe_ntiles_ = (int*)falloc(1);
+      moe_act_ = operand(e_act);
+      moe_ye_ = operand(pairs * dp_);
+      e_.ws_bytes_ += pairs * 16;
+      if (f32_) {
+        moe_gu32_ = falloc(e_gu);
+        e_.ws_bytes_ += e_gu * 4;
+      }
+    }
+  }
   if (f32_) {
     h32_ = falloc((size_t)R * dp_);
     gu32_ = falloc((size_t)R * 2 * std::max(fp, 1));
@@ -311,23 +580,24 @@ void LayeredDecoder::finalize() {
     e_.ws_bytes_ += ((size_t)R * (dp_ + kout) + qa + (size_t)pf_max_ctx_ * (rp + kvw)) * 2;
     // expanded attention from the portion length where its operations (key and value projections of the
     // whole context + dim + vdim per pair) drop below the absorbed form's (2 x rank per pair)
-    pf_min_ = 0;
+    pf_min_ = rp ? 0 : 1 << 30;
     for (const Dims& D : dims_) {
+      if (!D.H) continue;
       const double s = D.dkp + D.dvp, gain = 2.0 * D.rp - s;
       const int t = gain > 0 ? (int)std::min(256.0, std::max(64.0, D.rp * s / gain)) : 256;
       pf_min_ = std::max(pf_min_, t);
-      if (!mha_prefill_supports(D.dkp, D.dvp)) pf_min_ = 1 << 30;
     }
-    if (const char* v = std::getenv("AIOS_LATENT_PF_MIN")) pf_min_ = std::max(1, std::atoi(v));
+    if (const char* v = std::getenv("AIOS_LATENT_PF_MIN"))
+      if (rp) pf_min_ = std::max(1, std::atoi(v));
     for (const Dims& D : dims_)
-      if (!mha_prefill_supports(D.dkp, D.dvp)) pf_min_ = 1 << 30;
+      if (D.H && !mha_prefill_supports(D.dkp, D.dvp)) pf_min_ = 1 << 30;
     // the skinny GEMM's split-K workspace (shared with the engine's other users of gemm())
     const int maxN = std::max({nin, dp_, vp_, (int)kvw});
     e_.gk_ws_bytes_ = gemm_skinny_ws_bytes(64, maxN);
     e_.gk_ws_ = falloc(e_.gk_ws_bytes_ / 4 + 1);
     e_.gk_cnt_len_ = gemm_skinny_cnt_len(maxN);
     e_.gk_cnt_ = (int*)falloc(e_.gk_cnt_len_);
-    if (nl_ > 0 && dp_ == d_ && d_ % 128 == 0 && env_or("AIOS_GEMM_NORM_FUSE", 1)) {
+    if (!seq_ && dp_ == d_ && d_ % 128 == 0 && env_or("AIOS_GEMM_NORM_FUSE", 1)) {
       GemmQArgs p;
       std::memset(&p, 0, sizeof(p));
       p.M = 64; p.N = dp_; p.K = dims_[0].kout; p.nseg = 1; p.seg[0] = mat(w_[owner_[0]].out, dp_, dims_[0].kout);
@@ -341,20 +611,24 @@ void LayeredDecoder::finalize() {
   }
   // step parameters
   std::set<int> hs;
-  for (const Dims& D : dims_) hs.insert(D.H);
+  for (const Dims& D : dims_)
+    if (D.H) hs.insert(D.H);
   size_t tiles = 0;
   for (int h : hs) tiles += (size_t)R * ((h + 15) / 16) + R;
-  step_ints_ = (size_t)4 * R + 2 * tiles;
+  const size_t chunk_ints = (size_t)max_chunks_ * (sizeof(ScanChunk) / 4);
+  step_ints_ = (size_t)5 * R + chunk_ints + 2 * tiles;
   HIP_CHECK(hipHostMalloc((void**)&h_step_, step_ints_ * 4, hipHostMallocDefault));
   d_step_ = (int*)falloc(step_ints_);
   st_tokens_ = d_step_;
   st_pos_ = st_tokens_ + R;
   st_slot_ = st_pos_ + R;
   st_want_ = st_slot_ + R;
-  st_tiles_ = (LatentTile*)(st_want_ + R);
+  st_run_ = st_want_ + R;
+  st_chunks_ = (ScanChunk*)(st_run_ + R);
+  st_tiles_ = (LatentTile*)(st_run_ + R + chunk_ints);
   gemv_ok_.assign(5, 0);
   for (int b = 1; b <= 4 && !f32_; ++b) {
-    bool ok = dp_ == d_ && env_or("AIOS_LAYERED_GEMV", 1);
+    bool ok = !seq_ && dp_ == d_ && env_or("AIOS_LAYERED_GEMV", 1);
     for (int i = 0; i < nl_ && ok; ++i) ok = gemv_fits(i, b);
     gemv_ok_[b] = ok;
   }
@@ -380,27 +654,38 @@ bool LayeredDecoder::gemv_fits(int i, int B) {
 void LayeredDecoder::tune() {
   if (!env_or("AIOS_GEMM_PF_TUNE", 1) || nl_ == 0) return;
   float* tmp = nullptr;
-  const size_t n = (size_t)step_rows_ * std::max({dp_, dims_[0].kout, 64});
-  HIP_CHECK(hipMalloc(&tmp, n * 4));
-  fill_random_f32(tmp, n, 0x7u, 0.f, 1.f, e_.stream_);
+  HIP_CHECK(hipMalloc(&tmp, (size_t)step_rows_ * dp_ * 4));
+  fill_random_f32(tmp, (size_t)step_rows_ * dp_, 0x7u, 0.f, 1.f, e_.stream_);
   launch_f32_to_bf16(tmp, h16_, (size_t)step_rows_ * dp_, e_.stream_);
-  for (int M = 64; M <= step_rows_; M *= 2)
+  for (int M = 64; M <= step_rows_; M *= 2) {
+    auto go = [&](const bf16_t* A, int lda, const bf16_t* wt, int N, int K, int epi, float* C, int ldc, bf16_t* C16, int act) {
+      GemmQArgs g;
+      std::memset(&g, 0, sizeof(g));
+      g.A = A; g.lda = lda; g.M = M; g.N = N; g.K = K; g.nseg = 1; g.seg[0] = mat(wt, N, K);
+      g.C = C; g.C16 = C16; g.ldc = ldc; g.epi = epi; g.act = act;
+      gemm_pf_autotune(g, e_.stream_);
+    };
+    if (loopw_) go((const bf16_t*)xin_, 2 * dp_, loopw_, dp_, 2 * dp_, GEPI_STORE, y_, dp_, nullptr, 0);
     for (int i = 0; i < nl_; ++i) {
       if (owner_[i] != i) continue;
       const Dims& D = dims_[i];
       const Weights& w = w_[i];
-      auto go = [&](const bf16_t* A, int lda, const bf16_t* wt, int N, int K, int epi, float* C, int ldc, bf16_t* C16) {
-        GemmQArgs g;
-        std::memset(&g, 0, sizeof(g));
-        g.A = A; g.lda = lda; g.M = M; g.N = N; g.K = K; g.nseg = 1; g.seg[0] = mat(wt, N, K);
-        g.C = C; g.C16 = C16; g.ldc = ldc; g.epi = epi; g.act = e_.cfg_.layers[i].act;
-        gemm_pf_autotune(g, e_.stream_);
-      };
-      go(h16_, dp_, w.in, D.n1, dp_, GEPI_STORE, qdg_, D.n1, nullptr);
-      if (D.fp) go(h16_, dp_, w.in + (size_t)D.n1 * dp_, 2 * D.fp, dp_, GEPI_SWIGLU_BF16, nullptr, D.kout, cat16_ + D.gn);
-      go(cat16_, D.kout, w.out, dp_, D.kout, GEPI_ACCUM, x_, dp_, nullptr);
-      if (M <= pf_max_ctx_) go(cfull_, D.rp, w.ukv, D.qn + D.gn, D.rp, GEPI_STORE16, nullptr, D.qn + D.gn, kv_);
+      const int act = e_.cfg_.layers[i].act;
+      go(h16_, dp_, w.in, D.n1, dp_, GEPI_STORE, qdg_, D.n1, nullptr, act);
+      if (seq_) {
+        go(cat16_, D.kout, w.out, dp_, D.kout, GEPI_STORE, y_, dp_, nullptr, act);
+        if (w.in2 && D.n2) go(h16_, dp_, w.in2, D.n2, dp_, GEPI_STORE, qdg_, D.n2, nullptr, act);
+        if (D.glu) {
+          go(h16_, dp_, w.in2 + (size_t)D.n2 * dp_, 2 * D.glu, dp_, GEPI_SWIGLU_BF16, nullptr, D.glu, cat16_, act);
+          go(cat16_, D.glu, w.out2, dp_, D.glu, GEPI_STORE, y_, dp_, nullptr, act);
+        }
+      } else {
+        if (D.fp) go(h16_, dp_, w.in + (size_t)D.n1 * dp_, 2 * D.fp, dp_, GEPI_SWIGLU_BF16, nullptr, D.kout, cat16_ + D.gn, act);
+        go(cat16_, D.kout, w.out, dp_, D.kout, GEPI_ACCUM, x_, dp_, nullptr, act);
+      }
+      if (D.H && M <= pf_max_ctx_) go(cfull_, D.rp, w.ukv, D.qn + D.gn, D.rp, GEPI_STORE16, nullptr, D.qn + D.gn, kv_, act);
     }
+  }
   HIP_CHECK(hipMemsetAsync(h16_, 0, (size_t)step_rows_ * dp_ * 2, e_.stream_));
   HIP_CHECK(hipStreamSynchronize(e_.stream_));
   HIP_CHECK(hipFree(tmp));
@@ -424,7 +709,8 @@ int LayeredDecoder::key_split(int tiles, int max_len) const {
   return std::max(1, std::min({want, (max_len + keys - 1) / keys, max_len <= 4096 ? 32 : 64}));
 }
 
-LatentAttnArgs LayeredDecoder::latent_args(int i, const RowSet& r) {
+LatentAttnArgs LayeredDecoder::latent_args(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
   const Dims& D = dims_[i];
   const LayerSpec& s = e_.cfg_.layers[i];
   const Weights& w = w_[owner_[i]];
@@ -432,13 +718,16 @@ LatentAttnArgs LayeredDecoder::latent_args(int i, const RowSet& r) {
   std::memset(&a, 0, sizeof(a));
   a.n = r.n_abs;
   a.H = D.H; a.dk = D.dk; a.dkp = D.dkp; a.dvp = D.dvp; a.rank = D.rank; a.rp = D.rp;
+  a.rot = D.rot; a.roff = D.roff; a.qrot = D.qrot; a.rope = rope_[i];
+  a.window = s.window;
+  a.head_gate = s.out_gate == GATE_HEAD;
   a.scale = s.scale;
   a.eps = e_.cfg_.norm_eps;
   a.norm_w = w.kv_norm;
   a.sink = s.sink ? w.sink : nullptr;
-  a.qdg = qdg_; a.ld = D.n1; a.dkv_off = D.qn; a.g_off = s.out_gate ? D.qn + D.rp : -1;
+  a.qdg = qdg_; a.ld = D.n1; a.dkv_off = D.qn; a.g_off = s.out_gate ? D.gate_off : -1;
   a.pos = r.pos; a.slot = r.slot;
-  a.pool = pool_[i];
+  a.pool = runs_[k].pool;
   a.bt = e_.d_bt_; a.maxb = e_.kv_maxb_; a.kvb = e_.kvb_; a.f32 = f32_;
   a.wukT = w.ukT;
   a.wuv = w.ukv + (size_t)D.qn * D.rp;
@@ -450,18 +739,21 @@ LatentAttnArgs LayeredDecoder::latent_args(int i, const RowSet& r) {
     a.tiles = st_tiles_ + t.first;
     a.n_tiles = t.second;
   }
-  a.nsplit = f32_ || !latent_attn_mfma(D.rp) ? 1 : key_split(a.n_tiles, r.max_len);
+  // (a tile's window reaches from its first row's first key to its last row: at most 15 tokens more)
+  const int keys = s.window ? std::min(r.max_len, s.window + 15) : r.max_len;
+  a.nsplit = f32_ || !latent_attn_mfma(D.rp) ? 1 : key_split(a.n_tiles, keys);
   a.opart = opart_; a.ml = ml_;
   a.out = f32_ ? (void*)cat32_ : (void*)cat16_;
   a.ldo = D.kout;
   return a;
 }
 
-void LayeredDecoder::attention(int i, const RowSet& r) {
+void LayeredDecoder::attention(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
   const Dims& D = dims_[i];
   const Weights& w = w_[owner_[i]];
   hipStream_t st = e_.stream_;
-  const LatentAttnArgs a = latent_args(i, r);
+  const LatentAttnArgs a = latent_args(k, r);
   launch_latent_prep(a, r.n, st);
   if (a.n > 0) {
     launch_latent_attn(a, st);
@@ -469,21 +761,204 @@ void LayeredDecoder::attention(int i, const RowSet& r) {
   }
   for (const auto& pf : r.pf) {
     const Piece& p = pf.second;
-    const int row0 = pf.first, S = p.start + p.n, nkv = D.qn + D.gn;
-    launch_latent_gather((const bf16_t*)pool_[i], e_.d_bt_, e_.kv_maxb_, e_.kvb_, p.slot, S, D.rp, cfull_, st);
+    const int row0 = pf.first, k0 = a.window ? std::max(0, p.start - a.window + 1) : 0;
+    const int S = p.start + p.n - k0, nkv = D.qn + D.gn;
+    launch_latent_gather((const bf16_t*)a.pool, e_.d_bt_, e_.kv_maxb_, e_.kvb_, p.slot, k0, S, D.rp, cfull_, st);
     gemm16(cfull_, D.rp, w.ukv, S, nkv, D.rp, GEPI_STORE16, nullptr, nkv, kv_);
     MhaPrefillArgs m;
+    std::memset(&m, 0, sizeof(m));
     m.q = qdg_ + (size_t)row0 * D.n1; m.ldq = D.n1;
     m.k = kv_; m.v = kv_ + D.qn; m.ldkv = nkv;
-    m.H = D.H; m.dkp = D.dkp; m.dvp = D.dvp; m.start = p.start; m.T = p.n;
+    m.H = D.H; m.dkp = D.dkp; m.dvp = D.dvp; m.start = p.start - k0; m.T = p.n;
+    m.window = a.window; m.rot = a.rot; m.qrot = a.qrot; m.pos0 = p.start; m.rope = a.rope;
     m.scale = a.scale; m.sink = a.sink;
     m.gate = a.g_off >= 0 ? qdg_ + (size_t)row0 * D.n1 + a.g_off : nullptr;
+    m.head_gate = a.head_gate;
     m.out = cat16_ + (size_t)row0 * D.kout; m.ldo = D.kout;
     launch_mha_prefill(m, st);
   }
 }
 
-void LayeredDecoder::layer16(int i, const RowSet& r) {
+void LayeredDecoder::recurrence(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
+  const Dims& D = dims_[i];
+  const Weights& w = w_[owner_[i]];
+  MinGruArgs a;
+  std::memset(&a, 0, sizeof(a));
+  a.in = qdg_; a.ld = D.n1; a.z_off = 0; a.u_off = D.wp; a.g_off = 2 * D.wp;
+  a.zb = w.zb; a.ub = w.ub;
+  a.w = D.wp;
+  a.state = runs_[k].state;
+  a.slots = e_.cfg_.max_slots;
+  a.chunks = r.decode ? nullptr : st_chunks_;
+  a.pos = r.pos; a.slot = r.slot;
+  a.n = r.decode ? r.n : r.n_chunks;
+  a.split = r.decode ? 0 : r.split;
+  a.agg = agg_;
+  a.out = f32_ ? (void*)cat32_ : (void*)cat16_;
+  a.ldo = D.kout;
+  a.f32 = f32_;
+  launch_mingru(a, e_.stream_);
+}
+
+// ---- sequential layers --------------------------------------------------------------------------------
+void LayeredDecoder::project(const void* a, int lda, const bf16_t* w, int n, int N, int K, float* y, int ldy) {
+  if (f32_) return launch_gemm_f32((const float*)a, lda, w, K, n, N, K, y, ldy, 0, e_.stream_);
+  if (n <= 4) {
+    GemvArgs g = e_.gemv_args({}, N, K, n, nullptr, lda, nullptr, y, ldy, EPI_STORE, 0);
+    g.nseg = 1;
+    g.seg[0] = mat(w, N, K);
+    g.x16 = (const bf16_t*)a;
+    if (gemv_bf16_engine_fits(g)) return launch_gemv(g, e_.stream_);
+  }
+  gemm16((const bf16_t*)a, lda, w, n, N, K, GEPI_STORE, y, ldy, nullptr);
+}
+
+NextArgs LayeredDecoder::next_of(int k, bool decode) {
+  NextArgs x;
+  if (k >= (int)runs_.size()) {
+    if (!decode) return x;  // (a step's head gathers and normalises the rows it is asked for)
+    x.kind = NEXT_NORM;
+    x.g = out_norm_;
+  } else if (runs_[k].pass >= 0 && runs_[k].layer == e_.cfg_.loop_start) {
+    x.kind = NEXT_RAW;
+    x.out = xin_;
+    x.ldo = 2 * dp_;
+    return x;
+  } else {
+    x.kind = NEXT_NORM;
+    x.g = w_[owner_[runs_[k].layer]].norm;
+  }
+  x.out = f32_ ? (void*)h32_ : (void*)h16_;
+  x.ldo = dp_;
+  return x;
+}
+
+RowCloseArgs LayeredDecoder::close_args() const {
+  RowCloseArgs c;
+  std::memset((void*)&c, 0, sizeof(c));
+  c.x = x_;
+  c.dp = dp_; c.d = d_;
+  c.eps = e_.cfg_.norm_eps;
+  c.y = y_;
+  c.f32 = f32_;
+  return c;
+}
+
+// the second sublayer's products up to its result: c.y, or c.y and the experts' rows
+void LayeredDecoder::feed_forward(int k, const RowSet& r, RowCloseArgs& c) {
+  const int i = runs_[k].layer, n = r.n;
+  const Dims& D = dims_[i];
+  const LayerSpec& s = e_.cfg_.layers[i];
+  const Weights& w = w_[owner_[i]];
+  const void* h = f32_ ? (const void*)h32_ : (const void*)h16_;
+  void* act = f32_ ? (void*)cat32_ : (void*)cat16_;
+  const bf16_t* wglu = w.in2 + (size_t)D.n2 * dp_;
+  bool done = false;
+  if (!f32_ && D.glu && n <= 64) {  // one launch over all rows of in2
+    const int N = D.n2 + 2 * D.glu;
+    if (n <= 4) {
+      GemvArgs a = e_.gemv_args({}, N, dp_, n, nullptr, dp_, nullptr, qdg_, D.n2, EPI_STORE_GLU, 0);
+      a.nseg = 1;
+      a.seg[0] = mat(w.in2, N, dp_);
+      a.x16 = h16_;
+      a.act = s.act;
+      a.glu_row0 = D.n2;
+      a.y16 = cat16_;
+      a.ldy16 = D.glu;
+      done = gemv_bf16_engine_fits(a);
+      if (done) launch_gemv(a, e_.stream_);
+    }
+    if (!done && D.n2) {
+      GemmQArgs g;
+      std::memset(&g, 0, sizeof(g));
+      g.A = h16_; g.lda = dp_; g.M = n; g.N = N; g.K = dp_; g.nseg = 1; g.seg[0] = mat(w.in2, N, dp_);
+      g.C = qdg_; g.ldc = D.n2; g.epi = GEPI_STORE_GLU; g.act = s.act;
+      g.glu_n0 = D.n2; g.C16 = cat16_; g.ldc16 = D.glu;
+      e_.gemm(g);
+      done = true;
+    }
+  }
+  if (!done) {
+    if (D.n2) project(h, dp_, w.in2, n, D.n2, dp_, qdg_, D.n2);
+    if (D.glu && f32_) {
+      launch_gemm_f32(h32_, dp_, wglu, dp_, n, 2 * D.glu, dp_, gu32_, 2 * D.glu, 0, e_.stream_);
+      launch_glu_f32(gu32_, 2 * D.glu, cat32_, D.glu, n, D.glu, s.act, e_.stream_);
+    } else if (D.glu) {
+      gemm16(h16_, dp_, wglu, n, 2 * D.glu, dp_, GEPI_SWIGLU_BF16, nullptr, D.glu, cat16_, s.act);
+    }
+  }
+  c.y = D.glu || s.mlp == MLP_GLU ? y_ : nullptr;
+  if (s.mlp == MLP_MOE) {
+    MoeArgs m;
+    std::memset(&m, 0, sizeof(m));
+    m.n = n; m.experts = s.experts; m.top = s.top; m.scale = s.router_scale;
+    m.logits = qdg_ + D.router_off; m.ldl = D.n2;
+    m.corr = s.correction ? w.corr : nullptr;
+    m.dp = dp_; m.ff = D.fp; m.act = s.act;
+    m.h = h; m.ldh = dp_;
+    m.wgu = w.egu; m.wdn = w.edn;
+    m.sel = moe_sel_; m.wt = moe_wt_; m.pair = moe_pair_; m.token = moe_token_;
+    m.tiles = moe_tiles_; m.n_tiles = moe_ntiles_; m.max_tiles = moe_max_tiles_;
+    m.act_out = moe_act_; m.ye = moe_ye_; m.gu32 = moe_gu32_;
+    m.f32 = f32_;
+    if (!f32_ && n <= MOE_FEW) {
+      if (D.glu) { m.sh_act = cat16_; m.ld_sh = D.glu; m.sh_ff = D.glu; m.sh_dn = w.out2; }
+      m.y = y_;
+      c.y = y_;
+      return launch_moe_few(m, e_.stream_);
+    }
+    launch_moe_grouped(m, e_.stream_);
+    c.ye = moe_ye_; c.pair = moe_pair_; c.wt = moe_wt_; c.top = s.top;
+  }
+  if (D.glu) project(act, D.glu, w.out2, n, dp_, D.glu, y_, dp_);
+}
+
+void LayeredDecoder::layer_seq(int k, const RowSet& r) {
+  const int i = runs_[k].layer, n = r.n;
+  const Dims& D = dims_[i];
+  const LayerSpec& s = e_.cfg_.layers[i];
+  const Weights& w = w_[owner_[i]];
+  hipStream_t st = e_.stream_;
+  const void* h = f32_ ? (const void*)h32_ : (const void*)h16_;
+  void* cat = f32_ ? (void*)cat32_ : (void*)cat16_;
+  if (runs_[k].pass >= 0 && i == e_.cfg_.loop_start) {  // a pass begins: x = W [x; x0] + step
+    project(xin_, 2 * dp_, loopw_, n, dp_, 2 * dp_, y_, dp_);
+    RowCloseArgs c = close_args();
+    c.replace = 1;
+    c.add = loop_step_ + (size_t)runs_[k].pass * dp_;
+    c.next.kind = NEXT_NORM;
+    c.next.g = w.norm;
+    c.next.out = f32_ ? (void*)h32_ : (void*)h16_;
+    c.next.ldo = dp_;
+    launch_row_close(c, n, st);
+  }
+  project(h, dp_, w.in, n, D.n1, dp_, qdg_, D.n1);
+  if (s.mixer == MIX_MINGRU) recurrence(k, r);
+  else attention(k, r);
+  project(cat, D.kout, w.out, n, dp_, D.kout, y_, dp_);
+  RowCloseArgs c = close_args();
+  if (s.resid_gate) { c.gate = qdg_ + D.rg_off; c.ldg = D.n1; c.gate_bias = w.rgb; }
+  if (s.post_norm) c.post = w.post;
+  if (s.mlp == MLP_NONE) {
+    c.next = next_of(k + 1, r.decode);
+    return launch_row_close(c, n, st);
+  }
+  c.next.kind = NEXT_NORM;
+  c.next.g = w.norm2;
+  c.next.out = f32_ ? (void*)h32_ : (void*)h16_;
+  c.next.ldo = dp_;
+  launch_row_close(c, n, st);
+  RowCloseArgs f = close_args();
+  feed_forward(k, r, f);
+  if (s.resid_gate) { f.gate = qdg_; f.ldg = D.n2; f.gate_bias = w.rgb2; }
+  if (s.post_norm) f.post = w.post2;
+  f.next = next_of(k + 1, r.decode);
+  launch_row_close(f, n, st);
+}
+
+void LayeredDecoder::layer16(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
   const Dims& D = dims_[i];
   const LayerSpec& s = e_.cfg_.layers[i];
   const Weights& w = w_[owner_[i]];
@@ -499,7 +974,7 @@ void LayeredDecoder::layer16(int i, const RowSet& r) {
     a.y16 = D.fp ? cat16_ + D.gn : nullptr;
     a.ldy16 = D.kout;
     launch_gemv(a, st);
-    attention(i, r);
+    attention(k, r);
     GemvArgs b = e_.gemv_args({}, dp_, D.kout, n, nullptr, D.kout, nullptr, x_, dp_, EPI_RESID, 0);
     b.nseg = 1;
     b.seg[0] = mat(w.out, dp_, D.kout);
@@ -522,7 +997,7 @@ void LayeredDecoder::layer16(int i, const RowSet& r) {
     if (D.fp)
       gemm16(h16_, dp_, w.in + (size_t)D.n1 * dp_, n, 2 * D.fp, dp_, GEPI_SWIGLU_BF16, nullptr, D.kout, cat16_ + D.gn, s.act);
   }
-  attention(i, r);
+  attention(k, r);
   GemmQArgs g;
   std::memset(&g, 0, sizeof(g));
   g.A = cat16_; g.lda = D.kout; g.M = n; g.N = dp_; g.K = D.kout; g.nseg = 1; g.seg[0] = mat(w.out, dp_, D.kout);
@@ -536,7 +1011,8 @@ void LayeredDecoder::layer16(int i, const RowSet& r) {
   norm_ready_ = fuse;
 }
 
-void LayeredDecoder::layer32(int i, const RowSet& r) {
+void LayeredDecoder::layer32(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
   const Dims& D = dims_[i];
   const Weights& w = w_[owner_[i]];
   hipStream_t st = e_.stream_;
@@ -546,30 +1022,53 @@ void LayeredDecoder::layer32(int i, const RowSet& r) {
     launch_gemm_f32(h32_, dp_, w.in + (size_t)D.n1 * dp_, dp_, r.n, 2 * D.fp, dp_, gu32_, 2 * D.fp, 0, st);
     launch_glu_f32(gu32_, 2 * D.fp, cat32_ + D.gn, D.kout, r.n, D.fp, e_.cfg_.layers[i].act, st);
   }
-  attention(i, r);
+  attention(k, r);
   launch_gemm_f32(cat32_, D.kout, w.out, D.kout, r.n, dp_, D.kout, x_, dp_, 1, st);
 }
 
 void LayeredDecoder::run(const RowSet& r) {
-  launch_embed_pos(embd_, posw_, r.tokens, r.pos, r.n, dp_, x_, e_.stream_);
+  const EngineConfig& c = e_.cfg_;
+  EmbedArgs e;
+  std::memset((void*)&e, 0, sizeof(e));
+  e.table = embd_; e.scale = c.embed_scale; e.pos_table = posw_;
+  e.pair_table = pairw_; e.buckets = c.bigram_buckets; e.mul_prev = c.bigram_prev; e.mul_cur = c.bigram_cur;
+  e.tokens = r.tokens; e.pos = r.pos; e.slot = r.slot; e.run = r.run;
+  e.last = last_tok_; e.slots = c.max_slots;
+  e.dp = dp_; e.d = d_; e.eps = c.norm_eps;
+  e.x = x_;
+  if (xin_) {
+    e.keep = f32_ ? (void*)((float*)xin_ + dp_) : (void*)((bf16_t*)xin_ + dp_);
+    e.ld_keep = 2 * dp_;
+  }
+  e.f32 = f32_;
+  if (seq_) e.next = next_of(0, r.decode);
+  launch_embed_rows(e, r.n, e_.stream_);
   norm_ready_ = false;
-  for (int i = 0; i < nl_; ++i) {
-    if (f32_) layer32(i, r);
-    else layer16(i, r);
+  const int n = run_limit_ < 0 ? (int)runs_.size() : std::min(run_limit_, (int)runs_.size());
+  for (int k = 0; k < n; ++k) {
+    if (seq_) layer_seq(k, r);
+    else if (f32_) layer32(k, r);
+    else layer16(k, r);
   }
 }
 
 void LayeredDecoder::decode_forward(int B) {
   RowSet r;
-  r.tokens = e_.d_tokens_; r.pos = e_.d_pos_; r.slot = e_.d_slot_;
+  r.tokens = e_.d_tokens_; r.pos = e_.d_pos_; r.slot = e_.d_slot_; r.run = nullptr;
+  r.n_chunks = r.split = 0;
   r.n = r.n_abs = B;
   r.decode = true;
   r.max_len = e_.cfg_.max_ctx;
   run(r);
+  head_ready_ = seq_;  // (the last layer left the head's operand)
   // (the head reads the residual in place: the decode rows are x rows 0 .. B-1)
   std::swap(x_, xh_);
   head(B);
   std::swap(x_, xh_);
+}
+
+int LayeredDecoder::span(const Piece& p) const {
+  return max_window_ ? std::min(p.start + p.n, p.n + max_window_ - 1) : p.start + p.n;
 }
 
 void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>& first_row) {
@@ -581,7 +1080,7 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
   for (int p = 0; p < (int)pieces.size(); ++p) {
     const Piece& q = pieces[p];
     r.n += q.n;
-    if (q.n < pf_min_ || q.start + q.n > pf_max_ctx_) {
+    if (q.n < pf_min_ || span(q) > pf_max_ctx_) {
       order.push_back(p);
       r.n_abs += q.n;
       r.max_len = std::max(r.max_len, q.start + q.n);
@@ -592,8 +1091,10 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
   for (int p = 0; p < (int)pieces.size(); ++p)
     if (std::find(order.begin(), order.begin() + n_small, p) == order.begin() + n_small) order.push_back(p);
   first_row.assign(pieces.size(), 0);
-  int *ht = h_step_, *hp = ht + R, *hs = hp + R;
-  LatentTile* tiles = (LatentTile*)(hs + 2 * R);
+  int *ht = h_step_, *hp = ht + R, *hs = hp + R, *hr = hs + 2 * R;
+  ScanChunk* chunks = (ScanChunk*)(hr + R);
+  LatentTile* tiles = (LatentTile*)(h_step_ + ((const int*)st_tiles_ - d_step_));
+  r.n_chunks = r.split = 0;
   int row = 0, nt = 0;
   for (int o = 0; o < (int)order.size(); ++o) {
     const Piece& q = pieces[order[o]];
@@ -602,12 +1103,18 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
       ht[row + k] = q.tokens[k];
       hp[row + k] = q.start + k;
       hs[row + k] = q.slot;
+      hr[row + k] = k ? 0 : q.n;
     }
+    const int c0 = r.n_chunks;
+    if (c0 + (q.n + SCAN_CHUNK - 1) / SCAN_CHUNK > max_chunks_) throw std::runtime_error("layered forward: too many pieces");
+    for (int k = 0; k < q.n; k += SCAN_CHUNK)
+      chunks[r.n_chunks++] = ScanChunk{row + k, std::min(SCAN_CHUNK, q.n - k), q.slot, q.start + k, c0, k + SCAN_CHUNK >= q.n};
+    if (q.n > SCAN_CHUNK) r.split = 1;
     if (o >= n_small) r.pf.push_back({row, q});
     row += q.n;
   }
   for (const Dims& D : dims_) {
-    if (r.tiles.count(D.H)) continue;
+    if (!D.H || r.tiles.count(D.H)) continue;
     const int t0 = nt;
     for (int o = 0; o < n_small; ++o) {
       const int f0 = first_row[order[o]] * D.H, f1 = f0 + pieces[order[o]].n * D.H;
@@ -615,9 +1122,11 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
     }
     r.tiles[D.H] = {t0, nt - t0};
   }
-  r.tokens = st_tokens_; r.pos = st_pos_; r.slot = st_slot_;
-  HIP_CHECK(hipMemcpyAsync(d_step_, h_step_, ((size_t)4 * R + 2 * (size_t)nt) * 4, hipMemcpyHostToDevice, e_.stream_));
+  r.tokens = st_tokens_; r.pos = st_pos_; r.slot = st_slot_; r.run = st_run_;
+  const size_t ints = (size_t)((const int*)st_tiles_ - d_step_) + 2 * (size_t)nt;
+  HIP_CHECK(hipMemcpyAsync(d_step_, h_step_, ints * 4, hipMemcpyHostToDevice, e_.stream_));
   run(r);
+  head_ready_ = false;
   norm_ready_ = false;  // (the head normalises the rows it is asked for)
 }
 
@@ -636,6 +1145,15 @@ void LayeredDecoder::head(int B, int from) {
   hipStream_t st = e_.stream_;
   const float eps = e_.cfg_.norm_eps;
   float* y = e_.logits_;
+  if (seq_) {
+    void* h = f32_ ? (void*)h32_ : (void*)h16_;
+    if (!head_ready_) {
+      if (f32_) launch_rmsnorm(x, dp_, out_norm_, h32_, dp_, B, d_, eps, st);
+      else launch_rmsnorm_bf16(x, dp_, out_norm_, h16_, dp_, B, d_, eps, st);
+    }
+    head_ready_ = false;
+    return project(h, dp_, headw_, B, vp_, dp_, y, vp_);
+  }
   if (f32_) {
     launch_rmsnorm(x, dp_, out_norm_, h32_, dp_, B, d_, eps, st);
     launch_gemm_f32(h32_, dp_, headw_, dp_, B, vp_, dp_, y, vp_, 0, st);
@@ -661,6 +1179,18 @@ void LayeredDecoder::head(int B, int from) {
     launch_rmsnorm_bf16(x, dp_, out_norm_, h16_, dp_, B, d_, eps, st);
   }
   e_.gemm(g);
+}
+
+void LayeredDecoder::copy_state(int src, int dst) {
+  const int slots = e_.cfg_.max_slots;
+  auto copy = [&](void* base, size_t row) {
+    for (int p = 0; p < 2; ++p)
+      HIP_CHECK(hipMemcpyAsync((char*)base + ((size_t)p * slots + dst) * row, (char*)base + ((size_t)p * slots + src) * row, row,
+                               hipMemcpyDeviceToDevice, e_.stream_));
+  };
+  for (const Run& k : runs_)
+    if (k.state) copy(k.state, (size_t)dims_[k.layer].wp * 4);
+  if (last_tok_) copy(last_tok_, 4);
 }
 
 std::vector<float> LayeredDecoder::residual(int rows) {

@@ -43,6 +43,8 @@ void launch_rmsnorm(const float* x, int ldx, const float* w, float* y, int ldy, 
 void launch_rmsnorm_bf16(const float* x, int ldx, const float* w, bf16_t* y, int ldy, int rows, int n, float eps,
                          hipStream_t st);
 void launch_f32_to_bf16(const float* x, bf16_t* y, size_t n, hipStream_t st);
+// rows of n columns (n % 4 == 0, 16-byte aligned rows) to zero
+void launch_zero_rows(float* y, int ldy, int rows, int n, hipStream_t st);
 void launch_add(float* y, const float* x, size_t n, hipStream_t st);
 
 // Producer side of the split RMSNorm after a TP all-reduce (the skinny GEMM's nrm_in contract,

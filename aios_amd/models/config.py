@@ -25,16 +25,32 @@ ROPE_NEOX = 2   # qwen: (x[i], x[i + rot/2])
 @dataclasses.dataclass(frozen=True)
 class LayerConfig:
     """One layer of a model described layer by layer (csrc/layered.h LayerSpec)."""
-    mixer: str = "latent"          # latent attention
+    mixer: str = "latent"          # "latent" attention | "mingru"
+    # parallel: mixer and MLP read one norm and are added together; else one after the other, each with a norm
+    # of its own before it, and (post_norm) after it, and (resid_gate) its result times sigmoid(W h + b)
+    parallel: bool = True
+    norm_scalar: bool = False      # those norms have one number for all columns
+    post_norm: bool = False
+    resid_gate: bool = False
     heads: int = 1
-    dim: int = 64                  # query-key dimensions per head
+    dim: int = 64                  # (unrotated) query-key dimensions per head
     vdim: int = 64                 # value dimensions per head
     kv_rank: int = 64              # width of the cached latent
+    rot_dim: int = 0               # rotated query-key dimensions; their key part is shared by all heads
+    rot_dims: int = 0              # of which the first so many turn
+    rot_base: float = 10000.0
+    window: int = 0                # keys a token sees, itself included; 0: all before it
     scale: float = 0.125           # of q . k
     sink: bool = True              # a learned logit per head in the softmax's denominator
-    out_gate: bool = True          # head outputs times sigmoid(Wg h)
-    ff: int = 256                  # hidden width of the gated MLP; 0: none
+    out_gate: str = "element"      # head outputs times sigmoid(Wg h): "none" | "element" | "head" (one number)
+    width: int = 64                # of the state (mingru)
+    ff: int = 256                  # hidden width of the gated MLP, or of every expert; 0: none
     act: str = "gelu_tanh"         # of the gate: "gelu_tanh" | "silu"
+    experts: int = 0               # mixture of experts (0: a dense MLP), of which every token uses `top`
+    top: int = 0
+    router_scale: float = 1.0
+    correction: bool = False       # a learned number per expert joins the choice, not the weights
+    shared_ff: int = 0             # hidden width of the expert every token runs; 0: none
     weights_of: int = -1           # layer whose weights this one uses, or -1
 
 
@@ -62,6 +78,12 @@ class ModelConfig:
     chat_template: str = "zephyr"
     # models described layer by layer; empty: a llama-family decoder of the sizes above
     layers: Tuple[LayerConfig, ...] = ()
+    learned_pos: bool = True       # a table of max_ctx learned positions
+    embed_scale: float = 1.0       # of the token embedding
+    logit_scale: float = 1.0
+    # embedding of token pairs, row (previous * mul_prev + current * mul_cur) mod buckets: (buckets, mul_prev, mul_cur)
+    bigram: Optional[Tuple[int, int, int]] = None
+    loop: Optional[Tuple[int, int, int]] = None  # layers [start, stop) run `times` times: (start, stop, times)
 
     @property
     def q_dim(self) -> int:
@@ -77,15 +99,29 @@ class ModelConfig:
 
     def n_params(self) -> int:
         if self.layers:
-            n = 2 * self.vocab_size * self.d_model + self.max_ctx * self.d_model
-            for l in self.layers:
-                if l.weights_of < 0:
-                    n += self.d_model * (l.heads * (l.dim + 2 * l.vdim) + l.kv_rank + 3 * l.ff)
-                    n += l.kv_rank * l.heads * (l.dim + l.vdim)
-            return n
+            return self._layered_params()
         per_layer = self.d_model * (self.qkv_dim + self.q_dim) + 3 * self.d_model * self.d_ff + 2 * self.d_model
         emb = self.vocab_size * self.d_model * (1 if self.tie_embeddings else 2)
         return self.n_layers * per_layer + emb + self.d_model
+
+    def _layered_params(self) -> int:
+        d = self.d_model
+        n = 2 * self.vocab_size * d + (self.max_ctx * d if self.learned_pos else 0)
+        n += (self.bigram[0] + 1) * d if self.bigram else 0
+        n += 2 * d * d + self.loop[2] * d if self.loop else 0
+        for l in self.layers:
+            if l.weights_of >= 0:
+                continue
+            if l.mixer == "mingru":
+                n += 4 * l.width * d
+            else:
+                gate = {"none": 0, "element": l.heads * l.vdim, "head": l.heads}[l.out_gate]
+                n += d * (l.heads * (l.dim + l.rot_dim + l.vdim) + gate + l.kv_rank + l.rot_dim)
+                n += l.kv_rank * l.heads * (l.dim + l.vdim)
+            if l.resid_gate:
+                n += d * d * (2 if l.ff else 1)
+            n += 3 * d * (l.ff * max(1, l.experts) + l.shared_ff) + l.experts * d
+        return n
 
     def scaled(self, **kw) -> "ModelConfig":
         return dataclasses.replace(self, **kw)
@@ -131,6 +167,26 @@ def _gefazen(name: str, vocab: int, width: int, n_layers: int, max_ctx: int, **l
     return ModelConfig(name=name, arch="gefazen", vocab_size=vocab, d_model=width, n_layers=n_layers, n_heads=l.heads,
                        n_kv_heads=1, head_dim=l.dim, d_ff=l.ff, max_ctx=max_ctx, bos_id=-1, eos_id=-1,
                        layers=(l,) * n_layers)
+
+
+def _movalorn(name: str, vocab: int, width: int, n_layers: int, ff: int, experts: int, top: int, expert_ff: int,
+              window: int, loop: Tuple[int, int, int], max_ctx: int, state: int, **attn) -> ModelConfig:
+    """Every third layer latent attention, the others minGRU; the first MLP dense, then experts."""
+    common = dict(parallel=False, norm_scalar=True, post_norm=True, resid_gate=True, sink=False, out_gate="head")
+    dense = dict(ff=ff, act="gelu_tanh")
+    moe = dict(ff=expert_ff, act="silu", experts=experts, top=top, router_scale=1.5, correction=True, shared_ff=expert_ff)
+    layers = []
+    for i in range(n_layers):
+        mlp = dense if i == 0 else moe
+        if i % 3 == 1:
+            layers.append(LayerConfig(mixer="latent", window=window, scale=(attn["dim"] + attn["rot_dim"]) ** -0.5,
+                                      rot_dims=attn["rot_dim"], **attn, **common, **mlp))
+        else:
+            layers.append(LayerConfig(mixer="mingru", width=state, **common, **mlp))
+    return ModelConfig(name=name, arch="movalorn", vocab_size=vocab, d_model=width, n_layers=n_layers,
+                       n_heads=attn["heads"], n_kv_heads=1, head_dim=attn["dim"] + attn["rot_dim"], d_ff=ff, max_ctx=max_ctx,
+                       bos_id=-1, eos_id=-1, layers=tuple(layers), learned_pos=False, embed_scale=0.7, logit_scale=0.4,
+                       bigram=(4 * vocab + 1, 31, 17), loop=loop)
 
 
 PRESETS: Dict[str, ModelConfig] = {
@@ -185,6 +241,13 @@ PRESETS: Dict[str, ModelConfig] = {
     "gefazen-1b": _gefazen("gefazen-1b", 32000, 2048, 22, 4096, heads=32, dim=64, vdim=64, kv_rank=512, ff=5632),
     "gefazen-7b": _gefazen("gefazen-7b", 32000, 4096, 32, 32768, heads=32, dim=128, vdim=128, kv_rank=512, ff=14336),
     "test-gefazen": _gefazen("test-gefazen", 700, 512, 3, 512, heads=4, dim=64, vdim=32, kv_rank=64, ff=1024),
+    # Movalorn at the same widths, depths and active MLP sizes (layer runs, of which a loop repeats some)
+    "movalorn-1b": _movalorn("movalorn-1b", 32000, 2048, 18, 5632, 16, 3, 1408, 1024, (4, 8, 2), 4096, 2048, heads=32,
+                             dim=64, vdim=64, kv_rank=512, rot_dim=32),
+    "movalorn-7b": _movalorn("movalorn-7b", 32000, 4096, 26, 14336, 16, 3, 3584, 2048, (4, 10, 2), 32768, 4096, heads=32,
+                             dim=128, vdim=128, kv_rank=512, rot_dim=64),
+    "test-movalorn": _movalorn("test-movalorn", 600, 384, 5, 512, 6, 2, 128, 50, (1, 3, 2), 512, 320, heads=3, dim=40,
+                               vdim=32, kv_rank=72, rot_dim=24),
     "test-mistral-shape": ModelConfig(
         name="test-mistral-shape", vocab_size=1024, d_model=1024, n_layers=2, n_heads=8, n_kv_heads=2,
         head_dim=128, d_ff=2048, rope_theta=1e6, max_ctx=512, chat_template="mistral"),

@@ -41,7 +41,7 @@ def _layer(i: int, entry: dict) -> LayerConfig:
         raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
     w = entry.get("weights_of")
     return LayerConfig(mixer="latent", heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
-                       kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), sink=True, out_gate=True,
+                       kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), sink=True, out_gate="element",
                        ff=0 if mlp is None else int(mlp["ff"]), act="gelu_tanh", weights_of=-1 if w is None else int(w))
 
 

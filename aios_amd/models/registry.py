@@ -22,7 +22,7 @@ class Architecture:
 
 
 # architecture -> module under aios_amd.models that defines ARCHITECTURE
-_MODULES = {"gefazen": "gefazen"}
+_MODULES = {"gefazen": "gefazen", "movalorn": "movalorn"}
 
 
 def architectures():

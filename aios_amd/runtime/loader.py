@@ -96,7 +96,8 @@ def _load_dir(path: str, max_ctx: Optional[int], name: Optional[str], verbose: b
     t0 = time.time()
     cfg, raw, arch = registry.load_config(path, name or "")
     m = native.require()
-    eng = m.Engine(native.engine_config(cfg, max_ctx=min(max_ctx or cfg.max_ctx, cfg.max_ctx), **engine_kw))
+    ctx = max_ctx or cfg.max_ctx  # (a table of positions bounds the context)
+    eng = m.Engine(native.engine_config(cfg, max_ctx=min(ctx, cfg.max_ctx) if cfg.learned_pos else ctx, **engine_kw))
     r = SafetensorsReader(os.path.join(path, "model.safetensors"))
     for src, dst in arch.tensor_names(raw).items():
         if src not in r.tensors:
@@ -104,7 +105,7 @@ def _load_dir(path: str, max_ctx: Optional[int], name: Optional[str], verbose: b
         t = r.tensors[src]
         if t.dtype not in _ST_TYPES:
             raise ValueError(f"{path}: tensor {src} has unsupported dtype {t.dtype}")
-        rows, cols = (1, t.shape[0]) if len(t.shape) == 1 else t.shape
+        rows, cols = (1, int(np.prod(t.shape))) if len(t.shape) < 2 else t.shape
         eng.set_tensor(dst, int(_ST_TYPES[t.dtype]), rows, cols, r.raw(src))
     finalize(eng)
     if verbose:

@@ -144,18 +144,30 @@ def engine_config(cfg, max_ctx: Optional[int] = None, max_slots: int = 4, max_ba
             raise ValueError(f"{cfg.name}: layered models run on one GPU (no tensor parallelism)")
         if ec.kv_fp8:
             raise ValueError(f"{cfg.name}: the latent cache has no fp8 form (kv_dtype bf16)")
-        ec.max_positions = int(cfg.max_ctx)
+        ec.max_positions = int(cfg.max_ctx) if cfg.learned_pos else 0
+        ec.embed_scale, ec.logit_scale = float(cfg.embed_scale), float(cfg.logit_scale)
+        if cfg.bigram:
+            ec.bigram_buckets, ec.bigram_prev, ec.bigram_cur = (int(v) for v in cfg.bigram)
+        if cfg.loop:
+            ec.loop_start, ec.loop_stop, ec.loop_times = (int(v) for v in cfg.loop)
         ec.layers = [_layer_spec(m, l) for l in cfg.layers]
     return ec
 
 
 def _layer_spec(m, l):
     s = m.LayerSpec()
-    s.mixer = {"latent": m.MIX_LATENT}[l.mixer]
+    s.mixer = {"latent": m.MIX_LATENT, "mingru": m.MIX_MINGRU}[l.mixer]
+    s.parallel, s.norm_scalar = int(l.parallel), int(l.norm_scalar)
+    s.post_norm, s.resid_gate = int(l.post_norm), int(l.resid_gate)
     s.heads, s.dim, s.vdim, s.kv_rank = l.heads, l.dim, l.vdim, l.kv_rank
+    s.rot_dim, s.rot_dims, s.rot_base, s.window = l.rot_dim, l.rot_dims, float(l.rot_base), l.window
     s.scale = float(l.scale)
-    s.sink, s.out_gate = int(l.sink), int(l.out_gate)
-    s.mlp, s.ff = (m.MLP_GLU, l.ff) if l.ff else (m.MLP_NONE, 0)
+    s.sink = int(l.sink)
+    s.out_gate = {"none": m.GATE_NONE, "element": m.GATE_ELEMENT, "head": m.GATE_HEAD}[l.out_gate]
+    s.width = l.width
+    s.mlp, s.ff = (m.MLP_MOE if l.experts else m.MLP_GLU, l.ff) if l.ff else (m.MLP_NONE, 0)
     s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU}[l.act]
+    s.experts, s.top, s.shared_ff = l.experts, l.top, l.shared_ff
+    s.router_scale, s.correction = float(l.router_scale), int(l.correction)
     s.weights_of = l.weights_of
     return s
