@@ -14,6 +14,8 @@ with an in-process worker per model that owns the native Engine:
   prefill; with nothing decoding the prompt goes through in one call;
 * engines that run mixed batches (Engine.mixed_steps) take the prompt chunks of several admitted
   sequences and the decode token of every running one in ONE step instead of alternating the two;
+* a model with a recurrent state (Engine.recurrent) reuses a cached prefix only where some slot's state stands
+  at its end (Engine.resumable); a queued step that is dropped leaves the state it started from in place;
 * a cache pool smaller than every slot's full context (kv_pool_tokens) admits a request only when its
   blocks are certain to be available, and takes cached prefixes of idle slots back for it;
 * each iteration runs ONE batched decode step (hipGraph replay) for every decoding sequence, so
@@ -128,6 +130,8 @@ class Scheduler:
         self.step_log: Deque = collections.deque(maxlen=4096)  # (end time, batch) per decode step
         self.share_prefix = hasattr(engine, "copy_slot")
         self.mixed = bool(getattr(engine, "mixed_steps", False))
+        # a recurrent state stands at one position: a cached prefix is reusable only where the state can go on
+        self.recurrent = bool(getattr(engine, "recurrent", False))
         # a pool that cannot hold every slot's full context: blocks are reserved per request
         self.kv_block = int(getattr(engine, "kv_block_tokens", 0) or 0)
         self.kv_total = int(getattr(engine, "kv_blocks_total", 0) or 0)
@@ -273,21 +277,26 @@ class Scheduler:
             n += 1
         return n
 
+    def _reusable(self, slot: int, ids: List[int]) -> int:
+        """Leading tokens of ids that `slot` has already taken in and can go on from."""
+        n = self._common(self.slot_cache[slot], ids)
+        return n if not self.recurrent or self.engine.resumable(slot, n) else 0
+
     def _pick_slot(self, ids: List[int]):
         """(slot, reused tokens): the free slot whose own cache matches best, or -- when another
         slot (free or decoding) holds a longer matching prefix -- the free slot with the least
         cached content, which then shares that prefix through the paged KV."""
         best, best_len = None, -1
         for s in self.free_slots:
-            n = self._common(self.slot_cache[s], ids)
+            n = self._reusable(s, ids)
             if n > best_len:
                 best, best_len = s, n
         best_len = max(best_len, 0)
         if self.share_prefix:
             src, src_len = None, best_len
-            for s, c in self.slot_cache.items():
+            for s in self.slot_cache:
                 if s != best:
-                    n = self._common(c, ids)
+                    n = self._reusable(s, ids)
                     if n > src_len:
                         src, src_len = s, n
             if src is not None and src_len >= best_len + self.min_shared_prefix:
@@ -568,7 +577,7 @@ class Scheduler:
             self.engine.decode_sample(self._masks(rows))
             self._pending = rows
         # (spec and a row finished: the queued forward is dropped -- its KV writes at the next
-        # position are rewritten by whatever runs there next)
+        # position are rewritten by whatever runs there next, and so is a recurrent state)
         t3 = time.perf_counter()
         tm = self.timing
         tm["mask_s"] += (t3 - t2b) + (t1 - t0)   # masks + submit / sampler enqueue

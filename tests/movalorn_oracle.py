@@ -115,6 +115,14 @@ def route(h: torch.Tensor, w: Dict[str, torch.Tensor], p: str, r: dict):
     return pick, torch.gather(s, 1, pick) * r["scale"]
 
 
+def choice_gap(h: torch.Tensor, w: Dict[str, torch.Tensor], p: str, r: dict) -> torch.Tensor:
+    """How far the last chosen expert's choice score is above the first one left out [T]."""
+    if r["top"] == r["experts"]:
+        return torch.ones(h.shape[0], dtype=h.dtype)
+    c = torch.sort(torch.softmax(h @ w[p + "router"].T, -1) + w[p + "correction"], -1, descending=True).values
+    return c[:, r["top"] - 1] - c[:, r["top"]]
+
+
 def moe(h: torch.Tensor, w: Dict[str, torch.Tensor], p: str, m: dict) -> torch.Tensor:
     pick, wt = route(h, w, p, m["router"])
     y = torch.zeros_like(h)
@@ -150,8 +158,9 @@ def schedule(cfg: dict) -> List[tuple]:
 
 
 def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int], trace: Optional[list] = None,
-            dtype=DT) -> torch.Tensor:
-    """Logits [T, vocab]; `trace` collects the residual stream after every layer run."""
+            dtype=DT, gaps: Optional[list] = None) -> torch.Tensor:
+    """Logits [T, vocab]; `trace` collects the residual stream after every layer run, `gaps` the experts' choice
+    gaps of every layer run that has a router."""
     w = {k: v.to(dtype) for k, v in w.items()}
     eps = cfg["norm"]["eps"]
     x = x0 = embed(tokens, w, cfg["embedding"])
@@ -165,6 +174,8 @@ def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int], trace: Opt
             mix = lambda h: latent_attention(h, w, p + "mix.", layer["mixer"], eps)
         x = sublayer(x, w, p, 1, eps, mix)
         if layer.get("mlp") is not None:
+            if gaps is not None and layer["mlp"]["kind"] == "moe":
+                gaps.append(choice_gap(scalar_norm(x, w[p + "norm2"], eps), w, p + "mlp.", layer["mlp"]["router"]))
             x = sublayer(x, w, p, 2, eps, lambda h: feed_forward(h, w, p + "mlp.", layer["mlp"]))
         if trace is not None:
             trace.append(x)
@@ -176,3 +187,109 @@ def greedy(cfg: dict, w: Dict[str, torch.Tensor], prompt: List[int], n: int) -> 
     for _ in range(n):
         ids.append(int(forward(cfg, w, ids)[-1].argmax()))
     return ids[len(prompt):]
+
+
+# ---- random models of any size ------------------------------------------------------------------
+def make_config(width=96, vocab=211, eps=3e-5, layers=None, loop=None, scale=0.8, bigram=(101, 7, 3),
+                logit_scale=0.6) -> dict:
+    return {"architecture": "Movalorn", "width": width, "vocab": vocab, "norm": {"eps": eps},
+            "embedding": {"scale": scale, "bigram": dict(zip(("buckets", "mul_prev", "mul_cur"), bigram))},
+            "loop": None if loop is None else dict(zip(("start", "stop", "times"), loop)), "layers": layers,
+            "logit_scale": logit_scale}
+
+
+def dense(ff: int) -> dict:
+    return {"kind": "dense", "ff": ff}
+
+
+def experts(n: int, top: int, ff: int, shared: Optional[int], scale=1.3) -> dict:
+    m = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": n, "top": top, "scale": scale}}
+    return dict(m, shared={"ff": shared}) if shared else m
+
+
+def attention_layer(mlp, heads=3, dim=24, rot_dim=8, vdim=40, kv_rank=56, scale=0.17, window=17, base=3000.0) -> dict:
+    return {"type": "latent_attention", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "scale": scale,
+                      "mask": {"size": window}, "rot": {"base": base, "dims": rot_dim}}}
+
+
+def gru_layer(mlp, width=80) -> dict:
+    return {"type": "mingru", "mlp": mlp, "mixer": {"width": width}}
+
+
+def tensor_shapes(cfg: dict) -> Dict[str, tuple]:
+    d, V = cfg["width"], cfg["vocab"]
+    out = {"embed": (V, d), "bigram": (cfg["embedding"]["bigram"]["buckets"] + 1, d), "final.norm": (), "head": (V, d)}
+    if cfg.get("loop"):
+        out.update({"loop.in": (d, 2 * d), "loop.step": (cfg["loop"]["times"], d)})
+
+    def ffn(p, ff):
+        out.update({p + "gate": (ff, d), p + "up": (ff, d), p + "down": (d, ff)})
+
+    for i, layer in enumerate(cfg["layers"]):
+        m, p, mlp = layer["mixer"], f"l{i}.", layer.get("mlp")
+        for n in (1, 2) if mlp is not None else (1,):
+            out.update({f"{p}norm{n}": (), f"{p}norm{n}b": (), f"{p}rg{n}": (d, d), f"{p}rg{n}.b": (d,)})
+        if layer["type"] == "mingru":
+            n = m["width"]
+            out.update({p + "mix.z": (n, d), p + "mix.z.b": (n,), p + "mix.x": (n, d), p + "mix.x.b": (n,),
+                        p + "mix.g": (n, d), p + "mix.o": (d, n)})
+        else:
+            H, dk, dr, dv, r = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+            out.update({p + "mix.q": (H * (dk + dr), d), p + "mix.dkv": (r + dr, d), p + "mix.dkv.norm": (r,),
+                        p + "mix.uk": (H * dk, r), p + "mix.uv": (H * dv, r), p + "mix.g": (H, d),
+                        p + "mix.o": (d, H * dv)})
+        if mlp is None:
+            continue
+        if mlp["kind"] == "dense":
+            ffn(p + "mlp.", mlp["ff"])
+            continue
+        E = mlp["router"]["experts"]
+        out.update({p + "mlp.router": (E, d), p + "mlp.correction": (E,)})
+        for e in range(E):
+            ffn(f"{p}mlp.e{e}.", mlp["expert"]["ff"])
+        if mlp.get("shared"):
+            ffn(p + "mlp.shared.", mlp["shared"]["ff"])
+    return out
+
+
+def random_weights(cfg: dict, seed: int = 0, qk_gain: float = 1.0, classes: int = 0) -> Dict[str, torch.Tensor]:
+    """bf16 weights; qk_gain > 1 sharpens the attention (single keys stand out).  classes > 0: a token's class
+    (token mod classes) stands in columns of its own through all layers, and the routers go mostly by it, so that
+    hardly any choice of experts is close."""
+    g = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, shape in tensor_shapes(cfg).items():
+        t = torch.randn(shape, generator=g, dtype=torch.float32)
+        if name.split(".")[-1].startswith("norm"):
+            t = 1.0 + 0.3 * t
+        elif name in ("embed", "bigram"):
+            t = t * (1.0 if name == "embed" else 0.7)
+        elif name.endswith(".b"):
+            t = t * 0.7
+        elif name.endswith("correction"):
+            t = t * 0.2
+        elif name.endswith("router"):
+            t = t * 2 / math.sqrt(shape[1])
+        elif name == "loop.step":
+            t = t * 0.5
+        else:
+            t = t / math.sqrt(shape[1])
+            if name.endswith((".q", ".uk", ".dkv")):
+                t = t * qk_gain
+        if classes:
+            if name in ("embed", "bigram", "loop.step"):
+                t[:, :classes] = 0
+            if name == "embed":
+                for c in range(classes):
+                    t[c::classes, c] = 8.0
+            elif name.endswith((".o", ".down", "loop.in")):
+                t[:classes] = 0
+                if name == "loop.in":
+                    t[:classes, shape[0]:shape[0] + classes] = torch.eye(classes)
+            elif name.endswith("router"):
+                t *= 0.05
+                for c in range(classes):
+                    t[:, c] = torch.linspace(-1, 1, shape[0])[torch.randperm(shape[0], generator=g)]
+        out[name] = t.to(torch.bfloat16)
+    return out

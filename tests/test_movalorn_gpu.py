@@ -1,0 +1,743 @@
+"""Movalorn on the GPU against the plain oracle (movalorn_oracle.py): each kernel alone, then the engine in fp32 and
+bf16 -- whole prompts, portions, decoding (eager and captured), mixed batches, reused slots and blocks, keys just
+inside and outside a window, long decoding, the recurrent state's rules, generation through the scheduler."""
+import math
+import threading
+
+import numpy as np
+import pytest
+import torch
+
+import movalorn_oracle as O
+from test_gefazen import rel, write_model
+from test_movalorn import MIXED
+
+pytestmark = pytest.mark.gpu
+
+F32_TOL, BF16_TOL = 3e-5, 5e-2
+TOL = {"float32": F32_TOL, "bfloat16": BF16_TOL}
+DT = list(TOL)
+# positions whose experts are chosen by less than this (of scores between 0 and 1) may take others in bf16
+CLOSE = 0.004
+
+# the aligned shape takes the decode GEMVs and the prefill GEMMs' own tiles; wide: more than 16 heads, more than
+# 64 experts, no loop; deep: long rotated parts, cached rows above 512, a window of one token
+ALIGNED = O.make_config(width=512, vocab=640, eps=1e-5, loop=(0, 2, 3), bigram=(997, 1000003, 77), layers=[
+    O.gru_layer(O.experts(8, 3, 128, 192), width=512),
+    O.attention_layer(O.dense(768), heads=4, dim=64, rot_dim=32, vdim=64, kv_rank=128, scale=0.11, window=100),
+    O.gru_layer(O.dense(512), width=512)])
+WIDE = O.make_config(width=320, vocab=333, eps=1e-6, scale=1.7, bigram=(50, 1, 1), layers=[
+    O.attention_layer(O.dense(200), heads=20, dim=32, rot_dim=16, vdim=16, kv_rank=160, scale=0.15, window=200),
+    O.attention_layer(O.experts(70, 5, 72, 40), heads=1, dim=96, rot_dim=2, vdim=160, kv_rank=40, scale=0.09, window=33),
+    O.gru_layer(O.experts(4, 4, 64, None, scale=0.7), width=200)])
+DEEP = O.make_config(width=200, vocab=150, loop=(2, 3, 1), layers=[
+    O.attention_layer(O.experts(6, 2, 100, 60), heads=3, dim=144, rot_dim=64, vdim=72, kv_rank=300, scale=0.08, window=64),
+    O.attention_layer(None, heads=2, dim=20, rot_dim=40, vdim=200, kv_rank=520, scale=0.25, window=1),
+    O.attention_layer(O.dense(33), heads=7, dim=13, rot_dim=6, vdim=9, kv_rank=21, scale=0.3, window=90, base=20.0)])
+CONFIGS = {"mixed": MIXED, "aligned": ALIGNED, "wide": WIDE, "deep": DEEP}
+SEEDS = {"mixed": 12, "aligned": 11, "wide": 12, "deep": 11}  # (no close choices of experts)
+_cache, _want = {}, {}
+
+
+def model(name, tmp_models, qk_gain=1.5):
+    """(folder, config, weights) of a configuration, written once."""
+    if name not in _cache:
+        cfg = CONFIGS[name]
+        w = O.random_weights(cfg, seed=SEEDS[name], qk_gain=qk_gain, classes=3)
+        _cache[name] = (write_model(tmp_models / ("movalorn-" + name), cfg, w), cfg, w)
+    return _cache[name]
+
+
+def oracle(name, cfg, w, ids):
+    """(logits, positions whose experts are not a close call), computed once per model and prompt."""
+    key = (name, tuple(ids))
+    if key not in _want:
+        gaps = []
+        lg = O.forward(cfg, w, ids, gaps=gaps)
+        far = torch.stack(gaps).min(0).values > CLOSE if gaps else torch.ones(len(ids), dtype=torch.bool)
+        _want[key] = (lg, far)
+    return _want[key]
+
+
+def same(got, want, far, dtype):
+    if dtype == "float32":
+        return rel(got, want) < F32_TOL
+    assert len(far) < 30 or far.float().mean() > 0.9
+    return not far.any() or rel(got[far], want[far]) < BF16_TOL
+
+
+def engine(path, dtype="bfloat16", **kw):
+    from aios_amd.runtime.loader import load_engine
+
+    kw = dict(dict(max_slots=4, max_batch=8, max_ctx=512), **kw)
+    return load_engine(path, compute=dtype, **kw)[0]
+
+
+def ids_of(cfg, n, seed=0):
+    return [int(t) for t in np.random.default_rng(seed).integers(0, cfg["vocab"], n)]
+
+
+def run(eng, slot, ids, sizes, start=0):
+    """Feed ids in portions of the given sizes (the last repeats); logits of every position."""
+    out, at, k = [], 0, 0
+    while at < len(ids):
+        n = min(sizes[min(k, len(sizes) - 1)], len(ids) - at)
+        out.append(eng.step([slot], [start + at], [n], ids[at:at + n], list(range(n))))
+        at += n
+        k += 1
+    return torch.from_numpy(np.concatenate(out))
+
+
+# ---- kernels alone -----------------------------------------------------------------------------------
+def dev(t):
+    return t.cuda().contiguous()
+
+
+def E():
+    from aios_amd.runtime import native
+
+    return native.require()
+
+
+def stream():
+    return torch.cuda.current_stream().cuda_stream
+
+
+def pad(n, m):
+    return (n + m - 1) // m * m
+
+
+def bf(t):
+    return t.to(torch.bfloat16).float()
+
+
+def padded(t, n):
+    return torch.nn.functional.pad(t, (0, n - t.shape[-1]))
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+def test_embedding_rows_kernel(f32):
+    """Two portions and a single token, then their next tokens, one of which runs twice."""
+    V, d, dp, slots, bk = 50, 200, 256, 4, 13
+    g = torch.Generator().manual_seed(3)
+    tab, pair = torch.randn(V, d, generator=g).bfloat16(), torch.randn(bk + 1, d, generator=g).bfloat16()
+    seqs = {0: ids_of({"vocab": V}, 9, 1), 3: ids_of({"vocab": V}, 6, 2), 1: ids_of({"vocab": V}, 4, 3)}
+    want = {s: O.embed(t, {"embed": tab.double(), "bigram": pair.double()},
+                       {"scale": 0.75, "bigram": {"mul_prev": 10 ** 9 + 7, "mul_cur": 5, "buckets": bk}}) for s, t in seqs.items()}
+    last = torch.full((2, slots), -12345, dtype=torch.int32, device="cuda")
+    tabd, paird, gd = dev(padded(tab, dp)), dev(padded(pair, dp)), dev(padded(torch.full((d,), 0.5), dp))
+    dt = torch.float32 if f32 else torch.bfloat16
+
+    def go(entries, decode):  # (slot, start, n)
+        tok, pos, slot, rn = [], [], [], []
+        for s, st, n in entries:
+            tok += seqs[s][st:st + n]
+            pos += range(st, st + n)
+            slot += [s] * n
+            rn += [n] + [0] * (n - 1)
+        D = [torch.tensor(v, dtype=torch.int32, device="cuda") for v in (tok, pos, slot, rn)]
+        n = len(tok)
+        x, keep, out = torch.zeros(n, dp, device="cuda"), torch.zeros(n, 2 * dp, dtype=dt, device="cuda"), torch.zeros(n, dp, dtype=dt, device="cuda")
+        E().embed_rows(n, tabd.data_ptr(), 0.75, paird.data_ptr(), bk, 10 ** 9 + 7, 5, D[0].data_ptr(), D[1].data_ptr(),
+                       D[2].data_ptr(), 0 if decode else D[3].data_ptr(), last.data_ptr(), slots, dp, d, 1e-4, x.data_ptr(),
+                       keep.data_ptr() + keep.element_size() * dp, 2 * dp, f32, E().NEXT_NORM, gd.data_ptr(), out.data_ptr(),
+                       dp, stream())
+        torch.cuda.synchronize()
+        w = torch.cat([want[s][st:st + n] for s, st, n in entries])
+        assert (x.cpu()[:, :d].double() - w).abs().max() < 1e-6 and (x[:, d:] == 0).all()
+        tol = 1e-5 if f32 else 2e-2
+        assert (keep.cpu()[:, dp:dp + d].double() - w).abs().max() < tol and (keep[:, :dp] == 0).all()
+        assert (out.cpu()[:, :d].double() - 0.5 * O.rms(w, 1e-4)).abs().max() < tol and (out[:, d:] == 0).all()
+
+    go([(0, 0, 2), (3, 0, 3), (1, 0, 1)], False)
+    go([(0, 2, 1), (1, 1, 1), (3, 3, 1)], True)
+    go([(3, 3, 1), (0, 2, 1)], True)          # the same tokens once more
+    go([(1, 1, 3), (0, 3, 4), (3, 4, 2)], False)
+    seqs[0] = seqs[0][::-1]                   # a new sequence in the slot
+    want[0] = O.embed(seqs[0], {"embed": tab.double(), "bigram": pair.double()},
+                      {"scale": 0.75, "bigram": {"mul_prev": 10 ** 9 + 7, "mul_cur": 5, "buckets": bk}})
+    go([(0, 0, 1)], True)
+    go([(0, 1, 8)], False)
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+@pytest.mark.parametrize("d, rows", [(50, 3), (256, 70), (1000, 5), (5000, 2), (9000, 3)])
+def test_row_close_kernel(d, rows, f32):
+    m, g = E(), torch.Generator().manual_seed(d)
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    dp, top, dt, eps = pad(d, 64), 5, torch.float32 if f32 else torch.bfloat16, 1e-3
+    x, y, gate, gb, post, nx, add = rnd(rows, d), rnd(rows, d), rnd(rows, d), rnd(d), rnd(d), rnd(d), rnd(d)
+    ye, wt = rnd(rows * top, d).to(dt), rnd(rows, top)
+    pair = torch.randperm(rows * top, generator=g).view(rows, top).int()
+    D = [dev(padded(t, dp)) for t in (x, y, ye)]
+    V = [dev(padded(t, dp)) for t in (gb, post, nx, add)]
+    gd = dev(torch.cat([rnd(rows, 64), padded(gate, dp)], 1))
+    pd, wd = dev(pair), dev(wt)
+    moe = (wt[..., None].double() * ye.double()[pair.long()]).sum(1)
+    cases = [(True, True, True, True), (False, True, False, True), (True, False, True, False), (True, False, False, False)]
+    for use_y, use_e, use_gate, use_post in cases:
+        v = (y.double() if use_y else 0) + (moe if use_e else 0)
+        if use_gate:
+            v = v * torch.sigmoid(gate.double() + gb.double())
+        if use_post:
+            v = O.rms(v, eps) * post.double()
+        for replace in (0, 1):
+            want = (y.double() + add.double()) if replace else x.double() + v
+            for kind in (m.NEXT_NONE, m.NEXT_NORM, m.NEXT_RAW):
+                xd, out = D[0].clone(), torch.zeros(rows, dp + 64, dtype=dt, device="cuda")
+                kw = dict(replace=1, add=V[3].data_ptr()) if replace else dict(
+                    ye=D[2].data_ptr() if use_e else 0, pair=pd.data_ptr(), wt=wd.data_ptr(), top=top,
+                    gate=gd.data_ptr() + 256 if use_gate else 0, ldg=dp + 64, gate_bias=V[0].data_ptr(),
+                    post=V[1].data_ptr() if use_post else 0)
+                m.row_close(rows, xd.data_ptr(), dp, d, eps, D[1].data_ptr() if use_y or replace else 0, f32=f32, next=kind,
+                            g=V[2].data_ptr(), out=out.data_ptr(), ldo=dp + 64, stream=stream(), **kw)
+                torch.cuda.synchronize()
+                assert (xd.cpu()[:, :d].double() - want).abs().max() < 2e-5 and (xd[:, d:] == 0).all()
+                nxt = {m.NEXT_NONE: want * 0, m.NEXT_NORM: O.rms(want, eps) * nx.double(), m.NEXT_RAW: want}[kind]
+                tol = 3e-5 if f32 else 1e-2 * float(nxt.abs().max()) + 1e-6
+                assert (out.cpu()[:, :d].double() - nxt).abs().max() <= tol and (out[:, d:] == 0).all()
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+@pytest.mark.parametrize("w", [64, 320])
+def test_mingru_kernel(w, f32):
+    """Portions of unequal lengths at chunk borders, continued by others; single tokens, one of them twice; a slot
+    taken over by a new sequence."""
+    g = torch.Generator().manual_seed(w)
+    slots, ld = 6, 3 * w + 64
+    dt = torch.float32 if f32 else torch.bfloat16
+    zb, ub = torch.randn(w, generator=g), torch.randn(w, generator=g)
+    lens = {0: 400, 2: 300, 5: 200, 3: 150}
+    X = {s: torch.randn(n, 3, w, generator=g) * 2 for s, n in lens.items()}
+    ref = lambda x: O.mingru_states(x[:, 0].double() + zb.double(), x[:, 1].double() + ub.double()) * O.silu(x[:, 2].double())
+    want = {s: ref(x) for s, x in X.items()}
+    state = torch.full((2, slots, w), 1e30, device="cuda")
+    agg, work = torch.zeros(64, 3, w, device="cuda"), torch.zeros(64 * 6, dtype=torch.int32, device="cuda")
+    zd, ud = dev(zb), dev(ub)
+
+    def go(entries, decode=False):
+        rows = torch.cat([X[s][st:st + n] for s, st, n in entries])
+        n = rows.shape[0]
+        inp = torch.zeros(n, ld)
+        inp[:, :w], inp[:, w:2 * w], inp[:, 2 * w + 64:] = rows[:, 1], rows[:, 0], rows[:, 2]
+        inp, out = dev(inp), torch.zeros(n, w + 64, dtype=dt, device="cuda")
+        pieces, at, pos, slot = [], 0, [], []
+        for s, st, k in entries:
+            pieces.append([at, k, s, st])
+            pos.append(st)
+            slot.append(s)
+            at += k
+        pd, sd = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in (pos, slot))
+        E().mingru([] if decode else pieces, n, pd.data_ptr(), sd.data_ptr(), inp.data_ptr(), ld, w, 0, 2 * w + 64, zd.data_ptr(),
+                   ud.data_ptr(), w, state.data_ptr(), slots, agg.data_ptr(), work.data_ptr(), out.data_ptr(), w + 64, f32, stream())
+        torch.cuda.synchronize()
+        ref = torch.cat([want[s][st:st + k] for s, st, k in entries])
+        err = (out.cpu()[:, :w].double() - ref).abs().max() / ref.abs().max()
+        assert err < (2e-6 if f32 else 6e-3), (entries, float(err))
+
+    go([(0, 0, 1), (2, 0, 64), (5, 0, 2), (3, 0, 63)])
+    go([(0, 1, 130), (2, 64, 65), (5, 2, 1)])
+    go([(0, 131, 1), (5, 3, 1), (3, 63, 1), (2, 129, 1)], True)
+    go([(5, 3, 1), (0, 131, 1), (2, 129, 1)], True)                 # once more at the same positions
+    go([(5, 4, 1), (2, 130, 1)], True)
+    go([(2, 131, 128), (0, 132, 200), (3, 64, 86), (5, 5, 3)])      # even lengths: in and out at one parity
+    go([(0, 332, 68), (2, 259, 41)])
+    X[0] = torch.randn(140, 3, w, generator=g)
+    want[0] = ref(X[0])
+    go([(0, 0, 129), (5, 8, 192)])
+    go([(0, 129, 11)])
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+@pytest.mark.parametrize("H, dk, dr, dv, rank, window, gate", [
+    (4, 64, 16, 48, 96, 40, "head"), (20, 24, 8, 40, 150, 64, "element"), (1, 128, 64, 128, 512, 7, "head"),
+    (33, 13, 6, 16, 700, 65, "none"), (2, 32, 32, 32, 1000, 130, "head"), (3, 20, 10, 20, 33, 1, "head"), (5, 16, 4, 16, 60, 0, "head")])
+def test_latent_attention_kernel_with_a_rotated_part_and_a_window(H, dk, dr, dv, rank, window, gate, f32):
+    """Absorbed attention over a paged cache whose blocks are scattered: unequal sequences (one token each, as in
+    decoding, and a portion of several), several key splits, windows that end at tile and block borders."""
+    g = torch.Generator().manual_seed(H * 1000 + rank)
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    qrot, roff = pad(dk, 8), pad(rank, 8)
+    dkp, dvp = pad(qrot + dr, 32), pad(dv, 32)
+    rp = next(64 * t for t in (2, 4, 6, 8, 10, 12, 16, 32) if roff + dr <= 64 * t)
+    lens, portion, kvb, maxb = [1, 64, 65, 200, 129], 7, 64, 6
+    seqs = [(i, l - 1, 1) for i, l in enumerate(lens)] + [(5, 122, portion)]  # slot, start, new tokens
+    n, nslot = sum(s[2] for s in seqs), 6
+    uk, uv = bf(rnd(H, dk, rank) / math.sqrt(rank)), bf(rnd(H, dv, rank) / math.sqrt(rank))
+    kvn, base = 1 + 0.2 * rnd(rank), 300.0
+    scale, eps = 1.5 / math.sqrt(dk + dr), 1e-5
+    perm = torch.randperm(nslot * maxb, generator=g).view(nslot, maxb)
+    P = maxb * kvb
+    ang = torch.arange(P, dtype=O.DT)[:, None] * base ** (-2.0 * torch.arange(dr // 2, dtype=O.DT) / dr)
+    rope = torch.stack([ang.cos(), ang.sin()], -1).float()
+    turn = lambda v, p: O.rotate(torch.cat([torch.zeros(p, *v.shape[1:], dtype=O.DT), v.double()]), base, dr)[p:]
+    pool = torch.zeros(nslot * maxb + 1, kvb, rp)
+    ctx = {s: (bf(rnd(st, rank)), bf(rnd(st, dr))) for s, st, _ in seqs}
+    for s, st, _ in seqs:
+        for p in range(st):
+            pool[perm[s, p // kvb], p % kvb, :rank] = ctx[s][0][p]
+            pool[perm[s, p // kvb], p % kvb, roff:roff + dr] = ctx[s][1][p]
+    gn = {"head": pad(H, 64), "element": pad(H * dvp, 64), "none": 0}[gate]
+    dkv_off = pad(H * dkp, 64)
+    g_off, ld = dkv_off + rp, dkv_off + rp + gn
+    qdg = torch.zeros(n, ld)
+    q, dkv, gt = rnd(n, H, dk + dr) * 2, rnd(n, rank + dr), rnd(n, H, dv)
+    qv = qdg[:, :H * dkp].view(n, H, dkp)
+    qv[:, :, :dk], qv[:, :, qrot:qrot + dr] = q[..., :dk], q[..., dk:]
+    qdg[:, dkv_off:dkv_off + rank], qdg[:, dkv_off + roff:dkv_off + roff + dr] = dkv[:, :rank], dkv[:, rank:]
+    if gate == "head":
+        qdg[:, g_off:g_off + H] = gt[..., 0]
+        gt = gt[..., :1].expand(n, H, dv)
+    elif gate == "element":
+        qdg[:, g_off:g_off + H * dvp].view(n, H, dvp)[:, :, :dv] = gt
+    pos, slot, tiles, row = [], [], [], 0
+    want = torch.zeros(n, H, dv, dtype=O.DT)
+    for s, st, k in seqs:
+        pos += list(range(st, st + k))
+        slot += [s] * k
+        tiles += [(f, min(16, (row + k) * H - f)) for f in range(row * H, (row + k) * H, 16)]
+        c_new = O.rms(dkv[row:row + k, :rank].double(), eps) * kvn.double()
+        r_new = turn(dkv[row:row + k, rank:], st)
+        if not f32:
+            c_new, r_new = c_new.to(torch.bfloat16).double(), r_new.to(torch.bfloat16).double()
+        c, r = torch.cat([ctx[s][0].double(), c_new]), torch.cat([ctx[s][1].double(), r_new])
+        qr = turn(q[row:row + k, :, dk:], st)
+        for i in range(k):
+            see = O.visible(st + i, window or P)
+            a, b = see.start, see.stop
+            for h in range(H):
+                sc = (c[a:b] @ uk[h].double().T) @ q[row + i, h, :dk].double() + r[a:b] @ qr[i, h]
+                o = torch.softmax(sc * scale, 0) @ (c[a:b] @ uv[h].double().T)
+                want[row + i, h] = o * torch.sigmoid(gt[row + i, h].double()) if gate != "none" else o
+        row += k
+    dt = torch.float32 if f32 else torch.bfloat16
+    wukT, wuv = torch.zeros(H, rp, dkp), torch.zeros(H, dvp, rp)
+    wukT[:, :rank, :dk] = uk.transpose(1, 2)
+    for i in range(dr):
+        wukT[:, roff + i, qrot + i] = 1
+    wuv[:, :dv, :rank] = uv
+    D = dict(norm=padded(kvn, rp), pool=pool.to(dt), wukT=wukT.bfloat16(), wuv=wuv.bfloat16(), qdg=qdg, bt=perm.int(), rope=rope,
+             pos=torch.tensor(pos, dtype=torch.int32), slot=torch.tensor(slot, dtype=torch.int32),
+             tiles=torch.tensor(tiles, dtype=torch.int32))
+    D = {k: dev(v) for k, v in D.items()}
+    for nsplit in (1,) if f32 or rp > 1024 else (1, 3, 64):
+        out = torch.zeros(n, H * dvp, dtype=dt, device="cuda")
+        qa = torch.zeros(n, H, rp, dtype=dt, device="cuda")
+        part = torch.zeros(nsplit, n * H, rp, device="cuda")
+        ml = torch.zeros(nsplit, n * H, 2, device="cuda")
+        E().latent_attention(n, n, H, dk, dkp, dvp, rank, rp, scale, eps, D["norm"].data_ptr(), 0, D["qdg"].data_ptr(), ld, dkv_off,
+                             g_off if gate != "none" else -1, D["pos"].data_ptr(), D["slot"].data_ptr(), D["pool"].data_ptr(),
+                             D["bt"].data_ptr(), maxb, kvb, f32, D["wukT"].data_ptr(), D["wuv"].data_ptr(), qa.data_ptr(),
+                             D["tiles"].data_ptr(), len(tiles), nsplit, part.data_ptr(), ml.data_ptr(), out.data_ptr(), H * dvp,
+                             stream(), rot=dr, roff=roff, qrot=qrot, rope=D["rope"].data_ptr(), window=window,
+                             head_gate=int(gate == "head"))
+        torch.cuda.synchronize()
+        got = out.float().cpu().view(n, H, dvp)
+        assert (got[:, :, dv:] == 0).all()
+        err = (got[:, :, :dv].double() - want).abs().max() / want.abs().max()
+        assert err < (2e-5 if f32 else 3e-2), (nsplit, float(err))
+
+
+@pytest.mark.parametrize("H, dk, dr, dv, start, T, window, pos0", [
+    (2, 64, 32, 64, 0, 300, 100, 0), (3, 24, 8, 40, 77, 2, 40, 500), (1, 96, 32, 128, 63, 130, 64, 63), (2, 160, 64, 96, 128, 65, 1, 700),
+    (4, 40, 0, 64, 190, 164, 129, 190), (2, 13, 6, 16, 39, 257, 40, 1000)])
+def test_mha_prefill_kernel_with_a_rotated_part_and_a_window(H, dk, dr, dv, start, T, window, pos0):
+    """Queries are rotated in the kernel, by their own positions (the keys' buffer starts anywhere)."""
+    g = torch.Generator().manual_seed(T * 7 + dk)
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    qrot = pad(dk, 8)
+    dkp, dvp, S = pad(qrot + dr, 32), pad(dv, 32), start + T
+    q, k, v, gt = rnd(T, H, dk + dr), bf(rnd(S, H, dk + dr)), bf(rnd(S, H, dv)), rnd(T, H)
+    base, P = 700.0, pos0 + T
+    scale = 2 / math.sqrt(dk + dr)
+    qr = q.double()
+    if dr:
+        qr = torch.cat([qr[..., :dk], O.rotate(torch.cat([torch.zeros(pos0, H, dr, dtype=O.DT), qr[..., dk:]]), base, dr)[pos0:]], -1)
+    want = torch.zeros(T, H, dv, dtype=O.DT)
+    for i in range(T):
+        see = O.visible(start + i, window)
+        for h in range(H):
+            p = torch.softmax((k[see.start:see.stop, h].double() @ qr[i, h]) * scale, 0)
+            want[i, h] = p @ v[see.start:see.stop, h].double() * torch.sigmoid(gt[i, h].double())
+    ang = torch.arange(P, dtype=O.DT)[:, None] * base ** (-2.0 * torch.arange(dr // 2, dtype=O.DT) / max(dr, 1))
+    rope = dev(torch.stack([ang.cos(), ang.sin()], -1).float()) if dr else torch.zeros(1, device="cuda")
+
+    def spread(t, n):
+        o = torch.zeros(n, H, dkp)
+        o[..., :dk], o[..., qrot:qrot + dr] = t[..., :dk], t[..., dk:]
+        return o.view(n, H * dkp)
+
+    ldq, ldkv = H * dkp + 64, H * (dkp + dvp)
+    qb, kv = torch.zeros(T, ldq), torch.zeros(S, ldkv, dtype=torch.bfloat16)
+    qb[:, :H * dkp], qb[:, H * dkp:H * dkp + H] = spread(q, T), gt
+    kv[:, :H * dkp] = spread(k, S).bfloat16()
+    kv[:, H * dkp:].view(S, H, dvp)[:, :, :dv] = v.bfloat16()
+    qb, kv = dev(qb), dev(kv)
+    out = torch.zeros(T, H * dvp, dtype=torch.bfloat16, device="cuda")
+    E().mha_prefill(qb.data_ptr(), ldq, kv.data_ptr(), kv.data_ptr() + 2 * H * dkp, ldkv, H, dkp, dvp, start, T, scale, 0,
+                    qb.data_ptr() + 4 * H * dkp, out.data_ptr(), H * dvp, stream(), window=window, rot=dr, qrot=qrot, pos0=pos0,
+                    rope=rope.data_ptr(), head_gate=1)
+    torch.cuda.synchronize()
+    got = out.float().cpu().view(T, H, dvp)[:, :, :dv].double()
+    err = (got - want).abs().max() / want.abs().max()
+    assert err < 2e-2, float(err)
+
+
+@pytest.mark.parametrize("kind", ["few", "grouped", "f32"])
+@pytest.mark.parametrize("n, experts, top, ff, d, skew", [
+    (1, 12, 3, 96, 256, 0), (4, 5, 1, 64, 320, 0), (3, 3, 3, 200, 512, 0), (2, 300, 8, 64, 128, 0), (40, 6, 2, 72, 192, 0),
+    (64, 70, 5, 128, 256, 0), (65, 8, 2, 128, 448, 4), (300, 4, 2, 192, 320, 0), (500, 9, 3, 130, 192, 3), (130, 1000, 2, 64, 64, 0)])
+def test_experts_kernels(n, experts, top, ff, d, skew, kind):
+    """Every form of the routed experts; skew: most tokens want the same experts, some experts have none."""
+    if kind == "few" and n > E().MOE_FEW:
+        pytest.skip("more tokens than this form takes")
+    m, g = E(), torch.Generator().manual_seed(n * 31 + experts)
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    f32 = int(kind == "f32")
+    dt = torch.float32 if f32 else torch.bfloat16
+    dp, fp, shf = pad(d, 64), pad(ff, 64), 64
+    h = padded(rnd(n, d), dp).to(dt)
+    logits = rnd(n, experts) * 1.5
+    logits[:, :2] += skew
+    corr = rnd(experts) * 0.2
+    wg, wu, wd = (bf(rnd(experts, ff, d) / math.sqrt(d)), bf(rnd(experts, ff, d) / math.sqrt(d)), bf(rnd(experts, d, ff) / math.sqrt(ff)))
+    s = torch.softmax(logits.double(), -1)
+    pick = torch.topk(s + corr.double(), top, -1).indices
+    wt = torch.gather(s, 1, pick) * 1.7
+    want = torch.zeros(n, d, dtype=O.DT)
+    for t in range(n):
+        for k in range(top):
+            e, x = int(pick[t, k]), h[t, :d].double()
+            want[t] += wt[t, k] * ((O.silu(wg[e].double() @ x) * (wu[e].double() @ x)) @ wd[e].double().T)
+    wgu, wdn = torch.zeros(experts, 2 * fp, dp), torch.zeros(experts, dp, fp)
+    wgu[:, 0:2 * ff:2, :d], wgu[:, 1:2 * ff:2, :d], wdn[:, :d, :ff] = wg, wu, wd
+    sh_act, sh_dn = bf(rnd(n, shf)), bf(padded(rnd(d, shf) / 8, shf))
+    lpad = torch.zeros(n, experts + 64)
+    lpad[:, 64:] = logits
+    D = dict(h=h, l=lpad, corr=corr, wgu=wgu.bfloat16(), wdn=wdn.bfloat16(), sa=sh_act.bfloat16(),
+             sd=torch.nn.functional.pad(sh_dn, (0, 0, 0, dp - d)).bfloat16())
+    D = {k: dev(v) for k, v in D.items()}
+    P, tiles = n * top, experts + n * top // 16 + 1
+    I = lambda *s: torch.full(s, -7, dtype=torch.int32, device="cuda")
+    sel, pair, token, tl, nt = I(P), I(P), I(P), I(tiles, 4), I(1)
+    wtd, act, ye = torch.zeros(P, device="cuda"), torch.zeros(P, fp, dtype=dt, device="cuda"), torch.zeros(P, dp, dtype=dt, device="cuda")
+    gu, y = torch.zeros(P, 2 * fp, device="cuda"), torch.zeros(n, dp, device="cuda")
+    kw = dict(sh_act=D["sa"].data_ptr(), ld_sh=shf, sh_ff=shf, sh_dn=D["sd"].data_ptr(), y=y.data_ptr()) if kind == "few" else {}
+    m.moe(kind == "few", n, experts, top, 1.7, D["l"].data_ptr() + 256, experts + 64, D["corr"].data_ptr(), dp, fp, m.ACT_SILU,
+          D["h"].data_ptr(), dp, D["wgu"].data_ptr(), D["wdn"].data_ptr(), sel.data_ptr(), wtd.data_ptr(), pair.data_ptr(),
+          token.data_ptr(), tl.data_ptr(), nt.data_ptr(), tiles, act.data_ptr(), ye.data_ptr(), gu.data_ptr(), f32, stream=stream(), **kw)
+    torch.cuda.synchronize()
+    assert torch.equal(sel.cpu().view(n, top).long(), pick)
+    assert (wtd.cpu().view(n, top).double() - wt).abs().max() < 1e-6
+    if kind == "few":
+        got = y.cpu().double()
+        want = want + sh_act.double() @ sh_dn.double().T
+    else:
+        at = pair.cpu().view(n, top).long()
+        assert sorted(at.view(-1).tolist()) == list(range(P))
+        assert torch.equal(token.cpu()[at.view(-1)], torch.arange(n, dtype=torch.int32).repeat_interleave(top))
+        got = (ye.cpu().double()[at] * wtd.cpu().view(n, top, 1).double()).sum(1)
+    assert (got[:, d:] == 0).all()
+    err = (got[:, :d] - want).abs().max() / want.abs().max()
+    assert err < (3e-6 if f32 else 1.5e-2), float(err)
+
+
+# ---- the engine against the oracle ----------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_whole_prompt_portions_and_decode(name, dtype, tmp_models):
+    path, cfg, w = model(name, tmp_models)
+    ids = ids_of(cfg, 270)
+    want, far = oracle(name, cfg, w, ids)
+    eng = engine(path, dtype)
+    assert same(run(eng, 0, ids, [len(ids)]), want, far, dtype)
+    for slot, sizes in ((1, [2]), (2, [3, 61, 64, 1, 128, 5, 7]), (3, [130, 1]), (1, [1])):
+        n = 40 if sizes in ([2], [1]) else 160
+        eng.release_slot(slot)
+        assert same(run(eng, slot, ids[:n], sizes), want[:n], far[:n], dtype), sizes
+
+
+def test_residual_after_every_layer_run(tmp_models):
+    path, cfg, w = model("aligned", tmp_models)
+    ids, trace = ids_of(cfg, 50, 9), []
+    O.forward(cfg, w, ids, trace)
+    eng = engine(path, "float32")
+    assert eng.layer_runs == len(trace) == 7
+    for k in range(7):
+        eng.set_run_limit(k + 1)
+        eng.step([0], [0], [50], ids, [])
+        assert (torch.from_numpy(eng.last_residual(50)).double() - trace[k]).abs().max() < 1e-4
+    eng.set_run_limit(-1)
+    assert rel(run(eng, 0, ids, [50]), oracle("aligned", cfg, w, ids)[0]) < F32_TOL
+
+
+@pytest.mark.parametrize("name", ["aligned", "wide", "deep"])
+def test_long_portions_on_a_long_context(name, tmp_models, monkeypatch):
+    """Expanded attention from 32-token portions on, and passes of at most 96 rows: every border between the two
+    forms and between the passes of one step."""
+    monkeypatch.setenv("AIOS_LATENT_PF_MIN", "32")
+    monkeypatch.setenv("AIOS_STEP_ROWS", "96")
+    path, cfg, w = model(name, tmp_models)
+    ids = ids_of(cfg, 390, 3)
+    want, far = oracle(name, cfg, w, ids)
+    eng = engine(path)
+    assert same(run(eng, 0, ids, [390]), want, far, "bfloat16")
+    assert same(run(eng, 1, ids, [33, 31, 64, 2, 100, 97, 32]), want, far, "bfloat16")
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("name", ["mixed", "aligned"])
+def test_mixed_batches_equal_each_alone(name, dtype, tmp_models):
+    """Portions of some requests beside decoded tokens of others; a request pauses; slots and blocks are reused."""
+    path, cfg, w = model(name, tmp_models)
+    lens = [150, 9, 70, 33, 101, 64]
+    seqs = [ids_of(cfg, n, 20 + i) for i, n in enumerate(lens)]
+    want = [oracle(name, cfg, w, s) for s in seqs]
+    eng = engine(path, dtype, kv_pool_tokens=7 * 64)
+    rng = np.random.default_rng(4)
+    free, live, todo, got = [0, 1, 2, 3], {}, list(range(6)), [[] for _ in seqs]
+    while todo or live:
+        while todo and free and sum(-(-lens[i] // 64) for i in list(live) + todo[:1]) <= 7:
+            i = todo.pop(0)
+            live[i] = [free.pop(), 0]
+        entries = [i for i in live if rng.random() < 0.8] or list(live)[:1]
+        counts = [min(int(rng.choice([1, 1, 2, 5, 40, 66])), lens[i] - live[i][1]) for i in entries]
+        toks = [t for i, n in zip(entries, counts) for t in seqs[i][live[i][1]:live[i][1] + n]]
+        out = eng.step([live[i][0] for i in entries], [live[i][1] for i in entries], counts, toks, list(range(len(toks))))
+        at = 0
+        for i, n in zip(entries, counts):
+            got[i].append(torch.from_numpy(out[at:at + n].copy()))
+            at += n
+            live[i][1] += n
+            if live[i][1] == lens[i]:
+                eng.release_slot(live[i][0])
+                free.append(live.pop(i)[0])
+    assert eng.kv_blocks_free == 7
+    for i in range(6):
+        assert same(torch.cat(got[i]), *want[i], dtype), i
+
+
+@pytest.mark.parametrize("name", ["mixed", "aligned"])
+@pytest.mark.parametrize("dtype", DT)
+def test_captured_decode_equals_the_oracle(name, dtype, tmp_models):
+    """The decode graphs (every batch size's kernels: GEMV, skinny and prefill GEMM, both forms of the experts) replayed
+    step after step with other engine work in between, across a block border; logits of every replay."""
+    path, cfg, w = model(name, tmp_models)
+    seqs = [ids_of(cfg, 60 + 3 * (i % 6), 50 + i % 6) for i in range(40)]
+    want = [oracle(name, cfg, w, s) for s in seqs[:6]]
+    eng = engine(path, dtype, max_slots=41, max_batch=40, max_ctx=128)
+    for B in (1, 2, 4, 5, 6, 40):
+        start = [len(s) - 9 for s in seqs[:B]]
+        for b in range(B):
+            eng.release_slot(b)
+            eng.prefill(b, seqs[b][:start[b]], 0, False)
+        got = [[] for _ in range(B)]
+        for t in range(9):
+            eng.decode(list(range(B)), [seqs[b][start[b] + t] for b in range(B)], [start[b] + t for b in range(B)])
+            lg = torch.from_numpy(eng.last_logits(B))
+            for b in range(B):
+                got[b].append(lg[b:b + 1])
+            if t == 4:
+                eng.prefill(40, seqs[0][:5], 0, True)  # eager work between two replays
+        for b in range(B):
+            wl, far = want[b % 6]
+            assert same(torch.cat(got[b]), wl[start[b]:], far[start[b]:], dtype), (B, b)
+
+
+WINDOW = 70
+
+
+def window_model(tmp_models):
+    """Token 1 asks for token 0: the first layer's head 0 gives that pair a score far above all others, at any
+    distance inside the window (the rotated part is left out of it)."""
+    cfg = O.make_config(width=128, vocab=90, eps=1e-5, layers=[
+        O.attention_layer(O.dense(96), heads=2, dim=32, rot_dim=8, vdim=48, kv_rank=64, scale=0.3, window=WINDOW),
+        O.attention_layer(None, heads=3, dim=16, rot_dim=4, vdim=16, kv_rank=24, window=5)])
+    w = {k: v.float() for k, v in O.random_weights(cfg, 77).items()}
+    w["bigram"] *= 0.1
+    w["embed"][0, :], w["embed"][1, :] = 0.0, 0.0
+    w["embed"][0, 5], w["embed"][1, 9] = 12.0, 12.0
+    w["l0.mix.dkv"][:, 5] = 0
+    w["l0.mix.dkv"][3, 5] = 3.0
+    w["l0.mix.uk"][7, 3] = 2.0
+    w["l0.mix.q"][7, 9] = 2.0
+    w["l0.mix.uv"][:48, 3] *= 3
+    w["l0.mix.g"][0] = 0
+    return write_model(tmp_models / "movalorn-window", cfg, {k: v.to(torch.bfloat16) for k, v in w.items()}), cfg, \
+        {k: v.to(torch.bfloat16) for k, v in w.items()}
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_keys_just_inside_and_outside_the_window(dtype, tmp_models, monkeypatch):
+    path, cfg, w = window_model(tmp_models)
+    engs = [engine(path, dtype)]
+    if dtype == "bfloat16":
+        monkeypatch.setenv("AIOS_LATENT_PF_MIN", "2")  # the expanded form for every portion
+        engs.append(engine(path, dtype))
+    for n in (WINDOW + 3, 129, 192, 193, 300):
+        for dist in (0, 1, 31, 63, 64, WINDOW - 2, WINDOW - 1, WINDOW, WINDOW + 1):
+            if dist == 0 or dist >= n:
+                continue
+            ids = [2 + t % 88 for t in ids_of(cfg, n, 300 + n)]
+            ids[-1 - dist], ids[-1] = 0, 1
+            want = O.forward(cfg, w, ids)[-1:]
+            if n == 129:
+                without = O.forward(cfg, w, ids[:-1 - dist] + [50] + ids[n - dist:])[-1:]
+                if dist < WINDOW:
+                    assert rel(without, want) > 0.15  # the key is what the last position's logits rest on
+                elif dist > WINDOW + 5:
+                    assert rel(without, want) < 0.1
+            for eng in engs:
+                for slot, sizes in ((0, [n]), (1, [n - 1, 1]), (2, [40, 29, 2, 100, 1])):
+                    eng.release_slot(slot)
+                    assert rel(run(eng, slot, ids, sizes)[-1:], want) < 2 * TOL[dtype], (n, dist, sizes)
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_the_first_tokens_of_a_sequence(dtype, tmp_models):
+    path, cfg, w = model("mixed", tmp_models)
+    eng = engine(path, dtype)
+    for seed in range(4):
+        ids = ids_of(cfg, 5, 700 + seed)
+        want, far = oracle("mixed", cfg, w, ids)
+        for slot, sizes in ((0, [5]), (0, [1]), (1, [2, 3]), (1, [1, 4])):  # (slots are taken over without a release)
+            assert same(run(eng, slot, ids, sizes), want, far, dtype)
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_long_decoding_and_the_context_limit(dtype, tmp_models):
+    path, cfg, w = model("mixed", tmp_models)
+    P = 450
+    ids = ids_of(cfg, P, 8)
+    want, far = oracle("mixed", cfg, w, ids)
+    eng = engine(path, dtype, max_ctx=P)
+    run(eng, 0, ids[:P - 250], [P - 250])
+    assert same(run(eng, 0, ids[P - 250:], [1], start=P - 250), want[P - 250:], far[P - 250:], dtype)
+    with pytest.raises(RuntimeError, match="overflow"):
+        eng.step([0], [P], [1], [0], [])
+    with pytest.raises(RuntimeError):
+        eng.step([1], [0], [1], [cfg["vocab"]], [])
+
+
+def test_the_recurrent_state_stands_at_one_position(tmp_models):
+    """Where a slot may go on, a dropped single token, copies; anything else is refused before it runs."""
+    path, cfg, w = model("mixed", tmp_models)
+    a, b = ids_of(cfg, 140, 1), ids_of(cfg, 60, 2)
+    eng = engine(path, "float32")
+    assert eng.recurrent and eng.resumable(0, 0) and not eng.resumable(0, 1)
+    run(eng, 0, a, [140])
+    assert eng.resumable(0, 140) and not eng.resumable(0, 139) and not eng.resumable(0, 100)
+    for start in (100, 139, 141):
+        with pytest.raises(RuntimeError, match="state stands"):
+            eng.step([0], [start], [1], [0], [])
+        with pytest.raises(RuntimeError, match="state stands"):
+            eng.decode([0], [0], [start], [0.0], [0], 0, b"")
+        with pytest.raises(RuntimeError, match="state"):
+            eng.copy_slot(0, 1, start)
+    eng.copy_slot(0, 1, 140)
+    assert rel(run(eng, 1, b, [60], start=140), O.forward(cfg, w, a + b)[140:]) < F32_TOL
+    # a single token whose result is dropped, then another in its place; the copy's state is its own
+    run(eng, 0, [5], [1], start=140)
+    assert eng.resumable(0, 141) and eng.resumable(0, 140)
+    more = ids_of(cfg, 20, 3)
+    assert rel(run(eng, 0, more, [1], start=140), O.forward(cfg, w, a + more)[140:]) < F32_TOL
+    run(eng, 0, more, [20], start=160)
+    assert not eng.resumable(0, 179)
+
+
+def test_tensor_errors(tmp_models):
+    path, cfg, w = model("mixed", tmp_models)
+    bad = write_model(tmp_models / "mv-bad", cfg, {k: v for k, v in w.items() if k != "l1.mlp.e3.up"})
+    with pytest.raises(ValueError, match="l1.mlp.e3.up"):
+        engine(bad)
+    bad = write_model(tmp_models / "mv-bad2", cfg, dict(w, **{"l1.mix.g": w["l1.mix.g"][:2]}))
+    with pytest.raises(RuntimeError, match="attn_gate"):
+        engine(bad)
+    with pytest.raises(ValueError, match="fp8"):
+        engine(path, kv_dtype="fp8")
+
+
+# ---- generation through the framework's entry points -----------------------------------------------------
+def generate(mgr_path, reqs, max_batch):
+    """Results of several requests submitted at once, through ModelManager and its Scheduler; each list in `reqs`
+    after the one before it has ended."""
+    import asyncio
+
+    from aios_amd.runtime.model_manager import ModelManager
+
+    mgr = ModelManager(max_batch=max_batch, max_slots=max_batch)
+    m = asyncio.run(mgr.load_model("movalorn-test", mgr_path))
+    assert m.status == "ready", m.error
+    try:
+        out = []
+        for batch in reqs:
+            batch = batch(out) if callable(batch) else batch
+            res, ev = {}, threading.Event()
+
+            def done(i):
+                def f(r):
+                    res[i] = r
+                    if len(res) == len(batch):
+                        ev.set()
+                return f
+
+            for i, r in enumerate(batch):
+                r.on_done = done(i)
+            with m.scheduler.cv:
+                m.scheduler.queue.extend(batch)
+                m.scheduler.cv.notify()
+            assert ev.wait(100)
+            out.append([res[i] for i in range(len(batch))])
+        return out
+    finally:
+        asyncio.run(mgr.unload_model("movalorn-test"))
+
+
+@pytest.mark.parametrize("opts", ["#compute=float32", "#compute=float32&kv_tokens=256", ""])
+def test_greedy_generation_through_the_scheduler(opts, tmp_models, monkeypatch):
+    """Unequal prompts, some of which stop early (the others' queued step is dropped and run again); then a follow-up
+    that goes on where the first one's state stands."""
+    from aios_amd.runtime.scheduler import GenRequest
+
+    monkeypatch.setenv("AIOS_PREFILL_CHUNK", "48")
+    path, cfg, w = model("mixed", tmp_models)
+    prompts = [ids_of(cfg, n, 90 + n) for n in (3, 130, 50, 64, 20)]
+    n = 12
+    full = [O.greedy(cfg, w, p, n) for p in prompts]
+    stop = [full[i][5] if i in (1, 3) else None for i in range(5)]
+    reqs = [GenRequest(prompt_ids=p, max_tokens=n, stop_ids=[s] if s is not None else None) for p, s in zip(prompts, stop)]
+
+    def follow(out):
+        ids = prompts[0] + out[0][0].token_ids[:-1]
+        return [GenRequest(prompt_ids=ids + [7, 8], max_tokens=4)]
+
+    first, second = generate(path + opts, [reqs, follow], 4)
+    for p, r, s, f in zip(prompts, first, stop, full):
+        if opts:  # 32-bit: the oracle's own choice at every step
+            assert r.token_ids == (f if s is None else f[:f.index(s)])
+        else:     # bf16: a choice within rounding of the oracle's best, most of the time
+            lg = O.forward(cfg, w, p + r.token_ids)[len(p) - 1:-1]
+            if len(r.token_ids):
+                gap = lg.max(-1).values - lg.gather(1, torch.tensor(r.token_ids)[:, None])[:, 0]
+                assert float((gap / lg.std(-1)).median()) < 0.1
+    ids = prompts[0] + first[0].token_ids[:-1] + [7, 8]
+    if opts:
+        assert second[0].token_ids == O.greedy(cfg, w, ids, 4)
+    assert len(second[0].token_ids) == 4
+
+
+def test_synthetic_preset_decodes_and_matches_its_steps():
+    """Random-init preset: the captured decode loop's history equals single steps' argmax."""
+    from aios_amd.models.config import get_preset
+    from aios_amd.runtime.loader import random_engine
+
+    cfg = get_preset("test-movalorn")
+    eng = random_engine(cfg, seed=3, max_ctx=256, max_slots=2, max_batch=2, compute="float32")
+    ids = [int(t) for t in np.random.default_rng(0).integers(0, cfg.vocab_size, 30)]
+    first = int(np.asarray(eng.prefill(0, ids, 0, True)).argmax())
+    eng.decode_loop_prepare([0], [first], [30])
+    eng.decode_loop_run(1, 40, True)
+    hist = eng.decode_loop_history(1, 31, 40)
+    lg = eng.step([1], [0], [30 + 40], ids + [first] + hist[:39], list(range(29, 70)))
+    gap = lg.max(-1) - lg[np.arange(41), [first] + hist]
+    assert float((gap / lg.std(-1)).max()) < 1e-3
