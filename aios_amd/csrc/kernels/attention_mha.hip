@@ -49,6 +49,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
   const int tql = qvalid ? tq : a.T - 1;
   const int qpos = a.start + tql;
   const int qlow = a.window ? max(0, qpos - a.window + 1) : 0;  // first visible key
+  const uint32_t qspan = (uint32_t)(qpos - qlow);
   gbf16x8 qf[KS];
   const float sc = a.scale * 1.4426950408889634f;
   {
@@ -143,13 +144,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
     }
     const int kbase = kt * MH_KT;
     const bool full = kbase + MH_KT - 1 <= qpos && kbase >= qlow;
+    const int krel = kbase + 4 * half - qlow;
     float mx = -INFINITY;
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
-        const int key = kbase + t * 32 + (r & 3) + 8 * (r >> 2) + 4 * half;
-        if (!full && (key > qpos || key < qlow)) st[t][r] = -INFINITY;
+        // (visible: 0 <= key - qlow <= qpos - qlow, one unsigned comparison)
+        if (!full && (uint32_t)(krel + t * 32 + (r & 3) + 8 * (r >> 2)) > qspan) st[t][r] = -INFINITY;
         mx = fmaxf(mx, st[t][r]);
       }
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));

@@ -5,8 +5,8 @@
 //                             cycles) instead of waiting for a launch that does it; the second sums a token's
 //                             experts, and the shared one, into one row.
 //   more                      routing and a counting sort of the pairs by expert, then two grouped products
-//                             over tiles of one expert's rows: 16-row tiles streamed by waves while
-//                             experts have few rows, 128 x 128 tiles through LDS beyond.
+//                             over tiles of one expert's rows: weights streamed by waves while
+//                             experts have few rows (up to 64), 128 x 128 tiles through LDS beyond.
 // Router scores, their softmax and the weighted sums are fp32.  A row's result does not depend on its place in
 // a tile, so the order inside an expert is free.
 #include <algorithm>
@@ -17,6 +17,10 @@
 #include "gemm_common.h"
 
 namespace aios {
+
+__device__ __forceinline__ float lane_value(float v, int lane) {
+  return __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(v), lane));
+}
 
 // ---- routing: one wave per token ------------------------------------------------------------------
 // lane l holds experts l, l + 64, ..; NE >= experts / 64.  Lane k < top leaves with the k-th choice and its weight
@@ -77,8 +81,37 @@ __device__ __forceinline__ void moe_route_token(const MoeArgs& a, int t, int& my
       if (lane + 64 * i == bi) ch[i] = -INFINITY;
   }
 }
+// up to 64 experts, one a lane: an expert's place is the number of choices above its own, counted from scalar
+// copies of them (no chain of lane exchanges)
+__device__ __forceinline__ void moe_route_rank(const MoeArgs& a, int t, int& my_e, float& my_w) {
+  const int lane = threadIdx.x & 63;
+  const bool on = lane < a.experts;
+  const float z = on ? a.logits[(size_t)t * a.ldl + lane] : -INFINITY;
+  const float corr = on && a.corr ? a.corr[lane] : 0.f;
+  float mx = -INFINITY;
+  for (int e = 0; e < a.experts; ++e) mx = fmaxf(mx, lane_value(z, e));
+  const float p = expf(z - mx);
+  float sum = 0.f;
+  for (int e = 0; e < a.experts; ++e) sum += lane_value(p, e);
+  const float s = p / sum, ch = on ? s + corr : -INFINITY;
+  int place = on ? 0 : 64;
+  for (int e = 0; e < a.experts; ++e) {
+    const float c = lane_value(ch, e);
+    place += c > ch || (c == ch && e < lane);
+  }
+  my_e = 0;
+  my_w = 0.f;
+  for (int k = 0; k < a.top; ++k) {
+    const int e = __ffsll(__ballot(place == k)) - 1;
+    const float w = lane_value(s, e) * a.scale;
+    if (lane == k) {
+      my_e = e;
+      my_w = w;
+    }
+  }
+}
 __device__ __forceinline__ void moe_route(const MoeArgs& a, int t, int& e, float& w) {
-  if (a.experts <= 64) moe_route_token<1>(a, t, e, w);
+  if (a.experts <= 64) moe_route_rank(a, t, e, w);
   else if (a.experts <= 256) moe_route_token<4>(a, t, e, w);
   else moe_route_token<MOE_MAX_EXPERTS / 64>(a, t, e, w);
 }
@@ -167,13 +200,20 @@ __device__ __forceinline__ bool moe_place(const MoeArgs& a, int w, int nb, int4&
 // ---- few tokens -------------------------------------------------------------------------------------
 __device__ __forceinline__ gbf16x8 ldfrag(const bf16_t* p) { return __builtin_bit_cast(gbf16x8, *(const gu32x4*)p); }
 
-constexpr int MF_B = 8, MF_D = 4;  // 64-column items (two MFMA steps) in flight per wave: up, down
+constexpr int MF_B = 8;  // 64-column items (two MFMA steps) in flight per wave
+
+// n bf16 numbers (a multiple of 8) into LDS
+__device__ __forceinline__ void moe_stage(bf16_t* dst, const bf16_t* src, int n) {
+  for (int i = 8 * threadIdx.x; i < n; i += 8 * blockDim.x) *(gu32x4*)(dst + i) = *(const gu32x4*)(src + i);
+}
 
 // gate / up of every (token, expert) pair: 16 interleaved columns per workgroup, the width over its 4 waves
 __global__ void __launch_bounds__(256) moe_few_up_kernel(MoeArgs a) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t mf_smem[];  // the token's input [dp]
   __shared__ float red[4][16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
   const int t = blockIdx.y / a.top, k = blockIdx.y - t * a.top;
+  moe_stage(mf_smem, (const bf16_t*)a.h + (size_t)t * a.ldh, a.dp);
   int e;
   float w;
   moe_route(a, t, e, w);
@@ -184,25 +224,27 @@ __global__ void __launch_bounds__(256) moe_few_up_kernel(MoeArgs a) {
   e = __builtin_amdgcn_readlane(e, k);
   const int items = a.dp >> 6;
   const bf16_t* wp = a.wgu + ((size_t)e * 2 * a.ff + blockIdx.x * 16 + r16) * a.dp + 8 * q;
-  const bf16_t* hp = (const bf16_t*)a.h + (size_t)t * a.ldh + 8 * q;
+  const bf16_t* hp = mf_smem + 8 * q;
   gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
   for (int i0 = wave; i0 < items; i0 += 4 * MF_B) {
-    gbf16x8 wf[2 * MF_B], hf[2 * MF_B];
+    gbf16x8 wf[2 * MF_B];
 #pragma unroll
     for (int i = 0; i < MF_B; ++i) {
       const int c = 64 * min(i0 + 4 * i, items - 1);
       wf[2 * i] = ldfrag(wp + c);
       wf[2 * i + 1] = ldfrag(wp + c + 32);
-      hf[2 * i] = ldfrag(hp + c);
-      hf[2 * i + 1] = ldfrag(hp + c + 32);
     }
+    __builtin_amdgcn_sched_barrier(0);
+    if (i0 == wave) __syncthreads();  // (every wave has at least one item: the input is staged)
 #pragma unroll
     for (int i = 0; i < MF_B; ++i)
       if (i0 + 4 * i < items) {
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i], hf[2 * i], acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i + 1], hf[2 * i + 1], acc, 0, 0, 0);
+        const int c = 64 * (i0 + 4 * i);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i], ldfrag(hp + c), acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i + 1], ldfrag(hp + c + 32), acc, 0, 0, 0);
       }
   }
+  if (wave >= items) __syncthreads();
   // every lane of a quarter holds the same token: columns 4 q + j
   if (r16 == 0) *(gf32x4*)&red[wave][4 * q] = acc;
   __syncthreads();
@@ -217,63 +259,67 @@ __global__ void __launch_bounds__(256) moe_few_up_kernel(MoeArgs a) {
   }
 }
 
-// down of a token's experts and the shared one, weighted and summed: 16 columns per workgroup, the (expert,
-// 64-column) items over its 16 waves
+// down of a token's experts and the shared one, weighted and summed: 8 columns per workgroup, two waves each.  A
+// wave takes every other item of its column: 512 numbers of one expert's row, 8 a lane
+constexpr int MD_B = 8;  // items in flight per wave
+
+__device__ __forceinline__ float moe_dot8(gu32x4 w, gu32x4 x) {
+  float d = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const uint32_t a = w[j], b = x[j];
+    d = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(gbf16x2, a), __builtin_bit_cast(gbf16x2, b), d, false);
+  }
+  return d;
+}
+
 __global__ void __launch_bounds__(1024) moe_few_down_kernel(MoeArgs a) {
-  __shared__ float red[16][16];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
-  const int t = blockIdx.y, row = blockIdx.x * 16 + r16;
-  const int per = a.ff >> 6, routed = a.top * per, items = routed + (a.sh_dn ? a.sh_ff >> 6 : 0);
+  extern __shared__ __attribute__((aligned(16))) bf16_t mf_smem[];  // activations [top][ff] | shared [sh_ff]
+  __shared__ float red[16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int t = blockIdx.y, row = blockIdx.x * 8 + (wave >> 1);
+  const int per = (a.ff + 511) >> 9, routed = a.top * per, items = routed + (a.sh_dn ? (a.sh_ff + 511) >> 9 : 0);
   int my_e = 0;
   float my_w = 0.f;
   if (lane < a.top) {
     my_e = a.sel[t * a.top + lane];
     my_w = a.wt[t * a.top + lane];
   }
-  gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int i0 = wave; i0 < items; i0 += 16 * MF_D) {
-    gbf16x8 wf[2 * MF_D], hf[2 * MF_D];
-    float wt[MF_D];
+  moe_stage(mf_smem, (const bf16_t*)a.act_out + (size_t)t * a.top * a.ff, a.top * a.ff);
+  if (a.sh_dn) moe_stage(mf_smem + a.top * a.ff, a.sh_act + (size_t)t * a.ld_sh, a.sh_ff);
+  float acc = 0.f;
+  for (int i0 = wave & 1; i0 < items; i0 += 2 * MD_B) {
+    gu32x4 wv[MD_B];
+    float wt[MD_B];
+    int at[MD_B];  // this lane's place in the staged activations
 #pragma unroll
-    for (int i = 0; i < MF_D; ++i) {
-      const int it = __builtin_amdgcn_readfirstlane(min(i0 + 16 * i, items - 1));
-      const bf16_t *wp, *hp;
-      if (it < routed) {
-        const int k = it / per, c = 64 * (it - k * per);
-        const int e = __builtin_amdgcn_readlane(my_e, k);
-        wt[i] = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(my_w), k));
-        wp = a.wdn + ((size_t)e * a.dp + row) * a.ff + c;
-        hp = (const bf16_t*)a.act_out + ((size_t)t * a.top + k) * a.ff + c;
-      } else {
-        const int c = 64 * (it - routed);
-        wt[i] = 1.f;
-        wp = a.sh_dn + (size_t)row * a.sh_ff + c;
-        hp = a.sh_act + (size_t)t * a.ld_sh + c;
-      }
-      wf[2 * i] = ldfrag(wp + 8 * q);
-      wf[2 * i + 1] = ldfrag(wp + 8 * q + 32);
-      hf[2 * i] = ldfrag(hp + 8 * q);
-      hf[2 * i + 1] = ldfrag(hp + 8 * q + 32);
+    for (int i = 0; i < MD_B; ++i) {
+      const int it = i0 + 2 * i, in = min(it, items - 1);
+      const bool sh = in >= routed;
+      const int k = sh ? a.top : in / per, c = 512 * (in - k * per) + 8 * lane, n = sh ? a.sh_ff : a.ff;
+      const int cc = min(c, n - 8);  // (past the end, as past the last item: weight 0)
+      wt[i] = it < items && c < n ? (sh ? 1.f : lane_value(my_w, sh ? 0 : k)) : 0.f;
+      const int e = __builtin_amdgcn_readlane(my_e, sh ? 0 : k);
+      const bf16_t* base = sh ? a.sh_dn + (size_t)row * a.sh_ff : a.wdn + ((size_t)e * a.dp + row) * a.ff;
+      wv[i] = *(const gu32x4*)(base + cc);
+      at[i] = k * a.ff + cc;
     }
+    __builtin_amdgcn_sched_barrier(0);
+    if (i0 == (wave & 1)) __syncthreads();
 #pragma unroll
-    for (int i = 0; i < MF_D; ++i)
-      if (i0 + 16 * i < items) {
-        gf32x4 p = {0.f, 0.f, 0.f, 0.f};
-        p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i], hf[2 * i], p, 0, 0, 0);
-        p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i + 1], hf[2 * i + 1], p, 0, 0, 0);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) acc[j] = fmaf(wt[i], p[j], acc[j]);
-      }
+    for (int i = 0; i < MD_B; ++i) acc = fmaf(wt[i], moe_dot8(wv[i], *(const gu32x4*)(mf_smem + at[i])), acc);
   }
-  if (r16 == 0) *(gf32x4*)&red[wave][4 * q] = acc;
+  if ((wave & 1) >= items) __syncthreads();
+  acc = wave_sum(acc);
+  if (lane == 0) red[wave] = acc;
   __syncthreads();
-  if (threadIdx.x < 16) {
-    float s = 0.f;
-#pragma unroll
-    for (int v = 0; v < 16; ++v) s += red[v][threadIdx.x];
-    a.y[(size_t)t * a.dp + blockIdx.x * 16 + threadIdx.x] = s;
-  }
+  if (tid < 8) a.y[(size_t)t * a.dp + blockIdx.x * 8 + tid] = red[2 * tid] + red[2 * tid + 1];
 }
+
+static size_t moe_few_lds(const MoeArgs& a) {
+  return (size_t)2 * std::max(a.dp, a.top * a.ff + (a.sh_dn ? a.sh_ff : 0));
+}
+bool moe_few_fits(const MoeArgs& a) { return !a.f32 && a.n <= MOE_FEW && moe_few_lds(a) <= 128 * 1024; }
 
 static void moe_check(const MoeArgs& a) {
   if (a.experts < 1 || a.experts > MOE_MAX_EXPERTS || a.top < 1 || a.top > std::min(a.experts, MOE_MAX_TOP))
@@ -284,10 +330,10 @@ static void moe_check(const MoeArgs& a) {
 
 void launch_moe_few(const MoeArgs& a, hipStream_t st) {
   moe_check(a);
-  if (a.f32 || a.n > MOE_FEW) throw std::runtime_error("moe: not a few-token call");
+  if (!moe_few_fits(a)) throw std::runtime_error("moe: not a few-token call");
   if (a.n < 1) return;
-  hipLaunchKernelGGL(moe_few_up_kernel, dim3(2 * a.ff / 16, a.n * a.top), dim3(256), 0, st, a);
-  hipLaunchKernelGGL(moe_few_down_kernel, dim3(a.dp / 16, a.n), dim3(1024), 0, st, a);
+  hipLaunchKernelGGL(moe_few_up_kernel, dim3(2 * a.ff / 16, a.n * a.top), dim3(256), (size_t)2 * a.dp, st, a);
+  hipLaunchKernelGGL(moe_few_down_kernel, dim3(a.dp / 8, a.n), dim3(1024), moe_few_lds(a), st, a);
 }
 
 // ---- grouped, 16-row tiles ------------------------------------------------------------------------------
@@ -295,20 +341,32 @@ void launch_moe_few(const MoeArgs& a, hipStream_t st) {
 // 16-column block's K (4: 16 columns per workgroup; 1: 64)
 constexpr int MG_B = 4;  // 64-column items in flight per wave
 
+template <bool UP>
+__device__ __forceinline__ const bf16_t* moe_row(const MoeArgs& a, int r) {
+  return UP ? (const bf16_t*)a.h + (size_t)a.token[r] * a.ldh : (const bf16_t*)a.act_out + (size_t)r * a.ff;
+}
+// columns col .. col + 3 of row `row`
+template <bool UP>
+__device__ __forceinline__ void moe_store(const MoeArgs& a, size_t row, int col, gf32x4 v) {
+  if constexpr (UP)
+    *(uint32_t*)((bf16_t*)a.act_out + row * a.ff + col / 2) = pk_bf16(glu_act(v[0], a.act) * v[1], glu_act(v[2], a.act) * v[3]);
+  else
+    *(uint2*)((bf16_t*)a.ye + row * a.dp + col) = make_uint2(pk_bf16(v[0], v[1]), pk_bf16(v[2], v[3]));
+}
+
 template <bool UP, int KW>
 __global__ void __launch_bounds__(256) moe_tile16_kernel(MoeArgs a) {
-  __shared__ float red[KW == 4 ? 4 : 1][16][17];
   constexpr int NB = KW == 4 ? 16 : 64;
+  __shared__ float red[KW == 4 ? 4 : 1][16][17];
   const int N = UP ? 2 * a.ff : a.dp, K = UP ? a.dp : a.ff;
   int4 tile;
   int cb;
   if (!moe_place(a, blockIdx.x, N / NB, tile, cb)) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
   const int col = cb * NB + (KW == 4 ? 0 : wave * 16);
-  const int m = tile.y + min(r16, tile.z - 1);  // (rows past the tile repeat its last and are not stored)
-  const bf16_t* hp = UP ? (const bf16_t*)a.h + (size_t)a.token[m] * a.ldh : (const bf16_t*)a.act_out + (size_t)m * a.ff;
+  // (rows past the tile repeat its last and are not stored)
+  const bf16_t* hp = moe_row<UP>(a, tile.y + min(r16, tile.z - 1)) + 8 * q;
   const bf16_t* wp = (UP ? a.wgu : a.wdn) + ((size_t)tile.x * N + col + r16) * K + 8 * q;
-  hp += 8 * q;
   const int items = K >> 6;
   gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
   for (int i0 = KW == 4 ? wave : 0; i0 < items; i0 += KW * MG_B) {
@@ -321,6 +379,7 @@ __global__ void __launch_bounds__(256) moe_tile16_kernel(MoeArgs a) {
       hf[2 * i] = ldfrag(hp + c);
       hf[2 * i + 1] = ldfrag(hp + c + 32);
     }
+    __builtin_amdgcn_sched_barrier(0);  // (all of them in flight before the first is used)
 #pragma unroll
     for (int i = 0; i < MG_B; ++i)
       if (i0 + KW * i < items) {
@@ -338,13 +397,87 @@ __global__ void __launch_bounds__(256) moe_tile16_kernel(MoeArgs a) {
     for (int j = 0; j < 4; ++j)
       acc[j] = (red[0][r16][4 * q + j] + red[1][r16][4 * q + j]) + (red[2][r16][4 * q + j] + red[3][r16][4 * q + j]);
   }
-  if (r16 >= tile.z) return;
-  const size_t row = tile.y + r16;
-  if constexpr (UP)
-    *(uint32_t*)((bf16_t*)a.act_out + row * a.ff + (col + 4 * q) / 2) =
-        pk_bf16(glu_act(acc[0], a.act) * acc[1], glu_act(acc[2], a.act) * acc[3]);
-  else
-    *(uint2*)((bf16_t*)a.ye + row * a.dp + col + 4 * q) = make_uint2(pk_bf16(acc[0], acc[1]), pk_bf16(acc[2], acc[3]));
+  if (r16 < tile.z) moe_store<UP>(a, tile.y + r16, col + 4 * q, acc);
+}
+
+// ---- grouped, tiles of 16 MT rows ---------------------------------------------------------------------------
+// Weights are still what these read, but a fragment of them now serves MT row fragments: the rows go through LDS in
+// 256-column slices (two buffers, one barrier a slice), the weights straight to registers one slice ahead.  64
+// columns per workgroup, 16 a wave.
+constexpr int MS_K = 256, MS_LD = MS_K + 16;
+
+template <bool UP, int MT>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) moe_tile_rows_kernel(MoeArgs a) {
+  constexpr int ROWS = 16 * MT, RP = ROWS * MS_K / 8 / 256;  // 16-byte row pieces per thread and slice
+  __shared__ __attribute__((aligned(16))) bf16_t sm[2][ROWS * MS_LD];
+  const int N = UP ? 2 * a.ff : a.dp, K = UP ? a.dp : a.ff;
+  const int per_xcd = gridDim.x >> 3;  // (neighbours in work order on one XCD)
+  int4 tile;
+  int cb;
+  if (!moe_place(a, (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3), N / 64, tile, cb)) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, q = lane >> 4;
+  const int col = cb * 64 + wave * 16;
+  const bf16_t* wp = (UP ? a.wgu : a.wdn) + ((size_t)tile.x * N + col + r16) * K + 8 * q;
+  const int pr = tid >> 5, pc = 8 * (tid & 31);  // this thread's first row (then every 8th) and column in a slice
+  const bf16_t* hp[RP];
+  static_for<RP>([&](auto I) {
+    constexpr int i = decltype(I)::value;
+    hp[i] = moe_row<UP>(a, tile.y + min(pr + 8 * i, tile.z - 1));
+  });
+  gu32x4 rh[RP];
+  auto load_rows = [&](int k0) {
+    const int c = min(k0 + pc, K - 8);  // (K is a multiple of 64: columns past it are not multiplied)
+    static_for<RP>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      rh[i] = *(const gu32x4*)(hp[i] + c);
+    });
+  };
+  auto stage = [&](int b) {
+    static_for<RP>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      *(gu32x4*)(&sm[b][(pr + 8 * i) * MS_LD + pc]) = rh[i];
+    });
+  };
+  gbf16x8 wa[8], wb[8];
+  auto load_w = [&](gbf16x8(&w)[8], int k0) {
+    static_for<8>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      w[i] = ldfrag(wp + min(k0 + 32 * i, K - 32));
+    });
+  };
+  gf32x4 acc[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) acc[m] = gf32x4{0.f, 0.f, 0.f, 0.f};
+  const int slices = (K + MS_K - 1) / MS_K;
+  load_w(wa, 0);
+  load_rows(0);
+  stage(0);
+  __syncthreads();
+  auto step = [&](int s, gbf16x8(&w)[8], gbf16x8(&next)[8]) {
+    if (s + 1 < slices) {
+      load_w(next, (s + 1) * MS_K);
+      load_rows((s + 1) * MS_K);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+    const bf16_t* x = &sm[s & 1][r16 * MS_LD + 8 * q];
+    static_for<8>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      if (s * MS_K + 32 * i < K) {
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+          acc[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[i], ldfrag(x + 16 * m * MS_LD + 32 * i), acc[m], 0, 0, 0);
+      }
+    });
+    if (s + 1 < slices) stage((s + 1) & 1);
+    __syncthreads();
+  };
+  for (int s = 0; s < slices; s += 2) {
+    step(s, wa, wb);
+    if (s + 1 < slices) step(s + 1, wb, wa);
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+    if (16 * m + r16 < tile.z) moe_store<UP>(a, tile.y + 16 * m + r16, col + 4 * q, acc[m]);
 }
 
 // ---- grouped, 128 x 128 tiles -----------------------------------------------------------------------------
@@ -368,7 +501,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int r = (tid >> 3) + 32 * i, m = tile.y + min(r, tile.z - 1);
-    hp[i] = (UP ? (const bf16_t*)a.h + (size_t)a.token[m] * a.ldh : (const bf16_t*)a.act_out + (size_t)m * a.ff) + 8 * (tid & 7);
+    hp[i] = moe_row<UP>(a, m) + 8 * (tid & 7);
     wp[i] = w0 + (size_t)min(n0 + r, N - 1) * K + 8 * (tid & 7);
   }
   gu32x4 rh[4], rw[4];
@@ -429,24 +562,22 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
       for (int e = 0; e < 16; e += 4) {
         const int c = n0 + wn + 32 * i + 8 * (e >> 2) + 4 * half;
         if (c >= N) continue;
-        const float v0 = acc[i][j][e], v1 = acc[i][j][e + 1], v2 = acc[i][j][e + 2], v3 = acc[i][j][e + 3];
-        if constexpr (UP)
-          *(uint32_t*)((bf16_t*)a.act_out + row * a.ff + c / 2) = pk_bf16(glu_act(v0, a.act) * v1, glu_act(v2, a.act) * v3);
-        else
-          *(uint2*)((bf16_t*)a.ye + row * a.dp + c) = make_uint2(pk_bf16(v0, v1), pk_bf16(v2, v3));
+        moe_store<UP>(a, row, c, gf32x4{acc[i][j][e], acc[i][j][e + 1], acc[i][j][e + 2], acc[i][j][e + 3]});
       }
   }
 }
 
-// average rows per expert from which the 128-row tiles pay
-static int moe_big_rows() {
-  static const int v = [] {
-    const char* e = std::getenv("AIOS_MOE_BIG_ROWS");
-    return e ? std::atoi(e) : 24;
+// rows per tile by the average rows per expert (AIOS_MOE_TILE pins 16, 32, 64 or 128)
+int moe_tile_rows(int n, int top, int experts) {
+  static const int pin = [] {
+    const char* e = std::getenv("AIOS_MOE_TILE");
+    const int v = e ? std::atoi(e) : 0;
+    return v == 16 || v == 32 || v == 64 || v == MB_T ? v : 0;
   }();
-  return v;
+  if (pin) return pin;
+  const double rows = (double)n * top / experts;
+  return rows <= 10 ? 16 : rows <= 24 ? 32 : rows <= 100 ? 64 : MB_T;
 }
-int moe_tile_rows(int n, int top, int experts) { return (double)n * top / experts >= moe_big_rows() ? MB_T : 16; }
 int moe_max_tiles(int n, int top, int experts) {
   const int bm = moe_tile_rows(n, top, experts), p = n * top;
   return std::min(p, experts) + p / bm;
@@ -470,25 +601,30 @@ void launch_moe_grouped(const MoeArgs& a, hipStream_t st) {
     launch_gemm_f32_grouped((const float*)a.act_out, a.ff, nullptr, a.wdn, a.tiles, a.n_tiles, tiles, a.dp, a.ff, (float*)a.ye, st);
     return;
   }
-  auto t16 = [&](auto up, int N) {
+  auto t16 = [&](auto up, auto, int N) {
     constexpr bool UP = decltype(up)::value;
     if (tiles * (N / 64) >= 2 * device_cu_count())
       hipLaunchKernelGGL((moe_tile16_kernel<UP, 1>), dim3(tiles * (N / 64)), dim3(256), 0, st, a);
     else
       hipLaunchKernelGGL((moe_tile16_kernel<UP, 4>), dim3(tiles * (N / 16)), dim3(256), 0, st, a);
   };
-  auto t128 = [&](auto up, int N) {
+  auto trows = [&](auto up, auto mt, int N) {
+    constexpr bool UP = decltype(up)::value;
+    hipLaunchKernelGGL((moe_tile_rows_kernel<UP, decltype(mt)::value>), dim3((tiles * (N / 64) + 7) / 8 * 8), dim3(256), 0, st, a);
+  };
+  auto t128 = [&](auto up, auto, int N) {
     constexpr bool UP = decltype(up)::value;
     const int grid = (tiles * ((N + MB_T - 1) / MB_T) + 7) / 8 * 8;
     hipLaunchKernelGGL((moe_tile128_kernel<UP>), dim3(grid), dim3(256), 0, st, a);
   };
-  if (bm == 16) {
-    t16(std::true_type{}, 2 * a.ff);
-    t16(std::false_type{}, a.dp);
-  } else {
-    t128(std::true_type{}, 2 * a.ff);
-    t128(std::false_type{}, a.dp);
-  }
+  auto both = [&](auto go, auto mt) {
+    go(std::true_type{}, mt, 2 * a.ff);
+    go(std::false_type{}, mt, a.dp);
+  };
+  if (bm == 16) both(t16, 0);
+  else if (bm == 32) both(trows, std::integral_constant<int, 2>{});
+  else if (bm == 64) both(trows, std::integral_constant<int, 4>{});
+  else both(t128, 0);
 }
 
 }  // namespace aios

@@ -23,17 +23,41 @@ __device__ __forceinline__ float sig(float z) {
   return 1.f / (1.f + (F32 ? expf(-z) : __expf(-z)));
 }
 
+// sum over the workgroup: lane exchanges in registers, one LDS round over the waves (red: 16 floats a call)
+__device__ __forceinline__ float row_sum(float v, float* red) {
+  v += __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(v), 0xB1, 0xf, 0xf, true));   // quad_perm [1,0,3,2]
+  v += __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(v), 0x4E, 0xf, 0xf, true));   // quad_perm [2,3,0,1]
+  v += __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(v), 0x141, 0xf, 0xf, true));  // row_half_mirror
+  v += __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(v), 0x140, 0xf, 0xf, true));  // row_mirror
+  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  v = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  v = __uint_as_float(b[0]) + __uint_as_float(b[1]);
+  const int nw = blockDim.x >> 6;
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float t = 0.f;
+  for (int i = 0; i < nw; ++i) t += red[i];
+  return t;
+}
+
 // the next operand of row r from its residual v (NV float4 per thread at columns 4 (tid + i blockDim))
 template <int NV, bool F32>
 __device__ __forceinline__ void next_operand(const NextArgs& nx, int r, int dp, int d, float eps, const float4 (&v)[NV],
                                              float* red) {
   if (nx.kind == NEXT_NONE) return;
   float inv = 1.f;
+  float4 w[NV];  // (requested before the sum it is needed after)
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = 4 * ((int)threadIdx.x + i * (int)blockDim.x);
+    if (nx.kind == NEXT_NORM && c < dp) w[i] = *(const float4*)(nx.g + c);
+  }
   if (nx.kind == NEXT_NORM) {
     float s = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) s += sq4(v[i]);
-    inv = 1.f / sqrtf(block_sum(s, red) / (float)d + eps);
+    inv = 1.f / sqrtf(row_sum(s, red) / (float)d + eps);
   }
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
@@ -41,7 +65,7 @@ __device__ __forceinline__ void next_operand(const NextArgs& nx, int r, int dp, 
     if (c >= dp) break;
     float4 o = v[i];
     if (nx.kind == NEXT_NORM) {
-      const float4 g = *(const float4*)(nx.g + c);
+      const float4 g = w[i];
       o = make_float4(o.x * inv * g.x, o.y * inv * g.y, o.z * inv * g.z, o.w * inv * g.w);
     }
     put4<F32>(nx.out, (size_t)r * nx.ldo + c, o);
@@ -93,14 +117,16 @@ __global__ void embed_rows_kernel(EmbedArgs a) {
 
 template <int NV, bool F32>
 __global__ void row_close_kernel(RowCloseArgs a) {
-  __shared__ float red[16];
+  __shared__ float red[2][16];
   const int r = blockIdx.x;
-  float4 v[NV], x[NV];
+  float4 v[NV], x[NV], p[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = 4 * ((int)threadIdx.x + i * (int)blockDim.x);
     v[i] = x[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    p[i] = make_float4(1.f, 1.f, 1.f, 1.f);
     if (c >= a.dp) continue;
+    if (a.post) p[i] = *(const float4*)(a.post + c);
     const size_t at = (size_t)r * a.dp + c;
     if (a.y) v[i] = *(const float4*)(a.y + at);
     if (!a.replace) x[i] = *(const float4*)(a.x + at);
@@ -141,19 +167,18 @@ __global__ void row_close_kernel(RowCloseArgs a) {
     float s = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) s += sq4(v[i]);
-    inv = 1.f / sqrtf(block_sum(s, red) / (float)a.d + a.eps);
+    inv = 1.f / sqrtf(row_sum(s, red[0]) / (float)a.d + a.eps);
   }
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = 4 * ((int)threadIdx.x + i * (int)blockDim.x);
     if (c >= a.dp) continue;
-    float4 g = make_float4(1.f, 1.f, 1.f, 1.f);
-    if (a.post) g = *(const float4*)(a.post + c);
+    const float4 g = p[i];
     v[i].x = x[i].x + v[i].x * inv * g.x; v[i].y = x[i].y + v[i].y * inv * g.y;
     v[i].z = x[i].z + v[i].z * inv * g.z; v[i].w = x[i].w + v[i].w * inv * g.w;
     *(float4*)(a.x + (size_t)r * a.dp + c) = v[i];
   }
-  next_operand<NV, F32>(a.next, r, a.dp, a.d, a.eps, v, red);
+  next_operand<NV, F32>(a.next, r, a.dp, a.d, a.eps, v, red[1]);
 }
 
 template <bool F32, typename A, typename K1, typename K2, typename K4>

@@ -902,9 +902,9 @@ void LayeredDecoder::feed_forward(int k, const RowSet& r, RowCloseArgs& c) {
     m.tiles = moe_tiles_; m.n_tiles = moe_ntiles_; m.max_tiles = moe_max_tiles_;
     m.act_out = moe_act_; m.ye = moe_ye_; m.gu32 = moe_gu32_;
     m.f32 = f32_;
-    if (!f32_ && n <= MOE_FEW) {
-      if (D.glu) { m.sh_act = cat16_; m.ld_sh = D.glu; m.sh_ff = D.glu; m.sh_dn = w.out2; }
-      m.y = y_;
+    if (D.glu) { m.sh_act = cat16_; m.ld_sh = D.glu; m.sh_ff = D.glu; m.sh_dn = w.out2; }
+    m.y = y_;
+    if (moe_few_fits(m)) {
       c.y = y_;
       return launch_moe_few(m, e_.stream_);
     }

@@ -67,7 +67,7 @@ void launch_row_close(const RowCloseArgs& a, int rows, hipStream_t st);
 // by element in fp32; out_t = S_t * silu(g_t).  Portions are scanned in chunks of SCAN_CHUNK tokens side by
 // side.  The state is kept twice, by parity of the position it was left at: a single token that is run again
 // at the same position reads the same state.
-constexpr int SCAN_CHUNK = 64;
+constexpr int SCAN_CHUNK = 32;
 struct ScanChunk {
   int row0, n;      // rows of the step
   int slot, pos0;   // position of row0
@@ -126,9 +126,10 @@ struct MoeArgs {
   float* y;                   // [n][dp]
 };
 constexpr int MOE_FEW = 4;    // tokens up to which every (token, expert) pair is its own product
+bool moe_few_fits(const MoeArgs& a);                 // launch_moe_few takes these
 int moe_tile_rows(int n, int top, int experts);      // rows per tile the grouped path uses
 int moe_max_tiles(int n, int top, int experts);      // bound of the tile count
 void launch_moe_grouped(const MoeArgs& a, hipStream_t st);  // routing, grouping, experts -> ye
-void launch_moe_few(const MoeArgs& a, hipStream_t st);      // n <= MOE_FEW, bf16: routing, experts, weighted sum -> y
+void launch_moe_few(const MoeArgs& a, hipStream_t st);      // few tokens, bf16: routing, experts, weighted sum -> y
 
 }  // namespace aios
