@@ -6,7 +6,7 @@
 //                             experts, and the shared one, into one row.
 //   more                      routing and a counting sort of the pairs by expert, then two grouped products
 //                             over tiles of one expert's rows: weights streamed by waves while
-//                             experts have few rows (up to 64), 128 x 128 tiles through LDS beyond.
+//                             experts have few rows (up to 32), 128 x 128 tiles through LDS beyond.
 // Router scores, their softmax and the weighted sums are fp32.  A row's result does not depend on its place in
 // a tile, so the order inside an expert is free.
 #include <algorithm>
@@ -535,18 +535,20 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
   for (int s = 0; s < nk; ++s) {
     const int b = s & 1;
     if (s + 1 < nk) load((s + 1) * MB_K);
+    if (wm < tile.z) {  // (else none of this wave's rows exist)
 #pragma unroll
-    for (int k = 0; k < MB_K; k += 16) {
-      gbf16x8 hf[2], wf[2];
+      for (int k = 0; k < MB_K; k += 16) {
+        gbf16x8 hf[2], wf[2];
 #pragma unroll
-      for (int i = 0; i < 2; ++i) {
-        hf[i] = ldfrag(&sm[b][0][(wm + 32 * i + l32) * MB_LD + k + 8 * half]);
-        wf[i] = ldfrag(&sm[b][1][(wn + 32 * i + l32) * MB_LD + k + 8 * half]);
+        for (int i = 0; i < 2; ++i) {
+          hf[i] = ldfrag(&sm[b][0][(wm + 32 * i + l32) * MB_LD + k + 8 * half]);
+          wf[i] = ldfrag(&sm[b][1][(wn + 32 * i + l32) * MB_LD + k + 8 * half]);
+        }
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[i], hf[j], acc[i][j], 0, 0, 0);
       }
-#pragma unroll
-      for (int i = 0; i < 2; ++i)
-#pragma unroll
-        for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[i], hf[j], acc[i][j], 0, 0, 0);
     }
     if (s + 1 < nk) stage(b ^ 1);
     __syncthreads();
@@ -567,16 +569,16 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
   }
 }
 
-// rows per tile by the average rows per expert (AIOS_MOE_TILE pins 16, 32, 64 or 128)
+// rows per tile by the average rows per expert (AIOS_MOE_TILE pins 16, 32 or 128)
 int moe_tile_rows(int n, int top, int experts) {
   static const int pin = [] {
     const char* e = std::getenv("AIOS_MOE_TILE");
     const int v = e ? std::atoi(e) : 0;
-    return v == 16 || v == 32 || v == 64 || v == MB_T ? v : 0;
+    return v == 16 || v == 32 || v == MB_T ? v : 0;
   }();
   if (pin) return pin;
   const double rows = (double)n * top / experts;
-  return rows <= 10 ? 16 : rows <= 24 ? 32 : rows <= 100 ? 64 : MB_T;
+  return rows <= 6.5 ? 16 : rows <= 11 ? 32 : MB_T;
 }
 int moe_max_tiles(int n, int top, int experts) {
   const int bm = moe_tile_rows(n, top, experts), p = n * top;
@@ -623,7 +625,6 @@ void launch_moe_grouped(const MoeArgs& a, hipStream_t st) {
   };
   if (bm == 16) both(t16, 0);
   else if (bm == 32) both(trows, std::integral_constant<int, 2>{});
-  else if (bm == 64) both(trows, std::integral_constant<int, 4>{});
   else both(t128, 0);
 }
 

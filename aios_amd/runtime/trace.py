@@ -76,7 +76,7 @@ def main(argv=None) -> int:
     cfg, _, _ = registry.load_config(args.model)
     native.require("bf16")
     ctx = cfg.max_ctx if cfg.learned_pos else args.max_tokens
-    eng, _, _ = load_engine(args.model, max_ctx=ctx, max_slots=MAX_LIVE, max_batch=64, compute=args.dtype,
+    eng, _, _ = load_engine(args.model, max_ctx=ctx, max_slots=MAX_LIVE, max_batch=MAX_LIVE, compute=args.dtype,
                             kv_pool_tokens=args.max_tokens)
     replay = Replay(eng, MAX_LIVE)
     for line in sys.stdin:
