@@ -482,7 +482,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
 
 // ---- grouped, 128 x 128 tiles -----------------------------------------------------------------------------
 // Four waves of 64 x 64 (2 x 2 MFMA 32 x 32), the weights as the row operand so that a lane holds one token
-// and four consecutive columns.  64-wide K steps in two LDS buffers, the next one's loads in registers.
+// and four consecutive columns.  64-wide K steps in two LDS buffers, the loads of the three steps after the
+// current one in registers.
 constexpr int MB_T = 128, MB_K = 64, MB_LD = MB_K + 8;
 
 template <bool UP>
@@ -504,20 +505,24 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
     hp[i] = moe_row<UP>(a, m) + 8 * (tid & 7);
     wp[i] = w0 + (size_t)min(n0 + r, N - 1) * K + 8 * (tid & 7);
   }
-  gu32x4 rh[4], rw[4];
-  auto load = [&](int k) {
+  struct Regs {
+    gu32x4 h[4], w[4];
+  } rg[3];
+  const int nk = K / MB_K;
+  auto load = [&](Regs& r, int s) {
+    const int k = min(s, nk - 1) * MB_K;  // (the pipeline's tail requests are re-reads)
     static_for<4>([&](auto I) {
       constexpr int i = decltype(I)::value;
-      rh[i] = *(const gu32x4*)(hp[i] + k);
-      rw[i] = *(const gu32x4*)(wp[i] + k);
+      r.h[i] = *(const gu32x4*)(hp[i] + k);
+      r.w[i] = *(const gu32x4*)(wp[i] + k);
     });
   };
-  auto stage = [&](int b) {
+  auto stage = [&](const Regs& r, int b) {
     static_for<4>([&](auto I) {
       constexpr int i = decltype(I)::value;
       const int at = ((tid >> 3) + 32 * i) * MB_LD + 8 * (tid & 7);
-      *(gu32x4*)(&sm[b][0][at]) = rh[i];
-      *(gu32x4*)(&sm[b][1][at]) = rw[i];
+      *(gu32x4*)(&sm[b][0][at]) = r.h[i];
+      *(gu32x4*)(&sm[b][1][at]) = r.w[i];
     });
   };
   const int wm = (wave >> 1) * 64, wn = (wave & 1) * 64;
@@ -528,31 +533,39 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
     for (int j = 0; j < 2; ++j)
 #pragma unroll
       for (int e = 0; e < 16; ++e) acc[i][j][e] = 0.f;
-  load(0);
-  stage(0);
+  load(rg[0], 0);
+  load(rg[1], 1);
+  load(rg[2], 2);
+  stage(rg[0], 0);
   __syncthreads();
-  const int nk = K / MB_K;
-  for (int s = 0; s < nk; ++s) {
-    const int b = s & 1;
-    if (s + 1 < nk) load((s + 1) * MB_K);
+  // (six steps a turn: both the buffers and the register sets are then fixed names, with nothing to copy or wait for
+  // between steps)
+  auto step = [&](auto I, int s0) {
+    constexpr int i = decltype(I)::value, b = i & 1;
+    load(rg[i % 3], s0 + i + 3);
     if (wm < tile.z) {  // (else none of this wave's rows exist)
 #pragma unroll
       for (int k = 0; k < MB_K; k += 16) {
         gbf16x8 hf[2], wf[2];
 #pragma unroll
-        for (int i = 0; i < 2; ++i) {
-          hf[i] = ldfrag(&sm[b][0][(wm + 32 * i + l32) * MB_LD + k + 8 * half]);
-          wf[i] = ldfrag(&sm[b][1][(wn + 32 * i + l32) * MB_LD + k + 8 * half]);
+        for (int j = 0; j < 2; ++j) {
+          hf[j] = ldfrag(&sm[b][0][(wm + 32 * j + l32) * MB_LD + k + 8 * half]);
+          wf[j] = ldfrag(&sm[b][1][(wn + 32 * j + l32) * MB_LD + k + 8 * half]);
         }
 #pragma unroll
-        for (int i = 0; i < 2; ++i)
+        for (int c = 0; c < 2; ++c)
 #pragma unroll
-          for (int j = 0; j < 2; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[i], hf[j], acc[i][j], 0, 0, 0);
+          for (int j = 0; j < 2; ++j) acc[c][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[c], hf[j], acc[c][j], 0, 0, 0);
       }
     }
-    if (s + 1 < nk) stage(b ^ 1);
+    stage(rg[(i + 1) % 3], b ^ 1);  // (past the last step: never read)
     __syncthreads();
-  }
+  };
+  int s0 = 0;
+  for (; s0 + 6 <= nk; s0 += 6) static_for<6>([&](auto I) { step(I, s0); });
+  static_for<5>([&](auto I) {
+    if (s0 + decltype(I)::value < nk) step(I, s0);
+  });
 #pragma unroll
   for (int j = 0; j < 2; ++j) {
     const int r = wm + 32 * j + l32;
