@@ -5,8 +5,8 @@
 //                             cycles) instead of waiting for a launch that does it; the second sums a token's
 //                             experts, and the shared one, into one row.
 //   more                      routing and a counting sort of the pairs by expert, then two grouped products
-//                             over tiles of one expert's rows: weights streamed by waves while
-//                             experts have few rows (up to 32), 128 x 128 tiles through LDS beyond.
+//                             over tiles of one expert's rows: 32 rows with the weights streamed by waves
+//                             while experts have few, 128 x 128 through LDS beyond.
 // Router scores, their softmax and the weighted sums are fp32.  A row's result does not depend on its place in
 // a tile, so the order inside an expert is free.
 #include <algorithm>
@@ -185,11 +185,13 @@ __global__ void __launch_bounds__(1024) moe_group_kernel(MoeArgs a, int bm) {
   }
 }
 
-// workgroup w of a grouped product with nb column blocks -> (tile, column block): an expert's tiles run
-// together over each of its weight columns
-__device__ __forceinline__ bool moe_place(const MoeArgs& a, int w, int nb, int4& tile, int& cb) {
-  const int nt = *a.n_tiles, t = w / nb;
-  if (t >= nt) return false;
+// workgroup of a grouped product with nb column blocks -> (tile, column block): an expert's tiles run together over
+// each of its weight columns, and neighbours in that order on one XCD (workgroups are dealt round-robin over the
+// eight; the grid covers the most tiles there can be, the shares are of those there are)
+__device__ __forceinline__ bool moe_place(const MoeArgs& a, int nb, int4& tile, int& cb) {
+  const int total = *a.n_tiles * nb, per_xcd = (total + 7) >> 3;
+  const int w = (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3), t = w / nb;
+  if ((int)(blockIdx.x >> 3) >= per_xcd || w >= total) return false;
   const int4 x = a.tiles[t];
   const int first = x.w & 0xffff, per = x.w >> 16, local = w - first * nb;
   cb = local / per;
@@ -336,11 +338,8 @@ void launch_moe_few(const MoeArgs& a, hipStream_t st) {
   hipLaunchKernelGGL(moe_few_down_kernel, dim3(a.dp / 8, a.n), dim3(1024), moe_few_lds(a), st, a);
 }
 
-// ---- grouped, 16-row tiles ------------------------------------------------------------------------------
-// UP: rows gathered from h by token, GLU, act_out[row][ff]; else act_out -> ye.  KW: waves that share a
-// 16-column block's K (4: 16 columns per workgroup; 1: 64)
-constexpr int MG_B = 4;  // 64-column items in flight per wave
-
+// ---- grouped products -----------------------------------------------------------------------------------
+// UP: rows gathered from h by token, GLU, act_out[row][ff]; else act_out -> ye
 template <bool UP>
 __device__ __forceinline__ const bf16_t* moe_row(const MoeArgs& a, int r) {
   return UP ? (const bf16_t*)a.h + (size_t)a.token[r] * a.ldh : (const bf16_t*)a.act_out + (size_t)r * a.ff;
@@ -354,67 +353,19 @@ __device__ __forceinline__ void moe_store(const MoeArgs& a, size_t row, int col,
     *(uint2*)((bf16_t*)a.ye + row * a.dp + col) = make_uint2(pk_bf16(v[0], v[1]), pk_bf16(v[2], v[3]));
 }
 
-template <bool UP, int KW>
-__global__ void __launch_bounds__(256) moe_tile16_kernel(MoeArgs a) {
-  constexpr int NB = KW == 4 ? 16 : 64;
-  __shared__ float red[KW == 4 ? 4 : 1][16][17];
+// 32-row tiles, for experts with few rows: the weights are what this reads.  They go straight to registers, one
+// 256-column slice ahead, and every fragment of them serves both row fragments; the rows go through LDS (two
+// buffers, one barrier a slice).  64 columns per workgroup, 16 a wave.
+constexpr int MS_K = 256, MS_LD = MS_K + 16, MS_T = 32;
+
+template <bool UP>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) moe_tile32_kernel(MoeArgs a) {
+  constexpr int MT = MS_T / 16, RP = MS_T * MS_K / 8 / 256;  // row fragments; 16-byte row pieces per thread and slice
+  __shared__ __attribute__((aligned(16))) bf16_t sm[2][MS_T * MS_LD];
   const int N = UP ? 2 * a.ff : a.dp, K = UP ? a.dp : a.ff;
   int4 tile;
   int cb;
-  if (!moe_place(a, blockIdx.x, N / NB, tile, cb)) return;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
-  const int col = cb * NB + (KW == 4 ? 0 : wave * 16);
-  // (rows past the tile repeat its last and are not stored)
-  const bf16_t* hp = moe_row<UP>(a, tile.y + min(r16, tile.z - 1)) + 8 * q;
-  const bf16_t* wp = (UP ? a.wgu : a.wdn) + ((size_t)tile.x * N + col + r16) * K + 8 * q;
-  const int items = K >> 6;
-  gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int i0 = KW == 4 ? wave : 0; i0 < items; i0 += KW * MG_B) {
-    gbf16x8 wf[2 * MG_B], hf[2 * MG_B];
-#pragma unroll
-    for (int i = 0; i < MG_B; ++i) {
-      const int c = 64 * min(i0 + KW * i, items - 1);
-      wf[2 * i] = ldfrag(wp + c);
-      wf[2 * i + 1] = ldfrag(wp + c + 32);
-      hf[2 * i] = ldfrag(hp + c);
-      hf[2 * i + 1] = ldfrag(hp + c + 32);
-    }
-    __builtin_amdgcn_sched_barrier(0);  // (all of them in flight before the first is used)
-#pragma unroll
-    for (int i = 0; i < MG_B; ++i)
-      if (i0 + KW * i < items) {
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i], hf[2 * i], acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[2 * i + 1], hf[2 * i + 1], acc, 0, 0, 0);
-      }
-  }
-  // row r16 of the tile, columns 4 q + j
-  if constexpr (KW == 4) {
-#pragma unroll
-    for (int j = 0; j < 4; ++j) red[wave][r16][4 * q + j] = acc[j];
-    __syncthreads();
-    if (wave != 0) return;
-#pragma unroll
-    for (int j = 0; j < 4; ++j)
-      acc[j] = (red[0][r16][4 * q + j] + red[1][r16][4 * q + j]) + (red[2][r16][4 * q + j] + red[3][r16][4 * q + j]);
-  }
-  if (r16 < tile.z) moe_store<UP>(a, tile.y + r16, col + 4 * q, acc);
-}
-
-// ---- grouped, tiles of 16 MT rows ---------------------------------------------------------------------------
-// Weights are still what these read, but a fragment of them now serves MT row fragments: the rows go through LDS in
-// 256-column slices (two buffers, one barrier a slice), the weights straight to registers one slice ahead.  64
-// columns per workgroup, 16 a wave.
-constexpr int MS_K = 256, MS_LD = MS_K + 16;
-
-template <bool UP, int MT>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) moe_tile_rows_kernel(MoeArgs a) {
-  constexpr int ROWS = 16 * MT, RP = ROWS * MS_K / 8 / 256;  // 16-byte row pieces per thread and slice
-  __shared__ __attribute__((aligned(16))) bf16_t sm[2][ROWS * MS_LD];
-  const int N = UP ? 2 * a.ff : a.dp, K = UP ? a.dp : a.ff;
-  const int per_xcd = gridDim.x >> 3;  // (neighbours in work order on one XCD)
-  int4 tile;
-  int cb;
-  if (!moe_place(a, (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3), N / 64, tile, cb)) return;
+  if (!moe_place(a, N / 64, tile, cb)) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, q = lane >> 4;
   const int col = cb * 64 + wave * 16;
   const bf16_t* wp = (UP ? a.wgu : a.wdn) + ((size_t)tile.x * N + col + r16) * K + 8 * q;
@@ -480,8 +431,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
     if (16 * m + r16 < tile.z) moe_store<UP>(a, tile.y + 16 * m + r16, col + 4 * q, acc[m]);
 }
 
-// ---- grouped, 128 x 128 tiles -----------------------------------------------------------------------------
-// Four waves of 64 x 64 (2 x 2 MFMA 32 x 32), the weights as the row operand so that a lane holds one token
+// 128 x 128 tiles: four waves of 64 x 64 (2 x 2 MFMA 32 x 32), the weights as the row operand so that a lane holds one token
 // and four consecutive columns.  64-wide K steps in two LDS buffers, the loads of the three steps after the
 // current one in registers.
 constexpr int MB_T = 128, MB_K = 64, MB_LD = MB_K + 8;
@@ -490,11 +440,9 @@ template <bool UP>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) moe_tile128_kernel(MoeArgs a) {
   __shared__ __attribute__((aligned(16))) bf16_t sm[2][2][MB_T * MB_LD];
   const int N = UP ? 2 * a.ff : a.dp, K = UP ? a.dp : a.ff, nb = (N + MB_T - 1) / MB_T;
-  // neighbours in work order on one XCD (workgroups are dealt round-robin over the eight)
-  const int per_xcd = gridDim.x >> 3;
   int4 tile;
   int cb;
-  if (!moe_place(a, (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3), nb, tile, cb)) return;
+  if (!moe_place(a, nb, tile, cb)) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l32 = lane & 31, half = lane >> 5;
   const int n0 = cb * MB_T;
   const bf16_t *hp[4], *wp[4];
@@ -582,16 +530,15 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) m
   }
 }
 
-// rows per tile by the average rows per expert (AIOS_MOE_TILE pins 16, 32 or 128)
+// rows per tile by the average rows per expert (AIOS_MOE_TILE pins 32 or 128)
 int moe_tile_rows(int n, int top, int experts) {
   static const int pin = [] {
     const char* e = std::getenv("AIOS_MOE_TILE");
     const int v = e ? std::atoi(e) : 0;
-    return v == 16 || v == 32 || v == MB_T ? v : 0;
+    return v == MS_T || v == MB_T ? v : 0;
   }();
   if (pin) return pin;
-  const double rows = (double)n * top / experts;
-  return rows <= 6.5 ? 16 : rows <= 11 ? 32 : MB_T;
+  return (double)n * top / experts <= 14 ? MS_T : MB_T;
 }
 int moe_max_tiles(int n, int top, int experts) {
   const int bm = moe_tile_rows(n, top, experts), p = n * top;
@@ -616,29 +563,15 @@ void launch_moe_grouped(const MoeArgs& a, hipStream_t st) {
     launch_gemm_f32_grouped((const float*)a.act_out, a.ff, nullptr, a.wdn, a.tiles, a.n_tiles, tiles, a.dp, a.ff, (float*)a.ye, st);
     return;
   }
-  auto t16 = [&](auto up, auto, int N) {
-    constexpr bool UP = decltype(up)::value;
-    if (tiles * (N / 64) >= 2 * device_cu_count())
-      hipLaunchKernelGGL((moe_tile16_kernel<UP, 1>), dim3(tiles * (N / 64)), dim3(256), 0, st, a);
-    else
-      hipLaunchKernelGGL((moe_tile16_kernel<UP, 4>), dim3(tiles * (N / 16)), dim3(256), 0, st, a);
-  };
-  auto trows = [&](auto up, auto mt, int N) {
-    constexpr bool UP = decltype(up)::value;
-    hipLaunchKernelGGL((moe_tile_rows_kernel<UP, decltype(mt)::value>), dim3((tiles * (N / 64) + 7) / 8 * 8), dim3(256), 0, st, a);
-  };
-  auto t128 = [&](auto up, auto, int N) {
-    constexpr bool UP = decltype(up)::value;
-    const int grid = (tiles * ((N + MB_T - 1) / MB_T) + 7) / 8 * 8;
-    hipLaunchKernelGGL((moe_tile128_kernel<UP>), dim3(grid), dim3(256), 0, st, a);
-  };
-  auto both = [&](auto go, auto mt) {
-    go(std::true_type{}, mt, 2 * a.ff);
-    go(std::false_type{}, mt, a.dp);
-  };
-  if (bm == 16) both(t16, 0);
-  else if (bm == 32) both(trows, std::integral_constant<int, 2>{});
-  else both(t128, 0);
+  const int nu = 2 * a.ff, nd = a.dp;
+  auto grid = [&](int blocks) { return dim3((tiles * blocks + 7) / 8 * 8); };
+  if (bm == MS_T) {
+    hipLaunchKernelGGL((moe_tile32_kernel<true>), grid(nu / 64), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((moe_tile32_kernel<false>), grid(nd / 64), dim3(256), 0, st, a);
+  } else {
+    hipLaunchKernelGGL((moe_tile128_kernel<true>), grid((nu + MB_T - 1) / MB_T), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((moe_tile128_kernel<false>), grid((nd + MB_T - 1) / MB_T), dim3(256), 0, st, a);
+  }
 }
 
 }  // namespace aios

@@ -518,7 +518,7 @@ void LayeredDecoder::finalize() {
       pairs = std::max(pairs, P);
       e_act = std::max(e_act, P * D.fp);
       e_gu = std::max(e_gu, P * 2 * D.fp);
-      moe_max_tiles_ = std::max(moe_max_tiles_, s.experts + (int)(P / 16));
+      moe_max_tiles_ = std::max(moe_max_tiles_, s.experts + (int)(P / 32));
     }
     if (s.mixer != MIX_LATENT) continue;
     rp = std::max(rp, D.rp);

@@ -417,7 +417,7 @@ def test_experts_kernels(n, experts, top, ff, d, skew, kind):
     D = dict(h=h, l=lpad, corr=corr, wgu=wgu.bfloat16(), wdn=wdn.bfloat16(), sa=sh_act.bfloat16(),
              sd=torch.nn.functional.pad(sh_dn, (0, 0, 0, dp - d)).bfloat16())
     D = {k: dev(v) for k, v in D.items()}
-    P, tiles = n * top, experts + n * top // 16 + 1
+    P, tiles = n * top, experts + n * top // 32 + 1
     I = lambda *s: torch.full(s, -7, dtype=torch.int32, device="cuda")
     sel, pair, token, tl, nt = I(P), I(P), I(P), I(tiles, 4), I(1)
     wtd, act, ye = torch.zeros(P, device="cuda"), torch.zeros(P, fp, dtype=dt, device="cuda"), torch.zeros(P, dp, dtype=dt, device="cuda")
