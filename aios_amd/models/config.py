@@ -174,7 +174,7 @@ def _movalorn(name: str, vocab: int, width: int, n_layers: int, ff: int, experts
     """Every third layer latent attention, the others minGRU; the first MLP dense, then experts."""
     common = dict(parallel=False, norm_scalar=True, post_norm=True, resid_gate=True, sink=False, out_gate="head")
     dense = dict(ff=ff, act="gelu_tanh")
-    moe = dict(ff=expert_ff, act="silu", experts=experts, top=top, router_scale=1.5, correction=True, shared_ff=expert_ff)
+    moe = dict(ff=expert_ff, act="silu", experts=experts, top=top, router_scale=1.2, correction=True, shared_ff=expert_ff)
     layers = []
     for i in range(n_layers):
         mlp = dense if i == 0 else moe
@@ -186,7 +186,7 @@ def _movalorn(name: str, vocab: int, width: int, n_layers: int, ff: int, experts
     return ModelConfig(name=name, arch="movalorn", vocab_size=vocab, d_model=width, n_layers=n_layers,
                        n_heads=attn["heads"], n_kv_heads=1, head_dim=attn["dim"] + attn["rot_dim"], d_ff=ff, max_ctx=max_ctx,
                        bos_id=-1, eos_id=-1, layers=tuple(layers), learned_pos=False, embed_scale=0.7, logit_scale=0.4,
-                       bigram=(4 * vocab + 1, 31, 17), loop=loop)
+                       bigram=(4 * vocab + 1, 37, 11), loop=loop)
 
 
 PRESETS: Dict[str, ModelConfig] = {
