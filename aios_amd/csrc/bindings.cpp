@@ -145,12 +145,28 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.attr("MLP_NONE") = (int)MLP_NONE;
   m.attr("MLP_GLU") = (int)MLP_GLU;
   m.attr("MLP_MOE") = (int)MLP_MOE;
+  m.attr("MLP_ACT") = (int)MLP_ACT;
+  m.attr("MIX_NONE") = (int)MIX_NONE;
   m.attr("MIX_MINGRU") = (int)MIX_MINGRU;
+  m.attr("MIX_GQA") = (int)MIX_GQA;
+  m.attr("MIX_MAMBA2") = (int)MIX_MAMBA2;
+  m.attr("MIX_GLA") = (int)MIX_GLA;
   m.attr("GATE_NONE") = (int)GATE_NONE;
   m.attr("GATE_ELEMENT") = (int)GATE_ELEMENT;
   m.attr("GATE_HEAD") = (int)GATE_HEAD;
   m.attr("ACT_SILU") = (int)ACT_SILU;
   m.attr("ACT_GELU_TANH") = (int)ACT_GELU_TANH;
+  m.attr("ACT_RELU2") = (int)ACT_RELU2;
+  py::class_<LinSpec>(m, "LinSpec")
+      .def(py::init<>())
+      .def_readwrite("heads", &LinSpec::heads)
+      .def_readwrite("groups", &LinSpec::groups)
+      .def_readwrite("dim", &LinSpec::dim)
+      .def_readwrite("vdim", &LinSpec::vdim)
+      .def_readwrite("conv", &LinSpec::conv)
+      .def_readwrite("norm_groups", &LinSpec::norm_groups)
+      .def_readwrite("rank", &LinSpec::rank)
+      .def_readwrite("tau", &LinSpec::tau);
   py::class_<LayerSpec>(m, "LayerSpec")
       .def(py::init<>())
       .def_readwrite("mixer", &LayerSpec::mixer)
@@ -173,6 +189,15 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       .def_readwrite("rot_base", &LayerSpec::rot_base)
       .def_readwrite("window", &LayerSpec::window)
       .def_readwrite("width", &LayerSpec::width)
+      .def_readwrite("kv_heads", &LayerSpec::kv_heads)
+      .def_readwrite("chunk", &LayerSpec::chunk)
+      .def_readwrite("softcap", &LayerSpec::softcap)
+      .def_readwrite("attn_bias", &LayerSpec::attn_bias)
+      .def_readwrite("lin", &LayerSpec::lin)
+      .def_readwrite("beside", &LayerSpec::beside)
+      .def_readwrite("mixer_scale", &LayerSpec::mixer_scale)
+      .def_readwrite("beside_scale", &LayerSpec::beside_scale)
+      .def_readwrite("mlp_bias", &LayerSpec::mlp_bias)
       .def_readwrite("experts", &LayerSpec::experts)
       .def_readwrite("top", &LayerSpec::top)
       .def_readwrite("shared_ff", &LayerSpec::shared_ff)
@@ -216,6 +241,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       .def_readwrite("loop_start", &EngineConfig::loop_start)
       .def_readwrite("loop_stop", &EngineConfig::loop_stop)
       .def_readwrite("loop_times", &EngineConfig::loop_times)
+      .def_readwrite("loop_add", &EngineConfig::loop_add)
       .def_readwrite("compute_f32", &EngineConfig::compute_f32)
       .def_readwrite("kv_pool_tokens", &EngineConfig::kv_pool_tokens);
 

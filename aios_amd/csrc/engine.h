@@ -58,11 +58,12 @@ struct EngineConfig {
   int max_positions = 0;   // rows of the learned position table (layered models; 0: none)
   // layered models: scale of the token embedding and of the logits; an embedding of (previous, current) token
   // pairs, row (previous * bigram_prev + token * bigram_cur) mod bigram_buckets (0: none); layers
-  // [loop_start, loop_stop) run loop_times times in a row, every pass entered by x = W_in [x; embedding] + step
+  // [loop_start, loop_stop) run loop_times times in a row, every pass entered by x = W_in [x; embedding] + step, or
+  // (loop_add) every pass but the first by x += embedding
   float embed_scale = 1.f, logit_scale = 1.f;
   int bigram_buckets = 0;
   long long bigram_prev = 0, bigram_cur = 0;
-  int loop_start = 0, loop_stop = 0, loop_times = 0;
+  int loop_start = 0, loop_stop = 0, loop_times = 0, loop_add = 0;
   int compute_f32 = 0;     // everything in 32 bits (layered models)
   // tokens the cache pool holds (whole blocks); 0: every slot's full context at once
   int kv_pool_tokens = 0;

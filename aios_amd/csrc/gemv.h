@@ -16,6 +16,7 @@ enum GemvEpilogue : int {
                      //   all-reduce in the row-pair kernel's epilogue, GemvArgs::tp, gemv_q8.h)
   EPI_STORE_GLU = 5,  // rows below glu_row0: y[b][n] = acc; above: interleaved gate/up pairs through the GLU
                       //   to y16[b][(n - glu_row0) / 2] (row stride ldy16) -- the BF16 engine only
+  EPI_ACT16 = 6,      // y16[b][n] = act(acc + bias[n]) (bias or null; row stride ldy16) -- the BF16 engine only
 };
 
 struct ArDevCtx;  // comm.h

@@ -8,6 +8,8 @@
 // O^T += V^T P^T arrangement it shares: a lane holds one query row's scores, and P^T goes from the score
 // accumulators into the value product without leaving registers.  The softmax weights enter that product
 // as two bf16 terms (hi + lo).
+//
+// PG: grouped-query attention over its paged cache -- a 64-key tile is one cache block -- with a soft cap and chunks.
 #include <algorithm>
 
 #include "../latent.h"
@@ -19,7 +21,7 @@ typedef short mv4i16 __attribute__((ext_vector_type(4)));
 
 constexpr int MH_KT = 64;  // keys per tile
 
-template <int DK, int DV>
+template <int DK, int DV, bool PG>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + DV <= 256 ? 2 : 1))) attn_mha_kernel(MhaPrefillArgs a) {
   constexpr int KS = DK / 16, OT = DV / 32;
   constexpr int KROW = DK + 8, VROW = DV + 32;  // (conflict-free row-major and transposed reads)
@@ -48,11 +50,20 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
   const bool qvalid = tq < a.T;
   const int tql = qvalid ? tq : a.T - 1;
   const int qpos = a.start + tql;
-  const int qlow = a.window ? max(0, qpos - a.window + 1) : 0;  // first visible key
+  int qlow = a.window ? max(0, qpos - a.window + 1) : 0;  // first visible key
+  if (PG && a.chunk) qlow = max(qlow, qpos - qpos % a.chunk);
   const uint32_t qspan = (uint32_t)(qpos - qlow);
   gbf16x8 qf[KS];
   const float sc = a.scale * 1.4426950408889634f;
-  {
+  if constexpr (PG) {
+    const bf16_t* qp = a.q16 + ((size_t)tql * a.H + h) * a.dkp + 8 * half;
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+      uint4 u = make_uint4(0, 0, 0, 0);
+      if (16 * s < a.dkp) u = *(const uint4*)(qp + 16 * s);
+      qf[s] = __builtin_bit_cast(gbf16x8, u);
+    }
+  } else {
     const float* qp = a.q + (size_t)tql * a.ldq + h * a.dkp + 8 * half;
 #pragma unroll
     for (int s = 0; s < KS; ++s) {
@@ -88,31 +99,39 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
   float m_run = a.sink ? a.sink[h] * 1.4426950408889634f : -INFINITY;
   float l_run = a.sink ? 1.f : 0.f;
 
+  const float cap = PG ? a.softcap * 1.4426950408889634f : 0.f;
   const int last_pos = a.start + min(a.T, t0 + 128) - 1;  // highest query position of the block
   const int ntiles = last_pos / MH_KT + 1;
-  const int kt0 = a.window ? max(0, a.start + t0 - a.window + 1) / MH_KT : 0;  // tile of the block's first visible key
+  int klow = a.window ? max(0, a.start + t0 - a.window + 1) : 0;  // the block's first visible key
+  if (PG && a.chunk) klow = max(klow, (a.start + t0) / a.chunk * a.chunk);
+  const int kt0 = klow / MH_KT;
   const int last_key = a.start + a.T - 1;
   constexpr int KP = MH_KT * DK / 8 / 256, VP = MH_KT * DV / 8 / 256;  // 16-B pieces per thread
   struct Regs {
     gu32x4 k[KP], v[VP];
   };
-  const bf16_t* kb = a.k + (size_t)h * a.dkp;
-  const bf16_t* vb = a.v + (size_t)h * a.dvp;
+  const int kvh = PG ? h / (a.H / a.G) : h, ldk = PG ? a.dkp : a.ldkv, ldv = PG ? a.dvp : a.ldkv;
+  const size_t belems = PG ? (size_t)a.G * MH_KT * (a.dkp + a.dvp) : 0;
+  const bf16_t* kb = PG ? a.pool + (size_t)kvh * MH_KT * a.dkp : a.k + (size_t)h * a.dkp;
+  const bf16_t* vb = PG ? a.pool + (size_t)a.G * MH_KT * a.dkp + (size_t)kvh * MH_KT * a.dvp : a.v + (size_t)h * a.dvp;
+  int next = PG ? a.bt[min(kt0, ntiles - 1)] : 0;  // block of the tile that is requested next
   auto load = [&](Regs& r, int kt) {
     kt = min(kt, ntiles - 1);  // (the pipeline's tail requests are re-reads)
+    const size_t blk = PG ? (size_t)next * belems : 0;
+    if constexpr (PG) next = a.bt[min(kt + 1, ntiles - 1)];
     static_for<KP>([&](auto I) {
       constexpr int i = decltype(I)::value;
       const int idx = tid + 256 * i, c = idx % (DK / 8);
-      const int key = min(kt * MH_KT + idx / (DK / 8), last_key);
+      const int key = PG ? idx / (DK / 8) : min(kt * MH_KT + idx / (DK / 8), last_key);
       r.k[i] = gu32x4{0, 0, 0, 0};
-      if (c * 8 < a.dkp) r.k[i] = *(const gu32x4*)(kb + (size_t)key * a.ldkv + c * 8);
+      if (c * 8 < a.dkp) r.k[i] = *(const gu32x4*)(kb + blk + (size_t)key * ldk + c * 8);
     });
     static_for<VP>([&](auto I) {
       constexpr int i = decltype(I)::value;
       const int idx = tid + 256 * i, c = idx % (DV / 8);
-      const int key = min(kt * MH_KT + idx / (DV / 8), last_key);
+      const int key = PG ? idx / (DV / 8) : min(kt * MH_KT + idx / (DV / 8), last_key);
       r.v[i] = gu32x4{0, 0, 0, 0};
-      if (c * 8 < a.dvp) r.v[i] = *(const gu32x4*)(vb + (size_t)key * a.ldkv + c * 8);
+      if (c * 8 < a.dvp) r.v[i] = *(const gu32x4*)(vb + blk + (size_t)key * ldv + c * 8);
     });
   };
   auto stage = [&](const Regs& r, bf16_t* buf) {
@@ -150,6 +169,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
+        if (PG && a.softcap > 0.f)  // (the product is the exponent of tanh's exponential)
+          st[t][r] = fmaf(-2.f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(st[t][r]) + 1.f), cap);
         // (visible: 0 <= key - qlow <= qpos - qlow, one unsigned comparison)
         if (!full && (uint32_t)(krel + t * 32 + (r & 3) + 8 * (r >> 2)) > qspan) st[t][r] = -INFINITY;
         mx = fmaxf(mx, st[t][r]);
@@ -217,7 +238,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK + D
     __syncthreads();
   }
   if (!qvalid) return;
-  const float inv = 1.f / l_run;
+  const float inv = (PG ? a.out_scale : 1.f) / l_run;
   bf16_t* op = a.out + (size_t)tq * a.ldo + (size_t)h * a.dvp;
   const float* gp = a.gate ? a.gate + (size_t)tq * a.ldq + (a.head_gate ? h : (size_t)h * a.dvp) : nullptr;
 #pragma unroll
@@ -245,28 +266,35 @@ bool mha_prefill_supports(int dkp, int dvp) {
   return dkp > 0 && dvp > 0 && dkp <= 256 && dvp <= 256 && dkp % 32 == 0 && dvp % 32 == 0;
 }
 
-template <int DK, int DV>
+template <int DK, int DV, bool PG>
 static void mha_go(const MhaPrefillArgs& a, hipStream_t st) {
   constexpr size_t lds = (size_t)2 * MH_KT * ((DK + 8) + (DV + 32)) * sizeof(bf16_t);
   static_assert(lds <= 160 * 1024, "LDS");
-  hipLaunchKernelGGL((attn_mha_kernel<DK, DV>), dim3((a.T + 127) / 128, a.H), dim3(256), lds, st, a);
+  hipLaunchKernelGGL((attn_mha_kernel<DK, DV, PG>), dim3((a.T + 127) / 128, a.H), dim3(256), lds, st, a);
 }
-template <int DK>
+template <int DK, bool PG>
 static void mha_dv(const MhaPrefillArgs& a, hipStream_t st) {
-  if (a.dvp <= 64) mha_go<DK, 64>(a, st);
-  else if (a.dvp <= 128) mha_go<DK, 128>(a, st);
-  else mha_go<DK, 256>(a, st);
+  if (a.dvp <= 64) mha_go<DK, 64, PG>(a, st);
+  else if (a.dvp <= 128) mha_go<DK, 128, PG>(a, st);
+  else mha_go<DK, 256, PG>(a, st);
+}
+template <bool PG>
+static void mha_dk(const MhaPrefillArgs& a, hipStream_t st) {
+  if (a.dkp <= 64) mha_dv<64, PG>(a, st);
+  else if (a.dkp <= 128) mha_dv<128, PG>(a, st);
+  else if (a.dkp <= 192) mha_dv<192, PG>(a, st);
+  else mha_dv<256, PG>(a, st);
 }
 
 void launch_mha_prefill(const MhaPrefillArgs& a, hipStream_t st) {
   if (!mha_prefill_supports(a.dkp, a.dvp)) throw std::runtime_error("mha_prefill: unsupported head dimensions");
   if (a.rot % 2 || a.qrot % 8) throw std::runtime_error("mha_prefill: bad rotated part");
-  if (a.ldkv % 8 || a.ldq % 4 || a.ldo % 4) throw std::runtime_error("mha_prefill: misaligned rows");
+  if (a.pool ? a.H % std::max(1, a.G) || !a.q16 || !a.bt || a.rot || a.ldo % 4 || (a.gate && !a.head_gate)
+             : a.ldkv % 8 || a.ldq % 4 || a.ldo % 4)
+    throw std::runtime_error("mha_prefill: misaligned rows");
   if (a.T < 1) return;
-  if (a.dkp <= 64) mha_dv<64>(a, st);
-  else if (a.dkp <= 128) mha_dv<128>(a, st);
-  else if (a.dkp <= 192) mha_dv<192>(a, st);
-  else mha_dv<256>(a, st);
+  if (a.pool) mha_dk<true>(a, st);
+  else mha_dk<false>(a, st);
 }
 
 }  // namespace aios

@@ -158,7 +158,7 @@ __global__ void __launch_bounds__(BM * BN / 64) gemm_big_kernel(GemmQArgs a) {
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
           if (m < a.M && !(l32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
         } else if constexpr (EPI == GEPI_STORE16) {
-          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
         } else if (m < a.M) {
           float* c = a.C + (size_t)m * a.ldc + n;
           if (S > 1) unsafeAtomicAdd(c, v);

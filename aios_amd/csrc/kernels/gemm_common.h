@@ -20,6 +20,12 @@ __device__ __forceinline__ uint32_t pk_bf16(float a, float b) {
   return __builtin_bit_cast(uint32_t, __builtin_convertvector(v, gbf16x2));
 }
 
+// GEPI_STORE16: what column n's sum becomes
+__device__ __forceinline__ float store16_val(const GemmQArgs& a, int n, float v) {
+  if (a.bias16) v += a.bias16[n];
+  return a.unary ? unary_act(v, a.unary - 1) : v;
+}
+
 // 8 dequantised weights w = sc * q - of (q raw unsigned codes) -> one bf16x8 MFMA fragment
 __device__ __forceinline__ gbf16x8 dq8_frag(const float (&q)[8], float sc, float of) {
   gbf16x8 r;

@@ -394,7 +394,7 @@ __device__ __forceinline__ void pf_body(const GemmQArgs& a, int m0, int n0, int 
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
           if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
         } else if constexpr (EPI == GEPI_STORE16) {
-          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r16 & 1));
         } else if (m < a.M) {
@@ -594,7 +594,7 @@ __device__ __forceinline__ void pf_body32(const GemmQArgs& a, int m0, int n0, in
         const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
         if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
       } else if constexpr (EPI == GEPI_STORE16) {
-        if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+        if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
       } else if (m < a.M) {
         float* cp = a.C + (size_t)m * a.ldc + n;
         if (S > 1) unsafeAtomicAdd(cp, v);
@@ -905,7 +905,7 @@ __device__ __forceinline__ void pf4_body(const GemmQArgs& a, int m0, int n0, int
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
           if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
         } else if constexpr (EPI == GEPI_STORE16) {
-          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r32 & 1));
         } else if (m < a.M) {
@@ -1083,7 +1083,7 @@ __device__ __forceinline__ void pf8_body(const GemmQArgs& a, int m0, int n0, int
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
           if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
         } else if constexpr (EPI == GEPI_STORE16) {
-          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r16 & 1));
         } else if (m < a.M) {
@@ -1372,7 +1372,7 @@ __device__ __forceinline__ void pf8c_body(const GemmQArgs& a, int m0, int n0, in
           const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
           if (m < a.M && !(r16 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
         } else if constexpr (EPI == GEPI_STORE16) {
-          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+          if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
         } else if constexpr (EPI == GEPI_QKV) {
           pf_qkv_out(a, m, n, v, !(r16 & 1));
         } else if (m < a.M) {
@@ -1567,7 +1567,7 @@ __device__ __forceinline__ void pf8d_body(const GemmQArgs& a, int m0, int n0, in
         const float up = __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xF, 0xF, false));
         if (m < a.M && !(r32 & 1)) a.C16[(size_t)m * a.ldc + (n >> 1)] = f32_to_bf16(glu_act(v, a.act) * up);
       } else if constexpr (EPI == GEPI_STORE16) {
-        if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(v);
+        if (m < a.M) a.C16[(size_t)m * a.ldc + n] = f32_to_bf16(store16_val(a, n, v));
       } else if (m < a.M) {
         float* cp = a.C + (size_t)m * a.ldc + n;
         if (S > 1) unsafeAtomicAdd(cp, v);

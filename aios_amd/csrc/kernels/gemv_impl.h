@@ -206,6 +206,11 @@ __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b
       if (grow < a.glu_row0) *(float2*)(a.y + (size_t)b * a.ldy + grow) = make_float2(v0, v1);
       else a.y16[(size_t)b * a.ldy16 + ((grow - a.glu_row0) >> 1)] = f32_to_bf16(glu_act(v0, a.act) * v1);
     } break;
+    case EPI_ACT16: {
+      if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[grow + 1]; }
+      *(uint32_t*)(a.y16 + (size_t)b * a.ldy16 + grow) =
+          (uint32_t)f32_to_bf16(unary_act(v0, a.act)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act)) << 16;
+    } break;
     case EPI_QKV: {
       if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[grow + 1]; }
       const int hd = a.head_dim, qd = a.q_dim, kvd = a.kv_dim;
@@ -585,7 +590,7 @@ void launch_gemv_pair(const GemvArgs& a, hipStream_t st) {
   if constexpr (QT0 == QT_BF16 && QT1 == QT_BF16) {
     if (!a.force_v1 && launch_gemv_lds16(a, st)) return;  // B = 1..4: the BF16 LDS-DMA engine
   }
-  if (a.epi == EPI_STORE_GLU) throw std::runtime_error("gemv: the store + GLU epilogue is the BF16 engine's");
+  if (a.epi == EPI_STORE_GLU || a.epi == EPI_ACT16) throw std::runtime_error("gemv: this epilogue is the BF16 engine's");
   if (a.epi == EPI_TP_RESID)  // only the row-pair int8 kernel does the fused all-reduce epilogue
     throw std::runtime_error("gemv: EPI_TP_RESID launch not taken by the row-pair kernel (use launch_gemv_tp_fused)");
   if (a.x16 || a.y16) throw std::runtime_error("bf16 GEMV input / SwiGLU output: int8-activation kernels only");

@@ -486,6 +486,14 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
       if (grow < a.glu_row0) *(float2*)(a.y + grow) = make_float2(v0, v1);
       else a.y16[(grow - a.glu_row0) >> 1] = f32_to_bf16(glu_act(v0, a.act) * v1);
     } break;
+    case EPI_ACT16: {
+      if (a.bias) {
+        v0 += a.bias[grow];
+        v1 += a.bias[grow + 1];
+      }
+      *(uint32_t*)(a.y16 + grow) =
+          (uint32_t)f32_to_bf16(unary_act(v0, a.act)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act)) << 16;
+    } break;
     case EPI_QKV: {
       if (a.bias) {
         v0 += a.bias[grow];

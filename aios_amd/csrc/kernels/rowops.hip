@@ -111,6 +111,7 @@ __global__ void embed_rows_kernel(EmbedArgs a) {
     }
     *(float4*)(a.x + (size_t)r * a.dp + c) = v[i];
     if (a.keep) put4<F32>(a.keep, (size_t)r * a.ld_keep + c, v[i]);
+    if (a.keep32) *(float4*)(a.keep32 + (size_t)r * a.dp + c) = v[i];
   }
   next_operand<NV, F32>(a.next, r, a.dp, a.d, a.eps, v, red);
 }
@@ -130,6 +131,10 @@ __global__ void row_close_kernel(RowCloseArgs a) {
     const size_t at = (size_t)r * a.dp + c;
     if (a.y) v[i] = *(const float4*)(a.y + at);
     if (!a.replace) x[i] = *(const float4*)(a.x + at);
+    if (a.y_bias) {
+      const float4 b = *(const float4*)(a.y_bias + c);
+      v[i].x += b.x; v[i].y += b.y; v[i].z += b.z; v[i].w += b.w;
+    }
     if (a.ye) {
       for (int k0 = 0; k0 < a.top; k0 += 4) {
         float4 u[4];
@@ -176,6 +181,10 @@ __global__ void row_close_kernel(RowCloseArgs a) {
     const float4 g = p[i];
     v[i].x = x[i].x + v[i].x * inv * g.x; v[i].y = x[i].y + v[i].y * inv * g.y;
     v[i].z = x[i].z + v[i].z * inv * g.z; v[i].w = x[i].w + v[i].w * inv * g.w;
+    if (a.extra) {
+      const float4 b = *(const float4*)(a.extra + (size_t)r * a.dp + c);
+      v[i].x += b.x; v[i].y += b.y; v[i].z += b.z; v[i].w += b.w;
+    }
     *(float4*)(a.x + (size_t)r * a.dp + c) = v[i];
   }
   next_operand<NV, F32>(a.next, r, a.dp, a.d, a.eps, v, red[1]);

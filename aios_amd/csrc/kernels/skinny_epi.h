@@ -33,6 +33,9 @@ __device__ __forceinline__ bool sk_epilogue(const GemmQArgs& a, gf32x4 (&acc)[MT
       const uint32_t pk = pk_bf16(glu_act(v[0], a.act) * v[1], glu_act(v[2], a.act) * v[3]);
       *(uint32_t*)(a.C16 + (size_t)m * a.ldc + (n >> 1)) = pk;
     } else if constexpr (EPI == GEPI_STORE16) {
+      if (a.bias16 || a.unary)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = store16_val(a, n + j, v[j]);
       *(uint2*)(a.C16 + (size_t)m * a.ldc + n) = make_uint2(pk_bf16(v[0], v[1]), pk_bf16(v[2], v[3]));
     } else if constexpr (EPI == GEPI_STORE_GLU) {
       if (n < a.glu_n0)  // (a multiple of 4: the lane's 4 columns are on one side)

@@ -68,8 +68,16 @@ void launch_latent_gather(const bf16_t* pool, const int* bt, int maxb, int kvb, 
 
 // causal flash attention of one sequence's T new tokens at positions [start, start + T) over contiguous
 // per-head keys and values [0, start + T), with a sink and an output gate
+// paged (pool set): keys and values from the blocks of grouped-query attention's cache (mixers.h GqaArgs), whose
+// positions are the sequence's; queries q16 with the score's factor folded in
 struct MhaPrefillArgs {
   const float* q;        // [T][ldq], head h at h * dkp
+  const bf16_t* q16;     // paged: [T][H dkp]
+  const bf16_t* pool;
+  const int* bt;         // paged: block table of the sequence
+  int G;                 // paged: key / value heads
+  int chunk;             // paged: keys before the query's chunk of this many positions are out (0: none)
+  float softcap, out_scale;  // paged
   int ldq;
   const bf16_t *k, *v;   // [S][ldkv]: key of head h at k + h * dkp, value at v + h * dvp
   int ldkv;
@@ -80,7 +88,7 @@ struct MhaPrefillArgs {
   const float2* rope;
   float scale;
   const float* sink;     // [H] or null
-  const float* gate;     // [T][ldq], head h at h * dvp (head_gate: at h): the output times sigmoid(gate); or null
+  const float* gate;     // [T][ldq] (paged: ldq of the gate alone), head h at h * dvp (head_gate: at h): the output times sigmoid(gate); or null
   int head_gate;
   bf16_t* out;           // [T][ldo], head h at h * dvp
   int ldo;

@@ -5,6 +5,7 @@
 // layers' weights and cache pools and enqueues the forward pass of a set of rows.  A row is one token of
 // one slot at one position, so a batch may mix portions of prompts and single decoded tokens.
 #pragma once
+#include <algorithm>
 #include <map>
 #include <set>
 #include <string>
@@ -17,14 +18,24 @@
 
 namespace aios {
 
-enum MixerKind : int { MIX_LATENT = 1, MIX_MINGRU = 2 };
-enum MlpKind : int { MLP_NONE = 0, MLP_GLU = 1, MLP_MOE = 2 };
+enum MixerKind : int { MIX_NONE = 0, MIX_LATENT = 1, MIX_MINGRU = 2, MIX_GQA = 3, MIX_MAMBA2 = 4, MIX_GLA = 5 };
+enum MlpKind : int { MLP_NONE = 0, MLP_GLU = 1, MLP_MOE = 2, MLP_ACT = 3 };
 enum OutGate : int { GATE_NONE = 0, GATE_ELEMENT = 1, GATE_HEAD = 2 };
 
 // One layer: a mixer and a feed-forward.  Parallel: both read the same normalised input and are added to the
 // residual together (x += mixer(norm(x)) + mlp(norm(x))).  Otherwise one after the other, each
 //   x += post( f(h) * sigmoid(Wr h + br) ),  h = norm(x)
 // with the gate (resid_gate) and the norm of the result (post_norm) where the layer has them.
+
+// A linear recurrence (mixers.h LinScanArgs).
+struct LinSpec {
+  int heads = 1, groups = 1;           // groups: MIX_MAMBA2, heads that share B and C
+  int dim = 64, vdim = 64;             // state rows (key channels) and columns per head
+  int conv = 4;                        // MIX_MAMBA2: taps
+  int norm_groups = 1;                 // MIX_MAMBA2: parts of the gated norm
+  int rank = 16;                       // MIX_GLA: width of the decay's first projection
+  double tau = 16.0;                   // MIX_GLA
+};
 struct LayerSpec {
   int mixer = MIX_LATENT;
   int parallel = 1;
@@ -39,11 +50,23 @@ struct LayerSpec {
   float scale = 0.125f;                // of q . k
   int sink = 1;                        // a learned logit per head joins the softmax's denominator
   int out_gate = GATE_ELEMENT;         // head outputs times sigmoid(Wg h): a number each, or one per head
+  // MIX_GQA: heads, dim, vdim, the first rot_dims dimensions turn (in halves), window, scale, sink, out_gate, and
+  int kv_heads = 1;
+  int chunk = 0;                       // keys before a token's chunk of so many positions are out (0: no chunks)
+  float softcap = 0.f;                 // of the scores (0: none)
+  int attn_bias = 0;                   // biases of q, k, v and the output projection
   // MIX_MINGRU
   int width = 64;                      // of the state
+  // MIX_MAMBA2, MIX_GLA
+  LinSpec lin;
+  // a second mixer that reads the same input (MIX_MAMBA2 or MIX_GLA, sizes in lin): mixer_scale * first + beside_scale *
+  // second
+  int beside = MIX_NONE;
+  float mixer_scale = 1.f, beside_scale = 1.f;
   int mlp = MLP_GLU;
-  int ff = 256;                        // MLP_GLU: hidden width; MLP_MOE: of every expert
-  int act = ACT_GELU_TANH;             // GluAct of the gate
+  int ff = 256;                        // MLP_GLU, MLP_ACT: hidden width; MLP_MOE: of every expert
+  int act = ACT_GELU_TANH;             // GluAct of the gate; MLP_ACT: of the hidden layer
+  int mlp_bias = 0;                    // MLP_ACT
   int experts = 0, top = 0;            // MLP_MOE
   int shared_ff = 0;                   // hidden width of the expert that runs for every token (0: none)
   int correction = 0;                  // a learned number per expert joins the choice, not the weights
@@ -92,6 +115,10 @@ class LayeredDecoder {
     // [latent | rotated at roff]; qn / gn: rows of all heads' queries / values (gn: columns the mixer leaves)
     int H, dk, dv, rank, rot, qrot, roff, dkp, dvp, rp, qn, gn;
     int wp;                   // minGRU: padded width
+    int G, koff, voff;        // grouped-query attention: key / value heads, their columns (q at 0)
+    // linear recurrence: kind (0: none), heads, groups, state rows and columns (padded: np, vp), its columns in the
+    // input product and in the joint output matrix
+    int lin, lH, lG, lN, lnp, ldv, lvp, lin_off, lin_out;
     int ff, fp, shf, shp;     // feed-forward and shared expert, padded
     int gate_off, rg_off;     // columns of the output gate and of the residual gate in the input product
     int n1;                   // input product without gate / up
@@ -111,12 +138,18 @@ class LayeredDecoder {
     bf16_t *edn = nullptr;   // [experts][dp][fp]
     bf16_t *ukv = nullptr;   // [qn + gn][rp]: key | value up-projections
     bf16_t *ukT = nullptr;   // [H][rp][dkp]
+    // biases: q, k, v, output projection (times mixer_scale), MLP up and down
+    float *qb = nullptr, *kb = nullptr, *vb = nullptr, *ob = nullptr, *upb = nullptr, *dnb = nullptr;
+    // linear recurrence (mixers.h LinScanArgs)
+    float *conv_w = nullptr, *conv_b = nullptr, *dt_b = nullptr, *a_log = nullptr, *lin_d = nullptr, *lin_norm = nullptr,
+          *a2 = nullptr, *a2_b = nullptr;
   };
   // one pass of one layer; a looped layer has a cache or state per pass
   struct Run {
     int layer, pass;         // pass: -1 outside the loop
-    char* pool;              // cache (latent attention)
-    float* state;            // [2][slots][wp] (minGRU)
+    char* pool;              // cache (attention)
+    float* state;            // [2][slots][state numbers]
+    float* ring;             // [slots][taps][columns]: the convolution's last inputs
   };
   struct RowSet {
     const int *tokens, *pos, *slot, *run;  // run: rows of the sequence from its first row (null: one each)
@@ -125,18 +158,24 @@ class LayeredDecoder {
     std::map<int, std::pair<int, int>> tiles;  // step batches: heads -> (first tile, count)
     int max_len;                          // of the absorbed rows
     std::vector<std::pair<int, Piece>> pf;  // expanded path: first row, piece
-    int n_chunks, split;                  // step batches: chunks of the recurrences
+    int n_chunks, split, n_seqs;          // step batches: chunks of the recurrences, pieces
   };
   void layer16(int k, const RowSet& r);  // k: run
   void layer32(int k, const RowSet& r);
   void layer_seq(int k, const RowSet& r);
   void feed_forward(int k, const RowSet& r, RowCloseArgs& c);
   void recurrence(int k, const RowSet& r);
+  void linear(int k, const RowSet& r);
+  void grouped_attention(int k, const RowSet& r);
+  size_t state_floats(int i) const;      // of one slot and parity
+  size_t ring_floats(int i) const;       // of one slot
+  bool enters_pass(int k) const;         // run k begins a pass but the first, entered by adding the embedding
   void attention(int k, const RowSet& r);
   void run(const RowSet& r);
   NextArgs next_of(int k, bool decode);  // what the residual becomes before run k (the head's input after the last)
   RowCloseArgs close_args() const;
   LatentAttnArgs latent_args(int k, const RowSet& r);
+  int runs_to_do() const { return run_limit_ < 0 ? (int)runs_.size() : std::min(run_limit_, (int)runs_.size()); }
   // y[n][N] (ldy) = operand rows x w^T, through the GEMV, the short or the prefill GEMM
   void project(const void* a, int lda, const bf16_t* w, int n, int N, int K, float* y, int ldy);
   void alloc_layer(int i);
@@ -164,7 +203,7 @@ class LayeredDecoder {
   bool seq_ = false, recurrent_ = false, head_ready_ = false;
   int run_limit_ = -1, max_window_ = 0;  // max_window_: largest window, 0 if a layer has none
   bf16_t *embd_ = nullptr, *posw_ = nullptr, *headw_ = nullptr, *pairw_ = nullptr, *loopw_ = nullptr;
-  float *out_norm_ = nullptr, *loop_step_ = nullptr;
+  float *out_norm_ = nullptr, *loop_step_ = nullptr, *x0_ = nullptr;  // x0_: embedding rows (loops that add them)
   std::vector<float2*> rope_;            // per layer
   int* last_tok_ = nullptr;              // [2][slots]
   std::vector<std::pair<std::string, std::pair<int, int>>> tensors_;  // name, (rows, columns)
@@ -182,6 +221,9 @@ class LayeredDecoder {
   void *xin_ = nullptr, *moe_act_ = nullptr, *moe_ye_ = nullptr;
   int *moe_sel_ = nullptr, *moe_pair_ = nullptr, *moe_token_ = nullptr, *moe_ntiles_ = nullptr;
   int4* moe_tiles_ = nullptr;
+  // linear recurrences: operands of the blocks, outputs before the norm
+  void *lin_qo_ = nullptr, *lin_ko_ = nullptr, *lin_kr_ = nullptr, *lin_vo_ = nullptr, *lin_so_ = nullptr;
+  float *lin_dec_ = nullptr, *lin_y_ = nullptr;
   int moe_max_tiles_ = 0;
   // RMSNorm split across the short GEMMs (GemmQArgs nrm_*): set when the residual in x_ already went
   // through bf16(x * g_next) and per-tile sums
@@ -194,6 +236,7 @@ class LayeredDecoder {
   size_t step_ints_ = 0;
   int *st_tokens_ = nullptr, *st_pos_ = nullptr, *st_slot_ = nullptr, *st_want_ = nullptr, *st_run_ = nullptr;
   ScanChunk* st_chunks_ = nullptr;
+  ScanSeq* st_seqs_ = nullptr;
   int max_chunks_ = 0;
   LatentTile* st_tiles_ = nullptr;
 };

@@ -10,6 +10,8 @@
 // bf16 operand that the row operation before it wrote (mixers.h), so a layer is
 //   input product (+ residual gate rows) | mixer | output product | close | input product (+ residual gate and
 //   router rows, GLU in its epilogue) | experts | down product | close
+// Mixers that read the same input share the input product and the output product: a layer's attention and linear
+// recurrence leave their results side by side in one operand.
 // 32-bit engine: the same steps in fp32, absorbed attention for every row.
 #include "layered.h"
 
@@ -47,7 +49,7 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
   f32_ = c.compute_f32;
   if (d_ < 1 || v_ < 1 || c.max_positions < 0 || c.max_ctx < 1) throw std::runtime_error("layered model: bad sizes");
   if (c.tp_size > 1) throw std::runtime_error("layered models run on one GPU (no tensor parallelism)");
-  if (c.kv_fp8) throw std::runtime_error("layered models: the latent cache has no fp8 form");
+  if (c.kv_fp8) throw std::runtime_error("layered models: the cache has no fp8 form");
   if (c.loop_times > 0 && !(c.loop_start >= 0 && c.loop_start < c.loop_stop && c.loop_stop <= nl_))
     throw std::runtime_error("layered model: bad loop");
   if (c.bigram_buckets < 0) throw std::runtime_error("layered model: bad pair table");
@@ -71,13 +73,16 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
     if (s.mixer != t.mixer || s.heads != t.heads || s.dim != t.dim || s.vdim != t.vdim || s.kv_rank != t.kv_rank ||
         s.rot_dim != t.rot_dim || s.out_gate != t.out_gate || s.sink != t.sink || s.width != t.width || s.mlp != t.mlp ||
         s.post_norm != t.post_norm || s.resid_gate != t.resid_gate || s.norm_scalar != t.norm_scalar ||
+        s.kv_heads != t.kv_heads || s.attn_bias != t.attn_bias || s.beside != t.beside || s.lin.heads != t.lin.heads ||
+        s.lin.groups != t.lin.groups || s.lin.dim != t.lin.dim || s.lin.vdim != t.lin.vdim || s.lin.conv != t.lin.conv ||
+        s.lin.rank != t.lin.rank || s.mixer_scale != t.mixer_scale || s.mlp_bias != t.mlp_bias ||
         (s.mlp != MLP_NONE && (s.ff != t.ff || s.experts != t.experts || s.shared_ff != t.shared_ff || s.correction != t.correction)))
       throw std::runtime_error(at + "sizes differ from the layer whose weights it uses");
     if (s.mlp != MLP_NONE && s.ff < 1) throw std::runtime_error(at + "bad sizes");
     if (s.mlp == MLP_MOE && (s.experts < 1 || s.experts > MOE_MAX_EXPERTS || s.top < 1 || s.top > std::min(s.experts, MOE_MAX_TOP) ||
                              s.shared_ff < 0))
       throw std::runtime_error(at + "bad number of experts");
-    if (s.parallel && (s.mixer != MIX_LATENT || s.mlp == MLP_MOE || s.post_norm || s.resid_gate))
+    if (s.parallel && (s.mixer != MIX_LATENT || s.beside || s.mlp == MLP_MOE || s.mlp == MLP_ACT || s.post_norm || s.resid_gate))
       throw std::runtime_error(at + "a parallel layer is latent attention beside a dense MLP");
     Dims& D = dims_[i];
     std::memset(&D, 0, sizeof(D));
@@ -108,9 +113,55 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
       D.gn = D.wp;
       n = 3 * D.wp;
       recurrent_ = true;
+    } else if (s.mixer == MIX_GQA) {
+      if (s.heads < 1 || s.kv_heads < 1 || s.heads % s.kv_heads || s.dim < 1 || s.vdim < 1 || s.window < 0 || s.chunk < 0 ||
+          s.rot_dims < 0 || s.rot_dims % 2 || s.rot_dims > s.dim || s.out_gate == GATE_ELEMENT)
+        throw std::runtime_error(at + "bad sizes");
+      D.H = s.heads;
+      D.G = s.kv_heads;
+      D.dk = s.dim;
+      D.dv = s.vdim;
+      D.rot = s.rot_dims;
+      D.dkp = up(D.dk, 32);
+      D.dvp = up(D.dv, 32);
+      if (!gqa_supports(D.dkp, D.dvp)) throw std::runtime_error(at + "attention heads above 256 dimensions");
+      D.gn = up(D.H * D.dvp, 64);
+      D.koff = D.H * D.dk;
+      D.voff = D.koff + D.G * D.dk;
+      D.gate_off = D.voff + D.G * D.dv;
+      n = D.gate_off + (s.out_gate == GATE_HEAD ? D.H : 0);
+      const int w = s.window && s.chunk ? std::min(s.window, s.chunk) : s.window + s.chunk;
+      if (w) max_window_ = std::max(max_window_, w);
+      else all_windowed = false;
+    } else if (s.mixer == MIX_MAMBA2 || s.mixer == MIX_GLA) {
+      n = 0;
     } else {
       throw std::runtime_error("unknown mixer kind");
     }
+    const int lin = s.mixer == MIX_MAMBA2 || s.mixer == MIX_GLA ? s.mixer : s.beside;
+    if (s.beside && s.mixer != MIX_GQA) throw std::runtime_error(at + "a second mixer stands beside grouped-query attention only");
+    if (lin) {
+      const LinSpec& l = s.lin;
+      const bool key = lin == MIX_GLA;
+      if (lin != MIX_MAMBA2 && lin != MIX_GLA) throw std::runtime_error(at + "unknown second mixer");
+      if (l.heads < 1 || l.dim < 1 || l.vdim < 1 || !lin_pad_n(l.dim) || l.vdim > 1024 ||
+          (key ? l.rank < 1 || l.tau <= 0 : l.groups < 1 || l.heads % l.groups || l.conv < 1 || l.conv > 16 || l.norm_groups < 1 ||
+                                               (l.heads * l.vdim) % l.norm_groups))
+        throw std::runtime_error(at + "bad sizes of the linear recurrence");
+      D.lin = key ? LIN_KEY : LIN_HEAD;
+      D.lH = l.heads;
+      D.lG = key ? l.heads : l.groups;
+      D.lN = l.dim;
+      D.lnp = lin_pad_n(l.dim);
+      D.ldv = l.vdim;
+      D.lvp = up(l.vdim, 16);
+      D.lin_off = n;
+      D.lin_out = D.gn;
+      n += key ? D.lH * (2 * D.lN + 2 * D.ldv) + l.rank : 2 * D.lH * D.ldv + 2 * D.lG * D.lN + D.lH;
+      D.gn += up(D.lH * D.ldv, 64);
+      recurrent_ = true;
+    }
+    n = up(n, 64);
     D.ff = s.mlp != MLP_NONE ? s.ff : 0;
     D.fp = up(D.ff, 64);
     if (s.parallel) {
@@ -124,6 +175,7 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
     D.kout = D.gn;
     D.shf = s.mlp == MLP_MOE ? s.shared_ff : 0;
     D.shp = up(D.shf, 64);
+    if (s.mlp == MLP_ACT) D.fp = up_n(D.ff);
     D.glu = s.mlp == MLP_MOE ? D.shp : D.fp;
     D.router_off = s.resid_gate ? dp_ : 0;
     D.n2 = up_n(D.router_off + (s.mlp == MLP_MOE ? up(s.experts, 64) : 0));
@@ -133,14 +185,14 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
     const bool looped = c.loop_times > 0 && i >= c.loop_start && i < c.loop_stop;
     if (looped && i == c.loop_start)
       for (int t = 0; t < c.loop_times; ++t)
-        for (int j = c.loop_start; j < c.loop_stop; ++j) runs_.push_back({j, t, nullptr, nullptr});
-    if (!looped) runs_.push_back({i, -1, nullptr, nullptr});
+        for (int j = c.loop_start; j < c.loop_stop; ++j) runs_.push_back({j, t, nullptr, nullptr, nullptr});
+    if (!looped) runs_.push_back({i, -1, nullptr, nullptr, nullptr});
   }
   if (c.loop_times > 0 && !seq_) throw std::runtime_error("layered model: a loop of parallel layers");
   embd_ = balloc((size_t)v_ * dp_);
   if (c.max_positions) posw_ = balloc((size_t)c.max_positions * dp_);
   if (c.bigram_buckets) pairw_ = balloc((size_t)(c.bigram_buckets + 1) * dp_);
-  if (c.loop_times > 0) {
+  if (c.loop_times > 0 && !c.loop_add) {
     loopw_ = balloc((size_t)dp_ * 2 * dp_);
     loop_step_ = falloc((size_t)c.loop_times * dp_);
   }
@@ -164,9 +216,30 @@ void LayeredDecoder::alloc_layer(int i) {
     w.sink = falloc(D.H);
     w.ukv = balloc((size_t)(D.qn + D.gn) * D.rp);
     w.ukT = balloc((size_t)D.H * D.rp * D.dkp);
-  } else {
+  } else if (s.mixer == MIX_MINGRU) {
     w.zb = falloc(D.wp);
     w.ub = falloc(D.wp);
+  } else if (s.mixer == MIX_GQA) {
+    w.sink = falloc(D.H);
+    if (s.attn_bias) {
+      w.qb = falloc(D.H * D.dk);
+      w.kb = falloc(D.G * D.dk);
+      w.vb = falloc(D.G * D.dv);
+      w.ob = falloc(dp_);
+    }
+  }
+  if (D.lin == LIN_HEAD) {
+    const int C = D.lH * D.ldv + 2 * D.lG * D.lN;
+    w.conv_w = falloc((size_t)C * s.lin.conv);
+    w.conv_b = falloc(C);
+    w.dt_b = falloc(D.lH);
+    w.a_log = falloc(D.lH);
+    w.lin_d = falloc(D.lH);
+    w.lin_norm = falloc((size_t)D.lH * D.ldv);
+  } else if (D.lin == LIN_KEY) {
+    w.a2 = falloc((size_t)D.lH * D.lN * s.lin.rank);
+    w.a2_b = falloc((size_t)D.lH * D.lN);
+    w.lin_norm = falloc(D.ldv);
   }
   if (s.parallel) {
     w.in = balloc((size_t)D.nin * dp_);
@@ -181,7 +254,11 @@ void LayeredDecoder::alloc_layer(int i) {
   w.norm2 = falloc(dp_);
   if (s.post_norm) w.post2 = falloc(dp_);
   if (s.resid_gate) w.rgb2 = falloc(dp_);
-  w.in2 = balloc((size_t)(D.n2 + 2 * D.glu) * dp_);
+  w.in2 = balloc((size_t)(D.n2 + (s.mlp == MLP_ACT ? 1 : 2) * D.glu) * dp_);
+  if (s.mlp == MLP_ACT && s.mlp_bias) {
+    w.upb = falloc(D.fp);
+    w.dnb = falloc(dp_);
+  }
   if (D.glu) w.out2 = balloc((size_t)dp_ * D.glu);
   if (s.mlp == MLP_MOE) {
     w.corr = falloc(s.experts);
@@ -261,13 +338,44 @@ void LayeredDecoder::list_tensors() {
       if (s.sink) add(p + "attn_sinks.weight", 1, D.H);
       if (s.out_gate) add(p + "attn_gate.weight", s.out_gate == GATE_HEAD ? D.H : D.H * D.dv, d_);
       add(p + "attn_output.weight", d_, D.H * D.dv);
-    } else {
+    } else if (s.mixer == MIX_GQA) {
+      const struct { const char* n; int rows, cols; } mats[] = {
+          {"attn_q", D.H * D.dk, d_}, {"attn_k", D.G * D.dk, d_}, {"attn_v", D.G * D.dv, d_}, {"attn_output", d_, D.H * D.dv}};
+      for (const auto& m : mats) {
+        add(p + m.n + ".weight", m.rows, m.cols);
+        if (s.attn_bias) add(p + m.n + ".bias", 1, m.rows);
+      }
+      if (s.sink) add(p + "attn_sinks.weight", 1, D.H);
+      if (s.out_gate) add(p + "attn_gate.weight", D.H, d_);
+    } else if (s.mixer == MIX_MINGRU) {
       for (const char* n : {"z", "x"}) {
         add(p + "rnn_" + n + ".weight", s.width, d_);
         add(p + "rnn_" + n + ".bias", 1, s.width);
       }
       add(p + "rnn_gate.weight", s.width, d_);
       add(p + "rnn_output.weight", d_, s.width);
+    }
+    if (D.lin == LIN_HEAD) {
+      const int inner = D.lH * D.ldv, C = inner + 2 * D.lG * D.lN;
+      add(p + "ssm_in.weight", inner + C + D.lH, d_);
+      add(p + "ssm_conv1d.weight", C, s.lin.conv);
+      add(p + "ssm_conv1d.bias", 1, C);
+      add(p + "ssm_dt.bias", 1, D.lH);
+      add(p + "ssm_a_log.bias", 1, D.lH);
+      add(p + "ssm_d.bias", 1, D.lH);
+      add(p + "ssm_norm.weight", 1, inner);
+      add(p + "ssm_out.weight", d_, inner);
+    } else if (D.lin == LIN_KEY) {
+      const int nk = D.lH * D.lN, nv = D.lH * D.ldv;
+      add(p + "gla_q.weight", nk, d_);
+      add(p + "gla_k.weight", nk, d_);
+      add(p + "gla_v.weight", nv, d_);
+      add(p + "gla_gate.weight", nv, d_);
+      add(p + "gla_a1.weight", s.lin.rank, d_);
+      add(p + "gla_a2.weight", nk, s.lin.rank);
+      add(p + "gla_a2.bias", 1, nk);
+      add(p + "gla_norm.weight", 1, D.ldv);
+      add(p + "gla_output.weight", d_, nv);
     }
     auto closing = [&](const std::string& sub) {
       if (s.post_norm) add(p + sub + "_post_norm.weight", 1, nw);
@@ -286,6 +394,15 @@ void LayeredDecoder::list_tensors() {
       add(p + "ffn_gate.weight", D.ff, d_);
       add(p + "ffn_up.weight", D.ff, d_);
       add(p + "ffn_down.weight", d_, D.ff);
+      continue;
+    }
+    if (s.mlp == MLP_ACT) {
+      add(p + "ffn_up.weight", D.ff, d_);
+      add(p + "ffn_down.weight", d_, D.ff);
+      if (s.mlp_bias) {
+        add(p + "ffn_up.bias", 1, D.ff);
+        add(p + "ffn_down.bias", 1, d_);
+      }
       continue;
     }
     add(p + "ffn_gate_inp.weight", s.experts, d_);
@@ -345,6 +462,30 @@ void LayeredDecoder::put(const std::string& name, int rows, int cols, const bf16
   else if (t == "ffn_post_norm.weight") norm(w.post2);
   else if (t == "attn_kv_a_norm.weight") put_vec(w.kv_norm, cols, src, device);
   else if (t == "attn_sinks.weight") put_vec(w.sink, cols, src, device);
+  else if (s.mixer == MIX_GQA && t == "attn_q.weight") rows_at(w.in, 0);
+  else if (s.mixer == MIX_GQA && t == "attn_k.weight") rows_at(w.in, D.koff);
+  else if (s.mixer == MIX_GQA && t == "attn_v.weight") rows_at(w.in, D.voff);
+  else if (t == "attn_q.bias") put_vec(w.qb, cols, src, device);
+  else if (t == "attn_k.bias") put_vec(w.kb, cols, src, device);
+  else if (t == "attn_v.bias") put_vec(w.vb, cols, src, device);
+  else if (t == "attn_output.bias") put_vec(w.ob, cols, src, device, 0, s.mixer_scale);
+  else if (t == "ssm_in.weight" || t == "gla_q.weight") rows_at(w.in, D.lin_off);
+  else if (t == "gla_k.weight") rows_at(w.in, D.lin_off + D.lH * D.lN);
+  else if (t == "gla_v.weight") rows_at(w.in, D.lin_off + 2 * D.lH * D.lN);
+  else if (t == "gla_gate.weight") rows_at(w.in, D.lin_off + 2 * D.lH * D.lN + D.lH * D.ldv);
+  else if (t == "gla_a1.weight") rows_at(w.in, D.lin_off + 2 * D.lH * (D.lN + D.ldv));
+  else if (t == "gla_a2.weight") put_vec(w.a2, rows * cols, src, device);
+  else if (t == "gla_a2.bias") put_vec(w.a2_b, cols, src, device);
+  else if (t == "ssm_conv1d.weight") put_vec(w.conv_w, rows * cols, src, device);
+  else if (t == "ssm_conv1d.bias") put_vec(w.conv_b, cols, src, device);
+  else if (t == "ssm_dt.bias") put_vec(w.dt_b, cols, src, device);
+  else if (t == "ssm_a_log.bias") put_vec(w.a_log, cols, src, device);
+  else if (t == "ssm_d.bias") put_vec(w.lin_d, cols, src, device);
+  else if (t == "ssm_norm.weight" || t == "gla_norm.weight") put_vec(w.lin_norm, cols, src, device);
+  else if (t == "ssm_out.weight" || t == "gla_output.weight") place(w.out + D.lin_out, D.kout, src, cols, cols, rows, device);
+  else if (s.mlp == MLP_ACT && t == "ffn_up.weight") rows_at(w.in2, D.n2);
+  else if (t == "ffn_up.bias") put_vec(w.upb, cols, src, device);
+  else if (t == "ffn_down.bias") put_vec(w.dnb, cols, src, device);
   else if (t == "attn_q.weight") {
     heads(w.in, dp_, D.dk + D.rot, D.dkp, 0, D.dk);
     if (D.rot) heads(w.in + (size_t)D.qrot * dp_, dp_, D.dk + D.rot, D.dkp, D.dk, D.rot);
@@ -462,17 +603,17 @@ void LayeredDecoder::finalize() {
   for (int i = 0; i < nl_; ++i) {
     const Dims& D = dims_[i];
     const LayerSpec& s = c.layers[i];
-    if (s.mixer != MIX_LATENT) continue;
+    if (!D.H) continue;
     if (D.rot) {
-      float2*& t = ropes[{{s.rot_dim, s.rot_dims}, s.rot_base}];
+      float2*& t = ropes[{{D.rot, s.rot_dims}, s.rot_base}];
       if (!t) {
-        const std::vector<float> h = rope_table(s.rot_dim, s.rot_dims, s.rot_base);
+        const std::vector<float> h = rope_table(D.rot, s.rot_dims, s.rot_base);
         t = (float2*)e_.dmalloc(h.size() * 4);
         HIP_CHECK(hipMemcpy(t, h.data(), h.size() * 4, hipMemcpyHostToDevice));
       }
       rope_[i] = t;
     }
-    if (!w_[i].own) continue;
+    if (!w_[i].own || s.mixer != MIX_LATENT) continue;
     if (D.rot) {  // the rotated part of the cached row is a head's rotated key as it is
       std::vector<bf16_t> one((size_t)D.rot * D.rot, 0);
       for (int k = 0; k < D.rot; ++k) one[(size_t)k * D.rot + k] = 0x3f80;
@@ -486,12 +627,17 @@ void LayeredDecoder::finalize() {
   e_.kv_bytes_ = 0;
   for (Run& k : runs_) {
     const Dims& D = dims_[k.layer];
-    if (c.layers[k.layer].mixer == MIX_MINGRU) {
-      k.state = falloc((size_t)2 * c.max_slots * D.wp);
-      e_.kv_bytes_ += (size_t)2 * c.max_slots * D.wp * 4;
-      continue;
+    if (const size_t n = state_floats(k.layer)) {
+      k.state = falloc((size_t)2 * c.max_slots * n);
+      e_.kv_bytes_ += (size_t)2 * c.max_slots * n * 4;
     }
-    const size_t block = (size_t)e_.kvb_ * D.rp * es, bytes = (size_t)(e_.kv_nblocks_ + 1) * block;
+    if (const size_t n = ring_floats(k.layer)) {
+      k.ring = falloc((size_t)c.max_slots * n);
+      e_.kv_bytes_ += (size_t)c.max_slots * n * 4;
+    }
+    if (!D.H) continue;
+    if (D.G && e_.kvb_ != GQA_BLOCK) throw std::runtime_error("grouped-query attention: cache block size");
+    const size_t block = (D.G ? gqa_block_elems(D.G, D.dkp, D.dvp) : (size_t)e_.kvb_ * D.rp) * es, bytes = (size_t)(e_.kv_nblocks_ + 1) * block;
     k.pool = (char*)e_.dmalloc(bytes);
     HIP_CHECK(hipMemset(k.pool, 0, bytes));
     e_.pools_.push_back({k.pool, block});
@@ -504,12 +650,20 @@ void LayeredDecoder::finalize() {
   int n1 = 0, nin = 0, kout = 0, fp = 0, wp = 0;
   size_t qa = 0, part = 0, kvw = 0, flat = 0;
   size_t e_act = 0, e_gu = 0, pairs = 0;  // experts
+  LinWs lw = {0, 0, 0, 0, 0, 0};
+  size_t lin_y = 0;
   int rp = 0;
   for (int i = 0; i < nl_; ++i) {
     const Dims& D = dims_[i];
     const LayerSpec& s = c.layers[i];
     n1 = std::max({n1, D.n1, D.n2});
     nin = std::max({nin, D.nin, D.n1, D.n2 + 2 * D.glu});
+    if (D.lin) {
+      const LinWs l = lin_ws(D.lin, D.lH, D.lG, D.lnp, D.lvp, f32_);
+      lw = LinWs{std::max(lw.qo, l.qo), std::max(lw.ko, l.ko), std::max(lw.kr, l.kr),
+                 std::max(lw.vo, l.vo), std::max(lw.so, l.so), std::max(lw.dec, l.dec)};
+      lin_y = std::max(lin_y, (size_t)R * D.lH * D.ldv);
+    }
     kout = std::max({kout, D.kout, D.glu});
     fp = std::max(fp, seq_ ? D.glu : D.fp);
     wp = std::max(wp, D.wp);
@@ -519,6 +673,12 @@ void LayeredDecoder::finalize() {
       e_act = std::max(e_act, P * D.fp);
       e_gu = std::max(e_gu, P * 2 * D.fp);
       moe_max_tiles_ = std::max(moe_max_tiles_, s.experts + (int)(P / 32));
+    }
+    if (D.G) {
+      qa = std::max(qa, (size_t)R * D.H * D.dkp);
+      const size_t fl = std::max((size_t)R * D.H, (size_t)16 * 1024);  // (key_split: rows x splits)
+      flat = std::max(flat, fl);
+      part = std::max(part, fl * D.dvp);
     }
     if (s.mixer != MIX_LATENT) continue;
     rp = std::max(rp, D.rp);
@@ -544,6 +704,21 @@ void LayeredDecoder::finalize() {
     y_ = falloc((size_t)R * dp_);
     e_.ws_bytes_ += (size_t)R * dp_ * 4;
     if (loopw_) xin_ = operand((size_t)R * 2 * dp_);
+    if (c.loop_times > 1 && c.loop_add) {
+      x0_ = falloc((size_t)R * dp_);
+      e_.ws_bytes_ += (size_t)R * dp_ * 4;
+    }
+    if (lin_y) {
+      const size_t nb = (size_t)2 * max_chunks_;  // (a chunk is two blocks)
+      lin_qo_ = operand(nb * lw.qo);
+      lin_ko_ = operand(nb * lw.ko);
+      lin_kr_ = operand(nb * lw.kr);
+      lin_vo_ = operand(nb * lw.vo);
+      lin_so_ = operand(nb * lw.so);
+      lin_dec_ = falloc(nb * lw.dec);
+      lin_y_ = falloc(lin_y);
+      e_.ws_bytes_ += (nb * lw.dec + lin_y) * 4;
+    }
     if (wp) {
       agg_ = falloc((size_t)max_chunks_ * 3 * wp);
       e_.ws_bytes_ += (size_t)max_chunks_ * 3 * wp * 4;
@@ -582,13 +757,17 @@ void LayeredDecoder::finalize() {
     // whole context + dim + vdim per pair) drop below the absorbed form's (2 x rank per pair)
     pf_min_ = rp ? 0 : 1 << 30;
     for (const Dims& D : dims_) {
-      if (!D.H) continue;
+      if (!D.H || D.G) continue;
       const double s = D.dkp + D.dvp, gain = 2.0 * D.rp - s;
       const int t = gain > 0 ? (int)std::min(256.0, std::max(64.0, D.rp * s / gain)) : 256;
       pf_min_ = std::max(pf_min_, t);
     }
     if (const char* v = std::getenv("AIOS_LATENT_PF_MIN"))
       if (rp) pf_min_ = std::max(1, std::atoi(v));
+    // grouped-query attention: the flash kernel's 128-row blocks from half a block on
+    for (const Dims& D : dims_)
+      if (D.G) pf_min_ = rp ? std::max(pf_min_, 64) : env_or("AIOS_GQA_PF_MIN", 64);
+    if (!rp) pf_max_ctx_ = 1 << 30;  // (no context is expanded)
     for (const Dims& D : dims_)
       if (D.H && !mha_prefill_supports(D.dkp, D.dvp)) pf_min_ = 1 << 30;
     // the skinny GEMM's split-K workspace (shared with the engine's other users of gemm())
@@ -610,13 +789,14 @@ void LayeredDecoder::finalize() {
     }
   }
   // step parameters
-  std::set<int> hs;
+  std::set<int> hs;  // rows of a token that read the same keys
   for (const Dims& D : dims_)
-    if (D.H) hs.insert(D.H);
+    if (D.H) hs.insert(D.G ? D.H / D.G : D.H);
   size_t tiles = 0;
   for (int h : hs) tiles += (size_t)R * ((h + 15) / 16) + R;
   const size_t chunk_ints = (size_t)max_chunks_ * (sizeof(ScanChunk) / 4);
-  step_ints_ = (size_t)5 * R + chunk_ints + 2 * tiles;
+  const size_t seq_ints = (size_t)std::min(R, max_chunks_) * (sizeof(ScanSeq) / 4);
+  step_ints_ = (size_t)5 * R + chunk_ints + seq_ints + 1 + 2 * tiles;
   HIP_CHECK(hipHostMalloc((void**)&h_step_, step_ints_ * 4, hipHostMallocDefault));
   d_step_ = (int*)falloc(step_ints_);
   st_tokens_ = d_step_;
@@ -625,7 +805,8 @@ void LayeredDecoder::finalize() {
   st_want_ = st_slot_ + R;
   st_run_ = st_want_ + R;
   st_chunks_ = (ScanChunk*)(st_run_ + R);
-  st_tiles_ = (LatentTile*)(st_run_ + R + chunk_ints);
+  st_seqs_ = (ScanSeq*)(st_run_ + R + chunk_ints);
+  st_tiles_ = (LatentTile*)(st_run_ + R + chunk_ints + seq_ints);
   gemv_ok_.assign(5, 0);
   for (int b = 1; b <= 4 && !f32_; ++b) {
     bool ok = !seq_ && dp_ == d_ && env_or("AIOS_LAYERED_GEMV", 1);
@@ -675,7 +856,10 @@ void LayeredDecoder::tune() {
       if (seq_) {
         go(cat16_, D.kout, w.out, dp_, D.kout, GEPI_STORE, y_, dp_, nullptr, act);
         if (w.in2 && D.n2) go(h16_, dp_, w.in2, D.n2, dp_, GEPI_STORE, qdg_, D.n2, nullptr, act);
-        if (D.glu) {
+        if (D.glu && e_.cfg_.layers[i].mlp == MLP_ACT) {
+          go(h16_, dp_, w.in2 + (size_t)D.n2 * dp_, D.glu, dp_, GEPI_STORE16, nullptr, D.glu, cat16_, 0);
+          go(cat16_, D.glu, w.out2, dp_, D.glu, GEPI_STORE, y_, dp_, nullptr, act);
+        } else if (D.glu) {
           go(h16_, dp_, w.in2 + (size_t)D.n2 * dp_, 2 * D.glu, dp_, GEPI_SWIGLU_BF16, nullptr, D.glu, cat16_, act);
           go(cat16_, D.glu, w.out2, dp_, D.glu, GEPI_STORE, y_, dp_, nullptr, act);
         }
@@ -683,7 +867,7 @@ void LayeredDecoder::tune() {
         if (D.fp) go(h16_, dp_, w.in + (size_t)D.n1 * dp_, 2 * D.fp, dp_, GEPI_SWIGLU_BF16, nullptr, D.kout, cat16_ + D.gn, act);
         go(cat16_, D.kout, w.out, dp_, D.kout, GEPI_ACCUM, x_, dp_, nullptr, act);
       }
-      if (D.H && M <= pf_max_ctx_) go(cfull_, D.rp, w.ukv, D.qn + D.gn, D.rp, GEPI_STORE16, nullptr, D.qn + D.gn, kv_, act);
+      if (D.rp && M <= pf_max_ctx_) go(cfull_, D.rp, w.ukv, D.qn + D.gn, D.rp, GEPI_STORE16, nullptr, D.qn + D.gn, kv_, act);
     }
   }
   HIP_CHECK(hipMemsetAsync(h16_, 0, (size_t)step_rows_ * dp_ * 2, e_.stream_));
@@ -801,6 +985,124 @@ void LayeredDecoder::recurrence(int k, const RowSet& r) {
   launch_mingru(a, e_.stream_);
 }
 
+size_t LayeredDecoder::state_floats(int i) const {
+  const Dims& D = dims_[i];
+  return (size_t)D.wp + (D.lin ? (size_t)D.lH * D.lnp * D.lvp : 0);
+}
+size_t LayeredDecoder::ring_floats(int i) const {
+  const Dims& D = dims_[i];
+  return D.lin == LIN_HEAD ? (size_t)e_.cfg_.layers[i].lin.conv * (D.lH * D.ldv + 2 * D.lG * D.lN) : 0;
+}
+
+void LayeredDecoder::linear(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
+  const Dims& D = dims_[i];
+  const LayerSpec& s = e_.cfg_.layers[i];
+  const Weights& w = w_[owner_[i]];
+  const int nk = D.lH * D.lN, nv = D.lH * D.ldv, c0 = D.lin_off;
+  LinScanArgs a;
+  std::memset(&a, 0, sizeof(a));
+  a.kind = D.lin;
+  a.H = D.lH; a.G = D.lG; a.N = D.lN; a.np = D.lnp; a.dv = D.ldv; a.vp = D.lvp;
+  a.in = qdg_; a.ld = D.n1;
+  if (D.lin == LIN_HEAD) {  // [z | x | B | C | dt]
+    a.z_off = c0;
+    a.x_off = c0 + nv;
+    a.dt_off = c0 + 2 * nv + 2 * D.lG * D.lN;
+    a.taps = s.lin.conv;
+    a.norm_parts = s.lin.norm_groups;
+  } else {  // [q | k | v | gate | a]
+    a.q_off = c0;
+    a.k_off = c0 + nk;
+    a.v_off = c0 + 2 * nk;
+    a.z_off = c0 + 2 * nk + nv;
+    a.a_off = c0 + 2 * nk + 2 * nv;
+    a.rank = s.lin.rank;
+    a.q_scale = (float)(1.0 / std::sqrt((double)D.lN));
+    a.inv_tau = (float)(1.0 / s.lin.tau);
+  }
+  a.conv_w = w.conv_w; a.conv_b = w.conv_b; a.dt_b = w.dt_b; a.a_log = w.a_log; a.D = w.lin_d;
+  a.a2 = w.a2; a.a2_b = w.a2_b;
+  a.ring = runs_[k].ring;
+  a.state = runs_[k].state; a.slots = e_.cfg_.max_slots;
+  if (!r.decode) {
+    a.seqs = st_seqs_; a.n_seqs = r.n_seqs;
+    a.chunks = st_chunks_; a.n_chunks = r.n_chunks;
+  }
+  a.pos = r.pos; a.slot = r.slot; a.n = a.rows = r.n;
+  a.qo = lin_qo_; a.ko = lin_ko_; a.kr = lin_kr_; a.vo = lin_vo_; a.so = lin_so_; a.dec = lin_dec_;
+  a.y = lin_y_;
+  a.norm_w = w.lin_norm;
+  a.eps = e_.cfg_.norm_eps;
+  a.out_scale = s.beside ? s.beside_scale : s.mixer_scale;
+  a.out = f32_ ? (void*)(cat32_ + D.lin_out) : (void*)(cat16_ + D.lin_out);
+  a.ldo = D.kout;
+  a.f32 = f32_;
+  launch_lin_scan(a, e_.stream_);
+}
+
+void LayeredDecoder::grouped_attention(int k, const RowSet& r) {
+  const int i = runs_[k].layer;
+  const Dims& D = dims_[i];
+  const LayerSpec& s = e_.cfg_.layers[i];
+  const Weights& w = w_[owner_[i]];
+  hipStream_t st = e_.stream_;
+  GqaArgs a;
+  std::memset(&a, 0, sizeof(a));
+  a.rows = r.n; a.n = f32_ ? r.n : r.n_abs;
+  a.H = D.H; a.G = D.G; a.dk = D.dk; a.dkp = D.dkp; a.dv = D.dv; a.dvp = D.dvp;
+  a.rot = D.rot; a.rope = rope_[i];
+  a.window = s.window; a.chunk = s.chunk;
+  a.scale = s.scale; a.softcap = s.softcap;
+  a.sink = s.sink ? w.sink : nullptr;
+  a.qb = w.qb; a.kb = w.kb; a.vb = w.vb;
+  a.in = qdg_; a.ld = D.n1; a.k_off = D.koff; a.v_off = D.voff; a.g_off = s.out_gate == GATE_HEAD ? D.gate_off : -1;
+  a.out_scale = s.mixer_scale;
+  a.pos = r.pos; a.slot = r.slot;
+  a.pool = runs_[k].pool; a.bt = e_.d_bt_; a.maxb = e_.kv_maxb_; a.f32 = f32_;
+  a.q = qa_;
+  const int rep = D.H / D.G;
+  if (r.decode) {
+    a.n_tiles = r.n * ((rep + 15) / 16);
+  } else {
+    const auto t = r.tiles.at(rep);
+    a.tiles = st_tiles_ + t.first;
+    a.n_tiles = t.second;
+  }
+  // (a tile's keys reach from its first row's first one to its last row: at most 15 tokens more)
+  const int w1 = s.window ? s.window : 1 << 30, w2 = s.chunk ? s.chunk : 1 << 30;
+  const int keys = std::min(r.max_len, std::min(w1, w2) + 15);
+  a.nsplit = f32_ ? 1 : std::min(64, key_split(a.n_tiles * D.G, (keys + 3) / 4));  // (four waves share a split's keys)
+  a.opart = opart_; a.ml = ml_;
+  a.out = f32_ ? (void*)cat32_ : (void*)cat16_;
+  a.ldo = D.kout;
+  launch_gqa_prep(a, st);
+  if (a.n > 0) launch_gqa_attn(a, st);
+  for (const auto& pf : r.pf) {
+    if (f32_) break;
+    const Piece& p = pf.second;
+    const int row0 = pf.first;
+    MhaPrefillArgs m;
+    std::memset(&m, 0, sizeof(m));
+    m.q16 = (const bf16_t*)qa_ + (size_t)row0 * D.H * D.dkp;
+    m.pool = (const bf16_t*)a.pool;
+    m.bt = e_.d_bt_ + (size_t)p.slot * e_.kv_maxb_;
+    m.G = D.G; m.H = D.H; m.dkp = D.dkp; m.dvp = D.dvp;
+    m.start = p.start; m.T = p.n;
+    m.window = s.window; m.chunk = s.chunk;
+    m.softcap = s.softcap; m.out_scale = s.mixer_scale;
+    m.sink = a.sink;
+    m.gate = a.g_off >= 0 ? qdg_ + (size_t)row0 * D.n1 + a.g_off : nullptr;
+    m.ldq = D.n1; m.head_gate = 1;
+    m.out = cat16_ + (size_t)row0 * D.kout; m.ldo = D.kout;
+    launch_mha_prefill(m, st);
+  }
+}
+
+bool LayeredDecoder::enters_pass(int k) const {
+  return x0_ && k < runs_to_do() && runs_[k].pass > 0 && runs_[k].layer == e_.cfg_.loop_start;
+}
+
 // ---- sequential layers --------------------------------------------------------------------------------
 void LayeredDecoder::project(const void* a, int lda, const bf16_t* w, int n, int N, int K, float* y, int ldy) {
   if (f32_) return launch_gemm_f32((const float*)a, lda, w, K, n, N, K, y, ldy, 0, e_.stream_);
@@ -820,7 +1122,7 @@ NextArgs LayeredDecoder::next_of(int k, bool decode) {
     if (!decode) return x;  // (a step's head gathers and normalises the rows it is asked for)
     x.kind = NEXT_NORM;
     x.g = out_norm_;
-  } else if (runs_[k].pass >= 0 && runs_[k].layer == e_.cfg_.loop_start) {
+  } else if (loopw_ && runs_[k].pass >= 0 && runs_[k].layer == e_.cfg_.loop_start) {
     x.kind = NEXT_RAW;
     x.out = xin_;
     x.ldo = 2 * dp_;
@@ -855,6 +1157,38 @@ void LayeredDecoder::feed_forward(int k, const RowSet& r, RowCloseArgs& c) {
   void* act = f32_ ? (void*)cat32_ : (void*)cat16_;
   const bf16_t* wglu = w.in2 + (size_t)D.n2 * dp_;
   bool done = false;
+  if (s.mlp == MLP_ACT) {
+    if (D.n2) project(h, dp_, w.in2, n, D.n2, dp_, qdg_, D.n2);
+    if (f32_) {
+      launch_gemm_f32(h32_, dp_, wglu, dp_, n, D.fp, dp_, gu32_, D.fp, 0, e_.stream_);
+      launch_bias_act_f32(gu32_, D.fp, w.upb, cat32_, D.fp, n, D.fp, s.act, e_.stream_);
+    } else {
+      if (n <= 4) {
+        GemvArgs a = e_.gemv_args({}, D.fp, dp_, n, nullptr, dp_, nullptr, nullptr, D.fp, EPI_ACT16, 0);
+        a.nseg = 1;
+        a.seg[0] = mat(wglu, D.fp, dp_);
+        a.x16 = h16_;
+        a.act = s.act;
+        a.bias = w.upb;
+        a.y16 = cat16_;
+        a.ldy16 = D.fp;
+        done = gemv_bf16_engine_fits(a);
+        if (done) launch_gemv(a, e_.stream_);
+      }
+      if (!done) {
+        GemmQArgs g;
+        std::memset(&g, 0, sizeof(g));
+        g.A = h16_; g.lda = dp_; g.M = n; g.N = D.fp; g.K = dp_; g.nseg = 1; g.seg[0] = mat(wglu, D.fp, dp_);
+        g.C16 = cat16_; g.ldc = D.fp; g.epi = GEPI_STORE16;
+        g.bias16 = w.upb; g.unary = 1 + s.act;
+        e_.gemm(g);
+      }
+    }
+    project(act, D.fp, w.out2, n, dp_, D.fp, y_, dp_);
+    c.y = y_;
+    c.y_bias = w.dnb;
+    return;
+  }
   if (!f32_ && D.glu && n <= 64) {  // one launch over all rows of in2
     const int N = D.n2 + 2 * D.glu;
     if (n <= 4) {
@@ -922,7 +1256,7 @@ void LayeredDecoder::layer_seq(int k, const RowSet& r) {
   hipStream_t st = e_.stream_;
   const void* h = f32_ ? (const void*)h32_ : (const void*)h16_;
   void* cat = f32_ ? (void*)cat32_ : (void*)cat16_;
-  if (runs_[k].pass >= 0 && i == e_.cfg_.loop_start) {  // a pass begins: x = W [x; x0] + step
+  if (loopw_ && runs_[k].pass >= 0 && i == e_.cfg_.loop_start) {  // a pass begins: x = W [x; x0] + step
     project(xin_, 2 * dp_, loopw_, n, dp_, 2 * dp_, y_, dp_);
     RowCloseArgs c = close_args();
     c.replace = 1;
@@ -935,12 +1269,16 @@ void LayeredDecoder::layer_seq(int k, const RowSet& r) {
   }
   project(h, dp_, w.in, n, D.n1, dp_, qdg_, D.n1);
   if (s.mixer == MIX_MINGRU) recurrence(k, r);
-  else attention(k, r);
+  else if (s.mixer == MIX_GQA) grouped_attention(k, r);
+  else if (s.mixer == MIX_LATENT) attention(k, r);
+  if (D.lin) linear(k, r);
   project(cat, D.kout, w.out, n, dp_, D.kout, y_, dp_);
   RowCloseArgs c = close_args();
   if (s.resid_gate) { c.gate = qdg_ + D.rg_off; c.ldg = D.n1; c.gate_bias = w.rgb; }
   if (s.post_norm) c.post = w.post;
+  c.y_bias = w.ob;
   if (s.mlp == MLP_NONE) {
+    if (enters_pass(k + 1)) c.extra = x0_;
     c.next = next_of(k + 1, r.decode);
     return launch_row_close(c, n, st);
   }
@@ -953,6 +1291,7 @@ void LayeredDecoder::layer_seq(int k, const RowSet& r) {
   feed_forward(k, r, f);
   if (s.resid_gate) { f.gate = qdg_; f.ldg = D.n2; f.gate_bias = w.rgb2; }
   if (s.post_norm) f.post = w.post2;
+  if (enters_pass(k + 1)) f.extra = x0_;
   f.next = next_of(k + 1, r.decode);
   launch_row_close(f, n, st);
 }
@@ -1040,11 +1379,12 @@ void LayeredDecoder::run(const RowSet& r) {
     e.keep = f32_ ? (void*)((float*)xin_ + dp_) : (void*)((bf16_t*)xin_ + dp_);
     e.ld_keep = 2 * dp_;
   }
+  e.keep32 = x0_;
   e.f32 = f32_;
   if (seq_) e.next = next_of(0, r.decode);
   launch_embed_rows(e, r.n, e_.stream_);
   norm_ready_ = false;
-  const int n = run_limit_ < 0 ? (int)runs_.size() : std::min(run_limit_, (int)runs_.size());
+  const int n = runs_to_do();
   for (int k = 0; k < n; ++k) {
     if (seq_) layer_seq(k, r);
     else if (f32_) layer32(k, r);
@@ -1055,7 +1395,7 @@ void LayeredDecoder::run(const RowSet& r) {
 void LayeredDecoder::decode_forward(int B) {
   RowSet r;
   r.tokens = e_.d_tokens_; r.pos = e_.d_pos_; r.slot = e_.d_slot_; r.run = nullptr;
-  r.n_chunks = r.split = 0;
+  r.n_chunks = r.split = r.n_seqs = 0;
   r.n = r.n_abs = B;
   r.decode = true;
   r.max_len = e_.cfg_.max_ctx;
@@ -1093,8 +1433,9 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
   first_row.assign(pieces.size(), 0);
   int *ht = h_step_, *hp = ht + R, *hs = hp + R, *hr = hs + 2 * R;
   ScanChunk* chunks = (ScanChunk*)(hr + R);
+  ScanSeq* seqs = (ScanSeq*)(h_step_ + ((const int*)st_seqs_ - d_step_));
   LatentTile* tiles = (LatentTile*)(h_step_ + ((const int*)st_tiles_ - d_step_));
-  r.n_chunks = r.split = 0;
+  r.n_chunks = r.split = r.n_seqs = 0;
   int row = 0, nt = 0;
   for (int o = 0; o < (int)order.size(); ++o) {
     const Piece& q = pieces[order[o]];
@@ -1106,6 +1447,7 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
       hr[row + k] = k ? 0 : q.n;
     }
     const int c0 = r.n_chunks;
+    seqs[r.n_seqs++] = ScanSeq{row, q.n, q.slot, q.start, 2 * c0};
     if (c0 + (q.n + SCAN_CHUNK - 1) / SCAN_CHUNK > max_chunks_) throw std::runtime_error("layered forward: too many pieces");
     for (int k = 0; k < q.n; k += SCAN_CHUNK)
       chunks[r.n_chunks++] = ScanChunk{row + k, std::min(SCAN_CHUNK, q.n - k), q.slot, q.start + k, c0, k + SCAN_CHUNK >= q.n};
@@ -1114,13 +1456,14 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
     row += q.n;
   }
   for (const Dims& D : dims_) {
-    if (!D.H || r.tiles.count(D.H)) continue;
+    const int rep = D.G ? D.H / D.G : D.H;  // rows of a token that read the same keys
+    if (!D.H || r.tiles.count(rep)) continue;
     const int t0 = nt;
     for (int o = 0; o < n_small; ++o) {
-      const int f0 = first_row[order[o]] * D.H, f1 = f0 + pieces[order[o]].n * D.H;
+      const int f0 = first_row[order[o]] * rep, f1 = f0 + pieces[order[o]].n * rep;
       for (int f = f0; f < f1; f += 16) tiles[nt++] = LatentTile{f, std::min(16, f1 - f)};
     }
-    r.tiles[D.H] = {t0, nt - t0};
+    r.tiles[rep] = {t0, nt - t0};
   }
   r.tokens = st_tokens_; r.pos = st_pos_; r.slot = st_slot_; r.run = st_run_;
   const size_t ints = (size_t)((const int*)st_tiles_ - d_step_) + 2 * (size_t)nt;
@@ -1188,8 +1531,12 @@ void LayeredDecoder::copy_state(int src, int dst) {
       HIP_CHECK(hipMemcpyAsync((char*)base + ((size_t)p * slots + dst) * row, (char*)base + ((size_t)p * slots + src) * row, row,
                                hipMemcpyDeviceToDevice, e_.stream_));
   };
-  for (const Run& k : runs_)
-    if (k.state) copy(k.state, (size_t)dims_[k.layer].wp * 4);
+  for (const Run& k : runs_) {
+    if (k.state) copy(k.state, state_floats(k.layer) * 4);
+    if (k.ring)
+      HIP_CHECK(hipMemcpyAsync(k.ring + dst * ring_floats(k.layer), k.ring + src * ring_floats(k.layer), ring_floats(k.layer) * 4,
+                               hipMemcpyDeviceToDevice, e_.stream_));
+  }
   if (last_tok_) copy(last_tok_, 4);
 }
 

@@ -2,6 +2,7 @@
 // closing of a sublayer, gated recurrences, mixtures of experts.  Rows are tokens of any sequences; all
 // row lengths are padded with zeros to whole 64-column tiles, norms divide by the true width.
 #pragma once
+#include "latent.h"
 #include "ops.h"
 
 namespace aios {
@@ -35,18 +36,22 @@ struct EmbedArgs {
   float* x;                   // [rows][dp]
   void* keep;                 // the embedding for later passes, bf16 or fp32, or null
   int ld_keep;
+  float* keep32;              // the same in fp32 [rows][dp], or null
   int f32;
   NextArgs next;
 };
 void launch_embed_rows(const EmbedArgs& a, int rows, hipStream_t st);
 
-// Closes a sublayer: v = y (+ the weighted expert rows); v *= sigmoid(gate + bias); v = rms(v) * post;
-// x += v -- or, replacing the residual (loop entry), x = y + add -- and the next operand, in one pass.
+// Closes a sublayer: v = y + y_bias (+ the weighted expert rows); v *= sigmoid(gate + bias); v = rms(v) * post;
+// x += v (+ rows of its own, extra) -- or, replacing the residual (loop entry), x = y + add -- and the next
+// operand, in one pass.
 struct RowCloseArgs {
   float* x;                   // [rows][dp]
   int dp, d;
   float eps;
   const float* y;             // [rows][dp] or null
+  const float* y_bias;        // [dp] or null
+  const float* extra;         // [rows][dp] or null: added to the new residual
   const void* ye;             // [pairs][dp] expert outputs (bf16 or fp32) or null
   const int* pair;            // [rows][top] row in ye
   const float* wt;            // [rows][top] weight
@@ -90,6 +95,107 @@ struct MinGruArgs {
   int ldo, f32;
 };
 void launch_mingru(const MinGruArgs& a, hipStream_t st);
+
+// ---- grouped-query attention (kernels/gqa.hip) ------------------------------------------------------
+// Query head h reads key / value head h / (H / G).  Keys and values are cached per block of GQA_BLOCK tokens as
+// [G][block][dkp] keys, then [G][block][dvp] values.  Head sizes are padded to dkp / dvp (multiples of 32) there and in
+// q; the input product's columns are not.  Rotation turns the pairs (i, i + rot / 2) of a head's first rot dimensions.
+//   s = q . k * scale;  s = softcap tanh(s / softcap) (softcap > 0);  weights exp(s) / (exp(sink_h) + sum exp(s)) over the
+//   visible keys;  out_h = out_scale * sigmoid(gate_h) * sum weights v
+// A query at position i sees keys j <= i with j > i - window (window > 0) and floor(j / chunk) = floor(i / chunk)
+// (chunk > 0).
+constexpr int GQA_BLOCK = 64;
+struct GqaArgs {
+  int rows;                   // rows of the step
+  int n;                      // rows [0, n) take launch_gqa_attn
+  int H, G, dk, dkp, dv, dvp;
+  int rot;                    // even; (cos, sin) of pair i at position p: rope[p * rot / 2 + i]
+  const float2* rope;
+  int window, chunk;
+  float scale, softcap;
+  const float* sink;          // [H] or null
+  const float *qb, *kb, *vb;  // biases of q [H dk], k [G dk], v [G dv], or null
+  const float* in;            // [rows][ld]: q, k, v at their offsets, gates at g_off + h (g_off -1: none)
+  int ld, q_off, k_off, v_off, g_off;
+  float out_scale;
+  const int *pos, *slot;      // [rows]
+  void* pool;                 // bf16 or fp32 (f32)
+  const int* bt;              // [slots][maxb]
+  int maxb, f32;
+  void* q;                    // [rows][H dkp]: rotated queries; bf16 (the score's factor folded in) or fp32
+  // flat rows [f0, f0 + nv) of the [row][query head of one kv head] space, one sequence each; null: every row its own
+  const LatentTile* tiles;
+  int n_tiles, nsplit;        // key splits (at most 64)
+  float* opart;               // [nsplit][n * H][dvp]
+  float* ml;                  // [nsplit][n * H][2]
+  void* out;                  // [rows][ldo], head h at h * dvp, bf16 or fp32
+  int ldo;
+};
+inline size_t gqa_block_elems(int G, int dkp, int dvp) { return (size_t)G * GQA_BLOCK * (dkp + dvp); }
+// factor of q . k folded into the bf16 queries
+float gqa_q_factor(float scale, float softcap);
+void launch_gqa_prep(const GqaArgs& a, hipStream_t st);  // queries; keys and values into the cache
+void launch_gqa_attn(const GqaArgs& a, hipStream_t st);
+bool gqa_supports(int dkp, int dvp);
+
+// ---- linear recurrences with a matrix state (kernels/linear_scan.hip) ----------------------------------
+// Per head, S [N][dv] in fp32:  S_t = d_t S_{t-1} + k_t v_t^T,  o_t = S_t^T q_t.
+//   LIN_HEAD  d_t one number per head (state-space duality).  x, B, C: a causal convolution per channel and SiLU of the
+//             input columns [x: H dv | B: G N | C: G N];  dt = softplus(in + dt_b);  d = exp(-exp(a_log) dt),
+//             k = dt B, q = C (group h / (H / G)), v = x;  y = o + D x.  out = rms over norm_parts equal parts of
+//             (y silu(z)) * norm_w [H dv].
+//   LIN_KEY   d_t one number per key channel (gated linear attention): d = sigmoid(a2 a + a2_b)^(1 / tau), k and v
+//             the input columns, q times q_scale (G = H).  out = rms(o) per head * norm_w [dv] * silu(z).
+// Portions run in blocks of LIN_T tokens: what a block needs besides the state it starts from (operands, decays,
+// scores between its own tokens) is prepared for all blocks side by side; then one wave per head and 16 columns of
+// v walks the blocks with its part of S in registers.  The state is kept twice, by parity of the position it was left
+// at, and the convolution's inputs in a ring of `taps` positions, so that a single token that is run again at the
+// same position finds what it started from.
+enum LinKind : int { LIN_HEAD = 1, LIN_KEY = 2 };
+constexpr int LIN_T = 16;
+struct ScanSeq {
+  int row0, n, slot, pos0;
+  int b0;           // index of its first block in the operand buffers
+};
+struct LinScanArgs {
+  int kind;
+  int H, G, N, np, dv, vp;    // np, vp: N and dv padded (lin_pad_n, multiple of 16)
+  const float* in;            // [rows][ld] input product
+  int ld, z_off;              // output gate [H dv]
+  int x_off, taps, dt_off;    // LIN_HEAD: convolved columns, step sizes [H]
+  const float *conv_w, *conv_b;        // [H dv + 2 G N][taps], last tap the current token's; bias
+  const float *dt_b, *a_log, *D;       // [H]
+  float* ring;                // [slots][taps][H dv + 2 G N]
+  int q_off, k_off, v_off, a_off, rank;  // LIN_KEY
+  float q_scale, inv_tau;
+  const float *a2, *a2_b;     // [H N][rank], [H N]
+  float* state;               // [2][slots][H][np][vp]
+  int slots;
+  // portions (seqs, and chunks: the same tokens in SCAN_CHUNK pieces); or n single tokens (pos, slot)
+  const ScanSeq* seqs;
+  int n_seqs;
+  const ScanChunk* chunks;
+  int n_chunks;
+  const int *pos, *slot;
+  int n;
+  // operands of the blocks (bf16 or fp32), see lin_ws
+  void *qo, *ko, *kr, *vo, *so;
+  float* dec;
+  float* y;                   // [rows][H dv]
+  const float* norm_w;
+  int norm_parts;
+  float eps, out_scale;
+  int rows;
+  void* out;                  // [rows][ldo], bf16 or fp32
+  int ldo, f32;
+};
+int lin_pad_n(int n);                                // 0: not served
+struct LinWs { size_t qo, ko, kr, vo, so, dec; };    // numbers per block
+LinWs lin_ws(int kind, int H, int G, int np, int vp, bool f32);
+void launch_lin_scan(const LinScanArgs& a, hipStream_t st);
+
+// y[r][i] = act(x[r][i] + bias[i]) in fp32
+void launch_bias_act_f32(const float* x, int ldx, const float* bias, float* y, int ldy, int rows, int n, int act, hipStream_t st);
 
 // ---- mixture of experts (kernels/moe.hip) -----------------------------------------------------------
 // Router: s = softmax(logits), the `top` largest of s + correction, weights s * scale.  The (token, expert) pairs

@@ -192,7 +192,7 @@ void launch_gemm(const GemmArgs& a, hipStream_t st);
 bool gemm_supports(int qt);
 
 // multi-segment GEMM with fused epilogues (the prefill path): C = A x [W0; W1; W2]^T
-// GEPI_STORE16 (bf16 weights): C16[m][n] = bf16.  GEPI_STORE_GLU (bf16 weights, M <= 64): one launch for
+// GEPI_STORE16 (bf16 weights): C16[m][n] = bf16, after bias16[n] and the activation `unary` (GluAct + 1) if set.  GEPI_STORE_GLU (bf16 weights, M <= 64): one launch for
 // projections that share their input -- columns below glu_n0 to C in fp32, the interleaved gate / up
 // columns from there on through the GLU to C16[m][(n - glu_n0) / 2] (row stride ldc16).
 enum GemmEpi {
@@ -212,6 +212,8 @@ struct GemmQArgs {
   int epi;
   int act;           // gate activation of the GLU epilogues (GluAct)
   int glu_n0, ldc16; // GEPI_STORE_GLU
+  const float* bias16;  // GEPI_STORE16: [N] or null
+  int unary;            // GEPI_STORE16: 0 none, else 1 + GluAct
   int ksplit;        // K split over workgroups: 0 = auto, 1 = off
   // skinny (M <= 64) split-K: fp32 partial slabs [S][tiles][16*Mt][rows] + per-tile arrival
   // tickets (zero-initialised, re-armed by each tile's last arriver).  Null -> no split.

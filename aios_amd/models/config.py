@@ -23,9 +23,28 @@ ROPE_NEOX = 2   # qwen: (x[i], x[i + rot/2])
 
 
 @dataclasses.dataclass(frozen=True)
+class LinConfig:
+    """A linear recurrence with a matrix state (csrc/layered.h LinSpec)."""
+    heads: int = 1
+    groups: int = 1                # heads that share B and C (mamba2)
+    dim: int = 64                  # state rows (key channels) per head
+    vdim: int = 64                 # state columns per head
+    conv: int = 4                  # taps (mamba2)
+    norm_groups: int = 1           # parts of the gated norm (mamba2)
+    rank: int = 16                 # width of the decay's first projection (gla)
+    tau: float = 16.0              # root taken of the decay (gla)
+
+
+@dataclasses.dataclass(frozen=True)
 class LayerConfig:
     """One layer of a model described layer by layer (csrc/layered.h LayerSpec)."""
-    mixer: str = "latent"          # "latent" attention | "mingru"
+    # "latent" attention | "mingru" | "gqa" attention | "mamba2" | "gla"
+    mixer: str = "latent"
+    # a second mixer reading the same input ("mamba2" | "gla"; "": none): mixer_scale * first + beside_scale * second
+    beside: str = ""
+    mixer_scale: float = 1.0
+    beside_scale: float = 1.0
+    lin: Optional[LinConfig] = None  # sizes of the linear recurrence among the two
     # parallel: mixer and MLP read one norm and are added together; else one after the other, each with a norm
     # of its own before it, and (post_norm) after it, and (resid_gate) its result times sigmoid(W h + b)
     parallel: bool = True
@@ -42,10 +61,16 @@ class LayerConfig:
     window: int = 0                # keys a token sees, itself included; 0: all before it
     scale: float = 0.125           # of q . k
     sink: bool = True              # a learned logit per head in the softmax's denominator
+    kv_heads: int = 1              # key / value heads (gqa), whose first rot_dims dimensions turn in halves
+    chunk: int = 0                 # gqa: keys before a token's chunk of so many positions are out; 0: no chunks
+    softcap: float = 0.0           # gqa: of the scores; 0: none
+    attn_bias: bool = False        # gqa: biases of q, k, v and the output projection
     out_gate: str = "element"      # head outputs times sigmoid(Wg h): "none" | "element" | "head" (one number)
     width: int = 64                # of the state (mingru)
-    ff: int = 256                  # hidden width of the gated MLP, or of every expert; 0: none
-    act: str = "gelu_tanh"         # of the gate: "gelu_tanh" | "silu"
+    ff: int = 256                  # hidden width of the MLP, or of every expert; 0: none
+    gated: bool = True             # the MLP has a gate; else W_down act(W_up h + b) + b
+    act: str = "gelu_tanh"         # of the gate or the hidden layer: "gelu_tanh" | "silu" | "relu2" (no gate)
+    mlp_bias: bool = False         # without a gate
     experts: int = 0               # mixture of experts (0: a dense MLP), of which every token uses `top`
     top: int = 0
     router_scale: float = 1.0
@@ -84,6 +109,9 @@ class ModelConfig:
     # embedding of token pairs, row (previous * mul_prev + current * mul_cur) mod buckets: (buckets, mul_prev, mul_cur)
     bigram: Optional[Tuple[int, int, int]] = None
     loop: Optional[Tuple[int, int, int]] = None  # layers [start, stop) run `times` times: (start, stop, times)
+    # how a pass of the loop is entered: False: every pass by a projection of the residual and the embedding; True:
+    # every pass but the first by adding the embedding
+    loop_add: bool = False
 
     @property
     def q_dim(self) -> int:
@@ -108,19 +136,28 @@ class ModelConfig:
         d = self.d_model
         n = 2 * self.vocab_size * d + (self.max_ctx * d if self.learned_pos else 0)
         n += (self.bigram[0] + 1) * d if self.bigram else 0
-        n += 2 * d * d + self.loop[2] * d if self.loop else 0
+        n += 2 * d * d + self.loop[2] * d if self.loop and not self.loop_add else 0
         for l in self.layers:
             if l.weights_of >= 0:
                 continue
+            for kind in (l.mixer, l.beside):
+                if kind == "mamba2":
+                    inner, gn = l.lin.heads * l.lin.vdim, 2 * l.lin.groups * l.lin.dim
+                    n += d * (3 * inner + gn + l.lin.heads) + (inner + gn) * (l.lin.conv + 1) + inner
+                elif kind == "gla":
+                    nk, nv = l.lin.heads * l.lin.dim, l.lin.heads * l.lin.vdim
+                    n += d * (2 * nk + 3 * nv + l.lin.rank) + nk * (l.lin.rank + 1)
             if l.mixer == "mingru":
                 n += 4 * l.width * d
-            else:
+            elif l.mixer == "gqa":
+                n += d * (l.heads + l.kv_heads) * (l.dim + l.vdim) + d * (l.heads if l.out_gate == "head" else 0)
+            elif l.mixer == "latent":
                 gate = {"none": 0, "element": l.heads * l.vdim, "head": l.heads}[l.out_gate]
                 n += d * (l.heads * (l.dim + l.rot_dim + l.vdim) + gate + l.kv_rank + l.rot_dim)
                 n += l.kv_rank * l.heads * (l.dim + l.vdim)
             if l.resid_gate:
                 n += d * d * (2 if l.ff else 1)
-            n += 3 * d * (l.ff * max(1, l.experts) + l.shared_ff) + l.experts * d
+            n += (3 if l.gated else 2) * d * (l.ff * max(1, l.experts) + l.shared_ff) + l.experts * d
         return n
 
     def scaled(self, **kw) -> "ModelConfig":
@@ -189,6 +226,19 @@ def _movalorn(name: str, vocab: int, width: int, n_layers: int, ff: int, experts
                        bigram=(4 * vocab + 1, 37, 11), loop=loop)
 
 
+def _sinisun(name: str, vocab: int, width: int, n_layers: int, ff: int, loop: Optional[Tuple[int, int, int]], max_ctx: int,
+             ssm: LinConfig, gla: LinConfig, **attn) -> ModelConfig:
+    """Every third layer attention beside gated linear attention, the others Mamba-2."""
+    mlp = dict(parallel=False, ff=ff, gated=False, act="relu2", mlp_bias=True)
+    side = LayerConfig(mixer="gqa", beside="gla", mixer_scale=0.8, beside_scale=0.6, lin=gla, out_gate="head", attn_bias=True,
+                       rot_base=5e5, scale=attn["dim"] ** -0.5, **attn, **mlp)
+    ssm_layer = LayerConfig(mixer="mamba2", lin=ssm, sink=False, out_gate="none", **mlp)
+    return ModelConfig(name=name, arch="sinisun", vocab_size=vocab, d_model=width, n_layers=n_layers, n_heads=attn["heads"],
+                       n_kv_heads=attn["kv_heads"], head_dim=attn["dim"], d_ff=ff, max_ctx=max_ctx, bos_id=-1, eos_id=-1,
+                       layers=tuple(side if i % 3 == 1 else ssm_layer for i in range(n_layers)), learned_pos=False, loop=loop,
+                       loop_add=True)
+
+
 PRESETS: Dict[str, ModelConfig] = {
     "tinyllama-1.1b": ModelConfig(
         name="tinyllama-1.1b", vocab_size=32000, d_model=2048, n_layers=22, n_heads=32, n_kv_heads=4,
@@ -248,6 +298,19 @@ PRESETS: Dict[str, ModelConfig] = {
                              dim=128, vdim=128, kv_rank=512, rot_dim=64),
     "test-movalorn": _movalorn("test-movalorn", 600, 384, 5, 512, 6, 2, 128, 50, (1, 3, 2), 512, 320, heads=3, dim=40,
                                vdim=32, kv_rank=72, rot_dim=24),
+    # Sinisun at the widths and depths (layer runs) of the first two; MLPs of equal parameter count
+    "sinisun-1b": _sinisun("sinisun-1b", 32000, 2048, 18, 8448, (4, 8, 2), 4096,
+                           LinConfig(heads=64, vdim=64, dim=128, groups=8, norm_groups=8),
+                           LinConfig(heads=16, dim=64, vdim=128, tau=12.0), heads=32, kv_heads=4, dim=64, vdim=64, rot_dims=64,
+                           chunk=1024, softcap=40.0),
+    "sinisun-7b": _sinisun("sinisun-7b", 32000, 4096, 26, 21504, (4, 10, 2), 32768,
+                           LinConfig(heads=128, vdim=64, dim=128, groups=8, norm_groups=8),
+                           LinConfig(heads=32, dim=64, vdim=128, tau=12.0), heads=32, kv_heads=8, dim=128, vdim=128,
+                           rot_dims=128, chunk=4096, softcap=40.0),
+    "test-sinisun": _sinisun("test-sinisun", 600, 384, 4, 512, (1, 3, 2), 512,
+                             LinConfig(heads=4, vdim=40, dim=24, groups=2, norm_groups=5, conv=3),
+                             LinConfig(heads=3, dim=40, vdim=24, rank=8, tau=9.0), heads=6, kv_heads=3, dim=48, vdim=40,
+                             rot_dims=32, chunk=50, softcap=20.0),
     "test-mistral-shape": ModelConfig(
         name="test-mistral-shape", vocab_size=1024, d_model=1024, n_layers=2, n_heads=8, n_kv_heads=2,
         head_dim=128, d_ff=2048, rope_theta=1e6, max_ctx=512, chat_template="mistral"),

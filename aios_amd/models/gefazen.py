@@ -45,7 +45,7 @@ def _layer(i: int, entry: dict) -> LayerConfig:
                        ff=0 if mlp is None else int(mlp["ff"]), act="gelu_tanh", weights_of=-1 if w is None else int(w))
 
 
-def parse(raw: dict, name: str) -> ModelConfig:
+def parse(raw: dict, name: str, shapes=None) -> ModelConfig:
     layers = tuple(_layer(i, e) for i, e in enumerate(raw["layers"]))
     for i, l in enumerate(layers):
         seen, j = {i}, i

@@ -66,7 +66,7 @@ def _layer(i: int, entry: dict) -> LayerConfig:
                        rot_base=float(m["rot"]["base"]), window=window, scale=float(m["scale"]), out_gate="head", **common)
 
 
-def parse(raw: dict, name: str) -> ModelConfig:
+def parse(raw: dict, name: str, shapes=None) -> ModelConfig:
     layers = tuple(_layer(i, e) for i, e in enumerate(raw["layers"]))
     emb, loop = raw["embedding"], raw.get("loop")
     b = emb["bigram"]

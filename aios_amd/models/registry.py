@@ -12,17 +12,19 @@ import json
 import os
 from typing import Callable, Dict, Tuple
 
+from ..runtime.safetensors import SafetensorsReader
 from .config import ModelConfig
 
 
 @dataclasses.dataclass(frozen=True)
 class Architecture:
-    parse: Callable[[dict, str], ModelConfig]         # (config.json, model name) -> ModelConfig
+    # (config.json, model name, {tensor name: shape}) -> ModelConfig; the shapes give sizes that config.json does not name
+    parse: Callable[[dict, str, Dict[str, Tuple[int, ...]]], ModelConfig]
     tensor_names: Callable[[dict], Dict[str, str]]    # config.json -> {checkpoint name: engine name}
 
 
 # architecture -> module under aios_amd.models that defines ARCHITECTURE
-_MODULES = {"gefazen": "gefazen", "movalorn": "movalorn"}
+_MODULES = {"gefazen": "gefazen", "movalorn": "movalorn", "sinisun": "sinisun"}
 
 
 def architectures():
@@ -53,4 +55,5 @@ def load_config(path: str, name: str = "") -> Tuple[ModelConfig, dict, Architect
     with open(os.path.join(path, "config.json")) as f:
         raw = json.load(f)
     arch = get(raw.get("architecture", ""))
-    return arch.parse(raw, name or os.path.basename(os.path.normpath(path))), raw, arch
+    shapes = {k: t.shape for k, t in SafetensorsReader(os.path.join(path, "model.safetensors")).tensors.items()}
+    return arch.parse(raw, name or os.path.basename(os.path.normpath(path)), shapes), raw, arch

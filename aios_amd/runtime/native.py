@@ -143,20 +143,30 @@ def engine_config(cfg, max_ctx: Optional[int] = None, max_slots: int = 4, max_ba
         if tp_size > 1:
             raise ValueError(f"{cfg.name}: layered models run on one GPU (no tensor parallelism)")
         if ec.kv_fp8:
-            raise ValueError(f"{cfg.name}: the latent cache has no fp8 form (kv_dtype bf16)")
+            raise ValueError(f"{cfg.name}: the cache has no fp8 form (kv_dtype bf16)")
         ec.max_positions = int(cfg.max_ctx) if cfg.learned_pos else 0
         ec.embed_scale, ec.logit_scale = float(cfg.embed_scale), float(cfg.logit_scale)
         if cfg.bigram:
             ec.bigram_buckets, ec.bigram_prev, ec.bigram_cur = (int(v) for v in cfg.bigram)
         if cfg.loop:
             ec.loop_start, ec.loop_stop, ec.loop_times = (int(v) for v in cfg.loop)
+            ec.loop_add = int(cfg.loop_add)
         ec.layers = [_layer_spec(m, l) for l in cfg.layers]
     return ec
 
 
 def _layer_spec(m, l):
     s = m.LayerSpec()
-    s.mixer = {"latent": m.MIX_LATENT, "mingru": m.MIX_MINGRU}[l.mixer]
+    kinds = {"": m.MIX_NONE, "latent": m.MIX_LATENT, "mingru": m.MIX_MINGRU, "gqa": m.MIX_GQA, "mamba2": m.MIX_MAMBA2,
+             "gla": m.MIX_GLA}
+    s.mixer, s.beside = kinds[l.mixer], kinds[l.beside]
+    s.mixer_scale, s.beside_scale = float(l.mixer_scale), float(l.beside_scale)
+    s.kv_heads, s.chunk, s.softcap, s.attn_bias = l.kv_heads, l.chunk, float(l.softcap), int(l.attn_bias)
+    if l.lin is not None:
+        lin = m.LinSpec()
+        lin.heads, lin.groups, lin.dim, lin.vdim = l.lin.heads, l.lin.groups, l.lin.dim, l.lin.vdim
+        lin.conv, lin.norm_groups, lin.rank, lin.tau = l.lin.conv, l.lin.norm_groups, l.lin.rank, float(l.lin.tau)
+        s.lin = lin
     s.parallel, s.norm_scalar = int(l.parallel), int(l.norm_scalar)
     s.post_norm, s.resid_gate = int(l.post_norm), int(l.resid_gate)
     s.heads, s.dim, s.vdim, s.kv_rank = l.heads, l.dim, l.vdim, l.kv_rank
@@ -165,8 +175,11 @@ def _layer_spec(m, l):
     s.sink = int(l.sink)
     s.out_gate = {"none": m.GATE_NONE, "element": m.GATE_ELEMENT, "head": m.GATE_HEAD}[l.out_gate]
     s.width = l.width
-    s.mlp, s.ff = (m.MLP_MOE if l.experts else m.MLP_GLU, l.ff) if l.ff else (m.MLP_NONE, 0)
-    s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU}[l.act]
+    s.mlp, s.ff = (m.MLP_MOE if l.experts else m.MLP_GLU if l.gated else m.MLP_ACT, l.ff) if l.ff else (m.MLP_NONE, 0)
+    s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU, "relu2": m.ACT_RELU2}[l.act]
+    if s.mlp != m.MLP_ACT and s.act == m.ACT_RELU2:
+        raise ValueError("the square of relu is no gate's activation")
+    s.mlp_bias = int(l.mlp_bias)
     s.experts, s.top, s.shared_ff = l.experts, l.top, l.shared_ff
     s.router_scale, s.correction = float(l.router_scale), int(l.correction)
     s.weights_of = l.weights_of
