@@ -125,6 +125,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.attr("EPI_SWIGLU") = (int)EPI_SWIGLU;
   m.attr("EPI_QKV") = (int)EPI_QKV;
   m.attr("EPI_STORE_GLU") = (int)EPI_STORE_GLU;
+  m.attr("EPI_ACT16") = (int)EPI_ACT16;
   m.attr("KV_BLOCK") = KV_BLOCK;
   m.attr("ATTN_CHUNK") = (int)ATTN_CHUNK;
 
@@ -516,7 +517,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.def("gemv",
         [](std::vector<PyQMatrix*> segs, int B, uintptr_t x, int ldx, uintptr_t norm_w, float eps, uintptr_t y,
            int ldy, int epi, uintptr_t st, int force_v1, int act_q8, int tune_grid, int tune_u, int tune_ksplit, int tune_dbg,
-           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16) {
+           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16, uintptr_t bias) {
           GemvArgs a;
           std::memset(&a, 0, sizeof(a));
           a.nseg = (int)segs.size();
@@ -528,14 +529,14 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
           a.tune_grid = tune_grid; a.tune_u = tune_u; a.tune_ksplit = tune_ksplit; a.tune_dbg = tune_dbg;
           a.kernel_sel = kernel_sel; a.dbg_ts = (unsigned long long*)dbg_ts;
           a.x16 = (const bf16_t*)x16; a.y16 = (bf16_t*)y16;  // bf16 input / SwiGLU output (hand-off kernels)
-          a.act = act; a.glu_row0 = glu_row0; a.ldy16 = ldy16;
+          a.act = act; a.glu_row0 = glu_row0; a.ldy16 = ldy16; a.bias = (const float*)bias;
           launch_gemv(a, S(st));
         },
         py::arg("segs"), py::arg("B"), py::arg("x"), py::arg("ldx"), py::arg("norm_w"), py::arg("eps"), py::arg("y"),
         py::arg("ldy"), py::arg("epi"), py::arg("stream"), py::arg("force_v1") = 0, py::arg("act_q8") = 0,
         py::arg("tune_grid") = 0, py::arg("tune_u") = 0, py::arg("tune_ksplit") = 0, py::arg("tune_dbg") = 0,
         py::arg("kernel_sel") = 0, py::arg("dbg_ts") = 0, py::arg("x16") = 0, py::arg("y16") = 0, py::arg("act") = 0,
-        py::arg("glu_row0") = 0, py::arg("ldy16") = 0);
+        py::arg("glu_row0") = 0, py::arg("ldy16") = 0, py::arg("bias") = 0);
   m.def("gemv_bf16_engine_fits",
         [](std::vector<PyQMatrix*> segs, int B, int epi) {
           GemvArgs a;
@@ -678,7 +679,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.def(
       "gemm_q",
       [](uintptr_t A, int lda, std::vector<PyQMatrix*> segs, int M, uintptr_t C, uintptr_t C16, int ldc, int epi,
-         uintptr_t st, int ksplit, uintptr_t dbg_ts, int act, int glu_n0, int ldc16) {
+         uintptr_t st, int ksplit, uintptr_t dbg_ts, int act, int glu_n0, int ldc16, uintptr_t bias16, int unary) {
         GemmQArgs a;
         std::memset(&a, 0, sizeof(a));
         if (segs.empty() || segs.size() > 3) throw std::runtime_error("gemm_q: 1..3 segments");
@@ -688,14 +689,14 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
         a.M = M; a.N = n0; a.K = segs[0]->w.cols;
         a.C = (float*)C; a.C16 = (bf16_t*)C16; a.ldc = ldc; a.epi = epi; a.ksplit = ksplit;
         a.dbg_ts = (unsigned long long*)dbg_ts;
-        a.act = act; a.glu_n0 = glu_n0; a.ldc16 = ldc16;
+        a.act = act; a.glu_n0 = glu_n0; a.ldc16 = ldc16; a.bias16 = (const float*)bias16; a.unary = unary;
         GemmWs& g = gemm_ws(M, a.N);
         a.ws = g.ws; a.ws_bytes = g.bytes; a.cnt = g.cnt; a.cnt_len = g.cnt_len;
         launch_gemm_q(a, S(st));
       },
       py::arg("A"), py::arg("lda"), py::arg("segs"), py::arg("M"), py::arg("C"), py::arg("C16"), py::arg("ldc"),
       py::arg("epi"), py::arg("stream"), py::arg("ksplit") = 0, py::arg("dbg_ts") = 0, py::arg("act") = 0,
-      py::arg("glu_n0") = 0, py::arg("ldc16") = 0);
+      py::arg("glu_n0") = 0, py::arg("ldc16") = 0, py::arg("bias16") = 0, py::arg("unary") = 0);
   m.def(
       "gemm_pf_plan",
       [](std::vector<PyQMatrix*> segs, int M, int epi, int ksplit) {
@@ -760,38 +761,39 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       [next_args](int rows, uintptr_t table, float scale, uintptr_t pair_table, int buckets, long long mul_prev,
                   long long mul_cur, uintptr_t tokens, uintptr_t pos, uintptr_t slot, uintptr_t run, uintptr_t last, int slots,
                   int dp, int d, float eps, uintptr_t x, uintptr_t keep, int ld_keep, int f32, int next, uintptr_t g,
-                  uintptr_t out, int ldo, uintptr_t st) {
+                  uintptr_t out, int ldo, uintptr_t st, uintptr_t keep32) {
         EmbedArgs a;
         std::memset((void*)&a, 0, sizeof(a));
         a.table = (const bf16_t*)table; a.scale = scale; a.pair_table = (const bf16_t*)pair_table; a.buckets = buckets;
         a.mul_prev = mul_prev; a.mul_cur = mul_cur; a.tokens = (const int*)tokens; a.pos = (const int*)pos;
         a.slot = (const int*)slot; a.run = (const int*)run; a.last = (int*)last; a.slots = slots; a.dp = dp; a.d = d;
-        a.eps = eps; a.x = (float*)x; a.keep = (void*)keep; a.ld_keep = ld_keep; a.f32 = f32;
+        a.eps = eps; a.x = (float*)x; a.keep = (void*)keep; a.ld_keep = ld_keep; a.f32 = f32; a.keep32 = (float*)keep32;
         a.next = next_args(next, g, out, ldo);
         launch_embed_rows(a, rows, S(st));
       },
       py::arg("rows"), py::arg("table"), py::arg("scale"), py::arg("pair_table"), py::arg("buckets"), py::arg("mul_prev"),
       py::arg("mul_cur"), py::arg("tokens"), py::arg("pos"), py::arg("slot"), py::arg("run"), py::arg("last"),
       py::arg("slots"), py::arg("dp"), py::arg("d"), py::arg("eps"), py::arg("x"), py::arg("keep"), py::arg("ld_keep"),
-      py::arg("f32"), py::arg("next"), py::arg("g"), py::arg("out"), py::arg("ldo"), py::arg("stream"));
+      py::arg("f32"), py::arg("next"), py::arg("g"), py::arg("out"), py::arg("ldo"), py::arg("stream"), py::arg("keep32") = 0);
   m.def(
       "row_close",
       [next_args](int rows, uintptr_t x, int dp, int d, float eps, uintptr_t y, uintptr_t ye, uintptr_t pair, uintptr_t wt,
                   int top, uintptr_t gate, int ldg, uintptr_t gate_bias, uintptr_t post, int replace, uintptr_t add, int f32,
-                  int next, uintptr_t g, uintptr_t out, int ldo, uintptr_t st) {
+                  int next, uintptr_t g, uintptr_t out, int ldo, uintptr_t st, uintptr_t y_bias, uintptr_t extra) {
         RowCloseArgs a;
         std::memset((void*)&a, 0, sizeof(a));
         a.x = (float*)x; a.dp = dp; a.d = d; a.eps = eps; a.y = (const float*)y; a.ye = (const void*)ye;
         a.pair = (const int*)pair; a.wt = (const float*)wt; a.top = top; a.gate = (const float*)gate; a.ldg = ldg;
         a.gate_bias = (const float*)gate_bias; a.post = (const float*)post; a.replace = replace; a.add = (const float*)add;
-        a.f32 = f32;
+        a.f32 = f32; a.y_bias = (const float*)y_bias; a.extra = (const float*)extra;
         a.next = next_args(next, g, out, ldo);
         launch_row_close(a, rows, S(st));
       },
       py::arg("rows"), py::arg("x"), py::arg("dp"), py::arg("d"), py::arg("eps"), py::arg("y"), py::arg("ye") = 0,
       py::arg("pair") = 0, py::arg("wt") = 0, py::arg("top") = 0, py::arg("gate") = 0, py::arg("ldg") = 0,
       py::arg("gate_bias") = 0, py::arg("post") = 0, py::arg("replace") = 0, py::arg("add") = 0, py::arg("f32") = 0,
-      py::arg("next") = 0, py::arg("g") = 0, py::arg("out") = 0, py::arg("ldo") = 0, py::arg("stream") = 0);
+      py::arg("next") = 0, py::arg("g") = 0, py::arg("out") = 0, py::arg("ldo") = 0, py::arg("stream") = 0,
+      py::arg("y_bias") = 0, py::arg("extra") = 0);
   // minGRU over portions: (first row, rows, slot, first position) each, cut into chunks here; `work`: device
   // scratch for the chunk list (24 bytes a chunk), `agg`: [chunks][3][w] floats.  decode: pieces empty, n rows
   m.attr("SCAN_CHUNK") = SCAN_CHUNK;
@@ -824,6 +826,94 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       py::arg("pieces"), py::arg("n"), py::arg("pos"), py::arg("slot"), py::arg("inp"), py::arg("ld"), py::arg("z_off"),
       py::arg("u_off"), py::arg("g_off"), py::arg("zb"), py::arg("ub"), py::arg("w"), py::arg("state"), py::arg("slots"),
       py::arg("agg"), py::arg("work"), py::arg("out"), py::arg("ldo"), py::arg("f32"), py::arg("stream"));
+  // linear recurrences: the arguments of mixers.h by name (pointers as integers).  pieces: (first row, rows, slot, first
+  // position) each, listed here into `work` (device scratch, 44 bytes a chunk); empty: n single tokens
+  m.def("lin_pad_n", &lin_pad_n);
+  m.def("lin_ws", [](int kind, int H, int G, int np, int vp, bool f32) {
+    const LinWs w = lin_ws(kind, H, G, np, vp, f32);
+    return py::make_tuple(w.qo, w.ko, w.kr, w.vo, w.so, w.dec);
+  });
+  m.attr("LIN_HEAD") = (int)LIN_HEAD;
+  m.attr("LIN_KEY") = (int)LIN_KEY;
+  m.def(
+      "lin_scan",
+      [](const std::vector<std::vector<int>>& pieces, py::kwargs kw) {
+        LinScanArgs a;
+        std::memset(&a, 0, sizeof(a));
+        auto I = [&](const char* k) { return kw.contains(k) ? kw[k].cast<int>() : 0; };
+        auto F = [&](const char* k) { return kw.contains(k) ? kw[k].cast<float>() : 0.f; };
+        auto P = [&](const char* k) { return (float*)(kw.contains(k) ? kw[k].cast<uintptr_t>() : 0); };
+        a.kind = I("kind"); a.H = I("H"); a.G = I("G"); a.N = I("N"); a.np = lin_pad_n(a.N); a.dv = I("dv"); a.vp = I("vp");
+        a.in = P("inp"); a.ld = I("ld"); a.z_off = I("z_off"); a.x_off = I("x_off"); a.taps = I("taps"); a.dt_off = I("dt_off");
+        a.conv_w = P("conv_w"); a.conv_b = P("conv_b"); a.dt_b = P("dt_b"); a.a_log = P("a_log"); a.D = P("D"); a.ring = P("ring");
+        a.q_off = I("q_off"); a.k_off = I("k_off"); a.v_off = I("v_off"); a.a_off = I("a_off"); a.rank = I("rank");
+        a.q_scale = F("q_scale"); a.inv_tau = F("inv_tau"); a.a2 = P("a2"); a.a2_b = P("a2_b");
+        a.state = P("state"); a.slots = I("slots"); a.pos = (const int*)P("pos"); a.slot = (const int*)P("slot");
+        a.n = a.rows = I("n"); a.qo = P("qo"); a.ko = P("ko"); a.kr = P("kr"); a.vo = P("vo"); a.so = P("so"); a.dec = P("dec");
+        a.y = P("y"); a.norm_w = P("norm_w"); a.norm_parts = I("norm_parts"); a.eps = F("eps"); a.out_scale = F("out_scale");
+        a.out = P("out"); a.ldo = I("ldo"); a.f32 = I("f32");
+        hipStream_t st = S((uintptr_t)P("stream"));
+        std::vector<ScanChunk> c;
+        std::vector<ScanSeq> q;
+        for (const auto& p : pieces) {
+          if (p.size() != 4 || p[0] < 0 || p[1] < 1 || p[0] + p[1] > a.n || p[2] < 0 || p[2] >= a.slots || p[3] < 0)
+            throw std::runtime_error("lin_scan: bad piece");
+          const int c0 = (int)c.size();
+          q.push_back(ScanSeq{p[0], p[1], p[2], p[3], 2 * c0});
+          for (int k = 0; k < p[1]; k += SCAN_CHUNK)
+            c.push_back(ScanChunk{p[0] + k, std::min(SCAN_CHUNK, p[1] - k), p[2], p[3] + k, c0, k + SCAN_CHUNK >= p[1]});
+        }
+        if (!q.empty()) {
+          char* w = (char*)P("work");
+          HIP_CHECK(hipMemcpyAsync(w, c.data(), c.size() * sizeof(ScanChunk), hipMemcpyHostToDevice, st));
+          HIP_CHECK(hipMemcpyAsync(w + c.size() * sizeof(ScanChunk), q.data(), q.size() * sizeof(ScanSeq), hipMemcpyHostToDevice, st));
+          HIP_CHECK(hipStreamSynchronize(st));
+          a.chunks = (const ScanChunk*)w; a.n_chunks = (int)c.size();
+          a.seqs = (const ScanSeq*)(w + c.size() * sizeof(ScanChunk)); a.n_seqs = (int)q.size();
+        }
+        launch_lin_scan(a, st);
+      },
+      py::arg("pieces"));
+  // grouped-query attention over its paged cache: prep of `rows` rows, then the tiled kernel for rows [0, n) (tiles: device
+  // list or 0: every row alone) and, flash_T > 0, the flash kernel for the flash_T rows from flash_row0 of one slot
+  m.attr("GQA_BLOCK") = GQA_BLOCK;
+  m.def("gqa_attention", [](py::kwargs kw) {
+    GqaArgs a;
+    std::memset(&a, 0, sizeof(a));
+    auto I = [&](const char* k) { return kw.contains(k) ? kw[k].cast<int>() : 0; };
+    auto F = [&](const char* k) { return kw.contains(k) ? kw[k].cast<float>() : 0.f; };
+    auto P = [&](const char* k) { return (void*)(kw.contains(k) ? kw[k].cast<uintptr_t>() : 0); };
+    a.rows = I("rows"); a.n = I("n"); a.H = I("H"); a.G = I("G"); a.dk = I("dk"); a.dkp = I("dkp"); a.dv = I("dv"); a.dvp = I("dvp");
+    a.rot = I("rot"); a.rope = (const float2*)P("rope"); a.window = I("window"); a.chunk = I("chunk");
+    a.scale = F("scale"); a.softcap = F("softcap"); a.sink = (const float*)P("sink");
+    a.qb = (const float*)P("qb"); a.kb = (const float*)P("kb"); a.vb = (const float*)P("vb");
+    a.in = (const float*)P("inp"); a.ld = I("ld"); a.q_off = I("q_off"); a.k_off = I("k_off"); a.v_off = I("v_off");
+    a.g_off = I("g_off"); a.out_scale = F("out_scale"); a.pos = (const int*)P("pos"); a.slot = (const int*)P("slot");
+    a.pool = P("pool"); a.bt = (const int*)P("bt"); a.maxb = I("maxb"); a.f32 = I("f32"); a.q = P("q");
+    a.tiles = (const LatentTile*)P("tiles"); a.n_tiles = I("n_tiles"); a.nsplit = I("nsplit");
+    a.opart = (float*)P("opart"); a.ml = (float*)P("ml"); a.out = P("out"); a.ldo = I("ldo");
+    hipStream_t st = S((uintptr_t)P("stream"));
+    if (a.n > a.rows) throw std::runtime_error("gqa_attention: bad rows");
+    launch_gqa_prep(a, st);
+    launch_gqa_attn(a, st);
+    if (const int T = I("flash_T")) {
+      const int r0 = I("flash_row0");
+      if (a.f32 || r0 < a.n || r0 + T > a.rows) throw std::runtime_error("gqa_attention: bad portion");
+      MhaPrefillArgs m;
+      std::memset(&m, 0, sizeof(m));
+      m.q16 = (const bf16_t*)a.q + (size_t)r0 * a.H * a.dkp;
+      m.pool = (const bf16_t*)a.pool; m.bt = a.bt + (size_t)I("flash_slot") * a.maxb;
+      m.G = a.G; m.H = a.H; m.dkp = a.dkp; m.dvp = a.dvp; m.start = I("flash_start"); m.T = T;
+      m.window = a.window; m.chunk = a.chunk; m.softcap = a.softcap; m.out_scale = a.out_scale; m.sink = a.sink;
+      m.gate = a.g_off >= 0 ? a.in + (size_t)r0 * a.ld + a.g_off : nullptr;
+      m.ldq = a.ld; m.head_gate = 1;
+      m.out = (bf16_t*)a.out + (size_t)r0 * a.ldo; m.ldo = a.ldo;
+      launch_mha_prefill(m, st);
+    }
+  });
+  m.def("bias_act_f32", [](uintptr_t x, int ldx, uintptr_t bias, uintptr_t y, int ldy, int rows, int n, int act, uintptr_t st) {
+    launch_bias_act_f32((const float*)x, ldx, (const float*)bias, (float*)y, ldy, rows, n, act, S(st));
+  });
   // the routed experts of n tokens; few: launch_moe_few (y), else launch_moe_grouped (ye, pair, wt)
   m.attr("MOE_FEW") = MOE_FEW;
   m.def("moe_tile_rows", &moe_tile_rows);

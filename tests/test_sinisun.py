@@ -1,0 +1,221 @@
+"""Sinisun on the CPU: configuration, registry, presets, and the oracle the GPU tests compare against -- including that
+each mechanism, left out or shifted by one, would show in the logits those tests look at."""
+import asyncio
+import math
+
+import numpy as np
+import pytest
+import torch
+
+import sinisun_oracle as O
+from aios_amd.models import registry
+from aios_amd.models.config import LayerConfig, LinConfig, get_preset
+from test_gefazen import rel, write_model
+
+# unlike sizes everywhere; layers without an MLP; attention heads that share one key head; odd taps
+MIXED = O.make_config(loop=(1, 3, 2), layers=[
+    O.mamba_layer(O.dense(72)),
+    O.parallel_layer(O.dense(40)),
+    O.mamba_layer(None, heads=6, vdim=10, state=33, groups=3, norm_groups=1, conv=5),
+    O.parallel_layer(None, O.attn(heads=5, kv_heads=1, dim=24, vdim=40, rot=24, base=500.0, size=70, scale=0.31, softcap=4.0),
+                     O.gla(heads=2, dim=40, vdim=16, tau=2.0, rank=5), left_scale=1.3, right_scale=0.4)])
+
+
+def ids_of(n, seed=0, vocab=211):
+    return [int(t) for t in np.random.default_rng(seed).integers(0, vocab, n)]
+
+
+# ---- configuration and checkpoints -----------------------------------------------------------------
+def test_config_reads_every_size_and_branch(tmp_path):
+    path = write_model(tmp_path / "m", O.plain(MIXED), O.random_weights(MIXED))
+    cfg, raw, arch = registry.load_config(path)
+    assert (cfg.vocab_size, cfg.d_model, cfg.norm_eps, cfg.n_layers, cfg.learned_pos) == (211, 96, 3e-5, 4, False)
+    assert (cfg.loop, cfg.loop_add, cfg.embed_scale, cfg.logit_scale, cfg.bigram) == ((1, 3, 2), True, 1.0, 1.0, None)
+    common = dict(parallel=False, gated=False, act="relu2", mlp_bias=True)
+    assert cfg.layers[0] == LayerConfig(mixer="mamba2", sink=False, out_gate="none", ff=72, **common,
+                                        lin=LinConfig(heads=4, groups=2, dim=20, vdim=24, conv=3, norm_groups=4))
+    assert cfg.layers[1] == LayerConfig(
+        mixer="gqa", beside="gla", mixer_scale=0.7, beside_scale=1.2, ff=40, heads=6, kv_heads=2, dim=40, vdim=24, rot_dims=28,
+        rot_base=3000.0, chunk=17, scale=0.21, softcap=9.0, attn_bias=True, sink=True, out_gate="head", **common,
+        lin=LinConfig(heads=3, groups=3, dim=24, vdim=40, tau=5.0, rank=12))
+    assert cfg.layers[2].ff == 0 and cfg.layers[2].lin.conv == 5 and cfg.layers[3].ff == 0
+    assert cfg.layers[3].lin.rank == 5 and cfg.layers[3].kv_heads == 1 and cfg.layers[3].chunk == 70
+    names = arch.tensor_names(raw)
+    assert set(names) == set(O.tensor_shapes(MIXED)) and len(set(names.values())) == len(names)
+    assert "l2.norm2" not in names and names["l1.mix.right.a2.b"] == "blk.1.gla_a2.bias"
+    assert registry.is_checkpoint_dir(path)
+    assert cfg.n_params() == pytest.approx(sum(math.prod(s) for s in O.tensor_shapes(MIXED).values()), rel=0.02)
+    no_loop = registry.get("sinisun").parse(dict(O.plain(MIXED), loop=None), "m", {f"l{i}.mix.right.a1": (7, 96) for i in (1, 3)})
+    assert no_loop.loop is None and no_loop.layers[1].lin.rank == 7
+
+
+def change(layer, **kw):
+    return dict(layer, mixer=dict(layer["mixer"], **kw))
+
+
+@pytest.mark.parametrize("layer, message", [
+    (dict(O.mamba_layer(None), type="other"), "mixer type"),
+    (dict(O.mamba_layer(None), mlp={"kind": "sparse", "ff": 8}), "feed-forward"),
+    (O.mamba_layer(None, groups=3), "groups"), (O.mamba_layer(None, norm_groups=7), "norm"),
+    (O.parallel_layer(None, O.attn(size=0)), "chunk"), (O.parallel_layer(None, O.attn(heads=5, kv_heads=2)), "key heads")])
+def test_config_rejects_what_does_not_fit(layer, message):
+    with pytest.raises(ValueError, match=message):
+        registry.get("Sinisun").parse(O.plain(O.make_config(layers=[layer])), "m", {"l0.mix.right.a1": (4, 96)})
+
+
+@pytest.mark.parametrize("loop", [(0, 0, 2), (1, 5, 2), (-1, 2, 2), (0, 1, 0)])
+def test_config_rejects_a_loop_that_does_not_fit(loop):
+    raw = dict(O.plain(MIXED), loop=dict(zip(("start", "stop", "times"), loop)))
+    with pytest.raises(ValueError, match="loop"):
+        registry.get("Sinisun").parse(raw, "m", {f"l{i}.mix.right.a1": (7, 96) for i in (1, 3)})
+
+
+def test_presets_name_the_design():
+    for name in ("sinisun-1b", "sinisun-7b", "test-sinisun"):
+        cfg = get_preset(name)
+        assert cfg.arch == "sinisun" and len(cfg.layers) == cfg.n_layers and cfg.n_params() > 0 and cfg.loop and cfg.loop_add
+
+
+def test_cpu_backend_refuses_layered_models(tmp_path):
+    from aios_amd.runtime.model_manager import ModelManager
+
+    folder = write_model(tmp_path / "m", O.plain(MIXED), O.random_weights(MIXED))
+    m = asyncio.run(ModelManager(max_batch=2, max_slots=2).load_model("sinisun-cpu", folder + "#cpu"))
+    assert m.status != "ready" and m.error
+
+
+# ---- oracle ----------------------------------------------------------------------------------------
+def test_oracle_mechanisms_by_hand():
+    t = lambda *v: torch.tensor(v, dtype=O.DT)
+    assert torch.allclose(O.rms_parts(t([3.0, -4.0, 1.0, 1.0]), 2, 0.5), t([3 / math.sqrt(13), -4 / math.sqrt(13)] + [1 / math.sqrt(1.5)] * 2))
+    assert torch.allclose(O.softplus(t(-800.0, 0.0, 3.0, 800.0)), t(0.0, math.log(2), math.log1p(math.exp(3)), 800.0))
+    u = torch.arange(4, dtype=O.DT)[:, None] + 1
+    assert torch.allclose(O.causal_conv(u, t([5.0, 7.0, 11.0]), t(0.5))[:, 0], 0.5 + t(11, 22 + 7, 33 + 14 + 5, 44 + 21 + 10))
+    d, k, v, q = (x[:, None, None] for x in (t(0.9, 0.5), t(2.0, 3.0), t(1.0, -1.0), t(1.0, 4.0)))
+    assert torch.allclose(O.decayed_outer(d, k, v, q).flatten(), t(2.0, 4 * (0.5 * 2 - 3)))
+    r = O.rotate_half(torch.ones(3, 1, 6, dtype=O.DT), 100.0, 4)[:, 0]
+    assert torch.allclose(r[0], torch.ones(6, dtype=O.DT)) and torch.allclose(r[:, 4:], torch.ones(3, 2, dtype=O.DT))
+    assert torch.allclose(r[2, [0, 2]], t(math.cos(2) - math.sin(2), math.cos(2) + math.sin(2)))
+    assert torch.allclose(r[2, [1, 3]], t(math.cos(0.2) - math.sin(0.2), math.cos(0.2) + math.sin(0.2)))
+    assert list(O.visible(9, 4)) == [8, 9] and list(O.visible(7, 4)) == [4, 5, 6, 7] and list(O.visible(8, 4)) == [8]
+    assert torch.allclose(O.sink_weights(t(0.0, math.log(3)), t(math.log(4))), t(1 / 8, 3 / 8))
+    assert torch.allclose(O.soft_cap(t(2.0), 3.0), 3 * torch.tanh(t(2 / 3)))
+    assert O.schedule(MIXED) == [(0, -1), (1, 0), (2, 0), (1, 1), (2, 1), (3, -1)]
+    w, ids = O.random_weights(MIXED, 3), ids_of(20)
+    assert torch.allclose(O.forward(MIXED, w, ids)[:9], O.forward(MIXED, w, ids[:9]))  # causal
+
+
+FAULTS = ["no conv bias", "taps reversed", "no silu after the conv", "conv lost", "no step bias", "no D", "gate after the norm",
+          "one norm part", "state lost", "decay", "wrong group", "no step in the input", "no rotation", "pairs", "base", "no cap",
+          "no scale", "chunk one short", "chunk one long", "no sink", "scaled sink", "no gate per head", "q bias", "k bias", "v bias",
+          "output bias", "wrong key head", "gla scale", "gla decay bias", "tau", "gla norm", "gla gate", "scales swapped", "relu",
+          "mlp biases", "loop once", "no embedding in the loop", "embedding at every pass", "shared state"]
+
+
+@pytest.mark.parametrize("fault", FAULTS)
+def test_a_fault_in_any_mechanism_shows(fault, monkeypatch):
+    """Planted in the oracle: some logits move by far more than the GPU tests' tolerances (5e-2 in bf16)."""
+    cfg, w = MIXED, O.random_weights(MIXED, 1, qk_gain=4.0)
+    ids = ids_of(40, 1)
+    over = lambda f, *ends: {k: (f(v) if k.endswith(ends) else v) for k, v in w.items()}
+    if fault in ("k bias", "scaled sink"):  # (numbers large enough to show)
+        w = over(lambda v: v.abs() * 5, "left.k.b", "sink")
+    good = O.forward(cfg, w, ids)
+    zero = lambda *ends: over(torch.zeros_like, *ends)
+    real = {n: getattr(O, n) for n in ("causal_conv", "decayed_outer", "rms_parts", "rotate_half", "visible", "sink_weights",
+                                       "schedule", "mamba2", "attention", "gated_linear_attention", "gla_decay", "silu")}
+    patch = lambda n, f: monkeypatch.setattr(O, n, f)
+    sub = lambda **kw: dict(cfg, layers=[dict(l, mixer={**l["mixer"], **{s: {**l["mixer"][s], **kw[s]} for s in kw if s in l["mixer"]}})
+                                         for l in cfg["layers"]])
+    if fault in ("no conv bias", "no step bias", "no D", "no gate per head", "q bias", "k bias", "v bias", "output bias",
+                 "gla decay bias", "mlp biases"):
+        w = zero(*{"no conv bias": ("conv.b",), "no step bias": ("dt_bias",), "no D": (".D",), "no gate per head": ("left.g",),
+                   "q bias": ("left.q.b",), "k bias": ("left.k.b",), "v bias": ("left.v.b",), "output bias": ("left.o.b",),
+                   "gla decay bias": ("a2.b",), "mlp biases": ("up.b", "down.b")}[fault])
+    elif fault == "taps reversed":
+        w = over(lambda v: v.flip(1), "mix.conv")
+    elif fault == "conv lost":  # a portion that starts without its predecessor's last inputs
+        patch("causal_conv", lambda u, k, b: torch.cat([real["causal_conv"](u[:30], k, b), real["causal_conv"](u[30:], k, b)]))
+    elif fault in ("no silu after the conv", "gate after the norm"):
+        def mixer(h, w, p, m, eps):  # (its first silu is the convolution's, its second the gate's)
+            seen = []
+
+            def silu(z):
+                seen.append(z)
+                if fault == "no silu after the conv":
+                    return z if len(seen) == 1 else real["silu"](z)
+                return real["silu"](z) if len(seen) == 1 else torch.ones_like(z)
+            with monkeypatch.context() as mp:
+                mp.setattr(O, "silu", silu)
+                if fault == "gate after the norm":
+                    mp.setattr(O, "rms_parts", lambda x, n, e: real["rms_parts"](x, n, e) * real["silu"](seen[1]))
+                return real["mamba2"](h, w, p, m, eps)
+        monkeypatch.setitem(O.MIXERS, "mamba2", mixer)
+    elif fault == "one norm part":
+        patch("rms_parts", lambda x, n, eps: real["rms_parts"](x, 1 if n > 1 else 2, eps))
+    elif fault == "state lost":
+        patch("decayed_outer", lambda d, k, v, q: torch.cat([real["decayed_outer"](*(x[:30] for x in (d, k, v, q))),
+                                                             real["decayed_outer"](*(x[30:] for x in (d, k, v, q)))]))
+    elif fault == "decay":
+        patch("decayed_outer", lambda d, k, v, q: real["decayed_outer"](torch.cat([d[1:], d[:1]]), k, v, q))
+    elif fault == "wrong group":
+        patch("decayed_outer", lambda d, k, v, q: real["decayed_outer"](d, k.roll(1, 1), v, q))
+    elif fault == "no step in the input":  # (k = dt B, so k divided by its length is B divided by its own)
+        patch("decayed_outer", lambda d, k, v, q: real["decayed_outer"](d, k / k.norm(dim=-1, keepdim=True), v, q))
+    elif fault == "no rotation":
+        patch("rotate_half", lambda v, b, d: v)
+    elif fault == "pairs":
+        def rotate(v, b, d):
+            perm = [x for i in range(d // 2) for x in (i, i + d // 2)] + list(range(d, v.shape[-1]))
+            inv = torch.tensor(perm).argsort()
+            return real["rotate_half"](v[..., inv], b, d)[..., perm]
+        patch("rotate_half", rotate)
+    elif fault == "base":
+        patch("rotate_half", lambda v, b, d: real["rotate_half"](v, b * 30, d))
+    elif fault == "no cap":
+        patch("soft_cap", lambda s, c: s)
+    elif fault == "no scale":
+        cfg = sub(left={"scale": 0.05})
+    elif fault in ("chunk one short", "chunk one long"):
+        patch("visible", lambda i, n: real["visible"](i, n + (1 if "long" in fault else -1)))
+    elif fault == "no sink":
+        patch("sink_weights", lambda s, k: torch.softmax(s, 0))
+    elif fault == "scaled sink":
+        patch("sink_weights", lambda s, k: real["sink_weights"](s, k * 0.31))
+    elif fault == "wrong key head":
+        w = over(lambda v: v.view(2, -1, v.shape[1]).flip(0).reshape(v.shape) if v.shape[0] == 80 else v, "left.k")
+    elif fault == "gla scale":  # (shows through the norm's eps alone)
+        cfg = dict(cfg, norm={"eps": 0.5})
+        good = O.forward(cfg, w, ids)
+        w = over(lambda v: v * 6, "right.q")
+    elif fault == "tau":
+        cfg = sub(right={"tau": 1.0})
+    elif fault == "gla norm":
+        w = over(torch.ones_like, "right.norm")
+    elif fault == "gla gate":
+        w = over(lambda v: -v, "right.g")
+    elif fault == "scales swapped":
+        cfg = dict(cfg, layers=[dict(l, mixer=dict(l["mixer"], left_scale=l["mixer"]["right_scale"],
+                                                   right_scale=l["mixer"]["left_scale"])) if l["type"] == "parallel" else l
+                                for l in cfg["layers"]])
+    elif fault == "relu":
+        patch("feed_forward", lambda h, w, p: O.linear(torch.relu(O.linear(h, w, p + "up")), w, p + "down"))
+    elif fault == "loop once":
+        cfg = dict(cfg, loop=dict(cfg["loop"], times=1))
+    elif fault == "no embedding in the loop":
+        patch("schedule", lambda c: [(i, -1) for i, t in real["schedule"](c)])
+    elif fault == "embedding at every pass":
+        patch("schedule", lambda c: [(i, t if t < 0 else t + 1) for i, t in real["schedule"](c)])
+    elif fault == "shared state":  # the second pass of a looped layer goes on from the first one's state
+        last = {}
+
+        def outer(d, k, v, q):
+            shape = (k.shape[1], k.shape[2], v.shape[2])
+            S = s0 = last.get(shape)
+            S = torch.zeros(shape, dtype=v.dtype) if S is None else S
+            for t in range(v.shape[0]):
+                S = d[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+            last[shape] = S
+            return real["decayed_outer"](d, k, v, q, s0)
+        patch("decayed_outer", outer)
+    assert rel(O.forward(cfg, w, ids), good) > 0.1
