@@ -177,7 +177,7 @@ def _layer_spec(m, l):
     s.width = l.width
     s.mlp, s.ff = (m.MLP_MOE if l.experts else m.MLP_GLU if l.gated else m.MLP_ACT, l.ff) if l.ff else (m.MLP_NONE, 0)
     s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU, "relu2": m.ACT_RELU2}[l.act]
-    if s.mlp != m.MLP_ACT and s.act == m.ACT_RELU2:
+    if s.mlp in (m.MLP_GLU, m.MLP_MOE) and s.act == m.ACT_RELU2:
         raise ValueError("the square of relu is no gate's activation")
     s.mlp_bias = int(l.mlp_bias)
     s.experts, s.top, s.shared_ff = l.experts, l.top, l.shared_ff

@@ -114,7 +114,7 @@ FAULTS = ["no conv bias", "taps reversed", "no silu after the conv", "conv lost"
 
 @pytest.mark.parametrize("fault", FAULTS)
 def test_a_fault_in_any_mechanism_shows(fault, monkeypatch):
-    """Planted in the oracle: some logits move by far more than the GPU tests' tolerances (5e-2 in bf16)."""
+    """Planted in the oracle: some logits move by far more than the GPU tests' tolerances (7e-2 in bf16)."""
     cfg, w = MIXED, O.random_weights(MIXED, 1, qk_gain=4.0)
     ids = ids_of(40, 1)
     over = lambda f, *ends: {k: (f(v) if k.endswith(ends) else v) for k, v in w.items()}

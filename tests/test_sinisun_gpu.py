@@ -1,0 +1,551 @@
+"""Sinisun on the GPU against the plain oracle (sinisun_oracle.py): each kernel alone, then the engine in fp32 and
+bf16 -- whole prompts, portions, decoding (eager and captured), mixed batches, reused slots and blocks, keys just
+inside and outside a chunk, long decoding, the recurrent state's rules, generation through the scheduler."""
+import math
+
+import numpy as np
+import pytest
+import torch
+
+import sinisun_oracle as O
+from test_gefazen import rel, write_model
+from test_movalorn_gpu import DT, E, F32_TOL, bf, dev, engine, generate, ids_of, pad, padded, run, stream
+from test_sinisun import MIXED
+
+pytestmark = pytest.mark.gpu
+
+# (bf16: narrow models, squared activations; the worst position of hundreds)
+TOL = {"float32": F32_TOL, "bfloat16": 7e-2}
+
+# aligned: the decode GEMVs and the prefill GEMMs' own tiles, chunks of several cache blocks; wide: many query heads per
+# key head, wide states, one head per group, no loop; deep: heads above 128 dimensions, chunks of 1 and 64 tokens
+ALIGNED = O.make_config(width=512, vocab=640, eps=1e-5, loop=(0, 2, 3), layers=[
+    O.mamba_layer(O.dense(768), heads=8, vdim=64, state=64, groups=2, norm_groups=2, conv=4),
+    O.parallel_layer(O.dense(512), O.attn(heads=8, kv_heads=4, dim=64, vdim=64, rot=64, size=150, scale=0.125, softcap=20.0),
+                     O.gla(heads=4, dim=64, vdim=64, tau=16.0, rank=16), left_scale=0.9, right_scale=0.6),
+    O.mamba_layer(O.dense(1024), heads=4, vdim=128, state=128, groups=1, norm_groups=1, conv=4)])
+WIDE = O.make_config(width=320, vocab=333, eps=1e-6, layers=[
+    O.parallel_layer(O.dense(200), O.attn(heads=34, kv_heads=2, dim=32, vdim=16, rot=2, size=100, scale=0.3, softcap=50.0),
+                     O.gla(heads=1, dim=130, vdim=200, tau=1.0, rank=40), left_scale=1.0, right_scale=1.0),
+    O.mamba_layer(O.dense(72), heads=5, vdim=72, state=150, groups=5, norm_groups=5, conv=2),
+    O.mamba_layer(None, heads=1, vdim=320, state=16, groups=1, norm_groups=8, conv=1)])
+DEEP = O.make_config(width=200, vocab=150, loop=(2, 3, 1), layers=[
+    O.mamba_layer(O.dense(100), heads=9, vdim=13, state=70, groups=3, norm_groups=9, conv=8),
+    O.parallel_layer(None, O.attn(heads=3, kv_heads=3, dim=144, vdim=72, rot=100, size=64, scale=0.08, softcap=5.0, base=20.0),
+                     O.gla(heads=5, dim=10, vdim=21, tau=30.0, rank=3), left_scale=-0.8, right_scale=2.0),
+    O.parallel_layer(O.dense(33), O.attn(heads=4, kv_heads=2, dim=20, vdim=200, rot=20, size=1, scale=0.25, softcap=2.0),
+                     O.gla(heads=2, dim=33, vdim=9, tau=0.5, rank=1), left_scale=0.5, right_scale=0.5)])
+CONFIGS = {"mixed": MIXED, "aligned": ALIGNED, "wide": WIDE, "deep": DEEP}
+_cache, _want = {}, {}
+
+
+def model(name, tmp_models, qk_gain=1.5):
+    """(folder, config, weights) of a configuration, written once."""
+    if name not in _cache:
+        cfg = CONFIGS[name]
+        w = O.random_weights(cfg, seed=11, qk_gain=qk_gain)
+        _cache[name] = (write_model(tmp_models / ("sinisun-" + name), O.plain(cfg), w), cfg, w)
+    return _cache[name]
+
+
+def oracle(name, cfg, w, ids):
+    key = (name, tuple(ids))
+    if key not in _want:
+        _want[key] = O.forward(cfg, w, ids)
+    return _want[key]
+
+
+# ---- kernels alone -----------------------------------------------------------------------------------
+HEAD = [(4, 2, 20, 24, 3, 4), (6, 6, 48, 32, 4, 2), (3, 1, 128, 64, 1, 3), (2, 1, 200, 16, 16, 1), (5, 5, 70, 200, 2, 10),
+        (8, 2, 33, 300, 7, 1), (1, 1, 64, 640, 4, 1)]
+KEY = [(3, 3, 24, 40, 12, 5.0), (6, 6, 32, 64, 16, 16.0), (1, 1, 130, 200, 40, 1.0), (2, 2, 256, 16, 5, 0.5), (4, 4, 70, 9, 1, 30.0)]
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+@pytest.mark.parametrize("kind, sizes", [("head", s) for s in HEAD] + [("key", s) for s in KEY])
+def test_linear_scan_kernels(kind, sizes, f32):
+    """Portions of unequal lengths at block and chunk borders, continued by others; single tokens, some of them twice;
+    slots taken over by a new sequence; state and convolution inputs that no earlier sequence may leak."""
+    m = E()
+    H, G, N, dv = sizes[:4]
+    g = torch.Generator().manual_seed(H * 1000 + N)
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    head, eps, slots, osc = kind == "head", 3e-4, 6, 0.7
+    np_, vp, inner = m.lin_pad_n(N), pad(dv, 16), H * dv
+    dt = torch.float32 if f32 else torch.bfloat16
+    norm_w = 1 + 0.3 * rnd(inner if head else dv)
+    if head:
+        taps, parts = sizes[4:]
+        C = inner + 2 * G * N
+        w = dict(conv_w=rnd(C, taps) / math.sqrt(taps), conv_b=rnd(C) * 0.4, dt_b=rnd(H) - 1.5, a_log=rnd(H) - 1, D=1 + rnd(H) / 2)
+        width = 2 * inner + 2 * G * N + H
+        off = dict(z_off=5, x_off=5 + inner, dt_off=5 + 2 * inner + 2 * G * N, taps=taps, norm_parts=parts)
+    else:
+        rank, tau = sizes[4:]
+        w = dict(a2=rnd(H * N, rank) / math.sqrt(rank), a2_b=2 + rnd(H * N))
+        width = H * (2 * N + 2 * dv) + rank
+        off = dict(q_off=5, k_off=5 + H * N, v_off=5 + 2 * H * N, z_off=5 + 2 * H * N + inner, a_off=5 + 2 * H * N + 2 * inner,
+                   rank=rank, q_scale=N ** -0.5, inv_tau=1 / tau)
+
+    def ref(x):
+        x = x.double()
+        T = x.shape[0]
+        W = {k: v.double() for k, v in w.items()}
+        if head:
+            z, u, st = x[:, :inner], x[:, inner:-H], x[:, -H:]
+            u = O.silu(O.causal_conv(u, W["conv_w"], W["conv_b"]))
+            X = u[:, :inner].view(T, H, dv)
+            B, Cc = (u[:, inner + i * G * N:inner + (i + 1) * G * N].reshape(T, G, N).repeat_interleave(H // G, 1) for i in (0, 1))
+            st = O.softplus(st + W["dt_b"])
+            d = torch.exp(-torch.exp(W["a_log"]) * st)[..., None].expand(T, H, N)
+            o = O.decayed_outer(d, B * st[..., None], X, Cc) + W["D"][:, None] * X
+            return osc * O.rms_parts(o.reshape(T, inner) * O.silu(z), parts, eps) * norm_w.double()
+        q, k, v, z, a = torch.split(x, [H * N, H * N, inner, inner, rank], 1)
+        al = torch.sigmoid(a @ W["a2"].T + W["a2_b"]).pow(1 / tau).view(T, H, N)
+        o = O.decayed_outer(al, k.reshape(T, H, N), v.reshape(T, H, dv), q.reshape(T, H, N) * N ** -0.5)
+        return osc * (O.rms(o, eps) * norm_w.double()).reshape(T, inner) * O.silu(z)
+
+    X = {s: bf(rnd(n, width)) for s, n in {0: 230, 2: 140, 5: 90, 3: 100}.items()}
+    want = {s: ref(x) for s, x in X.items()}
+    D = {k: dev(v) for k, v in dict(w, norm_w=norm_w).items()}
+    state = torch.full((2, slots, H, np_, vp), 1e30, device="cuda")
+    ring = torch.full((slots, sizes[4], inner + 2 * G * N), 1e30, device="cuda") if head else None
+    ws = m.lin_ws(m.LIN_HEAD if head else m.LIN_KEY, H, G, np_, vp, bool(f32))
+    buf = {k: torch.full((2 * 24 * n + 4096,), float("nan"), dtype=torch.float32 if k == "dec" else dt, device="cuda")
+           for k, n in zip(("qo", "ko", "kr", "vo", "so", "dec"), ws)}
+    work, ld = torch.zeros(24 * 16, dtype=torch.int32, device="cuda"), 5 + width + 3
+
+    def go(entries, decode=False):
+        rows = torch.cat([X[s][st:st + n] for s, st, n in entries])
+        n = rows.shape[0]
+        inp = torch.full((n, ld), 1e30)
+        inp[:, 5:5 + width] = rows
+        inp, out, y = dev(inp), torch.zeros(n, inner + 64, dtype=dt, device="cuda"), torch.zeros(n, inner, device="cuda")
+        pieces, at = [], 0
+        for s, st, k in entries:
+            pieces.append([at, k, s, st])
+            at += k
+        pd, sd = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in zip(*[(p[3], p[2]) for p in pieces]))
+        print(kind, sizes, f32, entries, flush=True)
+        m.lin_scan([] if decode else pieces, kind=m.LIN_HEAD if head else m.LIN_KEY, H=H, G=G, N=N, dv=dv, vp=vp, inp=inp.data_ptr(),
+                   ld=ld, **off, **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr() if head else 0,
+                   state=state.data_ptr(), slots=slots, pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
+                   **{k: v.data_ptr() for k, v in buf.items()}, y=y.data_ptr(), eps=eps, out_scale=osc, out=out.data_ptr(),
+                   ldo=inner + 64, f32=f32, work=work.data_ptr(), stream=stream())
+        torch.cuda.synchronize()
+        ref = torch.cat([want[s][st:st + k] for s, st, k in entries])
+        got = out.cpu()[:, :inner].double()
+        err, rms = float((got - ref).abs().max() / ref.abs().max()), float((got - ref).pow(2).mean().sqrt() / ref.pow(2).mean().sqrt())
+        print(err, rms, flush=True)
+        assert (out[:, inner:] == 0).all() and err < (2e-5 if f32 else 3e-2) and rms < (4e-6 if f32 else 5e-3), (entries, err, rms)
+
+    go([(0, 0, 1), (2, 0, 64), (5, 0, 2), (3, 0, 31)])
+    go([(0, 1, 100), (2, 64, 17), (5, 2, 1)])
+    go([(0, 101, 1), (5, 3, 1), (3, 31, 1), (2, 81, 1)], True)
+    go([(5, 3, 1), (0, 101, 1), (2, 81, 1)], True)                  # once more at the same positions
+    go([(5, 4, 1), (2, 82, 1)], True)
+    go([(5, 4, 1), (2, 82, 1)])                                     # again, as portions of one token
+    go([(2, 83, 48), (0, 102, 128), (3, 32, 66), (5, 5, 3)])        # even lengths: in and out at one parity
+    X[0] = bf(rnd(70, width))
+    want[0] = ref(X[0])
+    go([(0, 0, 2), (5, 8, 82)])
+    go([(0, 2, 1)], True)
+    go([(0, 3, 49)])
+    X[3] = bf(rnd(9, width))
+    want[3] = ref(X[3])
+    for t in range(9):
+        go([(3, t, 1)], True)
+
+
+GQA = [(6, 2, 40, 24, 28, 0, 17, 9.0), (8, 4, 96, 96, 96, 0, 100, 30.0), (20, 1, 64, 64, 2, 0, 64, 3.0), (3, 3, 144, 72, 100, 0, 1, 5.0),
+       (34, 2, 20, 200, 0, 45, 0, 0.0), (4, 2, 256, 256, 256, 130, 96, 15.0), (32, 8, 128, 128, 64, 0, 0, 0.0)]
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+@pytest.mark.parametrize("H, G, dk, dv, rot, window, chunk, cap", GQA)
+def test_grouped_query_attention_kernels(H, G, dk, dv, rot, window, chunk, cap, f32):
+    """Unequal sequences over scattered blocks: single tokens, portions of several through the tiled kernel (key splits)
+    and the flash kernel; windows and chunks that end at tile and block borders; one dominant sink."""
+    m, g = E(), torch.Generator().manual_seed(H * 1000 + dk)
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    dkp, dvp, maxb, rep = pad(dk, 32), pad(dv, 32), 6, H // G
+    lens = [1, 64, 65, 200, 129, 101]
+    seqs = [(i, l - 1, 1) for i, l in enumerate(lens)] + [(6, 90, 47)]
+    flash = (7, 60, 150)  # (the flash kernel, 16-bit)
+    tot = seqs + [flash]
+    n, nall, nslot = sum(s[2] for s in seqs), sum(s[2] for s in tot), 8
+    scale, osc, base, P = 2.0 / math.sqrt(dk), 0.6, 300.0, maxb * 64
+    perm = torch.randperm(nslot * maxb, generator=g).view(nslot, maxb)
+    qb, kb, vb, sink = rnd(H * dk), rnd(G * dk), rnd(G * dv), rnd(H)
+    sink[H // 2] = 6.0
+    ld, cols = H * dk + G * (dk + dv) + H + 7, H * dk + G * (dk + dv)
+    inp = rnd(nall, ld)
+    ctx = {s: (bf(rnd(st, G, dk)), bf(rnd(st, G, dv))) for s, st, _ in tot}
+    turn = lambda v, p: O.rotate_half(torch.cat([torch.zeros(p, *v.shape[1:], dtype=O.DT), v.double()]), base, rot)[p:]
+    blk = torch.zeros(nslot * maxb + 1, G * 64 * (dkp + dvp))
+    kview, vview = blk[:, :G * 64 * dkp].view(-1, G, 64, dkp), blk[:, G * 64 * dkp:].view(-1, G, 64, dvp)
+    for s, st, _ in tot:
+        for p in range(st):
+            kview[perm[s, p // 64], :, p % 64, :dk], vview[perm[s, p // 64], :, p % 64, :dv] = ctx[s][0][p], ctx[s][1][p]
+    want, pos, slot, tiles, row = torch.zeros(nall, H, dv, dtype=O.DT), [], [], [], 0
+    r16 = (lambda t: t) if f32 else (lambda t: t.float().bfloat16().double())
+    for s, st, k in tot:
+        pos += range(st, st + k)
+        slot += [s] * k
+        if s != flash[0]:
+            tiles += [(f, min(16, (row + k) * rep - f)) for f in range(row * rep, (row + k) * rep, 16)]
+        x = inp[row:row + k]
+        q = turn((x[:, :H * dk] + qb).view(k, H, dk), st)
+        kn = r16(turn((x[:, H * dk:(H + G) * dk] + kb).view(k, G, dk), st))
+        K = torch.cat([ctx[s][0].double(), kn])
+        V = torch.cat([ctx[s][1].double(), r16((x[:, (H + G) * dk:cols] + vb).view(k, G, dv).double())])
+        gate = torch.sigmoid(x[:, cols:cols + H].double())
+        for i in range(k):
+            p = st + i
+            a, b = max(p // chunk * chunk if chunk else 0, p - window + 1 if window else 0), p + 1
+            for h in range(H):
+                sc = (K[a:b, h // rep] @ q[i, h]) * scale
+                sc = O.soft_cap(sc, cap) if cap else sc
+                want[row + i, h] = osc * gate[i, h] * (O.sink_weights(sc, sink[h].double()) @ V[a:b, h // rep])
+        row += k
+    ang = torch.arange(P, dtype=O.DT)[:, None] * base ** (-2.0 * torch.arange(rot // 2, dtype=O.DT) / max(rot, 1))
+    dt = torch.float32 if f32 else torch.bfloat16
+    D = dict(rope=torch.stack([ang.cos(), ang.sin()], -1).float() if rot else torch.zeros(2), sink=sink, qb=qb, kb=kb, vb=vb, inp=inp,
+             pos=torch.tensor(pos, dtype=torch.int32), slot=torch.tensor(slot, dtype=torch.int32), bt=perm.int(),
+             tiles=torch.tensor(tiles, dtype=torch.int32))
+    D = {k: dev(v) for k, v in D.items()}
+    for nsplit in (1,) if f32 else (1, 3, 64):
+        pool = dev(blk.to(dt))
+        out = torch.zeros(nall, H * dvp, dtype=dt, device="cuda")
+        q = torch.zeros(nall, H, dkp, dtype=dt, device="cuda")
+        na = nall if f32 else n
+        part, ml = torch.zeros(nsplit, na * H, dvp, device="cuda"), torch.zeros(nsplit, na * H, 2, device="cuda")
+        kw = {} if f32 else dict(flash_T=flash[2], flash_row0=n, flash_slot=flash[0], flash_start=flash[1])
+        print(H, G, dk, dv, rot, window, chunk, cap, f32, nsplit, flush=True)
+        m.gqa_attention(rows=nall, n=na, H=H, G=G, dk=dk, dkp=dkp, dv=dv, dvp=dvp, rot=rot, window=window, chunk=chunk, scale=scale,
+                        softcap=cap, ld=ld, q_off=0, k_off=H * dk, v_off=(H + G) * dk, g_off=cols, out_scale=osc, pool=pool.data_ptr(),
+                        maxb=maxb, f32=f32, q=q.data_ptr(), n_tiles=len(tiles), nsplit=nsplit, opart=part.data_ptr(),
+                        ml=ml.data_ptr(), out=out.data_ptr(), ldo=H * dvp, stream=stream(),
+                        **{k: v.data_ptr() for k, v in D.items()}, **kw)
+        torch.cuda.synchronize()
+        got = out.float().cpu().view(nall, H, dvp)
+        assert (got[:, :, dv:] == 0).all()
+        err = (got[:, :, :dv].double() - want).abs().amax((1, 2)) / want.abs().max()
+        assert float(err.max()) < (2e-5 if f32 else 2.5e-2), (nsplit, int(err.argmax()), float(err.max()))
+
+
+@pytest.mark.parametrize("M", [1, 2, 3, 4, 5, 33, 64, 65, 300])
+@pytest.mark.parametrize("act", ["relu2", "silu"])
+def test_activation_epilogues(M, act):
+    """act(W x + b) in the product's epilogue: GEMV engine, skinny and prefill GEMM, fp32."""
+    m, g = E(), torch.Generator().manual_seed(M)
+    K, N = 512, 768
+    x, w, b = bf(torch.randn(M, K, generator=g)), bf(torch.randn(N, K, generator=g) / math.sqrt(K)), torch.randn(N, generator=g)
+    want = x.double() @ w.double().T + b.double()
+    want = torch.relu(want) ** 2 if act == "relu2" else O.silu(want)
+    kind = {"relu2": m.ACT_RELU2, "silu": m.ACT_SILU}[act]
+    wb = w.bfloat16()
+    q = m.QMatrix(int(m.QT_BF16), N, K, wb.view(torch.int16).numpy())
+    xd, bd = dev(x.bfloat16()), dev(b)
+
+    def check(y, tol):
+        assert (y.cpu().double() - want).abs().max() / want.abs().max() < tol
+
+    y = torch.zeros(M, N, dtype=torch.bfloat16, device="cuda")
+    if M <= 4:
+        m.gemv([q], M, 0, K, 0, 1e-5, 0, N, m.EPI_ACT16, stream(), x16=xd.data_ptr(), y16=y.data_ptr(), ldy16=N, act=kind, bias=bd.data_ptr())
+        torch.cuda.synchronize()
+        check(y, 5e-3)
+    y.zero_()
+    m.gemm_q(xd.data_ptr(), K, [q], M, 0, y.data_ptr(), N, m.GEPI_STORE16, stream(), bias16=bd.data_ptr(), unary=1 + kind)
+    torch.cuda.synchronize()
+    check(y, 5e-3)
+    y32, z = torch.zeros(M, N, device="cuda"), dev((x.double() @ w.double().T).float())
+    m.bias_act_f32(z.data_ptr(), N, bd.data_ptr(), y32.data_ptr(), N, M, N, kind, stream())
+    torch.cuda.synchronize()
+    check(y32, 2e-6)
+
+
+@pytest.mark.parametrize("f32", [0, 1])
+def test_bias_and_loop_entry_in_the_row_operations(f32):
+    m, g = E(), torch.Generator().manual_seed(5)
+    rows, d = 7, 200
+    dp, dt, eps = pad(d, 64), torch.float32 if f32 else torch.bfloat16, 1e-3
+    rnd = lambda *s: torch.randn(*s, generator=g)
+    x, y, x0, yb, nx = rnd(rows, d), rnd(rows, d), rnd(rows, d), rnd(d), rnd(d)
+    xd, yd, ed, bd, nd = (dev(padded(t, dp)) for t in (x, y, x0, yb, nx))
+    out = torch.zeros(rows, dp, dtype=dt, device="cuda")
+    m.row_close(rows, xd.data_ptr(), dp, d, eps, yd.data_ptr(), f32=f32, next=m.NEXT_NORM, g=nd.data_ptr(), out=out.data_ptr(),
+                ldo=dp, stream=stream(), y_bias=bd.data_ptr(), extra=ed.data_ptr())
+    torch.cuda.synchronize()
+    want = (x + y + x0).double() + yb.double()
+    assert (xd.cpu()[:, :d].double() - want).abs().max() < 1e-5
+    nxt = O.rms(want, eps) * nx.double()
+    assert (out.cpu()[:, :d].double() - nxt).abs().max() < (1e-5 if f32 else 1e-2) * nxt.abs().max() and (out[:, d:] == 0).all()
+    tab, tok = rnd(9, d).bfloat16(), torch.tensor([3, 8, 0], dtype=torch.int32, device="cuda")
+    td, keep, e = dev(padded(tab, dp)), torch.zeros(3, dp, device="cuda"), torch.zeros(3, dp, device="cuda")
+    m.embed_rows(3, td.data_ptr(), 1.0, 0, 0, 0, 0, tok.data_ptr(), tok.data_ptr(), tok.data_ptr(), 0, 0, 4, dp, d, eps, e.data_ptr(), 0, 0, f32,
+                 m.NEXT_NORM, nd.data_ptr(), out.data_ptr(), dp, stream(), keep32=keep.data_ptr())
+    torch.cuda.synchronize()
+    assert torch.equal(keep, e) and torch.equal(e.cpu()[:, :d], tab[[3, 8, 0]].float())
+
+
+# ---- the engine against the oracle ----------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_whole_prompt_portions_and_decode(name, dtype, tmp_models):
+    path, cfg, w = model(name, tmp_models)
+    ids = ids_of(cfg, 270)
+    want = oracle(name, cfg, w, ids)
+    eng = engine(path, dtype)
+    assert rel(run(eng, 0, ids, [len(ids)]), want) < TOL[dtype]
+    for slot, sizes in ((1, [2]), (2, [3, 61, 64, 1, 128, 5, 7]), (3, [130, 1]), (1, [1]), (2, [150, 17, 16, 33, 32])):
+        n = 40 if sizes in ([2], [1]) else 170
+        eng.release_slot(slot)
+        assert rel(run(eng, slot, ids[:n], sizes), want[:n]) < TOL[dtype], sizes
+
+
+@pytest.mark.parametrize("name", ["aligned", "mixed"])
+def test_residual_after_every_layer_run(name, tmp_models):
+    path, cfg, w = model(name, tmp_models)
+    ids, trace = ids_of(cfg, 50, 9), []
+    O.forward(cfg, w, ids, trace)
+    eng = engine(path, "float32")
+    assert eng.layer_runs == len(trace) == len(O.schedule(cfg))
+    for k in range(len(trace)):
+        eng.set_run_limit(k + 1)
+        eng.step([0], [0], [50], ids, [])
+        assert (torch.from_numpy(eng.last_residual(50)).double() - trace[k]).abs().max() < 1e-4 * max(1.0, float(trace[k].abs().max()))
+    eng.set_run_limit(-1)
+    assert rel(run(eng, 0, ids, [50]), oracle(name, cfg, w, ids)) < F32_TOL
+
+
+@pytest.mark.parametrize("name", ["aligned", "wide", "deep"])
+def test_long_portions_on_a_long_context(name, tmp_models, monkeypatch):
+    """The flash kernel from 32-token portions on, and passes of at most 96 rows: every border between the two
+    kernels and between the passes of one step."""
+    monkeypatch.setenv("AIOS_GQA_PF_MIN", "32")
+    monkeypatch.setenv("AIOS_STEP_ROWS", "96")
+    path, cfg, w = model(name, tmp_models)
+    ids = ids_of(cfg, 390, 3)
+    want = oracle(name, cfg, w, ids)
+    eng = engine(path)
+    assert rel(run(eng, 0, ids, [390]), want) < TOL["bfloat16"]
+    assert rel(run(eng, 1, ids, [33, 31, 64, 2, 100, 97, 32]), want) < TOL["bfloat16"]
+
+
+@pytest.mark.parametrize("dtype", DT)
+@pytest.mark.parametrize("name", ["mixed", "aligned"])
+def test_mixed_batches_equal_each_alone(name, dtype, tmp_models):
+    """Portions of some requests beside decoded tokens of others; a request pauses; slots and blocks are reused."""
+    path, cfg, w = model(name, tmp_models)
+    lens = [150, 9, 70, 33, 101, 64]
+    seqs = [ids_of(cfg, n, 20 + i) for i, n in enumerate(lens)]
+    want = [oracle(name, cfg, w, s) for s in seqs]
+    eng = engine(path, dtype, kv_pool_tokens=7 * 64)
+    rng = np.random.default_rng(4)
+    free, live, todo, got = [0, 1, 2, 3], {}, list(range(6)), [[] for _ in seqs]
+    while todo or live:
+        while todo and free and sum(-(-lens[i] // 64) for i in list(live) + todo[:1]) <= 7:
+            i = todo.pop(0)
+            live[i] = [free.pop(), 0]
+        entries = [i for i in live if rng.random() < 0.8] or list(live)[:1]
+        counts = [min(int(rng.choice([1, 1, 2, 5, 40, 66])), lens[i] - live[i][1]) for i in entries]
+        toks = [t for i, n in zip(entries, counts) for t in seqs[i][live[i][1]:live[i][1] + n]]
+        out = eng.step([live[i][0] for i in entries], [live[i][1] for i in entries], counts, toks, list(range(len(toks))))
+        at = 0
+        for i, n in zip(entries, counts):
+            got[i].append(torch.from_numpy(out[at:at + n].copy()))
+            at += n
+            live[i][1] += n
+            if live[i][1] == lens[i]:
+                eng.release_slot(live[i][0])
+                free.append(live.pop(i)[0])
+    assert eng.kv_blocks_free == 7
+    for i in range(6):
+        assert rel(torch.cat(got[i]), want[i]) < TOL[dtype], i
+
+
+@pytest.mark.parametrize("name", ["mixed", "aligned"])
+@pytest.mark.parametrize("dtype", DT)
+def test_captured_decode_equals_the_oracle(name, dtype, tmp_models):
+    """The decode graphs (every batch size's kernels) replayed step after step with other engine work in between, across
+    block and chunk borders; logits of every replay."""
+    path, cfg, w = model(name, tmp_models)
+    seqs = [ids_of(cfg, 60 + 3 * (i % 6), 50 + i % 6) for i in range(40)]
+    want = [oracle(name, cfg, w, s) for s in seqs[:6]]
+    eng = engine(path, dtype, max_slots=41, max_batch=40, max_ctx=128)
+    for B in (1, 2, 4, 5, 6, 40):
+        start = [len(s) - 9 for s in seqs[:B]]
+        for b in range(B):
+            eng.release_slot(b)
+            eng.prefill(b, seqs[b][:start[b]], 0, False)
+        got = [[] for _ in range(B)]
+        for t in range(9):
+            eng.decode(list(range(B)), [seqs[b][start[b] + t] for b in range(B)], [start[b] + t for b in range(B)])
+            lg = torch.from_numpy(eng.last_logits(B))
+            for b in range(B):
+                got[b].append(lg[b:b + 1])
+            if t == 4:
+                eng.prefill(40, seqs[0][:5], 0, True)  # eager work between two replays
+        for b in range(B):
+            assert rel(torch.cat(got[b]), want[b % 6][start[b]:]) < TOL[dtype], (B, b)
+
+
+CHUNK = 70
+
+
+def chunk_model(tmp_models):
+    """Token 1 asks for token 0: the first layer's head 0 gives that pair a score far above all others (through
+    dimensions that do not turn), and the linear attention beside it stays small and forgets at once."""
+    cfg = O.make_config(width=128, vocab=90, eps=1e-5, layers=[
+        O.parallel_layer(O.dense(96), O.attn(heads=2, kv_heads=1, dim=32, vdim=48, rot=8, size=CHUNK, scale=0.3, softcap=25.0),
+                         O.gla(heads=2, dim=8, vdim=16, tau=0.2, rank=2), left_scale=1.5, right_scale=0.01),
+        O.parallel_layer(None, O.attn(heads=3, kv_heads=3, dim=16, vdim=16, rot=4, size=5),
+                         O.gla(heads=2, dim=8, vdim=16, tau=0.2, rank=2), right_scale=0.01)])
+    w = {k: v.float() for k, v in O.random_weights(cfg, 77).items()}
+    w["embed"][0, :], w["embed"][1, :] = 0.0, 0.0
+    w["embed"][0, 5], w["embed"][1, 9] = 12.0, 12.0
+    q = "l0.mix.left."
+    w[q + "k"][:, 5], w[q + "k"][20, 5], w[q + "q"][20, 9] = 0.0, 2.0, 2.0
+    w[q + "k"][20, 9] = 0.0
+    w[q + "v"][:, 5] *= 3
+    w[q + "g"][0], w[q + "sink"][0] = 0.0, 3.0
+    w = {k: v.to(torch.bfloat16) for k, v in w.items()}
+    return write_model(tmp_models / "sinisun-chunk", O.plain(cfg), w), cfg, w
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_keys_just_inside_and_outside_a_chunk(dtype, tmp_models, monkeypatch):
+    path, cfg, w = chunk_model(tmp_models)
+    engs = [engine(path, dtype)]
+    if dtype == "bfloat16":
+        monkeypatch.setenv("AIOS_GQA_PF_MIN", "2")  # the flash kernel for every portion
+        engs.append(engine(path, dtype))
+    for n in (CHUNK, CHUNK + 1, CHUNK + 2, 129, 2 * CHUNK, 2 * CHUNK + 1, 193, 300):
+        low = (n - 1) // CHUNK * CHUNK
+        for key in sorted({0, low - 1, low, low + 1, 63, 64, 127, 128, n - 2} & set(range(n - 1))):
+            ids = [2 + t % 88 for t in ids_of(cfg, n, 300 + n)]
+            ids[key], ids[-1] = 0, 1
+            want = O.forward(cfg, w, ids)[-1:]
+            if n in (129, 2 * CHUNK):
+                without = O.forward(cfg, w, ids[:key] + [50] + ids[key + 1:])[-1:]
+                if key >= low:
+                    assert rel(without, want) > 0.15  # the key is what the last position's logits rest on
+                elif key < n - 8:
+                    assert rel(without, want) < 0.05
+            for eng in engs:
+                for slot, sizes in ((0, [n]), (1, [n - 1, 1]), (2, [40, 29, 2, 100, 1])):
+                    eng.release_slot(slot)
+                    assert rel(run(eng, slot, ids, sizes)[-1:], want) < 2 * TOL[dtype], (n, key, sizes)
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_the_first_tokens_of_a_sequence(dtype, tmp_models):
+    path, cfg, w = model("mixed", tmp_models)
+    eng = engine(path, dtype)
+    for seed in range(4):
+        ids = ids_of(cfg, 5, 700 + seed)
+        want = oracle("mixed", cfg, w, ids)
+        for slot, sizes in ((0, [5]), (0, [1]), (1, [2, 3]), (1, [1, 4])):  # (slots are taken over without a release)
+            assert rel(run(eng, slot, ids, sizes), want) < TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DT)
+def test_long_decoding_and_the_context_limit(dtype, tmp_models):
+    path, cfg, w = model("mixed", tmp_models)
+    P = 450
+    ids = ids_of(cfg, P, 8)
+    want = oracle("mixed", cfg, w, ids)
+    eng = engine(path, dtype, max_ctx=P)
+    run(eng, 0, ids[:P - 250], [P - 250])
+    assert rel(run(eng, 0, ids[P - 250:], [1], start=P - 250), want[P - 250:]) < TOL[dtype]
+    with pytest.raises(RuntimeError, match="overflow"):
+        eng.step([0], [P], [1], [0], [])
+    with pytest.raises(RuntimeError):
+        eng.step([1], [0], [1], [cfg["vocab"]], [])
+
+
+def test_the_recurrent_state_stands_at_one_position(tmp_models):
+    """Where a slot may go on, a dropped single token, copies; anything else is refused before it runs."""
+    path, cfg, w = model("mixed", tmp_models)
+    a, b = ids_of(cfg, 140, 1), ids_of(cfg, 60, 2)
+    eng = engine(path, "float32")
+    assert eng.recurrent and eng.resumable(0, 0) and not eng.resumable(0, 1)
+    run(eng, 0, a, [140])
+    assert eng.resumable(0, 140) and not eng.resumable(0, 139) and not eng.resumable(0, 100)
+    for start in (100, 139, 141):
+        with pytest.raises(RuntimeError, match="state stands"):
+            eng.step([0], [start], [1], [0], [])
+    eng.copy_slot(0, 1, 140)
+    assert rel(run(eng, 1, b, [60], start=140), O.forward(cfg, w, a + b)[140:]) < F32_TOL
+    # a single token whose result is dropped, then another in its place; the copy's state is its own
+    run(eng, 0, [5], [1], start=140)
+    assert eng.resumable(0, 141) and eng.resumable(0, 140)
+    more = ids_of(cfg, 20, 3)
+    assert rel(run(eng, 0, more, [1], start=140), O.forward(cfg, w, a + more)[140:]) < F32_TOL
+
+
+def test_tensor_errors(tmp_models):
+    path, cfg, w = model("mixed", tmp_models)
+    bad = write_model(tmp_models / "sn-bad", O.plain(cfg), {k: v for k, v in w.items() if k != "l1.mix.right.a2.b"})
+    with pytest.raises(ValueError, match="l1.mix.right.a2.b"):
+        engine(bad)
+    bad = write_model(tmp_models / "sn-bad2", O.plain(cfg), dict(w, **{"l1.mix.left.g": w["l1.mix.left.g"][:2]}))
+    with pytest.raises(RuntimeError, match="attn_gate"):
+        engine(bad)
+    with pytest.raises(ValueError, match="fp8"):
+        engine(path, kv_dtype="fp8")
+
+
+# ---- generation through the framework's entry points -----------------------------------------------------
+@pytest.mark.parametrize("opts", ["#compute=float32", "#compute=float32&kv_tokens=256", ""])
+def test_greedy_generation_through_the_scheduler(opts, tmp_models, monkeypatch):
+    """Unequal prompts, some of which stop early (the others' queued step is dropped and run again); then a follow-up
+    that goes on where the first one's state stands."""
+    from aios_amd.runtime.scheduler import GenRequest
+
+    monkeypatch.setenv("AIOS_PREFILL_CHUNK", "48")
+    path, cfg, w = model("mixed", tmp_models)
+    prompts = [ids_of(cfg, n, 90 + n) for n in (3, 130, 50, 64, 20)]
+    n = 12
+    key = ("greedy", "mixed")
+    if key not in _want:
+        _want[key] = [O.greedy(cfg, w, p, n) for p in prompts]
+    full = _want[key]
+    stop = [full[i][5] if i in (1, 3) else None for i in range(5)]
+    reqs = [GenRequest(prompt_ids=p, max_tokens=n, stop_ids=[s] if s is not None else None) for p, s in zip(prompts, stop)]
+
+    def follow(out):
+        ids = prompts[0] + out[0][0].token_ids[:-1]
+        return [GenRequest(prompt_ids=ids + [7, 8], max_tokens=4)]
+
+    first, second = generate(path + opts, [reqs, follow], 4)
+    for p, r, s, f in zip(prompts, first, stop, full):
+        if opts:  # 32-bit: the oracle's own choice at every step
+            assert r.token_ids == (f if s is None else f[:f.index(s)])
+        elif len(r.token_ids):  # bf16: a choice within rounding of the oracle's best, most of the time
+            lg = O.forward(cfg, w, p + r.token_ids)[len(p) - 1:-1]
+            gap = lg.max(-1).values - lg.gather(1, torch.tensor(r.token_ids)[:, None])[:, 0]
+            assert float((gap / lg.std(-1)).median()) < 0.1
+    ids = prompts[0] + first[0].token_ids[:-1] + [7, 8]
+    if opts:
+        assert second[0].token_ids == O.greedy(cfg, w, ids, 4)
+    assert len(second[0].token_ids) == 4
+
+
+def test_synthetic_preset_decodes_and_matches_its_steps():
+    """Random-init preset: the captured decode loop's history equals single steps' argmax."""
+    from aios_amd.models.config import get_preset
+    from aios_amd.runtime.loader import random_engine
+
+    cfg = get_preset("test-sinisun")
+    eng = random_engine(cfg, seed=3, max_ctx=256, max_slots=2, max_batch=2, compute="float32")
+    ids = [int(t) for t in np.random.default_rng(0).integers(0, cfg.vocab_size, 30)]
+    first = int(np.asarray(eng.prefill(0, ids, 0, True)).argmax())
+    eng.decode_loop_prepare([0], [first], [30])
+    eng.decode_loop_run(1, 40, True)
+    hist = eng.decode_loop_history(1, 31, 40)
+    lg = eng.step([1], [0], [30 + 40], ids + [first] + hist[:39], list(range(29, 70)))
+    gap = lg.max(-1) - lg[np.arange(41), [first] + hist]
+    assert float((gap / lg.std(-1)).max()) < 1e-3
