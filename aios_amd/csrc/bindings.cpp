@@ -850,6 +850,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
         a.q_scale = F("q_scale"); a.inv_tau = F("inv_tau"); a.a2 = P("a2"); a.a2_b = P("a2_b");
         a.state = P("state"); a.slots = I("slots"); a.pos = (const int*)P("pos"); a.slot = (const int*)P("slot");
         a.n = a.rows = I("n"); a.qo = P("qo"); a.ko = P("ko"); a.kr = P("kr"); a.vo = P("vo"); a.so = P("so"); a.dec = P("dec");
+        a.nseg = std::max(1, I("nseg")); a.seg = P("seg"); a.seg_dec = P("seg_dec");
         a.y = P("y"); a.norm_w = P("norm_w"); a.norm_parts = I("norm_parts"); a.eps = F("eps"); a.out_scale = F("out_scale");
         a.out = P("out"); a.ldo = I("ldo"); a.f32 = I("f32");
         hipStream_t st = S((uintptr_t)P("stream"));

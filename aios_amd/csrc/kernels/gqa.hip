@@ -45,7 +45,7 @@ __global__ void __launch_bounds__(256) gqa_prep_kernel(GqaArgs a, float qf) {
     if constexpr (F32) ((float*)base)[i] = v;
     else ((bf16_t*)base)[i] = f32_to_bf16(v);
   };
-  for (int i = threadIdx.x; i < nall; i += 256) {
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < nall; i += 256 * gridDim.y) {
     if (i >= nk) {
       const int v = i - nk, g = v / (a.dvp >> 1), c = 2 * (v - g * (a.dvp >> 1));
       const size_t at = blk + (size_t)a.G * GQA_BLOCK * a.dkp + ((size_t)g * GQA_BLOCK + key) * a.dvp + c;
@@ -86,8 +86,10 @@ void launch_gqa_prep(const GqaArgs& a, hipStream_t st) {
   if (a.rows < 1) return;
   if (!gqa_supports(a.dkp, a.dvp) || a.H % a.G || a.rot % 2 || a.rot > a.dk || (a.rot && !a.rope))
     throw std::runtime_error("gqa: bad sizes");
-  if (a.f32) hipLaunchKernelGGL((gqa_prep_kernel<true>), dim3(a.rows), dim3(256), 0, st, a, 1.f);
-  else hipLaunchKernelGGL((gqa_prep_kernel<false>), dim3(a.rows), dim3(256), 0, st, a, gqa_q_factor(a.scale, a.softcap));
+  const int pieces = ((a.H + a.G) * (a.dkp / 2) + a.G * (a.dvp / 2) + 255) / 256;
+  const dim3 grid(a.rows, a.rows <= 64 ? pieces : (pieces + 3) / 4);
+  if (a.f32) hipLaunchKernelGGL((gqa_prep_kernel<true>), grid, dim3(256), 0, st, a, 1.f);
+  else hipLaunchKernelGGL((gqa_prep_kernel<false>), grid, dim3(256), 0, st, a, gqa_q_factor(a.scale, a.softcap));
 }
 
 // ---- attention ------------------------------------------------------------------------------------

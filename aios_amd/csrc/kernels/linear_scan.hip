@@ -7,7 +7,10 @@
 //                        o = (q with the decay since the block's start) S + A v,
 //                        S = (decay of the block) S + (k with the decay to the block's end)^T v.
 //                      A 16 x 16 accumulator tile is, lane for lane, the second operand of the 16-deep product, so S never
-//                      leaves registers and the waves need no barrier.
+//                      leaves registers and the waves need no barrier.  Operands are requested several blocks ahead.
+//                      Where heads and columns leave compute units idle, a portion is walked in segments side by side: a
+//                      first walk takes every segment but the last from zero (the first one from the state) to its end,
+//                      without outputs; the second starts each segment from what those before it make together.
 //   norm               root-mean-square of the parts, weight, output gate
 // Single tokens: lin_step, one workgroup per head and row (convolution, decays, state and, for LIN_KEY, the norm).
 //
@@ -244,9 +247,9 @@ __global__ void __launch_bounds__(256) lin_key_prep_kernel(LinScanArgs a) {
   const LinBlock bl = lin_block(a, blk);
   if (bl.n < 1) return;
   const float* in = a.in + (size_t)bl.row0 * a.ld;
-  for (int i = tid; i < bl.n * a.rank; i += 256) {
+  for (int i = tid; i < 16 * a.rank; i += 256) {
     const int t = i / a.rank;
-    sa[i] = in[(size_t)t * a.ld + a.a_off + i - t * a.rank];
+    sa[i] = t < bl.n ? in[(size_t)t * a.ld + a.a_off + i - t * a.rank] : 0.f;
   }
   for (int j = tid; j < a.vp; j += 256) {
     float v[16];
@@ -255,20 +258,40 @@ __global__ void __launch_bounds__(256) lin_key_prep_kernel(LinScanArgs a) {
     put16<F32>(a.vo, ((blk * a.H + h) * a.vp + j) * 16, v);
   }
   __syncthreads();
-  for (int i = tid; i < 16 * NP; i += 256) {  // log decays
-    const int t = i / NP, n = i - t * NP;
-    float ld = 0.f, qv = 0.f, kv = 0.f;
-    if (t < bl.n && n < a.N) {
-      const int c = h * a.N + n;
-      float z = a.a2_b[c];
-      for (int r = 0; r < a.rank; ++r) z = fmaf(a.a2[(size_t)c * a.rank + r], sa[t * a.rank + r], z);
-      ld = -ls_softplus(-z) * a.inv_tau;
-      qv = in[(size_t)t * a.ld + a.q_off + c] * a.q_scale;
-      kv = in[(size_t)t * a.ld + a.k_off + c];
+  // log decays: a thread owns TG tokens of a channel
+  constexpr int GR = NP <= 32 ? 8 : NP <= 64 ? 4 : NP <= 128 ? 2 : 1, TG = 16 / GR;
+  if (tid < GR * NP) {
+    const int n = tid % NP, t0 = tid / NP * TG;
+    const bool real = n < a.N;
+    const int c = h * a.N + (real ? n : 0);
+    float z[TG], qv[TG], kv[TG];
+#pragma unroll
+    for (int t = 0; t < TG; ++t) {
+      const bool ok = real && t0 + t < bl.n;
+      qv[t] = ok ? in[(size_t)(t0 + t) * a.ld + a.q_off + c] : 0.f;
+      kv[t] = ok ? in[(size_t)(t0 + t) * a.ld + a.k_off + c] : 0.f;
+      z[t] = a.a2_b[c];
     }
-    sd[i] = ld;
-    sq[i] = qv;
-    sk[i] = kv;
+    const float *w = a.a2 + (size_t)c * a.rank, *ar = sa + t0 * a.rank;
+    int r = 0;
+    for (; r + 4 <= a.rank; r += 4) {
+      const float w0 = w[r], w1 = w[r + 1], w2 = w[r + 2], w3 = w[r + 3];
+#pragma unroll
+      for (int t = 0; t < TG; ++t) {
+        const float* x = ar + t * a.rank + r;
+        z[t] = fmaf(w3, x[3], fmaf(w2, x[2], fmaf(w1, x[1], fmaf(w0, x[0], z[t]))));
+      }
+    }
+    for (; r < a.rank; ++r)
+#pragma unroll
+      for (int t = 0; t < TG; ++t) z[t] = fmaf(w[r], ar[t * a.rank + r], z[t]);
+#pragma unroll
+    for (int t = 0; t < TG; ++t) {
+      const int i = (t0 + t) * NP + n;
+      sd[i] = real && t0 + t < bl.n ? -ls_softplus(-z[t]) * a.inv_tau : 0.f;
+      sq[i] = qv[t] * a.q_scale;
+      sk[i] = kv[t];
+    }
   }
   __syncthreads();
   const size_t base = (blk * a.H + h) * NP, plane = (size_t)2 * a.n_chunks * a.H * NP * 16;
@@ -333,9 +356,27 @@ struct LinOps<true, KEY, NT> {
   float tot;
 };
 
+// buffers of operands in registers: requests run that many blocks ahead, less one
 template <bool F32, bool KEY, int NT>
+constexpr int lin_depth() {
+  if (F32) return 2;
+  return KEY ? (NT <= 6 ? 4 : NT <= 8 ? 3 : 2) : (NT <= 8 ? 4 : NT <= 12 ? 3 : 2);
+}
+
+// the blocks of a portion that a segment walks: [i0, i1), and how many segments there are
+struct LinSeg {
+  int i0, i1, n;
+};
+__device__ __forceinline__ LinSeg lin_seg(int nb, int nseg, int seg) {
+  const int per = max(LIN_SEG_MIN, (nb + nseg - 1) / nseg);
+  return LinSeg{seg * per, min(nb, (seg + 1) * per), (nb + per - 1) / per};
+}
+
+// ENDS: the first walk of a portion in segments (no outputs; segment s leaves what it ends with at seg[s + 1], its decay
+// at seg_dec[s + 1]; the first one also copies the state it starts from to seg[0])
+template <bool F32, bool KEY, int NT, bool ENDS>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) lin_walk_kernel(LinScanArgs a) {
-  constexpr int NP = 16 * NT;
+  constexpr int NP = 16 * NT, DEPTH = lin_depth<F32, KEY, NT>();
   using T = std::conditional_t<F32, float, bf16_t>;
   using V = std::conditional_t<F32, gf32x4, uint2>;
   const int lane = threadIdx.x & 63, nvt = a.vp >> 4;
@@ -344,55 +385,94 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
   const int h = w / nvt, vt = w - h * nvt, g = KEY ? h : h / (a.H / a.G), ng = KEY ? a.H : a.G;
   const int r16 = lane & 15, q = lane >> 4;
   const ScanSeq sq = a.seqs[blockIdx.y];
-  const int nb = (sq.n + LIN_T - 1) / LIN_T, col = 16 * vt + r16;
+  const int nb = (sq.n + LIN_T - 1) / LIN_T, col = 16 * vt + r16, seg = blockIdx.z;
+  const LinSeg sg = lin_seg(nb, a.nseg, seg);
+  if (seg >= sg.n) return;
+  const size_t hs = (size_t)a.np * a.vp, half = (size_t)a.slots * a.H * hs;
+  const size_t at = (size_t)(4 * q) * a.vp + col;  // of this lane in a head's state
+  float* st = a.state + ((size_t)sq.slot * a.H + h) * hs + at;
+  // segment j of this portion and head
+  auto seg_at = [&](int j) { return a.seg + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * hs + at; };
+  auto dec_at = [&](int j) { return a.seg_dec + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * a.np; };
   const size_t plane = (size_t)2 * a.n_chunks * a.H * NP * 16;
   using Ops = LinOps<F32, KEY, NT>;
   auto load = [&](Ops& o, int i) {
-    const size_t b = sq.b0 + min(i, nb - 1);  // (past the end: re-reads)
+    const size_t b = sq.b0 + min(i, sg.i1 - 1);  // (past the end: re-reads)
     const T* qo = (const T*)a.qo + (b * ng + g) * NP * 16 + r16 * 16 + 4 * q;
     const T* ko = (const T*)a.ko + (b * ng + g) * NP * 16 + r16 * 16 + 4 * q;
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      o.q[t] = *(const V*)(qo + 256 * t);
       o.k[t] = *(const V*)(ko + 256 * t);
-      if constexpr (KEY && !F32) {
-        o.ql[t] = *(const V*)(qo + plane + 256 * t);
-        o.kl[t] = *(const V*)(ko + plane + 256 * t);
-      }
+      if constexpr (KEY && !F32) o.kl[t] = *(const V*)(ko + plane + 256 * t);
+      if constexpr (ENDS) continue;
+      o.q[t] = *(const V*)(qo + 256 * t);
+      if constexpr (KEY && !F32) o.ql[t] = *(const V*)(qo + plane + 256 * t);
     }
     const T* so = (const T*)a.so + (b * a.H + h) * (F32 ? 256 : 512) + r16 * 16 + 4 * q;
-    o.s = *(const V*)so;
-    if constexpr (!F32) o.sl = *(const V*)(so + 256);
+    if constexpr (!ENDS) {
+      o.s = *(const V*)so;
+      if constexpr (!F32) o.sl = *(const V*)(so + 256);
+    }
     o.v = *(const V*)((const T*)a.vo + ((b * a.H + h) * a.vp + col) * 16 + 4 * q);
     if constexpr (KEY) {
 #pragma unroll
       for (int t = 0; t < NT; ++t) o.d[t] = *(const gf32x4*)(a.dec + (b * a.H + h) * NP + 16 * t + 4 * q);
     } else {
       const float* d = a.dec + (b * a.H + h) * 48;
-      o.d[0] = *(const gf32x4*)(d + 4 * q);
+      if constexpr (!ENDS) o.d[0] = *(const gf32x4*)(d + 4 * q);
       o.d[1] = *(const gf32x4*)(d + 16 + 4 * q);
       o.tot = d[32];
     }
   };
-  Ops A, B;
-  load(A, 0);
+  Ops o[DEPTH];
+#pragma unroll
+  for (int d = 0; d < DEPTH - 1; ++d) load(o[d], sg.i0 + d);
   // S[t]: rows 16 t + 4 q + r, column r16 of this wave's 16
   gf32x4 S[NT];
-  const size_t hs = (size_t)a.np * a.vp, half = (size_t)a.slots * a.H * hs;
-  float* st = a.state + ((size_t)sq.slot * a.H + h) * hs + (size_t)(4 * q) * a.vp + col;
-  {
-    const float* src = st + ((sq.pos0 - 1) & 1) * half;
+  auto read = [&](gf32x4 (&x)[NT], const float* src, bool live) {
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) S[t][r] = sq.pos0 > 0 ? src[(size_t)(16 * t + r) * a.vp] : 0.f;
+      for (int r = 0; r < 4; ++r) x[t][r] = live ? src[(size_t)(16 * t + r) * a.vp] : 0.f;
+  };
+  auto write = [&](float* dst) {
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) dst[(size_t)(16 * t + r) * a.vp] = S[t][r];
+  };
+  if (ENDS || a.nseg == 1 || sg.n == 1) {
+    read(S, st + ((sq.pos0 - 1) & 1) * half, sq.pos0 > 0 && seg == 0);
+    if constexpr (ENDS) {
+      if (seg == 0) write(seg_at(0));
+      if (seg + 1 >= sg.n) return;  // (the last one's end is the second walk's)
+    }
+  } else {
+    // (the state itself may already be the new one: the copies are read)
+    read(S, seg_at(min(seg, 1)), true);
+    for (int j = 2; j <= seg; ++j) {
+      gf32x4 e[NT];
+      read(e, seg_at(j), true);
+      const float* d = dec_at(j);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) S[t] = S[t] * *(const gf32x4*)(d + 16 * t + 4 * q) + e[t];
+    }
   }
-  const float skip = KEY ? 0.f : a.D[h];
+  gf32x4 D[ENDS && KEY ? NT : 1];  // decay of the segment
+  if constexpr (ENDS) {
+#pragma unroll
+    for (int t = 0; t < (KEY ? NT : 1); ++t) D[t] = gf32x4{1.f, 1.f, 1.f, 1.f};
+  }
+  const float skip = KEY || ENDS ? 0.f : a.D[h];
   auto step = [&](const Ops& o, int i) {
     gf32x4 y0 = {0.f, 0.f, 0.f, 0.f}, y1 = y0;
     gf32x4 vf;  // v in fp32: tokens 4 q + r, column r16
-    if constexpr (F32) {
-      vf = o.v;
+    if constexpr (F32) vf = o.v;
+    else
+      vf = gf32x4{__uint_as_float(o.v.x << 16), __uint_as_float(o.v.x & 0xffff0000u), __uint_as_float(o.v.y << 16),
+                  __uint_as_float(o.v.y & 0xffff0000u)};
+    if constexpr (ENDS) {
+    } else if constexpr (F32) {
 #pragma unroll
       for (int t = 0; t < NT; t += 2) {
         y0 = mfma4(o.q[t], S[t], y0);
@@ -402,8 +482,6 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
       if constexpr (!KEY) y0 *= o.d[0];
       y0 = mfma4(o.s, o.v, y0);
     } else {
-      vf = gf32x4{__uint_as_float(o.v.x << 16), __uint_as_float(o.v.x & 0xffff0000u), __uint_as_float(o.v.y << 16),
-                  __uint_as_float(o.v.y & 0xffff0000u)};
 #pragma unroll
       for (int t = 0; t < NT; t += 2) {
         uint2 h0, l0, h1, l1;
@@ -417,16 +495,18 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
       if constexpr (!KEY) y0 *= o.d[0];
       y0 = mfma32(o.s, o.sl, o.v, o.v, y0);
     }
-    if constexpr (!KEY) y0 += skip * vf;
+    if constexpr (!KEY && !ENDS) y0 += skip * vf;
     // the state at the block's end
     if constexpr (KEY) {
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         S[t] *= o.d[t];
+        if constexpr (ENDS) D[t] *= o.d[t];
         if constexpr (F32) S[t] = mfma4(o.k[t], o.v, S[t]);
         else S[t] = mfma32(o.k[t], o.kl[t], o.v, o.v, S[t]);
       }
     } else {
+      if constexpr (ENDS) D[0] *= o.tot;
       const gf32x4 vd = vf * o.d[1];
       uint2 vh, vl;
       if constexpr (!F32) split4(vd, vh, vl);
@@ -437,25 +517,30 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
         else S[t] = mfma32(o.k[t], o.k[t], vh, vl, S[t]);
       }
     }
-    if (col < a.dv) {
+    if (!ENDS && col < a.dv) {
       float* y = a.y + (size_t)(sq.row0 + 16 * i + 4 * q) * (a.H * a.dv) + h * a.dv + col;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (16 * i + 4 * q + r < sq.n) y[(size_t)r * a.H * a.dv] = y0[r];
     }
   };
-  for (int i = 0; i < nb; i += 2) {
-    load(B, i + 1);
-    step(A, i);
-    if (i + 1 >= nb) break;
-    load(A, i + 2);
-    step(B, i + 1);
+  for (int i = sg.i0; i < sg.i1; i += DEPTH) {
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) {
+      if (d && i + d >= sg.i1) break;
+      load(o[(d + DEPTH - 1) % DEPTH], i + d + DEPTH - 1);
+      step(o[d], i + d);
+    }
   }
-  float* dst = st + ((sq.pos0 + sq.n - 1) & 1) * half;
+  if constexpr (ENDS) {
+    write(seg_at(seg + 1));
+    if (vt == 0 && r16 == 0) {
 #pragma unroll
-  for (int t = 0; t < NT; ++t)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) dst[(size_t)(16 * t + r) * a.vp] = S[t][r];
+      for (int t = 0; t < NT; ++t) *(gf32x4*)(dec_at(seg + 1) + 16 * t + 4 * q) = D[KEY ? t : 0];
+    }
+  } else if (seg + 1 == sg.n) {
+    write(st + ((sq.pos0 + sq.n - 1) & 1) * half);
+  }
 }
 
 // ---- single tokens ----------------------------------------------------------------------------------
@@ -503,6 +588,7 @@ __global__ void __launch_bounds__(256) lin_step_kernel(LinScanArgs a) {
       if (n < a.N) {
         const int c = h * a.N + n;
         float z = a.a2_b[c];
+#pragma unroll 8
         for (int r = 0; r < a.rank; ++r) z = fmaf(a.a2[(size_t)c * a.rank + r], in[a.a_off + r], z);
         d = expf(-ls_softplus(-z) * a.inv_tau);
         k = in[a.k_off + c];
@@ -513,7 +599,7 @@ __global__ void __launch_bounds__(256) lin_step_kernel(LinScanArgs a) {
       sq[n] = q;
     }
   } else {
-    const int C = a.H * a.dv + 2 * a.G * a.N, rep = a.H / a.G, g = h / rep;
+    const int C = a.H * a.dv + 2 * a.G * a.N, rep = a.H / a.G, g = h / rep, p0 = pos % a.taps;
     const float dt = ls_softplus(in[a.dt_off + h] + a.dt_b[h]), dec = expf(-expf(a.a_log[h]) * dt);
     for (int i = tid; i < a.vp + 2 * a.np; i += 256) {
       int raw = -1;
@@ -528,11 +614,15 @@ __global__ void __launch_bounds__(256) lin_step_kernel(LinScanArgs a) {
         const float x = in[a.x_off + raw];
         u = fmaf(a.conv_w[(size_t)raw * a.taps + a.taps - 1], x, a.conv_b[raw]);
         float* ring = a.ring + (size_t)slot * a.taps * C + raw;
-        for (int d = 1; d < a.taps && d <= pos; ++d)
-          u = fmaf(a.conv_w[(size_t)raw * a.taps + a.taps - 1 - d], ring[(size_t)((pos - d) % a.taps) * C], u);
+#pragma unroll 4
+        for (int d = 1; d < a.taps; ++d) {
+          const int e = p0 - d + (p0 < d ? a.taps : 0);
+          const float xd = ring[(size_t)e * C];
+          u = fmaf(a.conv_w[(size_t)raw * a.taps + a.taps - 1 - d], d <= pos ? xd : 0.f, u);
+        }
         u = ls_silu<F32>(u);
         // (B and C are the group's: its first head keeps them; nobody reads this position's entry in this launch)
-        if (i < a.vp || h % rep == 0) ring[(size_t)(pos % a.taps) * C] = x;
+        if (i < a.vp || h % rep == 0) ring[(size_t)p0 * C] = x;
       }
       if (i < a.vp) {
         sv[i] = u;
@@ -585,8 +675,8 @@ __global__ void __launch_bounds__(256) lin_step_kernel(LinScanArgs a) {
 }
 
 // ---- norm and output gate ----------------------------------------------------------------------------
-// LANES threads per part of `n` numbers (64: four parts a workgroup, 256: one); PER numbers a thread
-template <bool F32, bool KEY, int LANES, int PER>
+// LANES threads per part of `n` numbers (64: four parts a workgroup, 256: one); PER pieces of V numbers a thread
+template <bool F32, bool KEY, int LANES, int PER, int V>
 __global__ void __launch_bounds__(256) lin_norm_kernel(LinScanArgs a, int parts, int n) {
   __shared__ float red[4];
   const int per = 256 / LANES, p = blockIdx.x * per + (int)threadIdx.x / LANES, lane = threadIdx.x % LANES, row = blockIdx.y;
@@ -594,22 +684,28 @@ __global__ void __launch_bounds__(256) lin_norm_kernel(LinScanArgs a, int parts,
   const int c0 = p * n;
   const float* y = a.y + (size_t)row * a.H * a.dv + c0;
   const float* z = a.in + (size_t)row * a.ld + a.z_off + c0;
-  float v[PER], gt[PER], ss = 0.f;
+  const float* nw = a.norm_w + (KEY ? 0 : c0);
+  typedef float vec __attribute__((ext_vector_type(V)));
+  vec v[PER], gt[PER], w[PER];
+  float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
-    const int c = lane + LANES * i;
-    v[i] = gt[i] = 0.f;
+    const int c = V * (lane + LANES * i);
+    v[i] = gt[i] = w[i] = vec(0.f);
     if (c < n) {
-      v[i] = y[c];
-      gt[i] = z[c];
+      v[i] = *(const vec*)(y + c);
+      gt[i] = *(const vec*)(z + c);
+      w[i] = *(const vec*)(nw + c);
     }
   }
 #pragma unroll
-  for (int i = 0; i < PER; ++i) {
-    gt[i] = ls_silu<F32>(gt[i]);
-    if constexpr (!KEY) v[i] *= gt[i];
-    ss += v[i] * v[i];
-  }
+  for (int i = 0; i < PER; ++i)
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      gt[i][e] = ls_silu<F32>(gt[i][e]);
+      if constexpr (!KEY) v[i][e] *= gt[i][e];
+      ss += v[i][e] * v[i][e];
+    }
   if constexpr (LANES == 64) {
 #pragma unroll
     for (int d = 32; d; d >>= 1) ss += __shfl_xor(ss, d, 64);
@@ -619,32 +715,44 @@ __global__ void __launch_bounds__(256) lin_norm_kernel(LinScanArgs a, int parts,
   const float inv = a.out_scale / sqrtf(ss / (float)n + a.eps);
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
-    const int c = lane + LANES * i;
+    const int c = V * (lane + LANES * i);
     if (c >= n) break;
-    const float w = a.norm_w[KEY ? c : c0 + c];
-    put1<F32>(a.out, (size_t)row * a.ldo + c0 + c, KEY ? v[i] * inv * w * gt[i] : v[i] * inv * w);
+    vec o = v[i] * inv * w[i];
+    if constexpr (KEY) o *= gt[i];
+    const size_t at = (size_t)row * a.ldo + c0 + c;
+    if constexpr (V == 1) put1<F32>(a.out, at, o[0]);
+    else if constexpr (F32) *(vec*)((float*)a.out + at) = o;
+    else *(uint2*)((bf16_t*)a.out + at) = make_uint2(pk_bf16(o[0], o[1]), pk_bf16(o[2], o[3]));
   }
+}
+
+template <bool F32, bool KEY, int V>
+static void lin_norm_v(const LinScanArgs& a, hipStream_t st) {
+  const int parts = KEY ? a.H : a.norm_parts, n = a.H * a.dv / parts, m = (n + V - 1) / V;
+  auto wave = [&](auto per) {
+    hipLaunchKernelGGL((lin_norm_kernel<F32, KEY, 64, decltype(per)::value, V>), dim3((parts + 3) / 4, a.rows), dim3(256), 0, st, a,
+                       parts, n);
+  };
+  auto block = [&](auto per) {
+    hipLaunchKernelGGL((lin_norm_kernel<F32, KEY, 256, decltype(per)::value, V>), dim3(parts, a.rows), dim3(256), 0, st, a, parts,
+                       n);
+  };
+  if (m <= 64) wave(std::integral_constant<int, 1>{});
+  else if (m <= 128) wave(std::integral_constant<int, 2>{});
+  else if (m <= 256) block(std::integral_constant<int, 1>{});
+  else if (m <= 512) block(std::integral_constant<int, 2>{});
+  else if (m <= 1024) block(std::integral_constant<int, 4>{});
+  else if (m <= 2048) block(std::integral_constant<int, 8>{});
+  else if (m <= 4096) block(std::integral_constant<int, 16>{});
+  else block(std::integral_constant<int, 64>{});
 }
 
 template <bool F32, bool KEY>
 static void lin_norm(const LinScanArgs& a, hipStream_t st) {
-  const int parts = KEY ? a.H : a.norm_parts, n = a.H * a.dv / parts;
-  auto wave = [&](auto per) {
-    hipLaunchKernelGGL((lin_norm_kernel<F32, KEY, 64, decltype(per)::value>), dim3((parts + 3) / 4, a.rows), dim3(256), 0, st, a,
-                       parts, n);
-  };
-  auto block = [&](auto per) {
-    hipLaunchKernelGGL((lin_norm_kernel<F32, KEY, 256, decltype(per)::value>), dim3(parts, a.rows), dim3(256), 0, st, a, parts, n);
-  };
-  if (n <= 64) wave(std::integral_constant<int, 1>{});
-  else if (n <= 128) wave(std::integral_constant<int, 2>{});
-  else if (n <= 256) wave(std::integral_constant<int, 4>{});
-  else if (n <= 512) wave(std::integral_constant<int, 8>{});
-  else if (n <= 1024) block(std::integral_constant<int, 4>{});
-  else if (n <= 2048) block(std::integral_constant<int, 8>{});
-  else if (n <= 4096) block(std::integral_constant<int, 16>{});
-  else if (n <= 8192) block(std::integral_constant<int, 32>{});
-  else block(std::integral_constant<int, 64>{});
+  const int n = a.H * a.dv / (KEY ? a.H : a.norm_parts);
+  const bool wide = n % 4 == 0 && a.ld % 4 == 0 && a.z_off % 4 == 0 && a.ldo % 4 == 0 && ((uintptr_t)a.out & 15) == 0;
+  if (wide) lin_norm_v<F32, KEY, 4>(a, st);
+  else lin_norm_v<F32, KEY, 1>(a, st);
 }
 
 template <bool F32, bool KEY>
@@ -663,7 +771,10 @@ static void lin_go(const LinScanArgs& a, hipStream_t st) {
       if (lds > 150 * 1024) throw std::runtime_error("linear scan: decay projection too wide");
       hipLaunchKernelGGL((lin_key_prep_kernel<F32, NT>), dim3(a.H, nblk), dim3(256), lds, st, a);
     }
-    hipLaunchKernelGGL((lin_walk_kernel<F32, KEY, NT>), dim3((a.H * (a.vp / 16) + 3) / 4, a.n_seqs), dim3(256), 0, st, a);
+    const int wg = (a.H * (a.vp / 16) + 3) / 4;
+    if (a.nseg > 1)
+      hipLaunchKernelGGL((lin_walk_kernel<F32, KEY, NT, true>), dim3(wg, a.n_seqs, a.nseg - 1), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((lin_walk_kernel<F32, KEY, NT, false>), dim3(wg, a.n_seqs, a.nseg), dim3(256), 0, st, a);
   };
   if constexpr (!KEY) {
     const dim3 grid((a.H * a.vp + 2 * a.G * a.np + LC_T - 1) / LC_T, nblk);
@@ -683,6 +794,12 @@ static void lin_go(const LinScanArgs& a, hipStream_t st) {
   lin_norm<F32, KEY>(a, st);
 }
 
+// segments a portion of at most `blocks` blocks is walked in: enough waves for the chip, one a SIMD
+int lin_segments(int H, int vp, int n_seqs, int blocks) {
+  const int waves = std::max(1, H * (vp / 16) * n_seqs);
+  return std::max(1, std::min({(1024 + waves / 2) / waves, LIN_SEGS / std::max(1, n_seqs), blocks / LIN_SEG_MIN, 8}));
+}
+
 void launch_lin_scan(const LinScanArgs& a, hipStream_t st) {
   const bool key = a.kind == LIN_KEY;
   if (a.H < 1 || a.G < 1 || a.H % a.G || (key && a.G != a.H) || a.np != lin_pad_n(a.N) || !a.np || a.vp % 16 || a.vp < a.dv ||
@@ -691,6 +808,8 @@ void launch_lin_scan(const LinScanArgs& a, hipStream_t st) {
   if (!key && (a.taps < 1 || a.taps > 16 || a.norm_parts < 1 || (a.H * a.dv) % a.norm_parts || a.H * a.dv / a.norm_parts > 16384))
     throw std::runtime_error("linear scan: bad convolution or norm");
   if ((a.seqs ? a.n_seqs : a.n) < 1) return;
+  if (a.seqs && (a.nseg < 1 || (a.nseg > 1 && (!a.seg || !a.seg_dec || a.nseg * a.n_seqs > LIN_SEGS))))
+    throw std::runtime_error("linear scan: bad segments");
   if (key) {
     if (a.f32) lin_go<true, true>(a, st);
     else lin_go<false, true>(a, st);

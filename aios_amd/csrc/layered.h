@@ -159,6 +159,7 @@ class LayeredDecoder {
     int max_len;                          // of the absorbed rows
     std::vector<std::pair<int, Piece>> pf;  // expanded path: first row, piece
     int n_chunks, split, n_seqs;          // step batches: chunks of the recurrences, pieces
+    int longest;                          // tokens of the longest piece
   };
   void layer16(int k, const RowSet& r);  // k: run
   void layer32(int k, const RowSet& r);
@@ -223,7 +224,7 @@ class LayeredDecoder {
   int4* moe_tiles_ = nullptr;
   // linear recurrences: operands of the blocks, outputs before the norm
   void *lin_qo_ = nullptr, *lin_ko_ = nullptr, *lin_kr_ = nullptr, *lin_vo_ = nullptr, *lin_so_ = nullptr;
-  float *lin_dec_ = nullptr, *lin_y_ = nullptr;
+  float *lin_dec_ = nullptr, *lin_y_ = nullptr, *lin_seg_ = nullptr, *lin_seg_dec_ = nullptr;
   int moe_max_tiles_ = 0;
   // RMSNorm split across the short GEMMs (GemmQArgs nrm_*): set when the residual in x_ already went
   // through bf16(x * g_next) and per-tile sums

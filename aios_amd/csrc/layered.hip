@@ -175,7 +175,7 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
     D.kout = D.gn;
     D.shf = s.mlp == MLP_MOE ? s.shared_ff : 0;
     D.shp = up(D.shf, 64);
-    if (s.mlp == MLP_ACT) D.fp = up_n(D.ff);
+    if (s.mlp == MLP_ACT) D.fp = D.ff > 4096 ? up(D.ff, 512) : up_n(D.ff);  // (the GEMV engine's K: whole 512s)
     D.glu = s.mlp == MLP_MOE ? D.shp : D.fp;
     D.router_off = s.resid_gate ? dp_ : 0;
     D.n2 = up_n(D.router_off + (s.mlp == MLP_MOE ? up(s.experts, 64) : 0));
@@ -651,7 +651,7 @@ void LayeredDecoder::finalize() {
   size_t qa = 0, part = 0, kvw = 0, flat = 0;
   size_t e_act = 0, e_gu = 0, pairs = 0;  // experts
   LinWs lw = {0, 0, 0, 0, 0, 0};
-  size_t lin_y = 0;
+  size_t lin_y = 0, lin_seg = 0, lin_seg_dec = 0;
   int rp = 0;
   for (int i = 0; i < nl_; ++i) {
     const Dims& D = dims_[i];
@@ -663,6 +663,8 @@ void LayeredDecoder::finalize() {
       lw = LinWs{std::max(lw.qo, l.qo), std::max(lw.ko, l.ko), std::max(lw.kr, l.kr),
                  std::max(lw.vo, l.vo), std::max(lw.so, l.so), std::max(lw.dec, l.dec)};
       lin_y = std::max(lin_y, (size_t)R * D.lH * D.ldv);
+      lin_seg = std::max(lin_seg, (size_t)LIN_SEGS * D.lH * D.lnp * D.lvp);
+      lin_seg_dec = std::max(lin_seg_dec, (size_t)LIN_SEGS * D.lH * D.lnp);
     }
     kout = std::max({kout, D.kout, D.glu});
     fp = std::max(fp, seq_ ? D.glu : D.fp);
@@ -717,7 +719,9 @@ void LayeredDecoder::finalize() {
       lin_so_ = operand(nb * lw.so);
       lin_dec_ = falloc(nb * lw.dec);
       lin_y_ = falloc(lin_y);
-      e_.ws_bytes_ += (nb * lw.dec + lin_y) * 4;
+      lin_seg_ = falloc(lin_seg);
+      lin_seg_dec_ = falloc(lin_seg_dec);
+      e_.ws_bytes_ += (nb * lw.dec + lin_y + lin_seg + lin_seg_dec) * 4;
     }
     if (wp) {
       agg_ = falloc((size_t)max_chunks_ * 3 * wp);
@@ -1028,6 +1032,8 @@ void LayeredDecoder::linear(int k, const RowSet& r) {
   if (!r.decode) {
     a.seqs = st_seqs_; a.n_seqs = r.n_seqs;
     a.chunks = st_chunks_; a.n_chunks = r.n_chunks;
+    a.nseg = lin_segments(D.lH, D.lvp, r.n_seqs, (r.longest + LIN_T - 1) / LIN_T);
+    a.seg = lin_seg_; a.seg_dec = lin_seg_dec_;
   }
   a.pos = r.pos; a.slot = r.slot; a.n = a.rows = r.n;
   a.qo = lin_qo_; a.ko = lin_ko_; a.kr = lin_kr_; a.vo = lin_vo_; a.so = lin_so_; a.dec = lin_dec_;
@@ -1395,7 +1401,7 @@ void LayeredDecoder::run(const RowSet& r) {
 void LayeredDecoder::decode_forward(int B) {
   RowSet r;
   r.tokens = e_.d_tokens_; r.pos = e_.d_pos_; r.slot = e_.d_slot_; r.run = nullptr;
-  r.n_chunks = r.split = r.n_seqs = 0;
+  r.n_chunks = r.split = r.n_seqs = r.longest = 0;
   r.n = r.n_abs = B;
   r.decode = true;
   r.max_len = e_.cfg_.max_ctx;
@@ -1435,7 +1441,7 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
   ScanChunk* chunks = (ScanChunk*)(hr + R);
   ScanSeq* seqs = (ScanSeq*)(h_step_ + ((const int*)st_seqs_ - d_step_));
   LatentTile* tiles = (LatentTile*)(h_step_ + ((const int*)st_tiles_ - d_step_));
-  r.n_chunks = r.split = r.n_seqs = 0;
+  r.n_chunks = r.split = r.n_seqs = r.longest = 0;
   int row = 0, nt = 0;
   for (int o = 0; o < (int)order.size(); ++o) {
     const Piece& q = pieces[order[o]];
@@ -1447,6 +1453,7 @@ void LayeredDecoder::forward(const std::vector<Piece>& pieces, std::vector<int>&
       hr[row + k] = k ? 0 : q.n;
     }
     const int c0 = r.n_chunks;
+    r.longest = std::max(r.longest, q.n);
     seqs[r.n_seqs++] = ScanSeq{row, q.n, q.slot, q.start, 2 * c0};
     if (c0 + (q.n + SCAN_CHUNK - 1) / SCAN_CHUNK > max_chunks_) throw std::runtime_error("layered forward: too many pieces");
     for (int k = 0; k < q.n; k += SCAN_CHUNK)

@@ -148,11 +148,12 @@ bool gqa_supports(int dkp, int dvp);
 //             the input columns, q times q_scale (G = H).  out = rms(o) per head * norm_w [dv] * silu(z).
 // Portions run in blocks of LIN_T tokens: what a block needs besides the state it starts from (operands, decays,
 // scores between its own tokens) is prepared for all blocks side by side; then one wave per head and 16 columns of
-// v walks the blocks with its part of S in registers.  The state is kept twice, by parity of the position it was left
+// v walks the blocks with its part of S in registers, long portions in segments side by side.  The state is kept twice, by parity of the position it was left
 // at, and the convolution's inputs in a ring of `taps` positions, so that a single token that is run again at the
 // same position finds what it started from.
 enum LinKind : int { LIN_HEAD = 1, LIN_KEY = 2 };
 constexpr int LIN_T = 16;
+constexpr int LIN_SEGS = 16, LIN_SEG_MIN = 8;  // segments of a step at most; blocks of a segment at least
 struct ScanSeq {
   int row0, n, slot, pos0;
   int b0;           // index of its first block in the operand buffers
@@ -181,6 +182,8 @@ struct LinScanArgs {
   // operands of the blocks (bf16 or fp32), see lin_ws
   void *qo, *ko, *kr, *vo, *so;
   float* dec;
+  int nseg;                   // segments a portion is walked in (lin_segments); more than 1: the states and decays at
+  float *seg, *seg_dec;       // their borders, [n_seqs][nseg][H] x [np][vp] and x [np]
   float* y;                   // [rows][H dv]
   const float* norm_w;
   int norm_parts;
@@ -191,6 +194,7 @@ struct LinScanArgs {
 };
 int lin_pad_n(int n);                                // 0: not served
 struct LinWs { size_t qo, ko, kr, vo, so, dec; };    // numbers per block
+int lin_segments(int H, int vp, int n_seqs, int blocks);  // blocks: of the longest portion
 LinWs lin_ws(int kind, int H, int G, int np, int vp, bool f32);
 void launch_lin_scan(const LinScanArgs& a, hipStream_t st);
 

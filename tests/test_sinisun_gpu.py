@@ -62,9 +62,10 @@ KEY = [(3, 3, 24, 40, 12, 5.0), (6, 6, 32, 64, 16, 16.0), (1, 1, 130, 200, 40, 1
 
 
 @pytest.mark.parametrize("f32", [0, 1])
+@pytest.mark.parametrize("nseg, shift", [(1, 5), (4, 4)])
 @pytest.mark.parametrize("kind, sizes", [("head", s) for s in HEAD] + [("key", s) for s in KEY])
-def test_linear_scan_kernels(kind, sizes, f32):
-    """Portions of unequal lengths at block and chunk borders, continued by others; single tokens, some of them twice;
+def test_linear_scan_kernels(kind, sizes, nseg, shift, f32):
+    """Columns at any offset and at aligned ones; portions in segments; portions of unequal lengths at block and chunk borders, continued by others; single tokens, some of them twice;
     slots taken over by a new sequence; state and convolution inputs that no earlier sequence may leak."""
     m = E()
     H, G, N, dv = sizes[:4]
@@ -79,21 +80,24 @@ def test_linear_scan_kernels(kind, sizes, f32):
         C = inner + 2 * G * N
         w = dict(conv_w=rnd(C, taps) / math.sqrt(taps), conv_b=rnd(C) * 0.4, dt_b=rnd(H) - 1.5, a_log=rnd(H) - 1, D=1 + rnd(H) / 2)
         width = 2 * inner + 2 * G * N + H
-        off = dict(z_off=5, x_off=5 + inner, dt_off=5 + 2 * inner + 2 * G * N, taps=taps, norm_parts=parts)
+        off = dict(z_off=shift, x_off=shift + inner, dt_off=shift + 2 * inner + 2 * G * N, taps=taps, norm_parts=parts)
     else:
         rank, tau = sizes[4:]
         w = dict(a2=rnd(H * N, rank) / math.sqrt(rank), a2_b=2 + rnd(H * N))
         width = H * (2 * N + 2 * dv) + rank
-        off = dict(q_off=5, k_off=5 + H * N, v_off=5 + 2 * H * N, z_off=5 + 2 * H * N + inner, a_off=5 + 2 * H * N + 2 * inner,
+        off = dict(q_off=shift, k_off=shift + H * N, v_off=shift + 2 * H * N, z_off=shift + 2 * H * N + inner,
+                   a_off=shift + 2 * H * N + 2 * inner,
                    rank=rank, q_scale=N ** -0.5, inv_tau=1 / tau)
 
-    def ref(x):
+    def ref(x, rounded=False):
         x = x.double()
         T = x.shape[0]
         W = {k: v.double() for k, v in w.items()}
         if head:
             z, u, st = x[:, :inner], x[:, inner:-H], x[:, -H:]
             u = O.silu(O.causal_conv(u, W["conv_w"], W["conv_b"]))
+            if rounded:
+                u = u.float().bfloat16().double()
             X = u[:, :inner].view(T, H, dv)
             B, Cc = (u[:, inner + i * G * N:inner + (i + 1) * G * N].reshape(T, G, N).repeat_interleave(H // G, 1) for i in (0, 1))
             st = O.softplus(st + W["dt_b"])
@@ -105,39 +109,42 @@ def test_linear_scan_kernels(kind, sizes, f32):
         o = O.decayed_outer(al, k.reshape(T, H, N), v.reshape(T, H, dv), q.reshape(T, H, N) * N ** -0.5)
         return osc * (O.rms(o, eps) * norm_w.double()).reshape(T, inner) * O.silu(z)
 
-    X = {s: bf(rnd(n, width)) for s, n in {0: 230, 2: 140, 5: 90, 3: 100}.items()}
-    want = {s: ref(x) for s, x in X.items()}
+    X = {s: bf(rnd(n, width)) for s, n in {0: 230, 2: 140, 5: 90, 3: 100, 4: 700, 1: 420}.items()}
+    # 16-bit portions round the convolution's outputs: where an output nearly cancels, that is what is left of it
+    soft = lambda x: (ref(x, True) - ref(x)).abs().amax(1, keepdim=True) * (2 if head and not f32 else 0)
+    want = {s: (ref(x), soft(x)) for s, x in X.items()}
     D = {k: dev(v) for k, v in dict(w, norm_w=norm_w).items()}
     state = torch.full((2, slots, H, np_, vp), 1e30, device="cuda")
     ring = torch.full((slots, sizes[4], inner + 2 * G * N), 1e30, device="cuda") if head else None
+    seg, seg_dec = (torch.full((16, H, np_) + e, float("nan"), device="cuda") for e in ((vp,), ()))
     ws = m.lin_ws(m.LIN_HEAD if head else m.LIN_KEY, H, G, np_, vp, bool(f32))
-    buf = {k: torch.full((2 * 24 * n + 4096,), float("nan"), dtype=torch.float32 if k == "dec" else dt, device="cuda")
+    buf = {k: torch.full((2 * 40 * n + 4096,), float("nan"), dtype=torch.float32 if k == "dec" else dt, device="cuda")
            for k, n in zip(("qo", "ko", "kr", "vo", "so", "dec"), ws)}
-    work, ld = torch.zeros(24 * 16, dtype=torch.int32, device="cuda"), 5 + width + 3
+    work, ld = torch.zeros(64 * 16, dtype=torch.int32, device="cuda"), pad(shift + width + 3, 4) + shift % 4
 
     def go(entries, decode=False):
         rows = torch.cat([X[s][st:st + n] for s, st, n in entries])
         n = rows.shape[0]
         inp = torch.full((n, ld), 1e30)
-        inp[:, 5:5 + width] = rows
+        inp[:, shift:shift + width] = rows
         inp, out, y = dev(inp), torch.zeros(n, inner + 64, dtype=dt, device="cuda"), torch.zeros(n, inner, device="cuda")
         pieces, at = [], 0
         for s, st, k in entries:
             pieces.append([at, k, s, st])
             at += k
         pd, sd = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in zip(*[(p[3], p[2]) for p in pieces]))
-        print(kind, sizes, f32, entries, flush=True)
+        print(kind, sizes, nseg, shift, f32, entries, flush=True)
         m.lin_scan([] if decode else pieces, kind=m.LIN_HEAD if head else m.LIN_KEY, H=H, G=G, N=N, dv=dv, vp=vp, inp=inp.data_ptr(),
                    ld=ld, **off, **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr() if head else 0,
-                   state=state.data_ptr(), slots=slots, pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
+                   state=state.data_ptr(), slots=slots, nseg=nseg, seg=seg.data_ptr(), seg_dec=seg_dec.data_ptr(), pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
                    **{k: v.data_ptr() for k, v in buf.items()}, y=y.data_ptr(), eps=eps, out_scale=osc, out=out.data_ptr(),
                    ldo=inner + 64, f32=f32, work=work.data_ptr(), stream=stream())
         torch.cuda.synchronize()
-        ref = torch.cat([want[s][st:st + k] for s, st, k in entries])
-        got = out.cpu()[:, :inner].double()
-        err, rms = float((got - ref).abs().max() / ref.abs().max()), float((got - ref).pow(2).mean().sqrt() / ref.pow(2).mean().sqrt())
+        exact, slack = (torch.cat([want[s][i][st:st + k] for s, st, k in entries]) for i in (0, 1))
+        miss = ((out.cpu()[:, :inner].double() - exact).abs() - slack).clamp(min=0)
+        err, rms = float(miss.max() / exact.abs().max()), float(miss.pow(2).mean().sqrt() / exact.pow(2).mean().sqrt())
         print(err, rms, flush=True)
-        assert (out[:, inner:] == 0).all() and err < (2e-5 if f32 else 3e-2) and rms < (4e-6 if f32 else 5e-3), (entries, err, rms)
+        assert (out[:, inner:] == 0).all() and err < (2e-5 if f32 else 3e-2) and rms < (1e-5 if f32 else 5e-3), (entries, err, rms)
 
     go([(0, 0, 1), (2, 0, 64), (5, 0, 2), (3, 0, 31)])
     go([(0, 1, 100), (2, 64, 17), (5, 2, 1)])
@@ -146,13 +153,16 @@ def test_linear_scan_kernels(kind, sizes, f32):
     go([(5, 4, 1), (2, 82, 1)], True)
     go([(5, 4, 1), (2, 82, 1)])                                     # again, as portions of one token
     go([(2, 83, 48), (0, 102, 128), (3, 32, 66), (5, 5, 3)])        # even lengths: in and out at one parity
+    go([(4, 0, 390), (1, 0, 130)])                                  # several segments, the last one short
+    go([(1, 130, 290), (4, 390, 1), (5, 8, 2)])                     # ... from a state, in place (even length)
+    go([(4, 391, 309), (5, 10, 6)])
     X[0] = bf(rnd(70, width))
-    want[0] = ref(X[0])
-    go([(0, 0, 2), (5, 8, 82)])
+    want[0] = ref(X[0]), soft(X[0])
+    go([(0, 0, 2), (5, 16, 74)])
     go([(0, 2, 1)], True)
     go([(0, 3, 49)])
     X[3] = bf(rnd(9, width))
-    want[3] = ref(X[3])
+    want[3] = ref(X[3]), soft(X[3])
     for t in range(9):
         go([(3, t, 1)], True)
 
