@@ -25,7 +25,7 @@
 
 namespace aios {
 
-typedef short ls16x4 __attribute__((ext_vector_type(4)));
+typedef unsigned int lu2 __attribute__((ext_vector_type(2)));
 
 int lin_pad_n(int n) {
   for (int t : {32, 64, 96, 128, 192, 256})
@@ -58,11 +58,14 @@ __device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t&
   hi = pk_bf16(a, b);
   lo = pk_bf16(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
 }
-__device__ __forceinline__ void split4(gf32x4 v, uint2& hi, uint2& lo) {
-  split2(v[0], v[1], hi.x, lo.x);
-  split2(v[2], v[3], hi.y, lo.y);
+__device__ __forceinline__ void split4(gf32x4 v, lu2& hi, lu2& lo) {
+  uint32_t h0, l0, h1, l1;
+  split2(v[0], v[1], h0, l0);
+  split2(v[2], v[3], h1, l1);
+  hi = lu2{h0, h1};
+  lo = lu2{l0, l1};
 }
-__device__ __forceinline__ gf32x4 mfma32(uint2 a0, uint2 a1, uint2 b0, uint2 b1, gf32x4 c) {
+__device__ __forceinline__ gf32x4 mfma32(lu2 a0, lu2 a1, lu2 b0, lu2 b1, gf32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(gbf16x8, make_uint4(a0.x, a0.y, a1.x, a1.y)),
                                                  __builtin_bit_cast(gbf16x8, make_uint4(b0.x, b0.y, b1.x, b1.y)), c, 0, 0, 0);
 }
@@ -208,7 +211,7 @@ __global__ void __launch_bounds__(256) lin_score_kernel(LinScanArgs a, int nscor
       acc = mfma4(*(const gf32x4*)((const float*)a.kr + at + 256), *(const gf32x4*)((const float*)a.qo + at + 256), acc);
     } else {
       const bf16_t *kr = (const bf16_t*)a.kr + at, *qr = (const bf16_t*)a.qo + at;
-      acc = mfma32(*(const uint2*)kr, *(const uint2*)(kr + 256), *(const uint2*)qr, *(const uint2*)(qr + 256), acc);
+      acc = mfma32(*(const lu2*)kr, *(const lu2*)(kr + 256), *(const lu2*)qr, *(const lu2*)(qr + 256), acc);
     }
   }
 #pragma unroll
@@ -221,10 +224,10 @@ __global__ void __launch_bounds__(256) lin_score_kernel(LinScanArgs a, int nscor
   if constexpr (F32) {
     *(gf32x4*)((float*)a.so + at) = acc;
   } else {
-    uint2 hi, lo;
+    lu2 hi, lo;
     split4(acc, hi, lo);
-    *(uint2*)((bf16_t*)a.so + at) = hi;
-    *(uint2*)((bf16_t*)a.so + at + 256) = lo;
+    *(lu2*)((bf16_t*)a.so + at) = hi;
+    *(lu2*)((bf16_t*)a.so + at + 256) = lo;
   }
 }
 
@@ -346,7 +349,7 @@ template <bool F32, bool KEY, int NT>
 struct LinOps;
 template <bool KEY, int NT>
 struct LinOps<false, KEY, NT> {
-  uint2 q[NT], ql[KEY ? NT : 1], k[NT], kl[KEY ? NT : 1], s, sl, v;
+  lu2 q[NT], ql[KEY ? NT : 1], k[NT], kl[KEY ? NT : 1], s, sl, v;
   gf32x4 d[KEY ? NT : 2];
   float tot;
 };
@@ -378,7 +381,7 @@ template <bool F32, bool KEY, int NT, bool ENDS>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) lin_walk_kernel(LinScanArgs a) {
   constexpr int NP = 16 * NT, DEPTH = lin_depth<F32, KEY, NT>();
   using T = std::conditional_t<F32, float, bf16_t>;
-  using V = std::conditional_t<F32, gf32x4, uint2>;
+  using V = std::conditional_t<F32, gf32x4, lu2>;
   const int lane = threadIdx.x & 63, nvt = a.vp >> 4;
   const int w = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
   if (w >= a.H * nvt) return;
@@ -396,7 +399,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
   auto dec_at = [&](int j) { return a.seg_dec + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * a.np; };
   const size_t plane = (size_t)2 * a.n_chunks * a.H * NP * 16;
   using Ops = LinOps<F32, KEY, NT>;
-  auto load = [&](Ops& o, int i) {
+  auto load = [&](Ops& o, int i) __attribute__((always_inline)) {
     const size_t b = sq.b0 + min(i, sg.i1 - 1);  // (past the end: re-reads)
     const T* qo = (const T*)a.qo + (b * ng + g) * NP * 16 + r16 * 16 + 4 * q;
     const T* ko = (const T*)a.ko + (b * ng + g) * NP * 16 + r16 * 16 + 4 * q;
@@ -425,15 +428,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
     }
   };
   Ops o[DEPTH];
-#pragma unroll
-  for (int d = 0; d < DEPTH - 1; ++d) load(o[d], sg.i0 + d);
+  static_for<DEPTH - 1>([&](auto d) { load(o[d], sg.i0 + d); });
   // S[t]: rows 16 t + 4 q + r, column r16 of this wave's 16
   gf32x4 S[NT];
-  auto read = [&](gf32x4 (&x)[NT], const float* src, bool live) {
+  auto read = [&](gf32x4 (&x)[NT], const float* src) __attribute__((always_inline)) {
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) x[t][r] = live ? src[(size_t)(16 * t + r) * a.vp] : 0.f;
+      for (int r = 0; r < 4; ++r) x[t][r] = src[(size_t)(16 * t + r) * a.vp];
   };
   auto write = [&](float* dst) {
 #pragma unroll
@@ -442,17 +444,22 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
       for (int r = 0; r < 4; ++r) dst[(size_t)(16 * t + r) * a.vp] = S[t][r];
   };
   if (ENDS || a.nseg == 1 || sg.n == 1) {
-    read(S, st + ((sq.pos0 - 1) & 1) * half, sq.pos0 > 0 && seg == 0);
+    if (sq.pos0 > 0 && seg == 0) {
+      read(S, st + ((sq.pos0 - 1) & 1) * half);
+    } else {
+#pragma unroll
+      for (int t = 0; t < NT; ++t) S[t] = gf32x4{0.f, 0.f, 0.f, 0.f};
+    }
     if constexpr (ENDS) {
       if (seg == 0) write(seg_at(0));
       if (seg + 1 >= sg.n) return;  // (the last one's end is the second walk's)
     }
   } else {
     // (the state itself may already be the new one: the copies are read)
-    read(S, seg_at(min(seg, 1)), true);
+    read(S, seg_at(min(seg, 1)));
     for (int j = 2; j <= seg; ++j) {
       gf32x4 e[NT];
-      read(e, seg_at(j), true);
+      read(e, seg_at(j));
       const float* d = dec_at(j);
 #pragma unroll
       for (int t = 0; t < NT; ++t) S[t] = S[t] * *(const gf32x4*)(d + 16 * t + 4 * q) + e[t];
@@ -464,7 +471,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
     for (int t = 0; t < (KEY ? NT : 1); ++t) D[t] = gf32x4{1.f, 1.f, 1.f, 1.f};
   }
   const float skip = KEY || ENDS ? 0.f : a.D[h];
-  auto step = [&](const Ops& o, int i) {
+  auto step = [&](const Ops& o, int i) __attribute__((always_inline)) {
     gf32x4 y0 = {0.f, 0.f, 0.f, 0.f}, y1 = y0;
     gf32x4 vf;  // v in fp32: tokens 4 q + r, column r16
     if constexpr (F32) vf = o.v;
@@ -484,7 +491,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
     } else {
 #pragma unroll
       for (int t = 0; t < NT; t += 2) {
-        uint2 h0, l0, h1, l1;
+        lu2 h0, l0, h1, l1;
         split4(S[t], h0, l0);
         split4(S[t + 1], h1, l1);
         y0 = mfma32(o.q[t], o.q[t + 1], h0, h1, y0);
@@ -508,7 +515,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
     } else {
       if constexpr (ENDS) D[0] *= o.tot;
       const gf32x4 vd = vf * o.d[1];
-      uint2 vh, vl;
+      lu2 vh, vl;
       if constexpr (!F32) split4(vd, vh, vl);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
@@ -519,19 +526,25 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) l
     }
     if (!ENDS && col < a.dv) {
       float* y = a.y + (size_t)(sq.row0 + 16 * i + 4 * q) * (a.H * a.dv) + h * a.dv + col;
+      if (16 * i + 16 <= sq.n) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (16 * i + 4 * q + r < sq.n) y[(size_t)r * a.H * a.dv] = y0[r];
+        for (int r = 0; r < 4; ++r) y[(size_t)r * a.H * a.dv] = y0[r];
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (16 * i + 4 * q + r < sq.n) y[(size_t)r * a.H * a.dv] = y0[r];
+      }
     }
   };
-  for (int i = sg.i0; i < sg.i1; i += DEPTH) {
-#pragma unroll
-    for (int d = 0; d < DEPTH; ++d) {
-      if (d && i + d >= sg.i1) break;
+  int i = sg.i0;
+  for (; i + DEPTH <= sg.i1; i += DEPTH)
+    static_for<DEPTH>([&](auto d) __attribute__((always_inline)) {
       load(o[(d + DEPTH - 1) % DEPTH], i + d + DEPTH - 1);
       step(o[d], i + d);
-    }
-  }
+    });
+  static_for<DEPTH - 1>([&](auto d) __attribute__((always_inline)) {
+    if (i + d < sg.i1) step(o[d], i + d);
+  });
   if constexpr (ENDS) {
     write(seg_at(seg + 1));
     if (vt == 0 && r16 == 0) {
@@ -722,7 +735,7 @@ __global__ void __launch_bounds__(256) lin_norm_kernel(LinScanArgs a, int parts,
     const size_t at = (size_t)row * a.ldo + c0 + c;
     if constexpr (V == 1) put1<F32>(a.out, at, o[0]);
     else if constexpr (F32) *(vec*)((float*)a.out + at) = o;
-    else *(uint2*)((bf16_t*)a.out + at) = make_uint2(pk_bf16(o[0], o[1]), pk_bf16(o[2], o[3]));
+    else *(lu2*)((bf16_t*)a.out + at) = lu2{pk_bf16(o[0], o[1]), pk_bf16(o[2], o[3])};
   }
 }
 
