@@ -363,8 +363,10 @@ struct LinOps<true, KEY, NT> {
 template <bool F32, bool KEY, int NT>
 constexpr int lin_depth() {
   if (F32) return 2;
-  return KEY ? (NT <= 6 ? 4 : NT <= 8 ? 3 : 2) : (NT <= 8 ? 4 : NT <= 12 ? 3 : 2);
+  return KEY ? (NT <= 2 ? 4 : NT <= 4 ? 3 : NT <= 6 ? 4 : NT <= 8 ? 3 : 2) : (NT <= 4 ? 4 : NT <= 6 ? 3 : NT <= 8 ? 2 : NT <= 12 ? 3 : 2);
 }
+// waves a SIMD whose registers fit
+constexpr int lin_waves(bool key, int nt) { return nt <= (key ? 4 : 8) ? 2 : 1; }
 
 // the blocks of a portion that a segment walks: [i0, i1), and how many segments there are
 struct LinSeg {
@@ -378,7 +380,7 @@ __device__ __forceinline__ LinSeg lin_seg(int nb, int nseg, int seg) {
 // ENDS: the first walk of a portion in segments (no outputs; segment s leaves what it ends with at seg[s + 1], its decay
 // at seg_dec[s + 1]; the first one also copies the state it starts from to seg[0])
 template <bool F32, bool KEY, int NT, bool ENDS>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) lin_walk_kernel(LinScanArgs a) {
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 1 : lin_waves(KEY, NT)))) lin_walk_kernel(LinScanArgs a) {
   constexpr int NP = 16 * NT, DEPTH = lin_depth<F32, KEY, NT>();
   using T = std::conditional_t<F32, float, bf16_t>;
   using V = std::conditional_t<F32, gf32x4, lu2>;
@@ -807,10 +809,10 @@ static void lin_go(const LinScanArgs& a, hipStream_t st) {
   lin_norm<F32, KEY>(a, st);
 }
 
-// segments a portion of at most `blocks` blocks is walked in: enough waves for the chip, one a SIMD
-int lin_segments(int H, int vp, int n_seqs, int blocks) {
-  const int waves = std::max(1, H * (vp / 16) * n_seqs);
-  return std::max(1, std::min({(1024 + waves / 2) / waves, LIN_SEGS / std::max(1, n_seqs), blocks / LIN_SEG_MIN, 8}));
+// segments a portion of at most `blocks` blocks is walked in: as many waves as the chip holds
+int lin_segments(int kind, int H, int np, int vp, int n_seqs, int blocks) {
+  const int waves = std::max(1, H * (vp / 16) * n_seqs), want = 1024 * lin_waves(kind == LIN_KEY, np / 16);
+  return std::max(1, std::min({(want + waves / 2) / waves, LIN_SEGS / std::max(1, n_seqs), blocks / LIN_SEG_MIN, 8}));
 }
 
 void launch_lin_scan(const LinScanArgs& a, hipStream_t st) {

@@ -1032,7 +1032,7 @@ void LayeredDecoder::linear(int k, const RowSet& r) {
   if (!r.decode) {
     a.seqs = st_seqs_; a.n_seqs = r.n_seqs;
     a.chunks = st_chunks_; a.n_chunks = r.n_chunks;
-    a.nseg = lin_segments(D.lH, D.lvp, r.n_seqs, (r.longest + LIN_T - 1) / LIN_T);
+    a.nseg = lin_segments(D.lin, D.lH, D.lnp, D.lvp, r.n_seqs, (r.longest + LIN_T - 1) / LIN_T);
     a.seg = lin_seg_; a.seg_dec = lin_seg_dec_;
   }
   a.pos = r.pos; a.slot = r.slot; a.n = a.rows = r.n;

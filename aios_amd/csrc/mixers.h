@@ -194,7 +194,7 @@ struct LinScanArgs {
 };
 int lin_pad_n(int n);                                // 0: not served
 struct LinWs { size_t qo, ko, kr, vo, so, dec; };    // numbers per block
-int lin_segments(int H, int vp, int n_seqs, int blocks);  // blocks: of the longest portion
+int lin_segments(int kind, int H, int np, int vp, int n_seqs, int blocks);  // blocks: of the longest portion
 LinWs lin_ws(int kind, int H, int G, int np, int vp, bool f32);
 void launch_lin_scan(const LinScanArgs& a, hipStream_t st);
 
