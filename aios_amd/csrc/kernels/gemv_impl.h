@@ -192,6 +192,7 @@ __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b
       if (grow + 1 < nrow) y[grow + 1] = v1;
     } break;
     case EPI_RESID: {
+      if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[min(grow + 1, nrow - 1)]; }
       float* y = a.y + (size_t)b * a.ldy;
       y[grow] += v0;
       if (grow + 1 < nrow) y[grow + 1] += v1;

@@ -474,6 +474,10 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
       if (grow + 1 < nrow) a.y[grow + 1] = v1;
       break;
     case EPI_RESID:
+      if (a.bias) {
+        v0 += a.bias[grow];
+        v1 += a.bias[min(grow + 1, nrow - 1)];
+      }
       unsafeAtomicAdd(a.y + grow, v0);
       if (grow + 1 < nrow) unsafeAtomicAdd(a.y + grow + 1, v1);
       break;

@@ -71,6 +71,7 @@ __device__ __forceinline__ bool sk_epilogue(const GemmQArgs& a, gf32x4 (&acc)[MT
     } else {
       float4* c = (float4*)(a.C + (size_t)m * a.ldc + n);
       if constexpr (EPI == GEPI_ACCUM_NORM) {
+        if (a.bias16) v += *(const gf32x4*)(a.bias16 + n);
         const float4 o = *c;
         const float4 x = make_float4(o.x + v[0], o.y + v[1], o.z + v[2], o.w + v[3]);
         *c = x;

@@ -164,6 +164,9 @@ class LayeredDecoder {
   void layer16(int k, const RowSet& r);  // k: run
   void layer32(int k, const RowSet& r);
   void layer_seq(int k, const RowSet& r);
+  // few rows: norms in the products that read the residual, sums and biases in those that add to it
+  void layer_fused(int k, const RowSet& r);
+  bool fused(int n) const { return plain_ && (n <= 4 ? (bool)gemv_ok_[n] : n <= 64 && nparts_ > 0); }
   void feed_forward(int k, const RowSet& r, RowCloseArgs& c);
   void recurrence(int k, const RowSet& r);
   void linear(int k, const RowSet& r);
@@ -201,6 +204,7 @@ class LayeredDecoder {
   std::vector<int> owner_;
   std::vector<Weights> w_;
   std::vector<Run> runs_;
+  bool plain_ = false;  // 16-bit sequential layers that add a sublayer's result as it is
   bool seq_ = false, recurrent_ = false, head_ready_ = false;
   int run_limit_ = -1, max_window_ = 0;  // max_window_: largest window, 0 if a layer has none
   bf16_t *embd_ = nullptr, *posw_ = nullptr, *headw_ = nullptr, *pairw_ = nullptr, *loopw_ = nullptr;

@@ -780,7 +780,10 @@ void LayeredDecoder::finalize() {
     e_.gk_ws_ = falloc(e_.gk_ws_bytes_ / 4 + 1);
     e_.gk_cnt_len_ = gemm_skinny_cnt_len(maxN);
     e_.gk_cnt_ = (int*)falloc(e_.gk_cnt_len_);
-    if (!seq_ && dp_ == d_ && d_ % 128 == 0 && env_or("AIOS_GEMM_NORM_FUSE", 1)) {
+    plain_ = seq_ && !loopw_ && dp_ == d_;
+    for (const LayerSpec& l : c.layers)
+      if (l.parallel || l.post_norm || l.resid_gate || (l.mlp != MLP_ACT && l.mlp != MLP_NONE)) plain_ = false;
+    if ((!seq_ || plain_) && dp_ == d_ && d_ % 128 == 0 && env_or("AIOS_GEMM_NORM_FUSE", 1)) {
       GemmQArgs p;
       std::memset(&p, 0, sizeof(p));
       p.M = 64; p.N = dp_; p.K = dims_[0].kout; p.nseg = 1; p.seg[0] = mat(w_[owner_[0]].out, dp_, dims_[0].kout);
@@ -813,7 +816,7 @@ void LayeredDecoder::finalize() {
   st_tiles_ = (LatentTile*)(st_run_ + R + chunk_ints + seq_ints);
   gemv_ok_.assign(5, 0);
   for (int b = 1; b <= 4 && !f32_; ++b) {
-    bool ok = !seq_ && dp_ == d_ && env_or("AIOS_LAYERED_GEMV", 1);
+    bool ok = (!seq_ || plain_) && dp_ == d_ && env_or("AIOS_LAYERED_GEMV", 1);
     for (int i = 0; i < nl_ && ok; ++i) ok = gemv_fits(i, b);
     gemv_ok_[b] = ok;
   }
@@ -824,15 +827,14 @@ void LayeredDecoder::finalize() {
 bool LayeredDecoder::gemv_fits(int i, int B) {
   const Dims& D = dims_[i];
   const Weights& w = w_[owner_[i]];
-  GemvArgs a = e_.gemv_args({}, D.nin, dp_, B, x_, dp_, w.norm, qdg_, D.n1, EPI_STORE, 0);
-  a.nseg = 1;
-  a.seg[0] = mat(w.in, D.nin, dp_);
-  if (!gemv_bf16_engine_fits(a)) return false;
-  a.seg[0] = mat(w.out, dp_, D.kout);
-  a.N = dp_;
-  a.K = D.kout;
-  a.ldx = D.kout;
-  return gemv_bf16_engine_fits(a);
+  auto fits = [&](const bf16_t* m, int N, int K, const float* norm) {
+    GemvArgs a = e_.gemv_args({}, N, K, B, x_, K, norm, qdg_, N, EPI_STORE, 0);
+    a.nseg = 1;
+    a.seg[0] = mat(m, N, K);
+    return gemv_bf16_engine_fits(a);
+  };
+  return fits(w.in, seq_ ? D.n1 : D.nin, dp_, w.norm) && fits(w.out, dp_, D.kout, nullptr) &&
+         (!seq_ || !D.glu || (fits(w.in2, D.glu, dp_, w.norm2) && fits(w.out2, dp_, D.glu, nullptr)));
 }
 
 // measured prefill-GEMM plans for the layers' shapes (as Engine::tune_prefill_gemm)
@@ -1371,6 +1373,79 @@ void LayeredDecoder::layer32(int k, const RowSet& r) {
   launch_gemm_f32(cat32_, D.kout, w.out, D.kout, r.n, dp_, D.kout, x_, dp_, 1, st);
 }
 
+void LayeredDecoder::layer_fused(int k, const RowSet& r) {
+  const int i = runs_[k].layer, n = r.n;
+  const Dims& D = dims_[i];
+  const LayerSpec& s = e_.cfg_.layers[i];
+  const Weights& w = w_[owner_[i]];
+  hipStream_t st = e_.stream_;
+  const float eps = e_.cfg_.norm_eps;
+  const bool few = n <= 4;
+  // y = W norm(x) in fp32, or (y16) act(W norm(x) + bias)
+  auto from_residual = [&](const bf16_t* m, int N, const float* g, float* y, bf16_t* y16, const float* bias) {
+    if (few) {
+      GemvArgs a = e_.gemv_args({}, N, dp_, n, x_, dp_, g, y, N, y16 ? EPI_ACT16 : EPI_STORE, 0);
+      a.nseg = 1;
+      a.seg[0] = mat(m, N, dp_);
+      a.act = s.act;
+      a.bias = bias;
+      a.y16 = y16;
+      a.ldy16 = N;
+      return launch_gemv(a, st);
+    }
+    GemmQArgs a;
+    std::memset(&a, 0, sizeof(a));
+    a.A = h16_; a.lda = dp_; a.M = n; a.N = N; a.K = dp_; a.nseg = 1; a.seg[0] = mat(m, N, dp_);
+    a.C = y; a.C16 = y16; a.ldc = N; a.epi = y16 ? GEPI_STORE16 : GEPI_STORE;
+    a.bias16 = bias;
+    if (y16) a.unary = 1 + s.act;
+    if (norm_ready_) { a.A = xn16_; a.nrm_in = npart_; a.nrm_parts = nparts_; a.nrm_eps = eps; }
+    e_.gemm(a);
+  };
+  // x += W cat + bias; g: weight of the norm that reads it next; enter: the loop's embedding joins
+  auto to_residual = [&](const bf16_t* m, int K, const float* bias, const float* g, bool enter) {
+    if (few) {
+      GemvArgs a = e_.gemv_args({}, dp_, K, n, nullptr, K, nullptr, x_, dp_, EPI_RESID, 0);
+      a.nseg = 1;
+      a.seg[0] = mat(m, dp_, K);
+      a.x16 = cat16_;
+      a.bias = bias;
+      launch_gemv(a, st);
+      if (!enter) return;
+    } else if (!enter) {
+      GemmQArgs a;
+      std::memset(&a, 0, sizeof(a));
+      a.A = cat16_; a.lda = K; a.M = n; a.N = dp_; a.K = K; a.nseg = 1; a.seg[0] = mat(m, dp_, K);
+      a.C = x_; a.ldc = dp_; a.epi = GEPI_ACCUM_NORM;
+      a.bias16 = bias;
+      a.nrm_g = g; a.nrm_out16 = xn16_; a.nrm_part = npart_; a.nrm_parts = nparts_;
+      e_.gemm(a);
+      norm_ready_ = true;
+      return;
+    }
+    RowCloseArgs c = close_args();
+    c.extra = x0_;
+    if (!few) {
+      project(cat16_, K, m, n, dp_, K, y_, dp_);
+      c.y = y_;
+      c.y_bias = bias;
+      c.next = next_of(k + 1, r.decode);
+      norm_ready_ = false;
+    }
+    launch_row_close(c, n, st);
+  };
+  from_residual(w.in, D.n1, w.norm, qdg_, nullptr, nullptr);
+  if (s.mixer == MIX_MINGRU) recurrence(k, r);
+  else if (s.mixer == MIX_GQA) grouped_attention(k, r);
+  else if (s.mixer == MIX_LATENT) attention(k, r);
+  if (D.lin) linear(k, r);
+  const float* after = k + 1 < runs_to_do() ? w_[owner_[runs_[k + 1].layer]].norm : out_norm_;
+  to_residual(w.out, D.kout, w.ob, D.glu ? w.norm2 : after, !D.glu && enters_pass(k + 1));
+  if (!D.glu) return;
+  from_residual(w.in2, D.glu, w.norm2, nullptr, cat16_, w.upb);
+  to_residual(w.out2, D.glu, w.dnb, after, enters_pass(k + 1));
+}
+
 void LayeredDecoder::run(const RowSet& r) {
   const EngineConfig& c = e_.cfg_;
   EmbedArgs e;
@@ -1387,12 +1462,14 @@ void LayeredDecoder::run(const RowSet& r) {
   }
   e.keep32 = x0_;
   e.f32 = f32_;
-  if (seq_) e.next = next_of(0, r.decode);
+  const bool few = fused(r.n);
+  if (seq_ && !(few && r.n <= 4)) e.next = next_of(0, r.decode);
   launch_embed_rows(e, r.n, e_.stream_);
   norm_ready_ = false;
   const int n = runs_to_do();
   for (int k = 0; k < n; ++k) {
-    if (seq_) layer_seq(k, r);
+    if (few) layer_fused(k, r);
+    else if (seq_) layer_seq(k, r);
     else if (f32_) layer32(k, r);
     else layer16(k, r);
   }
@@ -1406,7 +1483,7 @@ void LayeredDecoder::decode_forward(int B) {
   r.decode = true;
   r.max_len = e_.cfg_.max_ctx;
   run(r);
-  head_ready_ = seq_;  // (the last layer left the head's operand)
+  head_ready_ = seq_ && !fused(B);  // (the last layer left the head's operand)
   // (the head reads the residual in place: the decode rows are x rows 0 .. B-1)
   std::swap(x_, xh_);
   head(B);
@@ -1495,19 +1572,15 @@ void LayeredDecoder::head(int B, int from) {
   hipStream_t st = e_.stream_;
   const float eps = e_.cfg_.norm_eps;
   float* y = e_.logits_;
-  if (seq_) {
-    void* h = f32_ ? (void*)h32_ : (void*)h16_;
-    if (!head_ready_) {
-      if (f32_) launch_rmsnorm(x, dp_, out_norm_, h32_, dp_, B, d_, eps, st);
-      else launch_rmsnorm_bf16(x, dp_, out_norm_, h16_, dp_, B, d_, eps, st);
-    }
-    head_ready_ = false;
-    return project(h, dp_, headw_, B, vp_, dp_, y, vp_);
-  }
   if (f32_) {
-    launch_rmsnorm(x, dp_, out_norm_, h32_, dp_, B, d_, eps, st);
+    if (!head_ready_) launch_rmsnorm(x, dp_, out_norm_, h32_, dp_, B, d_, eps, st);
+    head_ready_ = false;
     launch_gemm_f32(h32_, dp_, headw_, dp_, B, vp_, dp_, y, vp_, 0, st);
     return;
+  }
+  if (head_ready_) {
+    head_ready_ = false;
+    return project(h16_, dp_, headw_, B, vp_, dp_, y, vp_);
   }
   if (B <= 4 && dp_ == d_ && !norm_ready_) {
     GemvArgs a = e_.gemv_args({}, vp_, dp_, B, x, dp_, out_norm_, y, vp_, EPI_STORE, 0);
