@@ -33,8 +33,8 @@ struct LinSpec {
   int dim = 64, vdim = 64;             // state rows (key channels) and columns per head
   int conv = 4;                        // MIX_MAMBA2: taps
   int norm_groups = 1;                 // MIX_MAMBA2: parts of the gated norm
-  int rank = 16;                       // MIX_GLA: width of the decay's first projection
-  double tau = 16.0;                   // MIX_GLA
+  int rank = 8;                        // MIX_GLA: width of the decay's first projection
+  double tau = 1.0;                    // MIX_GLA
 };
 struct LayerSpec {
   int mixer = MIX_LATENT;

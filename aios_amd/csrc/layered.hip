@@ -10,6 +10,8 @@
 // bf16 operand that the row operation before it wrote (mixers.h), so a layer is
 //   input product (+ residual gate rows) | mixer | output product | close | input product (+ residual gate and
 //   router rows, GLU in its epilogue) | experts | down product | close
+// Where a sublayer's result is added as it is (no gate, no norm of it), batches up to 64 rows need no row operations: as
+// above, the product that reads the residual normalises it and the one before adds to it (layer_fused).
 // Mixers that read the same input share the input product and the output product: a layer's attention and linear
 // recurrence leave their results side by side in one operand.
 // 32-bit engine: the same steps in fp32, absorbed attention for every row.

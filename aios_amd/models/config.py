@@ -31,8 +31,8 @@ class LinConfig:
     vdim: int = 64                 # state columns per head
     conv: int = 4                  # taps (mamba2)
     norm_groups: int = 1           # parts of the gated norm (mamba2)
-    rank: int = 16                 # width of the decay's first projection (gla)
-    tau: float = 16.0              # root taken of the decay (gla)
+    rank: int = 8                  # width of the decay's first projection (gla)
+    tau: float = 1.0               # root taken of the decay (gla)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -301,11 +301,11 @@ PRESETS: Dict[str, ModelConfig] = {
     # Sinisun at the widths and depths (layer runs) of the first two; MLPs of equal parameter count
     "sinisun-1b": _sinisun("sinisun-1b", 32000, 2048, 18, 8448, (4, 8, 2), 4096,
                            LinConfig(heads=64, vdim=64, dim=128, groups=8, norm_groups=8),
-                           LinConfig(heads=16, dim=64, vdim=128, tau=12.0), heads=32, kv_heads=4, dim=64, vdim=64, rot_dims=64,
+                           LinConfig(heads=16, dim=64, vdim=128, rank=16, tau=12.0), heads=32, kv_heads=4, dim=64, vdim=64, rot_dims=64,
                            chunk=1024, softcap=40.0),
     "sinisun-7b": _sinisun("sinisun-7b", 32000, 4096, 26, 21504, (4, 10, 2), 32768,
                            LinConfig(heads=128, vdim=64, dim=128, groups=8, norm_groups=8),
-                           LinConfig(heads=32, dim=64, vdim=128, tau=12.0), heads=32, kv_heads=8, dim=128, vdim=128,
+                           LinConfig(heads=32, dim=64, vdim=128, rank=16, tau=12.0), heads=32, kv_heads=8, dim=128, vdim=128,
                            rot_dims=128, chunk=4096, softcap=40.0),
     "test-sinisun": _sinisun("test-sinisun", 600, 384, 4, 512, (1, 3, 2), 512,
                              LinConfig(heads=4, vdim=40, dim=24, groups=2, norm_groups=5, conv=3),
