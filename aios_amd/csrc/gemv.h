@@ -9,7 +9,7 @@ constexpr int GEMV_MAX_SEGS = 3;
 
 enum GemvEpilogue : int {
   EPI_STORE = 0,   // y[b][n]  = acc
-  EPI_RESID = 1,   // y[b][n] += acc        (residual stream update; + bias[n], the BF16 engine only)
+  EPI_RESID = 1,   // y[b][n] += acc        (residual stream update)
   EPI_SWIGLU = 2,  // y[b][n/2] = silu(acc[2i]) * acc[2i+1]   (rows interleaved gate/up)
   EPI_QKV = 3,     // (+bias) RoPE on Q/K, Q -> y, K/V -> bf16 KV cache at pos[b]
   EPI_TP_RESID = 4,  // TP row-parallel O / down at batch 1: y[n] += sum over ranks of acc (the one-shot
@@ -17,6 +17,7 @@ enum GemvEpilogue : int {
   EPI_STORE_GLU = 5,  // rows below glu_row0: y[b][n] = acc; above: interleaved gate/up pairs through the GLU
                       //   to y16[b][(n - glu_row0) / 2] (row stride ldy16) -- the BF16 engine only
   EPI_ACT16 = 6,      // y16[b][n] = act(acc + bias[n]) (bias or null; row stride ldy16) -- the BF16 engine only
+  EPI_RESID_BIAS = 7,  // y[b][n] += acc + bias[n] -- the BF16 engine only
 };
 
 struct ArDevCtx;  // comm.h

@@ -192,7 +192,6 @@ __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b
       if (grow + 1 < nrow) y[grow + 1] = v1;
     } break;
     case EPI_RESID: {
-      if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[min(grow + 1, nrow - 1)]; }
       float* y = a.y + (size_t)b * a.ldy;
       y[grow] += v0;
       if (grow + 1 < nrow) y[grow + 1] += v1;
@@ -206,6 +205,11 @@ __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b
     case EPI_STORE_GLU: {
       if (grow < a.glu_row0) *(float2*)(a.y + (size_t)b * a.ldy + grow) = make_float2(v0, v1);
       else a.y16[(size_t)b * a.ldy16 + ((grow - a.glu_row0) >> 1)] = f32_to_bf16(glu_act(v0, a.act) * v1);
+    } break;
+    case EPI_RESID_BIAS: {
+      float2* y = (float2*)(a.y + (size_t)b * a.ldy + grow);
+      const float2 o = *y, c = *(const float2*)(a.bias + grow);
+      *y = make_float2(o.x + v0 + c.x, o.y + v1 + c.y);
     } break;
     case EPI_ACT16: {
       if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[grow + 1]; }

@@ -321,6 +321,7 @@ inline bool launch_gemv_lds16(const GemvArgs& a, hipStream_t st, bool dry = fals
   for (int s = 0; s < a.nseg; ++s)
     if (a.seg[s].qtype != QT_BF16 || a.seg[s].cols != a.K || (s > 0 && a.seg_row0[s] % 2)) return false;
   if (a.epi == EPI_STORE_GLU && (a.glu_row0 % 2 || a.ldy % 2)) return false;
+  if (a.epi == EPI_RESID_BIAS && (!a.bias || a.ldy % 2)) return false;
   if (a.epi == EPI_ACT16 && (!a.y16 || a.ldy16 % 2)) return false;
   const int npairs = a.N / 2;
   const int G = std::min(a.tune_grid > 0 ? a.tune_grid : device_cu_count(), npairs);

@@ -474,10 +474,6 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
       if (grow + 1 < nrow) a.y[grow + 1] = v1;
       break;
     case EPI_RESID:
-      if (a.bias) {
-        v0 += a.bias[grow];
-        v1 += a.bias[min(grow + 1, nrow - 1)];
-      }
       unsafeAtomicAdd(a.y + grow, v0);
       if (grow + 1 < nrow) unsafeAtomicAdd(a.y + grow + 1, v1);
       break;
@@ -489,6 +485,11 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
     case EPI_STORE_GLU: {
       if (grow < a.glu_row0) *(float2*)(a.y + grow) = make_float2(v0, v1);
       else a.y16[(grow - a.glu_row0) >> 1] = f32_to_bf16(glu_act(v0, a.act) * v1);
+    } break;
+    case EPI_RESID_BIAS: {
+      float2* y = (float2*)(a.y + grow);
+      const float2 o = *y, c = *(const float2*)(a.bias + grow);
+      *y = make_float2(o.x + v0 + c.x, o.y + v1 + c.y);
     } break;
     case EPI_ACT16: {
       if (a.bias) {

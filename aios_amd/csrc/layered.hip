@@ -1407,7 +1407,7 @@ void LayeredDecoder::layer_fused(int k, const RowSet& r) {
   // x += W cat + bias; g: weight of the norm that reads it next; enter: the loop's embedding joins
   auto to_residual = [&](const bf16_t* m, int K, const float* bias, const float* g, bool enter) {
     if (few) {
-      GemvArgs a = e_.gemv_args({}, dp_, K, n, nullptr, K, nullptr, x_, dp_, EPI_RESID, 0);
+      GemvArgs a = e_.gemv_args({}, dp_, K, n, nullptr, K, nullptr, x_, dp_, bias ? EPI_RESID_BIAS : EPI_RESID, 0);
       a.nseg = 1;
       a.seg[0] = mat(m, dp_, K);
       a.x16 = cat16_;
