@@ -152,12 +152,14 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.attr("MIX_GQA") = (int)MIX_GQA;
   m.attr("MIX_MAMBA2") = (int)MIX_MAMBA2;
   m.attr("MIX_GLA") = (int)MIX_GLA;
+  m.attr("MIX_DELTA") = (int)MIX_DELTA;
   m.attr("GATE_NONE") = (int)GATE_NONE;
   m.attr("GATE_ELEMENT") = (int)GATE_ELEMENT;
   m.attr("GATE_HEAD") = (int)GATE_HEAD;
   m.attr("ACT_SILU") = (int)ACT_SILU;
   m.attr("ACT_GELU_TANH") = (int)ACT_GELU_TANH;
   m.attr("ACT_RELU2") = (int)ACT_RELU2;
+  m.attr("ACT_XIELU") = (int)ACT_XIELU;
   py::class_<LinSpec>(m, "LinSpec")
       .def(py::init<>())
       .def_readwrite("heads", &LinSpec::heads)
@@ -194,11 +196,16 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       .def_readwrite("chunk", &LayerSpec::chunk)
       .def_readwrite("softcap", &LayerSpec::softcap)
       .def_readwrite("attn_bias", &LayerSpec::attn_bias)
+      .def_readwrite("qk_norm", &LayerSpec::qk_norm)
+      .def_readwrite("v_norm", &LayerSpec::v_norm)
+      .def_readwrite("v_mix", &LayerSpec::v_mix)
+      .def_readwrite("head_temp", &LayerSpec::head_temp)
       .def_readwrite("lin", &LayerSpec::lin)
       .def_readwrite("beside", &LayerSpec::beside)
       .def_readwrite("mixer_scale", &LayerSpec::mixer_scale)
       .def_readwrite("beside_scale", &LayerSpec::beside_scale)
       .def_readwrite("mlp_bias", &LayerSpec::mlp_bias)
+      .def_readwrite("mlp_scale", &LayerSpec::mlp_scale)
       .def_readwrite("experts", &LayerSpec::experts)
       .def_readwrite("top", &LayerSpec::top)
       .def_readwrite("shared_ff", &LayerSpec::shared_ff)
@@ -517,7 +524,8 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.def("gemv",
         [](std::vector<PyQMatrix*> segs, int B, uintptr_t x, int ldx, uintptr_t norm_w, float eps, uintptr_t y,
            int ldy, int epi, uintptr_t st, int force_v1, int act_q8, int tune_grid, int tune_u, int tune_ksplit, int tune_dbg,
-           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16, uintptr_t bias) {
+           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16, uintptr_t bias, float pos, float neg,
+           float scale) {
           GemvArgs a;
           std::memset(&a, 0, sizeof(a));
           a.nseg = (int)segs.size();
@@ -530,13 +538,15 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
           a.kernel_sel = kernel_sel; a.dbg_ts = (unsigned long long*)dbg_ts;
           a.x16 = (const bf16_t*)x16; a.y16 = (bf16_t*)y16;  // bf16 input / SwiGLU output (hand-off kernels)
           a.act = act; a.glu_row0 = glu_row0; a.ldy16 = ldy16; a.bias = (const float*)bias;
+          a.act_n = ActNum{pos, neg, scale};
           launch_gemv(a, S(st));
         },
         py::arg("segs"), py::arg("B"), py::arg("x"), py::arg("ldx"), py::arg("norm_w"), py::arg("eps"), py::arg("y"),
         py::arg("ldy"), py::arg("epi"), py::arg("stream"), py::arg("force_v1") = 0, py::arg("act_q8") = 0,
         py::arg("tune_grid") = 0, py::arg("tune_u") = 0, py::arg("tune_ksplit") = 0, py::arg("tune_dbg") = 0,
         py::arg("kernel_sel") = 0, py::arg("dbg_ts") = 0, py::arg("x16") = 0, py::arg("y16") = 0, py::arg("act") = 0,
-        py::arg("glu_row0") = 0, py::arg("ldy16") = 0, py::arg("bias") = 0);
+        py::arg("glu_row0") = 0, py::arg("ldy16") = 0, py::arg("bias") = 0, py::arg("pos") = 0.f, py::arg("neg") = 0.f,
+        py::arg("scale") = 1.f);
   m.def("gemv_bf16_engine_fits",
         [](std::vector<PyQMatrix*> segs, int B, int epi) {
           GemvArgs a;
@@ -679,7 +689,8 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.def(
       "gemm_q",
       [](uintptr_t A, int lda, std::vector<PyQMatrix*> segs, int M, uintptr_t C, uintptr_t C16, int ldc, int epi,
-         uintptr_t st, int ksplit, uintptr_t dbg_ts, int act, int glu_n0, int ldc16, uintptr_t bias16, int unary) {
+         uintptr_t st, int ksplit, uintptr_t dbg_ts, int act, int glu_n0, int ldc16, uintptr_t bias16, int unary,
+         float pos, float neg, float scale) {
         GemmQArgs a;
         std::memset(&a, 0, sizeof(a));
         if (segs.empty() || segs.size() > 3) throw std::runtime_error("gemm_q: 1..3 segments");
@@ -690,13 +701,15 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
         a.C = (float*)C; a.C16 = (bf16_t*)C16; a.ldc = ldc; a.epi = epi; a.ksplit = ksplit;
         a.dbg_ts = (unsigned long long*)dbg_ts;
         a.act = act; a.glu_n0 = glu_n0; a.ldc16 = ldc16; a.bias16 = (const float*)bias16; a.unary = unary;
+        a.act_n = ActNum{pos, neg, scale};
         GemmWs& g = gemm_ws(M, a.N);
         a.ws = g.ws; a.ws_bytes = g.bytes; a.cnt = g.cnt; a.cnt_len = g.cnt_len;
         launch_gemm_q(a, S(st));
       },
       py::arg("A"), py::arg("lda"), py::arg("segs"), py::arg("M"), py::arg("C"), py::arg("C16"), py::arg("ldc"),
       py::arg("epi"), py::arg("stream"), py::arg("ksplit") = 0, py::arg("dbg_ts") = 0, py::arg("act") = 0,
-      py::arg("glu_n0") = 0, py::arg("ldc16") = 0, py::arg("bias16") = 0, py::arg("unary") = 0);
+      py::arg("glu_n0") = 0, py::arg("ldc16") = 0, py::arg("bias16") = 0, py::arg("unary") = 0,
+      py::arg("pos") = 0.f, py::arg("neg") = 0.f, py::arg("scale") = 1.f);
   m.def(
       "gemm_pf_plan",
       [](std::vector<PyQMatrix*> segs, int M, int epi, int ksplit) {
@@ -835,6 +848,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   });
   m.attr("LIN_HEAD") = (int)LIN_HEAD;
   m.attr("LIN_KEY") = (int)LIN_KEY;
+  m.attr("LIN_DELTA") = (int)LIN_DELTA;
   m.def(
       "lin_scan",
       [](const std::vector<std::vector<int>>& pieces, py::kwargs kw) {
@@ -847,7 +861,7 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
         a.in = P("inp"); a.ld = I("ld"); a.z_off = I("z_off"); a.x_off = I("x_off"); a.taps = I("taps"); a.dt_off = I("dt_off");
         a.conv_w = P("conv_w"); a.conv_b = P("conv_b"); a.dt_b = P("dt_b"); a.a_log = P("a_log"); a.D = P("D"); a.ring = P("ring");
         a.q_off = I("q_off"); a.k_off = I("k_off"); a.v_off = I("v_off"); a.a_off = I("a_off"); a.rank = I("rank");
-        a.q_scale = F("q_scale"); a.inv_tau = F("inv_tau"); a.a2 = P("a2"); a.a2_b = P("a2_b");
+        a.b_off = I("b_off"); a.q_scale = F("q_scale"); a.inv_tau = F("inv_tau"); a.a2 = P("a2"); a.a2_b = P("a2_b");
         a.state = P("state"); a.slots = I("slots"); a.pos = (const int*)P("pos"); a.slot = (const int*)P("slot");
         a.n = a.rows = I("n"); a.qo = P("qo"); a.ko = P("ko"); a.kr = P("kr"); a.vo = P("vo"); a.so = P("so"); a.dec = P("dec");
         a.nseg = std::max(1, I("nseg")); a.seg = P("seg"); a.seg_dec = P("seg_dec");
@@ -887,6 +901,8 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
     a.rows = I("rows"); a.n = I("n"); a.H = I("H"); a.G = I("G"); a.dk = I("dk"); a.dkp = I("dkp"); a.dv = I("dv"); a.dvp = I("dvp");
     a.rot = I("rot"); a.rope = (const float2*)P("rope"); a.window = I("window"); a.chunk = I("chunk");
     a.scale = F("scale"); a.softcap = F("softcap"); a.sink = (const float*)P("sink");
+    a.qn = (const float*)P("qn"); a.kn = (const float*)P("kn"); a.temp = (const float*)P("temp"); a.v_norm = I("v_norm");
+    a.eps = F("eps"); a.first = (float*)P("first"); a.lambda = (const float*)P("lambda_");
     a.qb = (const float*)P("qb"); a.kb = (const float*)P("kb"); a.vb = (const float*)P("vb");
     a.in = (const float*)P("inp"); a.ld = I("ld"); a.q_off = I("q_off"); a.k_off = I("k_off"); a.v_off = I("v_off");
     a.g_off = I("g_off"); a.out_scale = F("out_scale"); a.pos = (const int*)P("pos"); a.slot = (const int*)P("slot");
@@ -912,9 +928,14 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
       launch_mha_prefill(m, st);
     }
   });
-  m.def("bias_act_f32", [](uintptr_t x, int ldx, uintptr_t bias, uintptr_t y, int ldy, int rows, int n, int act, uintptr_t st) {
-    launch_bias_act_f32((const float*)x, ldx, (const float*)bias, (float*)y, ldy, rows, n, act, S(st));
-  });
+  m.def(
+      "bias_act_f32",
+      [](uintptr_t x, int ldx, uintptr_t bias, uintptr_t y, int ldy, int rows, int n, int act, uintptr_t st, float pos, float neg,
+         float scale) {
+        launch_bias_act_f32((const float*)x, ldx, (const float*)bias, (float*)y, ldy, rows, n, act, ActNum{pos, neg, scale}, S(st));
+      },
+      py::arg("x"), py::arg("ldx"), py::arg("bias"), py::arg("y"), py::arg("ldy"), py::arg("rows"), py::arg("n"), py::arg("act"),
+      py::arg("stream"), py::arg("pos") = 0.f, py::arg("neg") = 0.f, py::arg("scale") = 1.f);
   // the routed experts of n tokens; few: launch_moe_few (y), else launch_moe_grouped (ye, pair, wt)
   m.attr("MOE_FEW") = MOE_FEW;
   m.def("moe_tile_rows", &moe_tile_rows);

@@ -73,16 +73,25 @@ __device__ __forceinline__ uint16_t f32_to_bf16(float f) {
 }
 // activation of a gated MLP's gate: z * sigmoid(z) (SiLU), or GELU in its tanh form, which is
 // z * sigmoid(2 sqrt(2 / pi) (z + 0.044715 z^3)) since (1 + tanh u) / 2 = sigmoid(2 u)
-enum GluAct : int { ACT_SILU = 0, ACT_GELU_TANH = 1, ACT_RELU2 = 2 };  // (ACT_RELU2: the square of relu)
+// (ACT_RELU2: the square of relu; ACT_XIELU: z / 2 + pos z^2 for z > 0, z / 2 + neg (e^z - 1 - z) below: both without a gate)
+enum GluAct : int { ACT_SILU = 0, ACT_GELU_TANH = 1, ACT_RELU2 = 2, ACT_XIELU = 3 };
+// numbers of an activation without a gate: ACT_XIELU's two, and what the result is multiplied by
+struct ActNum {
+  float pos, neg, scale;
+};
 __device__ __forceinline__ float glu_act(float z, int act) {
   const float u = act == ACT_GELU_TANH ? 1.5957691216057308f * fmaf(0.044715f * z * z, z, z) : z;
   return z / (1.f + __expf(-u));
 }
 // activation of an MLP without a gate
-__device__ __forceinline__ float unary_act(float z, int act) {
-  if (act != ACT_RELU2) return glu_act(z, act);
+__device__ __forceinline__ float unary_act(float z, int act, const ActNum& n) {
+  if (act == ACT_XIELU) {
+    const float m = fminf(z, 0.f);
+    return n.scale * fmaf(0.5f, z, z > 0.f ? n.pos * z * z : n.neg * (__expf(m) - 1.f - m));
+  }
+  if (act != ACT_RELU2) return n.scale * glu_act(z, act);
   const float r = fmaxf(z, 0.f);
-  return r * r;
+  return n.scale * r * r;
 }
 __device__ __forceinline__ float h2f(uint16_t h) { return __half2float(__ushort_as_half(h)); }
 

@@ -49,6 +49,7 @@ struct GemvArgs {
   bf16_t* y16;                  // EPI_SWIGLU: bf16 output [B][ldy] written instead of y (or null)
   int epi;
   int act;                      // gate activation of the GLU epilogues (GluAct)
+  ActNum act_n;                 // EPI_ACT16
   int glu_row0, ldy16;          // EPI_STORE_GLU
   // QKV epilogue
   const float* bias;            // [N] or null

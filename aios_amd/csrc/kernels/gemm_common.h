@@ -23,7 +23,7 @@ __device__ __forceinline__ uint32_t pk_bf16(float a, float b) {
 // GEPI_STORE16: what column n's sum becomes
 __device__ __forceinline__ float store16_val(const GemmQArgs& a, int n, float v) {
   if (a.bias16) v += a.bias16[n];
-  return a.unary ? unary_act(v, a.unary - 1) : v;
+  return a.unary ? unary_act(v, a.unary - 1, a.act_n) : v;
 }
 
 // 8 dequantised weights w = sc * q - of (q raw unsigned codes) -> one bf16x8 MFMA fragment

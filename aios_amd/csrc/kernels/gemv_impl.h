@@ -214,7 +214,7 @@ __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b
     case EPI_ACT16: {
       if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[grow + 1]; }
       *(uint32_t*)(a.y16 + (size_t)b * a.ldy16 + grow) =
-          (uint32_t)f32_to_bf16(unary_act(v0, a.act)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act)) << 16;
+          (uint32_t)f32_to_bf16(unary_act(v0, a.act, a.act_n)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act, a.act_n)) << 16;
     } break;
     case EPI_QKV: {
       if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[grow + 1]; }

@@ -497,7 +497,7 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
         v1 += a.bias[grow + 1];
       }
       *(uint32_t*)(a.y16 + grow) =
-          (uint32_t)f32_to_bf16(unary_act(v0, a.act)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act)) << 16;
+          (uint32_t)f32_to_bf16(unary_act(v0, a.act, a.act_n)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act, a.act_n)) << 16;
     } break;
     case EPI_QKV: {
       if (a.bias) {

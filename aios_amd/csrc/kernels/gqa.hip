@@ -1,7 +1,8 @@
 // Grouped-query attention of the layered decoders (mixers.h GqaArgs) over a paged cache: soft cap, sink, window or
 // chunks, a gate per head.
 //
-//   gqa_prep   biases, rotation, queries (the score's factor folded in) and the cache's new keys and values
+//   gqa_prep   biases, norms, rotation, mixing of values, queries (the score's factor folded in) and the cache's new keys
+//              and values
 //   gqa_attn   rows of one sequence that read the same key / value head, 16 to a tile (the query heads of a token,
 //              then further tokens): S^T = K Q^T per 32-key tile and wave, P^T goes from the accumulators into
 //              O^T += V^T P^T without leaving registers (V through a wave's own slice of LDS); the four waves take the
@@ -82,10 +83,118 @@ __global__ void __launch_bounds__(256) gqa_prep_kernel(GqaArgs a, float qf) {
   }
 }
 
+// with norms of q, k or v, numbers per head or mixed values: workgroups y < nq take a row's queries (each sums them all for the
+// norm and writes its share), y = nq its keys, the others four heads' values, a wave each
+template <bool F32>
+__global__ void __launch_bounds__(256) gqa_norm_prep_kernel(GqaArgs a, float qf, int nq) {
+  __shared__ float red[4];
+  const int row = blockIdx.x, y = blockIdx.y, tid = threadIdx.x, pos = a.pos[row], slot = a.slot[row], key = pos % GQA_BLOCK;
+  const float* in = a.in + (size_t)row * a.ld;
+  const size_t blk = (size_t)a.bt[(size_t)slot * a.maxb + pos / GQA_BLOCK] * a.G * GQA_BLOCK * (a.dkp + a.dvp);
+  if (y > nq) {
+    const int g = (y - nq - 1) * 4 + (tid >> 6), lane = tid & 63;
+    if (g >= a.G) return;
+    float v[4], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = lane + 64 * i;
+      v[i] = 0.f;
+      if (c < a.dv) v[i] = in[a.v_off + g * a.dv + c] + (a.vb ? a.vb[g * a.dv + c] : 0.f);
+      ss = fmaf(v[i], v[i], ss);
+    }
+#pragma unroll
+    for (int d = 32; d; d >>= 1) ss += __shfl_xor(ss, d, 64);
+    const float inv = a.v_norm ? 1.f / sqrtf(ss / (float)a.dv + a.eps) : 1.f, lam = a.lambda ? *a.lambda : 0.f;
+    const size_t at = blk + (size_t)a.G * GQA_BLOCK * a.dkp + ((size_t)g * GQA_BLOCK + key) * a.dvp;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int c = lane + 64 * i;
+      if (c >= a.dvp) break;
+      float x = v[i] * inv;
+      if (a.first && c < a.dv) {
+        float* f = a.first + ((size_t)row * a.G + g) * a.dv + c;
+        if (a.lambda) x = (1.f - lam) * x + lam * *f;
+        else *f = x;
+      }
+      if constexpr (F32) ((float*)a.pool)[at + c] = x;
+      else ((bf16_t*)a.pool)[at + c] = f32_to_bf16(x);
+    }
+    return;
+  }
+  const bool isq = y < nq;
+  const int heads = isq ? a.H : a.G, n = heads * a.dk, half = a.rot >> 1;
+  const float *x = in + (isq ? a.q_off : a.k_off), *b = isq ? a.qb : a.kb, *w = isq ? a.qn : a.kn;
+  const float2* cs = a.rope + (size_t)pos * half;
+  const bool vec = ((a.dk | a.ld | a.q_off | a.k_off) & 3) == 0;  // (whole 16-byte pieces)
+  float inv = 1.f;
+  if (w) {
+    float ss = 0.f;
+    if (vec) {
+      for (int i = 4 * tid; i < n; i += 1024) {
+        gf32x4 u = *(const gf32x4*)(x + i);
+        if (b) u += *(const gf32x4*)(b + i);
+        ss += (u[0] * u[0] + u[1] * u[1]) + (u[2] * u[2] + u[3] * u[3]);
+      }
+    } else {
+      for (int i = tid; i < n; i += 256) {
+        const float u = x[i] + (b ? b[i] : 0.f);
+        ss = fmaf(u, u, ss);
+      }
+    }
+#pragma unroll
+    for (int d = 32; d; d >>= 1) ss += __shfl_xor(ss, d, 64);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    inv = 1.f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)n + a.eps);
+  }
+  auto at = [&](int i) { return (x[i] + (b ? b[i] : 0.f)) * inv * (w ? w[i] : 1.f); };
+  for (int i = 4 * ((isq ? y * 256 : 0) + tid); i < heads * a.dkp; i += 1024 * (isq ? nq : 1)) {
+    const int h = i / a.dkp, c = i - h * a.dkp, k = h * a.dk + c;  // (padded head sizes are whole fours)
+    gf32x4 u = {0.f, 0.f, 0.f, 0.f};
+    if (vec && c < a.dk) {
+      u = *(const gf32x4*)(x + k);
+      if (b) u += *(const gf32x4*)(b + k);
+      u *= inv;
+      if (w) u *= *(const gf32x4*)(w + k);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (c + e < a.dk) u[e] = at(k + e);
+    }
+    if (c < a.rot) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int j = c + e;
+        if (j >= a.rot) break;
+        const float2 t = cs[j < half ? j : j - half];
+        u[e] = j < half ? u[e] * t.x - at(k + e + half) * t.y : u[e] * t.x + at(k + e - half) * t.y;
+      }
+    }
+    if (isq) {
+      u *= (a.temp ? a.temp[h] : 1.f) * (F32 ? 1.f : qf);
+      const size_t o = ((size_t)row * a.H + h) * a.dkp + c;
+      if constexpr (F32) *(gf32x4*)((float*)a.q + o) = u;
+      else *(uint2*)((bf16_t*)a.q + o) = make_uint2(pk_bf16(u[0], u[1]), pk_bf16(u[2], u[3]));
+    } else {
+      const size_t o = blk + ((size_t)h * GQA_BLOCK + key) * a.dkp + c;
+      if constexpr (F32) *(gf32x4*)((float*)a.pool + o) = u;
+      else *(uint2*)((bf16_t*)a.pool + o) = make_uint2(pk_bf16(u[0], u[1]), pk_bf16(u[2], u[3]));
+    }
+  }
+}
+
 void launch_gqa_prep(const GqaArgs& a, hipStream_t st) {
   if (a.rows < 1) return;
   if (!gqa_supports(a.dkp, a.dvp) || a.H % a.G || a.rot % 2 || a.rot > a.dk || (a.rot && !a.rope))
     throw std::runtime_error("gqa: bad sizes");
+  if (a.lambda && !a.first) throw std::runtime_error("gqa: no values to mix with");
+  if (a.qn || a.kn || a.temp || a.v_norm || a.first) {
+    const int nq = a.rows <= 64 ? (a.H * a.dkp + 1023) / 1024 : 1;
+    const dim3 grid(a.rows, nq + 1 + (a.G + 3) / 4);
+    if (a.f32) hipLaunchKernelGGL((gqa_norm_prep_kernel<true>), grid, dim3(256), 0, st, a, 1.f, nq);
+    else hipLaunchKernelGGL((gqa_norm_prep_kernel<false>), grid, dim3(256), 0, st, a, gqa_q_factor(a.scale, a.softcap), nq);
+    return;
+  }
   const int pieces = ((a.H + a.G) * (a.dkp / 2) + a.G * (a.dvp / 2) + 255) / 256;
   const dim3 grid(a.rows, a.rows <= 64 ? pieces : (pieces + 3) / 4);
   if (a.f32) hipLaunchKernelGGL((gqa_prep_kernel<true>), grid, dim3(256), 0, st, a, 1.f);

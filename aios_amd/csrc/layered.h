@@ -18,7 +18,7 @@
 
 namespace aios {
 
-enum MixerKind : int { MIX_NONE = 0, MIX_LATENT = 1, MIX_MINGRU = 2, MIX_GQA = 3, MIX_MAMBA2 = 4, MIX_GLA = 5 };
+enum MixerKind : int { MIX_NONE = 0, MIX_LATENT = 1, MIX_MINGRU = 2, MIX_GQA = 3, MIX_MAMBA2 = 4, MIX_GLA = 5, MIX_DELTA = 6 };
 enum MlpKind : int { MLP_NONE = 0, MLP_GLU = 1, MLP_MOE = 2, MLP_ACT = 3 };
 enum OutGate : int { GATE_NONE = 0, GATE_ELEMENT = 1, GATE_HEAD = 2 };
 
@@ -29,9 +29,9 @@ enum OutGate : int { GATE_NONE = 0, GATE_ELEMENT = 1, GATE_HEAD = 2 };
 
 // A linear recurrence (mixers.h LinScanArgs).
 struct LinSpec {
-  int heads = 1, groups = 1;           // groups: MIX_MAMBA2, heads that share B and C
+  int heads = 1, groups = 1;           // groups: heads that share B and C (MIX_MAMBA2) or a query and a key (MIX_DELTA)
   int dim = 64, vdim = 64;             // state rows (key channels) and columns per head
-  int conv = 4;                        // MIX_MAMBA2: taps
+  int conv = 4;                        // MIX_MAMBA2, MIX_DELTA: taps
   int norm_groups = 1;                 // MIX_MAMBA2: parts of the gated norm
   int rank = 8;                        // MIX_GLA: width of the decay's first projection
   double tau = 1.0;                    // MIX_GLA
@@ -48,18 +48,24 @@ struct LayerSpec {
   double rot_base = 10000.0;
   int window = 0;                      // keys a token sees, itself included (0: all before it)
   float scale = 0.125f;                // of q . k
-  int sink = 1;                        // a learned logit per head joins the softmax's denominator
+  int sink = 1;                        // 1: a learned logit per head joins the softmax's denominator; 2 (MIX_GQA): the logit 0
   int out_gate = GATE_ELEMENT;         // head outputs times sigmoid(Wg h): a number each, or one per head
   // MIX_GQA: heads, dim, vdim, the first rot_dims dimensions turn (in halves), window, scale, sink, out_gate, and
   int kv_heads = 1;
   int chunk = 0;                       // keys before a token's chunk of so many positions are out (0: no chunks)
   float softcap = 0.f;                 // of the scores (0: none)
-  int attn_bias = 0;                   // biases of q, k, v and the output projection
+  int attn_bias = 0;                   // 1: biases of q, k, v and the output projection; 2: of q, k, v
+  int qk_norm = 0;                     // RMS norm of all queries of a token at once, and of all keys, with weights
+  int v_norm = 0;                      // RMS norm of every head's value, without weights
+  int head_temp = 0;                   // a learned number per query head multiplies its scores
+  // from the second layer with v_mix on: values (1 - lambda) v + lambda v_first, lambda learned, v_first the values of the
+  // first such layer
+  int v_mix = 0;
   // MIX_MINGRU
   int width = 64;                      // of the state
-  // MIX_MAMBA2, MIX_GLA
+  // MIX_MAMBA2, MIX_GLA, MIX_DELTA
   LinSpec lin;
-  // a second mixer that reads the same input (MIX_MAMBA2 or MIX_GLA, sizes in lin): mixer_scale * first + beside_scale *
+  // a second mixer that reads the same input (MIX_MAMBA2, MIX_GLA or MIX_DELTA, sizes in lin): mixer_scale * first + beside_scale *
   // second
   int beside = MIX_NONE;
   float mixer_scale = 1.f, beside_scale = 1.f;
@@ -67,6 +73,7 @@ struct LayerSpec {
   int ff = 256;                        // MLP_GLU, MLP_ACT: hidden width; MLP_MOE: of every expert
   int act = ACT_GELU_TANH;             // GluAct of the gate; MLP_ACT: of the hidden layer
   int mlp_bias = 0;                    // MLP_ACT
+  float mlp_scale = 1.f;               // MLP_ACT: of the result
   int experts = 0, top = 0;            // MLP_MOE
   int shared_ff = 0;                   // hidden width of the expert that runs for every token (0: none)
   int correction = 0;                  // a learned number per expert joins the choice, not the weights
@@ -141,6 +148,8 @@ class LayeredDecoder {
     // biases: q, k, v, output projection (times mixer_scale), MLP up and down
     float *qb = nullptr, *kb = nullptr, *vb = nullptr, *ob = nullptr, *upb = nullptr, *dnb = nullptr;
     // linear recurrence (mixers.h LinScanArgs)
+    float *qn = nullptr, *kn = nullptr, *temp = nullptr, *lambda = nullptr;  // grouped-query attention's norms and numbers
+    ActNum act_n{0.f, 0.f, 1.f};
     float *conv_w = nullptr, *conv_b = nullptr, *dt_b = nullptr, *a_log = nullptr, *lin_d = nullptr, *lin_norm = nullptr,
           *a2 = nullptr, *a2_b = nullptr;
   };
@@ -167,6 +176,7 @@ class LayeredDecoder {
   // few rows: norms in the products that read the residual, sums and biases in those that add to it
   void layer_fused(int k, const RowSet& r);
   bool fused(int n) const { return plain_ && (n <= 4 ? (bool)gemv_ok_[n] : n <= 64 && nparts_ > 0); }
+  const Weights& weights(int k) const { return w_[owner_[runs_[k].layer]]; }
   void feed_forward(int k, const RowSet& r, RowCloseArgs& c);
   void recurrence(int k, const RowSet& r);
   void linear(int k, const RowSet& r);
@@ -210,6 +220,9 @@ class LayeredDecoder {
   bf16_t *embd_ = nullptr, *posw_ = nullptr, *headw_ = nullptr, *pairw_ = nullptr, *loopw_ = nullptr;
   float *out_norm_ = nullptr, *loop_step_ = nullptr, *x0_ = nullptr;  // x0_: embedding rows (loops that add them)
   std::vector<float2*> rope_;            // per layer
+  float* v_first_ = nullptr;             // [rows][G dv] values of the first layer that mixes them (v_first_layer_; -1: none)
+  int v_first_layer_ = -1;
+  const float* zero_sink_ = nullptr;     // [heads] zeros
   int* last_tok_ = nullptr;              // [2][slots]
   std::vector<std::pair<std::string, std::pair<int, int>>> tensors_;  // name, (rows, columns)
   std::map<std::string, std::pair<int, int>> shape_;

@@ -75,12 +75,15 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
     if (s.mixer != t.mixer || s.heads != t.heads || s.dim != t.dim || s.vdim != t.vdim || s.kv_rank != t.kv_rank ||
         s.rot_dim != t.rot_dim || s.out_gate != t.out_gate || s.sink != t.sink || s.width != t.width || s.mlp != t.mlp ||
         s.post_norm != t.post_norm || s.resid_gate != t.resid_gate || s.norm_scalar != t.norm_scalar ||
-        s.kv_heads != t.kv_heads || s.attn_bias != t.attn_bias || s.beside != t.beside || s.lin.heads != t.lin.heads ||
+        s.kv_heads != t.kv_heads || s.attn_bias != t.attn_bias || s.qk_norm != t.qk_norm || s.head_temp != t.head_temp ||
+        s.v_mix != t.v_mix || s.mlp_scale != t.mlp_scale || s.act != t.act || s.beside != t.beside || s.lin.heads != t.lin.heads ||
         s.lin.groups != t.lin.groups || s.lin.dim != t.lin.dim || s.lin.vdim != t.lin.vdim || s.lin.conv != t.lin.conv ||
         s.lin.rank != t.lin.rank || s.mixer_scale != t.mixer_scale || s.mlp_bias != t.mlp_bias ||
         (s.mlp != MLP_NONE && (s.ff != t.ff || s.experts != t.experts || s.shared_ff != t.shared_ff || s.correction != t.correction)))
       throw std::runtime_error(at + "sizes differ from the layer whose weights it uses");
     if (s.mlp != MLP_NONE && s.ff < 1) throw std::runtime_error(at + "bad sizes");
+    if (s.mlp != MLP_ACT && (s.act == ACT_RELU2 || s.act == ACT_XIELU || s.mlp_scale != 1.f) && s.mlp != MLP_NONE)
+      throw std::runtime_error(at + "an activation without a gate, or a scale, in an MLP with one");
     if (s.mlp == MLP_MOE && (s.experts < 1 || s.experts > MOE_MAX_EXPERTS || s.top < 1 || s.top > std::min(s.experts, MOE_MAX_TOP) ||
                              s.shared_ff < 0))
       throw std::runtime_error(at + "bad number of experts");
@@ -119,6 +122,13 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
       if (s.heads < 1 || s.kv_heads < 1 || s.heads % s.kv_heads || s.dim < 1 || s.vdim < 1 || s.window < 0 || s.chunk < 0 ||
           s.rot_dims < 0 || s.rot_dims % 2 || s.rot_dims > s.dim || s.out_gate == GATE_ELEMENT)
         throw std::runtime_error(at + "bad sizes");
+      if (s.v_mix) {
+        if (v_first_layer_ < 0) v_first_layer_ = i;
+        const LayerSpec& f = c.layers[v_first_layer_];
+        if (s.kv_heads != f.kv_heads || s.vdim != f.vdim)
+          throw std::runtime_error(at + "values to mix differ in size from those of layer " + std::to_string(v_first_layer_));
+        if (c.loop_times > 0) throw std::runtime_error(at + "mixed values in a looped model");
+      }
       D.H = s.heads;
       D.G = s.kv_heads;
       D.dk = s.dim;
@@ -135,22 +145,22 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
       const int w = s.window && s.chunk ? std::min(s.window, s.chunk) : s.window + s.chunk;
       if (w) max_window_ = std::max(max_window_, w);
       else all_windowed = false;
-    } else if (s.mixer == MIX_MAMBA2 || s.mixer == MIX_GLA) {
+    } else if (s.mixer == MIX_MAMBA2 || s.mixer == MIX_GLA || s.mixer == MIX_DELTA) {
       n = 0;
     } else {
       throw std::runtime_error("unknown mixer kind");
     }
-    const int lin = s.mixer == MIX_MAMBA2 || s.mixer == MIX_GLA ? s.mixer : s.beside;
+    const int lin = s.mixer == MIX_MAMBA2 || s.mixer == MIX_GLA || s.mixer == MIX_DELTA ? s.mixer : s.beside;
     if (s.beside && s.mixer != MIX_GQA) throw std::runtime_error(at + "a second mixer stands beside grouped-query attention only");
     if (lin) {
       const LinSpec& l = s.lin;
-      const bool key = lin == MIX_GLA;
-      if (lin != MIX_MAMBA2 && lin != MIX_GLA) throw std::runtime_error(at + "unknown second mixer");
+      const bool key = lin == MIX_GLA, delta = lin == MIX_DELTA;
+      if (lin != MIX_MAMBA2 && !key && !delta) throw std::runtime_error(at + "unknown second mixer");
       if (l.heads < 1 || l.dim < 1 || l.vdim < 1 || !lin_pad_n(l.dim) || l.vdim > 1024 ||
-          (key ? l.rank < 1 || l.tau <= 0 : l.groups < 1 || l.heads % l.groups || l.conv < 1 || l.conv > 16 || l.norm_groups < 1 ||
-                                               (l.heads * l.vdim) % l.norm_groups))
+          (key ? l.rank < 1 || l.tau <= 0 : l.groups < 1 || l.heads % l.groups || l.conv < 1 || l.conv > 16) ||
+          (lin == MIX_MAMBA2 && (l.norm_groups < 1 || (l.heads * l.vdim) % l.norm_groups)))
         throw std::runtime_error(at + "bad sizes of the linear recurrence");
-      D.lin = key ? LIN_KEY : LIN_HEAD;
+      D.lin = key ? LIN_KEY : delta ? LIN_DELTA : LIN_HEAD;
       D.lH = l.heads;
       D.lG = key ? l.heads : l.groups;
       D.lN = l.dim;
@@ -159,7 +169,7 @@ LayeredDecoder::LayeredDecoder(Engine& e) : e_(e) {
       D.lvp = up(l.vdim, 16);
       D.lin_off = n;
       D.lin_out = D.gn;
-      n += key ? D.lH * (2 * D.lN + 2 * D.ldv) + l.rank : 2 * D.lH * D.ldv + 2 * D.lG * D.lN + D.lH;
+      n += key ? D.lH * (2 * D.lN + 2 * D.ldv) + l.rank : 2 * D.lH * D.ldv + 2 * D.lG * D.lN + (delta ? 2 : 1) * D.lH;
       D.gn += up(D.lH * D.ldv, 64);
       recurrent_ = true;
     }
@@ -227,17 +237,25 @@ void LayeredDecoder::alloc_layer(int i) {
       w.qb = falloc(D.H * D.dk);
       w.kb = falloc(D.G * D.dk);
       w.vb = falloc(D.G * D.dv);
-      w.ob = falloc(dp_);
+      if (s.attn_bias == 1) w.ob = falloc(dp_);
     }
+    if (s.qk_norm) {
+      w.qn = falloc(D.H * D.dk);
+      w.kn = falloc(D.G * D.dk);
+    }
+    if (s.head_temp) w.temp = falloc(D.H);
+    if (s.v_mix) w.lambda = falloc(1);
   }
-  if (D.lin == LIN_HEAD) {
+  if (D.lin == LIN_HEAD || D.lin == LIN_DELTA) {
     const int C = D.lH * D.ldv + 2 * D.lG * D.lN;
     w.conv_w = falloc((size_t)C * s.lin.conv);
-    w.conv_b = falloc(C);
     w.dt_b = falloc(D.lH);
     w.a_log = falloc(D.lH);
-    w.lin_d = falloc(D.lH);
-    w.lin_norm = falloc((size_t)D.lH * D.ldv);
+    w.lin_norm = falloc(D.lin == LIN_DELTA ? D.ldv : (size_t)D.lH * D.ldv);
+    if (D.lin == LIN_HEAD) {
+      w.conv_b = falloc(C);
+      w.lin_d = falloc(D.lH);
+    }
   } else if (D.lin == LIN_KEY) {
     w.a2 = falloc((size_t)D.lH * D.lN * s.lin.rank);
     w.a2_b = falloc((size_t)D.lH * D.lN);
@@ -257,6 +275,7 @@ void LayeredDecoder::alloc_layer(int i) {
   if (s.post_norm) w.post2 = falloc(dp_);
   if (s.resid_gate) w.rgb2 = falloc(dp_);
   w.in2 = balloc((size_t)(D.n2 + (s.mlp == MLP_ACT ? 1 : 2) * D.glu) * dp_);
+  w.act_n.scale = s.mlp_scale;
   if (s.mlp == MLP_ACT && s.mlp_bias) {
     w.upb = falloc(D.fp);
     w.dnb = falloc(dp_);
@@ -292,8 +311,7 @@ void LayeredDecoder::place(bf16_t* dst, int dpitch, const bf16_t* src, int spitc
                         device ? hipMemcpyDeviceToDevice : hipMemcpyHostToDevice));
 }
 
-// src's n numbers times `mul`, or (spread > 0) its one number that many times
-void LayeredDecoder::put_vec(float* dst, int n, const bf16_t* src, bool device, int spread, float mul) {
+static std::vector<float> numbers(const bf16_t* src, int n, bool device) {
   std::vector<bf16_t> h(n);
   std::vector<float> f(n);
   if (device) HIP_CHECK(hipMemcpy(h.data(), src, (size_t)n * 2, hipMemcpyDeviceToHost));
@@ -301,8 +319,14 @@ void LayeredDecoder::put_vec(float* dst, int n, const bf16_t* src, bool device, 
   for (int i = 0; i < n; ++i) {
     const uint32_t u = (uint32_t)h[i] << 16;
     std::memcpy(&f[i], &u, 4);
-    f[i] *= mul;
   }
+  return f;
+}
+
+// src's n numbers times `mul`, or (spread > 0) its one number that many times
+void LayeredDecoder::put_vec(float* dst, int n, const bf16_t* src, bool device, int spread, float mul) {
+  std::vector<float> f = numbers(src, n, device);
+  for (float& v : f) v *= mul;
   if (spread > 0) f.assign(spread, f[0]);
   HIP_CHECK(hipMemcpy(dst, f.data(), f.size() * 4, hipMemcpyHostToDevice));
 }
@@ -345,9 +369,15 @@ void LayeredDecoder::list_tensors() {
           {"attn_q", D.H * D.dk, d_}, {"attn_k", D.G * D.dk, d_}, {"attn_v", D.G * D.dv, d_}, {"attn_output", d_, D.H * D.dv}};
       for (const auto& m : mats) {
         add(p + m.n + ".weight", m.rows, m.cols);
-        if (s.attn_bias) add(p + m.n + ".bias", 1, m.rows);
+        if (s.attn_bias == 1 || (s.attn_bias && &m != &mats[3])) add(p + m.n + ".bias", 1, m.rows);
       }
-      if (s.sink) add(p + "attn_sinks.weight", 1, D.H);
+      if (s.qk_norm) {
+        add(p + "attn_q_norm.weight", 1, D.H * D.dk);
+        add(p + "attn_k_norm.weight", 1, D.G * D.dk);
+      }
+      if (s.head_temp) add(p + "attn_temp.weight", 1, D.H);
+      if (s.v_mix) add(p + "attn_v_mix.weight", 1, 1);
+      if (s.sink == 1) add(p + "attn_sinks.weight", 1, D.H);
       if (s.out_gate) add(p + "attn_gate.weight", D.H, d_);
     } else if (s.mixer == MIX_MINGRU) {
       for (const char* n : {"z", "x"}) {
@@ -367,6 +397,19 @@ void LayeredDecoder::list_tensors() {
       add(p + "ssm_d.bias", 1, D.lH);
       add(p + "ssm_norm.weight", 1, inner);
       add(p + "ssm_out.weight", d_, inner);
+    } else if (D.lin == LIN_DELTA) {
+      const int nk = D.lG * D.lN, nv = D.lH * D.ldv;
+      for (const char* n : {"q", "k", "v"}) {
+        add(p + "delta_" + n + ".weight", *n == 'v' ? nv : nk, d_);
+        add(p + "delta_" + n + "_conv1d.weight", *n == 'v' ? nv : nk, s.lin.conv);
+      }
+      add(p + "delta_b.weight", D.lH, d_);
+      add(p + "delta_a.weight", D.lH, d_);
+      add(p + "delta_dt.bias", 1, D.lH);
+      add(p + "delta_a_log.bias", 1, D.lH);
+      add(p + "delta_gate.weight", nv, d_);
+      add(p + "delta_norm.weight", 1, D.ldv);
+      add(p + "delta_output.weight", d_, nv);
     } else if (D.lin == LIN_KEY) {
       const int nk = D.lH * D.lN, nv = D.lH * D.ldv;
       add(p + "gla_q.weight", nk, d_);
@@ -405,6 +448,7 @@ void LayeredDecoder::list_tensors() {
         add(p + "ffn_up.bias", 1, D.ff);
         add(p + "ffn_down.bias", 1, d_);
       }
+      if (s.act == ACT_XIELU) add(p + "ffn_act.bias", 1, 2);
       continue;
     }
     add(p + "ffn_gate_inp.weight", s.experts, d_);
@@ -471,7 +515,29 @@ void LayeredDecoder::put(const std::string& name, int rows, int cols, const bf16
   else if (t == "attn_k.bias") put_vec(w.kb, cols, src, device);
   else if (t == "attn_v.bias") put_vec(w.vb, cols, src, device);
   else if (t == "attn_output.bias") put_vec(w.ob, cols, src, device, 0, s.mixer_scale);
-  else if (t == "ssm_in.weight" || t == "gla_q.weight") rows_at(w.in, D.lin_off);
+  else if (t == "attn_q_norm.weight") put_vec(w.qn, cols, src, device);
+  else if (t == "attn_k_norm.weight") put_vec(w.kn, cols, src, device);
+  else if (t == "attn_temp.weight") put_vec(w.temp, cols, src, device);
+  else if (t == "attn_v_mix.weight") put_vec(w.lambda, cols, src, device);
+  else if (t == "delta_v.weight") rows_at(w.in, D.lin_off);  // [v | k | q | gate | strengths | steps], convolved: [v | k | q]
+  else if (t == "delta_k.weight") rows_at(w.in, D.lin_off + D.lH * D.ldv);
+  else if (t == "delta_q.weight") rows_at(w.in, D.lin_off + D.lH * D.ldv + D.lG * D.lN);
+  else if (t == "delta_gate.weight") rows_at(w.in, D.lin_off + D.lH * D.ldv + 2 * D.lG * D.lN);
+  else if (t == "delta_b.weight") rows_at(w.in, D.lin_off + 2 * (D.lH * D.ldv + D.lG * D.lN));
+  else if (t == "delta_a.weight") rows_at(w.in, D.lin_off + 2 * (D.lH * D.ldv + D.lG * D.lN) + D.lH);
+  else if (t == "delta_v_conv1d.weight") put_vec(w.conv_w, rows * cols, src, device);
+  else if (t == "delta_k_conv1d.weight") put_vec(w.conv_w + (size_t)D.lH * D.ldv * cols, rows * cols, src, device);
+  else if (t == "delta_q_conv1d.weight") put_vec(w.conv_w + (size_t)(D.lH * D.ldv + D.lG * D.lN) * cols, rows * cols, src, device);
+  else if (t == "delta_dt.bias") put_vec(w.dt_b, cols, src, device);
+  else if (t == "delta_a_log.bias") put_vec(w.a_log, cols, src, device);
+  else if (t == "delta_norm.weight") put_vec(w.lin_norm, cols, src, device);
+  else if (t == "delta_output.weight") place(w.out + D.lin_out, D.kout, src, cols, cols, rows, device);
+  else if (t == "ffn_act.bias") {  // (its two numbers go into softplus)
+    const std::vector<float> f = numbers(src, 2, device);
+    auto softplus = [](double z) { return std::max(z, 0.0) + std::log1p(std::exp(-std::fabs(z))); };
+    w.act_n.pos = (float)softplus(f[0]);
+    w.act_n.neg = (float)(0.5 + softplus(f[1]));
+  } else if (t == "ssm_in.weight" || t == "gla_q.weight") rows_at(w.in, D.lin_off);
   else if (t == "gla_k.weight") rows_at(w.in, D.lin_off + D.lH * D.lN);
   else if (t == "gla_v.weight") rows_at(w.in, D.lin_off + 2 * D.lH * D.lN);
   else if (t == "gla_gate.weight") rows_at(w.in, D.lin_off + 2 * D.lH * D.lN + D.lH * D.ldv);
@@ -487,7 +553,7 @@ void LayeredDecoder::put(const std::string& name, int rows, int cols, const bf16
   else if (t == "ssm_out.weight" || t == "gla_output.weight") place(w.out + D.lin_out, D.kout, src, cols, cols, rows, device);
   else if (s.mlp == MLP_ACT && t == "ffn_up.weight") rows_at(w.in2, D.n2);
   else if (t == "ffn_up.bias") put_vec(w.upb, cols, src, device);
-  else if (t == "ffn_down.bias") put_vec(w.dnb, cols, src, device);
+  else if (t == "ffn_down.bias") put_vec(w.dnb, cols, src, device, 0, s.mlp_scale);
   else if (t == "attn_q.weight") {
     heads(w.in, dp_, D.dk + D.rot, D.dkp, 0, D.dk);
     if (D.rot) heads(w.in + (size_t)D.qrot * dp_, dp_, D.dk + D.rot, D.dkp, D.dk, D.rot);
@@ -543,7 +609,7 @@ void LayeredDecoder::init_random(uint64_t seed) {
   for (const auto& t : tensors_) {
     const int rows = t.second.first, cols = t.second.second;
     const size_t n = (size_t)rows * cols;
-    const bool norm = t.first.find("norm") != std::string::npos, sink = t.first.find("sinks") != std::string::npos;
+    const bool norm = t.first.find("norm") != std::string::npos || t.first.find("attn_temp") != std::string::npos, sink = t.first.find("sinks") != std::string::npos;
     const bool bias = t.first.find(".bias") != std::string::npos;
     bf16_t* tmp = nullptr;
     if (norm || sink || bias) {
@@ -645,6 +711,10 @@ void LayeredDecoder::finalize() {
     e_.pools_.push_back({k.pool, block});
     e_.kv_bytes_ += bytes;
   }
+  int heads = 0;
+  for (const LayerSpec& s : c.layers)
+    if (s.sink == 2) heads = std::max(heads, s.heads);
+  if (heads) zero_sink_ = falloc(heads);
   if (pairw_) last_tok_ = (int*)falloc((size_t)2 * c.max_slots);
   step_rows_ = std::max(Bm, std::min(2048, c.max_slots * c.max_ctx));
   if (const char* v = std::getenv("AIOS_STEP_ROWS")) step_rows_ = std::max(Bm, std::atoi(v));
@@ -691,6 +761,11 @@ void LayeredDecoder::finalize() {
     flat = std::max(flat, fl);
     part = std::max(part, fl * D.rp);
     kvw = std::max(kvw, (size_t)D.qn + D.gn);
+  }
+  if (v_first_layer_ >= 0) {
+    const size_t n = (size_t)R * dims_[v_first_layer_].G * dims_[v_first_layer_].dv;
+    v_first_ = falloc(n);
+    e_.ws_bytes_ += n * 4;
   }
   x_ = falloc((size_t)R * dp_);
   xh_ = falloc((size_t)R * dp_);
@@ -999,7 +1074,7 @@ size_t LayeredDecoder::state_floats(int i) const {
 }
 size_t LayeredDecoder::ring_floats(int i) const {
   const Dims& D = dims_[i];
-  return D.lin == LIN_HEAD ? (size_t)e_.cfg_.layers[i].lin.conv * (D.lH * D.ldv + 2 * D.lG * D.lN) : 0;
+  return D.lin == LIN_HEAD || D.lin == LIN_DELTA ? (size_t)e_.cfg_.layers[i].lin.conv * (D.lH * D.ldv + 2 * D.lG * D.lN) : 0;
 }
 
 void LayeredDecoder::linear(int k, const RowSet& r) {
@@ -1019,6 +1094,13 @@ void LayeredDecoder::linear(int k, const RowSet& r) {
     a.dt_off = c0 + 2 * nv + 2 * D.lG * D.lN;
     a.taps = s.lin.conv;
     a.norm_parts = s.lin.norm_groups;
+  } else if (D.lin == LIN_DELTA) {  // [v | k | q | gate | strengths | steps]
+    a.x_off = c0;
+    a.z_off = c0 + nv + 2 * D.lG * D.lN;
+    a.b_off = a.z_off + nv;
+    a.dt_off = a.b_off + D.lH;
+    a.taps = s.lin.conv;
+    a.q_scale = (float)(1.0 / std::sqrt((double)D.lN));
   } else {  // [q | k | v | gate | a]
     a.q_off = c0;
     a.k_off = c0 + nk;
@@ -1064,7 +1146,12 @@ void LayeredDecoder::grouped_attention(int k, const RowSet& r) {
   a.rot = D.rot; a.rope = rope_[i];
   a.window = s.window; a.chunk = s.chunk;
   a.scale = s.scale; a.softcap = s.softcap;
-  a.sink = s.sink ? w.sink : nullptr;
+  a.sink = s.sink == 2 ? zero_sink_ : s.sink ? w.sink : nullptr;
+  a.qn = w.qn; a.kn = w.kn; a.temp = w.temp;
+  a.v_norm = s.v_norm;
+  a.eps = e_.cfg_.norm_eps;
+  if (s.v_mix) a.first = v_first_;
+  a.lambda = s.v_mix && i != v_first_layer_ ? w.lambda : nullptr;
   a.qb = w.qb; a.kb = w.kb; a.vb = w.vb;
   a.in = qdg_; a.ld = D.n1; a.k_off = D.koff; a.v_off = D.voff; a.g_off = s.out_gate == GATE_HEAD ? D.gate_off : -1;
   a.out_scale = s.mixer_scale;
@@ -1171,7 +1258,7 @@ void LayeredDecoder::feed_forward(int k, const RowSet& r, RowCloseArgs& c) {
     if (D.n2) project(h, dp_, w.in2, n, D.n2, dp_, qdg_, D.n2);
     if (f32_) {
       launch_gemm_f32(h32_, dp_, wglu, dp_, n, D.fp, dp_, gu32_, D.fp, 0, e_.stream_);
-      launch_bias_act_f32(gu32_, D.fp, w.upb, cat32_, D.fp, n, D.fp, s.act, e_.stream_);
+      launch_bias_act_f32(gu32_, D.fp, w.upb, cat32_, D.fp, n, D.fp, s.act, w.act_n, e_.stream_);
     } else {
       if (n <= 4) {
         GemvArgs a = e_.gemv_args({}, D.fp, dp_, n, nullptr, dp_, nullptr, nullptr, D.fp, EPI_ACT16, 0);
@@ -1179,6 +1266,7 @@ void LayeredDecoder::feed_forward(int k, const RowSet& r, RowCloseArgs& c) {
         a.seg[0] = mat(wglu, D.fp, dp_);
         a.x16 = h16_;
         a.act = s.act;
+        a.act_n = w.act_n;
         a.bias = w.upb;
         a.y16 = cat16_;
         a.ldy16 = D.fp;
@@ -1190,7 +1278,7 @@ void LayeredDecoder::feed_forward(int k, const RowSet& r, RowCloseArgs& c) {
         std::memset(&g, 0, sizeof(g));
         g.A = h16_; g.lda = dp_; g.M = n; g.N = D.fp; g.K = dp_; g.nseg = 1; g.seg[0] = mat(wglu, D.fp, dp_);
         g.C16 = cat16_; g.ldc = D.fp; g.epi = GEPI_STORE16;
-        g.bias16 = w.upb; g.unary = 1 + s.act;
+        g.bias16 = w.upb; g.unary = 1 + s.act; g.act_n = w.act_n;
         e_.gemm(g);
       }
     }
@@ -1390,6 +1478,7 @@ void LayeredDecoder::layer_fused(int k, const RowSet& r) {
       a.nseg = 1;
       a.seg[0] = mat(m, N, dp_);
       a.act = s.act;
+      a.act_n = w.act_n;
       a.bias = bias;
       a.y16 = y16;
       a.ldy16 = N;
@@ -1401,6 +1490,7 @@ void LayeredDecoder::layer_fused(int k, const RowSet& r) {
     a.C = y; a.C16 = y16; a.ldc = N; a.epi = y16 ? GEPI_STORE16 : GEPI_STORE;
     a.bias16 = bias;
     if (y16) a.unary = 1 + s.act;
+    a.act_n = w.act_n;
     if (norm_ready_) { a.A = xn16_; a.nrm_in = npart_; a.nrm_parts = nparts_; a.nrm_eps = eps; }
     e_.gemm(a);
   };

@@ -100,8 +100,11 @@ void launch_mingru(const MinGruArgs& a, hipStream_t st);
 // Query head h reads key / value head h / (H / G).  Keys and values are cached per block of GQA_BLOCK tokens as
 // [G][block][dkp] keys, then [G][block][dvp] values.  Head sizes are padded to dkp / dvp (multiples of 32) there and in
 // q; the input product's columns are not.  Rotation turns the pairs (i, i + rot / 2) of a head's first rot dimensions.
-//   s = q . k * scale;  s = softcap tanh(s / softcap) (softcap > 0);  weights exp(s) / (exp(sink_h) + sum exp(s)) over the
-//   visible keys;  out_h = out_scale * sigmoid(gate_h) * sum weights v
+//   s = q . k * scale * temp_h;  s = softcap tanh(s / softcap) (softcap > 0);  weights exp(s) / (exp(sink_h) + sum exp(s)) over
+//   the visible keys;  out_h = out_scale * sigmoid(gate_h) * sum weights v
+// Before the rotation q and k may be divided by the root mean square of all their heads' columns together and multiplied by
+// weights (qn, kn); v may be divided, head by head, by its own (v_norm), and then mixed with another layer's values of the
+// same token (lambda).
 // A query at position i sees keys j <= i with j > i - window (window > 0) and floor(j / chunk) = floor(i / chunk)
 // (chunk > 0).
 constexpr int GQA_BLOCK = 64;
@@ -115,6 +118,12 @@ struct GqaArgs {
   float scale, softcap;
   const float* sink;          // [H] or null
   const float *qb, *kb, *vb;  // biases of q [H dk], k [G dk], v [G dv], or null
+  const float *qn, *kn;       // [H dk], [G dk] norm weights, or null
+  const float* temp;          // [H] or null
+  int v_norm;
+  float eps;                  // of these norms
+  float* first;               // [rows][G dv] or null: values kept for later layers, or (lambda set) those of that layer
+  const float* lambda;        // one number or null: v = (1 - lambda) v + lambda first
   const float* in;            // [rows][ld]: q, k, v at their offsets, gates at g_off + h (g_off -1: none)
   int ld, q_off, k_off, v_off, g_off;
   float out_scale;
@@ -146,12 +155,16 @@ bool gqa_supports(int dkp, int dvp);
 //             (y silu(z)) * norm_w [H dv].
 //   LIN_KEY   d_t one number per key channel (gated linear attention): d = sigmoid(a2 a + a2_b)^(1 / tau), k and v
 //             the input columns, q times q_scale (G = H).  out = rms(o) per head * norm_w [dv] * silu(z).
+//   LIN_DELTA d_t one number per head, as LIN_HEAD's; the convolved columns are v, k, q (group h / (H / G)), k and q made
+//             unit vectors, q times q_scale.  b_t = sigmoid(in), and instead of v_t the state takes
+//             u_t = b_t (v_t - d_t S_{t-1}^T k_t).  out as LIN_KEY's.
 // Portions run in blocks of LIN_T tokens: what a block needs besides the state it starts from (operands, decays,
 // scores between its own tokens) is prepared for all blocks side by side; then one wave per head and 16 columns of
 // v walks the blocks with its part of S in registers, long portions in segments side by side.  The state is kept twice, by parity of the position it was left
 // at, and the convolution's inputs in a ring of `taps` positions, so that a single token that is run again at the
 // same position finds what it started from.
-enum LinKind : int { LIN_HEAD = 1, LIN_KEY = 2 };
+enum LinKind : int { LIN_HEAD = 1, LIN_KEY = 2, LIN_DELTA = 3 };
+constexpr float LIN_UNIT_EPS = 1e-6f;  // of the unit vectors, beside the sum of squares
 constexpr int LIN_T = 16;
 constexpr int LIN_SEGS = 16, LIN_SEG_MIN = 8;  // segments of a step at most; blocks of a segment at least
 struct ScanSeq {
@@ -163,8 +176,9 @@ struct LinScanArgs {
   int H, G, N, np, dv, vp;    // np, vp: N and dv padded (lin_pad_n, multiple of 16)
   const float* in;            // [rows][ld] input product
   int ld, z_off;              // output gate [H dv]
-  int x_off, taps, dt_off;    // LIN_HEAD: convolved columns, step sizes [H]
-  const float *conv_w, *conv_b;        // [H dv + 2 G N][taps], last tap the current token's; bias
+  int x_off, taps, dt_off;    // LIN_HEAD, LIN_DELTA: convolved columns, step sizes [H]
+  int b_off;                  // LIN_DELTA: strengths [H]
+  const float *conv_w, *conv_b;        // [H dv + 2 G N][taps], last tap the current token's; bias or null
   const float *dt_b, *a_log, *D;       // [H]
   float* ring;                // [slots][taps][H dv + 2 G N]
   int q_off, k_off, v_off, a_off, rank;  // LIN_KEY
@@ -199,7 +213,8 @@ LinWs lin_ws(int kind, int H, int G, int np, int vp, bool f32);
 void launch_lin_scan(const LinScanArgs& a, hipStream_t st);
 
 // y[r][i] = act(x[r][i] + bias[i]) in fp32
-void launch_bias_act_f32(const float* x, int ldx, const float* bias, float* y, int ldy, int rows, int n, int act, hipStream_t st);
+void launch_bias_act_f32(const float* x, int ldx, const float* bias, float* y, int ldy, int rows, int n, int act, const ActNum& num,
+                         hipStream_t st);
 
 // ---- mixture of experts (kernels/moe.hip) -----------------------------------------------------------
 // Router: s = softmax(logits), the `top` largest of s + correction, weights s * scale.  The (token, expert) pairs

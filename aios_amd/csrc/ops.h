@@ -214,6 +214,7 @@ struct GemmQArgs {
   int glu_n0, ldc16; // GEPI_STORE_GLU
   const float* bias16;  // GEPI_STORE16, GEPI_ACCUM_NORM: [N] or null
   int unary;            // GEPI_STORE16: 0 none, else 1 + GluAct
+  ActNum act_n;         // its numbers
   int ksplit;        // K split over workgroups: 0 = auto, 1 = off
   // skinny (M <= 64) split-K: fp32 partial slabs [S][tiles][16*Mt][rows] + per-tile arrival
   // tickets (zero-initialised, re-armed by each tile's last arriver).  Null -> no split.

@@ -26,10 +26,10 @@ ROPE_NEOX = 2   # qwen: (x[i], x[i + rot/2])
 class LinConfig:
     """A linear recurrence with a matrix state (csrc/layered.h LinSpec)."""
     heads: int = 1
-    groups: int = 1                # heads that share B and C (mamba2)
+    groups: int = 1                # of heads that share B and C (mamba2) or a query and a key (delta)
     dim: int = 64                  # state rows (key channels) per head
     vdim: int = 64                 # state columns per head
-    conv: int = 4                  # taps (mamba2)
+    conv: int = 4                  # taps (mamba2, delta)
     norm_groups: int = 1           # parts of the gated norm (mamba2)
     rank: int = 8                  # width of the decay's first projection (gla)
     tau: float = 1.0               # root taken of the decay (gla)
@@ -38,9 +38,9 @@ class LinConfig:
 @dataclasses.dataclass(frozen=True)
 class LayerConfig:
     """One layer of a model described layer by layer (csrc/layered.h LayerSpec)."""
-    # "latent" attention | "mingru" | "gqa" attention | "mamba2" | "gla"
+    # "latent" attention | "mingru" | "gqa" attention | "mamba2" | "gla" | "delta" (gated delta rule)
     mixer: str = "latent"
-    # a second mixer reading the same input ("mamba2" | "gla"; "": none): mixer_scale * first + beside_scale * second
+    # a second mixer reading the same input ("mamba2" | "gla" | "delta"; "": none): mixer_scale * first + beside_scale * second
     beside: str = ""
     mixer_scale: float = 1.0
     beside_scale: float = 1.0
@@ -61,16 +61,24 @@ class LayerConfig:
     window: int = 0                # keys a token sees, itself included; 0: all before it
     scale: float = 0.125           # of q . k
     sink: bool = True              # a learned logit per head in the softmax's denominator
+    sink_one: bool = False         # gqa: one (the logit 0) in the denominator instead
     kv_heads: int = 1              # key / value heads (gqa), whose first rot_dims dimensions turn in halves
     chunk: int = 0                 # gqa: keys before a token's chunk of so many positions are out; 0: no chunks
     softcap: float = 0.0           # gqa: of the scores; 0: none
-    attn_bias: bool = False        # gqa: biases of q, k, v and the output projection
+    attn_bias: bool = False        # gqa: biases of q, k, v and (out_bias) the output projection
+    out_bias: bool = True
+    qk_norm: bool = False          # gqa: RMS norm of all of a token's queries at once, and of all its keys
+    v_norm: bool = False           # gqa: every head's value divided by its root mean square
+    head_temp: bool = False        # gqa: a learned number per head multiplies its scores
+    # gqa: from the second such layer on, values are mixed with the first such layer's by a learned number
+    v_mix: bool = False
     out_gate: str = "element"      # head outputs times sigmoid(Wg h): "none" | "element" | "head" (one number)
     width: int = 64                # of the state (mingru)
     ff: int = 256                  # hidden width of the MLP, or of every expert; 0: none
     gated: bool = True             # the MLP has a gate; else W_down act(W_up h + b) + b
-    act: str = "gelu_tanh"         # of the gate or the hidden layer: "gelu_tanh" | "silu" | "relu2" (no gate)
+    act: str = "gelu_tanh"         # of the gate or the hidden layer: "gelu_tanh" | "silu" | "relu2", "xielu" (no gate)
     mlp_bias: bool = False         # without a gate
+    mlp_scale: float = 1.0         # of the result, without a gate
     experts: int = 0               # mixture of experts (0: a dense MLP), of which every token uses `top`
     top: int = 0
     router_scale: float = 1.0
@@ -144,6 +152,9 @@ class ModelConfig:
                 if kind == "mamba2":
                     inner, gn = l.lin.heads * l.lin.vdim, 2 * l.lin.groups * l.lin.dim
                     n += d * (3 * inner + gn + l.lin.heads) + (inner + gn) * (l.lin.conv + 1) + inner
+                elif kind == "delta":
+                    nk, nv = l.lin.groups * l.lin.dim, l.lin.heads * l.lin.vdim
+                    n += d * (2 * nk + 3 * nv + 2 * l.lin.heads) + (2 * nk + nv) * l.lin.conv
                 elif kind == "gla":
                     nk, nv = l.lin.heads * l.lin.dim, l.lin.heads * l.lin.vdim
                     n += d * (2 * nk + 3 * nv + l.lin.rank) + nk * (l.lin.rank + 1)
@@ -239,6 +250,17 @@ def _sinisun(name: str, vocab: int, width: int, n_layers: int, ff: int, loop: Op
                        loop_add=True)
 
 
+def _seledra(name: str, vocab: int, width: int, n_layers: int, ff: int, max_ctx: int, delta: LinConfig, **attn) -> ModelConfig:
+    """Every third layer attention, the others the gated delta rule."""
+    mlp = dict(parallel=False, ff=ff, gated=False, act="xielu", mlp_scale=0.7, mixer_scale=0.7)
+    att = LayerConfig(mixer="gqa", sink=False, sink_one=True, out_gate="head", attn_bias=True, out_bias=False, qk_norm=True, v_norm=True,
+                      head_temp=True, v_mix=True, scale=attn["dim"] ** -0.5, **attn, **mlp)
+    rec = LayerConfig(mixer="delta", lin=delta, sink=False, out_gate="none", **mlp)
+    return ModelConfig(name=name, arch="seledra", vocab_size=vocab, d_model=width, n_layers=n_layers, n_heads=attn["heads"],
+                       n_kv_heads=attn["kv_heads"], head_dim=attn["dim"], d_ff=ff, max_ctx=max_ctx, bos_id=-1, eos_id=-1,
+                       layers=tuple(att if i % 3 == 1 else rec for i in range(n_layers)))
+
+
 PRESETS: Dict[str, ModelConfig] = {
     "tinyllama-1.1b": ModelConfig(
         name="tinyllama-1.1b", vocab_size=32000, d_model=2048, n_layers=22, n_heads=32, n_kv_heads=4,
@@ -311,6 +333,13 @@ PRESETS: Dict[str, ModelConfig] = {
                              LinConfig(heads=4, vdim=40, dim=24, groups=2, norm_groups=5, conv=3),
                              LinConfig(heads=3, dim=40, vdim=24, rank=8, tau=9.0), heads=6, kv_heads=3, dim=48, vdim=40,
                              rot_dims=32, chunk=50, softcap=20.0),
+    # as deep as the Sinisun presets are in layer runs
+    "seledra-1b": _seledra("seledra-1b", 32000, 2048, 22, 8448, 4096, LinConfig(heads=32, vdim=128, dim=128, groups=16),
+                           heads=32, kv_heads=4, dim=64, vdim=64),
+    "seledra-7b": _seledra("seledra-7b", 32000, 4096, 32, 21504, 8192, LinConfig(heads=64, vdim=128, dim=128, groups=32),
+                           heads=32, kv_heads=8, dim=128, vdim=128),
+    "test-seledra": _seledra("test-seledra", 600, 384, 4, 512, 512, LinConfig(heads=6, vdim=40, dim=24, groups=2, conv=3),
+                             heads=6, kv_heads=3, dim=48, vdim=40),
     "test-mistral-shape": ModelConfig(
         name="test-mistral-shape", vocab_size=1024, d_model=1024, n_layers=2, n_heads=8, n_kv_heads=2,
         head_dim=128, d_ff=2048, rope_theta=1e6, max_ctx=512, chat_template="mistral"),

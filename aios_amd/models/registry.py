@@ -24,7 +24,7 @@ class Architecture:
 
 
 # architecture -> module under aios_amd.models that defines ARCHITECTURE
-_MODULES = {"gefazen": "gefazen", "movalorn": "movalorn", "sinisun": "sinisun"}
+_MODULES = {"gefazen": "gefazen", "movalorn": "movalorn", "sinisun": "sinisun", "seledra": "seledra"}
 
 
 def architectures():

@@ -158,10 +158,11 @@ def engine_config(cfg, max_ctx: Optional[int] = None, max_slots: int = 4, max_ba
 def _layer_spec(m, l):
     s = m.LayerSpec()
     kinds = {"": m.MIX_NONE, "latent": m.MIX_LATENT, "mingru": m.MIX_MINGRU, "gqa": m.MIX_GQA, "mamba2": m.MIX_MAMBA2,
-             "gla": m.MIX_GLA}
+             "gla": m.MIX_GLA, "delta": m.MIX_DELTA}
     s.mixer, s.beside = kinds[l.mixer], kinds[l.beside]
     s.mixer_scale, s.beside_scale = float(l.mixer_scale), float(l.beside_scale)
-    s.kv_heads, s.chunk, s.softcap, s.attn_bias = l.kv_heads, l.chunk, float(l.softcap), int(l.attn_bias)
+    s.kv_heads, s.chunk, s.softcap, s.attn_bias = l.kv_heads, l.chunk, float(l.softcap), (1 if l.out_bias else 2) if l.attn_bias else 0
+    s.qk_norm, s.v_norm, s.head_temp, s.v_mix = int(l.qk_norm), int(l.v_norm), int(l.head_temp), int(l.v_mix)
     if l.lin is not None:
         lin = m.LinSpec()
         lin.heads, lin.groups, lin.dim, lin.vdim = l.lin.heads, l.lin.groups, l.lin.dim, l.lin.vdim
@@ -172,14 +173,15 @@ def _layer_spec(m, l):
     s.heads, s.dim, s.vdim, s.kv_rank = l.heads, l.dim, l.vdim, l.kv_rank
     s.rot_dim, s.rot_dims, s.rot_base, s.window = l.rot_dim, l.rot_dims, float(l.rot_base), l.window
     s.scale = float(l.scale)
-    s.sink = int(l.sink)
+    s.sink = 2 if l.sink_one else int(l.sink)
     s.out_gate = {"none": m.GATE_NONE, "element": m.GATE_ELEMENT, "head": m.GATE_HEAD}[l.out_gate]
     s.width = l.width
     s.mlp, s.ff = (m.MLP_MOE if l.experts else m.MLP_GLU if l.gated else m.MLP_ACT, l.ff) if l.ff else (m.MLP_NONE, 0)
-    s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU, "relu2": m.ACT_RELU2}[l.act]
-    if s.mlp in (m.MLP_GLU, m.MLP_MOE) and s.act == m.ACT_RELU2:
-        raise ValueError("the square of relu is no gate's activation")
-    s.mlp_bias = int(l.mlp_bias)
+    s.act = {"gelu_tanh": m.ACT_GELU_TANH, "silu": m.ACT_SILU, "relu2": m.ACT_RELU2,
+             "xielu": m.ACT_XIELU}[l.act]
+    if s.mlp in (m.MLP_GLU, m.MLP_MOE) and s.act in (m.ACT_RELU2, m.ACT_XIELU):
+        raise ValueError(f"{l.act} is no gate's activation")
+    s.mlp_bias, s.mlp_scale = int(l.mlp_bias), float(l.mlp_scale)
     s.experts, s.top, s.shared_ff = l.experts, l.top, l.shared_ff
     s.router_scale, s.correction = float(l.router_scale), int(l.correction)
     s.weights_of = l.weights_of
