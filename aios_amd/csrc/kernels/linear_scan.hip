@@ -1073,7 +1073,7 @@ void launch_lin_scan(const LinScanArgs& a, hipStream_t st) {
   if ((a.seqs ? a.n_seqs : a.n) < 1) return;
   if (a.seqs && (a.nseg < 1 || (a.nseg > 1 && (!a.seg || !a.seg_dec || a.nseg * a.n_seqs > LIN_SEGS))))
     throw std::runtime_error("linear scan: bad segments");
-  if (a.kind == LIN_DELTA && a.nseg != 1) throw std::runtime_error("linear scan: the delta rule is walked in one segment");
+  if (a.kind == LIN_DELTA && a.seqs && a.nseg != 1) throw std::runtime_error("linear scan: the delta rule is walked in one segment");
   switch (a.kind) {
     case LIN_KEY: return a.f32 ? lin_go<true, LIN_KEY>(a, st) : lin_go<false, LIN_KEY>(a, st);
     case LIN_DELTA: return a.f32 ? lin_go<true, LIN_DELTA>(a, st) : lin_go<false, LIN_DELTA>(a, st);

@@ -333,10 +333,10 @@ PRESETS: Dict[str, ModelConfig] = {
                              LinConfig(heads=4, vdim=40, dim=24, groups=2, norm_groups=5, conv=3),
                              LinConfig(heads=3, dim=40, vdim=24, rank=8, tau=9.0), heads=6, kv_heads=3, dim=48, vdim=40,
                              rot_dims=32, chunk=50, softcap=20.0),
-    # as deep as the Sinisun presets are in layer runs
-    "seledra-1b": _seledra("seledra-1b", 32000, 2048, 22, 8448, 4096, LinConfig(heads=32, vdim=128, dim=128, groups=16),
+    # as deep as the Sinisun presets are in layer runs, states and MLPs as large
+    "seledra-1b": _seledra("seledra-1b", 32000, 2048, 22, 8448, 4096, LinConfig(heads=32, vdim=128, dim=128, groups=8),
                            heads=32, kv_heads=4, dim=64, vdim=64),
-    "seledra-7b": _seledra("seledra-7b", 32000, 4096, 32, 21504, 8192, LinConfig(heads=64, vdim=128, dim=128, groups=32),
+    "seledra-7b": _seledra("seledra-7b", 32000, 4096, 32, 21504, 8192, LinConfig(heads=64, vdim=128, dim=128, groups=16),
                            heads=32, kv_heads=8, dim=128, vdim=128),
     "test-seledra": _seledra("test-seledra", 600, 384, 4, 512, 512, LinConfig(heads=6, vdim=40, dim=24, groups=2, conv=3),
                              heads=6, kv_heads=3, dim=48, vdim=40),

@@ -60,7 +60,7 @@ def parse():
                     help="skip the goal->plan latency secondary (BASELINE.json's agent metric)")
     ap.add_argument("--tp-model", default="llama3-70b")
     ap.add_argument("--tp-steps", type=int, default=64)
-    ap.add_argument("--design", default="", choices=("", "gefazen", "movalorn", "sinisun"),
+    ap.add_argument("--design", default="", choices=("", "gefazen", "movalorn", "sinisun", "seledra"),
                     help="instead of the headline: prefill and decode throughput of this design at the sizes of two real "
                          "models' layers (random weights), beside the closest other model of equal size with bf16 weights; "
                          "one JSON line per measurement, one GPU")
@@ -126,7 +126,8 @@ def measure(preset: str, recipe: str, batch: int, prompt: int, steps: int, warmu
 # numbers a token uses)
 DESIGN_PAIRS = {"gefazen": (("gefazen-1b", "tinyllama-1.1b"), ("gefazen-7b", "mistral-7b")),
                 "movalorn": (("movalorn-1b", "gefazen-1b"), ("movalorn-7b", "gefazen-7b")),
-                "sinisun": (("sinisun-1b", "tinyllama-1.1b"), ("sinisun-7b", "mistral-7b"))}
+                "sinisun": (("sinisun-1b", "tinyllama-1.1b"), ("sinisun-7b", "mistral-7b")),
+                "seledra": (("seledra-1b", "sinisun-1b"), ("seledra-7b", "sinisun-7b"))}
 DESIGN_DECODE = ((1, 128), (1, 2048), (4, 2048), (16, 1024), (32, 1024))   # (sequences, context)
 DESIGN_PREFILL = (128, 512, 2048)
 
