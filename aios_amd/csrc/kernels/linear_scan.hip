@@ -1,5 +1,4 @@
-// Linear recurrences with a matrix state (mixers.h LinScanArgs): per head S_t = d_t S_{t-1} + k_t v_t^T, o_t = S_t^T q_t;
-// LIN_DELTA with u_t = b_t (v_t - d_t S_{t-1}^T k_t) in the place of v_t.
+// Linear recurrences with a matrix state (mixers.h LinScanArgs): per head S_t = d_t S_{t-1} + k_t v_t^T, o_t = S_t^T q_t.
 //
 // Portions, in blocks of 16 tokens:
 //   conv (LIN_HEAD)    a thread per channel and block: convolution, SiLU, operands in the order the walk reads them
@@ -12,10 +11,8 @@
 //                      Where heads and columns leave compute units idle, a portion is walked in segments side by side: a
 //                      first walk takes every segment but the last from zero (the first one from the state) to its end,
 //                      without outputs; the second starts each segment from what those before it make together.
-//                      LIN_DELTA: within a block (I + L) U = diag(b) (V - decayed K S), L[t][s] = b_t (d_t .. d_{s+1}) k_t . k_s,
-//                        s < t; score leaves (I + L)^-1 diag(b), and U is one more product in the walk.  Lengths of k and q
-//                        are numbers per token and go with the decays.
 //   norm               root-mean-square of the parts, weight, output gate
+// LIN_DELTA has a score and a walk of its own (delta_rule.hip); convolution and norm are shared.
 // Single tokens: lin_step, one workgroup per head and row (convolution, decays, state and, for LIN_KEY, the norm).
 //
 // fp32: state, decays, step sizes, cumulative decays, scores, norms, gates.  The products take bf16 operands: q, k, v and
@@ -24,12 +21,9 @@
 #include <algorithm>
 #include <stdexcept>
 
-#include "../mixers.h"
-#include "gemm_common.h"
+#include "lin_common.h"
 
 namespace aios {
-
-typedef unsigned int lu2 __attribute__((ext_vector_type(2)));
 
 int lin_pad_n(int n) {
   for (int t : {32, 64, 96, 128, 192, 256})
@@ -37,91 +31,29 @@ int lin_pad_n(int n) {
   return 0;
 }
 
-// numbers a head's block keeps beside its operands (LIN_HEAD, LIN_DELTA): per token the decay since the block's start, and
-// to its end times what the input is multiplied by; LIN_DELTA: the first times the key's length; then the block's decay
-static constexpr int lin_decs(int kind) { return kind == LIN_DELTA ? 64 : 48; }
-
 // numbers per block of LIN_T tokens; bf16: decayed operands have a second plane behind the first
 LinWs lin_ws(int kind, int H, int G, int np, int vp, bool f32) {
-  const size_t g = kind == LIN_KEY ? H : G, two = f32 ? 1 : 2, q = g * np * LIN_T, delta = kind == LIN_DELTA ? 2 : 1;
+  const size_t g = kind == LIN_KEY ? H : G, two = f32 ? 1 : 2, q = g * np * LIN_T;
   LinWs w;
   w.qo = kind == LIN_KEY ? q * two : q;
   w.ko = w.qo;
   w.kr = kind != LIN_KEY ? q : 0;
   w.vo = (size_t)H * vp * LIN_T;
-  w.so = (size_t)H * 256 * two * delta;
-  w.dec = kind == LIN_KEY ? (size_t)H * np : (size_t)H * lin_decs(kind);
+  w.so = (size_t)H * 256 * two * (kind == LIN_DELTA ? 3 : 1);
+  w.dec = kind == LIN_KEY ? (size_t)H * np : (size_t)H * (kind == LIN_DELTA ? 64 : 48);
   return w;
-}
-
-template <bool F32>
-__device__ __forceinline__ float ls_exp(float x) { return F32 ? expf(x) : __expf(x); }
-template <bool F32>
-__device__ __forceinline__ float ls_silu(float z) { return z / (1.f + ls_exp<F32>(-z)); }
-// log(1 + e^z)
-__device__ __forceinline__ float ls_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-
-// two floats -> bf16 pairs (hi) and what the rounding left (lo)
-__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
-  hi = pk_bf16(a, b);
-  lo = pk_bf16(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
-}
-__device__ __forceinline__ void split4(gf32x4 v, lu2& hi, lu2& lo) {
-  uint32_t h0, l0, h1, l1;
-  split2(v[0], v[1], h0, l0);
-  split2(v[2], v[3], h1, l1);
-  hi = lu2{h0, h1};
-  lo = lu2{l0, l1};
-}
-__device__ __forceinline__ gf32x4 mfma32(lu2 a0, lu2 a1, lu2 b0, lu2 b1, gf32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(gbf16x8, make_uint4(a0.x, a0.y, a1.x, a1.y)),
-                                                 __builtin_bit_cast(gbf16x8, make_uint4(b0.x, b0.y, b1.x, b1.y)), c, 0, 0, 0);
-}
-// one 16-deep product in fp32: step r takes the depths 4 (lane / 16) + r
-__device__ __forceinline__ gf32x4 mfma4(gf32x4 a, gf32x4 b, gf32x4 c) {
-#pragma unroll
-  for (int r = 0; r < 4; ++r) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], c, 0, 0, 0);
-  return c;
-}
-
-// 16 numbers of one row of an operand
-template <bool F32>
-__device__ __forceinline__ void put16(void* base, size_t at, const float (&v)[16]) {
-  if constexpr (F32) {
-#pragma unroll
-    for (int i = 0; i < 16; i += 4) *(float4*)((float*)base + at + i) = make_float4(v[i], v[i + 1], v[i + 2], v[i + 3]);
-  } else {
-    uint32_t u[8];
-#pragma unroll
-    for (int i = 0; i < 8; ++i) u[i] = pk_bf16(v[2 * i], v[2 * i + 1]);
-    *(uint4*)((bf16_t*)base + at) = make_uint4(u[0], u[1], u[2], u[3]);
-    *(uint4*)((bf16_t*)base + at + 8) = make_uint4(u[4], u[5], u[6], u[7]);
-  }
-}
-template <bool F32>
-__device__ __forceinline__ void put1(void* base, size_t at, float v) {
-  if constexpr (F32) ((float*)base)[at] = v;
-  else ((bf16_t*)base)[at] = f32_to_bf16(v);
-}
-
-// a block's rows of the step
-struct LinBlock {
-  int row0, n, slot, pos0, seq_pos0;  // seq_pos0: the portion's first position
-};
-__device__ __forceinline__ LinBlock lin_block(const LinScanArgs& a, int b) {
-  const ScanChunk c = a.chunks[b >> 1];
-  const int t0 = (b & 1) * LIN_T;
-  return LinBlock{c.row0 + t0, min(LIN_T, c.n - t0), c.slot, c.pos0 + t0, a.chunks[c.first].pos0};
 }
 
 // ---- LIN_HEAD, LIN_DELTA: convolution --------------------------------------------------------------------------
 constexpr int LC_T = 128;
 
-// TM: taps at most
-template <bool F32, int TM>
+// TM: taps at most; PAIRS: a pair of blocks, in the operands' order of delta_rule.hip
+template <bool F32, int TM, bool PAIRS>
 __global__ void __launch_bounds__(LC_T) lin_conv_kernel(LinScanArgs a) {
-  const LinBlock bl = lin_block(a, blockIdx.y);
+  constexpr int TOK = PAIRS ? 2 * LIN_T : LIN_T;
+  LinBlock bl = lin_block(a, PAIRS ? 2 * blockIdx.y : blockIdx.y);
   if (bl.n < 1) return;
+  if (PAIRS) bl.n = a.chunks[blockIdx.y].n;
   const int nx = a.H * a.vp, ng = a.G * a.np;
   int c = blockIdx.x * LC_T + threadIdx.x;
   if (c >= nx + 2 * ng) return;
@@ -139,15 +71,15 @@ __global__ void __launch_bounds__(LC_T) lin_conv_kernel(LinScanArgs a) {
     i = k - hd * a.np;
     if (i < a.N) raw = a.H * a.dv + (sec - 1) * a.G * a.N + hd * a.N + i;
   }
-  float u[16];
+  float u[TOK];
 #pragma unroll
-  for (int t = 0; t < 16; ++t) u[t] = 0.f;
+  for (int t = 0; t < TOK; ++t) u[t] = 0.f;
   if (raw >= 0) {
-    float w[TM], x[16 + TM - 1];  // w[d]: tap of lag d
+    float w[TM], x[TOK + TM - 1];  // w[d]: tap of lag d
 #pragma unroll
     for (int d = 0; d < TM; ++d) w[d] = d < a.taps ? a.conv_w[(size_t)raw * a.taps + a.taps - 1 - d] : 0.f;
 #pragma unroll
-    for (int j = 0; j < 16 + TM - 1; ++j) {
+    for (int j = 0; j < TOK + TM - 1; ++j) {
       const int t = j - (TM - 1), p = bl.pos0 + t;  // token t of the block
       x[j] = 0.f;
       if (t >= bl.n || -t >= a.taps) continue;
@@ -156,7 +88,7 @@ __global__ void __launch_bounds__(LC_T) lin_conv_kernel(LinScanArgs a) {
     }
     const float b = a.conv_b ? a.conv_b[raw] : 0.f;
 #pragma unroll
-    for (int t = 0; t < 16; ++t) {
+    for (int t = 0; t < TOK; ++t) {
       float s = b;
 #pragma unroll
       for (int d = 0; d < TM; ++d) s = fmaf(w[d], x[t + TM - 1 - d], s);
@@ -164,28 +96,34 @@ __global__ void __launch_bounds__(LC_T) lin_conv_kernel(LinScanArgs a) {
     }
   }
   const size_t blk = blockIdx.y;
-  if (sec == 0) return put16<F32>(a.vo, ((blk * a.H + hd) * a.vp + i) * 16, u);
-  const size_t base = (blk * a.G + hd) * a.np;
-  if (sec == 1) put16<F32>(a.ko, (base + i) * 16, u);
-  void* rows = sec == 1 ? a.kr : a.qo;
+  if constexpr (PAIRS) {
+    if (sec < 2) {  // (four tokens of the first block, then the same of the second)
+      float o[2][16];
 #pragma unroll
-  for (int t = 0; t < 16; ++t) put1<F32>(rows, (base + (i & ~15)) * 16 + t * 16 + (i & 15), u[t]);
+      for (int t = 0; t < TOK; ++t) o[(t & 15) >> 3][((t >> 2) & 1) * 8 + (t >> 4) * 4 + (t & 3)] = u[t];
+      void* cols = sec == 0 ? a.vo : a.ko;
+      const size_t at = (sec == 0 ? (blk * a.H + hd) * a.vp + i : (blk * a.G + hd) * a.np + i) * TOK;
+      put16<F32>(cols, at, o[0]);
+      put16<F32>(cols, at + 16, o[1]);
+      if (sec == 0) return;
+    }
+#pragma unroll
+    for (int t = 0; t < TOK; ++t)
+      put1<F32>(sec == 1 ? a.kr : a.qo, ((2 * blk + (t >> 4)) * a.G + hd) * a.np * 16 + pair_row(i, t & 15), u[t]);
+  } else {
+    if (sec == 0) return put16<F32>(a.vo, ((blk * a.H + hd) * a.vp + i) * 16, u);
+    const size_t base = (blk * a.G + hd) * a.np;
+    if (sec == 1) put16<F32>(a.ko, (base + i) * 16, u);
+    void* rows = sec == 1 ? a.kr : a.qo;
+#pragma unroll
+    for (int t = 0; t < 16; ++t) put1<F32>(rows, (base + (i & ~15)) * 16 + t * 16 + (i & 15), u[t]);
+  }
 }
 
-// ---- LIN_HEAD, LIN_DELTA: decays and scores; the last inputs into the ring ---------------------------------
-template <bool F32, bool DELTA>
+// ---- LIN_HEAD: decays and scores; the last inputs into the ring -----------------------------------------
+template <bool F32>
 __global__ void __launch_bounds__(256) lin_score_kernel(LinScanArgs a, int nscore, int nkeep) {
-  if ((int)blockIdx.x >= nscore) {  // (the convolution, which reads the ring, is a launch before this one)
-    const int C = a.H * a.dv + 2 * a.G * a.N, k = blockIdx.x - nscore;
-    const ScanSeq s = a.seqs[k / nkeep];
-    const int c = (k % nkeep) * 256 + threadIdx.x;
-    if (c >= C) return;
-    for (int i = 0; i < min(s.n, a.taps); ++i) {
-      const int t = s.n - 1 - i;
-      a.ring[((size_t)s.slot * a.taps + (s.pos0 + t) % a.taps) * C + c] = a.in[(size_t)(s.row0 + t) * a.ld + a.x_off + c];
-    }
-    return;
-  }
+  if ((int)blockIdx.x >= nscore) return lin_keep(a, blockIdx.x - nscore, nkeep);
   const int lane = threadIdx.x & 63, idx = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int blk = idx / a.H, h = idx - blk * a.H;
   if (blk >= 2 * a.n_chunks) return;
@@ -203,83 +141,32 @@ __global__ void __launch_bounds__(256) lin_score_kernel(LinScanArgs a, int nscor
     if (r16 >= d) cum += o;
   }
   const float tot = __shfl(cum, 15, 16);
-  float* dec = a.dec + ((size_t)blk * a.H + h) * lin_decs(DELTA ? LIN_DELTA : LIN_HEAD);
+  float* dec = a.dec + ((size_t)blk * a.H + h) * 48;
+  if (q == 0) {
+    dec[r16] = expf(cum);
+    dec[16 + r16] = dt * expf(tot - cum);
+    if (r16 == 0) dec[32] = expf(tot);
+  }
   // A^T[s][t] = k_s . q_t: a lane holds s = 4 q + r, t = r16
   const size_t base = ((size_t)blk * a.G + h / (a.H / a.G)) * a.np * 16 + r16 * 16 + 4 * q;
-  gf32x4 acc = {0.f, 0.f, 0.f, 0.f}, kk = acc, qq = acc;  // (DELTA: k_s . k_t and q_s . q_t too)
+  gf32x4 acc = {0.f, 0.f, 0.f, 0.f};
   for (int i = 0; i < a.np / 16; i += 2) {
     const size_t at = base + (size_t)i * 256;
     if constexpr (F32) {
-#pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        const gf32x4 k = *(const gf32x4*)((const float*)a.kr + at + 256 * j), qv = *(const gf32x4*)((const float*)a.qo + at + 256 * j);
-        acc = mfma4(k, qv, acc);
-        if constexpr (DELTA) {
-          kk = mfma4(k, k, kk);
-          qq = mfma4(qv, qv, qq);
-        }
-      }
+      acc = mfma4(*(const gf32x4*)((const float*)a.kr + at), *(const gf32x4*)((const float*)a.qo + at), acc);
+      acc = mfma4(*(const gf32x4*)((const float*)a.kr + at + 256), *(const gf32x4*)((const float*)a.qo + at + 256), acc);
     } else {
       const bf16_t *kr = (const bf16_t*)a.kr + at, *qr = (const bf16_t*)a.qo + at;
-      const lu2 k0 = *(const lu2*)kr, k1 = *(const lu2*)(kr + 256), q0 = *(const lu2*)qr, q1 = *(const lu2*)(qr + 256);
-      acc = mfma32(k0, k1, q0, q1, acc);
-      if constexpr (DELTA) {
-        kk = mfma32(k0, k1, k0, k1, kk);
-        qq = mfma32(q0, q1, q0, q1, qq);
-      }
+      acc = mfma32(*(const lu2*)kr, *(const lu2*)(kr + 256), *(const lu2*)qr, *(const lu2*)(qr + 256), acc);
     }
   }
-  float iq = 1.f, ik = dt;  // what q and the state's input of token r16 are multiplied by
-  if constexpr (DELTA) {
-    float nk = 0.f, nq = 0.f;
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      if (4 * q + r == r16) {
-        nk = kk[r];
-        nq = qq[r];
-      }
-    const int diag = (r16 >> 2) * 16 + r16;
-    ik = 1.f / sqrtf(__shfl(nk, diag, 64) + LIN_UNIT_EPS);
-    iq = a.q_scale / sqrtf(__shfl(nq, diag, 64) + LIN_UNIT_EPS);
-  }
-  if (q == 0) {
-    dec[r16] = iq * expf(cum);
-    dec[16 + r16] = ik * expf(tot - cum);
-    if constexpr (DELTA) dec[32 + r16] = ik * expf(cum);
-    if (r16 == 0) dec[DELTA ? 48 : 32] = expf(tot);
-  }
-  const float beta = DELTA && r16 < bl.n ? 1.f / (1.f + expf(-a.in[(size_t)(bl.row0 + r16) * a.ld + a.b_off + h])) : 0.f;
-  gf32x4 low;
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int s = 4 * q + r;
-    const float cs = __shfl(cum, s, 16), is = __shfl(ik, s, 16), d = s <= r16 ? is * expf(cum - cs) : 0.f;
-    acc[r] *= d * iq;
-    if constexpr (DELTA) low[r] = s < r16 ? kk[r] * d * ik * beta : 0.f;
+    const float cs = __shfl(cum, s, 16), ds = __shfl(dt, s, 16);
+    acc[r] = s <= r16 ? acc[r] * ds * expf(cum - cs) : 0.f;
   }
-  if constexpr (DELTA) {  // column r16 of (I + low)^-1, row after row
-    __shared__ float sl[4][16][20];
-    float(*l)[20] = sl[threadIdx.x >> 6];
-    *(gf32x4*)(l[r16] + 4 * q) = low;
-    // (a wave's slice of LDS is its own and LDS executes a wave's accesses in order; the fence keeps the compiler to it)
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    float x[16];
-#pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      x[i] = i == r16 ? 1.f : 0.f;
-#pragma unroll
-      for (int s = 0; s < i; ++s) x[i] = fmaf(-l[i][s], x[s], x[i]);
-    }
-    const size_t at = ((size_t)blk * a.H + h) * (F32 ? 512 : 1024) + (F32 ? 256 : 512) + r16;
-#pragma unroll
-    for (int i = 0; i < 16; ++i)
-      if (i >> 2 == q) {
-        const float v = x[i] * beta;
-        put1<F32>(a.so, at + i * 16, v);
-        if constexpr (!F32) put1<F32>(a.so, at + 256 + i * 16, v - bf16_to_f32(f32_to_bf16(v)));
-      }
-  }
-  const size_t at = ((size_t)blk * a.H + h) * (F32 ? 256 : 512) * (DELTA ? 2 : 1) + r16 * 16 + 4 * q;
+  const size_t at = ((size_t)blk * a.H + h) * (F32 ? 256 : 512) + r16 * 16 + 4 * q;
   if constexpr (F32) {
     *(gf32x4*)((float*)a.so + at) = acc;
   } else {
@@ -404,32 +291,28 @@ __global__ void __launch_bounds__(256) lin_key_prep_kernel(LinScanArgs a) {
 }
 
 // ---- the walk ---------------------------------------------------------------------------------------
-// (kr: keys token by token, and i: the block's (I + L)^-1 diag(b), of LIN_DELTA)
-template <bool F32, int KIND, int NT>
+template <bool F32, bool KEY, int NT>
 struct LinOps;
-template <int KIND, int NT>
-struct LinOps<false, KIND, NT> {
-  static constexpr int K = KIND == LIN_KEY ? NT : 1, D = KIND == LIN_DELTA ? NT : 1;
-  lu2 q[NT], ql[K], k[NT], kl[K], kr[D], s, sl, i, il, v;
-  gf32x4 d[KIND == LIN_KEY ? NT : KIND == LIN_DELTA ? 3 : 2];
+template <bool KEY, int NT>
+struct LinOps<false, KEY, NT> {
+  lu2 q[NT], ql[KEY ? NT : 1], k[NT], kl[KEY ? NT : 1], s, sl, v;
+  gf32x4 d[KEY ? NT : 2];
   float tot;
 };
-template <int KIND, int NT>
-struct LinOps<true, KIND, NT> {
-  gf32x4 q[NT], k[NT], kr[KIND == LIN_DELTA ? NT : 1], s, i, v, d[KIND == LIN_KEY ? NT : KIND == LIN_DELTA ? 3 : 2];
+template <bool KEY, int NT>
+struct LinOps<true, KEY, NT> {
+  gf32x4 q[NT], k[NT], s, v, d[KEY ? NT : 2];
   float tot;
 };
 
 // buffers of operands in registers: requests run that many blocks ahead, less one
-template <bool F32, int KIND, int NT>
+template <bool F32, bool KEY, int NT>
 constexpr int lin_depth() {
-  constexpr bool KEY = KIND == LIN_KEY;
   if (F32) return 2;
-  if (KIND == LIN_DELTA) return NT <= 4 ? 4 : NT <= 8 ? 3 : 2;
   return KEY ? (NT <= 2 ? 4 : NT <= 4 ? 3 : NT <= 6 ? 4 : NT <= 8 ? 3 : 2) : (NT <= 4 ? 4 : NT <= 6 ? 3 : NT <= 8 ? 2 : NT <= 12 ? 3 : 2);
 }
 // waves a SIMD whose registers fit
-constexpr int lin_waves(int kind, int nt) { return kind == LIN_DELTA ? 1 : nt <= (kind == LIN_KEY ? 4 : 8) ? 2 : 1; }
+constexpr int lin_waves(bool key, int nt) { return nt <= (key ? 4 : 8) ? 2 : 1; }
 
 // the blocks of a portion that a segment walks: [i0, i1), and how many segments there are
 struct LinSeg {
@@ -442,19 +325,13 @@ __device__ __forceinline__ LinSeg lin_seg(int nb, int nseg, int seg) {
 
 // ENDS: the first walk of a portion in segments (no outputs; segment s leaves what it ends with at seg[s + 1], its decay
 // at seg_dec[s + 1]; the first one also copies the state it starts from to seg[0])
-template <bool F32, int KIND, int NT, bool ENDS>
-__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 1 : lin_waves(KIND, NT)))) lin_walk_kernel(LinScanArgs a) {
-  constexpr bool KEY = KIND == LIN_KEY, DELTA = KIND == LIN_DELTA;
-  constexpr int NP = 16 * NT, DEPTH = lin_depth<F32, KIND, NT>(), SO = (F32 ? 256 : 512) * (DELTA ? 2 : 1);
+template <bool F32, bool KEY, int NT, bool ENDS>
+__global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 1 : lin_waves(KEY, NT)))) lin_walk_kernel(LinScanArgs a) {
+  constexpr int NP = 16 * NT, DEPTH = lin_depth<F32, KEY, NT>();
   using T = std::conditional_t<F32, float, bf16_t>;
   using V = std::conditional_t<F32, gf32x4, lu2>;
   const int lane = threadIdx.x & 63, nvt = a.vp >> 4;
-  int w = __builtin_amdgcn_readfirstlane(blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6));
-  if (DELTA && blockDim.x == 64) {  // workgroups of one wave are dealt round-robin: a head's waves go to one XCD
-    const int per = (a.H * nvt + 7) >> 3;
-    w = (w & 7) * per + (w >> 3);
-    if ((int)(blockIdx.x >> 3) >= per) return;
-  }
+  const int w = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
   if (w >= a.H * nvt) return;
   const int h = w / nvt, vt = w - h * nvt, g = KEY ? h : h / (a.H / a.G), ng = KEY ? a.H : a.G;
   const int r16 = lane & 15, q = lane >> 4;
@@ -469,7 +346,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 
   auto seg_at = [&](int j) { return a.seg + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * hs + at; };
   auto dec_at = [&](int j) { return a.seg_dec + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * a.np; };
   const size_t plane = (size_t)2 * a.n_chunks * a.H * NP * 16;
-  using Ops = LinOps<F32, KIND, NT>;
+  using Ops = LinOps<F32, KEY, NT>;
   auto load = [&](Ops& o, int i) __attribute__((always_inline)) {
     const size_t b = sq.b0 + min(i, sg.i1 - 1);  // (past the end: re-reads)
     const T* qo = (const T*)a.qo + (b * ng + g) * NP * 16 + r16 * 16 + 4 * q;
@@ -482,28 +359,20 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 
       o.q[t] = *(const V*)(qo + 256 * t);
       if constexpr (KEY && !F32) o.ql[t] = *(const V*)(qo + plane + 256 * t);
     }
-    const T* so = (const T*)a.so + (b * a.H + h) * SO + r16 * 16 + 4 * q;
+    const T* so = (const T*)a.so + (b * a.H + h) * (F32 ? 256 : 512) + r16 * 16 + 4 * q;
     if constexpr (!ENDS) {
       o.s = *(const V*)so;
       if constexpr (!F32) o.sl = *(const V*)(so + 256);
-    }
-    if constexpr (DELTA) {
-      const T* kr = (const T*)a.kr + (b * ng + g) * NP * 16 + r16 * 16 + 4 * q;
-#pragma unroll
-      for (int t = 0; t < NT; ++t) o.kr[t] = *(const V*)(kr + 256 * t);
-      o.i = *(const V*)(so + SO / 2);
-      if constexpr (!F32) o.il = *(const V*)(so + SO / 2 + 256);
     }
     o.v = *(const V*)((const T*)a.vo + ((b * a.H + h) * a.vp + col) * 16 + 4 * q);
     if constexpr (KEY) {
 #pragma unroll
       for (int t = 0; t < NT; ++t) o.d[t] = *(const gf32x4*)(a.dec + (b * a.H + h) * NP + 16 * t + 4 * q);
     } else {
-      const float* d = a.dec + (b * a.H + h) * lin_decs(KIND);
+      const float* d = a.dec + (b * a.H + h) * 48;
       if constexpr (!ENDS) o.d[0] = *(const gf32x4*)(d + 4 * q);
       o.d[1] = *(const gf32x4*)(d + 16 + 4 * q);
-      if constexpr (DELTA) o.d[2] = *(const gf32x4*)(d + 32 + 4 * q);
-      o.tot = d[DELTA ? 48 : 32];
+      o.tot = d[32];
     }
   };
   Ops o[DEPTH];
@@ -549,7 +418,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 
 #pragma unroll
     for (int t = 0; t < (KEY ? NT : 1); ++t) D[t] = gf32x4{1.f, 1.f, 1.f, 1.f};
   }
-  const float skip = KIND != LIN_HEAD || ENDS ? 0.f : a.D[h];
+  const float skip = KEY || ENDS ? 0.f : a.D[h];
   auto step = [&](const Ops& o, int i) __attribute__((always_inline)) {
     gf32x4 y0 = {0.f, 0.f, 0.f, 0.f}, y1 = y0;
     gf32x4 vf;  // v in fp32: tokens 4 q + r, column r16
@@ -557,40 +426,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 
     else
       vf = gf32x4{__uint_as_float(o.v.x << 16), __uint_as_float(o.v.x & 0xffff0000u), __uint_as_float(o.v.y << 16),
                   __uint_as_float(o.v.y & 0xffff0000u)};
-    if constexpr (DELTA) {  // vf becomes u; y0 the state's part and the block's own
-      gf32x4 x0 = y0, x1 = y0;
-#pragma unroll
-      for (int t = 0; t < NT; t += 2) {
-        if constexpr (F32) {
-          x0 = mfma4(o.kr[t], S[t], x0);
-          x1 = mfma4(o.kr[t + 1], S[t + 1], x1);
-          y0 = mfma4(o.q[t], S[t], y0);
-          y1 = mfma4(o.q[t + 1], S[t + 1], y1);
-        } else {
-          lu2 h0, l0, h1, l1;
-          split4(S[t], h0, l0);
-          split4(S[t + 1], h1, l1);
-          x0 = mfma32(o.kr[t], o.kr[t + 1], h0, h1, x0);
-          x1 = mfma32(o.kr[t], o.kr[t + 1], l0, l1, x1);
-          y0 = mfma32(o.q[t], o.q[t + 1], h0, h1, y0);
-          y1 = mfma32(o.q[t], o.q[t + 1], l0, l1, y1);
-        }
-      }
-      y0 = (y0 + y1) * o.d[0];
-      vf -= o.d[2] * (x0 + x1);
-      if constexpr (F32) {
-        vf = mfma4(o.i, vf, gf32x4{0.f, 0.f, 0.f, 0.f});
-        y0 = mfma4(o.s, vf, y0);
-      } else {
-        lu2 h, l;
-        split4(vf, h, l);
-        vf = mfma32(o.i, o.il, l, l, gf32x4{0.f, 0.f, 0.f, 0.f});
-        vf = mfma32(o.i, o.il, h, h, vf);
-        split4(vf, h, l);
-        y0 = mfma32(o.s, o.sl, l, l, y0);
-        y0 = mfma32(o.s, o.sl, h, h, y0);
-      }
-    } else if constexpr (ENDS) {
+    if constexpr (ENDS) {
     } else if constexpr (F32) {
 #pragma unroll
       for (int t = 0; t < NT; t += 2) {
@@ -614,7 +450,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 
       if constexpr (!KEY) y0 *= o.d[0];
       y0 = mfma32(o.s, o.sl, o.v, o.v, y0);
     }
-    if constexpr (KIND == LIN_HEAD && !ENDS) y0 += skip * vf;
+    if constexpr (!KEY && !ENDS) y0 += skip * vf;
     // the state at the block's end
     if constexpr (KEY) {
 #pragma unroll
@@ -669,162 +505,6 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(F32 ? 
 }
 
 // ---- single tokens ----------------------------------------------------------------------------------
-// sum over the workgroup (red: 4 floats)
-__device__ __forceinline__ float lin_block_sum(float v, float* red) {
-#pragma unroll
-  for (int d = 32; d; d >>= 1) v += __shfl_xor(v, d, 64);
-  __syncthreads();
-  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-  __syncthreads();
-  float t = 0.f;
-  for (int i = 0; i < ((int)blockDim.x >> 6); ++i) t += red[i];
-  return t;
-}
-
-// the convolution of a token's columns for head h: put(i, value) for v's [0, vp), k's [vp, vp + np) and q's [vp + np, vp + 2 np)
-template <bool F32, class Put>
-__device__ __forceinline__ void lin_step_conv(const LinScanArgs& a, const float* in, int h, int pos, int slot, Put put) {
-  const int C = a.H * a.dv + 2 * a.G * a.N, rep = a.H / a.G, g = h / rep, p0 = pos % a.taps;
-  for (int i = threadIdx.x; i < a.vp + 2 * a.np; i += 256) {
-    int raw = -1;
-    if (i < a.vp) {
-      if (i < a.dv) raw = h * a.dv + i;
-    } else {
-      const int sec = i >= a.vp + a.np, n = i - a.vp - sec * a.np;
-      if (n < a.N) raw = a.H * a.dv + (sec * a.G + g) * a.N + n;
-    }
-    float u = 0.f;
-    if (raw >= 0) {
-      const float x = in[a.x_off + raw];
-      u = fmaf(a.conv_w[(size_t)raw * a.taps + a.taps - 1], x, a.conv_b ? a.conv_b[raw] : 0.f);
-      float* ring = a.ring + (size_t)slot * a.taps * C + raw;
-#pragma unroll 4
-      for (int d = 1; d < a.taps; ++d) {
-        const int e = p0 - d + (p0 < d ? a.taps : 0);
-        const float xd = ring[(size_t)e * C];
-        u = fmaf(a.conv_w[(size_t)raw * a.taps + a.taps - 1 - d], d <= pos ? xd : 0.f, u);
-      }
-      u = ls_silu<F32>(u);
-      // (k and q are the group's: its first head keeps them; nobody reads this position's entry in this launch)
-      if (i < a.vp || h % rep == 0) ring[(size_t)p0 * C] = x;
-    }
-    put(i, u);
-  }
-}
-__device__ __forceinline__ float lin_step_dt(const LinScanArgs& a, const float* in, int h) {
-  return ls_softplus(in[a.dt_off + h] + a.dt_b[h]);
-}
-
-// root mean square of a head's dv numbers in y (LDS), weight, output gate -> out
-template <bool F32>
-__device__ __forceinline__ void lin_step_norm(const LinScanArgs& a, const float* in, int h, int row, const float* y, float ss, float* red) {
-  const float inv = a.out_scale / sqrtf(lin_block_sum(ss, red) / (float)a.dv + a.eps);
-  for (int j = threadIdx.x; j < a.dv; j += 256)
-    put1<F32>(a.out, (size_t)row * a.ldo + h * a.dv + j, y[j] * inv * a.norm_w[j] * ls_silu<F32>(in[a.z_off + h * a.dv + j]));
-}
-
-// LIN_DELTA.  With x = S^T k and w = S^T q of the state as it was: u = b (v - d x), o = d w + (k . q) u.  ROWS: rows of the
-// state a thread asks for at once; a state of more (REREAD) is read a second time
-template <bool F32, int ROWS, bool REREAD>
-__global__ void __launch_bounds__(256) lin_delta_step_kernel(LinScanArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float ls_smem[];
-  __shared__ float red[4], dots[4][3];
-  const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
-  const int pos = a.pos[row], slot = a.slot[row];
-  const float* in = a.in + (size_t)row * a.ld;
-  const int c4 = a.vp >> 2, nr = 256 / c4, col = 4 * (tid % c4), r0 = tid / c4;
-  const bool mine = r0 < nr;
-  float *sv = ls_smem, *sk = sv + a.vp, *sq = sk + a.np, *sx = sq + a.np, *sw = sx + nr * a.vp, *so = sw + nr * a.vp;
-  const size_t hs = (size_t)a.np * a.vp, half = (size_t)a.slots * a.H * hs;
-  float* st = a.state + ((size_t)slot * a.H + h) * hs;
-  const float* src = st + ((pos - 1) & 1) * half;
-  float* dst = st + (pos & 1) * half;
-  float4 s[ROWS];
-  auto fetch = [&](int n0) __attribute__((always_inline)) {
-#pragma unroll
-    for (int u = 0; u < ROWS; ++u) {
-      const int n = n0 + u * nr;
-      s[u] = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (pos > 0 && mine && n < a.np) s[u] = *(const float4*)(src + (size_t)n * a.vp + col);
-    }
-  };
-  fetch(r0);  // (on its way while the operands are formed)
-  const float dec = expf(-expf(a.a_log[h]) * lin_step_dt(a, in, h)), beta = 1.f / (1.f + expf(-in[a.b_off + h]));
-  lin_step_conv<F32>(a, in, h, pos, slot, [&](int i, float u) { ls_smem[i] = u; });
-  __syncthreads();
-  float kk = 0.f, qq = 0.f, kq = 0.f;
-  for (int n = tid; n < a.np; n += 256) {
-    kk = fmaf(sk[n], sk[n], kk);
-    qq = fmaf(sq[n], sq[n], qq);
-    kq = fmaf(sk[n], sq[n], kq);
-  }
-#pragma unroll
-  for (int d = 32; d; d >>= 1) {
-    kk += __shfl_xor(kk, d, 64);
-    qq += __shfl_xor(qq, d, 64);
-    kq += __shfl_xor(kq, d, 64);
-  }
-  if ((tid & 63) == 0) {
-    dots[tid >> 6][0] = kk;
-    dots[tid >> 6][1] = qq;
-    dots[tid >> 6][2] = kq;
-  }
-  float4 x = make_float4(0.f, 0.f, 0.f, 0.f), w = x;
-  if (mine) {
-    for (int n0 = r0; n0 < a.np; n0 += ROWS * nr) {
-      if (REREAD && n0 != r0) fetch(n0);
-#pragma unroll
-      for (int u = 0; u < ROWS; ++u) {
-        const int n = min(n0 + u * nr, a.np - 1);  // (past the end: the rows are zeros)
-        const float k = sk[n], q = sq[n];
-        x.x = fmaf(k, s[u].x, x.x); x.y = fmaf(k, s[u].y, x.y); x.z = fmaf(k, s[u].z, x.z); x.w = fmaf(k, s[u].w, x.w);
-        w.x = fmaf(q, s[u].x, w.x); w.y = fmaf(q, s[u].y, w.y); w.z = fmaf(q, s[u].z, w.z); w.w = fmaf(q, s[u].w, w.w);
-      }
-    }
-    *(float4*)(sx + r0 * a.vp + col) = x;
-    *(float4*)(sw + r0 * a.vp + col) = w;
-  }
-  __syncthreads();
-  kk = (dots[0][0] + dots[1][0]) + (dots[2][0] + dots[3][0]);
-  qq = (dots[0][1] + dots[1][1]) + (dots[2][1] + dots[3][1]);
-  kq = (dots[0][2] + dots[1][2]) + (dots[2][2] + dots[3][2]);
-  const float ik = 1.f / sqrtf(kk + LIN_UNIT_EPS), iq = a.q_scale / sqrtf(qq + LIN_UNIT_EPS);
-  if (mine) {
-    x = make_float4(0.f, 0.f, 0.f, 0.f);
-    for (int r = 0; r < nr; ++r) {
-      const float4 p = *(const float4*)(sx + r * a.vp + col);
-      x.x += p.x; x.y += p.y; x.z += p.z; x.w += p.w;
-    }
-    const float4 v = *(const float4*)(sv + col);
-    const float f = -dec * ik, g = beta * ik;  // (the state takes k times ik)
-    x.x = g * fmaf(f, x.x, v.x); x.y = g * fmaf(f, x.y, v.y); x.z = g * fmaf(f, x.z, v.z); x.w = g * fmaf(f, x.w, v.w);
-    for (int n0 = r0; n0 < a.np; n0 += ROWS * nr) {
-      if (REREAD) fetch(n0);
-#pragma unroll
-      for (int u = 0; u < ROWS; ++u) {
-        const int n = n0 + u * nr;
-        if (n >= a.np) break;
-        const float k = sk[n];
-        *(float4*)(dst + (size_t)n * a.vp + col) =
-            make_float4(fmaf(k, x.x, dec * s[u].x), fmaf(k, x.y, dec * s[u].y), fmaf(k, x.z, dec * s[u].z), fmaf(k, x.w, dec * s[u].w));
-      }
-    }
-    if (r0 == 0) {
-      w = make_float4(0.f, 0.f, 0.f, 0.f);
-      for (int r = 0; r < nr; ++r) {
-        const float4 p = *(const float4*)(sw + r * a.vp + col);
-        w.x += p.x; w.y += p.y; w.z += p.z; w.w += p.w;
-      }
-      const float c = iq * kq, d = iq * dec;
-      *(float4*)(so + col) = make_float4(fmaf(c, x.x, d * w.x), fmaf(c, x.y, d * w.y), fmaf(c, x.z, d * w.z), fmaf(c, x.w, d * w.w));
-    }
-  }
-  __syncthreads();
-  float ss = 0.f;
-  for (int j = tid; j < a.dv; j += 256) ss = fmaf(so[j], so[j], ss);
-  lin_step_norm<F32>(a, in, h, row, so, ss, red);
-}
-
 template <bool F32, bool KEY>
 __global__ void __launch_bounds__(256) lin_step_kernel(LinScanArgs a) {
   extern __shared__ __attribute__((aligned(16))) float ls_smem[];
@@ -999,20 +679,10 @@ static void lin_norm(const LinScanArgs& a, hipStream_t st) {
   else lin_norm_v<F32, KEY, 1>(a, st);
 }
 
-template <bool F32>
-static void lin_delta_step(const LinScanArgs& a, hipStream_t st) {
-  const int nr = 256 / (a.vp / 4), rows = (a.np + nr - 1) / nr;
-  const size_t lds = (size_t)(2 * a.vp + 2 * a.np + 2 * nr * a.vp) * 4;
-  const dim3 grid(a.H, a.n);
-  if (rows <= 4) hipLaunchKernelGGL((lin_delta_step_kernel<F32, 4, false>), grid, dim3(256), lds, st, a);
-  else if (rows <= 16) hipLaunchKernelGGL((lin_delta_step_kernel<F32, 16, false>), grid, dim3(256), lds, st, a);
-  else hipLaunchKernelGGL((lin_delta_step_kernel<F32, 16, true>), grid, dim3(256), lds, st, a);
-}
-
 template <bool F32, int KIND>
 static void lin_go(const LinScanArgs& a, hipStream_t st) {
   constexpr bool KEY = KIND == LIN_KEY, DELTA = KIND == LIN_DELTA;
-  if (!a.seqs && DELTA) return lin_delta_step<F32>(a, st);
+  if (!a.seqs && DELTA) return launch_delta_step(a, st);
   if (!a.seqs) {
     const size_t lds = (size_t)(a.vp + 3 * a.np + 256 / (a.vp / 4) * a.vp) * 4;
     hipLaunchKernelGGL((lin_step_kernel<F32, KEY>), dim3(a.H, a.n), dim3(256), lds, st, a);
@@ -1027,22 +697,21 @@ static void lin_go(const LinScanArgs& a, hipStream_t st) {
       if (lds > 150 * 1024) throw std::runtime_error("linear scan: decay projection too wide");
       hipLaunchKernelGGL((lin_key_prep_kernel<F32, NT>), dim3(a.H, nblk), dim3(256), lds, st, a);
     }
-    const int waves = a.H * (a.vp / 16), wg = (waves + 3) / 4;
-    if constexpr (DELTA) {  // (few waves: one a workgroup, over as many compute units)
-      if (waves * a.n_seqs <= 1024) hipLaunchKernelGGL((lin_walk_kernel<F32, KIND, NT, false>), dim3((waves + 7) / 8 * 8, a.n_seqs), dim3(64), 0, st, a);
-      else hipLaunchKernelGGL((lin_walk_kernel<F32, KIND, NT, false>), dim3(wg, a.n_seqs), dim3(256), 0, st, a);
-      return;
-    }
-    if constexpr (!DELTA)
-      if (a.nseg > 1) hipLaunchKernelGGL((lin_walk_kernel<F32, KIND, NT, true>), dim3(wg, a.n_seqs, a.nseg - 1), dim3(256), 0, st, a);
-    hipLaunchKernelGGL((lin_walk_kernel<F32, KIND, NT, false>), dim3(wg, a.n_seqs, a.nseg), dim3(256), 0, st, a);
+    const int wg = (a.H * (a.vp / 16) + 3) / 4;
+    if (a.nseg > 1)
+      hipLaunchKernelGGL((lin_walk_kernel<F32, KEY, NT, true>), dim3(wg, a.n_seqs, a.nseg - 1), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((lin_walk_kernel<F32, KEY, NT, false>), dim3(wg, a.n_seqs, a.nseg), dim3(256), 0, st, a);
   };
   if constexpr (!KEY) {
-    const dim3 grid((a.H * a.vp + 2 * a.G * a.np + LC_T - 1) / LC_T, nblk);
-    if (a.taps <= 4) hipLaunchKernelGGL((lin_conv_kernel<F32, 4>), grid, dim3(LC_T), 0, st, a);
-    else hipLaunchKernelGGL((lin_conv_kernel<F32, 16>), grid, dim3(LC_T), 0, st, a);
+    const dim3 grid((a.H * a.vp + 2 * a.G * a.np + LC_T - 1) / LC_T, DELTA ? a.n_chunks : nblk);
+    if (a.taps <= 4) hipLaunchKernelGGL((lin_conv_kernel<F32, 4, DELTA>), grid, dim3(LC_T), 0, st, a);
+    else hipLaunchKernelGGL((lin_conv_kernel<F32, 16, DELTA>), grid, dim3(LC_T), 0, st, a);
+    if constexpr (DELTA) {
+      launch_delta_walk(a, st);
+      return lin_norm<F32, true>(a, st);
+    }
     const int nscore = (nblk * a.H + 3) / 4, nkeep = (a.H * a.dv + 2 * a.G * a.N + 255) / 256;
-    hipLaunchKernelGGL((lin_score_kernel<F32, DELTA>), dim3(nscore + nkeep * a.n_seqs), dim3(256), 0, st, a, nscore, nkeep);
+    hipLaunchKernelGGL((lin_score_kernel<F32>), dim3(nscore + nkeep * a.n_seqs), dim3(256), 0, st, a, nscore, nkeep);
   }
   switch (a.np / 16) {
     case 2: walk(std::integral_constant<int, 2>{}); break;
@@ -1052,13 +721,13 @@ static void lin_go(const LinScanArgs& a, hipStream_t st) {
     case 12: walk(std::integral_constant<int, 12>{}); break;
     default: walk(std::integral_constant<int, 16>{}); break;
   }
-  lin_norm<F32, KEY || DELTA>(a, st);
+  lin_norm<F32, KEY>(a, st);
 }
 
 // segments a portion of at most `blocks` blocks is walked in: as many waves as the chip holds
 int lin_segments(int kind, int H, int np, int vp, int n_seqs, int blocks) {
-  if (kind == LIN_DELTA) return 1;
-  const int waves = std::max(1, H * (vp / 16) * n_seqs), want = 1024 * lin_waves(kind, np / 16);
+  if (kind == LIN_DELTA) return delta_segments(H, np, vp, n_seqs, blocks);
+  const int waves = std::max(1, H * (vp / 16) * n_seqs), want = 1024 * lin_waves(kind == LIN_KEY, np / 16);
   return std::max(1, std::min({(want + waves / 2) / waves, LIN_SEGS / std::max(1, n_seqs), blocks / LIN_SEG_MIN, 8}));
 }
 
@@ -1073,7 +742,6 @@ void launch_lin_scan(const LinScanArgs& a, hipStream_t st) {
   if ((a.seqs ? a.n_seqs : a.n) < 1) return;
   if (a.seqs && (a.nseg < 1 || (a.nseg > 1 && (!a.seg || !a.seg_dec || a.nseg * a.n_seqs > LIN_SEGS))))
     throw std::runtime_error("linear scan: bad segments");
-  if (a.kind == LIN_DELTA && a.seqs && a.nseg != 1) throw std::runtime_error("linear scan: the delta rule is walked in one segment");
   switch (a.kind) {
     case LIN_KEY: return a.f32 ? lin_go<true, LIN_KEY>(a, st) : lin_go<false, LIN_KEY>(a, st);
     case LIN_DELTA: return a.f32 ? lin_go<true, LIN_DELTA>(a, st) : lin_go<false, LIN_DELTA>(a, st);

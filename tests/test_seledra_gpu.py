@@ -67,10 +67,10 @@ DELTA = [(6, 2, 20, 24, 3), (6, 6, 40, 32, 4), (3, 1, 128, 64, 2), (2, 1, 200, 1
 
 
 @pytest.mark.parametrize("f32", [0, 1])
-@pytest.mark.parametrize("shift", [5, 4])
+@pytest.mark.parametrize("nseg, shift", [(1, 5), (4, 4)])
 @pytest.mark.parametrize("sizes", DELTA)
-def test_delta_rule_kernels(sizes, shift, f32):
-    """Columns at any offset and at aligned ones; portions of unequal lengths at block and chunk borders, continued by others;
+def test_delta_rule_kernels(sizes, nseg, shift, f32):
+    """Columns at any offset and at aligned ones; portions in segments; portions of unequal lengths at block and chunk borders, continued by others;
     single tokens, some of them twice; slots taken over by a new sequence; state and convolution inputs that no earlier
     sequence may leak; strong and weak decays, and a run of equal keys written at nearly full strength."""
     m = E()
@@ -106,7 +106,7 @@ def test_delta_rule_kernels(sizes, shift, f32):
             x[20:70, C + inner:C + inner + H] += 5
         return bf(x)
 
-    X = {s: inputs(n, s == 1) for s, n in {0: 230, 2: 140, 5: 90, 3: 100, 4: 400, 1: 200}.items()}
+    X = {s: inputs(n, s == 1) for s, n in {0: 230, 2: 140, 5: 90, 3: 100, 4: 700, 1: 500}.items()}
     # 16-bit portions round the convolution's outputs: where an output nearly cancels, that is what is left of it
     soft = lambda x: (ref(x, True) - ref(x)).abs().amax(1, keepdim=True) * (0 if f32 else 2)
     want = {s: (ref(x), soft(x)) for s, x in X.items()}
@@ -119,7 +119,7 @@ def test_delta_rule_kernels(sizes, shift, f32):
            for k, n in zip(("qo", "ko", "kr", "vo", "so", "dec"), m.lin_ws(m.LIN_DELTA, H, G, np_, vp, bool(f32)))}
     work, ld = torch.zeros(64 * 16, dtype=torch.int32, device="cuda"), pad(shift + width + 3, 4) + shift % 4
 
-    def go(entries, decode=False, nseg=1):
+    def go(entries, decode=False):
         rows = torch.cat([X[s][st:st + n] for s, st, n in entries])
         n = rows.shape[0]
         inp = torch.full((n, ld), 1e30)
@@ -130,10 +130,10 @@ def test_delta_rule_kernels(sizes, shift, f32):
             pieces.append([at, k, s, st])
             at += k
         pd, sd = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in zip(*[(p[3], p[2]) for p in pieces]))
-        print(sizes, shift, f32, entries, flush=True)
+        print(sizes, nseg, shift, f32, entries, flush=True)
         m.lin_scan([] if decode else pieces, kind=m.LIN_DELTA, H=H, G=G, N=N, dv=dv, vp=vp, inp=inp.data_ptr(), ld=ld, **off,
                    **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr(), state=state.data_ptr(), slots=slots, nseg=nseg,
-                   seg=seg.data_ptr(), seg_mat=mat.data_ptr(), pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
+                   seg=seg.data_ptr(), seg_dec=mat.data_ptr(), pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
                    **{k: v.data_ptr() for k, v in buf.items()}, y=y.data_ptr(), eps=eps, out_scale=osc, out=out.data_ptr(),
                    ldo=inner + 64, f32=f32, work=work.data_ptr(), stream=stream())
         torch.cuda.synchronize()
@@ -150,11 +150,12 @@ def test_delta_rule_kernels(sizes, shift, f32):
     go([(5, 4, 1), (2, 82, 1)], True)
     go([(5, 4, 1), (2, 82, 1)])                                     # again, as portions of one token
     go([(2, 83, 48), (0, 102, 128), (3, 32, 66), (5, 5, 3)])        # even lengths: in and out at one parity
-    go([(1, 0, 30)])
-    go([(1, 30, 90)])
+    go([(4, 0, 390), (1, 0, 130)])                                  # several segments, the last one short
+    go([(1, 130, 370), (4, 390, 1), (5, 8, 2)])                     # ... from a state, in place (even length)
+    go([(4, 391, 309), (5, 10, 6)])
     X[0] = inputs(70)
     want[0] = ref(X[0]), soft(X[0])
-    go([(0, 0, 2), (5, 8, 74)])
+    go([(0, 0, 2), (5, 16, 74)])
     go([(0, 2, 1)], True)
     go([(0, 3, 49)])
     X[3] = inputs(9)
