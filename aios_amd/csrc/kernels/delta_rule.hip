@@ -11,9 +11,7 @@
 //   walk    a wave owns a head and 16 columns of v, its part of S in accumulators from pair to pair:
 //             u = T (v - D K S - ..),  o = D Q S + scores u,  S = (decay of the pair) S + K^T (decay to its end) u.
 //           A 16 x 16 accumulator tile is, lane for lane, the second operand of the 16-deep product, so neither S nor u
-//           leaves registers.  Where heads and columns leave compute units idle, a portion is walked in segments side by side: a
-//           segment's transition S -> M S + E is the walk of the unit matrix without values and the walk from zero, so a first
-//           walk finds M and E of all segments but the last, the second one starts each from what those before it make together.
+//           leaves registers; other waves bring the operands through LDS, pairs ahead.
 // Single tokens: delta_step, one workgroup per head and row, the norm included.
 //
 // fp32: state, decays, strengths, lengths, the system and its inverse, scores, norms, gates.  The products take bf16 operands:
@@ -22,6 +20,7 @@
 #include <algorithm>
 #include <stdexcept>
 
+#include "lds_dma.h"
 #include "lin_common.h"
 
 namespace aios {
@@ -233,153 +232,180 @@ __global__ void __launch_bounds__(256) delta_score_kernel(LinScanArgs a, int nsc
 }
 
 // ---- the walk ---------------------------------------------------------------------------------------
-// the pairs of a portion that a segment walks: [i0, i1), and how many segments there are
-constexpr int DELTA_SEG_MIN = 4;
-struct DeltaSeg {
-  int i0, i1, n;
+// A workgroup's DELTA_W walkers take neighbouring columns of one head.  Its loaders bring what they read of a pair to LDS: 1 KB
+// pieces, 16 bytes a lane in the order the products take them, pairs ahead.
+constexpr int DELTA_W = 2, DELTA_L = 2;
+
+template <bool F32, int NT>
+struct DeltaStage {
+  static constexpr int P = F32 ? 2 : 1;                                     // pieces of an Oct tile
+  static constexpr int KR = 0, Q = KR + NT * P, K = Q + NT * P, M = K + NT * P, D = M + DM_N, V = D + 1;  // first pieces
+  static constexpr int ALL = V + DELTA_W * P, EACH = (ALL + DELTA_L - 1) / DELTA_L;  // EACH: a loader requests
+  static constexpr int BYTES = ALL * 1024;
+  static constexpr int N = BYTES * 4 <= 150 * 1024 ? 4 : BYTES * 3 <= 150 * 1024 ? 3 : BYTES * 2 <= 150 * 1024 ? 2 : 1;
+  static_assert(BYTES * N <= 150 * 1024, "LDS");
 };
-__device__ __forceinline__ DeltaSeg delta_seg(int pairs, int nseg, int seg) {
-  const int per = max(DELTA_SEG_MIN, (pairs + nseg - 1) / nseg);
-  return DeltaSeg{seg * per, min(pairs, (seg + 1) * per), (pairs + per - 1) / per};
+
+// loader l's part of pair p -> the stage at LDS address `to`
+template <bool F32, int NT>
+__device__ __forceinline__ void delta_request(const LinScanArgs& a, size_t p, int h, int vt0, int l, int lane, uint32_t to) {
+  using L = DeltaStage<F32, NT>;
+  constexpr int ES = F32 ? 4 : 2, ROWS = NT * 256 * ES, TILE = 512 * ES, R = NT / 2 * L::P;  // bytes of a block's rows, of an Oct tile
+  const int nvt = a.vp >> 4, g = h / (a.H / a.G), r16 = lane & 15, q = lane >> 4;
+  // a lane's 16 bytes of a piece: of an Oct tile or matrix (32 numbers a row), of an fp32 matrix
+  const int by_oct = (r16 * 32 + 8 * q) * ES, by_mat = F32 ? (r16 * 16 + 4 * q) * 4 : by_oct;
+  const uint8_t *kr = (const uint8_t*)a.kr + (2 * p * a.G + g) * ROWS, *qo = (const uint8_t*)a.qo + (2 * p * a.G + g) * ROWS;
+  const uint8_t* ko = (const uint8_t*)a.ko + (p * a.G + g) * 2 * ROWS;
+  const uint8_t* so = (const uint8_t*)a.so + (p * a.H + h) * DM_N * mat_size(F32) * ES;
+  const uint8_t* vo = (const uint8_t*)a.vo + (p * a.H + h) * a.vp * 32 * ES;
+#pragma unroll
+  for (int j = 0; j < L::EACH; ++j) {
+    const int u = min(l + DELTA_L * j, L::ALL - 1);  // (the last piece twice: the same bytes)
+    const uint8_t* src;
+    if (u < L::K) {
+      const int r = u < L::Q ? u : u - L::Q, b = r >= R, t = r - b * R;
+      src = (u < L::Q ? kr : qo) + (size_t)b * a.G * ROWS + (t / L::P) * TILE + (t % L::P) * 16 + by_oct;
+    } else if (u < L::M) {
+      src = ko + ((u - L::K) / L::P) * TILE + ((u - L::K) % L::P) * 16 + by_oct;
+    } else if (u < L::D) {
+      src = so + (u - L::M) * mat_size(F32) * ES + by_mat;
+    } else if (u < L::V) {
+      src = (const uint8_t*)(a.dec + (p * a.H + h) * DD_N) + (lane & 31) * 16;
+    } else {
+      src = vo + min(vt0 + (u - L::V) / L::P, nvt - 1) * TILE + ((u - L::V) % L::P) * 16 + by_oct;
+    }
+    pf_glds16(src, to + u * 1024);
+  }
 }
 
-// Registers hold one pair's operands; each is requested anew as soon as the walk is through with it, half a step before it is
-// needed again.
-// ENDS: the first walk of a portion in segments, without outputs.  Segment s leaves what it ends with at seg[s + 1]: the first
-// one from the state it starts from (which it copies to seg[0]), the others from zero; waves of 16 more columns each take the
-// columns of the unit matrix, without values, to the segment's transition, at seg_dec[s + 1].
-template <bool F32, int NT, bool ENDS>
-__global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(!F32 && NT <= 8 ? 2 : 1))) delta_walk_kernel(LinScanArgs a) {
-  constexpr int NP = 16 * NT, MAT = mat_size(F32);
-  const int lane = threadIdx.x, nvt = a.vp >> 4, per_head = nvt + (ENDS ? NT : 0), waves = a.H * per_head;
+template <bool F32, int NT>
+__global__ void __launch_bounds__(64 * (DELTA_W + DELTA_L)) __attribute__((amdgpu_waves_per_eu(2))) delta_walk_kernel(LinScanArgs a) {
+  using L = DeltaStage<F32, NT>;
+  // What a step reads is in registers before it begins where they and LDS have room (AHEAD): its rows since the step before was
+  // half done, the rest since that one's end.
+  constexpr bool AHEAD = L::N >= 3;
+  extern __shared__ __attribute__((aligned(16))) uint8_t dw_smem[];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int nvt = a.vp >> 4, per_head = (nvt + DELTA_W - 1) / DELTA_W, groups = a.H * per_head;
   // (workgroups are dealt round-robin: a head's go to one XCD)
-  const int per_xcd = gridDim.x >> 3, w = (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3);
-  if (w >= waves) return;
-  const int h = w / per_head, wt = w - h * per_head, g = h / (a.H / a.G), seg = blockIdx.z;
-  const bool unit = wt >= nvt;
-  const int r16 = lane & 15, q = lane >> 4;
+  const int w = (blockIdx.x & 7) * (gridDim.x >> 3) + (blockIdx.x >> 3);
+  if (w >= groups) return;
+  const int h = w / per_head, vt0 = (w - h * per_head) * DELTA_W;
   const ScanSeq sq = a.seqs[blockIdx.y];
-  const DeltaSeg sg = delta_seg((sq.n + 2 * LIN_T - 1) / (2 * LIN_T), a.nseg, seg);
-  if (seg + (ENDS ? 1 : 0) >= sg.n || (ENDS && unit && seg == 0)) return;
-  const int p0 = sq.b0 / 2, col = 16 * (unit ? wt - nvt : wt) + r16;
+  const int np = (sq.n + 2 * LIN_T - 1) / (2 * LIN_T), p0 = sq.b0 / 2;
+  // Step i: the pieces it reads from LDS (its own, AHEAD the next one's) are there when all but the younger requests are; then one
+  // barrier, after which nobody reads the stage any more that is filled next.
+  if (wave >= DELTA_W) {
+    const uint32_t lds0 = pf_lds_addr(dw_smem);
+    auto request = [&](int i) __attribute__((always_inline)) {  // (past the end: the last one again)
+      delta_request<F32, NT>(a, (size_t)(p0 + min(i, np - 1)), h, vt0, wave - DELTA_W, lane, lds0 + (uint32_t)(i % L::N) * L::BYTES);
+    };
+#pragma unroll
+    for (int i = 0; i < (L::N > 1 ? L::N - 1 : 1); ++i) request(i);
+    if constexpr (AHEAD) {
+      pf_vmcnt<(L::N - 2) * L::EACH>();
+      pf_barrier();
+    }
+    for (int i = 0; i < np; ++i) {
+      pf_vmcnt<(AHEAD ? (L::N - 3) * L::EACH : 0)>();
+      pf_barrier();
+      if constexpr (L::N == 1) pf_barrier();
+      request(i + (L::N > 1 ? L::N - 1 : 1));
+    }
+    pf_vmcnt<0>();  // (nothing may arrive in LDS that is another workgroup's by then)
+    return;
+  }
+  const int r16 = lane & 15, q = lane >> 4;
+  const bool mine = vt0 + wave < nvt;  // (a walker past the last column goes along)
+  const int col = 16 * min(vt0 + wave, nvt - 1) + r16;
   const size_t hs = (size_t)a.np * a.vp, half = (size_t)a.slots * a.H * hs;
-  const size_t lane_at = (size_t)(4 * q) * a.vp + col;  // of this lane in a head's state
-  float* st = a.state + ((size_t)sq.slot * a.H + h) * hs + lane_at;
-  // segment j of this portion and head
-  auto seg_at = [&](int j) { return a.seg + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * hs + lane_at; };
-  auto mat_of = [&](int j) { return a.seg_dec + (((size_t)blockIdx.y * a.nseg + j) * a.H + h) * NP * NP; };
-  constexpr bool HOLD = !F32 || NT <= 8;  // (what registers have room for; else operands are read where they are used)
-  Oct<F32> kr[2][HOLD ? NT / 2 : 1], x[2][HOLD ? NT / 2 : 1], k[HOLD ? NT : 1], vo;
+  float* st = a.state + ((size_t)sq.slot * a.H + h) * hs + (size_t)(4 * q) * a.vp + col;
+  // S[t]: rows 16 t + 4 q + r, column r16 of this wave's 16
+  constexpr gf32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  gf32x4 S[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    S[t] = zero;
+    if (sq.pos0 > 0) {
+      const float* src = st + ((sq.pos0 - 1) & 1) * half + (size_t)(16 * t) * a.vp;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[t][r] = src[(size_t)r * a.vp];
+    }
+  }
+  Oct<F32> kr[2][AHEAD ? NT / 2 : 1], x[2][AHEAD ? NT / 2 : 1], k[AHEAD ? NT : 1], vo;
   Mat<F32> m[DM_N];
   gf32x4 d[2][3];
   float tot;
-  auto pair_of = [&](int i) { return (size_t)(p0 + min(i, sg.i1 - 1)); };  // (past the end: re-reads)
-  auto row_at = [&](size_t p, int b, int t) { return ((2 * p + b) * a.G + g) * NP * 16 + r16 * 32 + 8 * q + 256 * t; };
-  auto col_at = [&](size_t p, int t) { return ((p * a.G + g) * NP + 16 * t + r16) * 32 + 8 * q; };
-  auto load_rows = [&](int i) __attribute__((always_inline)) {
-    if constexpr (!HOLD) return;
-    const size_t p = pair_of(i);
-#pragma unroll
-    for (int t = 0; t < NT; t += 2)
-#pragma unroll
-      for (int b = 0; b < 2; ++b) {
-        kr[b][t / 2] = oct<F32>(a.kr, row_at(p, b, t));
-        if constexpr (!ENDS) x[b][t / 2] = oct<F32>(a.qo, row_at(p, b, t));
-      }
+  auto stage = [&](int i) { return dw_smem + (i % L::N) * L::BYTES + lane * 16; };
+  auto piece = [&](const uint8_t* sb, int u) __attribute__((always_inline)) {
+    Oct<F32> o;
+    if constexpr (F32) {
+      o.a = *(const gf32x4*)(sb + u * 1024);
+      o.b = *(const gf32x4*)(sb + (u + 1) * 1024);
+    } else {
+      o.u = *(const gu32x4*)(sb + u * 1024);
+    }
+    return o;
   };
-  auto load_rest = [&](int i) __attribute__((always_inline)) {
-    const size_t p = pair_of(i);
-    if (!ENDS || !unit) vo = oct<F32>(a.vo, ((p * a.H + h) * a.vp + col) * 32 + 8 * q);
-    const float* dec = a.dec + (p * a.H + h) * DD_N;
+  auto row = [&](int first, int b, int t) { return first + (b * NT + t) / 2 * L::P; };
+  auto read_rows = [&](int i) __attribute__((always_inline)) {
+    const uint8_t* sb = stage(i);
+    if constexpr (AHEAD) {
+#pragma unroll
+      for (int t = 0; t < NT; t += 2)
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+          kr[b][t / 2] = piece(sb, row(L::KR, b, t));
+          x[b][t / 2] = piece(sb, row(L::Q, b, t));
+        }
+    }
+  };
+  auto read_rest = [&](int i) __attribute__((always_inline)) {
+    const uint8_t* sb = stage(i);
+    const float* dec = (const float*)(sb - lane * 16 + L::D * 1024);
+    vo = piece(sb, L::V + wave * L::P);
 #pragma unroll
     for (int b = 0; b < 2; ++b)
 #pragma unroll
-      for (int j = ENDS ? 1 : 0; j < 3; ++j) d[b][j] = *(const gf32x4*)(dec + b * DD_BLOCK + 16 * j + 4 * q);
+      for (int j = 0; j < 3; ++j) d[b][j] = *(const gf32x4*)(dec + b * DD_BLOCK + 16 * j + 4 * q);
     tot = dec[DD_TOT];
 #pragma unroll
-    for (int j = DM_N - 1; j >= (ENDS ? DM_T0 : 0); --j) m[j] = mat<F32>(a.so, (p * a.H + h) * DM_N * MAT + j * MAT + mat_at<F32>(r16, 4 * q));
-    if constexpr (HOLD) {
+    for (int j = DM_N - 1; j >= 0; --j) {
+      if constexpr (F32) m[j].f = *(const gf32x4*)(sb + (L::M + j) * 1024);
+      else m[j].u = *(const gu32x4*)(sb + (L::M + j) * 1024);
+    }
+    if constexpr (AHEAD) {
 #pragma unroll
-      for (int t = 0; t < NT; ++t) k[t] = oct<F32>(a.ko, col_at(p, t));
+      for (int t = 0; t < NT; ++t) k[t] = piece(sb, L::K + t * L::P);
     }
   };
-  if constexpr (ENDS) vo = Oct<F32>{};
-  constexpr gf32x4 zero = {0.f, 0.f, 0.f, 0.f};
-  // S[t]: rows 16 t + 4 q + r, column r16 of this wave's 16
-  gf32x4 S[NT];
-#pragma unroll
-  for (int t = 0; t < NT; ++t) S[t] = zero;
-  auto read = [&](gf32x4 (&x)[NT], const float* src) __attribute__((always_inline)) {
-#pragma unroll
-    for (int t = 0; t < NT; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) x[t][r] = src[(size_t)(16 * t + r) * a.vp];
-  };
-  auto write = [&](float* dst) __attribute__((always_inline)) {
-#pragma unroll
-    for (int t = 0; t < NT; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) dst[(size_t)(16 * t + r) * a.vp] = S[t][r];
-  };
-  auto first = [&]() __attribute__((always_inline)) {
-    load_rows(sg.i0);
-    load_rest(sg.i0);
-  };
-  if (ENDS || sg.n == 1) {
-    first();
-    if (seg == 0 && sq.pos0 > 0) read(S, st + ((sq.pos0 - 1) & 1) * half);
-    if constexpr (ENDS) {
-      if (seg == 0) write(seg_at(0));
-      if (unit) {
-#pragma unroll
-        for (int t = 0; t < NT; ++t)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) S[t][r] = 16 * t + 4 * q + r == col ? 1.f : 0.f;
-      }
-    }
-  } else {
-    // (the state itself may already be the new one: the copies are read)
-    read(S, seg_at(min(seg, 1)));
-    for (int j = 2; j <= seg; ++j) {  // the transition of segment j - 1 times what was, and what it added itself
-      Tile<F32> s[NT];
-#pragma unroll
-      for (int t = 0; t < NT; ++t) s[t] = tile<F32>(S[t]);
-      read(S, seg_at(j));
-      const float* mt = mat_of(j) + r16 * NP + 4 * q;
-#pragma unroll
-      for (int t = 0; t < NT; ++t)
-#pragma unroll
-        for (int u = 0; u < NT; u += 2) {
-          const Tile<F32> m0 = tile<F32>(*(const gf32x4*)(mt + 16 * t * NP + 16 * u)), m1 = tile<F32>(*(const gf32x4*)(mt + 16 * t * NP + 16 * u + 16));
-          if constexpr (F32) {
-            S[t] = mfma4(m1.f, s[u + 1].f, mfma4(m0.f, s[u].f, S[t]));
-          } else {
-            S[t] = mul(join(m0.h, m1.h), s[u], s[u + 1], S[t]);
-            S[t] = mul8(join(m0.l, m1.l), join(s[u].h, s[u + 1].h), S[t]);
-          }
-        }
-    }
-    first();
+  if constexpr (AHEAD) {
+    pf_barrier();
+    read_rows(0);
+    read_rest(0);
   }
-  for (int i = sg.i0; i < sg.i1; ++i) {
+  for (int i = 0; i < np; ++i) {
+    __builtin_amdgcn_sched_barrier(0);
+    // (without AHEAD the last step's reads may not have come back yet)
+    if constexpr (!AHEAD) asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    pf_barrier();
+    const uint8_t* sb = stage(i);
+    if constexpr (!AHEAD) read_rest(i);
     gf32x4 c[2] = {zero, zero}, y[2] = {zero, zero};
 #pragma unroll
     for (int t = 0; t < NT; t += 2) {
       const Tile<F32> s0 = tile<F32>(S[t]), s1 = tile<F32>(S[t + 1]);
 #pragma unroll
       for (int b = 0; b < 2; ++b) {
-        if constexpr (HOLD) {
-          c[b] = mul(kr[b][t / 2], s0, s1, c[b]);
-          if constexpr (!ENDS) y[b] = mul(x[b][t / 2], s0, s1, y[b]);
-        } else {
-          c[b] = mul(oct<F32>(a.kr, row_at(p0 + i, b, t)), s0, s1, c[b]);
-          if constexpr (!ENDS) y[b] = mul(oct<F32>(a.qo, row_at(p0 + i, b, t)), s0, s1, y[b]);
-        }
+        c[b] = mul(AHEAD ? kr[b][AHEAD ? t / 2 : 0] : piece(sb, row(L::KR, b, t)), s0, s1, c[b]);
+        y[b] = mul(AHEAD ? x[b][AHEAD ? t / 2 : 0] : piece(sb, row(L::Q, b, t)), s0, s1, y[b]);
       }
     }
-    __builtin_amdgcn_sched_barrier(0);
-    load_rows(i + 1);
-    __builtin_amdgcn_sched_barrier(0);
+    if constexpr (AHEAD) {
+      __builtin_amdgcn_sched_barrier(0);
+      read_rows(i + 1);
+      __builtin_amdgcn_sched_barrier(0);
+    }
     gf32x4 v[2];  // in fp32: tokens 4 q + r, column r16
     if constexpr (F32) {
       v[0] = vo.a;
@@ -393,24 +419,24 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(!F32 &&
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
       v[b] -= d[b][2] * c[b];
-      if constexpr (!ENDS) y[b] *= d[b][0];
+      y[b] *= d[b][0];
     }
     const gf32x4 u0 = mul(m[DM_T0], tile<F32>(v[0]), zero);
     const Tile<F32> t0 = tile<F32>(u0);
     const gf32x4 u1 = mul(m[DM_T1], tile<F32>(mul(m[DM_L10], t0, v[1])), zero);
     const Tile<F32> t1 = tile<F32>(u1), e0 = tile<F32>(u0 * d[0][1]), e1 = tile<F32>(u1 * d[1][1]);
-    if constexpr (!ENDS) {
-      y[0] = mul(m[DM_A0], t0, y[0]);
-      y[1] = mul(m[DM_A10], t0, y[1]);
-      y[1] = mul(m[DM_A1], t1, y[1]);
-    }
     // the state at the pair's end
 #pragma unroll
-    for (int t = 0; t < NT; ++t) S[t] = mul(HOLD ? k[HOLD ? t : 0] : oct<F32>(a.ko, col_at(p0 + i, t)), e0, e1, S[t] * tot);
-    __builtin_amdgcn_sched_barrier(0);
-    load_rest(i + 1);
-    __builtin_amdgcn_sched_barrier(0);
-    if (!ENDS && col < a.dv) {
+    for (int t = 0; t < NT; ++t) S[t] = mul(AHEAD ? k[AHEAD ? t : 0] : piece(sb, L::K + t * L::P), e0, e1, S[t] * tot);
+    y[0] = mul(m[DM_A0], t0, y[0]);
+    y[1] = mul(m[DM_A10], t0, y[1]);
+    y[1] = mul(m[DM_A1], t1, y[1]);
+    if constexpr (AHEAD) {
+      __builtin_amdgcn_sched_barrier(0);
+      read_rest(i + 1);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    if (mine && col < a.dv) {
 #pragma unroll
       for (int b = 0; b < 2; ++b) {
         const int t = 32 * i + 16 * b + 4 * q;
@@ -420,17 +446,17 @@ __global__ void __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(!F32 &&
           if (t + r < sq.n) out[(size_t)r * a.H * a.dv] = y[b][r];
       }
     }
+    if constexpr (L::N == 1) {
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      pf_barrier();
+    }
   }
-  if constexpr (ENDS) {
-    if (!unit) return write(seg_at(seg + 1));
-    float* dst = mat_of(seg + 1) + 4 * q * NP + col;
+  if (!mine) return;
+  float* dst = st + ((sq.pos0 + sq.n - 1) & 1) * half;
 #pragma unroll
-    for (int t = 0; t < NT; ++t)
+  for (int t = 0; t < NT; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) dst[(16 * t + r) * NP] = S[t][r];
-  } else if (seg + 1 == sg.n) {
-    write(st + ((sq.pos0 + sq.n - 1) & 1) * half);
-  }
+    for (int r = 0; r < 4; ++r) dst[(size_t)(16 * t + r) * a.vp] = S[t][r];
 }
 
 template <bool F32>
@@ -439,10 +465,9 @@ static void delta_walk(const LinScanArgs& a, hipStream_t st) {
   hipLaunchKernelGGL((delta_score_kernel<F32>), dim3(nscore + nkeep * a.n_seqs), dim3(256), 0, st, a, nscore, nkeep);
   auto walk = [&](auto nt) {
     constexpr int NT = decltype(nt)::value;
-    const int n = a.H * (a.vp / 16), ne = n + a.H * NT;
-    if (a.nseg > 1)
-      hipLaunchKernelGGL((delta_walk_kernel<F32, NT, true>), dim3((ne + 7) / 8 * 8, a.n_seqs, a.nseg - 1), dim3(64), 0, st, a);
-    hipLaunchKernelGGL((delta_walk_kernel<F32, NT, false>), dim3((n + 7) / 8 * 8, a.n_seqs, a.nseg), dim3(64), 0, st, a);
+    using L = DeltaStage<F32, NT>;
+    const int groups = a.H * ((a.vp / 16 + DELTA_W - 1) / DELTA_W);
+    hipLaunchKernelGGL((delta_walk_kernel<F32, NT>), dim3((groups + 7) / 8 * 8, a.n_seqs), dim3(64 * (DELTA_W + DELTA_L)), L::N * L::BYTES, st, a);
   };
   switch (a.np / 16) {
     case 2: walk(std::integral_constant<int, 2>{}); break;
@@ -452,14 +477,6 @@ static void delta_walk(const LinScanArgs& a, hipStream_t st) {
     case 12: walk(std::integral_constant<int, 12>{}); break;
     default: walk(std::integral_constant<int, 16>{}); break;
   }
-}
-
-// Two walks of 1 / n of the pairs, the first over the transition's columns too, instead of one of them all: from three on, where
-// the chip has room
-int delta_segments(int H, int np, int vp, int n_seqs, int blocks) {
-  const int room = 4096 / std::max(1, H * (np + vp) / 16 * n_seqs);
-  const int n = std::min({room, LIN_SEGS / std::max(1, n_seqs), blocks / (2 * DELTA_SEG_MIN), 8});
-  return n < 3 ? 1 : n;
 }
 
 void launch_delta_walk(const LinScanArgs& a, hipStream_t st) { a.f32 ? delta_walk<true>(a, st) : delta_walk<false>(a, st); }

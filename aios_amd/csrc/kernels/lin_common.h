@@ -140,7 +140,6 @@ __device__ __forceinline__ void lin_step_norm(const LinScanArgs& a, const float*
 
 // delta_rule.hip: LIN_DELTA's part of a portion between the convolution and the norm, and its single tokens
 void launch_delta_walk(const LinScanArgs& a, hipStream_t st);
-int delta_segments(int H, int np, int vp, int n_seqs, int blocks);
 void launch_delta_step(const LinScanArgs& a, hipStream_t st);
 
 }  // namespace aios

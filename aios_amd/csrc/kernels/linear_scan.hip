@@ -726,7 +726,7 @@ static void lin_go(const LinScanArgs& a, hipStream_t st) {
 
 // segments a portion of at most `blocks` blocks is walked in: as many waves as the chip holds
 int lin_segments(int kind, int H, int np, int vp, int n_seqs, int blocks) {
-  if (kind == LIN_DELTA) return delta_segments(H, np, vp, n_seqs, blocks);
+  if (kind == LIN_DELTA) return 1;  // (a segment's transition is a whole matrix)
   const int waves = std::max(1, H * (vp / 16) * n_seqs), want = 1024 * lin_waves(kind == LIN_KEY, np / 16);
   return std::max(1, std::min({(want + waves / 2) / waves, LIN_SEGS / std::max(1, n_seqs), blocks / LIN_SEG_MIN, 8}));
 }
@@ -740,6 +740,7 @@ void launch_lin_scan(const LinScanArgs& a, hipStream_t st) {
   if (a.kind == LIN_HEAD && (a.norm_parts < 1 || (a.H * a.dv) % a.norm_parts || a.H * a.dv / a.norm_parts > 16384))
     throw std::runtime_error("linear scan: bad norm");
   if ((a.seqs ? a.n_seqs : a.n) < 1) return;
+  if (a.kind == LIN_DELTA && a.seqs && a.nseg != 1) throw std::runtime_error("linear scan: the delta rule takes one segment");
   if (a.seqs && (a.nseg < 1 || (a.nseg > 1 && (!a.seg || !a.seg_dec || a.nseg * a.n_seqs > LIN_SEGS))))
     throw std::runtime_error("linear scan: bad segments");
   switch (a.kind) {

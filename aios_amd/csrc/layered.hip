@@ -736,7 +736,7 @@ void LayeredDecoder::finalize() {
                  std::max(lw.vo, l.vo), std::max(lw.so, l.so), std::max(lw.dec, l.dec)};
       lin_y = std::max(lin_y, (size_t)R * D.lH * D.ldv);
       lin_seg = std::max(lin_seg, (size_t)LIN_SEGS * D.lH * D.lnp * D.lvp);
-      lin_seg_dec = std::max(lin_seg_dec, (size_t)LIN_SEGS * D.lH * D.lnp * (D.lin == LIN_DELTA ? D.lnp : 1));
+      lin_seg_dec = std::max(lin_seg_dec, (size_t)LIN_SEGS * D.lH * D.lnp);
     }
     kout = std::max({kout, D.kout, D.glu});
     fp = std::max(fp, seq_ ? D.glu : D.fp);

@@ -197,7 +197,7 @@ struct LinScanArgs {
   void *qo, *ko, *kr, *vo, *so;
   float* dec;
   int nseg;                   // segments a portion is walked in (lin_segments); more than 1: the states and decays at
-  float *seg, *seg_dec;       // their borders, [n_seqs][nseg][H] x [np][vp] and x [np] (LIN_DELTA: [np][np])
+  float *seg, *seg_dec;       // their borders, [n_seqs][nseg][H] x [np][vp] and x [np]
   float* y;                   // [rows][H dv]
   const float* norm_w;
   int norm_parts;

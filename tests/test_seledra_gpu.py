@@ -67,10 +67,10 @@ DELTA = [(6, 2, 20, 24, 3), (6, 6, 40, 32, 4), (3, 1, 128, 64, 2), (2, 1, 200, 1
 
 
 @pytest.mark.parametrize("f32", [0, 1])
-@pytest.mark.parametrize("nseg, shift", [(1, 5), (4, 4)])
+@pytest.mark.parametrize("shift", [5, 4])
 @pytest.mark.parametrize("sizes", DELTA)
-def test_delta_rule_kernels(sizes, nseg, shift, f32):
-    """Columns at any offset and at aligned ones; portions in segments; portions of unequal lengths at block and chunk borders, continued by others;
+def test_delta_rule_kernels(sizes, shift, f32):
+    """Columns at any offset and at aligned ones; portions of unequal lengths at block and chunk borders, continued by others;
     single tokens, some of them twice; slots taken over by a new sequence; state and convolution inputs that no earlier
     sequence may leak; strong and weak decays, and a run of equal keys written at nearly full strength."""
     m = E()
@@ -114,7 +114,6 @@ def test_delta_rule_kernels(sizes, nseg, shift, f32):
     state = torch.full((2, slots, H, np_, vp), 1e30, device="cuda")
     ring = torch.full((slots, taps, C), 1e30, device="cuda")
     nan = float("nan")
-    seg, mat = torch.full((16, H, np_, vp), nan, device="cuda"), torch.full((16, H, np_, np_), nan, device="cuda")
     buf = {k: torch.full((2 * 40 * n + 4096,), nan, dtype=torch.float32 if k == "dec" else dt, device="cuda")
            for k, n in zip(("qo", "ko", "kr", "vo", "so", "dec"), m.lin_ws(m.LIN_DELTA, H, G, np_, vp, bool(f32)))}
     work, ld = torch.zeros(64 * 16, dtype=torch.int32, device="cuda"), pad(shift + width + 3, 4) + shift % 4
@@ -130,10 +129,9 @@ def test_delta_rule_kernels(sizes, nseg, shift, f32):
             pieces.append([at, k, s, st])
             at += k
         pd, sd = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in zip(*[(p[3], p[2]) for p in pieces]))
-        print(sizes, nseg, shift, f32, entries, flush=True)
+        print(sizes, shift, f32, entries, flush=True)
         m.lin_scan([] if decode else pieces, kind=m.LIN_DELTA, H=H, G=G, N=N, dv=dv, vp=vp, inp=inp.data_ptr(), ld=ld, **off,
-                   **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr(), state=state.data_ptr(), slots=slots, nseg=nseg,
-                   seg=seg.data_ptr(), seg_dec=mat.data_ptr(), pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
+                   **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr(), state=state.data_ptr(), slots=slots, pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
                    **{k: v.data_ptr() for k, v in buf.items()}, y=y.data_ptr(), eps=eps, out_scale=osc, out=out.data_ptr(),
                    ldo=inner + 64, f32=f32, work=work.data_ptr(), stream=stream())
         torch.cuda.synchronize()
@@ -150,8 +148,8 @@ def test_delta_rule_kernels(sizes, nseg, shift, f32):
     go([(5, 4, 1), (2, 82, 1)], True)
     go([(5, 4, 1), (2, 82, 1)])                                     # again, as portions of one token
     go([(2, 83, 48), (0, 102, 128), (3, 32, 66), (5, 5, 3)])        # even lengths: in and out at one parity
-    go([(4, 0, 390), (1, 0, 130)])                                  # several segments, the last one short
-    go([(1, 130, 370), (4, 390, 1), (5, 8, 2)])                     # ... from a state, in place (even length)
+    go([(4, 0, 390), (1, 0, 130)])                                  # long, unequal
+    go([(1, 130, 370), (4, 390, 1), (5, 8, 2)])                     # from a state, in place (even length)
     go([(4, 391, 309), (5, 10, 6)])
     X[0] = inputs(70)
     want[0] = ref(X[0]), soft(X[0])
