@@ -279,7 +279,7 @@ __device__ __forceinline__ void delta_request(const LinScanArgs& a, size_t p, in
 }
 
 template <bool F32, int NT>
-__global__ void __launch_bounds__(64 * (DELTA_W + DELTA_L)) __attribute__((amdgpu_waves_per_eu(2))) delta_walk_kernel(LinScanArgs a) {
+__global__ void __launch_bounds__(64 * (DELTA_W + DELTA_L)) __attribute__((amdgpu_waves_per_eu(!F32 && NT <= 8 ? 2 : 1))) delta_walk_kernel(LinScanArgs a) {
   using L = DeltaStage<F32, NT>;
   // What a step reads is in registers before it begins where they and LDS have room (AHEAD): its rows since the step before was
   // half done, the rest since that one's end.

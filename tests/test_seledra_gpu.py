@@ -63,7 +63,7 @@ def oracle(name, cfg, w, ids):
 
 # ---- kernels alone -----------------------------------------------------------------------------------
 DELTA = [(6, 2, 20, 24, 3), (6, 6, 40, 32, 4), (3, 1, 128, 64, 2), (2, 1, 200, 16, 1), (5, 5, 70, 200, 10), (8, 2, 33, 300, 7),
-         (1, 1, 64, 640, 4), (32, 16, 128, 128, 4)]
+         (1, 1, 64, 640, 4), (4, 2, 180, 72, 4), (32, 16, 128, 128, 4)]
 
 
 @pytest.mark.parametrize("f32", [0, 1])
