@@ -524,8 +524,8 @@ PYBIND11_MODULE(AIOS_MODULE, m) {
   m.def("gemv",
         [](std::vector<PyQMatrix*> segs, int B, uintptr_t x, int ldx, uintptr_t norm_w, float eps, uintptr_t y,
            int ldy, int epi, uintptr_t st, int force_v1, int act_q8, int tune_grid, int tune_u, int tune_ksplit, int tune_dbg,
-           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16, uintptr_t bias, float pos, float neg,
-           float scale) {
+           int kernel_sel, uintptr_t dbg_ts, uintptr_t x16, uintptr_t y16, int act, int glu_row0, int ldy16, uintptr_t bias,
+           float pos, float neg, float scale) {
           GemvArgs a;
           std::memset(&a, 0, sizeof(a));
           a.nseg = (int)segs.size();

@@ -49,7 +49,6 @@ struct GemvArgs {
   bf16_t* y16;                  // EPI_SWIGLU: bf16 output [B][ldy] written instead of y (or null)
   int epi;
   int act;                      // gate activation of the GLU epilogues (GluAct)
-  ActNum act_n;                 // EPI_ACT16
   int glu_row0, ldy16;          // EPI_STORE_GLU
   // QKV epilogue
   const float* bias;            // [N] or null
@@ -62,8 +61,13 @@ struct GemvArgs {
   bf16_t* k_cache;              // layer base of the paged pool [blocks][n_kv][KV_BLOCK][hd]
   const int* block_table;       // [slots][max_ctx / KV_BLOCK] or null (identity)
   bf16_t* v_cache;
-  int kv_fp8;                   // KV pool in fp8 e4m3: stores code = value * kv_inv_{k,v}
-  float kv_inv_k, kv_inv_v;
+  union {                       // (of two epilogues: the batch-1 kernels' launches feel every argument byte)
+    struct {
+      int kv_fp8;               // EPI_QKV: KV pool in fp8 e4m3: stores code = value * kv_inv_{k,v}
+      float kv_inv_k, kv_inv_v;
+    };
+    ActNum act_n;               // EPI_ACT16
+  };
   // batch-1 decode: {pos, physical KV block} and the RoPE (cos, sin) row of this step's position,
   // prepared by the step's embedding launch (StepPrep, ops.h) -- no pos -> block table / rope chain
   // in the QKV kernel (null: looked up from pos / slot / block_table)

@@ -279,7 +279,8 @@ __device__ __forceinline__ void delta_request(const LinScanArgs& a, size_t p, in
 }
 
 template <bool F32, int NT>
-__global__ void __launch_bounds__(64 * (DELTA_W + DELTA_L)) __attribute__((amdgpu_waves_per_eu(!F32 && NT <= 8 ? 2 : 1))) delta_walk_kernel(LinScanArgs a) {
+__global__ void __launch_bounds__(64 * (DELTA_W + DELTA_L)) __attribute__((amdgpu_waves_per_eu(!F32 && NT <= 8 ? 2 : 1)))
+delta_walk_kernel(LinScanArgs a) {
   using L = DeltaStage<F32, NT>;
   // What a step reads is in registers before it begins where they and LDS have room (AHEAD): its rows since the step before was
   // half done, the rest since that one's end.
@@ -467,7 +468,8 @@ static void delta_walk(const LinScanArgs& a, hipStream_t st) {
     constexpr int NT = decltype(nt)::value;
     using L = DeltaStage<F32, NT>;
     const int groups = a.H * ((a.vp / 16 + DELTA_W - 1) / DELTA_W);
-    hipLaunchKernelGGL((delta_walk_kernel<F32, NT>), dim3((groups + 7) / 8 * 8, a.n_seqs), dim3(64 * (DELTA_W + DELTA_L)), L::N * L::BYTES, st, a);
+    hipLaunchKernelGGL((delta_walk_kernel<F32, NT>), dim3((groups + 7) / 8 * 8, a.n_seqs), dim3(64 * (DELTA_W + DELTA_L)),
+                       L::N * L::BYTES, st, a);
   };
   switch (a.np / 16) {
     case 2: walk(std::integral_constant<int, 2>{}); break;

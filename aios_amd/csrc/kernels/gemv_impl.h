@@ -183,6 +183,8 @@ __device__ __forceinline__ void gemv_tile(const QWeight& w, int row0, int k0, in
   }
 }
 
+// ACT: with EPI_ACT16 (the BF16 engine's)
+template <bool ACT = false>
 __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b, float v0, float v1) {
   const int nrow = a.row_base + a.N;
   switch (a.epi) {
@@ -212,6 +214,7 @@ __device__ __forceinline__ void gemv_epilogue(const GemvArgs& a, int grow, int b
       *y = make_float2(o.x + v0 + c.x, o.y + v1 + c.y);
     } break;
     case EPI_ACT16: {
+      if constexpr (!ACT) break;
       if (a.bias) { v0 += a.bias[grow]; v1 += a.bias[grow + 1]; }
       *(uint32_t*)(a.y16 + (size_t)b * a.ldy16 + grow) =
           (uint32_t)f32_to_bf16(unary_act(v0, a.act, a.act_n)) | (uint32_t)f32_to_bf16(unary_act(v1, a.act, a.act_n)) << 16;

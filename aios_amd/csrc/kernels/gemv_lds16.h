@@ -267,7 +267,7 @@ __global__ void __launch_bounds__(LG_THREADS) gemv_lds16(GemvArgs a, CuPlan pl) 
 #pragma unroll
       for (int bb = 1; bb < B; ++bb)
         if (b == bb) s_ = sb[bb];
-      gemv_epilogue(a, a.row_base + r0 + 2 * p, b, rowacc[b * pl.racc_n + 2 * p] * s_,
+      gemv_epilogue<true>(a, a.row_base + r0 + 2 * p, b, rowacc[b * pl.racc_n + 2 * p] * s_,
                     rowacc[b * pl.racc_n + 2 * p + 1] * s_);
     }
     return;
@@ -298,7 +298,7 @@ __global__ void __launch_bounds__(LG_THREADS) gemv_lds16(GemvArgs a, CuPlan pl) 
         }
         cu_qkv_epilogue(a, grow, v0, v1, t, pos0, kv_blk0);
       } else {
-        gemv_epilogue1(a, grow, v0, v1);
+        gemv_epilogue1<true>(a, grow, v0, v1);
       }
     }
   }

@@ -465,6 +465,8 @@ __device__ __forceinline__ void qkv_part(const GemvArgs& a, int grow, int& part,
   lr = r - head * hd;
 }
 // rope: (cos, sin) of this pair at pos0 (QKV; ignored for V rows and the other epilogues)
+// ACT: with EPI_ACT16 (the BF16 engine's)
+template <bool ACT = false>
 __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, float v0, float v1, float2 rope = {1.f, 0.f},
                                                int pos0 = 0, int kv_blk0 = 0) {
   const int nrow = a.row_base + a.N;
@@ -492,6 +494,7 @@ __device__ __forceinline__ void gemv_epilogue1(const GemvArgs& a, int grow, floa
       *y = make_float2(o.x + v0 + c.x, o.y + v1 + c.y);
     } break;
     case EPI_ACT16: {
+      if constexpr (!ACT) break;
       if (a.bias) {
         v0 += a.bias[grow];
         v1 += a.bias[grow + 1];

@@ -59,7 +59,9 @@ __device__ __forceinline__ void put1(void* base, size_t at, float v) {
 
 // Operands of delta_rule.hip are ordered so that the eight numbers a lane takes into a 32-deep product are neighbours: token t
 // of channel i in a block's and group's rows (a column's 32 tokens: four of the first block, the same four of the second, ..)
-__device__ __forceinline__ size_t pair_row(int i, int t) { return (i >> 5) * 512 + t * 32 + ((i >> 2) & 3) * 8 + ((i >> 4) & 1) * 4 + (i & 3); }
+__device__ __forceinline__ size_t pair_row(int i, int t) {
+  return (i >> 5) * 512 + t * 32 + ((i >> 2) & 3) * 8 + ((i >> 4) & 1) * 4 + (i & 3);
+}
 
 // a block's rows of the step
 struct LinBlock {

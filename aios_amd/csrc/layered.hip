@@ -609,7 +609,8 @@ void LayeredDecoder::init_random(uint64_t seed) {
   for (const auto& t : tensors_) {
     const int rows = t.second.first, cols = t.second.second;
     const size_t n = (size_t)rows * cols;
-    const bool norm = t.first.find("norm") != std::string::npos || t.first.find("attn_temp") != std::string::npos, sink = t.first.find("sinks") != std::string::npos;
+    const bool norm = t.first.find("norm") != std::string::npos || t.first.find("attn_temp") != std::string::npos;
+    const bool sink = t.first.find("sinks") != std::string::npos;
     const bool bias = t.first.find(".bias") != std::string::npos;
     bf16_t* tmp = nullptr;
     if (norm || sink || bias) {

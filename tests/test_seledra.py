@@ -105,8 +105,8 @@ def test_oracle_mechanisms_by_hand():
 
 FAULTS = ["no position", "position shifted", "q norm per head", "k norm per head", "norm weights", "one-plus norm", "no value norm",
           "value norm over all", "no temp", "temp per key head", "scale", "learned sink", "no sink", "q bias", "k bias", "v bias",
-          "wrong key head", "values not mixed", "mixed the other way", "mixed in the first", "mixed with the one before",
-          "mixed where not asked", "no gate per head", "gate of the residual", "taps reversed", "conv lost", "no silu after the conv",
+          "wrong key head", "values not mixed", "mixed the other way", "first mixed with zeros", "mixed with the one before",
+          "mixed where not asked", "no gate per head", "gate of another head", "taps reversed", "conv lost", "no silu after the conv",
           "conv of v left out", "no unit q", "no unit k", "q scale", "state lost", "decay", "decay after the write", "no decay in the read",
           "no strength", "strength shifted", "read before the write", "no delta", "wrong group", "no step bias", "delta norm per row",
           "delta norm weight", "delta gate", "xielu numbers swapped", "xielu below zero", "residual scale", "residual scale of the mlp",
@@ -133,8 +133,8 @@ def test_a_fault_in_any_mechanism_shows(fault, monkeypatch):
         w = over(lambda v: v + 1.5, "dt_bias")
     good = O.forward(cfg, w, ids)
     zero = lambda *ends: over(torch.zeros_like, *ends)
-    real = {n: getattr(O, n) for n in ("rms", "whole_norm", "value_norm", "mix_values", "scores", "weights", "attention", "causal_conv", "unit",
-                                       "decay", "delta_rule", "delta", "silu", "xielu", "embed", "feed_forward")}
+    real = {n: getattr(O, n) for n in ("rms", "whole_norm", "value_norm", "mix_values", "attention", "causal_conv", "unit", "decay",
+                                       "delta_rule", "delta", "silu", "xielu", "feed_forward")}
     patch = lambda n, f: monkeypatch.setattr(O, n, f)
     cut = lambda f: (lambda *a: torch.cat([f(*(x[:30] for x in a)), f(*(x[30:] for x in a))]))
 
@@ -192,9 +192,17 @@ def test_a_fault_in_any_mechanism_shows(fault, monkeypatch):
         patch("mix_values", lambda v, f, l: v)
     elif fault == "mixed the other way":
         patch("mix_values", lambda v, f, l: real["mix_values"](f, v, l + 0.2))
-    elif fault == "mixed in the first":  # (the first layer's number used on its own values)
-        w = over(lambda v: v * 1.7, "l2.mix.v")
-        patch("value_norm", lambda v, eps: real["rms"](v, eps) * (0.5 if v.shape[1] == 3 else 1))
+    elif fault == "first mixed with zeros":
+        def att(h, w, p, m, eps, shared):
+            if not m["v_mix"] or "values" in shared:
+                return real["attention"](h, w, p, m, eps, shared)
+            with monkeypatch.context() as mp:
+                seen = []
+                mp.setattr(O, "value_norm", lambda v, e: (seen.append(real["rms"](v, e)), (1 - w[p + "vmix"]) * seen[0])[1])
+                y = real["attention"](h, w, p, m, eps, shared)
+            shared["values"] = seen[0]
+            return y
+        monkeypatch.setitem(O.MIXERS, "attention", att)
     elif fault == "mixed with the one before":
         def att(h, w, p, m, eps, shared):
             with monkeypatch.context() as mp:
@@ -210,8 +218,10 @@ def test_a_fault_in_any_mechanism_shows(fault, monkeypatch):
                                 dict(l, mixer=dict(l["mixer"], v_mix=False)) if l["type"] == "attention" else l
                                 for i, l in enumerate(cfg["layers"])])
         w = dict(w, **{"l1.mix.vmix": torch.tensor(0.5)})
-    elif fault == "gate of the residual":
-        monkeypatch.setitem(O.MIXERS, "attention", lambda h, w, p, m, e, s: real["attention"](h, dict(w, **{p + "g": w[p + "g"].roll(1, 0)}), p, m, e, s))
+    elif fault == "gate of another head":
+        def att(h, w, p, m, eps, shared):
+            return real["attention"](h, dict(w, **{p + "g": w[p + "g"].roll(1, 0)}), p, m, eps, shared)
+        monkeypatch.setitem(O.MIXERS, "attention", att)
     elif fault == "taps reversed":
         w = over(lambda v: v.flip(1), ".conv")
     elif fault == "conv lost":  # a portion that starts without its predecessor's last inputs

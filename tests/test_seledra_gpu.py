@@ -131,7 +131,8 @@ def test_delta_rule_kernels(sizes, shift, f32):
         pd, sd = (torch.tensor(v, dtype=torch.int32, device="cuda") for v in zip(*[(p[3], p[2]) for p in pieces]))
         print(sizes, shift, f32, entries, flush=True)
         m.lin_scan([] if decode else pieces, kind=m.LIN_DELTA, H=H, G=G, N=N, dv=dv, vp=vp, inp=inp.data_ptr(), ld=ld, **off,
-                   **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr(), state=state.data_ptr(), slots=slots, pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
+                   **{k: v.data_ptr() for k, v in D.items()}, ring=ring.data_ptr(), state=state.data_ptr(), slots=slots,
+                   pos=pd.data_ptr(), slot=sd.data_ptr(), n=n,
                    **{k: v.data_ptr() for k, v in buf.items()}, y=y.data_ptr(), eps=eps, out_scale=osc, out=out.data_ptr(),
                    ldo=inner + 64, f32=f32, work=work.data_ptr(), stream=stream())
         torch.cuda.synchronize()
@@ -233,8 +234,8 @@ def test_attention_with_norms_temperatures_and_mixed_values(H, G, dk, dv, rot, w
              tiles=torch.tensor(tiles, dtype=torch.int32))
     D = {k: dev(v) for k, v in D.items()}
     part_of = dict(qn=dev(qn), kn=dev(kn), temp=dev(temp), lambda_=dev(lam))
-    small = H * dk <= 700
-    for qk, vn, tm, mix, nsplit in [(1, 1, 1, 2, 1), (1, 1, 1, 1, 3)] + ([(0, 0, 1, 0, 64), (1, 0, 0, 0, 1), (0, 1, 0, 2, 3)] if small else []):
+    some = [(0, 0, 1, 0, 64), (1, 0, 0, 0, 1), (0, 1, 0, 2, 3)] if H * dk <= 700 else []
+    for qk, vn, tm, mix, nsplit in [(1, 1, 1, 2, 1), (1, 1, 1, 1, 3)] + some:
         want, mine = ref(qk, vn, tm, mix)
         nsplit = 1 if f32 else nsplit
         pool, fd = dev(blk.to(dt)), dev(first if mix == 2 else torch.full_like(first, float("nan")))
