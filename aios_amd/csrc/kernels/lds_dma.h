@@ -18,7 +18,7 @@ __device__ __forceinline__ void pf_vmcnt() {
 // LDS-DMA through inline asm: hipcc's waitcnt pass then does not see the DMA, so it no longer puts
 // an `s_waitcnt vmcnt(0)` in front of the first ds_read after every issue (it cannot prove the read
 // misses the DMA's target slot -- measured: that drain serialised every K-step).  The counted
-// pf_vmcnt waits below are the only ordering these loads need.  M0 is set and restored inside the
+// pf_vmcnt waits are the only ordering these loads need.  M0 is set and restored inside the
 // statement.
 __device__ __forceinline__ uint32_t pf_lds_addr(const uint8_t* p) {
   return (uint32_t)(uintptr_t)(const __attribute__((address_space(3))) uint8_t*)p;
